@@ -42,6 +42,9 @@ enum {
     PIE_SAMPLER_KIND_DIST = 6, PIE_SAMPLER_KIND_RAW_LOGITS = 7, PIE_SAMPLER_KIND_LOGPROB = 8,
     PIE_SAMPLER_KIND_LOGPROBS = 9, PIE_SAMPLER_KIND_ENTROPY = 10
 };
+/* Bits of rs_slot_flags: the request's state starts from zero before its rows of this forward
+ * (also implied by a first position of 0). */
+enum { PIE_RS_RESET = 1 };
 enum { PIE_COPY_D2H = 0, PIE_COPY_H2D = 1, PIE_COPY_D2D = 2, PIE_COPY_H2H = 3 };
 enum { PIE_RESOURCE_KV = 0, PIE_RESOURCE_RS = 1 };
 enum { PIE_ADAPTER_LOAD = 0, PIE_ADAPTER_SAVE = 1, PIE_ADAPTER_ZO_INIT = 2,
@@ -244,6 +247,8 @@ PieHipDriver* pie_hip_driver_create(const char* config_toml, char* err, size_t e
 void pie_hip_driver_destroy(PieHipDriver* d);
 /* Capabilities JSON, valid for the driver's lifetime. */
 const char* pie_hip_driver_capabilities(const PieHipDriver* d);
+/* Message of the last failed forward ("" before one), valid until the next call. */
+const char* pie_hip_driver_last_error(const PieHipDriver* d);
 /* Handle one frame; *out stays valid until the next call on this driver.  Returns 0. */
 int pie_hip_driver_handle(PieHipDriver* d, const PieFrameDesc* frame, PieResponseFrameDesc* out);
 /*

@@ -45,8 +45,10 @@ extern "C" {
  *      argument of pie_hip_kv_write_quant / pie_hip_qkv_rope_kvwrite_quant; KV scale pools
  *      [pages, hk, page_size] (were [pages, page_size, hk]); int4 tile-major weights in decode
  *      order (pie_hip_repack_mfma_tiles_int4); pie_hip_gemv_time_next removed
- *   3  current */
-#define PIE_HIP_ABI_VERSION 3
+ *   3  lm_head argmax pairs, attention merge in the output projection, uniform-row hints
+ *   4  current: the `swiglu` argument of the linears is an epilogue code (PIE_HIP_EPI_*: 0 and 1
+ *      mean what they did, 2 is the squared ReLU); the layer-stack kernels */
+#define PIE_HIP_ABI_VERSION 4
 int pie_hip_abi_version(void);
 
 /* ---- W4A16 ("int4b8", symmetric, group-quantised) ------------------------- */
@@ -106,6 +108,11 @@ int pie_hip_gemv_w4a16_tuned(const uint16_t* act_bf16, const uint32_t* packed,
  * Replaces the rmsnorm -> gemm_act_x_w (-> swiglu) sequences of
  * driver/cuda/src/model/llama_like.cpp:370-705.
  */
+/* Epilogue codes, the `swiglu` argument of every linear entry point: PIE_HIP_EPI_RELU2 stores
+ * y[m, n] = bf16( max(sum, 0)^2 ) (all N columns; not combinable with beta). */
+#define PIE_HIP_EPI_NONE 0
+#define PIE_HIP_EPI_SWIGLU 1
+#define PIE_HIP_EPI_RELU2 2
 #define PIE_HIP_FMT_INT4B8 0
 #define PIE_HIP_FMT_INT8 1
 #define PIE_HIP_FMT_FP8 2
@@ -756,6 +763,107 @@ int pie_hip_quant_fp8_per_channel(const uint16_t* w_bf16, uint8_t* q_e4m3, float
  * layout (driver/cuda/src/kernels/dequant_wna16.cu:11-38) but ships no quantiser for it. */
 int pie_hip_quant_int4b8_group(const uint16_t* w_bf16, uint32_t* packed, uint16_t* scale_bf16,
                                int rows, int cols, int group_size, void* stream);
+
+/* ---- layer stacks --------------------------------------------------------------- */
+/*
+ * Kernels of models whose layers are listed one by one (latent attention, gated delta rule,
+ * squared-ReLU feed-forward, norms on the sublayers' outputs).  No counterpart in the reference.
+ * dtype: the compute type, i.e. the storage of activations, of the latent cache and of the
+ * convolution state (void pointers below).  Weights of products are bf16 in both types; norms,
+ * angles, softmax, recurrences and the residual stream are fp32 in both.
+ */
+#define PIE_HIP_DT_BF16 0
+#define PIE_HIP_DT_F32 1
+
+/* x[n, :] = table[token_ids[n], :] (ids >= vocab read row 0) in fp32 and, as x_act, in the compute
+ * type; rows of ld values, columns from the width on are zero. */
+int pie_hip_embed_stream(int dtype, const uint32_t* token_ids, const uint16_t* table_bf16, float* x,
+                         void* x_act, int num_tokens, int width, int ld, int vocab, void* stream);
+/* x += y / sqrt(mean(y^2) + eps) * weight; x_act = the new x in the compute type. */
+int pie_hip_norm_add(int dtype, const void* y, const float* weight, float* x, void* x_act, int rows, int width,
+                     int ldy, int ld, float eps, void* stream);
+/* out[s, :] = x[rows[s], :] / sqrt(mean(x^2) + eps) * weight in the compute type (zeros from the
+ * width to ld). */
+int pie_hip_norm_rows(int dtype, const float* x, const uint32_t* rows, const float* weight, void* out,
+                      int num_out, int width, int ld, int num_rows, float eps, void* stream);
+/* logits[s, v] = cap * tanh(y[s, v] * scale / cap) (cap 0: y * scale) in fp32, and tokens[s], the
+ * index of the largest (lowest among equals, NaN never wins). */
+int pie_hip_logits_finish(int dtype, const void* y, float* logits, uint32_t* tokens, int rows, int vocab,
+                          int ldy, float scale, float cap, void* stream);
+/* table[n, i] = cos(a) * mscale, table[n, dims/2 + i] = sin(a) * mscale with a = positions[n] *
+ * freq[i]; angles are formed and reduced in double. */
+int pie_hip_rotary_table(const int32_t* positions, const double* freq, float* table, int num_tokens, int dims,
+                         float mscale, void* stream);
+/* y[M, N] = act[M, K] . W[N, K]^T in fp32 over bf16 weights; epilogue PIE_HIP_EPI_NONE / _RELU2. */
+int pie_hip_linear_f32(const float* act, const uint16_t* w_bf16, float* y, int M, int N, int K, int epilogue,
+                       void* stream);
+
+/*
+ * Latent attention.  A cache row is [kvp latent | rotated key part] (ld_row values, zero padded);
+ * the pool is [pages * page_size, ld_row], one per layer, kv_slots / page lists as for the K / V
+ * pools.
+ * pie_hip_latent_prep: fused[n] = [query latent q_rank | .. | kv_off: latent kv_rank, rot_dim key
+ *   values]; cq[n] = the query latent normed (compact rows of ld_cq, zero padded); the token's
+ *   cache row = the normed latent and the key values rotated in adjacent pairs (first rot_dims of
+ *   them, table of pie_hip_rotary_table).
+ * pie_hip_head_linear: y[n, h, c] = sum_k W[h, c, k] act[n, h, k] (heads act_stride / y_stride
+ *   apart in rows of ld_act / ld_y; C % 16 == 0, K % 32 == 0).  With rope_table also
+ *   y[n, h, C + i] = the rotated act[n, h, rot_off + i], i < rot_dim, zeros to rotp.
+ * pie_hip_latent_attn_rows_plain: o[n, h, :] = softmax_j(q[n, h, :] . row_j * scale) . row_j[:kvp]
+ *   over the first row_kv_len[n] keys; q [rows, heads, ld_row], o [rows, heads, kvp].  Any sizes
+ *   (kvp <= 2048).
+ */
+int pie_hip_latent_prep(int dtype, const void* fused, const float* q_norm, const float* kv_norm,
+                        const float* rope_table, const int64_t* kv_slots, void* cq, void* pool, int num_tokens,
+                        int ld_fused, int kv_off, int q_rank, int ld_cq, int kv_rank, int kvp, int rot_dim,
+                        int rot_dims, int ld_row, float eps, void* stream);
+int pie_hip_head_linear(int dtype, const void* act, const uint16_t* w_bf16, void* y, const float* rope_table,
+                        int M, int heads, int C, int K, int ld_act, int act_stride, int ld_y, int y_stride,
+                        int rot_off, int rot_dim, int rot_dims, int rotp, void* stream);
+int pie_hip_latent_attn_rows_plain(int dtype, const void* q, const void* pool, void* o,
+                                   const uint32_t* kv_page_indices, const uint32_t* row_page_begin,
+                                   const int32_t* row_kv_len, int num_rows, int heads, int kvp, int ld_row,
+                                   int page_size, float scale, void* stream);
+
+/*
+ * Gated delta rule with a decay per head and key channel.  row_req [N]: request of each row;
+ * qo_indptr [R + 1]: rows of each request; rs_slot [R]: its slot of the state pool (rs_base + slot *
+ * rs_stride bytes); rs_fresh [R]: 1 = starts from zero.  The fp32 state [heads, dim, vdim] sits at
+ * state_offset of the slot, the last taps - 1 convolution inputs [taps - 1, channels] (compute type,
+ * channels = q | k | v) at conv_offset.
+ * pie_hip_delta_prep: fused[n] = [q | k | v | step sizes (heads) | .. decay_off: decay_rank | ..
+ *   gate_off: gate_rank].  q, k: causal convolution (conv_w [channels, taps], the last column is the
+ *   current token's), silu, unit vector x / sqrt(sum x^2 + 1e-6) per head, q also times dim^-1/2;
+ *   v: convolution, silu; beta = sigmoid(step size); a1, g1: the low-rank inputs, compact, zero
+ *   padded.  dim <= 512.
+ * pie_hip_delta_decay: g = exp(-exp(a_log[head]) * softplus(raw + dt_bias)), [N, heads * dim].
+ * pie_hip_delta_scan: per token S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q; head h
+ *   uses q / k head h / (heads / kv_heads).  Reads and writes the state.  dim <= 256.
+ * pie_hip_delta_out: y = o / sqrt(mean(o^2) + eps) * norm_w * sigmoid(gate) per head; writes the
+ *   convolution state.
+ */
+int pie_hip_delta_prep(int dtype, const void* fused, const float* conv_w, const void* rs_base, size_t rs_stride,
+                       size_t conv_offset, const int32_t* row_req, const int32_t* qo_indptr,
+                       const int32_t* rs_slot, const int32_t* rs_fresh, float* q, float* k, float* v, float* beta,
+                       void* a1, void* g1, int num_tokens, int ld, int heads, int kv_heads, int dim, int vdim,
+                       int taps, int decay_off, int decay_rank, int ld_a1, int gate_off, int gate_rank, int ld_g1,
+                       void* stream);
+int pie_hip_delta_decay(int dtype, const void* raw, const float* a_log, const float* dt_bias, float* g,
+                        int num_tokens, int ld_raw, int heads, int dim, void* stream);
+int pie_hip_delta_scan(const float* q, const float* k, const float* v, const float* g, const float* beta, float* o,
+                       void* rs_base, size_t rs_stride, size_t state_offset, const int32_t* qo_indptr,
+                       const int32_t* rs_slot, const int32_t* rs_fresh, int num_requests, int heads, int kv_heads,
+                       int dim, int vdim, void* stream);
+int pie_hip_delta_out(int dtype, const float* o, const void* gate, const float* norm_w, void* y, const void* fused,
+                      void* rs_base, size_t rs_stride, size_t conv_offset, const int32_t* row_req,
+                      const int32_t* qo_indptr, const int32_t* rs_slot, const int32_t* rs_fresh, int num_tokens,
+                      int ld_gate, int ld_y, int ld_fused, int heads, int kv_heads, int dim, int vdim, int taps,
+                      float eps, void* stream);
+
+/* pie_hip_sample_gather_logits over fp32 logits. */
+int pie_hip_sample_gather_logits_f32(const float* logits, const int32_t* rows, float* out_f32,
+                                     const uint32_t* mask_bounds, const int32_t* mask_bounds_indptr,
+                                     int num_slots, int vocab, void* stream);
 
 #ifdef __cplusplus
 }

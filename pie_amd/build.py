@@ -55,6 +55,10 @@ def _run(cmd: list[str]) -> None:
         sys.stderr.write(err + "\n")
 
 
+def _jobs() -> int:
+    return min(int(os.environ.get("MAX_JOBS", 8)), os.cpu_count() or 1)
+
+
 def hip_sources() -> list[Path]:
     return sorted(CSRC.glob("*.hip"))
 
@@ -69,7 +73,7 @@ def build_kernels(force: bool = False, jobs: int | None = None) -> Path:
         objs.append(obj)
         if force or not _newer(obj, [src] + headers):
             todo.append([HIPCC, *HIP_FLAGS, "-c", str(src), "-o", str(obj)])
-    jobs = jobs or min(8, os.cpu_count() or 1)
+    jobs = jobs or _jobs()
     with ThreadPoolExecutor(max_workers=jobs) as pool:
         list(pool.map(_run, todo))
     if force or todo or not KERNEL_LIB.exists():
@@ -90,7 +94,7 @@ def build_driver(force: bool = False, jobs: int | None = None) -> Path:
         objs.append(obj)
         if force or not _newer(obj, [src] + headers):
             todo.append([HIPCC, *HIP_FLAGS, f"-I{DRIVER_SRC}", "-c", str(src), "-o", str(obj)])
-    jobs = jobs or min(8, os.cpu_count() or 1)
+    jobs = jobs or _jobs()
     with ThreadPoolExecutor(max_workers=jobs) as pool:
         list(pool.map(_run, todo))
     if force or todo or not DRIVER_LIB.exists() or not _newer(DRIVER_LIB, [KERNEL_LIB]):
@@ -98,6 +102,20 @@ def build_driver(force: bool = False, jobs: int | None = None) -> Path:
               *map(str, objs), f"-L{KERNEL_LIB.parent}", "-lpie_hip_kernels",
               "-Wl,-rpath,$ORIGIN", "-lpthread"])
     return DRIVER_LIB
+
+
+def ensure_built() -> None:
+    """Builds what is missing (a fresh checkout); libraries that are there are used as they are.
+    Processes that start at once wait for one of them."""
+    if KERNEL_LIB.exists() and DRIVER_LIB.exists():
+        return
+    import fcntl
+
+    OBJ_DIR.mkdir(parents=True, exist_ok=True)
+    with open(OBJ_DIR / "lock", "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        if not (KERNEL_LIB.exists() and DRIVER_LIB.exists()):
+            build_all()
 
 
 def build_all(force: bool = False) -> None:

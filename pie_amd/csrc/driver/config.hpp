@@ -13,12 +13,51 @@
 #include <stdexcept>
 #include <cctype>
 #include <string>
+#include <vector>
 
 namespace pie_hip_driver {
 
+// ---- layer stacks: models whose layers differ from one another ----------------------------------
+// Each layer names a mixer (what exchanges information between tokens) with its own sizes, and an
+// optional feed-forward.  Mixers are listed here once, with every constant a parameter.
+
+// Rotary embedding of the first `dims` entries of a vector, adjacent pairs.
+struct RotarySpec {
+    int dims = 0;
+    double base = 10000.0;
+    bool yarn = false;   // frequencies ramped between f and f / factor, cos / sin scaled
+    double factor = 1.0, original = 0.0, fast = 32.0, slow = 1.0;
+    bool operator==(const RotarySpec& o) const {
+        return dims == o.dims && base == o.base && yarn == o.yarn && factor == o.factor && original == o.original &&
+               fast == o.fast && slow == o.slow;
+    }
+};
+
+// Attention over a cached low-rank latent per token and one rotated key part shared by the heads.
+struct LatentAttentionSpec {
+    int heads = 0, dim = 0, rot_dim = 0, vdim = 0, q_rank = 0, kv_rank = 0;
+    double scale = 0.0;
+    RotarySpec rot;
+};
+
+// Gated delta rule with one decay per head and key channel; a short causal convolution before it.
+struct ChannelDeltaSpec {
+    int heads = 0, kv_heads = 0, dim = 0, vdim = 0, taps = 1;
+    int decay_rank = 0, gate_rank = 0;   // low-rank decay and output gate (a checkpoint's tensors fix them)
+};
+
+enum class MixerKind { LatentAttention, ChannelDelta };
+
+struct LayerSpec {
+    MixerKind mixer = MixerKind::LatentAttention;
+    LatentAttentionSpec latent;
+    ChannelDeltaSpec delta;
+    int ff = 0;   // squared-ReLU feed-forward of this width; 0: the layer has none
+};
+
 struct ModelConfig {
     // architecture: "llama3" (dense, adjacent-pair RoPE) | "qwen3" (dense, qk-norm, half-split
-    // RoPE) | "qwen3_moe"
+    // RoPE) | "qwen3_moe" | "varasun" (layer stack)
     std::string arch = "llama3";
     int hidden = 0, layers = 0, q_heads = 0, kv_heads = 0, head_dim = 0, intermediate = 0;
     int vocab = 0;
@@ -51,6 +90,16 @@ struct ModelConfig {
     // Face snapshot directory; its config.json then fixes the shape fields above and the weights
     // come from its safetensors files instead of the synthetic initialiser
     std::string checkpoint_dir;
+    // with checkpoint_dir: take only config.json from it and fill the weights synthetically
+    bool random_weights = false;
+    // layer stacks: the layers, and what follows the last one (logits = cap * tanh(scale * y / cap);
+    // cap 0: no cap).  Empty for the uniform architectures above.
+    std::vector<LayerSpec> stack;
+    float logit_scale = 1.f, logit_softcap = 0.f;
+    bool is_stack() const { return !stack.empty(); }
+    // activations and products: "bfloat16" | "float32" (layer stacks only: true 32-bit throughout)
+    std::string compute_dtype = "bfloat16";
+    bool f32() const { return compute_dtype == "float32"; }
 };
 
 struct BatchingConfig {
@@ -59,6 +108,9 @@ struct BatchingConfig {
     int max_forward_tokens = 10240;
     int max_forward_requests = 512;
     int cpu_pages = 0;
+    // recurrent state of layer stacks: sequences that can hold state at a time (0: one per request
+    // of a batch), and host slots they can be swapped to
+    int rs_cache_slots = 0, cpu_rs_slots = 0;
     // KV-cache storage (driver/cuda/src/config.hpp:66, kv_cache_format.cpp:46-110): auto | bf16 |
     // bfloat16 | fp8_e4m3 | int8_per_token_head | fp8_per_token_head
     std::string kv_cache_dtype = "auto";
@@ -181,8 +233,52 @@ inline int kv_format_code(const std::string& value) {
 }
 
 // Shape and range checks, defaults that depend on other fields.
+inline void finalize_batching(const BatchingConfig& b) {
+    if (b.kv_page_size <= 0 || b.kv_page_size % 16 != 0)
+        throw std::runtime_error("config: kv_page_size must be a positive multiple of 16");
+    if (b.total_pages <= 0 || b.max_forward_tokens <= 0 || b.max_forward_requests <= 0)
+        throw std::runtime_error("config: [batching] sizes must be positive");
+    if (b.rs_cache_slots < 0 || b.cpu_rs_slots < 0)
+        throw std::runtime_error("config: rs_cache_slots and cpu_rs_slots must not be negative");
+    (void)kv_format_code(b.kv_cache_dtype);
+}
+
+// Layer stacks: every layer's sizes, and the storage choices the stack executor has.
+inline void finalize_stack(DriverConfig& c) {
+    auto& m = c.model;
+    if (m.hidden <= 0 || m.vocab <= 0) throw std::runtime_error("config: a layer stack needs a width and a vocabulary");
+    for (size_t i = 0; i < m.stack.size(); ++i) {
+        const LayerSpec& l = m.stack[i];
+        const std::string at = "config: layer " + std::to_string(i) + ": ";
+        if (l.ff < 0) throw std::runtime_error(at + "negative feed-forward width");
+        if (l.mixer == MixerKind::LatentAttention) {
+            const auto& a = l.latent;
+            if (a.heads <= 0 || a.dim <= 0 || a.rot_dim < 0 || a.vdim <= 0 || a.q_rank <= 0 || a.kv_rank <= 0)
+                throw std::runtime_error(at + "latent_attention needs heads, dim, vdim, q_rank, kv_rank");
+            if (a.rot.dims < 0 || a.rot.dims % 2 != 0 || a.rot.dims > a.rot_dim)
+                throw std::runtime_error(at + "rot.dims must be even and at most rot_dim");
+            if (a.rot.dims > 0 && !(a.rot.base > 0.0)) throw std::runtime_error(at + "rot.base must be positive");
+        } else {
+            const auto& d = l.delta;
+            if (d.heads <= 0 || d.kv_heads <= 0 || d.dim <= 0 || d.vdim <= 0 || d.taps <= 0)
+                throw std::runtime_error(at + "channel_delta needs heads, kv_heads, dim, vdim, conv");
+            if (d.heads % d.kv_heads != 0) throw std::runtime_error(at + "heads must be a multiple of kv_heads");
+        }
+    }
+    if (m.compute_dtype != "bfloat16" && m.compute_dtype != "float32")
+        throw std::runtime_error("config: compute_dtype must be bfloat16 or float32");
+    m.quant = "bf16";   // the linears of layer stacks are kept as stored
+    m.layers = static_cast<int>(m.stack.size());
+    if (kv_format_code(c.batching.kv_cache_dtype) != 0)
+        throw std::runtime_error("config: layer stacks keep their cache in the compute type (kv_cache_dtype = auto)");
+    if (c.batching.rs_cache_slots == 0) c.batching.rs_cache_slots = c.batching.max_forward_requests;
+    finalize_batching(c.batching);
+}
+
 inline void finalize_config(DriverConfig& c) {
     auto& m = c.model;
+    if (m.is_stack()) return finalize_stack(c);
+    if (m.f32()) throw std::runtime_error("config: compute_dtype float32 is available for layer stacks only");
     if (m.hidden <= 0 || m.layers <= 0 || m.q_heads <= 0 || m.kv_heads <= 0 || m.vocab <= 0)
         throw std::runtime_error("config: [model] needs hidden, layers, q_heads, kv_heads, vocab");
     if (m.head_dim <= 0) m.head_dim = m.hidden / m.q_heads;
@@ -206,12 +302,7 @@ inline void finalize_config(DriverConfig& c) {
     if (m.rope_scaling.empty()) m.rope_scaling = "llama3";
     if (m.rope_scaling != "llama3" && m.rope_scaling != "yarn")
         throw std::runtime_error("config: rope_scaling must be llama3 or yarn");
-    const auto& b = c.batching;
-    if (b.kv_page_size <= 0 || b.kv_page_size % 16 != 0)
-        throw std::runtime_error("config: kv_page_size must be a positive multiple of 16");
-    if (b.total_pages <= 0 || b.max_forward_tokens <= 0 || b.max_forward_requests <= 0)
-        throw std::runtime_error("config: [batching] sizes must be positive");
-    (void)kv_format_code(b.kv_cache_dtype);
+    finalize_batching(c.batching);
 }
 
 inline DriverConfig parse_config_text(const std::string& text) {
@@ -256,6 +347,8 @@ inline DriverConfig parse_config_text(const std::string& text) {
                 else if (k == "init_std") m.init_std = (float)to_float(v, key);
                 else if (k == "router_std") m.router_std = (float)to_float(v, key);
                 else if (k == "embed_std") m.embed_std = (float)to_float(v, key);
+                else if (k == "random_weights") m.random_weights = to_bool(v, key);
+                else if (k == "compute_dtype") m.compute_dtype = v;
                 else if (k == "hf_path" || k == "snapshot_dir") m.checkpoint_dir = v;
                 // other [model] keys (paths, dtype hints) belong to loaders this driver lacks
             } else if (sec == "batching") {
@@ -265,6 +358,8 @@ inline DriverConfig parse_config_text(const std::string& text) {
                 else if (k == "max_forward_tokens") b.max_forward_tokens = (int)to_int(v, key);
                 else if (k == "max_forward_requests") b.max_forward_requests = (int)to_int(v, key);
                 else if (k == "cpu_pages") b.cpu_pages = (int)to_int(v, key);
+                else if (k == "rs_cache_slots") b.rs_cache_slots = (int)to_int(v, key);
+                else if (k == "cpu_rs_slots") b.cpu_rs_slots = (int)to_int(v, key);
                 else if (k == "kv_cache_dtype") b.kv_cache_dtype = v;
                 else throw std::runtime_error("config: unknown [batching] key '" + k + "'");
             } else if (sec == "runtime") {

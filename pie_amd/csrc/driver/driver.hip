@@ -6,6 +6,7 @@
 //   response CSR shape             driver/bridge/include/pie_bridge/response_builder.hpp:52-271
 //   entry points                   driver/portable/src/entry.cpp:483-505, server/src/driver_ffi.rs:18-46
 //   offline generation harness     driver/portable/src/executor/executor.cpp:1439-1597
+#include <algorithm>
 #include <atomic>
 #include <chrono>
 #include <csignal>
@@ -246,7 +247,8 @@ struct PieHipDriver {
         if (hipStreamCreateWithFlags(&s, hipStreamNonBlocking) != hipSuccess)
             throw std::runtime_error("cannot create a HIP stream");
         try {
-            if (cfg.model.checkpoint_dir.empty()) model.init_synthetic(cfg.model, s);
+            if (cfg.model.is_stack()) model.load_stack(cfg.model, s);
+            else if (cfg.model.checkpoint_dir.empty() || cfg.model.random_weights) model.init_synthetic(cfg.model, s);
             else model.load_snapshot(cfg.model, s);
             if (cfg.runtime.tiled_weights) model.build_tiled_copies(s);
         } catch (...) {
@@ -268,14 +270,15 @@ struct PieHipDriver {
         std::ostringstream j;
         j << "{\"total_pages\":" << total_pages << ",\"kv_page_size\":" << ps
           << ",\"swap_pool_size\":" << cfg.batching.cpu_pages
-          << ",\"rs_cache_required\":false,\"rs_cache_slots\":0,\"rs_cache_slot_bytes\":0"
+          << ",\"rs_cache_required\":" << (exec->rs_slots() > 0 ? "true" : "false")
+          << ",\"rs_cache_slots\":" << exec->rs_slots() << ",\"rs_cache_slot_bytes\":" << exec->rs_slot_bytes()
           << ",\"max_forward_tokens\":" << cfg.batching.max_forward_tokens
           << ",\"max_forward_requests\":" << cfg.batching.max_forward_requests
           << ",\"max_page_refs\":" << total_pages << ",\"max_logit_rows\":" << umax
           << ",\"max_prob_rows\":" << umax << ",\"max_custom_mask_bytes\":" << umax
           << ",\"max_sampler_rows\":" << umax << ",\"max_logprob_labels\":" << umax
           << ",\"arch_name\":\"" << json_escape(m.arch) << "\",\"vocab_size\":" << m.vocab
-          << ",\"max_model_len\":" << total_pages * ps << ",\"activation_dtype\":\"bfloat16\""
+          << ",\"max_model_len\":" << total_pages * ps << ",\"activation_dtype\":\"" << m.compute_dtype << "\""
           << ",\"snapshot_dir\":\"" << json_escape(cfg.runtime.snapshot_dir) << "\"}";
         caps = j.str();
     }
@@ -318,7 +321,7 @@ struct PieHipDriver {
     // outside its pool is out of range (3); pairs before a bad one have been copied.
     int copy(const PieCopyRequestDesc& c, uint32_t method) {
         if (c.srcs.len != c.dsts.len) return PIE_STATUS_FAILED;
-        if (method >= PIE_METHOD_COPY_RS_D2H) return PIE_STATUS_UNSUPPORTED;  // no recurrent state
+        if (method >= PIE_METHOD_COPY_RS_D2H) return copy_rs(c, method);
         const uint32_t dev = static_cast<uint32_t>(exec->total_pages());
         const uint32_t host = static_cast<uint32_t>(exec->cpu_pages());
         if (method != PIE_METHOD_COPY_KV_D2D && host == 0) return PIE_STATUS_UNSUPPORTED;
@@ -337,6 +340,24 @@ struct PieHipDriver {
             default: return PIE_STATUS_UNSUPPORTED;
         }
         return good == c.srcs.len ? PIE_STATUS_OK : PIE_STATUS_OUT_OF_RANGE;
+    }
+
+    // Recurrent-state slots: same checks and codes; unsupported for models without such state.
+    int copy_rs(const PieCopyRequestDesc& c, uint32_t method) {
+        const uint32_t dev = static_cast<uint32_t>(exec->rs_slots()), host = static_cast<uint32_t>(exec->cpu_rs_slots());
+        if (dev == 0 || (method != PIE_METHOD_COPY_RS_D2D && host == 0)) return PIE_STATUS_UNSUPPORTED;
+        const uint32_t src_cap = (method == PIE_METHOD_COPY_RS_D2H || method == PIE_METHOD_COPY_RS_D2D) ? dev : host;
+        const uint32_t dst_cap = (method == PIE_METHOD_COPY_RS_H2D || method == PIE_METHOD_COPY_RS_D2D) ? dev : host;
+        for (size_t i = 0; i < c.srcs.len; ++i)
+            if (c.srcs.ptr[i] >= src_cap || c.dsts.ptr[i] >= dst_cap) return PIE_STATUS_OUT_OF_RANGE;
+        switch (method) {
+            case PIE_METHOD_COPY_RS_D2D: exec->copy_rs_d2d(c.srcs.ptr, c.dsts.ptr, c.srcs.len); break;
+            case PIE_METHOD_COPY_RS_D2H: exec->copy_rs_d2h(c.srcs.ptr, c.dsts.ptr, c.srcs.len); break;
+            case PIE_METHOD_COPY_RS_H2D: exec->copy_rs_h2d(c.srcs.ptr, c.dsts.ptr, c.srcs.len); break;
+            case PIE_METHOD_COPY_RS_H2H: exec->copy_rs_h2h(c.srcs.ptr, c.dsts.ptr, c.srcs.len); break;
+            default: return PIE_STATUS_UNSUPPORTED;
+        }
+        return PIE_STATUS_OK;
     }
 
     void handle(const PieFrameDesc& frame, PieResponseFrameDesc& out) {
@@ -384,7 +405,7 @@ void set_err(char* err, size_t cap, const std::string& msg) {
 // Fills a forward frame over borrowed vectors (the harness plays the runtime's role).
 struct FrameBuilder {
     std::vector<uint32_t> tokens, positions, pages, page_indptr, last_lens, qo_indptr, samp_idx,
-        samp_indptr, sampler_indptr;
+        samp_indptr, sampler_indptr, rs_slots;
     std::vector<PieSamplerDesc> samplers;
     std::vector<uint64_t> ctx_ids;
     PieFrameDesc frame;
@@ -403,6 +424,7 @@ struct FrameBuilder {
         f.samplers = {samplers.data(), samplers.size()};
         f.sampler_indptr = {sampler_indptr.data(), sampler_indptr.size()};
         f.context_ids = {ctx_ids.data(), ctx_ids.size()};
+        f.rs_slot_ids = {rs_slots.data(), rs_slots.size()};
         f.single_token_mode = 1;
     }
 };
@@ -457,6 +479,8 @@ extern "C" const char* pie_hip_driver_capabilities(const PieHipDriver* d) {
     return d ? d->caps.c_str() : nullptr;
 }
 
+extern "C" const char* pie_hip_driver_last_error(const PieHipDriver* d) { return d ? d->last_error.c_str() : nullptr; }
+
 extern "C" int pie_hip_driver_handle(PieHipDriver* d, const PieFrameDesc* frame,
                                      PieResponseFrameDesc* out) {
     if (!d || !frame || !out) return -1;
@@ -473,6 +497,17 @@ extern "C" int pie_hip_driver_handle(PieHipDriver* d, const PieFrameDesc* frame,
 extern "C" size_t pie_hip_driver_export_tensor(PieHipDriver* d, const char* name, void* dst,
                                                size_t cap) {
     if (!d || !name) return 0;
+    if (d->cfg.model.is_stack()) {
+        // layer stacks: fp32 logits of the last forward's (last chunk of) sampled rows, weights
+        // in their padded layouts
+        if (std::string(name) == "debug.logits") {
+            const size_t bytes = static_cast<size_t>(d->exec->last_logit_rows()) * d->cfg.model.vocab * 4;
+            if (dst && bytes && hipMemcpy(dst, d->exec->last_logits_f32(), std::min(bytes, cap), hipMemcpyDeviceToHost) != hipSuccess)
+                return 0;
+            return bytes;
+        }
+        if (std::string(name).rfind("debug.", 0) == 0 || std::string(name).rfind("info.", 0) == 0) return 0;
+    }
     if (std::string(name) == "debug.logits") {
         const size_t bytes = static_cast<size_t>(d->exec->last_logit_rows()) * d->cfg.model.vocab * 2;
         if (dst && bytes) {
@@ -589,6 +624,9 @@ extern "C" int pie_hip_driver_generate(PieHipDriver* d, const uint32_t* prompt, 
                                      " pages, pool has " + std::to_string(d->exec->total_pages()));
         if (replicate > d->cfg.batching.max_forward_requests)
             throw std::runtime_error("generate: replicate exceeds max_forward_requests");
+        const bool recurrent = d->exec->rs_slots() > 0;   // context c keeps its state in slot c
+        if (recurrent && replicate > d->exec->rs_slots())
+            throw std::runtime_error("generate: replicate exceeds the recurrent-state slots");
         PieResponseFrameDesc resp;
         std::vector<uint32_t> last(replicate);
         const int chunk_cap = d->cfg.batching.max_forward_tokens;
@@ -609,6 +647,7 @@ extern "C" int pie_hip_driver_generate(PieHipDriver* d, const uint32_t* prompt, 
                 fb.last_lens = {static_cast<uint32_t>(upto - (np - 1) * ps)};
                 fb.qo_indptr = {0u, static_cast<uint32_t>(n)};
                 fb.ctx_ids = {static_cast<uint64_t>(c)};
+                if (recurrent) fb.rs_slots = {static_cast<uint32_t>(c)};
                 const bool final_chunk = upto == n_prompt;
                 if (final_chunk) {
                     fb.samp_idx = {static_cast<uint32_t>(n - 1)};
@@ -640,6 +679,11 @@ extern "C" int pie_hip_driver_generate(PieHipDriver* d, const uint32_t* prompt, 
                     dsts.push_back(static_cast<uint32_t>(c * pages_per_ctx + p));
                 }
             d->exec->copy_pages_d2d(srcs.data(), dsts.data(), srcs.size());
+            if (recurrent) {
+                std::vector<uint32_t> from(static_cast<size_t>(replicate) - 1, 0u), to;
+                for (int c = 1; c < replicate; ++c) to.push_back(static_cast<uint32_t>(c));
+                d->exec->copy_rs_d2d(from.data(), to.data(), to.size());
+            }
             for (int c = 1; c < replicate; ++c) {
                 last[c] = last[0];
                 out_tokens[static_cast<size_t>(c) * max_new] = last[0];
@@ -675,6 +719,7 @@ extern "C" int pie_hip_driver_generate(PieHipDriver* d, const uint32_t* prompt, 
                 if (sd.seed != 0) sd.seed += static_cast<uint32_t>(s * replicate + c);   // a fresh draw per slot
                 fb.samplers.push_back(sd);
                 fb.ctx_ids.push_back(static_cast<uint64_t>(c));
+                if (recurrent) fb.rs_slots.push_back(static_cast<uint32_t>(c));
             }
             for (int c = 0; c <= replicate; ++c) {
                 fb.page_indptr.push_back(static_cast<uint32_t>(c * np));

@@ -130,9 +130,11 @@ bool routes_to_gemv(const Linear& w, int M, bool has_norm, size_t ws_bytes) {
 // `force`: -1 = pick (the start-up measurement when there is one, else the cost model); 0..3 = that
 // kernel whatever the costs (the tuner's own launches).  Returns false when a forced kernel does
 // not take the shape.
+}  // namespace
+
 bool linear_fused(const Linear& w, const uint16_t* act, const uint16_t* norm_w, float eps,
                   uint16_t* y, int M, int beta, int swiglu, uint16_t* norm_tmp, void* gemm_ws,
-                  size_t gemm_ws_bytes, hipStream_t s, int force = -1) {
+                  size_t gemm_ws_bytes, hipStream_t s, int force) {
     const int fmt = fmt_code(w.kind);
     const int sbf = w.scale_bf16 ? 1 : 0;
     const int forced_rows = forced_gemv_rows();
@@ -190,12 +192,10 @@ bool linear_fused(const Linear& w, const uint16_t* act, const uint16_t* norm_w, 
     return true;
 }
 
-}  // namespace
-
 // Staged inputs are packed back to back in an order that makes every offset a function of
 // (rows, sampled rows) only — the page list goes last — so one contiguous host-to-device copy
 // feeds a forward and a captured graph's pointers stay valid for its (rows, sampled rows) key.
-Executor::Inputs Executor::input_layout(int N, int S) {
+Executor::Inputs Executor::input_layout(int N, int S) const {
     Inputs in{};
     size_t off = 0;
     in.off_tokens = off;       off = align_up(off + static_cast<size_t>(N) * 4, 256);
@@ -204,6 +204,11 @@ Executor::Inputs Executor::input_layout(int N, int S) {
     in.off_row_begin = off;    off = align_up(off + static_cast<size_t>(N) * 4, 256);
     in.off_row_len = off;      off = align_up(off + static_cast<size_t>(N) * 4, 256);
     in.off_sample_rows = off;  off = align_up(off + static_cast<size_t>(S) * 4, 256);
+    const size_t per_row = model_.cfg().is_stack() ? 4 : 0;
+    in.off_row_req = off;      off = align_up(off + N * per_row, 256);
+    in.off_qo = off;           off = align_up(off + (N + 1) * per_row, 256);
+    in.off_rs_slot = off;      off = align_up(off + N * per_row, 256);
+    in.off_rs_fresh = off;     off = align_up(off + N * per_row, 256);
     in.off_pages = off;
     in.total = off;
     return in;
@@ -216,26 +221,41 @@ Executor::Executor(const DriverConfig& cfg, Model& model) : cfg_(cfg), model_(mo
     max_tokens_ = cfg.batching.max_forward_tokens;
     max_page_refs_ = 4 * total_pages_ + max_tokens_;
     kv_format_ = kv_format_code(cfg.batching.kv_cache_dtype);
+    dt_ = model.cfg().f32() ? PIE_HIP_DT_F32 : PIE_HIP_DT_BF16;
     alloc_kv();
     cpu_pages_ = std::max(0, cfg.batching.cpu_pages);
-    if (cpu_pages_ > 0) {
-        const size_t bytes = static_cast<size_t>(model.cfg().layers) * 2 * cpu_pages_ *
-                             (page_bytes() + scale_page_bytes());
+    if (cpu_pages_ > 0 && swap_page_bytes_ > 0) {
+        const size_t bytes = swap_page_bytes_ * static_cast<size_t>(cpu_pages_);
         PIE_HIP_CHECK(hipHostMalloc(reinterpret_cast<void**>(&swap_pool_), bytes, hipHostMallocDefault));
         std::memset(swap_pool_, 0, bytes);
     }
 
-    const ModelConfig& m = model.cfg();
+    if (model.cfg().is_stack()) alloc_stack();
+    else alloc_uniform();
+
+    in_ = input_layout(max_tokens_, max_tokens_);
+    in_.total = align_up(in_.off_pages + static_cast<size_t>(max_page_refs_) * 4, 256);
+    PIE_HIP_CHECK(hipHostMalloc(reinterpret_cast<void**>(&in_host_), in_.total, hipHostMallocDefault));
+    PIE_HIP_CHECK(hipMalloc(reinterpret_cast<void**>(&in_dev_), in_.total));
+    out_cap_ = static_cast<size_t>(max_tokens_);
+    out_tokens_ = dmalloc<uint32_t>(out_cap_);
+    PIE_HIP_CHECK(hipHostMalloc(reinterpret_cast<void**>(&out_host_), out_cap_ * 4, hipHostMallocDefault));
+    tune_linears();
+}
+
+// Activation workspaces of the uniform architectures.
+void Executor::alloc_uniform() {
+    const ModelConfig& m = model_.cfg();
     const size_t T = static_cast<size_t>(max_tokens_);
     const int H = m.hidden, d = m.head_dim, hq = m.q_heads, hk = m.kv_heads;
-    const int I = model.is_moe() ? m.expert_intermediate : m.intermediate;
+    const int I = model_.is_moe() ? m.expert_intermediate : m.intermediate;
     x_ = dmalloc<uint16_t>(T * H);
     xn_ = dmalloc<uint16_t>(T * H);
     qkv_ = dmalloc<uint16_t>(T * (hq + 2 * hk) * d);
     q_ = dmalloc<uint16_t>(T * hq * d);
     attn_ = dmalloc<uint16_t>(T * hq * d);
     gu_ = dmalloc<uint16_t>(T * 2 * I);
-    if (model.is_moe()) {
+    if (model_.is_moe()) {
         // one row per route (token, k): expert activations and per-route outputs, the router
         // logits, and the grouped layout the routing kernel builds
         const size_t R = T * m.top_k;
@@ -251,11 +271,9 @@ Executor::Executor(const DriverConfig& cfg, Model& model) : cfg_(cfg), model_(mo
         act_ = dmalloc<uint16_t>(T * I);
     }
     rope_tab_ = dmalloc<float>(T * d);
-    const size_t srows = std::min<size_t>(T, 2 * static_cast<size_t>(cfg.batching.max_forward_requests));
+    const size_t srows = std::min<size_t>(T, 2 * static_cast<size_t>(cfg_.batching.max_forward_requests));
     xs_ = dmalloc<uint16_t>(srows * H);
     logits_ = dmalloc<uint16_t>(srows * m.vocab);
-    out_tokens_ = dmalloc<uint32_t>(T);
-    out_cap_ = T;
     amax_ws_bytes_ = pie_hip_lm_head_argmax_workspace_bytes(4, m.vocab);
     if (amax_ws_bytes_) PIE_HIP_CHECK(hipMalloc(&amax_ws_, amax_ws_bytes_));
     // Bound of the split-K partial buffers over every (rows, context) the planner can pick:
@@ -271,8 +289,8 @@ Executor::Executor(const DriverConfig& cfg, Model& model) : cfg_(cfg), model_(mo
         PIE_HIP_CHECK(hipMemcpy(iota_slots_, iota.data(), T * sizeof(int64_t), hipMemcpyHostToDevice));
     }
     // fp32 partials of the split-K GEMM for decode batches of up to 128 rows (dense layers)
-    if (!model.layers.empty()) {
-        const LayerWeights& l0 = model.layers[0];
+    if (!model_.layers.empty()) {
+        const LayerWeights& l0 = model_.layers[0];
         for (const Linear* w : {&l0.wqkv, &l0.wo, &l0.wgu, &l0.wdown})
             for (int rows : {64, 128})
                 if (w->data && w->K % 64 == 0)
@@ -280,20 +298,15 @@ Executor::Executor(const DriverConfig& cfg, Model& model) : cfg_(cfg), model_(mo
         gemm_ws_bytes_ = std::min<size_t>(gemm_ws_bytes_, size_t(64) << 20);
         if (gemm_ws_bytes_) PIE_HIP_CHECK(hipMalloc(&gemm_ws_, gemm_ws_bytes_));
     }
-
-    in_ = input_layout(max_tokens_, max_tokens_);
-    in_.total = align_up(in_.off_pages + static_cast<size_t>(max_page_refs_) * 4, 256);
-    PIE_HIP_CHECK(hipHostMalloc(reinterpret_cast<void**>(&in_host_), in_.total, hipHostMallocDefault));
-    PIE_HIP_CHECK(hipMalloc(reinterpret_cast<void**>(&in_dev_), in_.total));
-    PIE_HIP_CHECK(hipHostMalloc(reinterpret_cast<void**>(&out_host_), T * 4, hipHostMallocDefault));
-    tune_linears();
 }
 
 Executor::~Executor() {
     if (stream_) (void)hipStreamSynchronize(stream_);
     for (auto& kv : graphs_) (void)hipGraphExecDestroy(kv.second);
-    for (auto* p : k_pool_) (void)hipFree(p);
-    for (auto* p : v_pool_) (void)hipFree(p);
+    for (const PagePool& p : page_pools_) (void)hipFree(p.base);
+    for (void* p : stack_.allocs) (void)hipFree(p);
+    if (rs_base_) (void)hipFree(rs_base_);
+    if (rs_host_) (void)hipHostFree(rs_host_);
     for (void* p : {static_cast<void*>(x_), static_cast<void*>(xn_), static_cast<void*>(qkv_),
                     static_cast<void*>(q_), static_cast<void*>(attn_), static_cast<void*>(gu_),
                     static_cast<void*>(act_), static_cast<void*>(xs_), static_cast<void*>(logits_),
@@ -305,8 +318,6 @@ Executor::~Executor() {
                     static_cast<void*>(moe_route_pos_), static_cast<void*>(k_rows_),
                     static_cast<void*>(v_rows_), static_cast<void*>(iota_slots_)})
         if (p) (void)hipFree(p);
-    for (auto* p : k_scale_pool_) (void)hipFree(p);
-    for (auto* p : v_scale_pool_) (void)hipFree(p);
     if (kv_shadow_k_) (void)hipFree(kv_shadow_k_);
     if (kv_shadow_v_) (void)hipFree(kv_shadow_v_);
     for (Growable* g : {&mask_in_host_, &mask_in_dev_, &mask_bitmap_, &tile_in_host_, &tile_in_dev_}) g->release();
@@ -442,68 +453,82 @@ void Executor::tune_linears() {
     PIE_HIP_CHECK(hipStreamSynchronize(s));
 }
 
-// Allocate the pool; on out-of-memory halve the page count down to 64 pages
+// Allocate the pools; on out-of-memory halve the page count down to 64 pages
 // (driver/portable/src/entry.cpp:327-348).
 void Executor::alloc_kv() {
-    const int L = model_.cfg().layers;
-    for (;;) {
-        const size_t bytes = page_bytes() * static_cast<size_t>(total_pages_);
-        const size_t sbytes = scale_page_bytes() * static_cast<size_t>(total_pages_);
-        bool ok = true;
-        for (int l = 0; l < L && ok; ++l) {
-            void *k = nullptr, *v = nullptr;
-            if (hipMalloc(&k, bytes) != hipSuccess) { ok = false; break; }
-            k_pool_.push_back(static_cast<uint16_t*>(k));
-            if (hipMalloc(&v, bytes) != hipSuccess) { ok = false; break; }
-            v_pool_.push_back(static_cast<uint16_t*>(v));
-            if (sbytes) {
-                if (hipMalloc(&k, sbytes) != hipSuccess) { ok = false; break; }
-                k_scale_pool_.push_back(static_cast<float*>(k));
-                if (hipMalloc(&v, sbytes) != hipSuccess) { ok = false; break; }
-                v_scale_pool_.push_back(static_cast<float*>(v));
-            }
-        }
-        if (ok && kv_format_ == PIE_HIP_KV_FP4_BLOCK) {
-            // the bf16 pages the attention kernels read (k_bf16_pages / v_bf16_pages of the
-            // reference's layer view, driver/cuda/src/kernels/kv_paged.cu:698-770)
-            const ModelConfig& m = model_.cfg();
-            const size_t shadow = static_cast<size_t>(total_pages_) * page_size_ * m.kv_heads * m.head_dim * 2;
-            void *k = nullptr, *v = nullptr;
-            if (hipMalloc(&k, shadow) != hipSuccess || hipMalloc(&v, shadow) != hipSuccess) {
-                if (k) (void)hipFree(k);
-                ok = false;
-            } else {
-                kv_shadow_k_ = static_cast<uint16_t*>(k);
-                kv_shadow_v_ = static_cast<uint16_t*>(v);
-                PIE_HIP_CHECK(hipMemsetAsync(kv_shadow_k_, 0, shadow, stream_));
-                PIE_HIP_CHECK(hipMemsetAsync(kv_shadow_v_, 0, shadow, stream_));
-            }
-        }
-        if (ok) {
-            // Pages start zeroed so slots no request has written hold finite values.
-            for (int l = 0; l < L; ++l) {
-                PIE_HIP_CHECK(hipMemsetAsync(k_pool_[l], 0, bytes, stream_));
-                PIE_HIP_CHECK(hipMemsetAsync(v_pool_[l], 0, bytes, stream_));
-                if (sbytes) {
-                    PIE_HIP_CHECK(hipMemsetAsync(k_scale_pool_[l], 0, sbytes, stream_));
-                    PIE_HIP_CHECK(hipMemsetAsync(v_scale_pool_[l], 0, sbytes, stream_));
-                }
-            }
-            PIE_HIP_CHECK(hipStreamSynchronize(stream_));
-            return;
-        }
+    while (!alloc_pools()) {
         (void)hipGetLastError();
-        for (auto* p : k_pool_) (void)hipFree(p);
-        for (auto* p : v_pool_) (void)hipFree(p);
-        for (auto* p : k_scale_pool_) (void)hipFree(p);
-        for (auto* p : v_scale_pool_) (void)hipFree(p);
+        if (total_pages_ <= 64) throw std::runtime_error("executor: cannot allocate the KV pool");
+        total_pages_ = std::max(64, total_pages_ / 2);
+    }
+    size_t off = 0;
+    for (PagePool& p : page_pools_) {
+        p.host_off = off;
+        off += p.page_bytes;
+        // Pages start zeroed so slots no request has written hold finite values.
+        PIE_HIP_CHECK(hipMemsetAsync(p.base, 0, p.page_bytes * static_cast<size_t>(total_pages_), stream_));
+    }
+    swap_page_bytes_ = off;
+    PIE_HIP_CHECK(hipStreamSynchronize(stream_));
+}
+
+bool Executor::alloc_pools() {
+    const ModelConfig& m = model_.cfg();
+    auto pool = [&](size_t bytes_per_page) -> unsigned char* {
+        void* p = nullptr;
+        if (hipMalloc(&p, bytes_per_page * static_cast<size_t>(total_pages_)) != hipSuccess) return nullptr;
+        page_pools_.push_back({static_cast<unsigned char*>(p), bytes_per_page, 0});
+        return static_cast<unsigned char*>(p);
+    };
+    auto give_up = [&] {
+        for (const PagePool& p : page_pools_) (void)hipFree(p.base);
+        page_pools_.clear();
         k_pool_.clear();
         v_pool_.clear();
         k_scale_pool_.clear();
         v_scale_pool_.clear();
-        if (total_pages_ <= 64) throw std::runtime_error("executor: cannot allocate the KV pool");
-        total_pages_ = std::max(64, total_pages_ / 2);
+        latent_pool_.clear();
+        return false;
+    };
+    if (m.is_stack()) {
+        for (const LayerSpec& l : m.stack) {
+            latent_pool_.push_back(nullptr);
+            if (l.mixer != MixerKind::LatentAttention) continue;
+            const size_t esize = m.f32() ? 4 : 2;
+            latent_pool_.back() = pool(static_cast<size_t>(page_size_) * LatentShape(l.latent).ld_row * esize);
+            if (!latent_pool_.back()) return give_up();
+        }
+        return true;
     }
+    for (int l = 0; l < m.layers; ++l) {
+        unsigned char* k = pool(page_bytes());
+        unsigned char* v = k ? pool(page_bytes()) : nullptr;
+        if (!v) return give_up();
+        k_pool_.push_back(reinterpret_cast<uint16_t*>(k));
+        v_pool_.push_back(reinterpret_cast<uint16_t*>(v));
+        if (scale_page_bytes()) {
+            k = pool(scale_page_bytes());
+            v = k ? pool(scale_page_bytes()) : nullptr;
+            if (!v) return give_up();
+            k_scale_pool_.push_back(reinterpret_cast<float*>(k));
+            v_scale_pool_.push_back(reinterpret_cast<float*>(v));
+        }
+    }
+    if (kv_format_ == PIE_HIP_KV_FP4_BLOCK) {
+        // the bf16 pages the attention kernels read (k_bf16_pages / v_bf16_pages of the
+        // reference's layer view, driver/cuda/src/kernels/kv_paged.cu:698-770)
+        const size_t shadow = static_cast<size_t>(total_pages_) * page_size_ * m.kv_heads * m.head_dim * 2;
+        void *k = nullptr, *v = nullptr;
+        if (hipMalloc(&k, shadow) != hipSuccess || hipMalloc(&v, shadow) != hipSuccess) {
+            if (k) (void)hipFree(k);
+            return give_up();
+        }
+        kv_shadow_k_ = static_cast<uint16_t*>(k);
+        kv_shadow_v_ = static_cast<uint16_t*>(v);
+        PIE_HIP_CHECK(hipMemsetAsync(kv_shadow_k_, 0, shadow, stream_));
+        PIE_HIP_CHECK(hipMemsetAsync(kv_shadow_v_, 0, shadow, stream_));
+    }
+    return true;
 }
 
 // x += sum_k w_k * down_e(swiglu(gate_up_e(norm(x)))) over each token's top-k experts
@@ -559,6 +584,7 @@ void Executor::moe_block(const LayerWeights& w, int N, const uint16_t* next_norm
 }
 
 void Executor::body(int N, int S, int max_kv_len) {
+    if (model_.cfg().is_stack()) return stack_body(N, S, max_kv_len);
     xn_holds_next_norm_ = false;
     const Inputs in_ = input_layout(N, S);
     const ModelConfig& m = model_.cfg();
@@ -983,9 +1009,12 @@ void Executor::enqueue_samplers() {
     auto* od = static_cast<unsigned char*>(samp_out_dev_.ptr);
     float* f32 = static_cast<float*>(samp_f32_.ptr);
     if (!samp_gather_in_body_) {
-        PIE_KERNEL(pie_hip_sample_gather_logits(
-            logits_, nullptr, f32, samp_.n_bounds ? reinterpret_cast<const uint32_t*>(in + samp_.bounds) : nullptr,
-            samp_.n_bounds ? reinterpret_cast<const int32_t*>(in + samp_.bounds_indptr) : nullptr, S, V, stream_));
+        const auto* bounds = samp_.n_bounds ? reinterpret_cast<const uint32_t*>(in + samp_.bounds) : nullptr;
+        const auto* indptr = samp_.n_bounds ? reinterpret_cast<const int32_t*>(in + samp_.bounds_indptr) : nullptr;
+        if (stack_.logits)
+            PIE_KERNEL(pie_hip_sample_gather_logits_f32(stack_.logits, nullptr, f32, bounds, indptr, S, V, stream_));
+        else
+            PIE_KERNEL(pie_hip_sample_gather_logits(logits_, nullptr, f32, bounds, indptr, S, V, stream_));
     }
     PIE_HIP_CHECK(hipMemsetAsync(od, 0, samp_.o_total, stream_));   // eager stage, never captured
     PIE_KERNEL(pie_hip_sample(
@@ -1062,6 +1091,7 @@ void Executor::forward(const BatchPlan& plan, std::vector<uint32_t>& tokens_out,
     std::memcpy(in_host_ + in.off_row_len, plan.row_kv_len.data(), static_cast<size_t>(N) * 4);
     if (S) std::memcpy(in_host_ + in.off_sample_rows, plan.sample_rows.data(), static_cast<size_t>(S) * 4);
     std::memcpy(in_host_ + in.off_pages, plan.page_indices.data(), plan.page_indices.size() * 4);
+    if (model_.cfg().is_stack()) prepare_stack(plan, in);
     PIE_HIP_CHECK(hipMemcpyAsync(in_dev_, in_host_, used, hipMemcpyHostToDevice, stream_));
     // a sliding window (driver/portable/src/plan.cpp:60-70: keys below p - W + 1 are hidden)
     // matters once some context is longer than the window; such batches take the masked kernels
@@ -1135,53 +1165,29 @@ void Executor::forward(const BatchPlan& plan, std::vector<uint32_t>& tokens_out,
         tokens_out = samples->tokens;
     }
     const int cap = static_cast<int>(std::min<size_t>(max_tokens_, 2 * static_cast<size_t>(cfg_.batching.max_forward_requests)));
+    if (model_.cfg().is_stack()) commit_stack(plan);
     last_logit_rows_ = S == 0 ? 0 : ((S - 1) % cap) + 1;
 }
 
-// A swap-pool slot holds a page's K (or V) bytes followed by its fp32 scales (scaled formats).
 void Executor::copy_pages_d2h(const uint32_t* dev_srcs, const uint32_t* host_dsts, size_t n) {
-    const size_t pb = page_bytes(), sb = scale_page_bytes();
     for (size_t i = 0; i < n; ++i)
-        for (size_t l = 0; l < k_pool_.size(); ++l)
-            for (int kv = 0; kv < 2; ++kv) {
-                unsigned char* dst = swap_slot(static_cast<int>(l), kv, host_dsts[i]);
-                const auto* pool = reinterpret_cast<const unsigned char*>(kv ? v_pool_[l] : k_pool_[l]);
-                PIE_HIP_CHECK(hipMemcpyAsync(dst, pool + static_cast<size_t>(dev_srcs[i]) * pb, pb,
-                                             hipMemcpyDeviceToHost, stream_));
-                if (sb) {
-                    const auto* sc = reinterpret_cast<const unsigned char*>(kv ? v_scale_pool_[l] : k_scale_pool_[l]);
-                    PIE_HIP_CHECK(hipMemcpyAsync(dst + pb, sc + static_cast<size_t>(dev_srcs[i]) * sb, sb,
-                                                 hipMemcpyDeviceToHost, stream_));
-                }
-            }
+        for (const PagePool& p : page_pools_)
+            PIE_HIP_CHECK(hipMemcpyAsync(swap_slot(p, host_dsts[i]), p.base + dev_srcs[i] * p.page_bytes, p.page_bytes,
+                                         hipMemcpyDeviceToHost, stream_));
     PIE_HIP_CHECK(hipStreamSynchronize(stream_));
 }
 
 void Executor::copy_pages_h2d(const uint32_t* host_srcs, const uint32_t* dev_dsts, size_t n) {
-    const size_t pb = page_bytes(), sb = scale_page_bytes();
     for (size_t i = 0; i < n; ++i)
-        for (size_t l = 0; l < k_pool_.size(); ++l)
-            for (int kv = 0; kv < 2; ++kv) {
-                const unsigned char* src = swap_slot(static_cast<int>(l), kv, host_srcs[i]);
-                auto* pool = reinterpret_cast<unsigned char*>(kv ? v_pool_[l] : k_pool_[l]);
-                PIE_HIP_CHECK(hipMemcpyAsync(pool + static_cast<size_t>(dev_dsts[i]) * pb, src, pb,
-                                             hipMemcpyHostToDevice, stream_));
-                if (sb) {
-                    auto* sc = reinterpret_cast<unsigned char*>(kv ? v_scale_pool_[l] : k_scale_pool_[l]);
-                    PIE_HIP_CHECK(hipMemcpyAsync(sc + static_cast<size_t>(dev_dsts[i]) * sb, src + pb, sb,
-                                                 hipMemcpyHostToDevice, stream_));
-                }
-            }
+        for (const PagePool& p : page_pools_)
+            PIE_HIP_CHECK(hipMemcpyAsync(p.base + dev_dsts[i] * p.page_bytes, swap_slot(p, host_srcs[i]), p.page_bytes,
+                                         hipMemcpyHostToDevice, stream_));
     PIE_HIP_CHECK(hipStreamSynchronize(stream_));
 }
 
 void Executor::copy_pages_h2h(const uint32_t* srcs, const uint32_t* dsts, size_t n) {
-    const size_t pb = page_bytes() + scale_page_bytes();
     for (size_t i = 0; i < n; ++i)
-        for (size_t l = 0; l < k_pool_.size(); ++l)
-            for (int kv = 0; kv < 2; ++kv)
-                std::memmove(swap_slot(static_cast<int>(l), kv, dsts[i]),
-                             swap_slot(static_cast<int>(l), kv, srcs[i]), pb);
+        for (const PagePool& p : page_pools_) std::memmove(swap_slot(p, dsts[i]), swap_slot(p, srcs[i]), p.page_bytes);
 }
 
 void Executor::copy_pages_d2d(const uint32_t* srcs, const uint32_t* dsts, size_t n) {
@@ -1195,18 +1201,9 @@ void Executor::copy_pages_d2d(const uint32_t* srcs, const uint32_t* dsts, size_t
     PIE_HIP_CHECK(hipMemcpyAsync(copy_ids_ + copy_ids_cap_, dsts, n * 4, hipMemcpyHostToDevice, stream_));
     for (size_t i = 0; i < n; i += 65535) {
         const int cnt = static_cast<int>(std::min<size_t>(65535, n - i));
-        for (size_t l = 0; l < k_pool_.size(); ++l) {
-            PIE_KERNEL(pie_hip_copy_kv_pages(k_pool_[l], copy_ids_ + i, copy_ids_ + copy_ids_cap_ + i,
-                                             cnt, page_bytes(), stream_));
-            PIE_KERNEL(pie_hip_copy_kv_pages(v_pool_[l], copy_ids_ + i, copy_ids_ + copy_ids_cap_ + i,
-                                             cnt, page_bytes(), stream_));
-            if (scale_page_bytes()) {
-                PIE_KERNEL(pie_hip_copy_kv_pages(k_scale_pool_[l], copy_ids_ + i, copy_ids_ + copy_ids_cap_ + i,
-                                                 cnt, scale_page_bytes(), stream_));
-                PIE_KERNEL(pie_hip_copy_kv_pages(v_scale_pool_[l], copy_ids_ + i, copy_ids_ + copy_ids_cap_ + i,
-                                                 cnt, scale_page_bytes(), stream_));
-            }
-        }
+        for (const PagePool& p : page_pools_)
+            PIE_KERNEL(pie_hip_copy_kv_pages(p.base, copy_ids_ + i, copy_ids_ + copy_ids_cap_ + i, cnt, p.page_bytes,
+                                             stream_));
     }
     PIE_HIP_CHECK(hipStreamSynchronize(stream_));
 }

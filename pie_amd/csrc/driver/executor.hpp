@@ -13,6 +13,13 @@
 //   gu   = xn · Wgu^T ; h = silu(gate) * up ; x = x + h · Wdown^T
 // tail: gather sampled rows -> final norm -> lm_head -> argmax (first index wins).
 //
+// Layer stacks (ModelConfig::stack; executor_stack.hip) keep an fp32 residual stream and run, per
+// layer, mixer -> norm-and-add -> feed-forward -> norm-and-add:
+//   latent attention  in-projection, norms + rotation + cache write, query up-projection, attention
+//                     over the latent pool, out-projection
+//   channel delta     in-projection, convolution + unit vectors, decay and gate projections, the
+//                     recurrence over the request's state slot, norm + gate, out-projection
+//
 // Split into a host `prepare` (plan upload, outside any capture) and a device-only `body`
 // that is captured into a HIP graph per (rows, sampled rows, context bucket) for pure decode,
 // the prepare/body split of driver/cuda/src/executor/executor.hpp:42-75.
@@ -27,6 +34,7 @@
 
 #include "config.hpp"
 #include "model.hpp"
+#include "pie_hip_kernels.h"
 #include "planner.hpp"
 
 namespace pie_hip_driver {
@@ -46,6 +54,11 @@ struct SampleOutputs {
     std::vector<int32_t> out_indptr;
     std::vector<float> raw_logits;
 };
+
+// y = epilogue(rmsnorm?(act) . W^T) through the bf16 / quantised kernels (executor.hip).
+bool linear_fused(const Linear& w, const uint16_t* act, const uint16_t* norm_w, float eps,
+                  uint16_t* y, int M, int beta, int epilogue, uint16_t* norm_tmp, void* gemm_ws,
+                  size_t gemm_ws_bytes, hipStream_t s, int force = -1);
 
 class Executor {
   public:
@@ -69,6 +82,14 @@ class Executor {
     void copy_pages_h2d(const uint32_t* host_srcs, const uint32_t* dev_dsts, size_t n);
     void copy_pages_h2h(const uint32_t* srcs, const uint32_t* dsts, size_t n);
     int cpu_pages() const { return cpu_pages_; }
+    // Recurrent-state slots of layer stacks: whole-slot copies, same four directions.
+    void copy_rs_d2d(const uint32_t* srcs, const uint32_t* dsts, size_t n);
+    void copy_rs_d2h(const uint32_t* dev_srcs, const uint32_t* host_dsts, size_t n);
+    void copy_rs_h2d(const uint32_t* host_srcs, const uint32_t* dev_dsts, size_t n);
+    void copy_rs_h2h(const uint32_t* srcs, const uint32_t* dsts, size_t n);
+    int rs_slots() const { return rs_slots_; }
+    int cpu_rs_slots() const { return cpu_rs_slots_; }
+    size_t rs_slot_bytes() const { return rs_stride_; }
 
     int total_pages() const { return total_pages_; }
     int page_size() const { return page_size_; }
@@ -88,6 +109,8 @@ class Executor {
         if (what == "act") return act_;
         return nullptr;
     }
+    // fp32 logits [rows, vocab] of the same rows (layer stacks; null otherwise)
+    const float* last_logits_f32() const { return stack_.logits; }
     int last_logit_rows() const { return last_logit_rows_; }
     const uint16_t* kv_pool(bool k, int layer) const {
         if (layer < 0 || layer >= static_cast<int>(k_pool_.size())) return nullptr;
@@ -95,6 +118,13 @@ class Executor {
     }
 
   private:
+    // staged inputs: one pinned host block mirrored by one device block.  Layer stacks add the
+    // rows' requests and the requests' row ranges and state slots.
+    struct Inputs {
+        size_t off_tokens, off_positions, off_slots, off_row_begin, off_row_len, off_sample_rows,
+            off_row_req, off_qo, off_rs_slot, off_rs_fresh, off_pages, total;
+    };
+    Inputs input_layout(int N, int S) const;
     void body(int N, int S, int max_kv_len);
     void grow_outputs(size_t slots);
     void prepare_masks(const BatchPlan& plan);
@@ -107,6 +137,15 @@ class Executor {
     static constexpr size_t kMergeProjMaxBytes = 64 * 1024;   // partial results a merging output projection reads per block
     bool xn_holds_next_norm_ = false;             // (while a forward is being enqueued) xn_ = the coming layer's normalised rows
     void alloc_kv();
+    bool alloc_pools();   // every page pool at total_pages_ pages; false (and nothing kept) when memory runs out
+    void alloc_uniform();
+    void alloc_stack();
+    void prepare_stack(const BatchPlan& plan, const Inputs& in);   // host half: checks, state slots, row ranges
+    void commit_stack(const BatchPlan& plan);                      // after success: the slots' new positions
+    void stack_body(int N, int S, int max_kv_len);
+    void stack_latent(const StackLayer& w, int layer, int N, int max_kv_len, const Inputs& in);
+    void stack_delta(const StackLayer& w, int layer, int N, const Inputs& in);
+    void stack_linear(const Linear& w, const void* act, void* y, int M, int epilogue = PIE_HIP_EPI_NONE);
     void tune_linears();
 
     DriverConfig cfg_;
@@ -123,11 +162,19 @@ class Executor {
     int n_page_refs_ = 0;                      // page list entries of the forward in flight
     uint16_t *k_rows_ = nullptr, *v_rows_ = nullptr;     // this step's rotated K / V rows before quantisation
     int64_t* iota_slots_ = nullptr;                      // 0, 1, 2, ...: row t of k_rows_ is "slot" t
-    unsigned char* swap_pool_ = nullptr;       // pinned: [layer][K|V][cpu_pages] pages (+ their scales)
+    // every paged allocation in copy order (K and V pools and their scales, or latent pools); page
+    // copies walk this list.  host_off: bytes per page of the pools before it, so that pool p's
+    // swap region starts at host_off * cpu_pages.
+    struct PagePool {
+        unsigned char* base;
+        size_t page_bytes, host_off;
+    };
+    std::vector<PagePool> page_pools_;
+    size_t swap_page_bytes_ = 0;               // all pools' bytes of one page
+    unsigned char* swap_pool_ = nullptr;       // pinned
     int cpu_pages_ = 0;
-    unsigned char* swap_slot(int layer, int kv, uint32_t slot) const {
-        return swap_pool_ + ((static_cast<size_t>(layer) * 2 + kv) * cpu_pages_ + slot) *
-                                (page_bytes() + scale_page_bytes());
+    unsigned char* swap_slot(const PagePool& p, uint32_t slot) const {
+        return swap_pool_ + p.host_off * cpu_pages_ + slot * p.page_bytes;
     }
     // activations
     uint16_t *x_ = nullptr, *xn_ = nullptr, *qkv_ = nullptr, *q_ = nullptr, *attn_ = nullptr;
@@ -149,12 +196,6 @@ class Executor {
     uint32_t* copy_ids_ = nullptr;  // staging for page-copy id lists
     size_t copy_ids_cap_ = 0;
 
-    // staged inputs: one pinned host block mirrored by one device block
-    struct Inputs {
-        size_t off_tokens, off_positions, off_slots, off_row_begin, off_row_len, off_sample_rows,
-            off_pages, total;
-    };
-    static Inputs input_layout(int N, int S);
     Inputs in_{};  // layout at capacity: sizes the staging buffers
     unsigned char* in_host_ = nullptr;
     unsigned char* in_dev_ = nullptr;
@@ -185,6 +226,27 @@ class Executor {
     } samp_{};
     bool samp_gather_in_body_ = false;
     uint64_t unseeded_draws_ = 0;
+
+    // ---- layer stacks ----
+    struct StackBuffers {
+        float *x = nullptr, *logits = nullptr;   // residual stream, finished logits
+        // compute type
+        void *xa = nullptr, *in = nullptr, *y = nullptr, *cq = nullptr, *q = nullptr, *q_lat = nullptr, *o_lat = nullptr,
+             *o = nullptr, *act = nullptr, *a1 = nullptr, *g1 = nullptr, *decay = nullptr, *gate = nullptr,
+             *xs = nullptr, *raw_logits = nullptr;
+        float *dq = nullptr, *dk = nullptr, *dv = nullptr, *dg = nullptr, *d_beta = nullptr, *d_o = nullptr;
+        std::vector<float*> rotary;              // tables of the step, one per distinct rotation
+        std::vector<void*> allocs;
+    } stack_;
+    int dt_ = PIE_HIP_DT_BF16;
+    const BatchPlan* plan_ = nullptr;            // (while a forward is being enqueued)
+    int n_requests_ = 0;
+    std::vector<unsigned char*> latent_pool_;    // per layer (null: no latent cache)
+    unsigned char *rs_base_ = nullptr, *rs_host_ = nullptr;
+    int rs_slots_ = 0, cpu_rs_slots_ = 0;
+    size_t rs_stride_ = 0;                       // bytes per slot
+    std::vector<size_t> rs_state_off_, rs_conv_off_;   // per layer
+    std::vector<int64_t> rs_pos_, rs_host_pos_;  // tokens a slot's state has seen (-1: nothing)
 
     std::map<std::tuple<int, int, int, int>, hipGraphExec_t> graphs_;   // (rows, sampling slots, context bucket, rows equally long)
     bool uniform_rows_ = false;   // this step's rows are about equally long (decode batches)

@@ -1,0 +1,312 @@
+// Layer stacks in the executor: workspaces, recurrent-state slots, and the forward body of models
+// whose layers are listed one by one (ModelConfig::stack).
+#include <algorithm>
+#include <cstring>
+#include <set>
+#include <stdexcept>
+#include <string>
+
+#include "executor.hpp"
+#include "pie_hip_kernels.h"
+
+namespace pie_hip_driver {
+
+#define PIE_HIP_CHECK(expr)                                                              \
+    do {                                                                                 \
+        hipError_t e_ = (expr);                                                          \
+        if (e_ != hipSuccess)                                                            \
+            throw std::runtime_error(std::string(#expr) + ": " + hipGetErrorString(e_)); \
+    } while (0)
+
+#define PIE_KERNEL(expr)                                                                     \
+    do {                                                                                     \
+        const int st_ = (expr);                                                              \
+        if (st_ != PIE_HIP_OK)                                                               \
+            throw std::runtime_error(std::string(#expr) + " failed with status " +          \
+                                     std::to_string(st_));                                   \
+    } while (0)
+
+// Workspaces at their largest over the layers, and the recurrent-state pool.
+void Executor::alloc_stack() {
+    const ModelConfig& m = model_.cfg();
+    const size_t T = static_cast<size_t>(max_tokens_), esize = m.f32() ? 4 : 2;
+    const size_t ld_x = static_cast<size_t>(model_.ld_x());
+    size_t in = 0, cq = 0, q = 0, q_lat = 0, o_lat = 0, o = 0, act = 0, a1 = 0, g1 = 0, decay = 0, gate = 0;
+    size_t kd = 0, vd = 0, gd = 0, heads = 0, state = 0;
+    auto up = [](size_t& v, int n) { v = std::max(v, static_cast<size_t>(n)); };
+    for (const StackLayer& l : model_.stack) {
+        rs_state_off_.push_back(0);
+        rs_conv_off_.push_back(0);
+        up(act, l.spec.ff > 0 ? pad_to(l.spec.ff, 128) : 0);
+        if (l.spec.mixer == MixerKind::LatentAttention) {
+            const LatentShape s(l.spec.latent);
+            up(in, s.ld_in);
+            up(cq, s.ld_cq);
+            up(q, s.ld_q);
+            up(q_lat, s.heads * s.ld_row);
+            up(o_lat, s.heads * s.kvp);
+            up(o, s.ld_o);
+        } else {
+            const ChannelDeltaSpec& d = l.spec.delta;
+            const DeltaShape s(d);
+            up(in, s.ld_in);
+            up(o, s.ld_o);
+            up(a1, s.ld_a1);
+            up(g1, s.ld_g1);
+            up(decay, s.ld_decay);
+            up(gate, s.ld_gate);
+            up(kd, s.kd);
+            up(vd, s.vd);
+            up(gd, d.heads * d.dim);
+            up(heads, d.heads);
+            auto place = [&](size_t bytes) {
+                const size_t at = state;
+                state = (state + bytes + 255) / 256 * 256;
+                return at;
+            };
+            rs_state_off_.back() = place(static_cast<size_t>(d.heads) * d.dim * d.vdim * 4);
+            rs_conv_off_.back() = place(static_cast<size_t>(d.taps - 1) * s.channels * esize);
+        }
+    }
+    // Zeroed: columns that pad a row to its product's K are written by nobody.
+    auto take = [&](size_t bytes) {
+        void* p = nullptr;
+        PIE_HIP_CHECK(hipMalloc(&p, std::max<size_t>(bytes, 16)));
+        stack_.allocs.push_back(p);
+        PIE_HIP_CHECK(hipMemsetAsync(p, 0, std::max<size_t>(bytes, 16), stream_));
+        return p;
+    };
+    auto f32 = [&](size_t n) { return static_cast<float*>(take(n * 4)); };
+    auto compute = [&](size_t n) { return take(n * esize); };
+    stack_.x = f32(T * ld_x);
+    stack_.xa = compute(T * ld_x);
+    stack_.in = compute(T * in);
+    stack_.y = compute(T * ld_x);
+    stack_.cq = compute(T * cq);
+    stack_.q = compute(T * q);
+    stack_.q_lat = compute(T * q_lat);
+    stack_.o_lat = compute(T * o_lat);
+    stack_.o = compute(T * o);
+    stack_.act = compute(T * act);
+    stack_.a1 = compute(T * a1);
+    stack_.g1 = compute(T * g1);
+    stack_.decay = compute(T * decay);
+    stack_.gate = compute(T * gate);
+    stack_.dq = f32(T * kd);
+    stack_.dk = f32(T * kd);
+    stack_.dv = f32(T * vd);
+    stack_.dg = f32(T * gd);
+    stack_.d_beta = f32(T * heads);
+    stack_.d_o = f32(T * vd);
+    const size_t srows = std::min<size_t>(T, 2 * static_cast<size_t>(cfg_.batching.max_forward_requests));
+    stack_.xs = compute(srows * ld_x);
+    stack_.raw_logits = compute(srows * static_cast<size_t>(model_.head.N));
+    stack_.logits = f32(srows * static_cast<size_t>(m.vocab));
+    for (const RotaryTable& r : model_.rotary) stack_.rotary.push_back(f32(T * static_cast<size_t>(r.spec.dims)));
+    for (StackLayer& l : model_.stack)
+        for (const Linear* w : {&l.w_in, &l.w_uq, &l.w_decay, &l.w_gate, &l.wo, &l.w_up, &l.w_down})
+            for (int rows : {64, 128})
+                if (!m.f32() && w->data && w->K % 64 == 0)
+                    gemm_ws_bytes_ = std::max(gemm_ws_bytes_, pie_hip_gemm_mfma_workspace_bytes(rows, w->N, w->K));
+    gemm_ws_bytes_ = std::min<size_t>(gemm_ws_bytes_, size_t(64) << 20);
+    if (gemm_ws_bytes_) PIE_HIP_CHECK(hipMalloc(&gemm_ws_, gemm_ws_bytes_));
+    rs_stride_ = state;
+    if (state) {
+        rs_slots_ = cfg_.batching.rs_cache_slots;
+        cpu_rs_slots_ = cfg_.batching.cpu_rs_slots;
+        void* p = nullptr;
+        PIE_HIP_CHECK(hipMalloc(&p, state * static_cast<size_t>(rs_slots_)));
+        rs_base_ = static_cast<unsigned char*>(p);
+        PIE_HIP_CHECK(hipMemsetAsync(rs_base_, 0, state * static_cast<size_t>(rs_slots_), stream_));
+        if (cpu_rs_slots_ > 0) {
+            PIE_HIP_CHECK(hipHostMalloc(&p, state * static_cast<size_t>(cpu_rs_slots_), hipHostMallocDefault));
+            rs_host_ = static_cast<unsigned char*>(p);
+            std::memset(rs_host_, 0, state * static_cast<size_t>(cpu_rs_slots_));
+        }
+        rs_pos_.assign(static_cast<size_t>(rs_slots_), -1);
+        rs_host_pos_.assign(static_cast<size_t>(cpu_rs_slots_), -1);
+    }
+    PIE_HIP_CHECK(hipStreamSynchronize(stream_));
+}
+
+// Whole slots move, with the number of tokens their state has seen.
+void Executor::copy_rs_d2d(const uint32_t* srcs, const uint32_t* dsts, size_t n) {
+    for (size_t i = 0; i < n; ++i) {
+        if (srcs[i] == dsts[i]) continue;
+        PIE_HIP_CHECK(hipMemcpyAsync(rs_base_ + dsts[i] * rs_stride_, rs_base_ + srcs[i] * rs_stride_, rs_stride_,
+                                     hipMemcpyDeviceToDevice, stream_));
+        rs_pos_[dsts[i]] = rs_pos_[srcs[i]];
+    }
+    PIE_HIP_CHECK(hipStreamSynchronize(stream_));
+}
+void Executor::copy_rs_d2h(const uint32_t* srcs, const uint32_t* dsts, size_t n) {
+    for (size_t i = 0; i < n; ++i) {
+        PIE_HIP_CHECK(hipMemcpyAsync(rs_host_ + dsts[i] * rs_stride_, rs_base_ + srcs[i] * rs_stride_, rs_stride_,
+                                     hipMemcpyDeviceToHost, stream_));
+        rs_host_pos_[dsts[i]] = rs_pos_[srcs[i]];
+    }
+    PIE_HIP_CHECK(hipStreamSynchronize(stream_));
+}
+void Executor::copy_rs_h2d(const uint32_t* srcs, const uint32_t* dsts, size_t n) {
+    for (size_t i = 0; i < n; ++i) {
+        PIE_HIP_CHECK(hipMemcpyAsync(rs_base_ + dsts[i] * rs_stride_, rs_host_ + srcs[i] * rs_stride_, rs_stride_,
+                                     hipMemcpyHostToDevice, stream_));
+        rs_pos_[dsts[i]] = rs_host_pos_[srcs[i]];
+    }
+    PIE_HIP_CHECK(hipStreamSynchronize(stream_));
+}
+void Executor::copy_rs_h2h(const uint32_t* srcs, const uint32_t* dsts, size_t n) {
+    for (size_t i = 0; i < n; ++i) {
+        std::memmove(rs_host_ + dsts[i] * rs_stride_, rs_host_ + srcs[i] * rs_stride_, rs_stride_);
+        rs_host_pos_[dsts[i]] = rs_host_pos_[srcs[i]];
+    }
+}
+
+// What a stack refuses, the state slots of the batch's requests and which of them start from zero.
+void Executor::prepare_stack(const BatchPlan& plan, const Inputs& in) {
+    if (plan.has_user_masks) throw std::runtime_error("executor: layer stacks take no custom attention masks");
+    auto* row_req = reinterpret_cast<int32_t*>(in_host_ + in.off_row_req);
+    auto* qo = reinterpret_cast<int32_t*>(in_host_ + in.off_qo);
+    auto* slot = reinterpret_cast<int32_t*>(in_host_ + in.off_rs_slot);
+    auto* fresh = reinterpret_cast<int32_t*>(in_host_ + in.off_rs_fresh);
+    const bool recurrent = rs_slots_ > 0;
+    if (recurrent && static_cast<int>(plan.rs_slots.size()) != plan.R)
+        throw std::runtime_error("executor: this model needs a recurrent-state slot per request (rs_slot_ids)");
+    std::set<uint32_t> seen;
+    for (int r = 0; r < plan.R; ++r) {
+        const int q0 = plan.qo_indptr[r], q1 = plan.qo_indptr[r + 1];
+        qo[r] = q0;
+        for (int i = q0; i < q1; ++i) {
+            row_req[i] = r;
+            if (i > q0 && plan.positions[i] != plan.positions[i - 1] + 1)
+                throw std::runtime_error("executor: a request's rows must be consecutive positions");
+        }
+        slot[r] = 0;
+        fresh[r] = 1;
+        if (!recurrent) continue;
+        const uint32_t s = plan.rs_slots[r];
+        if (s >= static_cast<uint32_t>(rs_slots_)) throw std::runtime_error("executor: recurrent-state slot out of range");
+        if (!seen.insert(s).second) throw std::runtime_error("executor: two requests of a batch share a recurrent-state slot");
+        // state cannot be rolled back to a rejected draft's predecessor
+        if (!plan.draft_tokens[r].empty()) throw std::runtime_error("executor: recurrent state cannot verify drafts");
+        const bool reset = plan.positions[q0] == 0 || (!plan.rs_flags.empty() && (plan.rs_flags[r] & PIE_RS_RESET));
+        if (!reset && rs_pos_[s] != plan.positions[q0])
+            throw std::runtime_error("executor: slot " + std::to_string(s) + " holds the state after " +
+                                     std::to_string(rs_pos_[s]) + " tokens, the request goes on at position " +
+                                     std::to_string(plan.positions[q0]));
+        slot[r] = static_cast<int32_t>(s);
+        fresh[r] = reset ? 1 : 0;
+    }
+    qo[plan.R] = plan.N;
+    if (recurrent)
+        for (int r = 0; r < plan.R; ++r) rs_pos_[plan.rs_slots[r]] = -1;   // (until the pass has succeeded)
+    plan_ = &plan;
+}
+
+void Executor::commit_stack(const BatchPlan& plan) {
+    plan_ = nullptr;
+    if (rs_slots_ == 0) return;
+    for (int r = 0; r < plan.R; ++r) rs_pos_[plan.rs_slots[r]] = plan.positions[plan.qo_indptr[r + 1] - 1] + 1;
+}
+
+void Executor::stack_linear(const Linear& w, const void* act, void* y, int M, int epilogue) {
+    if (dt_ == PIE_HIP_DT_F32)
+        PIE_KERNEL(pie_hip_linear_f32(static_cast<const float*>(act), static_cast<const uint16_t*>(w.data),
+                                      static_cast<float*>(y), M, w.N, w.K, epilogue, stream_));
+    else
+        linear_fused(w, static_cast<const uint16_t*>(act), nullptr, 0.f, static_cast<uint16_t*>(y), M, 0, epilogue,
+                     nullptr, gemm_ws_, gemm_ws_bytes_, stream_);
+}
+
+void Executor::stack_latent(const StackLayer& w, int layer, int N, int max_kv_len, const Inputs& in) {
+    const LatentAttentionSpec& a = w.spec.latent;
+    const LatentShape s(a);
+    const auto* slots = reinterpret_cast<const int64_t*>(in_dev_ + in.off_slots);
+    const auto* row_begin = reinterpret_cast<const uint32_t*>(in_dev_ + in.off_row_begin);
+    const auto* row_len = reinterpret_cast<const int32_t*>(in_dev_ + in.off_row_len);
+    const auto* pages = reinterpret_cast<const uint32_t*>(in_dev_ + in.off_pages);
+    const float* rope = w.rotary >= 0 ? stack_.rotary[static_cast<size_t>(w.rotary)] : nullptr;
+    (void)max_kv_len;
+    stack_linear(w.w_in, stack_.xa, stack_.in, N);
+    PIE_KERNEL(pie_hip_latent_prep(dt_, stack_.in, w.q_norm, w.kv_norm, rope, slots, stack_.cq, latent_pool_[layer], N,
+                                   s.ld_in, s.kv_off, a.q_rank, s.ld_cq, a.kv_rank, s.kvp, a.rot_dim, a.rot.dims,
+                                   s.ld_row, model_.cfg().rms_eps, stream_));
+    stack_linear(w.w_uq, stack_.cq, stack_.q, N);
+    PIE_KERNEL(pie_hip_head_linear(dt_, stack_.q, w.w_uk_t, stack_.q_lat, s.rotp ? rope : nullptr, N, s.heads, s.kvp,
+                                   s.dimp, s.ld_q, s.hd, s.heads * s.ld_row, s.ld_row, s.dimp, a.rot_dim, a.rot.dims,
+                                   s.rotp, stream_));
+    PIE_KERNEL(pie_hip_latent_attn_rows_plain(dt_, stack_.q_lat, latent_pool_[layer], stack_.o_lat, pages, row_begin,
+                                              row_len, N, s.heads, s.kvp, s.ld_row, page_size_,
+                                              static_cast<float>(a.scale), stream_));
+    PIE_KERNEL(pie_hip_head_linear(dt_, stack_.o_lat, w.w_uv, stack_.o, nullptr, N, s.heads, s.vdp, s.kvp,
+                                   s.heads * s.kvp, s.kvp, s.ld_o, s.vdp, 0, 0, 0, 0, stream_));
+    stack_linear(w.wo, stack_.o, stack_.y, N);
+}
+
+void Executor::stack_delta(const StackLayer& w, int layer, int N, const Inputs& in) {
+    const ChannelDeltaSpec& d = w.spec.delta;
+    const DeltaShape s(d);
+    const auto* row_req = reinterpret_cast<const int32_t*>(in_dev_ + in.off_row_req);
+    const auto* qo = reinterpret_cast<const int32_t*>(in_dev_ + in.off_qo);
+    const auto* slot = reinterpret_cast<const int32_t*>(in_dev_ + in.off_rs_slot);
+    const auto* fresh = reinterpret_cast<const int32_t*>(in_dev_ + in.off_rs_fresh);
+    stack_linear(w.w_in, stack_.xa, stack_.in, N);
+    PIE_KERNEL(pie_hip_delta_prep(dt_, stack_.in, w.conv_w, rs_base_, rs_stride_, rs_conv_off_[layer], row_req, qo, slot,
+                                  fresh, stack_.dq, stack_.dk, stack_.dv, stack_.d_beta, stack_.a1, stack_.g1, N, s.ld_in,
+                                  d.heads, d.kv_heads, d.dim, d.vdim, d.taps, s.decay_off, d.decay_rank, s.ld_a1,
+                                  s.gate_off, d.gate_rank, s.ld_g1, stream_));
+    stack_linear(w.w_decay, stack_.a1, stack_.decay, N);
+    stack_linear(w.w_gate, stack_.g1, stack_.gate, N);
+    PIE_KERNEL(pie_hip_delta_decay(dt_, stack_.decay, w.a_log, w.dt_bias, stack_.dg, N, s.ld_decay, d.heads, d.dim, stream_));
+    PIE_KERNEL(pie_hip_delta_scan(stack_.dq, stack_.dk, stack_.dv, stack_.dg, stack_.d_beta, stack_.d_o, rs_base_,
+                                  rs_stride_, rs_state_off_[layer], qo, slot, fresh, n_requests_, d.heads, d.kv_heads,
+                                  d.dim, d.vdim, stream_));
+    PIE_KERNEL(pie_hip_delta_out(dt_, stack_.d_o, stack_.gate, w.out_norm, stack_.o, stack_.in, rs_base_, rs_stride_,
+                                 rs_conv_off_[layer], row_req, qo, slot, fresh, N, s.ld_gate, s.ld_o, s.ld_in, d.heads,
+                                 d.kv_heads, d.dim, d.vdim, d.taps, model_.cfg().rms_eps, stream_));
+    stack_linear(w.wo, stack_.o, stack_.y, N);
+}
+
+void Executor::stack_body(int N, int S, int max_kv_len) {
+    const Inputs in = input_layout(N, S);
+    const ModelConfig& m = model_.cfg();
+    const int H = m.hidden, ld = model_.ld_x();
+    hipStream_t s = stream_;
+    n_requests_ = plan_->R;
+    PIE_KERNEL(pie_hip_embed_stream(dt_, reinterpret_cast<const uint32_t*>(in_dev_ + in.off_tokens), model_.embed,
+                                    stack_.x, stack_.xa, N, H, ld, m.vocab, s));
+    for (size_t i = 0; i < model_.rotary.size(); ++i)
+        PIE_KERNEL(pie_hip_rotary_table(reinterpret_cast<const int32_t*>(in_dev_ + in.off_positions),
+                                        model_.rotary[i].freq, stack_.rotary[i], N, model_.rotary[i].spec.dims,
+                                        model_.rotary[i].mscale, s));
+    for (size_t l = 0; l < model_.stack.size(); ++l) {
+        const StackLayer& w = model_.stack[l];
+        if (w.spec.mixer == MixerKind::LatentAttention) stack_latent(w, static_cast<int>(l), N, max_kv_len, in);
+        else stack_delta(w, static_cast<int>(l), N, in);
+        PIE_KERNEL(pie_hip_norm_add(dt_, stack_.y, w.norm1, stack_.x, stack_.xa, N, H, w.wo.N, ld, m.rms_eps, s));
+        if (w.spec.ff > 0) {
+            stack_linear(w.w_up, stack_.xa, stack_.act, N, PIE_HIP_EPI_RELU2);
+            stack_linear(w.w_down, stack_.act, stack_.y, N);
+            PIE_KERNEL(pie_hip_norm_add(dt_, stack_.y, w.norm2, stack_.x, stack_.xa, N, H, w.w_down.N, ld, m.rms_eps, s));
+        }
+    }
+    // the output norm and the head on the sampled rows only
+    const auto* sample_rows = reinterpret_cast<const uint32_t*>(in_dev_ + in.off_sample_rows);
+    const int cap = static_cast<int>(std::min<size_t>(max_tokens_, 2 * static_cast<size_t>(cfg_.batching.max_forward_requests)));
+    for (int s0 = 0; s0 < S; s0 += cap) {
+        const int n = std::min(cap, S - s0);
+        PIE_KERNEL(pie_hip_norm_rows(dt_, stack_.x, sample_rows + s0, model_.stack_norm, stack_.xs, n, H, ld, N, m.rms_eps, s));
+        stack_linear(model_.head, stack_.xs, stack_.raw_logits, n);
+        PIE_KERNEL(pie_hip_logits_finish(dt_, stack_.raw_logits, stack_.logits, out_tokens_ + s0, n, m.vocab,
+                                         model_.head.N, m.logit_scale, m.logit_softcap, s));
+        if (samp_gather_in_body_) {   // more sampled rows than one chunk: keep each chunk's rows
+            const auto* dev = static_cast<const unsigned char*>(samp_in_dev_.ptr);
+            PIE_KERNEL(pie_hip_sample_gather_logits_f32(
+                stack_.logits, nullptr, static_cast<float*>(samp_f32_.ptr) + static_cast<size_t>(s0) * m.vocab,
+                samp_.n_bounds ? reinterpret_cast<const uint32_t*>(dev + samp_.bounds) : nullptr,
+                samp_.n_bounds ? reinterpret_cast<const int32_t*>(dev + samp_.bounds_indptr) + s0 : nullptr, n, m.vocab, s));
+        }
+    }
+}
+
+}  // namespace pie_hip_driver

@@ -40,13 +40,6 @@ __global__ void fill_normal_bf16_kernel(uint16_t* __restrict__ out, size_t n, ui
     out[i] = __builtin_bit_cast(uint16_t, b);
 }
 
-void fill_normal(uint16_t* dst, size_t n, uint64_t seed, float mean, float std,
-                 hipStream_t stream) {
-    if (n == 0) return;
-    hipLaunchKernelGGL(fill_normal_bf16_kernel, dim3(static_cast<unsigned>((n + 255) / 256)),
-                       dim3(256), 0, stream, dst, n, seed, mean, std);
-    PIE_HIP_CHECK(hipGetLastError());
-}
 
 // Inside every block of 2*half rows: dst row 2i = src row i (gate_i), dst row 2i+1 = src row
 // half + i (up_i); rows of row_bytes bytes (always even), moved two bytes at a time — a
@@ -81,6 +74,13 @@ __global__ void f32_to_bf16_kernel(const float* __restrict__ in, uint16_t* __res
 }
 
 }  // namespace
+
+void fill_normal(uint16_t* dst, size_t n, uint64_t seed, float mean, float std, hipStream_t stream) {
+    if (n == 0) return;
+    hipLaunchKernelGGL(fill_normal_bf16_kernel, dim3(static_cast<unsigned>((n + 255) / 256)),
+                       dim3(256), 0, stream, dst, n, seed, mean, std);
+    PIE_HIP_CHECK(hipGetLastError());
+}
 
 std::vector<float> rope_inv_freq(const ModelConfig& cfg) {
     const int d = cfg.head_dim, half = d / 2;
@@ -134,25 +134,30 @@ Model::~Model() {
 }
 
 void Model::build_tiled_copies(hipStream_t stream) {
+    std::vector<Linear*> linears;
     for (LayerWeights& l : layers)
-        for (Linear* w : {&l.wqkv, &l.wo, &l.wgu, &l.wdown}) {
-            if (!w->data || w->data_tiled || w->N <= 0 || w->N % 16 != 0) continue;
-            const size_t row_bytes = w->data_bytes() / static_cast<size_t>(w->N);
-            if (row_bytes % 64 != 0) continue;
-            w->data_tiled = alloc(w->data_bytes(), "");
-            const int st = w->kind == Quant::Int4b8
-                               ? pie_hip_repack_mfma_tiles_int4(w->data, w->data_tiled, w->N, row_bytes, stream)
-                               : pie_hip_repack_mfma_tiles(w->data, w->data_tiled, w->N, row_bytes, stream);
-            if (st != PIE_HIP_OK)
-                throw std::runtime_error("model: weight repack failed");
-            if (w->kind == Quant::Int4b8) {
-                w->scale_tiled = alloc(w->scale_bytes(), "");
-                if (pie_hip_repack_scale_tiles(static_cast<const uint16_t*>(w->scale),
-                                               static_cast<uint16_t*>(w->scale_tiled), w->N, w->K / w->group,
-                                               stream) != PIE_HIP_OK)
-                    throw std::runtime_error("model: scale repack failed");
-            }
+        for (Linear* w : {&l.wqkv, &l.wo, &l.wgu, &l.wdown}) linears.push_back(w);
+    if (!cfg_.f32())   // (the fp32 products read the row-major weights)
+        for (StackLayer& l : stack)
+            for (Linear* w : {&l.w_in, &l.w_uq, &l.w_decay, &l.w_gate, &l.wo, &l.w_up, &l.w_down}) linears.push_back(w);
+    for (Linear* w : linears) {
+        if (!w->data || w->data_tiled || w->N <= 0 || w->N % 16 != 0) continue;
+        const size_t row_bytes = w->data_bytes() / static_cast<size_t>(w->N);
+        if (row_bytes % 64 != 0) continue;
+        w->data_tiled = alloc(w->data_bytes(), "");
+        const int st = w->kind == Quant::Int4b8
+                           ? pie_hip_repack_mfma_tiles_int4(w->data, w->data_tiled, w->N, row_bytes, stream)
+                           : pie_hip_repack_mfma_tiles(w->data, w->data_tiled, w->N, row_bytes, stream);
+        if (st != PIE_HIP_OK)
+            throw std::runtime_error("model: weight repack failed");
+        if (w->kind == Quant::Int4b8) {
+            w->scale_tiled = alloc(w->scale_bytes(), "");
+            if (pie_hip_repack_scale_tiles(static_cast<const uint16_t*>(w->scale),
+                                           static_cast<uint16_t*>(w->scale_tiled), w->N, w->K / w->group,
+                                           stream) != PIE_HIP_OK)
+                throw std::runtime_error("model: scale repack failed");
         }
+    }
     PIE_HIP_CHECK(hipStreamSynchronize(stream));
 }
 
@@ -341,64 +346,6 @@ void Model::init_synthetic(const ModelConfig& cfg, hipStream_t stream) {
     tmp_bf16_ = nullptr;
     pair_qk_rows(stream);
 }
-
-namespace {
-
-// Widens / narrows a checkpoint tensor to bf16 bits on the host when it is not bf16 already.
-const uint16_t* as_bf16(const StTensor& t, std::vector<uint16_t>& staging) {
-    const size_t n = static_cast<size_t>(t.elems());
-    if (t.dtype == "BF16") {
-        if (t.bytes != n * 2) throw std::runtime_error("snapshot: BF16 tensor with a wrong byte count");
-        return reinterpret_cast<const uint16_t*>(t.data);
-    }
-    staging.resize(n);
-    auto rne = [](float f) {
-        uint32_t u;
-        std::memcpy(&u, &f, 4);
-        if ((u & 0x7FFFFFFFu) > 0x7F800000u) return static_cast<uint16_t>((u >> 16) | 0x40u);
-        return static_cast<uint16_t>((u + 0x7FFFu + ((u >> 16) & 1u)) >> 16);
-    };
-    if (t.dtype == "F32") {
-        if (t.bytes != n * 4) throw std::runtime_error("snapshot: F32 tensor with a wrong byte count");
-        for (size_t i = 0; i < n; ++i) {
-            float f;
-            std::memcpy(&f, t.data + 4 * i, 4);
-            staging[i] = rne(f);
-        }
-    } else if (t.dtype == "F16") {
-        if (t.bytes != n * 2) throw std::runtime_error("snapshot: F16 tensor with a wrong byte count");
-        for (size_t i = 0; i < n; ++i) {
-            uint16_t h;
-            std::memcpy(&h, t.data + 2 * i, 2);
-            const uint32_t sign = (h & 0x8000u) << 16, exp = (h >> 10) & 0x1Fu, man = h & 0x3FFu;
-            uint32_t u;
-            if (exp == 0) {
-                if (man == 0) u = sign;
-                else {   // subnormal half: normalise
-                    int e = -1;
-                    uint32_t m2 = man;
-                    do { ++e; m2 <<= 1; } while (!(m2 & 0x400u));
-                    u = sign | ((127 - 15 - e) << 23) | ((m2 & 0x3FFu) << 13);
-                }
-            } else if (exp == 31) u = sign | 0x7F800000u | (man << 13);
-            else u = sign | ((exp + 112) << 23) | (man << 13);
-            float f;
-            std::memcpy(&f, &u, 4);
-            staging[i] = rne(f);
-        }
-    } else {
-        throw std::runtime_error("snapshot: dtype " + t.dtype + " is not a floating weight");
-    }
-    return staging.data();
-}
-
-void expect_shape(const StTensor& t, const std::string& name, int64_t rows, int64_t cols) {
-    const bool ok = cols < 0 ? (t.shape.size() == 1 && t.shape[0] == rows)
-                             : (t.shape.size() == 2 && t.shape[0] == rows && t.shape[1] == cols);
-    if (!ok) throw std::runtime_error("snapshot: tensor '" + name + "' has an unexpected shape");
-}
-
-}  // namespace
 
 void Model::load_snapshot(const ModelConfig& cfg, hipStream_t stream) {
     cfg_ = cfg;

@@ -65,6 +65,56 @@ struct LayerWeights {
     Linear router;                // MoE: [E, H] bf16
 };
 
+// Where everything sits in a layer-stack layer's padded matrices and rows.  Sizes that are the K of
+// a product are rounded up so that every product takes the matrix-core kernels (zero columns in
+// the weights, zero or ignored entries in the rows).
+constexpr int pad_to(int v, int a) { return (v + a - 1) / a * a; }
+struct LatentShape {
+    int heads, dimp, rotp, vdp, kvp;   // per-head sizes and the latent, rounded up
+    int kv_off, ld_in;                 // fused down projection: query latent | (kv_off) latent, rotated key part
+    int ld_cq, hd, ld_q;               // query latent rows; q rows: heads of [dimp | rotp]
+    int ld_row;                        // cache row: [kvp | rotp]
+    int ld_o;                          // attention output rows: heads of vdp
+    explicit LatentShape(const LatentAttentionSpec& a)
+        : heads(a.heads), dimp(pad_to(a.dim, 32)), rotp(pad_to(a.rot_dim, 32)), vdp(pad_to(a.vdim, 32)),
+          kvp(pad_to(a.kv_rank, 64)), kv_off(pad_to(a.q_rank, 16)), ld_in(pad_to(kv_off + a.kv_rank + a.rot_dim, 16)),
+          ld_cq(pad_to(a.q_rank, 128)), hd(dimp + rotp), ld_q(heads * hd), ld_row(kvp + rotp),
+          ld_o(pad_to(heads * vdp, 128)) {}
+};
+struct DeltaShape {
+    int kd, vd, channels;                       // q (= k) channels, v channels, all three
+    int decay_off, gate_off, ld_in;             // fused projection: q | k | v | step sizes | decay | gate inputs
+    int ld_a1, ld_g1, ld_decay, ld_gate, ld_o;  // low-rank inputs, their projections, output rows
+    explicit DeltaShape(const ChannelDeltaSpec& d)
+        : kd(d.kv_heads * d.dim), vd(d.heads * d.vdim), channels(2 * kd + vd), decay_off(pad_to(channels + d.heads, 8)),
+          gate_off(pad_to(decay_off + d.decay_rank, 8)), ld_in(pad_to(gate_off + d.gate_rank, 16)),
+          ld_a1(pad_to(d.decay_rank, 128)), ld_g1(pad_to(d.gate_rank, 128)), ld_decay(pad_to(d.heads * d.dim, 16)),
+          ld_gate(pad_to(vd, 16)), ld_o(pad_to(vd, 128)) {}
+};
+
+struct StackLayer {
+    LayerSpec spec;
+    float *norm1 = nullptr, *norm2 = nullptr;
+    Linear w_in;            // everything the mixer projects its input to, fused
+    Linear wo;
+    Linear w_up, w_down;    // feed-forward (none: data null)
+    // latent attention
+    Linear w_uq;
+    Linear w_ukv;                                // [heads * (dimp + vdp), kvp]: keys and values out of the latent
+    uint16_t *w_uk_t = nullptr, *w_uv = nullptr; // per head [kvp, dimp] (transposed keys) and [vdp, kvp]
+    float *q_norm = nullptr, *kv_norm = nullptr;
+    int rotary = -1;                             // index into Model::rotary
+    // channel delta
+    Linear w_decay, w_gate;                      // second factors of the low-rank decay and output gate
+    float *conv_w = nullptr, *a_log = nullptr, *dt_bias = nullptr, *out_norm = nullptr;
+};
+
+struct RotaryTable {
+    RotarySpec spec;
+    double* freq = nullptr;   // [dims / 2] device
+    float mscale = 1.f;
+};
+
 struct TensorRef {
     void* ptr;
     size_t bytes;
@@ -90,6 +140,9 @@ class Model {
     // Builds the tile-major copies of every decoder linear whose shape the skinny GEMM takes.
     void build_tiled_copies(hipStream_t stream);
 
+    // Layer stacks (cfg.stack): weights from the snapshot, or synthetic with cfg.random_weights.
+    void load_stack(const ModelConfig& cfg, hipStream_t stream);
+
     const ModelConfig& cfg() const { return cfg_; }
     bool is_moe() const { return cfg_.arch == "qwen3_moe"; }
     bool has_qk_norm() const { return cfg_.arch != "llama3"; }
@@ -104,6 +157,12 @@ class Model {
     uint16_t* final_norm = nullptr;
     float* inv_freq = nullptr;  // [d/2] device
     std::vector<LayerWeights> layers;
+    // layer stacks
+    std::vector<StackLayer> stack;
+    std::vector<RotaryTable> rotary;   // the stack's distinct rotations
+    Linear head;                       // lm_head, padded
+    float* stack_norm = nullptr;       // norm ahead of it
+    int ld_x() const { return pad_to(cfg_.hidden, 128); }
 
     // bytes streamed from HBM by one decode step at batch 1 (every weight once)
     size_t decode_weight_bytes() const { return decode_bytes_; }
@@ -131,6 +190,11 @@ class Model {
 // Host-side inv_freq table (theta^(-2i/d) with optional llama3 band scaling,
 // driver/portable/src/model.cpp:1414-1448: the stored factor divides the base frequency).
 std::vector<float> rope_inv_freq(const ModelConfig& cfg);
+// Frequencies of a rotation spec, and what its cos and sin are multiplied by.
+std::vector<double> rotary_frequencies(const RotarySpec& r);
+float rotary_mscale(const RotarySpec& r);
+// bf16 N(mean, std) on the device, a pure function of (seed, index)
+void fill_normal(uint16_t* dst, size_t n, uint64_t seed, float mean, float std, hipStream_t stream);
 // What cos and sin are multiplied by: YaRN's attention factor (0.1 ln(factor) + 1 unless the
 // config states one), 1 for every other scheme.
 float rope_mscale(const ModelConfig& cfg);

@@ -1,0 +1,268 @@
+// Weights of layer-stack models: checkpoint tensors ("embed", "l<i>.norm1", "l<i>.mix.*",
+// "l<i>.mlp.*", "final.norm", "head") into the padded, fused matrices the kernels read.
+#include <cmath>
+#include <cstring>
+#include <memory>
+#include <stdexcept>
+
+#include "model.hpp"
+#include "pie_hip_kernels.h"
+#include "snapshot.hpp"
+
+namespace pie_hip_driver {
+
+#define PIE_HIP_CHECK(expr)                                                              \
+    do {                                                                                 \
+        hipError_t e_ = (expr);                                                          \
+        if (e_ != hipSuccess)                                                            \
+            throw std::runtime_error(std::string(#expr) + ": " + hipGetErrorString(e_)); \
+    } while (0)
+
+// f_i = base^(-2i/dims); with YaRN scaling f_i / factor above the pair that turns `slow` times
+// over the original context, f_i below the one that turns `fast` times, a linear ramp between.
+std::vector<double> rotary_frequencies(const RotarySpec& r) {
+    std::vector<double> out(static_cast<size_t>(r.dims / 2));
+    double lo = 0.0, hi = 0.0;
+    if (r.yarn) {
+        auto pair_with_turns = [&](double turns) {
+            return r.dims * std::log(r.original / (2.0 * 3.14159265358979323846 * turns)) / (2.0 * std::log(r.base));
+        };
+        lo = std::max(std::floor(pair_with_turns(r.fast)), 0.0);
+        hi = std::min(std::ceil(pair_with_turns(r.slow)), static_cast<double>(r.dims) - 1.0);
+    }
+    for (size_t i = 0; i < out.size(); ++i) {
+        const double f = std::pow(r.base, -2.0 * static_cast<double>(i) / r.dims);
+        out[i] = f;
+        if (r.yarn) {
+            const double ramp = std::min(1.0, std::max(0.0, (static_cast<double>(i) - lo) / std::max(hi - lo, 0.001)));
+            out[i] = f / r.factor * ramp + f * (1.0 - ramp);
+        }
+    }
+    return out;
+}
+
+float rotary_mscale(const RotarySpec& r) {
+    return r.yarn ? static_cast<float>(0.1 * std::log(r.factor) + 1.0) : 1.f;
+}
+
+namespace {
+
+// A checkpoint matrix on the host: bf16 bits [rows, cols].
+struct HostMatrix {
+    std::vector<uint16_t> v;
+    int rows = 0, cols = 0;
+    const uint16_t* row(int r) const { return v.data() + static_cast<size_t>(r) * cols; }
+};
+
+float bf16_value(uint16_t b) {
+    const uint32_t u = static_cast<uint32_t>(b) << 16;
+    float f;
+    std::memcpy(&f, &u, 4);
+    return f;
+}
+
+}  // namespace
+
+void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
+    cfg_ = cfg;
+    quant_ = Quant::Bf16;
+    const bool random = cfg.random_weights;
+    std::unique_ptr<Snapshot> snap;
+    if (!random) snap = std::make_unique<Snapshot>(cfg.checkpoint_dir);
+    std::uint64_t seed = cfg.seed;
+    auto next_seed = [&]() { return seed += 0xA0761D6478BD642Full; };
+    const int H = cfg.hidden, Hp = ld_x(), V = cfg.vocab;
+
+    auto matrix = [&](const std::string& name, int rows, int cols) {
+        const StTensor& t = snap->at(name);
+        expect_shape(t, name, rows, cols);
+        HostMatrix m;
+        std::vector<uint16_t> staging;
+        const uint16_t* p = as_bf16(t, staging);
+        m.v.assign(p, p + t.elems());
+        m.rows = rows;
+        m.cols = cols;
+        return m;
+    };
+    // fp32 vector (or small matrix) parameter; `dflt` fills it for random weights
+    auto vec = [&](const std::string& name, size_t n, auto dflt) {
+        std::vector<float> v(n);
+        if (random) {
+            for (size_t i = 0; i < n; ++i) v[i] = dflt(i);
+        } else {
+            const StTensor& t = snap->at(name);
+            if (t.elems() != static_cast<int64_t>(n)) throw std::runtime_error("snapshot: tensor '" + name + "' has an unexpected shape");
+            if (t.dtype == "F32") {   // kept to the last bit
+                std::memcpy(v.data(), t.data, 4 * n);
+            } else {
+                std::vector<uint16_t> staging;
+                const uint16_t* p = as_bf16(t, staging);
+                for (size_t i = 0; i < n; ++i) v[i] = bf16_value(p[i]);
+            }
+        }
+        float* d = static_cast<float*>(alloc(4 * n, name));
+        PIE_HIP_CHECK(hipMemcpyAsync(d, v.data(), 4 * n, hipMemcpyHostToDevice, stream));
+        PIE_HIP_CHECK(hipStreamSynchronize(stream));
+        return d;
+    };
+    auto ones = [](size_t) { return 1.f; };
+    auto upload = [&](uint16_t* dst, const std::vector<uint16_t>& host) {
+        PIE_HIP_CHECK(hipMemcpyAsync(dst, host.data(), host.size() * 2, hipMemcpyHostToDevice, stream));
+        PIE_HIP_CHECK(hipStreamSynchronize(stream));
+    };
+    auto device_matrix = [&](const std::string& name, size_t elems, int fan_in, auto fill) {
+        auto* d = static_cast<uint16_t*>(alloc(elems * 2, name));
+        if (random) {
+            fill_normal(d, elems, next_seed(), 0.f, 0.7f / std::sqrt(static_cast<float>(fan_in)), stream);
+        } else {
+            std::vector<uint16_t> host(elems, 0);
+            fill(host);
+            upload(d, host);
+        }
+        return d;
+    };
+    // [N, K] zero-padded linear; fill(put) places checkpoint rows: put(row, first column, values, n)
+    auto linear = [&](Linear& lin, const std::string& name, int N, int K, int fan_in, auto fill) {
+        lin.kind = Quant::Bf16;
+        lin.N = N;
+        lin.K = K;
+        lin.data = device_matrix(name, static_cast<size_t>(N) * K, fan_in, [&](std::vector<uint16_t>& host) {
+            fill([&](int row, int col, const uint16_t* src, int n) {
+                std::memcpy(host.data() + static_cast<size_t>(row) * K + col, src, static_cast<size_t>(n) * 2);
+            });
+        });
+        decode_bytes_ += lin.data_bytes();
+    };
+    // rows [row0, row0 + rows) = the tensor's rows as they are
+    auto plain_rows = [&](const auto& put, const std::string& name, int row0, int rows, int cols) {
+        const HostMatrix m = matrix(name, rows, cols);
+        for (int r = 0; r < rows; ++r) put(row0 + r, 0, m.row(r), cols);
+    };
+    auto rotary_of = [&](const RotarySpec& spec) {
+        if (spec.dims == 0) return -1;
+        for (size_t i = 0; i < rotary.size(); ++i)
+            if (rotary[i].spec == spec) return static_cast<int>(i);
+        RotaryTable t;
+        t.spec = spec;
+        t.mscale = rotary_mscale(spec);
+        const std::vector<double> f = rotary_frequencies(spec);
+        t.freq = static_cast<double*>(alloc(f.size() * 8, "rotary." + std::to_string(rotary.size())));
+        PIE_HIP_CHECK(hipMemcpyAsync(t.freq, f.data(), f.size() * 8, hipMemcpyHostToDevice, stream));
+        PIE_HIP_CHECK(hipStreamSynchronize(stream));
+        rotary.push_back(t);
+        return static_cast<int>(rotary.size()) - 1;
+    };
+
+    embed = device_matrix("embed", static_cast<size_t>(V) * H, 1,
+                          [&](std::vector<uint16_t>& host) { host = matrix("embed", V, H).v; });
+    linear(head, "head", pad_to(V, 16), Hp, H, [&](auto put) { plain_rows(put, "head", 0, V, H); });
+    stack_norm = vec("final.norm", H, ones);
+
+    stack.resize(cfg.stack.size());
+    for (size_t l = 0; l < stack.size(); ++l) {
+        StackLayer& w = stack[l];
+        w.spec = cfg.stack[l];
+        const std::string p = "l" + std::to_string(l) + ".", mix = p + "mix.";
+        w.norm1 = vec(p + "norm1", H, ones);
+        if (w.spec.mixer == MixerKind::LatentAttention) {
+            const LatentAttentionSpec& a = w.spec.latent;
+            const LatentShape s(a);
+            w.rotary = rotary_of(a.rot);
+            w.q_norm = vec(mix + "dq.norm", a.q_rank, ones);
+            w.kv_norm = vec(mix + "dkv.norm", a.kv_rank, ones);
+            linear(w.w_in, mix + "in", s.ld_in, Hp, H, [&](auto put) {
+                plain_rows(put, mix + "dq", 0, a.q_rank, H);
+                plain_rows(put, mix + "dkv", s.kv_off, a.kv_rank + a.rot_dim, H);
+            });
+            linear(w.w_uq, mix + "uq", s.ld_q, s.ld_cq, a.q_rank, [&](auto put) {
+                const HostMatrix m = matrix(mix + "uq", a.heads * (a.dim + a.rot_dim), a.q_rank);
+                for (int h = 0; h < a.heads; ++h)
+                    for (int i = 0; i < a.dim + a.rot_dim; ++i)
+                        put(h * s.hd + (i < a.dim ? i : s.dimp + i - a.dim), 0, m.row(h * (a.dim + a.rot_dim) + i), a.q_rank);
+            });
+            HostMatrix uk, uv;
+            if (!random) {
+                uk = matrix(mix + "uk", a.heads * a.dim, a.kv_rank);
+                uv = matrix(mix + "uv", a.heads * a.vdim, a.kv_rank);
+            }
+            w.w_uk_t = device_matrix(mix + "uk_t", static_cast<size_t>(a.heads) * s.kvp * s.dimp, a.dim,
+                                     [&](std::vector<uint16_t>& host) {
+                                         for (int h = 0; h < a.heads; ++h)
+                                             for (int d = 0; d < a.dim; ++d)
+                                                 for (int r = 0; r < a.kv_rank; ++r)
+                                                     host[(static_cast<size_t>(h) * s.kvp + r) * s.dimp + d] = uk.row(h * a.dim + d)[r];
+                                     });
+            w.w_uv = device_matrix(mix + "uv", static_cast<size_t>(a.heads) * s.vdp * s.kvp, a.kv_rank,
+                                   [&](std::vector<uint16_t>& host) {
+                                       for (int h = 0; h < a.heads; ++h)
+                                           for (int c = 0; c < a.vdim; ++c)
+                                               std::memcpy(&host[(static_cast<size_t>(h) * s.vdp + c) * s.kvp],
+                                                           uv.row(h * a.vdim + c), static_cast<size_t>(a.kv_rank) * 2);
+                                   });
+            const size_t before = decode_bytes_;
+            linear(w.w_ukv, mix + "ukv", a.heads * (s.dimp + s.vdp), s.kvp, a.kv_rank, [&](auto put) {
+                for (int h = 0; h < a.heads; ++h) {
+                    for (int d = 0; d < a.dim; ++d) put(h * (s.dimp + s.vdp) + d, 0, uk.row(h * a.dim + d), a.kv_rank);
+                    for (int c = 0; c < a.vdim; ++c)
+                        put(h * (s.dimp + s.vdp) + s.dimp + c, 0, uv.row(h * a.vdim + c), a.kv_rank);
+                }
+            });
+            decode_bytes_ = before + static_cast<size_t>(a.heads) * s.kvp * (s.dimp + s.vdp) * 2;   // (decode reads uk_t and uv instead)
+            linear(w.wo, mix + "o", Hp, s.ld_o, a.heads * a.vdim, [&](auto put) {
+                const HostMatrix m = matrix(mix + "o", H, a.heads * a.vdim);
+                for (int r = 0; r < H; ++r)
+                    for (int h = 0; h < a.heads; ++h) put(r, h * s.vdp, m.row(r) + h * a.vdim, a.vdim);
+            });
+        } else {
+            ChannelDeltaSpec& d = w.spec.delta;
+            // the ranks of the decay and the output gate are the shapes of their first factors
+            auto rank_of = [&](const std::string& name, int dflt) {
+                if (random) return dflt;
+                const StTensor& t = snap->at(name);
+                if (t.shape.size() != 2 || t.shape[0] <= 0 || t.shape[0] > (1 << 20))
+                    throw std::runtime_error("snapshot: tensor '" + name + "' has an unexpected shape");
+                return static_cast<int>(t.shape[0]);
+            };
+            d.decay_rank = rank_of(mix + "a1", d.decay_rank > 0 ? d.decay_rank : d.dim);
+            d.gate_rank = rank_of(mix + "g1", d.gate_rank > 0 ? d.gate_rank : d.vdim);
+            const DeltaShape s(d);
+            linear(w.w_in, mix + "in", s.ld_in, Hp, H, [&](auto put) {
+                plain_rows(put, mix + "q", 0, s.kd, H);
+                plain_rows(put, mix + "k", s.kd, s.kd, H);
+                plain_rows(put, mix + "v", 2 * s.kd, s.vd, H);
+                plain_rows(put, mix + "b", s.channels, d.heads, H);
+                plain_rows(put, mix + "a1", s.decay_off, d.decay_rank, H);
+                plain_rows(put, mix + "g1", s.gate_off, d.gate_rank, H);
+            });
+            linear(w.w_decay, mix + "a2", s.ld_decay, s.ld_a1, d.decay_rank,
+                   [&](auto put) { plain_rows(put, mix + "a2", 0, d.heads * d.dim, d.decay_rank); });
+            linear(w.w_gate, mix + "g2", s.ld_gate, s.ld_g1, d.gate_rank,
+                   [&](auto put) { plain_rows(put, mix + "g2", 0, s.vd, d.gate_rank); });
+            linear(w.wo, mix + "o", Hp, s.ld_o, s.vd, [&](auto put) { plain_rows(put, mix + "o", 0, H, s.vd); });
+            w.a_log = vec(mix + "A_log", d.heads, [&](size_t i) { return std::log(1.f + static_cast<float>(i % 8)); });
+            w.dt_bias = vec(mix + "dt_bias", static_cast<size_t>(d.heads) * d.dim, [](size_t) { return -3.f; });
+            w.out_norm = vec(mix + "norm", d.vdim, ones);
+            // the three convolutions back to back, [channels, taps]
+            std::vector<float> conv(static_cast<size_t>(s.channels) * d.taps, 0.5f);
+            if (!random) {
+                size_t at = 0;
+                for (const auto& [name, ch] : {std::pair<const char*, int>{"q", s.kd}, {"k", s.kd}, {"v", s.vd}}) {
+                    const HostMatrix m = matrix(mix + name + ".conv", ch, d.taps);
+                    for (uint16_t b : m.v) conv[at++] = bf16_value(b);
+                }
+            }
+            w.conv_w = static_cast<float*>(alloc(conv.size() * 4, mix + "conv"));
+            PIE_HIP_CHECK(hipMemcpyAsync(w.conv_w, conv.data(), conv.size() * 4, hipMemcpyHostToDevice, stream));
+            PIE_HIP_CHECK(hipStreamSynchronize(stream));
+        }
+        if (w.spec.ff > 0) {
+            const int ff = w.spec.ff, ffp = pad_to(ff, 128);
+            w.norm2 = vec(p + "norm2", H, ones);
+            linear(w.w_up, p + "mlp.up", ffp, Hp, H, [&](auto put) { plain_rows(put, p + "mlp.up", 0, ff, H); });
+            linear(w.w_down, p + "mlp.down", Hp, ffp, ff, [&](auto put) { plain_rows(put, p + "mlp.down", 0, H, ff); });
+        }
+    }
+    PIE_HIP_CHECK(hipStreamSynchronize(stream));
+}
+
+}  // namespace pie_hip_driver

@@ -54,6 +54,8 @@ struct BatchPlan {
     std::vector<std::vector<uint32_t>> logit_mask_runs;  // [R] BRLE runs (empty = no constraint)
     std::vector<std::vector<uint32_t>> draft_tokens;     // [R] speculative drafts to verify
     std::vector<std::vector<uint32_t>> row_mask_runs;    // [N] when has_user_masks: BRLE runs per token row
+    std::vector<uint32_t> rs_slots;   // [R] recurrent-state slots, empty when the request names none
+    std::vector<uint8_t> rs_flags;    // [R] or empty
     int max_kv_len = 0;
     bool pure_decode = false;  // every request has exactly one token row, no user masks
     bool all_greedy = false;   // every sampling slot is a token sampler with temperature ~ 0
@@ -145,6 +147,8 @@ inline BatchPlan plan_forward(const PieForwardRequestDesc& f, int page_size, int
     p.seq_len.resize(R);
     p.qo_indptr.assign(f.qo_indptr.ptr, f.qo_indptr.ptr + R + 1);
     p.page_indices.assign(f.kv_page_indices.ptr, f.kv_page_indices.ptr + f.kv_page_indices.len);
+    p.rs_slots.assign(f.rs_slot_ids.ptr, f.rs_slot_ids.ptr + f.rs_slot_ids.len);
+    p.rs_flags.assign(f.rs_slot_flags.ptr, f.rs_slot_flags.ptr + f.rs_slot_flags.len);
     p.sample_indptr.assign(1, 0);
     p.logit_mask_runs.resize(R);
     p.draft_tokens.resize(R);

@@ -298,13 +298,166 @@ class Snapshot {
     std::map<std::string, StTensor> tensors_;
 };
 
+// ---- checkpoint tensors as weights -----------------------------------------------------------
+// Widens / narrows a checkpoint tensor to bf16 bits on the host when it is not bf16 already.
+inline const uint16_t* as_bf16(const StTensor& t, std::vector<uint16_t>& staging) {
+    const size_t n = static_cast<size_t>(t.elems());
+    if (t.dtype == "BF16") {
+        if (t.bytes != n * 2) throw std::runtime_error("snapshot: BF16 tensor with a wrong byte count");
+        return reinterpret_cast<const uint16_t*>(t.data);
+    }
+    staging.resize(n);
+    auto rne = [](float f) {
+        uint32_t u;
+        std::memcpy(&u, &f, 4);
+        if ((u & 0x7FFFFFFFu) > 0x7F800000u) return static_cast<uint16_t>((u >> 16) | 0x40u);
+        return static_cast<uint16_t>((u + 0x7FFFu + ((u >> 16) & 1u)) >> 16);
+    };
+    if (t.dtype == "F32") {
+        if (t.bytes != n * 4) throw std::runtime_error("snapshot: F32 tensor with a wrong byte count");
+        for (size_t i = 0; i < n; ++i) {
+            float f;
+            std::memcpy(&f, t.data + 4 * i, 4);
+            staging[i] = rne(f);
+        }
+    } else if (t.dtype == "F16") {
+        if (t.bytes != n * 2) throw std::runtime_error("snapshot: F16 tensor with a wrong byte count");
+        for (size_t i = 0; i < n; ++i) {
+            uint16_t h;
+            std::memcpy(&h, t.data + 2 * i, 2);
+            const uint32_t sign = (h & 0x8000u) << 16, exp = (h >> 10) & 0x1Fu, man = h & 0x3FFu;
+            uint32_t u;
+            if (exp == 0) {
+                if (man == 0) u = sign;
+                else {   // subnormal half: normalise
+                    int e = -1;
+                    uint32_t m2 = man;
+                    do { ++e; m2 <<= 1; } while (!(m2 & 0x400u));
+                    u = sign | ((127 - 15 - e) << 23) | ((m2 & 0x3FFu) << 13);
+                }
+            } else if (exp == 31) u = sign | 0x7F800000u | (man << 13);
+            else u = sign | ((exp + 112) << 23) | (man << 13);
+            float f;
+            std::memcpy(&f, &u, 4);
+            staging[i] = rne(f);
+        }
+    } else {
+        throw std::runtime_error("snapshot: dtype " + t.dtype + " is not a floating weight");
+    }
+    return staging.data();
+}
+
+inline void expect_shape(const StTensor& t, const std::string& name, int64_t rows, int64_t cols) {
+    const bool ok = cols < 0 ? (t.shape.size() == 1 && t.shape[0] == rows)
+                             : (t.shape.size() == 2 && t.shape[0] == rows && t.shape[1] == cols);
+    if (!ok) throw std::runtime_error("snapshot: tensor '" + name + "' has an unexpected shape");
+}
+
+// ---- config.json -> ModelConfig: layer stacks ---------------------------------------------------
+inline int json_size(const Json& j, const std::string& key, const std::string& at) {
+    const Json* v = j.get(key);
+    if (!v || v->kind != Json::Number || v->num != static_cast<double>(static_cast<int>(v->num)))
+        throw std::runtime_error("snapshot: " + at + " needs an integer '" + key + "'");
+    return static_cast<int>(v->num);
+}
+inline double json_number(const Json& j, const std::string& key, const std::string& at) {
+    const Json* v = j.get(key);
+    if (!v || v->kind != Json::Number) throw std::runtime_error("snapshot: " + at + " needs a number '" + key + "'");
+    return v->num;
+}
+
+inline RotarySpec parse_rotary(const Json& j, const std::string& at) {
+    RotarySpec r;
+    r.dims = json_size(j, "dims", at);
+    r.base = json_number(j, "base", at);
+    if (const Json* s = j.get("scaling"); s && s->kind == Json::Object) {
+        r.yarn = true;
+        r.factor = json_number(*s, "factor", at);
+        r.original = json_number(*s, "original", at);
+        r.fast = json_number(*s, "fast", at);
+        r.slow = json_number(*s, "slow", at);
+    }
+    return r;
+}
+
+// One entry per mixer kind: config name -> reader of its sizes.
+struct MixerReader {
+    const char* type;
+    void (*read)(LayerSpec& l, const Json& mixer, const std::string& at);
+};
+inline const std::vector<MixerReader>& mixer_registry() {
+    static const std::vector<MixerReader> table = {
+        {"latent_attention",
+         [](LayerSpec& l, const Json& j, const std::string& at) {
+             l.mixer = MixerKind::LatentAttention;
+             auto& a = l.latent;
+             a.heads = json_size(j, "heads", at);
+             a.dim = json_size(j, "dim", at);
+             a.rot_dim = json_size(j, "rot_dim", at);
+             a.vdim = json_size(j, "vdim", at);
+             a.q_rank = json_size(j, "q_rank", at);
+             a.kv_rank = json_size(j, "kv_rank", at);
+             a.scale = json_number(j, "scale", at);
+             const Json* rot = j.get("rot");
+             if (rot && rot->kind == Json::Object) a.rot = parse_rotary(*rot, at + " rot");
+         }},
+        {"channel_delta",
+         [](LayerSpec& l, const Json& j, const std::string& at) {
+             l.mixer = MixerKind::ChannelDelta;
+             auto& d = l.delta;
+             d.heads = json_size(j, "heads", at);
+             d.kv_heads = json_size(j, "kv_heads", at);
+             d.dim = json_size(j, "dim", at);
+             d.vdim = json_size(j, "vdim", at);
+             d.taps = json_size(j, "conv", at);
+         }},
+    };
+    return table;
+}
+
+// {"architecture", "width", "vocab", "norm": {"eps"}, "logit_scale", "logit_softcap",
+//  "layers": [{"type", "mixer": {...}, "mlp": {"kind", "ff"} | null}, ...]}
+inline void apply_stack_config(ModelConfig& m, const Json& c) {
+    m.arch = "varasun";
+    m.hidden = json_size(c, "width", "config.json");
+    m.vocab = json_size(c, "vocab", "config.json");
+    const Json* norm = c.get("norm");
+    if (!norm) throw std::runtime_error("snapshot: config.json needs 'norm'");
+    m.rms_eps = static_cast<float>(json_number(*norm, "eps", "norm"));
+    m.logit_scale = static_cast<float>(c.number_or("logit_scale", 1.0));
+    m.logit_softcap = static_cast<float>(c.number_or("logit_softcap", 0.0));
+    const Json* layers = c.get("layers");
+    if (!layers || layers->kind != Json::Array || layers->arr.empty())
+        throw std::runtime_error("snapshot: config.json needs a list 'layers'");
+    m.stack.clear();
+    for (const Json& j : layers->arr) {
+        const std::string at = "layer " + std::to_string(m.stack.size());
+        LayerSpec l;
+        const std::string type = j.string_or("type", "");
+        const Json* mixer = j.get("mixer");
+        if (!mixer || mixer->kind != Json::Object) throw std::runtime_error("snapshot: " + at + " needs 'mixer'");
+        bool known = false;
+        for (const MixerReader& r : mixer_registry())
+            if (type == r.type) {
+                r.read(l, *mixer, at);
+                known = true;
+            }
+        if (!known) throw std::runtime_error("snapshot: " + at + ": unknown mixer '" + type + "'");
+        if (const Json* mlp = j.get("mlp"); mlp && mlp->kind == Json::Object) {
+            const std::string kind = mlp->string_or("kind", "");
+            if (kind != "dense") throw std::runtime_error("snapshot: " + at + ": unknown mlp kind '" + kind + "'");
+            l.ff = json_size(*mlp, "ff", at + " mlp");
+            if (l.ff <= 0) throw std::runtime_error("snapshot: " + at + ": mlp.ff must be positive");
+        }
+        m.stack.push_back(l);
+    }
+}
+
 // ---- config.json -> ModelConfig ----------------------------------------------------------------
 // Field names as transformers writes them (llama / qwen3 / qwen3_moe); the reference reads the
 // same keys in driver/portable/src/hf_config.cpp.  Checkpoints use the half-split RoPE pairing
 // (the CUDA driver's default, driver/cuda/src/kernels/rope.cu:10-21) unless the TOML says otherwise.
-inline void apply_hf_config(ModelConfig& m, const std::string& dir) {
-    const Json c = parse_json_file(dir + "/config.json");
-    const std::string type = c.string_or("model_type", "");
+inline void apply_hf_fields(ModelConfig& m, const Json& c, const std::string& type) {
     if (type == "llama" || type == "mistral") m.arch = "llama3";
     else if (type == "qwen3") m.arch = "qwen3";
     else if (type == "qwen3_moe") m.arch = "qwen3_moe";
@@ -350,6 +503,17 @@ inline void apply_hf_config(ModelConfig& m, const std::string& dir) {
         m.norm_topk = c.bool_or("norm_topk_prob", true);
     }
     if (m.rope_interleaved < 0) m.rope_interleaved = 0;
+}
+
+// The registry of architectures: config.json's "model_type" (Hugging Face checkpoints) or
+// "architecture" (layer stacks) picks the reader.
+inline void apply_hf_config(ModelConfig& m, const std::string& dir) {
+    const Json c = parse_json_file(dir + "/config.json");
+    const std::string arch = c.string_or("architecture", "");
+    if (arch == "Varasun") return apply_stack_config(m, c);
+    const std::string type = c.string_or("model_type", "");
+    if (type.empty() && !arch.empty()) throw std::runtime_error("snapshot: unsupported architecture '" + arch + "'");
+    apply_hf_fields(m, c, type);
 }
 
 }  // namespace pie_hip_driver

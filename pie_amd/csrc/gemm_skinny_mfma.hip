@@ -125,6 +125,7 @@ struct SkinnyArgs {
     const int32_t* offsets;     // grouped: [P+1] first row of each problem; null: one problem
     int M;                      // rows when offsets == null
     int N, K, G, g_shift, beta, swiglu, scale_is_bf16;
+    int relu2;                  // 1: y = bf16(max(sum, 0)^2)
     int m_split;                // dense only: blockIdx.y = 16-row pass
     int tiled;                  // weights (and int4 group scales) in the tile-major layout
     size_t w_stride, scale_stride;  // bytes between problems
@@ -400,6 +401,10 @@ __global__ __launch_bounds__(KP* kWave) void skinny_kernel(const SkinnyArgs a) {
                 }
             } else if (ok) {
                 const size_t o = static_cast<size_t>(m) * nout + n;
+                if (a.relu2) {
+                    v = fmaxf(v, 0.f);
+                    v *= v;
+                }
                 if (a.beta) v += bf16_bits_to_f32(a.y[o]);
                 a.y[o] = f32_to_bf16_bits(v);
             }
@@ -750,6 +755,10 @@ __global__ __launch_bounds__(kSwWaves* kWave, NG == 1 && MT == 1 ? 4 : 2) void s
                 }
             } else if (ok) {
                 const size_t o = static_cast<size_t>(m) * nout + n;
+                if (a.relu2) {
+                    v = fmaxf(v, 0.f);
+                    v *= v;
+                }
                 if (a.beta) v += bf16_bits_to_f32(a.y[o]);
                 a.y[o] = f32_to_bf16_bits(v);
             }
@@ -865,6 +874,7 @@ int launch_skinny(SkinnyArgs a, int problems, hipStream_t stream) {
         a.g_shift = __builtin_ctz(static_cast<unsigned>(a.G));
     }
     if (a.swiglu && (a.N % 2 != 0 || a.beta)) return PIE_HIP_ERR_INVALID;
+    if (a.relu2 && a.beta) return PIE_HIP_ERR_INVALID;
     if (problems > 65535) return PIE_HIP_ERR_UNSUPPORTED;
     // Dense matrices with more than one 16-row pass: one block per (tile group, pass) instead
     // of a pass loop inside the block.  The passes then read the same weights at about the same
@@ -974,7 +984,8 @@ extern "C" int pie_hip_gemm_skinny(int format, const uint16_t* act_bf16, const v
     a.K = K;
     a.G = group_size;
     a.beta = beta;
-    a.swiglu = swiglu ? 1 : 0;
+    a.swiglu = swiglu == PIE_HIP_EPI_SWIGLU ? 1 : 0;
+    a.relu2 = swiglu == PIE_HIP_EPI_RELU2 ? 1 : 0;
     a.scale_is_bf16 = scale_is_bf16;
     return dispatch_skinny(format, a, 1, static_cast<hipStream_t>(stream));
 }
@@ -1002,7 +1013,8 @@ extern "C" int pie_hip_moe_grouped_gemm(int format, const uint16_t* act_bf16,
     a.N = N;
     a.K = K;
     a.G = group_size;
-    a.swiglu = swiglu ? 1 : 0;
+    a.swiglu = swiglu == PIE_HIP_EPI_SWIGLU ? 1 : 0;
+    a.relu2 = swiglu == PIE_HIP_EPI_RELU2 ? 1 : 0;
     a.scale_is_bf16 = scale_is_bf16;
     a.w_stride = weight_stride_bytes;
     a.scale_stride = scale_stride_bytes;
@@ -1027,7 +1039,8 @@ extern "C" int pie_hip_gemm_skinny_tiled(int format, const uint16_t* act_bf16, c
     a.K = K;
     a.G = group_size;
     a.beta = beta;
-    a.swiglu = swiglu ? 1 : 0;
+    a.swiglu = swiglu == PIE_HIP_EPI_SWIGLU ? 1 : 0;
+    a.relu2 = swiglu == PIE_HIP_EPI_RELU2 ? 1 : 0;
     a.scale_is_bf16 = scale_is_bf16;
     a.tiled = 1;
     return dispatch_skinny(format, a, 1, static_cast<hipStream_t>(stream));
@@ -1093,7 +1106,8 @@ extern "C" int pie_hip_moe_grouped_gemm_tiled(int format, const uint16_t* act_bf
     a.N = N;
     a.K = K;
     a.G = group_size;
-    a.swiglu = swiglu ? 1 : 0;
+    a.swiglu = swiglu == PIE_HIP_EPI_SWIGLU ? 1 : 0;
+    a.relu2 = swiglu == PIE_HIP_EPI_RELU2 ? 1 : 0;
     a.scale_is_bf16 = scale_is_bf16;
     a.tiled = 1;
     a.w_stride = weight_stride_bytes;

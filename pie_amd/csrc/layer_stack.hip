@@ -1,0 +1,278 @@
+// The kernels every layer of a layer-stack model shares: embedding into an fp32 residual stream,
+// the norm-and-add that ends a sublayer, the output norm, the logit finish (scale, soft cap,
+// argmax), the rotation table, and the fp32 linear of the 32-bit compute type.
+//
+// The residual stream x is fp32 [rows, ld]; the activations the products read are a copy of it in
+// the compute type, written by the kernel that last changed x, so no product starts with a
+// conversion.  Columns from the width to ld are zero in both.
+#include "act_type.hip.h"
+
+namespace pie_hip {
+namespace {
+
+template <class T>
+__global__ __launch_bounds__(256) void embed_stream_kernel(const uint32_t* __restrict__ tokens,
+                                                           const uint16_t* __restrict__ table,
+                                                           float* __restrict__ x, T* __restrict__ xa, int width,
+                                                           int ld, int vocab) {
+    const int n = blockIdx.x;
+    const uint32_t t = tokens[n];
+    const size_t row = t < static_cast<uint32_t>(vocab) ? t : 0;
+    for (int i = threadIdx.x; i < ld; i += blockDim.x) {
+        const float v = i < width ? bf16_bits_to_f32(table[row * width + i]) : 0.f;
+        x[static_cast<size_t>(n) * ld + i] = v;
+        xa[static_cast<size_t>(n) * ld + i] = act_put<T>(v);
+    }
+}
+
+// x += y / sqrt(mean(y^2) + eps) * w, and the compute-type copy of the new x.  One block per row;
+// a thread keeps the first kCache of its elements in registers between the two passes, requested
+// together with x and w so that the row waits for memory once.
+template <class T, int BLOCK>
+__global__ __launch_bounds__(BLOCK) void norm_add_kernel(const T* __restrict__ y, const float* __restrict__ w,
+                                                       float* __restrict__ x, T* __restrict__ xa, int width, int ldy,
+                                                       int ld, float eps) {
+    __shared__ float red[BLOCK / kWave];
+    const size_t n = blockIdx.x;
+    const T* yr = y + n * ldy;
+    float* xr = x + n * ld;
+    T* ar = xa + n * ld;
+    constexpr int kCache = 8;   // groups of four
+    f32x4_t yv[kCache], xv[kCache], wv[kCache];
+    float local = 0.f;
+    const int n4 = width / 4;
+#pragma unroll
+    for (int c = 0; c < kCache; ++c) {
+        const int i = threadIdx.x + c * BLOCK;
+        if (i < n4) {
+            if constexpr (sizeof(T) == 2) {
+                const u32x2_t r = *reinterpret_cast<const u32x2_t*>(yr + 4 * i);
+                yv[c] = f32x4_t{bf16_lo(r.x), bf16_hi(r.x), bf16_lo(r.y), bf16_hi(r.y)};
+            } else {
+                yv[c] = *reinterpret_cast<const f32x4_t*>(yr + 4 * i);
+            }
+            xv[c] = *reinterpret_cast<const f32x4_t*>(xr + 4 * i);
+            wv[c] = *reinterpret_cast<const f32x4_t*>(w + 4 * i);
+        }
+    }
+#pragma unroll
+    for (int c = 0; c < kCache; ++c)
+        if (threadIdx.x + c * BLOCK < n4)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) local += yv[c][e] * yv[c][e];
+    const int done = min(n4, kCache * BLOCK) * 4;   // the rest: wider rows and a width's last one to three
+    for (int i = done + threadIdx.x; i < width; i += BLOCK) {
+        const float v = act_get<T>(yr[i]);
+        local += v * v;
+    }
+    const float inv = 1.f / sqrtf(block_total(local, red) / static_cast<float>(width) + eps);
+#pragma unroll
+    for (int c = 0; c < kCache; ++c) {
+        const int i = threadIdx.x + c * BLOCK;
+        if (i < n4) {
+            f32x4_t o;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) o[e] = xv[c][e] + yv[c][e] * inv * wv[c][e];
+            *reinterpret_cast<f32x4_t*>(xr + 4 * i) = o;
+            if constexpr (sizeof(T) == 2)
+                *reinterpret_cast<u32x2_t*>(ar + 4 * i) = u32x2_t{pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3])};
+            else *reinterpret_cast<f32x4_t*>(ar + 4 * i) = o;
+        }
+    }
+    for (int i = done + threadIdx.x; i < width; i += BLOCK) {
+        const float v = xr[i] + act_get<T>(yr[i]) * inv * w[i];
+        xr[i] = v;
+        ar[i] = act_put<T>(v);
+    }
+}
+
+// out[s] = rmsnorm(x[rows[s]]) * w in the compute type; columns past the width are zero
+template <class T>
+__global__ __launch_bounds__(256) void norm_rows_kernel(const float* __restrict__ x, const uint32_t* __restrict__ rows,
+                                                        const float* __restrict__ w, T* __restrict__ out, int width,
+                                                        int ld, int num_rows, float eps) {
+    __shared__ float red[4];
+    const size_t s = blockIdx.x;
+    const uint32_t r = rows[s];
+    const float* xr = x + static_cast<size_t>(r < static_cast<uint32_t>(num_rows) ? r : 0) * ld;
+    float local = 0.f;
+    for (int i = threadIdx.x; i < width; i += 256) local += xr[i] * xr[i];
+    const float inv = 1.f / sqrtf(block_total(local, red) / static_cast<float>(width) + eps);
+    for (int i = threadIdx.x; i < ld; i += 256) out[s * ld + i] = i < width ? act_put<T>(xr[i] * inv * w[i]) : act_put<T>(0.f);
+}
+
+// logits f32 = cap * tanh(y * scale / cap) (cap 0: y * scale), and their argmax (the lowest index
+// among equals, NaN never wins).  One block per row.
+template <class T>
+__global__ __launch_bounds__(1024) void logits_finish_kernel(const T* __restrict__ y, float* __restrict__ logits,
+                                                             uint32_t* __restrict__ tokens, int vocab, int ldy,
+                                                             float scale, float cap) {
+    __shared__ float sv[16];
+    __shared__ int si[16];
+    const size_t s = blockIdx.x;
+    float bv = -INFINITY;
+    int bi = 0;
+    for (int i = threadIdx.x; i < vocab; i += blockDim.x) {
+        float v = act_get<T>(y[s * ldy + i]) * scale;
+        if (cap > 0.f) v = cap * tanhf(v / cap);
+        logits[s * vocab + i] = v;
+        if (v > bv) {   // (indices ascend inside a thread)
+            bv = v;
+            bi = i;
+        }
+    }
+    auto better = [&](float ov, int oi) {
+        if (ov > bv || (ov == bv && oi < bi)) {
+            bv = ov;
+            bi = oi;
+        }
+    };
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) better(__shfl_xor(bv, off, kWave), __shfl_xor(bi, off, kWave));
+    const int lane = threadIdx.x & (kWave - 1), wv = threadIdx.x / kWave;
+    if (lane == 0) {
+        sv[wv] = bv;
+        si[wv] = bi;
+    }
+    __syncthreads();
+    if (threadIdx.x == 0) {
+        for (int i = 1; i < static_cast<int>(blockDim.x) / kWave; ++i) better(sv[i], si[i]);
+        tokens[s] = static_cast<uint32_t>(bi);
+    }
+}
+
+// table[n, i] = cos(a) * mscale, table[n, half + i] = sin(a) * mscale, a = position * f_i.  The
+// angle is formed and reduced in double so that its fp32 value is right to the last bit at any
+// position.
+__global__ void rotary_table_kernel(const int32_t* __restrict__ positions, const double* __restrict__ freq,
+                                    float* __restrict__ table, int half, float mscale) {
+    const int n = blockIdx.x;
+    for (int i = threadIdx.x; i < half; i += blockDim.x) {
+        constexpr double kTwoPi = 6.283185307179586476925;
+        double a = static_cast<double>(positions[n]) * freq[i];
+        a -= rint(a / kTwoPi) * kTwoPi;
+        float s, c;
+        sincosf(static_cast<float>(a), &s, &c);
+        table[static_cast<size_t>(n) * 2 * half + i] = c * mscale;
+        table[static_cast<size_t>(n) * 2 * half + half + i] = s * mscale;
+    }
+}
+
+// y[M, N] = epilogue(act[M, K] fp32 . W[N, K]^T bf16), fp32 products and sums: 64 x 64 tiles of
+// 16-wide K steps through LDS, 4 x 4 outputs per thread.
+constexpr int kFT = 64, kFK = 16;
+__global__ __launch_bounds__(256) void linear_f32_kernel(const float* __restrict__ act, const uint16_t* __restrict__ w,
+                                                         float* __restrict__ y, int M, int N, int K, int relu2) {
+    __shared__ float as[kFK][kFT + 4];
+    __shared__ float ws[kFK][kFT + 4];
+    const int n0 = blockIdx.x * kFT, m0 = blockIdx.y * kFT;
+    const int tid = threadIdx.x, tx = tid & 15, ty = tid >> 4;
+    const int lr = tid >> 2, lk = (tid & 3) * 4;   // the row and the four k-values this thread stages
+    float acc[4][4] = {};
+    for (int k0 = 0; k0 < K; k0 += kFK) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int k = k0 + lk + e;
+            const bool kin = k < K;
+            as[lk + e][lr] = kin && m0 + lr < M ? act[static_cast<size_t>(m0 + lr) * K + k] : 0.f;
+            ws[lk + e][lr] = kin && n0 + lr < N ? bf16_bits_to_f32(w[static_cast<size_t>(n0 + lr) * K + k]) : 0.f;
+        }
+        __syncthreads();
+#pragma unroll
+        for (int k = 0; k < kFK; ++k) {
+            float a[4], b[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                a[i] = as[k][ty * 4 + i];
+                b[i] = ws[k][tx * 4 + i];
+            }
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) acc[i][j] = fmaf(a[i], b[j], acc[i][j]);
+        }
+        __syncthreads();
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int m = m0 + ty * 4 + i, n = n0 + tx * 4 + j;
+            if (m >= M || n >= N) continue;
+            float v = acc[i][j];
+            if (relu2) {
+                v = fmaxf(v, 0.f);
+                v *= v;
+            }
+            y[static_cast<size_t>(m) * N + n] = v;
+        }
+}
+
+}  // namespace
+}  // namespace pie_hip
+
+using namespace pie_hip;
+
+extern "C" int pie_hip_embed_stream(int dtype, const uint32_t* token_ids, const uint16_t* table_bf16, float* x,
+                                    void* x_act, int num_tokens, int width, int ld, int vocab, void* stream) {
+    if (!token_ids || !table_bf16 || !x || !x_act || num_tokens <= 0 || width <= 0 || ld < width || vocab <= 0)
+        return PIE_HIP_ERR_INVALID;
+    PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL(embed_stream_kernel<T>, dim3(num_tokens), dim3(256), 0,
+                                                  static_cast<hipStream_t>(stream), token_ids, table_bf16, x,
+                                                  static_cast<T*>(x_act), width, ld, vocab));
+    return launch_status();
+}
+
+extern "C" int pie_hip_norm_add(int dtype, const void* y, const float* weight, float* x, void* x_act, int rows,
+                                int width, int ldy, int ld, float eps, void* stream) {
+    if (!y || !weight || !x || !x_act || rows <= 0 || width <= 0 || ldy < width || ld < width) return PIE_HIP_ERR_INVALID;
+    if (ldy % 8 != 0 || ld % 8 != 0) return PIE_HIP_ERR_UNSUPPORTED;
+    // (few rows: wider blocks, so that a row's traffic is in flight at once)
+    if (width >= 2048)
+        PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL((norm_add_kernel<T, 1024>), dim3(rows), dim3(1024), 0,
+                                                      static_cast<hipStream_t>(stream), static_cast<const T*>(y),
+                                                      weight, x, static_cast<T*>(x_act), width, ldy, ld, eps));
+    else
+        PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL((norm_add_kernel<T, 256>), dim3(rows), dim3(256), 0,
+                                                      static_cast<hipStream_t>(stream), static_cast<const T*>(y),
+                                                      weight, x, static_cast<T*>(x_act), width, ldy, ld, eps));
+    return launch_status();
+}
+
+extern "C" int pie_hip_norm_rows(int dtype, const float* x, const uint32_t* rows, const float* weight, void* out,
+                                 int num_out, int width, int ld, int num_rows, float eps, void* stream) {
+    if (!x || !rows || !weight || !out || num_out <= 0 || width <= 0 || ld < width || num_rows <= 0)
+        return PIE_HIP_ERR_INVALID;
+    PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL(norm_rows_kernel<T>, dim3(num_out), dim3(256), 0,
+                                                  static_cast<hipStream_t>(stream), x, rows, weight,
+                                                  static_cast<T*>(out), width, ld, num_rows, eps));
+    return launch_status();
+}
+
+extern "C" int pie_hip_logits_finish(int dtype, const void* y, float* logits, uint32_t* tokens, int rows, int vocab,
+                                     int ldy, float scale, float cap, void* stream) {
+    if (!y || !logits || !tokens || rows <= 0 || vocab <= 0 || ldy < vocab) return PIE_HIP_ERR_INVALID;
+    PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL(logits_finish_kernel<T>, dim3(rows), dim3(1024), 0,
+                                                  static_cast<hipStream_t>(stream), static_cast<const T*>(y), logits,
+                                                  tokens, vocab, ldy, scale, cap));
+    return launch_status();
+}
+
+extern "C" int pie_hip_rotary_table(const int32_t* positions, const double* freq, float* table, int num_tokens,
+                                    int dims, float mscale, void* stream) {
+    if (!positions || !freq || !table || num_tokens <= 0 || dims <= 0 || dims % 2 != 0) return PIE_HIP_ERR_INVALID;
+    hipLaunchKernelGGL(rotary_table_kernel, dim3(num_tokens), dim3(64), 0, static_cast<hipStream_t>(stream), positions,
+                       freq, table, dims / 2, mscale);
+    return launch_status();
+}
+
+extern "C" int pie_hip_linear_f32(const float* act, const uint16_t* w_bf16, float* y, int M, int N, int K,
+                                  int epilogue, void* stream) {
+    if (!act || !w_bf16 || !y || M <= 0 || N <= 0 || K <= 0) return PIE_HIP_ERR_INVALID;
+    if (epilogue != PIE_HIP_EPI_NONE && epilogue != PIE_HIP_EPI_RELU2) return PIE_HIP_ERR_UNSUPPORTED;
+    const int gy = (M + kFT - 1) / kFT;
+    if (gy > 65535) return PIE_HIP_ERR_UNSUPPORTED;
+    hipLaunchKernelGGL(linear_f32_kernel, dim3((N + kFT - 1) / kFT, gy), dim3(256), 0, static_cast<hipStream_t>(stream),
+                       act, w_bf16, y, M, N, K, epilogue == PIE_HIP_EPI_RELU2 ? 1 : 0);
+    return launch_status();
+}

@@ -1107,14 +1107,17 @@ __global__ __launch_bounds__(kSampBlock) void sample_kernel(SampleArgs a) {
 // Sampled rows of the bf16 logits -> f32, BRLE logit mask applied.  bounds: per slot, the
 // cumulative ends of its runs (run j covers [bounds[j-1], bounds[j]) and allows its tokens
 // when j is odd); a slot without runs is unconstrained.
+__device__ __forceinline__ float logit_f32(uint16_t v) { return bf16_bits_to_f32(v); }
+__device__ __forceinline__ float logit_f32(float v) { return v; }
+template <class T>
 __global__ __launch_bounds__(256) void sample_gather_kernel(
-    const uint16_t* __restrict__ logits, const int32_t* __restrict__ rows, float* __restrict__ out,
+    const T* __restrict__ logits, const int32_t* __restrict__ rows, float* __restrict__ out,
     const uint32_t* __restrict__ bounds, const int32_t* __restrict__ bounds_indptr, int V) {
     const int s = blockIdx.y;
     const int v = blockIdx.x * blockDim.x + threadIdx.x;
     if (v >= V) return;
     const size_t src_row = rows ? static_cast<size_t>(rows[s]) : static_cast<size_t>(s);
-    float x = bf16_bits_to_f32(logits[src_row * V + v]);
+    float x = logit_f32(logits[src_row * V + v]);
     if (bounds_indptr) {
         const int b0 = bounds_indptr[s], b1 = bounds_indptr[s + 1];
         if (b1 > b0) {
@@ -1139,18 +1142,31 @@ extern "C" size_t pie_hip_sample_workspace_bytes(int num_slots, int vocab) {
     return static_cast<size_t>(num_slots) * vocab * 4 * sizeof(uint32_t);
 }
 
+namespace {
+template <class T>
+int gather_logits(const T* logits, const int32_t* rows, float* out_f32, const uint32_t* mask_bounds,
+                  const int32_t* mask_bounds_indptr, int num_slots, int vocab, void* stream) {
+    using namespace pie_hip;
+    if (!logits || !out_f32 || num_slots <= 0 || vocab <= 0) return PIE_HIP_ERR_INVALID;
+    if (num_slots > 65535) return PIE_HIP_ERR_UNSUPPORTED;
+    if (mask_bounds_indptr && !mask_bounds) mask_bounds_indptr = nullptr;
+    hipLaunchKernelGGL(sample_gather_kernel<T>, dim3((vocab + 255) / 256, num_slots), dim3(256), 0,
+                       static_cast<hipStream_t>(stream), logits, rows, out_f32, mask_bounds, mask_bounds_indptr, vocab);
+    return launch_status();
+}
+}  // namespace
+
 extern "C" int pie_hip_sample_gather_logits(const uint16_t* logits_bf16, const int32_t* rows,
                                             float* out_f32, const uint32_t* mask_bounds,
                                             const int32_t* mask_bounds_indptr, int num_slots,
                                             int vocab, void* stream) {
-    using namespace pie_hip;
-    if (!logits_bf16 || !out_f32 || num_slots <= 0 || vocab <= 0) return PIE_HIP_ERR_INVALID;
-    if (num_slots > 65535) return PIE_HIP_ERR_UNSUPPORTED;
-    if (mask_bounds_indptr && !mask_bounds) mask_bounds_indptr = nullptr;
-    hipLaunchKernelGGL(sample_gather_kernel, dim3((vocab + 255) / 256, num_slots), dim3(256), 0,
-                       static_cast<hipStream_t>(stream), logits_bf16, rows, out_f32, mask_bounds,
-                       mask_bounds_indptr, vocab);
-    return launch_status();
+    return gather_logits(logits_bf16, rows, out_f32, mask_bounds, mask_bounds_indptr, num_slots, vocab, stream);
+}
+
+extern "C" int pie_hip_sample_gather_logits_f32(const float* logits, const int32_t* rows, float* out_f32,
+                                                const uint32_t* mask_bounds, const int32_t* mask_bounds_indptr,
+                                                int num_slots, int vocab, void* stream) {
+    return gather_logits(logits, rows, out_f32, mask_bounds, mask_bounds_indptr, num_slots, vocab, stream);
 }
 
 extern "C" int pie_hip_sample(const float* logits_f32, const int32_t* kind, const float* temperature,

@@ -144,6 +144,8 @@ def lib() -> C.CDLL:
         l.pie_hip_driver_destroy.argtypes = [C.c_void_p]
         l.pie_hip_driver_capabilities.restype = C.c_char_p
         l.pie_hip_driver_capabilities.argtypes = [C.c_void_p]
+        l.pie_hip_driver_last_error.restype = C.c_char_p
+        l.pie_hip_driver_last_error.argtypes = [C.c_void_p]
         l.pie_hip_driver_handle.argtypes = [C.c_void_p, C.POINTER(FrameDesc), C.POINTER(ResponseFrameDesc)]
         l.pie_hip_driver_generate.argtypes = [C.c_void_p, C.c_void_p, C.c_int, C.c_int, C.c_int,
                                               C.c_int, C.c_void_p, C.c_void_p, C.c_char_p, C.c_size_t]
@@ -176,7 +178,7 @@ class ForwardFrame:
                  context_ids=None, masks: Optional[Sequence[Sequence[int]]] = None,
                  driver_id: int = 0, logit_masks: Optional[Sequence[Sequence[int]]] = None,
                  logit_mask_indptr=None, spec_token_ids=None, spec_position_ids=None,
-                 spec_indptr=None):
+                 spec_indptr=None, rs_slot_ids=None, rs_slot_flags=None):
         R = len(qo_indptr) - 1
         self._keep = []
 
@@ -243,6 +245,12 @@ class ForwardFrame:
             f.spec_token_ids = u32(spec_token_ids)
             f.spec_position_ids = u32(spec_position_ids)
             f.spec_indptr = u32(spec_indptr)
+        if rs_slot_ids is not None:   # recurrent-state slot of each request
+            f.rs_slot_ids = u32(rs_slot_ids)
+        if rs_slot_flags is not None:
+            fl = np.ascontiguousarray(np.asarray(rs_slot_flags, dtype=np.uint8))
+            self._keep.append(fl)
+            f.rs_slot_flags = U8Slice(fl.ctypes.data_as(C.POINTER(C.c_uint8)), fl.size)
         f.single_token_mode = 1 if len(token_ids) == R else 0
 
 
@@ -348,6 +356,10 @@ class Driver:
         import json
 
         return json.loads(lib().pie_hip_driver_capabilities(self._h).decode())
+
+    def last_error(self) -> str:
+        """Message of the last failed forward."""
+        return (lib().pie_hip_driver_last_error(self._h) or b"").decode()
 
     def handle(self, frame) -> ResponseFrameDesc:
         fr = frame.frame if isinstance(frame, ForwardFrame) else frame
