@@ -343,6 +343,75 @@ def other_configs_extra(drvmod):
     return out
 
 
+# --layer-stack: layers of a layer-stack model (latent attention, one channel-delta layer in three,
+# squared-ReLU feed-forward) beside bf16 llama-type layers of the same width, heads and feed-forward.
+STACK_SIZES = {
+    "width4096": dict(width=4096, heads=32, dim=128, rot_dim=64, vdim=128, q_rank=1536, kv_rank=512, ff=14336,
+                      kv_heads=8, vocab=32000, layers=6),
+    "width2048": dict(width=2048, heads=16, dim=128, rot_dim=64, vdim=128, q_rank=768, kv_rank=512, ff=8192,
+                      kv_heads=4, vocab=32000, layers=6),
+}
+
+
+def stack_config(z: dict) -> dict:
+    rot = dict(dims=z["rot_dim"], base=500000.0, scaling=dict(factor=4.0, original=4096, fast=32.0, slow=1.0))
+    latent = dict(type="latent_attention", mlp=dict(kind="dense", ff=z["ff"]),
+                  mixer=dict(heads=z["heads"], dim=z["dim"], rot_dim=z["rot_dim"], vdim=z["vdim"], q_rank=z["q_rank"],
+                             kv_rank=z["kv_rank"], rot=rot, scale=(z["dim"] + z["rot_dim"]) ** -0.5))
+    delta = dict(type="channel_delta", mlp=dict(kind="dense", ff=z["ff"]),
+                 mixer=dict(heads=z["heads"], kv_heads=z["heads"], dim=z["dim"], vdim=z["vdim"], conv=4))
+    layers = [delta if l % 3 == 2 else latent for l in range(z["layers"])]
+    return dict(architecture="Varasun", layers=layers, width=z["width"], vocab=z["vocab"], norm=dict(eps=1e-5),
+                logit_scale=0.5, logit_softcap=15.0)
+
+
+def stack_workload(args):
+    """Prefill and decode throughput of the layer stacks above and of the llama-type model of equal
+    size, both through the driver boundary on random bf16 weights."""
+    import tempfile
+
+    from pie_amd import driver as drvmod
+
+    n_prompt, page = args.prompt, 16
+    cases = [(1, n_prompt), (16, n_prompt), (64, n_prompt)]
+    out = {}
+    names = [args.layer_stack] if args.layer_stack != "all" else list(STACK_SIZES)
+    for name in names:
+        z = STACK_SIZES[name]
+        max_new = args.warmup + args.steps + 1
+        pages = (n_prompt + max_new + page - 1) // page * 64 + 8
+        with tempfile.TemporaryDirectory() as td:
+            (Path(td) / "config.json").write_text(json.dumps(stack_config(z)))
+            models = {
+                "varasun": dict(hf_path=td, random_weights=True, quant="bf16"),
+                "llama": dict(arch="llama3", hidden=z["width"], layers=z["layers"], q_heads=z["heads"],
+                              kv_heads=z["kv_heads"], head_dim=z["dim"], intermediate=z["ff"], vocab=z["vocab"],
+                              quant="bf16"),
+            }
+            res = {}
+            for which, model in models.items():
+                if args.layer_stack_only and which != args.layer_stack_only:
+                    continue
+                drv = drvmod.Driver(toml(model, page, pages, 2048, 64))
+                try:
+                    rng = np.random.default_rng(5)
+                    prompt = rng.integers(0, z["vocab"], n_prompt)
+                    drv.set_generate_divergence(7919)
+                    drv.generate(prompt, 2)
+                    prefill = min(drv.generate(prompt, 1)[1]["prefill_us"] for _ in range(5)) * 1e-6
+                    r = dict(prefill_tokens_per_s=round(n_prompt / prefill, 1), prefill_ms=round(prefill * 1e3, 3))
+                    for batch, _ in cases:
+                        _, tm = drv.generate(prompt, max_new, replicate=batch, warmup=args.warmup)
+                        wall = tm["decode_wall_us"] * 1e-6 / tm["decode_steps"]
+                        r[f"decode_batch{batch}"] = dict(tokens_per_s=round(batch / wall, 1), ms_per_step=round(wall * 1e3, 4))
+                    res[which] = r
+                finally:
+                    drv.close()
+            out[name] = dict(sizes=z, **res)
+    print(json.dumps({"layer_stack": out, "prompt_tokens": n_prompt, "steps": args.steps, "warmup": args.warmup,
+                      "dtype": "bf16", "data": "synthetic (random weights)"}))
+
+
 def lm_head_extra(drv, model):
     import torch
 
@@ -516,6 +585,11 @@ def main():
     ap.add_argument("--pmc-workload", action="store_true",
                     help="only launch what a `rocprofv3 --pmc FETCH_SIZE|WRITE_SIZE` run needs: a "
                          "256 MiB device copy (the counter's scale) and the four int4 GEMV shapes")
+    ap.add_argument("--layer-stack", default=None, choices=["all", *STACK_SIZES],
+                    help="measure layer-stack models (prefill and decode at batch 1, 16, 64) beside the llama-type "
+                         "model of equal size instead of the headline workload")
+    ap.add_argument("--layer-stack-only", default=None, choices=["varasun", "llama"],
+                    help="with --layer-stack: only this side (for profiles)")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this driver path is built and measured on one GPU; "
@@ -529,6 +603,9 @@ def main():
         sys.exit(1)
     from pie_amd import driver as drvmod
 
+    if args.layer_stack:
+        stack_workload(args)
+        return
     if args.pmc_workload:
         pmc_workload()
         return

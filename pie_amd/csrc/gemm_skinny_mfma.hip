@@ -523,7 +523,9 @@ __global__ __launch_bounds__(kSwWaves* kWave, NG == 1 && MT == 1 ? 4 : 2) void s
     // (the ring runs ahead of the arithmetic, so its last trips reach past the wave's K slice:
     // those requests repeat the slice's own last block — a cache hit — instead of fetching the
     // neighbour's blocks a second time)
-    const int b_last = max(b_lo, min(nb, b_lo + nch * CB) - 1);
+    // (a wave whose slice is empty — a K of fewer chunks than its waves' shares cover — starts at nb:
+    // its requests repeat the matrix's last block)
+    const int b_last = min(nb - 1, max(b_lo, min(nb, b_lo + nch * CB) - 1));
     // Group scales: one load per block for all NG tiles — lane 16 i + j fetches tile i's scale of
     // weight row j — carried in the ring slot of the block's first tile; a tile's step reads its
     // value across the wave.  (A load per tile and step made a third of the kernel's vector-memory

@@ -369,6 +369,7 @@ __global__ __launch_bounds__(kBlock) void gemv_kernel(const GemvArgs a) {
     const int row_end = row_begin + (a.slice_q + (wgi < a.slice_r ? 1 : 0)) * gran;
     const int ngroups = (row_end - row_begin + R - 1) / R;
     const int nunits = ngroups * nchunks;
+    const int idle_row = min(row_begin, N - gran);   // what units past the slice re-read (an empty slice starts at N)
 
     // Branch-free loads: lanes past K re-read lane 0's piece and are masked out in compute;
     // rows past the slice re-read its last row and are dropped at the store.
@@ -389,7 +390,7 @@ __global__ __launch_bounds__(kBlock) void gemv_kernel(const GemvArgs a) {
             gidx = (valid && live) ? (a.g_shift >= 0 ? kbase >> a.g_shift : kbase / a.G) : 0;
 #pragma unroll
         for (int r = 0; r < R; ++r) {
-            const int row = live ? min(row_begin + g * R + r, row_end - 1) : row_begin;
+            const int row = live ? min(row_begin + g * R + r, row_end - 1) : idle_row;
             u.w[r] = __builtin_nontemporal_load(a.w + static_cast<size_t>(row) * row_stride_v4 +
                                                 piece);
             if constexpr (F::kGroupScale && !one_gs)
@@ -398,7 +399,7 @@ __global__ __launch_bounds__(kBlock) void gemv_kernel(const GemvArgs a) {
         if constexpr (one_gs) {
             {
                 const int lr = min(lane >> gpc_shift, R - 1);
-                const int row = live ? min(row_begin + g * R + lr, row_end - 1) : row_begin;
+                const int row = live ? min(row_begin + g * R + lr, row_end - 1) : idle_row;
                 const int grp = live ? min(((c * kChunkK) >> a.g_shift) + (lane & ((1 << gpc_shift) - 1)), groups_per_row - 1) : 0;
                 u.gsv = a.gscale[static_cast<size_t>(row) * groups_per_row + grp];
             }
@@ -411,7 +412,7 @@ __global__ __launch_bounds__(kBlock) void gemv_kernel(const GemvArgs a) {
         const int li = lane < per ? lane / M : 0;
         const int lm = lane < per ? lane % M : 0;
         // (a wave whose slice is empty has no live unit: row_end - 1 may be -1 there)
-        const int lrow = !live ? row_begin
+        const int lrow = !live ? idle_row
                          : pairs ? min(row_begin + g * R + 2 * li, row_end - 2)
                                  : min(row_begin + g * R + li, row_end - 1);
         u.prev = a.y[pairs ? 0 : static_cast<size_t>(lm) * N + lrow];

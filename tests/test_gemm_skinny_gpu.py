@@ -33,6 +33,21 @@ def test_skinny_matches_oracle(gpu, oracle, kind, M, N, K):
 
 
 @pytest.mark.parametrize("kind", KINDS)
+@pytest.mark.parametrize("M,N,K", [(16, 6144, 1536), (5, 1600, 2560), (40, 6144, 1536)])
+def test_tile_major_weights_whose_k_chunks_do_not_fill_the_waves(gpu, oracle, kind, M, N, K):
+    """Six (ten) K chunks over four (eight) waves of a tile group: the last shares are empty and must
+    not reach past the matrix."""
+    import torch
+    from pie_amd import ops
+
+    rng = np.random.default_rng(330 + M)
+    wd, mk = make_weight(oracle, rng, kind, N, K)
+    x = oracle.f32_to_bf16(rng.standard_normal((M, K)).astype(np.float32))
+    got = bits(ops.gemm_skinny(dev(x, gpu, torch.bfloat16), ops.repack_mfma_tiles(mk(gpu))))
+    assert close_to_oracle(oracle, got, oracle_linear(oracle, wd, x))
+
+
+@pytest.mark.parametrize("kind", KINDS)
 def test_skinny_equals_gemv_path_rowwise(gpu, oracle, kind):
     """Same contract as the GEMV: every activation row gives the value the GEMV gives for it
     (sum order differs, so within one bf16 step on almost all elements)."""
