@@ -807,7 +807,7 @@ int pie_hip_linear_f32(const float* act, const uint16_t* w_bf16, float* y, int M
  *   cache row = the normed latent and the key values rotated in adjacent pairs (first rot_dims of
  *   them, table of pie_hip_rotary_table).
  * pie_hip_head_linear: y[n, h, c] = sum_k W[h, c, k] act[n, h, k] (heads act_stride / y_stride
- *   apart in rows of ld_act / ld_y; C % 16 == 0, K % 32 == 0).  With rope_table also
+ *   apart in rows of ld_act / ld_y; C % 16 == 0, K % 32 == 0).  With rotp > 0 also
  *   y[n, h, C + i] = the rotated act[n, h, rot_off + i], i < rot_dim, zeros to rotp.
  * pie_hip_latent_attn_rows_plain: o[n, h, :] = softmax_j(q[n, h, :] . row_j * scale) . row_j[:kvp]
  *   over the first row_kv_len[n] keys; q [rows, heads, ld_row], o [rows, heads, kvp].  Any sizes
@@ -824,6 +824,35 @@ int pie_hip_latent_attn_rows_plain(int dtype, const void* q, const void* pool, v
                                    const uint32_t* kv_page_indices, const uint32_t* row_page_begin,
                                    const int32_t* row_kv_len, int num_rows, int heads, int kvp, int ld_row,
                                    int page_size, float scale, void* stream);
+
+/* The same function on the matrix cores over bf16 pools, rows [row0, row0 + num_rows): weights
+ * enter the second product as hi + lo bf16 pairs.  rotp in {32, 64}, kvp in {64, 128, 192, 256, 384,
+ * 512} (pie_hip_latent_attn_rows_supported), page_size % 16 == 0.  max_tokens_per_req: the most
+ * rows a request brings (1: a decode batch; more: row_req / qo_indptr must cover the rows, whole
+ * requests only).  workspace: pie_hip_latent_attn_rows_workspace_bytes. */
+int pie_hip_latent_attn_rows_supported(int kvp, int rotp);
+size_t pie_hip_latent_attn_rows_workspace_bytes(int num_rows, int heads, int kvp, int max_kv_len,
+                                                int max_tokens_per_req);
+int pie_hip_latent_attn_rows(const uint16_t* q, const uint16_t* pool, uint16_t* o, const uint32_t* kv_page_indices,
+                             const uint32_t* row_page_begin, const int32_t* row_kv_len, const int32_t* row_req,
+                             const int32_t* qo_indptr, int row0, int num_rows, int heads, int kvp, int rotp,
+                             int page_size, float scale, int max_kv_len, int max_tokens_per_req, void* workspace,
+                             size_t workspace_bytes, void* stream);
+/* Long portions: keys and values projected out of the latents, then ordinary causal attention.
+ * pie_hip_latent_gather: the first num_keys cache rows of a page list as compact rows, lat [num_keys,
+ *   kvp] and rot [num_keys, rotp].
+ * pie_hip_latent_attn_prefill: rows [row0, row0 + num_rows) of one request, q [rows, heads, dimp +
+ *   rotp] (the rotated part not yet rotated: rope_table rows as for pie_hip_latent_prep), kv
+ *   [num_keys, heads, dimp + vdp] the projected keys and values, rot as gathered; row n sees its
+ *   first row_kv_len[n] keys; o [rows, ld_o], heads vdp apart.  (dimp + rotp) / 32 in 2..6, vdp / 32
+ *   in 1..4 (pie_hip_latent_attn_prefill_supported). */
+int pie_hip_latent_gather(const uint16_t* pool, const uint32_t* pages, uint16_t* lat, uint16_t* rot, int num_keys,
+                          int kvp, int rotp, int page_size, void* stream);
+int pie_hip_latent_attn_prefill_supported(int dimp, int rotp, int vdp);
+int pie_hip_latent_attn_prefill(const uint16_t* q, const uint16_t* kv, const uint16_t* rot, uint16_t* o,
+                                const float* rope_table, const int32_t* row_kv_len, int row0, int num_rows,
+                                int num_keys, int heads, int dimp, int rotp, int rot_dims, int vdp, int ld_o,
+                                float scale, void* stream);
 
 /*
  * Gated delta rule with a decay per head and key channel.  row_req [N]: request of each row;

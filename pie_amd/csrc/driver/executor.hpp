@@ -213,6 +213,8 @@ class Executor {
     // query-row tiles of the current forward for the matrix-core prefill attention (0 = per-row kernel)
     Growable tile_in_host_, tile_in_dev_;
     int n_tiles_ = 0, tile_rows_ = 0;
+    // keys and values projected out of cached latents (the longest portion so far)
+    Growable expand_lat_, expand_rot_, expand_kv_;
     // custom attention masks of the current forward (never part of a captured graph)
     Growable mask_in_host_, mask_in_dev_, mask_bitmap_;
     int mask_stride_ = 0;

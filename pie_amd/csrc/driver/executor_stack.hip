@@ -110,6 +110,15 @@ void Executor::alloc_stack() {
                     gemm_ws_bytes_ = std::max(gemm_ws_bytes_, pie_hip_gemm_mfma_workspace_bytes(rows, w->N, w->K));
     gemm_ws_bytes_ = std::min<size_t>(gemm_ws_bytes_, size_t(64) << 20);
     if (gemm_ws_bytes_) PIE_HIP_CHECK(hipMalloc(&gemm_ws_, gemm_ws_bytes_));
+    // partial results of the latent attention's splits: a plan with more than one split has at most
+    // 512 (tile, split) blocks of 32 (token, head) pairs
+    if (o_lat && !m.f32()) {
+        size_t kvp = 0;
+        for (const StackLayer& l : model_.stack)
+            if (l.spec.mixer == MixerKind::LatentAttention) up(kvp, LatentShape(l.spec.latent).kvp);
+        attn_ws_bytes_ = 512 * 32 * (kvp + 2) * sizeof(float);
+        PIE_HIP_CHECK(hipMalloc(&attn_ws_, attn_ws_bytes_));
+    }
     rs_stride_ = state;
     if (state) {
         rs_slots_ = cfg_.batching.rs_cache_slots;
@@ -226,20 +235,74 @@ void Executor::stack_latent(const StackLayer& w, int layer, int N, int max_kv_le
     const auto* row_len = reinterpret_cast<const int32_t*>(in_dev_ + in.off_row_len);
     const auto* pages = reinterpret_cast<const uint32_t*>(in_dev_ + in.off_pages);
     const float* rope = w.rotary >= 0 ? stack_.rotary[static_cast<size_t>(w.rotary)] : nullptr;
-    (void)max_kv_len;
     stack_linear(w.w_in, stack_.xa, stack_.in, N);
     PIE_KERNEL(pie_hip_latent_prep(dt_, stack_.in, w.q_norm, w.kv_norm, rope, slots, stack_.cq, latent_pool_[layer], N,
                                    s.ld_in, s.kv_off, a.q_rank, s.ld_cq, a.kv_rank, s.kvp, a.rot_dim, a.rot.dims,
                                    s.ld_row, model_.cfg().rms_eps, stream_));
     stack_linear(w.w_uq, stack_.cq, stack_.q, N);
-    PIE_KERNEL(pie_hip_head_linear(dt_, stack_.q, w.w_uk_t, stack_.q_lat, s.rotp ? rope : nullptr, N, s.heads, s.kvp,
-                                   s.dimp, s.ld_q, s.hd, s.heads * s.ld_row, s.ld_row, s.dimp, a.rot_dim, a.rot.dims,
-                                   s.rotp, stream_));
-    PIE_KERNEL(pie_hip_latent_attn_rows_plain(dt_, stack_.q_lat, latent_pool_[layer], stack_.o_lat, pages, row_begin,
-                                              row_len, N, s.heads, s.kvp, s.ld_row, page_size_,
-                                              static_cast<float>(a.scale), stream_));
-    PIE_KERNEL(pie_hip_head_linear(dt_, stack_.o_lat, w.w_uv, stack_.o, nullptr, N, s.heads, s.vdp, s.kvp,
-                                   s.heads * s.kvp, s.kvp, s.ld_o, s.vdp, 0, 0, 0, 0, stream_));
+
+    const size_t esize = dt_ == PIE_HIP_DT_F32 ? 4 : 2;
+    auto rows_of = [&](void* buf, int row, int ld) { return static_cast<unsigned char*>(buf) + static_cast<size_t>(row) * ld * esize; };
+    const bool matrix = dt_ == PIE_HIP_DT_BF16 && pie_hip_latent_attn_rows_supported(s.kvp, s.rotp);
+    // rows [r0, r0 + n): through the latent space
+    auto rows_form = [&](int r0, int n, int max_len, int max_tokens) {
+        if (n <= 0) return;
+        PIE_KERNEL(pie_hip_head_linear(dt_, rows_of(stack_.q, r0, s.ld_q), w.w_uk_t, rows_of(stack_.q_lat, r0, s.heads * s.ld_row),
+                                       rope ? rope + static_cast<size_t>(r0) * a.rot.dims : nullptr, n, s.heads, s.kvp, s.dimp,
+                                       s.ld_q, s.hd, s.heads * s.ld_row, s.ld_row, s.dimp, a.rot_dim, a.rot.dims, s.rotp, stream_));
+        if (matrix)
+            PIE_KERNEL(pie_hip_latent_attn_rows(static_cast<const uint16_t*>(stack_.q_lat),
+                                                reinterpret_cast<const uint16_t*>(latent_pool_[layer]),
+                                                static_cast<uint16_t*>(stack_.o_lat), pages, row_begin, row_len,
+                                                reinterpret_cast<const int32_t*>(in_dev_ + in.off_row_req),
+                                                reinterpret_cast<const int32_t*>(in_dev_ + in.off_qo), r0, n, s.heads, s.kvp,
+                                                s.rotp, page_size_, static_cast<float>(a.scale), max_len, max_tokens, attn_ws_,
+                                                attn_ws_bytes_, stream_));
+        else
+            PIE_KERNEL(pie_hip_latent_attn_rows_plain(dt_, rows_of(stack_.q_lat, r0, s.heads * s.ld_row), latent_pool_[layer],
+                                                      rows_of(stack_.o_lat, r0, s.heads * s.kvp), pages, row_begin + r0, row_len + r0, n,
+                                                      s.heads, s.kvp, s.ld_row, page_size_, static_cast<float>(a.scale), stream_));
+        PIE_KERNEL(pie_hip_head_linear(dt_, rows_of(stack_.o_lat, r0, s.heads * s.kvp), w.w_uv, rows_of(stack_.o, r0, s.ld_o), nullptr, n,
+                                       s.heads, s.vdp, s.kvp, s.heads * s.kvp, s.kvp, s.ld_o, s.vdp, 0, 0, 0, 0, stream_));
+    };
+    if (plan_->pure_decode) {
+        rows_form(0, N, max_kv_len, 1);
+    } else {
+        // Portions long enough take the expanded form: projecting `ctx` keys and values costs
+        // ctx kv_rank (dim + vdim) per head, what it saves per query and key is
+        // 2 kv_rank - (dim + vdim).
+        const int per_key = s.dimp + s.vdp, saved = 2 * s.kvp - per_key;
+        const bool can_expand = dt_ == PIE_HIP_DT_BF16 && saved > 0 && pie_hip_latent_attn_prefill_supported(s.dimp, s.rotp, s.vdp);
+        const int expand_min = can_expand ? std::max(64, static_cast<int>(static_cast<long long>(s.kvp) * per_key / saved)) : 0;
+        int run0 = 0, run_len = 0, run_tokens = 1;   // requests of the rows form, launched together
+        for (int r = 0; r < plan_->R; ++r) {
+            const int q0 = plan_->qo_indptr[r], q1 = plan_->qo_indptr[r + 1];
+            if (!can_expand || q1 - q0 < expand_min) {
+                run_len = std::max(run_len, plan_->row_kv_len[q1 - 1]);
+                run_tokens = std::max(run_tokens, q1 - q0);
+                continue;
+            }
+            rows_form(run0, q0 - run0, run_len, run_tokens);
+            run0 = q1;
+            run_len = 0;
+            run_tokens = 1;
+            const int ctx = plan_->row_kv_len[q1 - 1];
+            expand_lat_.ensure(static_cast<size_t>(ctx) * s.kvp * 2);
+            expand_rot_.ensure(static_cast<size_t>(ctx) * s.rotp * 2);
+            expand_kv_.ensure(static_cast<size_t>(ctx) * w.w_ukv.N * 2);
+            auto* lat = static_cast<uint16_t*>(expand_lat_.ptr);
+            auto* rot = static_cast<uint16_t*>(expand_rot_.ptr);
+            auto* kv = static_cast<uint16_t*>(expand_kv_.ptr);
+            PIE_KERNEL(pie_hip_latent_gather(reinterpret_cast<const uint16_t*>(latent_pool_[layer]),
+                                             pages + plan_->row_page_begin[q0], lat, rot, ctx, s.kvp, s.rotp, page_size_, stream_));
+            PIE_KERNEL(pie_hip_gemm_mfma(PIE_HIP_FMT_BF16, lat, w.w_ukv.data, nullptr, 0, 0, kv, ctx, w.w_ukv.N, w.w_ukv.K, 0,
+                                         PIE_HIP_EPI_NONE, stream_));
+            PIE_KERNEL(pie_hip_latent_attn_prefill(static_cast<const uint16_t*>(stack_.q), kv, rot, static_cast<uint16_t*>(stack_.o),
+                                                   rope, row_len, q0, q1 - q0, ctx, s.heads, s.dimp, s.rotp, a.rot.dims, s.vdp,
+                                                   s.ld_o, static_cast<float>(a.scale), stream_));
+        }
+        rows_form(run0, N - run0, run_len, run_tokens);
+    }
     stack_linear(w.wo, stack_.o, stack_.y, N);
 }
 

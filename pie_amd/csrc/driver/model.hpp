@@ -69,6 +69,10 @@ struct LayerWeights {
 // a product are rounded up so that every product takes the matrix-core kernels (zero columns in
 // the weights, zero or ignored entries in the rows).
 constexpr int pad_to(int v, int a) { return (v + a - 1) / a * a; }
+// (the latent ranks the matrix-core attention is built for; wider ones take the plain kernel)
+constexpr int pad_latent(int v) {
+    return v <= 256 ? pad_to(v, 64) : v <= 512 ? pad_to(v, 128) : pad_to(v, 64);
+}
 struct LatentShape {
     int heads, dimp, rotp, vdp, kvp;   // per-head sizes and the latent, rounded up
     int kv_off, ld_in;                 // fused down projection: query latent | (kv_off) latent, rotated key part
@@ -76,8 +80,8 @@ struct LatentShape {
     int ld_row;                        // cache row: [kvp | rotp]
     int ld_o;                          // attention output rows: heads of vdp
     explicit LatentShape(const LatentAttentionSpec& a)
-        : heads(a.heads), dimp(pad_to(a.dim, 32)), rotp(pad_to(a.rot_dim, 32)), vdp(pad_to(a.vdim, 32)),
-          kvp(pad_to(a.kv_rank, 64)), kv_off(pad_to(a.q_rank, 16)), ld_in(pad_to(kv_off + a.kv_rank + a.rot_dim, 16)),
+        : heads(a.heads), dimp(pad_to(a.dim, 32)), rotp(a.rot_dim > 0 ? pad_to(a.rot_dim, 32) : 32), vdp(pad_to(a.vdim, 32)),
+          kvp(pad_latent(a.kv_rank)), kv_off(pad_to(a.q_rank, 16)), ld_in(pad_to(kv_off + a.kv_rank + a.rot_dim, 16)),
           ld_cq(pad_to(a.q_rank, 128)), hd(dimp + rotp), ld_q(heads * hd), ld_row(kvp + rotp),
           ld_o(pad_to(heads * vdp, 128)) {}
 };

@@ -5,10 +5,10 @@
 // Two forms of the same function read it:
 //   rows form      the key projection is moved to the query side, q~ = W_uk^T q: the scores are
 //                  q~ . row and the weighted sum of the rows' latent parts goes through W_uv once
-//                  per query.  Reads each cached row once per (token, head group); decode and
+//                  per query (latent_attention_mfma.hip, any sizes here).  Reads each cached row once per (token, head group); decode and
 //                  short portions.
 //   expanded form  keys and values of all cached tokens are projected out of the latents first,
-//                  then ordinary attention runs on them (latent_attention_mfma.hip); long
+//                  then ordinary attention runs on them (latent_attention_prefill.hip); long
 //                  portions, where it needs a third of the arithmetic.
 #include "act_type.hip.h"
 
@@ -72,13 +72,13 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
 
 // y[n, h, :] = W[h] . act[n, h, :] for per-head matrices W [heads, C, K] bf16 (C, K multiples of
 // 16 and 32; act rows of `ld_act`, heads `act_stride` apart): the query's way into the latent
-// space and the latent sum's way out of it.  With rot_src the launch's last blocks along x copy the
+// space and the latent sum's way out of it.  With rotp > 0 the launch's last blocks along x write the
 // rotated part of the query: y[n, h, C + i] = rotated(act[n, h, rot_off + i]), zeros past rot_dim.
 struct HeadArgs {
     const void* act;
     const uint16_t* w;
     void* y;
-    const float* rope_table;   // null: no rotated part
+    const float* rope_table;   // (used when rotp > 0 and rot_dims > 0)
     int M, heads, C, K, ld_act, act_stride, ld_y, y_stride;
     int rot_off, rot_dim, rot_dims, rotp;
 };
@@ -105,7 +105,7 @@ __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const HeadArgs a)
     const int h = blockIdx.y, m0 = blockIdx.z * 16 * MT;
     const int lane = threadIdx.x & (kWave - 1), wv = threadIdx.x / kWave;
     const int l16 = lane & 15, g = lane >> 4;
-    if (a.rope_table && blockIdx.x == gridDim.x - 1) {
+    if (a.rotp > 0 && blockIdx.x == gridDim.x - 1) {
         head_rotated_part<uint16_t>(a, h, m0, min(m0 + 16 * MT, a.M));
         return;
     }
@@ -120,13 +120,24 @@ __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const HeadArgs a)
     f32x4_t acc[MT];
 #pragma unroll
     for (int t = 0; t < MT; ++t) acc[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-    for (int k = 0; k < a.K; k += 32) {
-        const bf16x8_t wf = __builtin_bit_cast(bf16x8_t, *reinterpret_cast<const u32x4_t*>(wp + k));
+    // (four k-steps requested together; past K a request repeats the last step and is not multiplied)
+    constexpr int U = 4;
+    for (int k0 = 0; k0 < a.K; k0 += 32 * U) {
+        u32x4_t wf[U], af[U][MT];
 #pragma unroll
-        for (int t = 0; t < MT; ++t) {
-            const bf16x8_t af = __builtin_bit_cast(bf16x8_t, *reinterpret_cast<const u32x4_t*>(ap[t] + k));
-            acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, af, acc[t], 0, 0, 0);
+        for (int u = 0; u < U; ++u) {
+            const int k = min(k0 + 32 * u, a.K - 32);
+            wf[u] = *reinterpret_cast<const u32x4_t*>(wp + k);
+#pragma unroll
+            for (int t = 0; t < MT; ++t) af[u][t] = *reinterpret_cast<const u32x4_t*>(ap[t] + k);
+        }
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            if (k0 + 32 * u >= a.K) break;
+#pragma unroll
+            for (int t = 0; t < MT; ++t)
+                acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, wf[u]),
+                                                                 __builtin_bit_cast(bf16x8_t, af[u][t]), acc[t], 0, 0, 0);
         }
     }
 #pragma unroll
@@ -157,7 +168,7 @@ __global__ __launch_bounds__(256) void head_linear_f32_kernel(const HeadArgs a) 
         }
         dst[c] = acc;
     }
-    if (a.rope_table) head_rotated_part<float>(a, h, m, m + 1);
+    if (a.rotp > 0) head_rotated_part<float>(a, h, m, m + 1);
 }
 
 // The rows form of the attention, any sizes and either compute type: one block per (head, row),
@@ -261,7 +272,7 @@ extern "C" int pie_hip_head_linear(int dtype, const void* act, const uint16_t* w
     if (C % 16 != 0 || K % 32 != 0 || ld_act % 8 != 0 || act_stride % 8 != 0 || ld_y % 8 != 0 || y_stride % 8 != 0)
         return PIE_HIP_ERR_UNSUPPORTED;
     if (ld_act < (heads - 1) * act_stride + K || ld_y < (heads - 1) * y_stride + C) return PIE_HIP_ERR_INVALID;
-    if (rope_table && (rot_dims > rot_dim || rot_dims % 2 != 0 || rotp < rot_dim || y_stride < C + rotp ||
+    if (rotp > 0 && ((rot_dims > 0 && !rope_table) || rot_dims > rot_dim || rot_dims % 2 != 0 || rotp < rot_dim || y_stride < C + rotp ||
                        act_stride < rot_off + rot_dim))
         return PIE_HIP_ERR_INVALID;
     const HeadArgs a{act, w_bf16, y, rope_table, M, heads, C, K, ld_act, act_stride, ld_y, y_stride, rot_off, rot_dim,
@@ -273,7 +284,7 @@ extern "C" int pie_hip_head_linear(int dtype, const void* act, const uint16_t* w
         return launch_status();
     }
     if (dtype != PIE_HIP_DT_BF16) return PIE_HIP_ERR_INVALID;
-    const int gx = (C + 63) / 64 + (rope_table ? 1 : 0);
+    const int gx = (C + 63) / 64 + (rotp > 0 ? 1 : 0);
     const int mt = M <= 16 ? 1 : M <= 32 ? 2 : 4;
     const int gz = (M + 16 * mt - 1) / (16 * mt);
     if (gz > 65535) return PIE_HIP_ERR_UNSUPPORTED;
