@@ -860,34 +860,55 @@ int pie_hip_latent_attn_prefill(const uint16_t* q, const uint16_t* kv, const uin
  * rs_stride bytes); rs_fresh [R]: 1 = starts from zero.  The fp32 state [heads, dim, vdim] sits at
  * state_offset of the slot, the last taps - 1 convolution inputs [taps - 1, channels] (compute type,
  * channels = q | k | v) at conv_offset.
- * pie_hip_delta_prep: fused[n] = [q | k | v | step sizes (heads) | .. decay_off: decay_rank | ..
- *   gate_off: gate_rank].  q, k: causal convolution (conv_w [channels, taps], the last column is the
- *   current token's), silu, unit vector x / sqrt(sum x^2 + 1e-6) per head, q also times dim^-1/2;
- *   v: convolution, silu; beta = sigmoid(step size); a1, g1: the low-rank inputs, compact, zero
- *   padded.  dim <= 512.
- * pie_hip_delta_decay: g = exp(-exp(a_log[head]) * softplus(raw + dt_bias)), [N, heads * dim].
- * pie_hip_delta_scan: per token S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q; head h
- *   uses q / k head h / (heads / kv_heads).  Reads and writes the state.  dim <= 256.
- * pie_hip_delta_out: y = o / sqrt(mean(o^2) + eps) * norm_w * sigmoid(gate) per head; writes the
- *   convolution state.
+ * pie_hip_delta_prep: fused[n] = [q | k | v | step sizes (heads) | ..].  q, k: causal convolution
+ *   (conv_w [channels, taps], the last column is the current token's), silu, unit vector
+ *   x / sqrt(sum x^2 + 1e-6) per head, q also times dim^-1/2; v: convolution, silu; beta =
+ *   sigmoid(step size).  dim <= 512.
+ * pie_hip_delta_conv_state: the last taps - 1 convolution inputs of every request (after prep).
+ * pie_hip_delta_lowrank: fused[n] also holds the low-rank inputs a1 (decay_off, decay_rank) and g1
+ *   (gate_off, gate_rank); log2_decay = -exp(a_log[head]) softplus(w_decay a1 + dt_bias) log2(e),
+ *   [N, heads * dim] fp32; gate = w_gate g1, [N, ld_gate] compute type.  Weights [.., ld_a1], [..,
+ *   ld_g1], zero past the ranks.
+ * pie_hip_delta_scan: per token S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q with g =
+ *   2^log2_decay; head h uses q / k head h / (heads / kv_heads).  Reads and writes the state.
+ *   dim <= 256.
+ * pie_hip_delta_chunked: the same recurrence sixteen tokens at a time on the fp32 matrix
+ *   instructions.  chunks [num_chunks][2] = (first row, rows <= 16), a request's in order;
+ *   req_chunks [R + 1].  dim <= 256; workspace pie_hip_delta_chunked_workspace_bytes.
+ * pie_hip_delta_out: y = o / sqrt(mean(o^2) + eps) * norm_w * sigmoid(gate) per head.
+ * pie_hip_delta_step: prep, scan and out for one token per request (row r = request r) in one launch;
+ *   write_conv (heads == kv_heads only) moves the convolution's state on too.  vdim a multiple of 4,
+ *   dim and vdim <= 256 (pie_hip_delta_step_supported).
  */
 int pie_hip_delta_prep(int dtype, const void* fused, const float* conv_w, const void* rs_base, size_t rs_stride,
                        size_t conv_offset, const int32_t* row_req, const int32_t* qo_indptr,
                        const int32_t* rs_slot, const int32_t* rs_fresh, float* q, float* k, float* v, float* beta,
-                       void* a1, void* g1, int num_tokens, int ld, int heads, int kv_heads, int dim, int vdim,
-                       int taps, int decay_off, int decay_rank, int ld_a1, int gate_off, int gate_rank, int ld_g1,
-                       void* stream);
-int pie_hip_delta_decay(int dtype, const void* raw, const float* a_log, const float* dt_bias, float* g,
-                        int num_tokens, int ld_raw, int heads, int dim, void* stream);
-int pie_hip_delta_scan(const float* q, const float* k, const float* v, const float* g, const float* beta, float* o,
-                       void* rs_base, size_t rs_stride, size_t state_offset, const int32_t* qo_indptr,
+                       int num_tokens, int ld, int heads, int kv_heads, int dim, int vdim, int taps, void* stream);
+int pie_hip_delta_conv_state(int dtype, const void* fused, void* rs_base, size_t rs_stride, size_t conv_offset,
+                             const int32_t* qo_indptr, const int32_t* rs_slot, const int32_t* rs_fresh,
+                             int num_requests, int ld, int channels, int taps, void* stream);
+int pie_hip_delta_lowrank(int dtype, const void* fused, const uint16_t* w_decay, const uint16_t* w_gate,
+                          const float* a_log, const float* dt_bias, float* log2_decay, void* gate, int num_tokens,
+                          int ld, int decay_off, int decay_rank, int ld_a1, int gate_off, int gate_rank, int ld_g1,
+                          int heads, int dim, int vdim, int ld_gate, void* stream);
+int pie_hip_delta_scan(const float* q, const float* k, const float* v, const float* log2_decay, const float* beta,
+                       float* o, void* rs_base, size_t rs_stride, size_t state_offset, const int32_t* qo_indptr,
                        const int32_t* rs_slot, const int32_t* rs_fresh, int num_requests, int heads, int kv_heads,
                        int dim, int vdim, void* stream);
-int pie_hip_delta_out(int dtype, const float* o, const void* gate, const float* norm_w, void* y, const void* fused,
-                      void* rs_base, size_t rs_stride, size_t conv_offset, const int32_t* row_req,
-                      const int32_t* qo_indptr, const int32_t* rs_slot, const int32_t* rs_fresh, int num_tokens,
-                      int ld_gate, int ld_y, int ld_fused, int heads, int kv_heads, int dim, int vdim, int taps,
-                      float eps, void* stream);
+size_t pie_hip_delta_chunked_workspace_bytes(int num_chunks, int heads, int dim);
+int pie_hip_delta_chunked(const float* q, const float* k, const float* v, const float* log2_decay, const float* beta,
+                          float* o, void* rs_base, size_t rs_stride, size_t state_offset, const int32_t* chunks,
+                          const int32_t* req_chunks, const int32_t* rs_slot, const int32_t* rs_fresh, int num_chunks,
+                          int num_requests, int heads, int kv_heads, int dim, int vdim, void* workspace,
+                          size_t workspace_bytes, void* stream);
+int pie_hip_delta_out(int dtype, const float* o, const void* gate, const float* norm_w, void* y, int num_tokens,
+                      int ld_gate, int ld_y, int heads, int vdim, float eps, void* stream);
+int pie_hip_delta_step_supported(int dim, int vdim);
+int pie_hip_delta_step(int dtype, const void* fused, const float* conv_w, const float* log2_decay, const void* gate,
+                       const float* norm_w, void* y, void* rs_base, size_t rs_stride, size_t state_offset,
+                       size_t conv_offset, const int32_t* rs_slot, const int32_t* rs_fresh, int num_requests, int ld,
+                       int ld_gate, int ld_y, int heads, int kv_heads, int dim, int vdim, int taps, int write_conv,
+                       float eps, void* stream);
 
 /* pie_hip_sample_gather_logits over fp32 logits. */
 int pie_hip_sample_gather_logits_f32(const float* logits, const int32_t* rows, float* out_f32,

@@ -321,7 +321,7 @@ Executor::~Executor() {
     if (kv_shadow_k_) (void)hipFree(kv_shadow_k_);
     if (kv_shadow_v_) (void)hipFree(kv_shadow_v_);
     for (Growable* g : {&mask_in_host_, &mask_in_dev_, &mask_bitmap_, &tile_in_host_, &tile_in_dev_, &expand_lat_, &expand_rot_,
-                        &expand_kv_}) g->release();
+                        &expand_kv_, &chunk_host_, &chunk_dev_, &delta_ws_}) g->release();
     for (Growable* g : {&samp_f32_, &samp_ws_, &samp_in_dev_, &samp_in_host_, &samp_out_dev_, &samp_out_host_})
         g->release();
     if (swap_pool_) (void)hipHostFree(swap_pool_);

@@ -215,6 +215,9 @@ class Executor {
     int n_tiles_ = 0, tile_rows_ = 0;
     // keys and values projected out of cached latents (the longest portion so far)
     Growable expand_lat_, expand_rot_, expand_kv_;
+    // delta rule over portions: the step's chunks and the chunk records
+    Growable chunk_host_, chunk_dev_, delta_ws_;
+    int n_chunks_ = 0;
     // custom attention masks of the current forward (never part of a captured graph)
     Growable mask_in_host_, mask_in_dev_, mask_bitmap_;
     int mask_stride_ = 0;
@@ -234,7 +237,7 @@ class Executor {
         float *x = nullptr, *logits = nullptr;   // residual stream, finished logits
         // compute type
         void *xa = nullptr, *in = nullptr, *y = nullptr, *cq = nullptr, *q = nullptr, *q_lat = nullptr, *o_lat = nullptr,
-             *o = nullptr, *act = nullptr, *a1 = nullptr, *g1 = nullptr, *decay = nullptr, *gate = nullptr,
+             *o = nullptr, *act = nullptr, *gate = nullptr,
              *xs = nullptr, *raw_logits = nullptr;
         float *dq = nullptr, *dk = nullptr, *dv = nullptr, *dg = nullptr, *d_beta = nullptr, *d_o = nullptr;
         std::vector<float*> rotary;              // tables of the step, one per distinct rotation

@@ -31,7 +31,7 @@ void Executor::alloc_stack() {
     const ModelConfig& m = model_.cfg();
     const size_t T = static_cast<size_t>(max_tokens_), esize = m.f32() ? 4 : 2;
     const size_t ld_x = static_cast<size_t>(model_.ld_x());
-    size_t in = 0, cq = 0, q = 0, q_lat = 0, o_lat = 0, o = 0, act = 0, a1 = 0, g1 = 0, decay = 0, gate = 0;
+    size_t in = 0, cq = 0, q = 0, q_lat = 0, o_lat = 0, o = 0, act = 0, gate = 0;
     size_t kd = 0, vd = 0, gd = 0, heads = 0, state = 0;
     auto up = [](size_t& v, int n) { v = std::max(v, static_cast<size_t>(n)); };
     for (const StackLayer& l : model_.stack) {
@@ -51,9 +51,6 @@ void Executor::alloc_stack() {
             const DeltaShape s(d);
             up(in, s.ld_in);
             up(o, s.ld_o);
-            up(a1, s.ld_a1);
-            up(g1, s.ld_g1);
-            up(decay, s.ld_decay);
             up(gate, s.ld_gate);
             up(kd, s.kd);
             up(vd, s.vd);
@@ -88,9 +85,6 @@ void Executor::alloc_stack() {
     stack_.o_lat = compute(T * o_lat);
     stack_.o = compute(T * o);
     stack_.act = compute(T * act);
-    stack_.a1 = compute(T * a1);
-    stack_.g1 = compute(T * g1);
-    stack_.decay = compute(T * decay);
     stack_.gate = compute(T * gate);
     stack_.dq = f32(T * kd);
     stack_.dk = f32(T * kd);
@@ -104,7 +98,7 @@ void Executor::alloc_stack() {
     stack_.logits = f32(srows * static_cast<size_t>(m.vocab));
     for (const RotaryTable& r : model_.rotary) stack_.rotary.push_back(f32(T * static_cast<size_t>(r.spec.dims)));
     for (StackLayer& l : model_.stack)
-        for (const Linear* w : {&l.w_in, &l.w_uq, &l.w_decay, &l.w_gate, &l.wo, &l.w_up, &l.w_down})
+        for (const Linear* w : {&l.w_in, &l.w_uq, &l.wo, &l.w_up, &l.w_down})
             for (int rows : {64, 128})
                 if (!m.f32() && w->data && w->K % 64 == 0)
                     gemm_ws_bytes_ = std::max(gemm_ws_bytes_, pie_hip_gemm_mfma_workspace_bytes(rows, w->N, w->K));
@@ -181,7 +175,7 @@ void Executor::prepare_stack(const BatchPlan& plan, const Inputs& in) {
     const bool recurrent = rs_slots_ > 0;
     if (recurrent && static_cast<int>(plan.rs_slots.size()) != plan.R)
         throw std::runtime_error("executor: this model needs a recurrent-state slot per request (rs_slot_ids)");
-    std::set<uint32_t> seen;
+    std::set<uint32_t> seen;   // (a slot's state is read and written by one request of a batch)
     for (int r = 0; r < plan.R; ++r) {
         const int q0 = plan.qo_indptr[r], q1 = plan.qo_indptr[r + 1];
         qo[r] = q0;
@@ -209,6 +203,24 @@ void Executor::prepare_stack(const BatchPlan& plan, const Inputs& in) {
     qo[plan.R] = plan.N;
     if (recurrent)
         for (int r = 0; r < plan.R; ++r) rs_pos_[plan.rs_slots[r]] = -1;   // (until the pass has succeeded)
+    if (recurrent && !plan.pure_decode) {
+        // the requests' rows in chunks of sixteen: (first row, rows), then each request's first chunk
+        std::vector<int32_t> chunks, first(1, 0);
+        for (int r = 0; r < plan.R; ++r) {
+            for (int i = plan.qo_indptr[r]; i < plan.qo_indptr[r + 1]; i += 16) {
+                chunks.push_back(i);
+                chunks.push_back(std::min(16, plan.qo_indptr[r + 1] - i));
+            }
+            first.push_back(static_cast<int32_t>(chunks.size() / 2));
+        }
+        n_chunks_ = static_cast<int>(chunks.size() / 2);
+        chunks.insert(chunks.end(), first.begin(), first.end());
+        chunk_host_.pinned = true;
+        chunk_host_.ensure(chunks.size() * 4);
+        chunk_dev_.ensure(chunks.size() * 4);
+        std::memcpy(chunk_host_.ptr, chunks.data(), chunks.size() * 4);
+        PIE_HIP_CHECK(hipMemcpyAsync(chunk_dev_.ptr, chunk_host_.ptr, chunks.size() * 4, hipMemcpyHostToDevice, stream_));
+    }
     plan_ = &plan;
 }
 
@@ -314,19 +326,41 @@ void Executor::stack_delta(const StackLayer& w, int layer, int N, const Inputs& 
     const auto* slot = reinterpret_cast<const int32_t*>(in_dev_ + in.off_rs_slot);
     const auto* fresh = reinterpret_cast<const int32_t*>(in_dev_ + in.off_rs_fresh);
     stack_linear(w.w_in, stack_.xa, stack_.in, N);
-    PIE_KERNEL(pie_hip_delta_prep(dt_, stack_.in, w.conv_w, rs_base_, rs_stride_, rs_conv_off_[layer], row_req, qo, slot,
-                                  fresh, stack_.dq, stack_.dk, stack_.dv, stack_.d_beta, stack_.a1, stack_.g1, N, s.ld_in,
-                                  d.heads, d.kv_heads, d.dim, d.vdim, d.taps, s.decay_off, d.decay_rank, s.ld_a1,
-                                  s.gate_off, d.gate_rank, s.ld_g1, stream_));
-    stack_linear(w.w_decay, stack_.a1, stack_.decay, N);
-    stack_linear(w.w_gate, stack_.g1, stack_.gate, N);
-    PIE_KERNEL(pie_hip_delta_decay(dt_, stack_.decay, w.a_log, w.dt_bias, stack_.dg, N, s.ld_decay, d.heads, d.dim, stream_));
-    PIE_KERNEL(pie_hip_delta_scan(stack_.dq, stack_.dk, stack_.dv, stack_.dg, stack_.d_beta, stack_.d_o, rs_base_,
-                                  rs_stride_, rs_state_off_[layer], qo, slot, fresh, n_requests_, d.heads, d.kv_heads,
-                                  d.dim, d.vdim, stream_));
-    PIE_KERNEL(pie_hip_delta_out(dt_, stack_.d_o, stack_.gate, w.out_norm, stack_.o, stack_.in, rs_base_, rs_stride_,
-                                 rs_conv_off_[layer], row_req, qo, slot, fresh, N, s.ld_gate, s.ld_o, s.ld_in, d.heads,
-                                 d.kv_heads, d.dim, d.vdim, d.taps, model_.cfg().rms_eps, stream_));
+    PIE_KERNEL(pie_hip_delta_lowrank(dt_, stack_.in, w.w_decay, w.w_gate, w.a_log, w.dt_bias, stack_.dg, stack_.gate, N,
+                                     s.ld_in, s.decay_off, d.decay_rank, s.ld_a1, s.gate_off, d.gate_rank, s.ld_g1, d.heads,
+                                     d.dim, d.vdim, s.ld_gate, stream_));
+    const float eps = model_.cfg().rms_eps;
+    auto conv_state = [&] {
+        PIE_KERNEL(pie_hip_delta_conv_state(dt_, stack_.in, rs_base_, rs_stride_, rs_conv_off_[layer], qo, slot, fresh,
+                                            n_requests_, s.ld_in, s.channels, d.taps, stream_));
+    };
+    if (plan_->pure_decode && pie_hip_delta_step_supported(d.dim, d.vdim)) {
+        // (heads that share q / k channels leave the convolution's state to a launch of its own)
+        const bool own = d.heads == d.kv_heads;
+        PIE_KERNEL(pie_hip_delta_step(dt_, stack_.in, w.conv_w, stack_.dg, stack_.gate, w.out_norm, stack_.o, rs_base_, rs_stride_,
+                                      rs_state_off_[layer], rs_conv_off_[layer], slot, fresh, N, s.ld_in, s.ld_gate, s.ld_o,
+                                      d.heads, d.kv_heads, d.dim, d.vdim, d.taps, own ? 1 : 0, eps, stream_));
+        if (!own) conv_state();
+    } else {
+        PIE_KERNEL(pie_hip_delta_prep(dt_, stack_.in, w.conv_w, rs_base_, rs_stride_, rs_conv_off_[layer], row_req, qo, slot,
+                                      fresh, stack_.dq, stack_.dk, stack_.dv, stack_.d_beta, N, s.ld_in, d.heads, d.kv_heads,
+                                      d.dim, d.vdim, d.taps, stream_));
+        conv_state();
+        if (plan_->pure_decode) {
+            PIE_KERNEL(pie_hip_delta_scan(stack_.dq, stack_.dk, stack_.dv, stack_.dg, stack_.d_beta, stack_.d_o, rs_base_,
+                                          rs_stride_, rs_state_off_[layer], qo, slot, fresh, n_requests_, d.heads, d.kv_heads,
+                                          d.dim, d.vdim, stream_));
+        } else {
+            delta_ws_.ensure(pie_hip_delta_chunked_workspace_bytes(n_chunks_, d.heads, d.dim));
+            const auto* chunks = static_cast<const int32_t*>(chunk_dev_.ptr);
+            PIE_KERNEL(pie_hip_delta_chunked(stack_.dq, stack_.dk, stack_.dv, stack_.dg, stack_.d_beta, stack_.d_o, rs_base_,
+                                             rs_stride_, rs_state_off_[layer], chunks, chunks + 2 * n_chunks_, slot, fresh,
+                                             n_chunks_, n_requests_, d.heads, d.kv_heads, d.dim, d.vdim, delta_ws_.ptr,
+                                             delta_ws_.cap, stream_));
+        }
+        PIE_KERNEL(pie_hip_delta_out(dt_, stack_.d_o, stack_.gate, w.out_norm, stack_.o, N, s.ld_gate, s.ld_o, d.heads, d.vdim,
+                                     eps, stream_));
+    }
     stack_linear(w.wo, stack_.o, stack_.y, N);
 }
 

@@ -88,11 +88,11 @@ struct LatentShape {
 struct DeltaShape {
     int kd, vd, channels;                       // q (= k) channels, v channels, all three
     int decay_off, gate_off, ld_in;             // fused projection: q | k | v | step sizes | decay | gate inputs
-    int ld_a1, ld_g1, ld_decay, ld_gate, ld_o;  // low-rank inputs, their projections, output rows
+    int ld_a1, ld_g1, ld_gate, ld_o;            // columns of the low-rank second factors, gate rows, output rows
     explicit DeltaShape(const ChannelDeltaSpec& d)
         : kd(d.kv_heads * d.dim), vd(d.heads * d.vdim), channels(2 * kd + vd), decay_off(pad_to(channels + d.heads, 8)),
           gate_off(pad_to(decay_off + d.decay_rank, 8)), ld_in(pad_to(gate_off + d.gate_rank, 16)),
-          ld_a1(pad_to(d.decay_rank, 128)), ld_g1(pad_to(d.gate_rank, 128)), ld_decay(pad_to(d.heads * d.dim, 16)),
+          ld_a1(pad_to(d.decay_rank, 32)), ld_g1(pad_to(d.gate_rank, 32)),
           ld_gate(pad_to(vd, 16)), ld_o(pad_to(vd, 128)) {}
 };
 
@@ -109,7 +109,7 @@ struct StackLayer {
     float *q_norm = nullptr, *kv_norm = nullptr;
     int rotary = -1;                             // index into Model::rotary
     // channel delta
-    Linear w_decay, w_gate;                      // second factors of the low-rank decay and output gate
+    uint16_t *w_decay = nullptr, *w_gate = nullptr;   // second factors of the low-rank decay and output gate
     float *conv_w = nullptr, *a_log = nullptr, *dt_bias = nullptr, *out_norm = nullptr;
 };
 

@@ -234,10 +234,15 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
                 plain_rows(put, mix + "a1", s.decay_off, d.decay_rank, H);
                 plain_rows(put, mix + "g1", s.gate_off, d.gate_rank, H);
             });
-            linear(w.w_decay, mix + "a2", s.ld_decay, s.ld_a1, d.decay_rank,
-                   [&](auto put) { plain_rows(put, mix + "a2", 0, d.heads * d.dim, d.decay_rank); });
-            linear(w.w_gate, mix + "g2", s.ld_gate, s.ld_g1, d.gate_rank,
-                   [&](auto put) { plain_rows(put, mix + "g2", 0, s.vd, d.gate_rank); });
+            auto low_rank = [&](const std::string& name, int rows, int rank, int ld) {
+                decode_bytes_ += static_cast<size_t>(rows) * ld * 2;
+                return device_matrix(name, static_cast<size_t>(rows) * ld, rank, [&](std::vector<uint16_t>& host) {
+                    const HostMatrix m = matrix(name, rows, rank);
+                    for (int r = 0; r < rows; ++r) std::memcpy(&host[static_cast<size_t>(r) * ld], m.row(r), static_cast<size_t>(rank) * 2);
+                });
+            };
+            w.w_decay = low_rank(mix + "a2", d.heads * d.dim, d.decay_rank, s.ld_a1);
+            w.w_gate = low_rank(mix + "g2", s.vd, d.gate_rank, s.ld_g1);
             linear(w.wo, mix + "o", Hp, s.ld_o, s.vd, [&](auto put) { plain_rows(put, mix + "o", 0, H, s.vd); });
             w.a_log = vec(mix + "A_log", d.heads, [&](size_t i) { return std::log(1.f + static_cast<float>(i % 8)); });
             w.dt_bias = vec(mix + "dt_bias", static_cast<size_t>(d.heads) * d.dim, [](size_t) { return -3.f; });
