@@ -866,8 +866,8 @@ int pie_hip_latent_attn_prefill(const uint16_t* q, const uint16_t* kv, const uin
  *   sigmoid(step size).  dim <= 512.
  * pie_hip_delta_conv_state: the last taps - 1 convolution inputs of every request (after prep).
  * pie_hip_delta_lowrank: fused[n] also holds the low-rank inputs a1 (decay_off, decay_rank) and g1
- *   (gate_off, gate_rank); log2_decay = -exp(a_log[head]) softplus(w_decay a1 + dt_bias) log2(e),
- *   [N, heads * dim] fp32; gate = w_gate g1, [N, ld_gate] compute type.  Weights [.., ld_a1], [..,
+ *   (gate_off, gate_rank); log2_decay = rate[head] softplus(w_decay a1 + dt_bias) with
+ *   rate = -exp(A_log) log2(e), [N, heads * dim] fp32; gate = w_gate g1, [N, ld_gate] compute type.  Weights [.., ld_a1], [..,
  *   ld_g1], zero past the ranks.
  * pie_hip_delta_scan: per token S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q with g =
  *   2^log2_decay; head h uses q / k head h / (heads / kv_heads).  Reads and writes the state.
@@ -888,7 +888,7 @@ int pie_hip_delta_conv_state(int dtype, const void* fused, void* rs_base, size_t
                              const int32_t* qo_indptr, const int32_t* rs_slot, const int32_t* rs_fresh,
                              int num_requests, int ld, int channels, int taps, void* stream);
 int pie_hip_delta_lowrank(int dtype, const void* fused, const uint16_t* w_decay, const uint16_t* w_gate,
-                          const float* a_log, const float* dt_bias, float* log2_decay, void* gate, int num_tokens,
+                          const float* rate, const float* dt_bias, float* log2_decay, void* gate, int num_tokens,
                           int ld, int decay_off, int decay_rank, int ld_a1, int gate_off, int gate_rank, int ld_g1,
                           int heads, int dim, int vdim, int ld_gate, void* stream);
 int pie_hip_delta_scan(const float* q, const float* k, const float* v, const float* log2_decay, const float* beta,
@@ -898,8 +898,8 @@ int pie_hip_delta_scan(const float* q, const float* k, const float* v, const flo
 size_t pie_hip_delta_chunked_workspace_bytes(int num_chunks, int heads, int dim);
 int pie_hip_delta_chunked(const float* q, const float* k, const float* v, const float* log2_decay, const float* beta,
                           float* o, void* rs_base, size_t rs_stride, size_t state_offset, const int32_t* chunks,
-                          const int32_t* req_chunks, const int32_t* rs_slot, const int32_t* rs_fresh, int num_chunks,
-                          int num_requests, int heads, int kv_heads, int dim, int vdim, void* workspace,
+                          const int32_t* req_chunks, const int32_t* qo_indptr, const int32_t* rs_slot,
+                          const int32_t* rs_fresh, int num_chunks, int num_requests, int heads, int kv_heads, int dim, int vdim, void* workspace,
                           size_t workspace_bytes, void* stream);
 int pie_hip_delta_out(int dtype, const float* o, const void* gate, const float* norm_w, void* y, int num_tokens,
                       int ld_gate, int ld_y, int heads, int vdim, float eps, void* stream);

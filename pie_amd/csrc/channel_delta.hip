@@ -78,14 +78,33 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(const DeltaPrepArgs a) 
                 w[e][j] = d < len && tap >= 0 ? a.conv_w[static_cast<size_t>(c0 + d) * a.taps + tap] : 0.f;
             }
     float win[PL][4] = {};   // inputs of the last four tokens, oldest first
-    int prev_req = -1;
     const float qk_scale = is_q ? 1.f / sqrtf(static_cast<float>(a.dim)) : 1.f;
+    int r = 0, row0 = 0, row1 = n0;   // the request in hand and its rows (re-read where it ends)
+    bool fresh = false;
+    const T* state = nullptr;
+    T now[PL];   // the row's own inputs, requested one row ahead
+    auto request = [&](int n) {
+#pragma unroll
+        for (int e = 0; e < PL; ++e) {
+            const int d = lane + e * kWave;
+            if (d < len) now[e] = fused[static_cast<size_t>(n) * a.ld + c0 + d];
+        }
+    };
+    request(n0);
     for (int n = n0; n < n1; ++n) {
-        const int r = a.rows.row_req[n];
-        const int row0 = a.rows.qo_indptr[r], i = n - row0;
-        const bool fresh = a.rows.rs_fresh[r] != 0;
-        const T* state = reinterpret_cast<const T*>(a.rs_base + static_cast<size_t>(a.rows.rs_slot[r]) * a.rs_stride + a.conv_offset);
-        float val[PL];
+        const bool enter = n >= row1;
+        if (enter) {
+            r = a.rows.row_req[n];
+            row0 = a.rows.qo_indptr[r];
+            row1 = a.rows.qo_indptr[r + 1];
+            fresh = a.rows.rs_fresh[r] != 0;
+            state = reinterpret_cast<const T*>(a.rs_base + static_cast<size_t>(a.rows.rs_slot[r]) * a.rs_stride + a.conv_offset);
+        }
+        const int i = n - row0;
+        float cur[PL], val[PL];
+#pragma unroll
+        for (int e = 0; e < PL; ++e) cur[e] = lane + e * kWave < len ? act_get<T>(now[e]) : 0.f;
+        if (n + 1 < n1) request(n + 1);
 #pragma unroll
         for (int e = 0; e < PL; ++e) {
             const int d = lane + e * kWave;
@@ -94,13 +113,13 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(const DeltaPrepArgs a) 
             auto input = [&](int at) { return conv_input<T>(fused, state, a.ld, row0, at, c0 + d, keep, channels, fresh); };
             float y = 0.f;
             if (windowed) {
-                if (r != prev_req) {
+                if (enter) {
 #pragma unroll
                     for (int j = 1; j < 4; ++j) win[e][j] = 4 - j <= keep ? input(i - (4 - j)) : 0.f;
                 }
 #pragma unroll
                 for (int j = 0; j < 3; ++j) win[e][j] = win[e][j + 1];
-                win[e][3] = act_get<T>(fused[static_cast<size_t>(n) * a.ld + c0 + d]);
+                win[e][3] = cur[e];
 #pragma unroll
                 for (int j = 0; j < 4; ++j) y = fmaf(w[e][j], win[e][j], y);
             } else {
@@ -108,7 +127,6 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(const DeltaPrepArgs a) 
             }
             val[e] = y * sigmoid_f32(y);
         }
-        prev_req = r;
         if (is_v) {
 #pragma unroll
             for (int e = 0; e < PL; ++e) {
@@ -146,22 +164,21 @@ __global__ __launch_bounds__(256) void delta_conv_state_kernel(const T* __restri
 }
 
 __device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
-constexpr float kLog2e = 1.4426950408889634f;
 
 // The second factors of the low-rank decay and output gate, straight from the fused projection's
-// columns: log2 of the decay, -exp(A_log) softplus(W_a2 a1 + dt_bias) log2(e), in fp32, and the
+// columns: log2 of the decay, rate[head] softplus(W_a2 a1 + dt_bias), in fp32, and the
 // gate's projection in the compute type.  The launch's first blocks along x take the decay's
 // outputs, the others the gate's, 64 each; MFMA as in the head-wise linears (weights the A operand).
 struct LowRankArgs {
     const void* fused;
     const uint16_t *w_decay, *w_gate;   // [.., ld_a1], [.., ld_g1], zero columns past the rank
-    const float *a_log, *dt_bias;
+    const float *rate, *dt_bias;        // [heads] -exp(A_log) log2(e); [heads * dim]
     float* lg;                          // [M, heads * dim]
     void* gate;                         // [M, ld_gate]
     int M, ld, decay_off, gate_off, decay_rank, gate_rank, ld_a1, ld_g1, dim, decay_n, gate_n, ld_gate, decay_blocks;
 };
 __device__ __forceinline__ float decay_log2(const LowRankArgs& a, int c, float raw) {
-    return -expf(a.a_log[c / a.dim]) * softplus_f32(raw + a.dt_bias[c]) * kLog2e;
+    return a.rate[c / a.dim] * softplus_f32(raw + a.dt_bias[c]);
 }
 typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
 template <int MT>
@@ -196,12 +213,19 @@ __global__ __launch_bounds__(256) void delta_lowrank_mfma_kernel(const LowRankAr
     for (int t = 0; t < MT; ++t) {
         const int m = m0 + 16 * t + l16;
         if (m >= a.M) continue;
+        const int c = c0 + 4 * g;
+        if (is_gate) {   // (ld_gate is a multiple of 16: whole pieces)
+            *reinterpret_cast<u32x2_t*>(static_cast<uint16_t*>(a.gate) + static_cast<size_t>(m) * a.ld_gate + c) =
+                u32x2_t{pack_bf16x2(acc[t][0], acc[t][1]), pack_bf16x2(acc[t][2], acc[t][3])};
+        } else if (N % 4 == 0 && c + 4 <= N) {
+            f32x4_t v;
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const int c = c0 + 4 * g + e;
-            if (c >= N) continue;
-            if (is_gate) static_cast<uint16_t*>(a.gate)[static_cast<size_t>(m) * a.ld_gate + c] = f32_to_bf16_bits(acc[t][e]);
-            else a.lg[static_cast<size_t>(m) * N + c] = decay_log2(a, c, acc[t][e]);
+            for (int e = 0; e < 4; ++e) v[e] = decay_log2(a, c + e, acc[t][e]);
+            *reinterpret_cast<f32x4_t*>(a.lg + static_cast<size_t>(m) * N + c) = v;
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                if (c + e < N) a.lg[static_cast<size_t>(m) * N + c + e] = decay_log2(a, c + e, acc[t][e]);
         }
     }
 }
@@ -618,8 +642,8 @@ struct DeltaWalkArgs {
     float* o;
     unsigned char* rs_base;
     size_t rs_stride, state_offset;
-    const int32_t* chunks;       // [num_chunks][2]
     const int32_t* req_chunks;   // [R + 1] chunks of each request
+    const int32_t* qo_indptr;    // [R + 1] rows of each request
     const int32_t *rs_slot, *rs_fresh;
     int heads, dim, vdim;
 };
@@ -638,6 +662,7 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(const DeltaWalkArgs a) 
     const int tid = threadIdx.x, lane = tid & (kWave - 1), l16 = lane & 15, g = lane >> 4;
     const int wv = __builtin_amdgcn_readfirstlane(tid / kWave);
     const int c_lo = a.req_chunks[r], c_hi = a.req_chunks[r + 1];
+    const int req_row0 = a.qo_indptr[r], req_row1 = a.qo_indptr[r + 1];
     const int vd = a.heads * a.vdim, col = col0 + l16;
     const bool live = col < a.vdim, fresh = a.rs_fresh[r] != 0;
     float* S = reinterpret_cast<float*>(a.rs_base + static_cast<size_t>(a.rs_slot[r]) * a.rs_stride + a.state_offset) +
@@ -667,8 +692,8 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(const DeltaWalkArgs a) 
         }
         f.tm = *reinterpret_cast<const f32x4_t*>(rec + Rec::tm + l16 * 16 + 4 * g);
         f.b = *reinterpret_cast<const f32x4_t*>(rec + Rec::b + l16 * 16 + 4 * g);
-        f.row0 = a.chunks[2 * c];
-        f.nt = a.chunks[2 * c + 1];
+        f.row0 = req_row0 + (c - c_lo) * kChunkTok;
+        f.nt = min(kChunkTok, req_row1 - f.row0);
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
             const int t = 4 * g + e;
@@ -790,18 +815,18 @@ extern "C" int pie_hip_delta_conv_state(int dtype, const void* fused, void* rs_b
 }
 
 extern "C" int pie_hip_delta_lowrank(int dtype, const void* fused, const uint16_t* w_decay, const uint16_t* w_gate,
-                                     const float* a_log, const float* dt_bias, float* log2_decay, void* gate,
+                                     const float* rate, const float* dt_bias, float* log2_decay, void* gate,
                                      int num_tokens, int ld, int decay_off, int decay_rank, int ld_a1, int gate_off,
                                      int gate_rank, int ld_g1, int heads, int dim, int vdim, int ld_gate, void* stream) {
-    if (!fused || !w_decay || !w_gate || !a_log || !dt_bias || !log2_decay || !gate || num_tokens <= 0 || heads <= 0 ||
+    if (!fused || !w_decay || !w_gate || !rate || !dt_bias || !log2_decay || !gate || num_tokens <= 0 || heads <= 0 ||
         dim <= 0 || vdim <= 0 || decay_rank <= 0 || gate_rank <= 0 || ld_a1 < decay_rank || ld_g1 < gate_rank ||
         decay_off + decay_rank > ld || gate_off + gate_rank > ld || ld_gate < heads * vdim)
         return PIE_HIP_ERR_INVALID;
     // whole 16-byte pieces of the low-rank columns must lie inside a row
-    if (ld % 8 != 0 || decay_off % 8 != 0 || gate_off % 8 != 0 || ld_a1 % 32 != 0 || ld_g1 % 32 != 0 ||
+    if (ld % 8 != 0 || ld_gate % 16 != 0 || decay_off % 8 != 0 || gate_off % 8 != 0 || ld_a1 % 32 != 0 || ld_g1 % 32 != 0 ||
         decay_off + (decay_rank + 7) / 8 * 8 > ld || gate_off + (gate_rank + 7) / 8 * 8 > ld)
         return PIE_HIP_ERR_UNSUPPORTED;
-    const LowRankArgs a{fused, w_decay, w_gate, a_log, dt_bias, log2_decay, gate, num_tokens, ld, decay_off, gate_off,
+    const LowRankArgs a{fused, w_decay, w_gate, rate, dt_bias, log2_decay, gate, num_tokens, ld, decay_off, gate_off,
                         decay_rank, gate_rank, ld_a1, ld_g1, dim, heads * dim, heads * vdim, ld_gate, (heads * dim + 63) / 64};
     const int gx = a.decay_blocks + (heads * vdim + 63) / 64;
     hipStream_t s = static_cast<hipStream_t>(stream);
@@ -852,17 +877,17 @@ extern "C" size_t pie_hip_delta_chunked_workspace_bytes(int num_chunks, int head
 
 extern "C" int pie_hip_delta_chunked(const float* q, const float* k, const float* v, const float* log2_decay,
                                      const float* beta, float* o, void* rs_base, size_t rs_stride, size_t state_offset,
-                                     const int32_t* chunks, const int32_t* req_chunks, const int32_t* rs_slot,
-                                     const int32_t* rs_fresh, int num_chunks, int num_requests, int heads, int kv_heads,
+                                     const int32_t* chunks, const int32_t* req_chunks, const int32_t* qo_indptr,
+                                     const int32_t* rs_slot, const int32_t* rs_fresh, int num_chunks, int num_requests, int heads, int kv_heads,
                                      int dim, int vdim, void* workspace, size_t workspace_bytes, void* stream) {
-    if (!q || !k || !v || !log2_decay || !beta || !o || !rs_base || !chunks || !req_chunks || !rs_slot || !rs_fresh ||
+    if (!q || !k || !v || !log2_decay || !beta || !o || !rs_base || !chunks || !req_chunks || !qo_indptr || !rs_slot || !rs_fresh ||
         num_chunks <= 0 || num_requests <= 0 || heads <= 0 || kv_heads <= 0 || heads % kv_heads != 0 || dim <= 0 || vdim <= 0)
         return PIE_HIP_ERR_INVALID;
     if (dim > 256 || num_chunks > 65535 || num_requests > 65535 || (vdim + 15) / 16 > 65535) return PIE_HIP_ERR_UNSUPPORTED;
     if (!workspace || workspace_bytes < pie_hip_delta_chunked_workspace_bytes(num_chunks, heads, dim)) return PIE_HIP_ERR_INVALID;
     float* rec = static_cast<float*>(workspace);
     const DeltaChunkArgs c{q, k, log2_decay, beta, chunks, rec, heads, kv_heads, dim};
-    const DeltaWalkArgs w{rec, v, o, static_cast<unsigned char*>(rs_base), rs_stride, state_offset, chunks, req_chunks,
+    const DeltaWalkArgs w{rec, v, o, static_cast<unsigned char*>(rs_base), rs_stride, state_offset, req_chunks, qo_indptr,
                           rs_slot, rs_fresh, heads, dim, vdim};
     hipStream_t s = static_cast<hipStream_t>(stream);
     switch ((dim + 63) / 64) {

@@ -326,7 +326,7 @@ void Executor::stack_delta(const StackLayer& w, int layer, int N, const Inputs& 
     const auto* slot = reinterpret_cast<const int32_t*>(in_dev_ + in.off_rs_slot);
     const auto* fresh = reinterpret_cast<const int32_t*>(in_dev_ + in.off_rs_fresh);
     stack_linear(w.w_in, stack_.xa, stack_.in, N);
-    PIE_KERNEL(pie_hip_delta_lowrank(dt_, stack_.in, w.w_decay, w.w_gate, w.a_log, w.dt_bias, stack_.dg, stack_.gate, N,
+    PIE_KERNEL(pie_hip_delta_lowrank(dt_, stack_.in, w.w_decay, w.w_gate, w.decay_rate, w.dt_bias, stack_.dg, stack_.gate, N,
                                      s.ld_in, s.decay_off, d.decay_rank, s.ld_a1, s.gate_off, d.gate_rank, s.ld_g1, d.heads,
                                      d.dim, d.vdim, s.ld_gate, stream_));
     const float eps = model_.cfg().rms_eps;
@@ -354,7 +354,7 @@ void Executor::stack_delta(const StackLayer& w, int layer, int N, const Inputs& 
             delta_ws_.ensure(pie_hip_delta_chunked_workspace_bytes(n_chunks_, d.heads, d.dim));
             const auto* chunks = static_cast<const int32_t*>(chunk_dev_.ptr);
             PIE_KERNEL(pie_hip_delta_chunked(stack_.dq, stack_.dk, stack_.dv, stack_.dg, stack_.d_beta, stack_.d_o, rs_base_,
-                                             rs_stride_, rs_state_off_[layer], chunks, chunks + 2 * n_chunks_, slot, fresh,
+                                             rs_stride_, rs_state_off_[layer], chunks, chunks + 2 * n_chunks_, qo, slot, fresh,
                                              n_chunks_, n_requests_, d.heads, d.kv_heads, d.dim, d.vdim, delta_ws_.ptr,
                                              delta_ws_.cap, stream_));
         }

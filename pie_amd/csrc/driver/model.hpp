@@ -110,7 +110,7 @@ struct StackLayer {
     int rotary = -1;                             // index into Model::rotary
     // channel delta
     uint16_t *w_decay = nullptr, *w_gate = nullptr;   // second factors of the low-rank decay and output gate
-    float *conv_w = nullptr, *a_log = nullptr, *dt_bias = nullptr, *out_norm = nullptr;
+    float *conv_w = nullptr, *decay_rate = nullptr /* -exp(A_log) log2(e) */, *dt_bias = nullptr, *out_norm = nullptr;
 };
 
 struct RotaryTable {

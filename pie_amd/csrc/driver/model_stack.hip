@@ -84,8 +84,9 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
         m.cols = cols;
         return m;
     };
-    // fp32 vector (or small matrix) parameter; `dflt` fills it for random weights
-    auto vec = [&](const std::string& name, size_t n, auto dflt) {
+    // fp32 vector parameter; `dflt` fills it for random weights, `map` changes its values
+    auto identity = [](float v) { return v; };
+    auto vec_mapped = [&](const std::string& name, size_t n, auto dflt, auto map) {
         std::vector<float> v(n);
         if (random) {
             for (size_t i = 0; i < n; ++i) v[i] = dflt(i);
@@ -100,11 +101,13 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
                 for (size_t i = 0; i < n; ++i) v[i] = bf16_value(p[i]);
             }
         }
+        for (float& x : v) x = map(x);
         float* d = static_cast<float*>(alloc(4 * n, name));
         PIE_HIP_CHECK(hipMemcpyAsync(d, v.data(), 4 * n, hipMemcpyHostToDevice, stream));
         PIE_HIP_CHECK(hipStreamSynchronize(stream));
         return d;
     };
+    auto vec = [&](const std::string& name, size_t n, auto dflt) { return vec_mapped(name, n, dflt, identity); };
     auto ones = [](size_t) { return 1.f; };
     auto upload = [&](uint16_t* dst, const std::vector<uint16_t>& host) {
         PIE_HIP_CHECK(hipMemcpyAsync(dst, host.data(), host.size() * 2, hipMemcpyHostToDevice, stream));
@@ -244,7 +247,8 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
             w.w_decay = low_rank(mix + "a2", d.heads * d.dim, d.decay_rank, s.ld_a1);
             w.w_gate = low_rank(mix + "g2", s.vd, d.gate_rank, s.ld_g1);
             linear(w.wo, mix + "o", Hp, s.ld_o, s.vd, [&](auto put) { plain_rows(put, mix + "o", 0, H, s.vd); });
-            w.a_log = vec(mix + "A_log", d.heads, [&](size_t i) { return std::log(1.f + static_cast<float>(i % 8)); });
+            w.decay_rate = vec_mapped(mix + "A_log", d.heads, [&](size_t i) { return std::log(1.f + static_cast<float>(i % 8)); },
+                               [](float v) { return static_cast<float>(-std::exp(static_cast<double>(v)) * 1.4426950408889634074); });
             w.dt_bias = vec(mix + "dt_bias", static_cast<size_t>(d.heads) * d.dim, [](size_t) { return -3.f; });
             w.out_norm = vec(mix + "norm", d.vdim, ones);
             // the three convolutions back to back, [channels, taps]

@@ -84,8 +84,8 @@ struct HeadArgs {
 };
 
 template <class T>
-__device__ __forceinline__ void head_rotated_part(const HeadArgs& a, int h, int m_begin, int m_end) {
-    for (int idx = threadIdx.x; idx < (m_end - m_begin) * a.rotp; idx += blockDim.x) {
+__device__ __forceinline__ void head_rotated_part(const HeadArgs& a, int h, int m_begin, int m_end, int part, int parts) {
+    for (int idx = part * blockDim.x + threadIdx.x; idx < (m_end - m_begin) * a.rotp; idx += parts * blockDim.x) {
         const int m = m_begin + idx / a.rotp, i = idx % a.rotp;
         const T* src = static_cast<const T*>(a.act) + static_cast<size_t>(m) * a.ld_act +
                        static_cast<size_t>(h) * a.act_stride + a.rot_off;
@@ -97,20 +97,21 @@ __device__ __forceinline__ void head_rotated_part(const HeadArgs& a, int h, int 
     }
 }
 
-// Matrix-core form: a wave takes 16 outputs of one head for MT tiles of 16 rows; the weight
+// Matrix-core form: a wave (a block of its own: with few rows these launches are small, and single
+// waves spread over the most CUs) takes 16 outputs of one head for MT tiles of 16 rows; the weight
 // fragment (A operand: output on lane%16, k in the lane) is read once for all of them, the rows
 // are the B operand, so a lane ends with four consecutive outputs of one row.
 template <int MT>
-__global__ __launch_bounds__(256) void head_linear_mfma_kernel(const HeadArgs a) {
+__global__ __launch_bounds__(kWave) void head_linear_mfma_kernel(const HeadArgs a) {
     const int h = blockIdx.y, m0 = blockIdx.z * 16 * MT;
-    const int lane = threadIdx.x & (kWave - 1), wv = threadIdx.x / kWave;
+    const int lane = threadIdx.x;
     const int l16 = lane & 15, g = lane >> 4;
-    if (a.rotp > 0 && blockIdx.x == gridDim.x - 1) {
-        head_rotated_part<uint16_t>(a, h, m0, min(m0 + 16 * MT, a.M));
+    const int cblocks = a.C / 16;
+    if (static_cast<int>(blockIdx.x) >= cblocks) {
+        head_rotated_part<uint16_t>(a, h, m0, min(m0 + 16 * MT, a.M), blockIdx.x - cblocks, gridDim.x - cblocks);
         return;
     }
-    const int c0 = (blockIdx.x * 4 + wv) * 16;
-    if (c0 >= a.C) return;
+    const int c0 = blockIdx.x * 16;
     const uint16_t* wp = a.w + (static_cast<size_t>(h) * a.C + c0 + l16) * a.K + 8 * g;
     const uint16_t* ap[MT];
 #pragma unroll
@@ -120,8 +121,8 @@ __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const HeadArgs a)
     f32x4_t acc[MT];
 #pragma unroll
     for (int t = 0; t < MT; ++t) acc[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    // (four k-steps requested together; past K a request repeats the last step and is not multiplied)
-    constexpr int U = 4;
+    // (eight k-steps requested together, four with many rows; past K a request repeats the last step and is not multiplied)
+    constexpr int U = MT == 1 ? 8 : 4;
     for (int k0 = 0; k0 < a.K; k0 += 32 * U) {
         u32x4_t wf[U], af[U][MT];
 #pragma unroll
@@ -168,7 +169,7 @@ __global__ __launch_bounds__(256) void head_linear_f32_kernel(const HeadArgs a) 
         }
         dst[c] = acc;
     }
-    if (a.rotp > 0) head_rotated_part<float>(a, h, m, m + 1);
+    if (a.rotp > 0) head_rotated_part<float>(a, h, m, m + 1, 0, 1);
 }
 
 // The rows form of the attention, any sizes and either compute type: one block per (head, row),
@@ -284,14 +285,14 @@ extern "C" int pie_hip_head_linear(int dtype, const void* act, const uint16_t* w
         return launch_status();
     }
     if (dtype != PIE_HIP_DT_BF16) return PIE_HIP_ERR_INVALID;
-    const int gx = (C + 63) / 64 + (rotp > 0 ? 1 : 0);
     const int mt = M <= 16 ? 1 : M <= 32 ? 2 : 4;
+    const int gx = C / 16 + (rotp > 0 ? mt : 0);
     const int gz = (M + 16 * mt - 1) / (16 * mt);
     if (gz > 65535) return PIE_HIP_ERR_UNSUPPORTED;
     switch (mt) {
-        case 1: hipLaunchKernelGGL(head_linear_mfma_kernel<1>, dim3(gx, heads, gz), dim3(256), 0, s, a); break;
-        case 2: hipLaunchKernelGGL(head_linear_mfma_kernel<2>, dim3(gx, heads, gz), dim3(256), 0, s, a); break;
-        default: hipLaunchKernelGGL(head_linear_mfma_kernel<4>, dim3(gx, heads, gz), dim3(256), 0, s, a); break;
+        case 1: hipLaunchKernelGGL(head_linear_mfma_kernel<1>, dim3(gx, heads, gz), dim3(64), 0, s, a); break;
+        case 2: hipLaunchKernelGGL(head_linear_mfma_kernel<2>, dim3(gx, heads, gz), dim3(64), 0, s, a); break;
+        default: hipLaunchKernelGGL(head_linear_mfma_kernel<4>, dim3(gx, heads, gz), dim3(64), 0, s, a); break;
     }
     return launch_status();
 }

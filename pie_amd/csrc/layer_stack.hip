@@ -11,17 +11,26 @@ namespace pie_hip {
 namespace {
 
 template <class T>
-__global__ __launch_bounds__(256) void embed_stream_kernel(const uint32_t* __restrict__ tokens,
-                                                           const uint16_t* __restrict__ table,
-                                                           float* __restrict__ x, T* __restrict__ xa, int width,
-                                                           int ld, int vocab) {
+__global__ __launch_bounds__(1024) void embed_stream_kernel(const uint32_t* __restrict__ tokens,
+                                                            const uint16_t* __restrict__ table,
+                                                            float* __restrict__ x, T* __restrict__ xa, int width,
+                                                            int ld, int vocab) {
     const int n = blockIdx.x;
     const uint32_t t = tokens[n];
     const size_t row = t < static_cast<uint32_t>(vocab) ? t : 0;
-    for (int i = threadIdx.x; i < ld; i += blockDim.x) {
-        const float v = i < width ? bf16_bits_to_f32(table[row * width + i]) : 0.f;
-        x[static_cast<size_t>(n) * ld + i] = v;
-        xa[static_cast<size_t>(n) * ld + i] = act_put<T>(v);
+    for (int i = 4 * threadIdx.x; i < ld; i += 4 * blockDim.x) {   // (ld is a multiple of 4)
+        f32x4_t v = {0.f, 0.f, 0.f, 0.f};
+        if (i + 4 <= width && width % 4 == 0) {
+            const u32x2_t r = *reinterpret_cast<const u32x2_t*>(table + row * width + i);
+            v = f32x4_t{bf16_lo(r.x), bf16_hi(r.x), bf16_lo(r.y), bf16_hi(r.y)};
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                if (i + e < width) v[e] = bf16_bits_to_f32(table[row * width + i + e]);
+        }
+        *reinterpret_cast<f32x4_t*>(x + static_cast<size_t>(n) * ld + i) = v;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) xa[static_cast<size_t>(n) * ld + i + e] = act_put<T>(v[e]);
     }
 }
 
@@ -88,17 +97,32 @@ __global__ __launch_bounds__(BLOCK) void norm_add_kernel(const T* __restrict__ y
 
 // out[s] = rmsnorm(x[rows[s]]) * w in the compute type; columns past the width are zero
 template <class T>
-__global__ __launch_bounds__(256) void norm_rows_kernel(const float* __restrict__ x, const uint32_t* __restrict__ rows,
-                                                        const float* __restrict__ w, T* __restrict__ out, int width,
-                                                        int ld, int num_rows, float eps) {
-    __shared__ float red[4];
+__global__ __launch_bounds__(1024) void norm_rows_kernel(const float* __restrict__ x, const uint32_t* __restrict__ rows,
+                                                         const float* __restrict__ w, T* __restrict__ out, int width,
+                                                         int ld, int num_rows, float eps) {
+    __shared__ float red[16];
     const size_t s = blockIdx.x;
     const uint32_t r = rows[s];
     const float* xr = x + static_cast<size_t>(r < static_cast<uint32_t>(num_rows) ? r : 0) * ld;
-    float local = 0.f;
-    for (int i = threadIdx.x; i < width; i += 256) local += xr[i] * xr[i];
+    constexpr int kCache = 8;
+    float xv[kCache], wv[kCache], local = 0.f;
+#pragma unroll
+    for (int c = 0; c < kCache; ++c) {
+        const int i = threadIdx.x + c * 1024;
+        xv[c] = i < width ? xr[i] : 0.f;
+        wv[c] = i < width ? w[i] : 0.f;
+    }
+#pragma unroll
+    for (int c = 0; c < kCache; ++c) local += xv[c] * xv[c];
+    for (int i = threadIdx.x + kCache * 1024; i < width; i += 1024) local += xr[i] * xr[i];
     const float inv = 1.f / sqrtf(block_total(local, red) / static_cast<float>(width) + eps);
-    for (int i = threadIdx.x; i < ld; i += 256) out[s * ld + i] = i < width ? act_put<T>(xr[i] * inv * w[i]) : act_put<T>(0.f);
+#pragma unroll
+    for (int c = 0; c < kCache; ++c) {
+        const int i = threadIdx.x + c * 1024;
+        if (i < ld) out[s * ld + i] = act_put<T>(xv[c] * inv * wv[c]);
+    }
+    for (int i = threadIdx.x + kCache * 1024; i < ld; i += 1024)
+        out[s * ld + i] = i < width ? act_put<T>(xr[i] * inv * w[i]) : act_put<T>(0.f);
 }
 
 // logits f32 = cap * tanh(y * scale / cap) (cap 0: y * scale), and their argmax (the lowest index
@@ -112,13 +136,22 @@ __global__ __launch_bounds__(1024) void logits_finish_kernel(const T* __restrict
     const size_t s = blockIdx.x;
     float bv = -INFINITY;
     int bi = 0;
-    for (int i = threadIdx.x; i < vocab; i += blockDim.x) {
-        float v = act_get<T>(y[s * ldy + i]) * scale;
-        if (cap > 0.f) v = cap * tanhf(v / cap);
-        logits[s * vocab + i] = v;
-        if (v > bv) {   // (indices ascend inside a thread)
-            bv = v;
-            bi = i;
+    constexpr int U = 8;   // values requested together
+    for (int i0 = threadIdx.x; i0 < vocab; i0 += U * 1024) {
+        T raw[U];
+#pragma unroll
+        for (int u = 0; u < U; ++u) raw[u] = y[s * ldy + min(i0 + u * 1024, vocab - 1)];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const int i = i0 + u * 1024;
+            if (i >= vocab) break;
+            float v = act_get<T>(raw[u]) * scale;
+            if (cap > 0.f) v = cap * tanhf(v / cap);
+            logits[s * vocab + i] = v;
+            if (v > bv) {   // (indices ascend inside a thread)
+                bv = v;
+                bi = i;
+            }
         }
     }
     auto better = [&](float ov, int oi) {
@@ -217,7 +250,9 @@ extern "C" int pie_hip_embed_stream(int dtype, const uint32_t* token_ids, const 
                                     void* x_act, int num_tokens, int width, int ld, int vocab, void* stream) {
     if (!token_ids || !table_bf16 || !x || !x_act || num_tokens <= 0 || width <= 0 || ld < width || vocab <= 0)
         return PIE_HIP_ERR_INVALID;
-    PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL(embed_stream_kernel<T>, dim3(num_tokens), dim3(256), 0,
+    if (ld % 4 != 0) return PIE_HIP_ERR_UNSUPPORTED;
+    const int threads = ld >= 4096 ? 1024 : 256;
+    PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL(embed_stream_kernel<T>, dim3(num_tokens), dim3(threads), 0,
                                                   static_cast<hipStream_t>(stream), token_ids, table_bf16, x,
                                                   static_cast<T*>(x_act), width, ld, vocab));
     return launch_status();
@@ -227,8 +262,8 @@ extern "C" int pie_hip_norm_add(int dtype, const void* y, const float* weight, f
                                 int width, int ldy, int ld, float eps, void* stream) {
     if (!y || !weight || !x || !x_act || rows <= 0 || width <= 0 || ldy < width || ld < width) return PIE_HIP_ERR_INVALID;
     if (ldy % 8 != 0 || ld % 8 != 0) return PIE_HIP_ERR_UNSUPPORTED;
-    // (few rows: wider blocks, so that a row's traffic is in flight at once)
-    if (width >= 2048)
+    // (few wide rows: wider blocks, so that a row's traffic is in flight at once)
+    if (width >= 2048 && rows < 512)
         PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL((norm_add_kernel<T, 1024>), dim3(rows), dim3(1024), 0,
                                                       static_cast<hipStream_t>(stream), static_cast<const T*>(y),
                                                       weight, x, static_cast<T*>(x_act), width, ldy, ld, eps));
@@ -243,7 +278,7 @@ extern "C" int pie_hip_norm_rows(int dtype, const float* x, const uint32_t* rows
                                  int num_out, int width, int ld, int num_rows, float eps, void* stream) {
     if (!x || !rows || !weight || !out || num_out <= 0 || width <= 0 || ld < width || num_rows <= 0)
         return PIE_HIP_ERR_INVALID;
-    PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL(norm_rows_kernel<T>, dim3(num_out), dim3(256), 0,
+    PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL(norm_rows_kernel<T>, dim3(num_out), dim3(1024), 0,
                                                   static_cast<hipStream_t>(stream), x, rows, weight,
                                                   static_cast<T*>(out), width, ld, num_rows, eps));
     return launch_status();
