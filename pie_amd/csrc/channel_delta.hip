@@ -697,7 +697,8 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(const DeltaWalkArgs a) 
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
             const int t = 4 * g + e;
-            f.v[e] = live && t < f.nt ? a.v[static_cast<size_t>(f.row0 + t) * vd + h * a.vdim + col] : 0.f;
+            // (columns and tokens past the end repeat the last one: they are not stored, their step size is 0)
+            f.v[e] = a.v[static_cast<size_t>(f.row0 + min(t, f.nt - 1)) * vd + h * a.vdim + min(col, a.vdim - 1)];
         }
     };
     auto run = [&](const Frags& f, int buf) {
@@ -738,14 +739,19 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(const DeltaWalkArgs a) 
             }
         }
     };
-    Frags f0, f1;
-    load(f0, c_lo);
-    for (int c = c_lo; c < c_hi; c += 2) {
-        load(f1, min(c + 1, c_hi - 1));
-        run(f0, 0);
-        if (c + 1 < c_hi) {
-            load(f0, min(c + 2, c_hi - 1));
-            run(f1, 1);
+    // (three chunks ahead: the records come from beyond the L2, a chunk's arithmetic is shorter than
+    // that takes)
+    constexpr int kAhead = 4;
+    Frags f[kAhead];
+#pragma unroll
+    for (int i = 0; i < kAhead - 1; ++i) load(f[i], min(c_lo + i, c_hi - 1));
+    for (int c = c_lo; c < c_hi; c += kAhead) {
+#pragma unroll
+        for (int i = 0; i < kAhead; ++i) {
+            load(f[(i + kAhead - 1) % kAhead], min(c + i + kAhead - 1, c_hi - 1));
+            __builtin_amdgcn_sched_barrier(0);
+            if (c + i < c_hi) run(f[i], i & 1);
+            __builtin_amdgcn_sched_barrier(0);
         }
     }
     if (live)

@@ -37,9 +37,17 @@ struct LatentRowsArgs {
     const int32_t* row_len;
     const int32_t* row_req;   // request of each row, qo_indptr its rows (null: every row its own request)
     const int32_t* qo_indptr;
-    int row0, num_rows, heads, head_groups, heads_per_tile, tokens_per_tile, ps, steps_per_split, nsplit;
+    int row0, num_rows, heads, head_groups, heads_per_tile, tokens_per_tile, ps, ps_shift, steps_per_split, nsplit;
     float scale_log2e;
 };
+
+// Keys of one split: a decode row cuts its own keys evenly (steps_per_split 0), whatever the bound
+// the launch was planned with; portions take the planned length.
+__device__ __forceinline__ int split_keys(int keys, int nsplit, int steps_per_split) {
+    if (steps_per_split > 0) return steps_per_split * kStep;
+    const int steps = (keys + kStep - 1) / kStep;
+    return max(1, (steps + nsplit - 1) / nsplit) * kStep;
+}
 
 // C: latent columns / 64; R: rotated columns / 32; MT: 16-pair tiles per block
 template <int C, int R, int MT>
@@ -67,8 +75,9 @@ __global__ __launch_bounds__(kBlock, 2) void latent_rows_kernel(const LatentRows
         nt = min(a.tokens_per_tile, a.qo_indptr[r + 1] - n);
     }
     const int kmax = a.row_len[n + nt - 1];   // (rows of a request are consecutive positions)
-    const int k_begin = blockIdx.y * a.steps_per_split * kStep;
-    const int k_end = min(kmax, k_begin + a.steps_per_split * kStep);
+    const int keys_per_split = split_keys(kmax, a.nsplit, a.steps_per_split);
+    const int k_begin = blockIdx.y * keys_per_split;
+    const int k_end = min(kmax, k_begin + keys_per_split);
     if (k_begin >= kmax && !(a.nsplit == 1 && kmax == 0)) return;
     const uint32_t* pages = a.page_indices + a.row_begin[n];
     // pair m of the tile -> token, head, visible keys
@@ -98,18 +107,22 @@ __global__ __launch_bounds__(kBlock, 2) void latent_rows_kernel(const LatentRows
 
     const int key = tid >> 3, piece0 = tid & 7;
     u32x4_t reg[NP];
-    auto issue = [&](int j0) {
-        const int jb = min(j0 + kStep - 1, kmax - 1);
-        const int page_a = j0 / a.ps, pa_end = (page_a + 1) * a.ps;
-        const uint32_t pid_a = __builtin_amdgcn_readfirstlane(pages[page_a]);
-        const uint32_t pid_b = __builtin_amdgcn_readfirstlane(pages[page_a + (jb >= pa_end ? 1 : 0)]);
+    // the page of this thread's key, requested a step ahead of the key itself: the two requests
+    // depend on each other and would otherwise stand in line in every step
+    uint32_t pid = 0;
+    int in_page = 0;
+    auto fetch_page = [&](int j0) {
         const int j = min(j0 + key, kmax - 1);   // (keys past the extent repeat the last: their weights are zero)
-        const bool in_a = j < pa_end;
-        const size_t slot = static_cast<size_t>(in_a ? pid_a : pid_b) * a.ps + (j - (in_a ? pa_end - a.ps : pa_end));
-        const uint16_t* row = a.pool + slot * LD + piece0 * 8;
+        const int page = a.ps_shift >= 0 ? j >> a.ps_shift : j / a.ps;
+        pid = pages[page];
+        in_page = j - page * a.ps;
+    };
+    auto issue = [&](int j0) {
+        const uint16_t* row = a.pool + (static_cast<size_t>(pid) * a.ps + in_page) * LD + piece0 * 8;
 #pragma unroll
         for (int u = 0; u < NP; ++u)
             if (PPR % 8 == 0 || piece0 + 8 * u < PPR) reg[u] = *reinterpret_cast<const u32x4_t*>(row + 64 * u);
+        fetch_page(j0 + kStep);
     };
     auto stage = [&]() {
         uint16_t* row = &tile[key * STRIDE + piece0 * 8];
@@ -124,21 +137,34 @@ __global__ __launch_bounds__(kBlock, 2) void latent_rows_kernel(const LatentRows
 #pragma unroll
         for (int t = 0; t < MT; ++t) acc[c][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 
-    if (k_begin < k_end) issue(k_begin);
+    if (k_begin < k_end) {
+        fetch_page(k_begin);
+        issue(k_begin);
+    }
     for (int j0 = k_begin; j0 < k_end; j0 += kStep) {
         stage();
         if (j0 + kStep < k_end) issue(j0 + kStep);
         __syncthreads();
         // scores
         {
-            f32x4_t st = {0.f, 0.f, 0.f, 0.f};
+            // (fragments requested KG at a time ahead of their products, two accumulator chains)
+            f32x4_t st = {0.f, 0.f, 0.f, 0.f}, st1 = st;
             const uint16_t* kp = &tile[(16 * kh + l16) * STRIDE + 8 * g];
+            constexpr int KG = 6;
 #pragma unroll
-            for (int ks = 0; ks < KSW; ++ks) {
-                if (MT == 1 && ks0 + ks >= KS) break;
-                const bf16x8_t kf = __builtin_bit_cast(bf16x8_t, *reinterpret_cast<const u32x4_t*>(kp + 32 * (ks0 + ks)));
-                st = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[ks], st, 0, 0, 0);
+            for (int k0 = 0; k0 < KSW; k0 += KG) {
+                u32x4_t kf[KG];
+#pragma unroll
+                for (int u = 0; u < KG; ++u)
+                    if (k0 + u < KSW) kf[u] = *reinterpret_cast<const u32x4_t*>(kp + 32 * min(ks0 + k0 + u, KS - 1));
+#pragma unroll
+                for (int u = 0; u < KG; ++u)
+                    if (k0 + u < KSW) {   // (a k-step past the row meets a zero query fragment)
+                        if (u & 1) st1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, kf[u]), qf[k0 + u], st1, 0, 0, 0);
+                        else st = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, kf[u]), qf[k0 + u], st, 0, 0, 0);
+                    }
             }
+            st += st1;
             *reinterpret_cast<f32x4_t*>(&sc[MT == 2 ? 0 : wv >> 1][(rt * 16 + l16) * SSTR + 16 * kh + 4 * g]) = st;
         }
         __syncthreads();
@@ -249,9 +275,10 @@ __global__ __launch_bounds__(kBlock, 2) void latent_rows_kernel(const LatentRows
 // thread.  A row has as many pieces as splits start before its last key.
 __global__ void latent_merge_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
                                     const int32_t* __restrict__ row_len, uint16_t* __restrict__ o, int row0, int heads,
-                                    int kvp, int nsplit, int keys_per_split) {
+                                    int kvp, int nsplit, int steps_per_split) {
     const size_t out = static_cast<size_t>(row0) * heads + blockIdx.x;
-    const int ns = min(nsplit, (row_len[out / heads] + keys_per_split - 1) / keys_per_split);
+    const int len = row_len[out / heads], keys_per_split = split_keys(len, nsplit, steps_per_split);
+    const int ns = min(nsplit, (len + keys_per_split - 1) / keys_per_split);
     const float* ml = part_ml + out * nsplit * 2;
     float mx = -INFINITY;
     for (int s = 0; s < ns; ++s) mx = fmaxf(mx, ml[2 * s]);
@@ -289,6 +316,7 @@ LatentPlan latent_plan(int num_rows, int heads, int max_kv_len, int max_tokens_p
     if (ns < 1) ns = 1;
     p.steps_per_split = static_cast<int>((steps + ns - 1) / ns);
     p.nsplit = (steps + p.steps_per_split - 1) / p.steps_per_split;
+    if (max_tokens_per_req == 1) p.steps_per_split = 0;
     return p;
 }
 
@@ -332,7 +360,8 @@ extern "C" int pie_hip_latent_attn_rows(const uint16_t* q, const uint16_t* pool,
     if (p.nsplit > 65535) return PIE_HIP_ERR_UNSUPPORTED;
     LatentRowsArgs a{q, pool, o, nullptr, nullptr, kv_page_indices, row_page_begin, row_kv_len,
                      max_tokens_per_req > 1 ? row_req : nullptr, qo_indptr, row0, num_rows, heads, p.head_groups,
-                     p.heads_per_tile, p.tokens_per_tile, page_size, p.steps_per_split, p.nsplit,
+                     p.heads_per_tile, p.tokens_per_tile, page_size,
+                     (page_size & (page_size - 1)) == 0 ? __builtin_ctz(static_cast<unsigned>(page_size)) : -1, p.steps_per_split, p.nsplit,
                      scale * 1.4426950408889634f};
     if (p.nsplit > 1) {
         if (!workspace || workspace_bytes < pie_hip_latent_attn_rows_workspace_bytes(num_rows, heads, kvp, max_kv_len, max_tokens_per_req))
@@ -352,6 +381,6 @@ extern "C" int pie_hip_latent_attn_rows(const uint16_t* q, const uint16_t* pool,
 #undef PIE_LATENT_CASE
     if (st != PIE_HIP_OK || p.nsplit == 1) return st;
     hipLaunchKernelGGL(latent_merge_kernel, dim3(num_rows * heads), dim3(kvp / 4), 0, s, a.part_o, a.part_ml, row_kv_len, o,
-                       row0, heads, kvp, p.nsplit, p.steps_per_split * kStep);
+                       row0, heads, kvp, p.nsplit, p.steps_per_split);
     return launch_status();
 }
