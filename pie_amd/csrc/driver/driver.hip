@@ -863,7 +863,22 @@ extern "C" long long pie_hip_driver_snapshot_info(const char* dir, char* out, si
           << ",\"rms_eps\":" << m.rms_eps << ",\"rope_theta\":" << m.rope_theta
           << ",\"rope_factor\":" << m.rope_factor << ",\"tie_embeddings\":" << (m.tie_embeddings ? "true" : "false")
           << ",\"num_experts\":" << m.num_experts << ",\"top_k\":" << m.top_k
-          << ",\"expert_intermediate\":" << m.expert_intermediate << ",\"tensors\":{";
+          << ",\"expert_intermediate\":" << m.expert_intermediate << ",\"logit_scale\":" << m.logit_scale
+          << ",\"logit_softcap\":" << m.logit_softcap << ",\"stack\":[";
+        for (size_t i = 0; i < m.stack.size(); ++i) {
+            const LayerSpec& l = m.stack[i];
+            j << (i ? ",{" : "{") << "\"ff\":" << l.ff;
+            if (l.mixer == MixerKind::LatentAttention)
+                j << ",\"type\":\"latent_attention\",\"heads\":" << l.latent.heads << ",\"dim\":" << l.latent.dim
+                  << ",\"rot_dim\":" << l.latent.rot_dim << ",\"vdim\":" << l.latent.vdim << ",\"q_rank\":" << l.latent.q_rank
+                  << ",\"kv_rank\":" << l.latent.kv_rank << ",\"scale\":" << l.latent.scale << ",\"rot_dims\":" << l.latent.rot.dims
+                  << ",\"rot_base\":" << l.latent.rot.base << ",\"yarn\":" << (l.latent.rot.yarn ? "true" : "false");
+            else
+                j << ",\"type\":\"channel_delta\",\"heads\":" << l.delta.heads << ",\"kv_heads\":" << l.delta.kv_heads
+                  << ",\"dim\":" << l.delta.dim << ",\"vdim\":" << l.delta.vdim << ",\"conv\":" << l.delta.taps;
+            j << "}";
+        }
+        j << "],\"tensors\":{";
         bool first = true;
         for (const auto& [name, t] : snap.tensors()) {
             j << (first ? "" : ",") << "\"" << json_escape(name) << "\":{\"dtype\":\"" << t.dtype << "\",\"shape\":[";

@@ -353,6 +353,8 @@ def copy_kv_pages(pool: torch.Tensor, srcs: torch.Tensor, dsts: torch.Tensor) ->
            "pie_hip_copy_kv_pages")
 
 
+RELU2 = 2   # `swiglu` argument of the linears: squared-ReLU epilogue, all N columns
+
 FMT = {"int4b8": 0, "int8": 1, "fp8": 2, "bf16": 3}
 
 
@@ -369,7 +371,7 @@ def linear_fused(act: torch.Tensor, w: WeightView, norm_weight: Optional[torch.T
         _dev(norm_weight, torch.bfloat16, "norm_weight")
         if norm_weight.numel() != K:
             raise KernelError("norm weight must have K entries")
-    n_out = w.N // 2 if swiglu else w.N
+    n_out = w.N // 2 if swiglu is True or swiglu == 1 else w.N
     if y is None:
         if beta:
             raise KernelError("beta=1 needs an existing y")
@@ -414,7 +416,7 @@ def gemm_skinny(act: torch.Tensor, w: WeightView, y: Optional[torch.Tensor] = No
     M, K = act.shape
     if K != w.K:
         raise KernelError("act K != weight K")
-    n_out = w.N // 2 if swiglu else w.N
+    n_out = w.N // 2 if swiglu is True or swiglu == 1 else w.N
     if y is None:
         if beta:
             raise KernelError("beta=1 needs an existing y")
@@ -566,7 +568,7 @@ def gemm_mfma(act: torch.Tensor, w: WeightView, y: Optional[torch.Tensor] = None
     M, K = act.shape
     if K != w.K:
         raise KernelError("act K != weight K")
-    n_out = w.N // 2 if swiglu else w.N
+    n_out = w.N // 2 if swiglu is True or swiglu == 1 else w.N
     if y is None:
         if beta:
             raise KernelError("beta=1 needs an existing y")
@@ -1070,3 +1072,143 @@ def attention_rows_paged_kvq(fmt: str, q: torch.Tensor, k_pages: torch.Tensor, v
               _ptr(lse_t), _ptr(kv_page_indices), _ptr(row_page_begin), _ptr(row_kv_len), rows, hq, hk, d, ps,
               C.c_float(-1.0), max_kv, _ptr(ws), C.c_size_t(need), _stream()), "pie_hip_attn_rows_paged_kvq")
     return o, lse_t
+
+
+# ---------------------------------------------------------------- layer-stack kernels
+def _dt(t: torch.Tensor) -> int:
+    """Compute-type code of an activation tensor."""
+    if t.dtype not in (torch.bfloat16, torch.float32):
+        raise KernelError("compute type must be bfloat16 or float32")
+    return 0 if t.dtype == torch.bfloat16 else 1
+
+
+def norm_add(y: torch.Tensor, weight: torch.Tensor, x: torch.Tensor, eps: float) -> torch.Tensor:
+    """x += rmsnorm(y) * weight in place (fp32); returns the new x in y's type.  Rows of x may be
+    longer than the width (= len(weight))."""
+    _dev(weight, torch.float32, "weight")
+    _dev(x, torch.float32, "x")
+    _dev(y, y.dtype, "y")
+    xa = torch.zeros(x.shape, dtype=y.dtype, device=x.device)
+    _check(kernels().pie_hip_norm_add(_dt(y), _ptr(y), _ptr(weight), _ptr(x), _ptr(xa), x.shape[0], weight.numel(),
+                                      y.shape[1], x.shape[1], C.c_float(eps), _stream()), "pie_hip_norm_add")
+    return xa
+
+
+def norm_rows(x: torch.Tensor, rows: torch.Tensor, weight: torch.Tensor, eps: float, dtype) -> torch.Tensor:
+    out = torch.full((rows.numel(), x.shape[1]), 7.0, dtype=dtype, device=x.device)
+    _check(kernels().pie_hip_norm_rows(_dt(out), _ptr(x), _ptr(rows), _ptr(weight), _ptr(out), rows.numel(),
+                                       weight.numel(), x.shape[1], x.shape[0], C.c_float(eps), _stream()), "pie_hip_norm_rows")
+    return out
+
+
+def logits_finish(y: torch.Tensor, vocab: int, scale: float, cap: float):
+    logits = torch.empty((y.shape[0], vocab), dtype=torch.float32, device=y.device)
+    tokens = torch.empty(y.shape[0], dtype=torch.int32, device=y.device)
+    _check(kernels().pie_hip_logits_finish(_dt(y), _ptr(y), _ptr(logits), _ptr(tokens), y.shape[0], vocab, y.shape[1],
+                                           C.c_float(scale), C.c_float(cap), _stream()), "pie_hip_logits_finish")
+    return logits, tokens
+
+
+def rotary_table(positions: torch.Tensor, freq: torch.Tensor, mscale: float) -> torch.Tensor:
+    _dev(positions, torch.int32, "positions")
+    _dev(freq, torch.float64, "freq")
+    table = torch.empty((positions.numel(), 2 * freq.numel()), dtype=torch.float32, device=freq.device)
+    _check(kernels().pie_hip_rotary_table(_ptr(positions), _ptr(freq), _ptr(table), positions.numel(), 2 * freq.numel(),
+                                          C.c_float(mscale), _stream()), "pie_hip_rotary_table")
+    return table
+
+
+def linear_f32(act: torch.Tensor, w: torch.Tensor, relu2: bool = False) -> torch.Tensor:
+    _dev(act, torch.float32, "act")
+    _dev(w, torch.bfloat16, "w")
+    y = torch.empty((act.shape[0], w.shape[0]), dtype=torch.float32, device=act.device)
+    _check(kernels().pie_hip_linear_f32(_ptr(act), _ptr(w), _ptr(y), act.shape[0], w.shape[0], act.shape[1],
+                                        2 if relu2 else 0, _stream()), "pie_hip_linear_f32")
+    return y
+
+
+def head_linear(act: torch.Tensor, w: torch.Tensor, rope_table: Optional[torch.Tensor] = None, rot_dim: int = 0,
+                rot_dims: int = 0, rotp: int = 0) -> torch.Tensor:
+    """act [M, heads, A], w [heads, C, K] -> [M, heads, C + rotp]; the rotated part starts at K."""
+    M, heads, A = act.shape
+    _, n, k = w.shape
+    y = torch.full((M, heads, n + rotp), 3.0, dtype=act.dtype, device=act.device)
+    _check(kernels().pie_hip_head_linear(_dt(act), _ptr(act), _ptr(w), _ptr(y), _ptr(rope_table), M, heads, n, k,
+                                         heads * A, A, heads * (n + rotp), n + rotp, k, rot_dim, rot_dims, rotp, _stream()),
+           "pie_hip_head_linear")
+    return y
+
+
+def latent_attn_rows(q: torch.Tensor, pool: torch.Tensor, kvp: int, page_indices: torch.Tensor, row_begin: torch.Tensor,
+                     row_len: torch.Tensor, page_size: int, scale: float, row_req: Optional[torch.Tensor] = None,
+                     qo_indptr: Optional[torch.Tensor] = None, max_tokens: int = 1, plain: bool = False,
+                     max_kv_len: Optional[int] = None) -> torch.Tensor:
+    """q [rows, heads, ld], pool [slots, ld] -> o [rows, heads, kvp]."""
+    rows, heads, ld = q.shape
+    o = torch.full((rows, heads, kvp), 3.0, dtype=q.dtype, device=q.device)
+    longest = int(row_len.max()) if max_kv_len is None else max_kv_len
+    lib = kernels()
+    if plain:
+        _check(lib.pie_hip_latent_attn_rows_plain(_dt(q), _ptr(q), _ptr(pool), _ptr(o), _ptr(page_indices), _ptr(row_begin),
+                                                  _ptr(row_len), rows, heads, kvp, ld, page_size, C.c_float(scale), _stream()),
+               "pie_hip_latent_attn_rows_plain")
+        return o
+    lib.pie_hip_latent_attn_rows_workspace_bytes.restype = C.c_size_t
+    need = int(lib.pie_hip_latent_attn_rows_workspace_bytes(rows, heads, kvp, longest, max_tokens))
+    ws = torch.empty(max(need, 16), dtype=torch.uint8, device=q.device)
+    _check(lib.pie_hip_latent_attn_rows(_ptr(q), _ptr(pool), _ptr(o), _ptr(page_indices), _ptr(row_begin), _ptr(row_len),
+                                        _ptr(row_req), _ptr(qo_indptr), 0, rows, heads, kvp, ld - kvp, page_size,
+                                        C.c_float(scale), longest, max_tokens, _ptr(ws), C.c_size_t(need), _stream()),
+           "pie_hip_latent_attn_rows")
+    return o
+
+
+def latent_gather(pool: torch.Tensor, pages: torch.Tensor, num_keys: int, kvp: int, page_size: int):
+    ld = pool.shape[-1]
+    lat = torch.empty((num_keys, kvp), dtype=torch.bfloat16, device=pool.device)
+    rot = torch.empty((num_keys, ld - kvp), dtype=torch.bfloat16, device=pool.device)
+    _check(kernels().pie_hip_latent_gather(_ptr(pool), _ptr(pages), _ptr(lat), _ptr(rot), num_keys, kvp, ld - kvp, page_size,
+                                           _stream()), "pie_hip_latent_gather")
+    return lat, rot
+
+
+def latent_attn_prefill(q: torch.Tensor, kv: torch.Tensor, rot: torch.Tensor, rope_table: Optional[torch.Tensor],
+                        rot_dims: int, row_len: torch.Tensor, dimp: int, scale: float) -> torch.Tensor:
+    """q [rows, heads, dimp + rotp], kv [keys, heads, dimp + vdp], rot [keys, rotp] -> o [rows, heads * vdp]."""
+    rows, heads, _ = q.shape
+    vdp = kv.shape[2] - dimp
+    o = torch.full((rows, heads * vdp), 3.0, dtype=torch.bfloat16, device=q.device)
+    if int(row_len.max()) > kv.shape[0]:
+        raise KernelError("a row sees more keys than there are")
+    _check(kernels().pie_hip_latent_attn_prefill(_ptr(q), _ptr(kv), _ptr(rot), _ptr(o), _ptr(rope_table), _ptr(row_len), 0, rows,
+                                                 kv.shape[0], heads, dimp, rot.shape[1], rot_dims, vdp, heads * vdp,
+                                                 C.c_float(scale), _stream()), "pie_hip_latent_attn_prefill")
+    return o
+
+
+def delta_scan(q, k, v, log2_decay, beta, state, qo_indptr, slots, fresh, heads, kv_heads, chunked: bool = False):
+    """The recurrence over a batch's rows; state [slots, heads, dim, vdim] fp32 is updated in place.
+    q, k [N, kv_heads * dim], v [N, heads * vdim], log2_decay [N, heads * dim], beta [N, heads]."""
+    dim, vdim = state.shape[2], state.shape[3]
+    o = torch.full_like(v, 3.0)
+    stride, R = C.c_size_t(state.stride(0) * 4), slots.numel()
+    if not chunked:
+        _check(kernels().pie_hip_delta_scan(_ptr(q), _ptr(k), _ptr(v), _ptr(log2_decay), _ptr(beta), _ptr(o), _ptr(state), stride,
+                                            C.c_size_t(0), _ptr(qo_indptr), _ptr(slots), _ptr(fresh), R, heads, kv_heads, dim,
+                                            vdim, _stream()), "pie_hip_delta_scan")
+        return o
+    qo = qo_indptr.tolist()
+    chunks, first = [], [0]
+    for r in range(R):
+        chunks += [(i, min(16, qo[r + 1] - i)) for i in range(qo[r], qo[r + 1], 16)]
+        first.append(len(chunks))
+    lib = kernels()
+    lib.pie_hip_delta_chunked_workspace_bytes.restype = C.c_size_t
+    need = int(lib.pie_hip_delta_chunked_workspace_bytes(len(chunks), heads, dim))
+    ws = torch.empty(max(need, 16), dtype=torch.uint8, device=q.device)
+    ct = torch.tensor(chunks, dtype=torch.int32, device=q.device)
+    ft = torch.tensor(first, dtype=torch.int32, device=q.device)
+    _check(lib.pie_hip_delta_chunked(_ptr(q), _ptr(k), _ptr(v), _ptr(log2_decay), _ptr(beta), _ptr(o), _ptr(state), stride,
+                                     C.c_size_t(0), _ptr(ct), _ptr(ft), _ptr(qo_indptr), _ptr(slots), _ptr(fresh), len(chunks), R,
+                                     heads, kv_heads, dim, vdim, _ptr(ws), C.c_size_t(need), _stream()), "pie_hip_delta_chunked")
+    return o
