@@ -354,15 +354,15 @@ STACK_SIZES = {
 
 
 def stack_config(z: dict) -> dict:
-    rot = dict(dims=z["rot_dim"], base=500000.0, scaling=dict(factor=4.0, original=4096, fast=32.0, slow=1.0))
+    rot = dict(dims=z["rot_dim"], base=10000.0, scaling=dict(factor=4.0, original=4096, fast=24.0, slow=2.0))
     latent = dict(type="latent_attention", mlp=dict(kind="dense", ff=z["ff"]),
                   mixer=dict(heads=z["heads"], dim=z["dim"], rot_dim=z["rot_dim"], vdim=z["vdim"], q_rank=z["q_rank"],
                              kv_rank=z["kv_rank"], rot=rot, scale=(z["dim"] + z["rot_dim"]) ** -0.5))
     delta = dict(type="channel_delta", mlp=dict(kind="dense", ff=z["ff"]),
                  mixer=dict(heads=z["heads"], kv_heads=z["heads"], dim=z["dim"], vdim=z["vdim"], conv=4))
     layers = [delta if l % 3 == 2 else latent for l in range(z["layers"])]
-    return dict(architecture="Varasun", layers=layers, width=z["width"], vocab=z["vocab"], norm=dict(eps=1e-5),
-                logit_scale=0.5, logit_softcap=15.0)
+    return dict(architecture="Varasun", layers=layers, width=z["width"], vocab=z["vocab"], norm=dict(eps=1e-6),
+                logit_scale=0.25, logit_softcap=30.0)
 
 
 def stack_workload(args):
