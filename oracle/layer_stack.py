@@ -1,5 +1,6 @@
-"""Plain, slow statement of the layer-stack models (per-layer mixers: latent attention and the
-channel-decay delta rule) in numpy double precision.
+"""Plain, slow statement of the layer-stack models in numpy double precision: Varasun (latent attention,
+the channel-decay delta rule) and Lofudra (windowed attention beside retention, mLSTM, Mamba-2, a loop
+over some of the layers).
 
 One function per mechanism, whole sequences only: no cache, no pages, no batches.  Nothing here is
 shared with the product path; the tests compare the driver with it and plant their mistakes here.
@@ -35,6 +36,18 @@ def softplus(z):
 
 def squared_relu(z):
     return np.square(np.maximum(z, 0.0))
+
+
+def gelu_erf(z):
+    return 0.5 * z * (1.0 + np.vectorize(math.erf)(z / math.sqrt(2.0)))
+
+
+def log_sigmoid(z):
+    return -np.logaddexp(0.0, -z)
+
+
+def divide_by_rms(x, eps):
+    return x / np.sqrt(np.mean(x * x, axis=-1, keepdims=True) + eps)
 
 
 def rotation_frequencies(rot: dict):
@@ -132,15 +145,145 @@ def channel_delta(h, w, p, m, eps):
     return (rms_norm(o, w[p + "norm"], eps) * gate).reshape(T, H * dv) @ w[p + "o"].T
 
 
-MIXERS = {"latent_attention": latent_attention, "channel_delta": channel_delta}
+def rotate_halves(x, positions, rot: dict):
+    """Rotation of the first rot['dims'] entries, entry i with entry i + dims/2; x is [T, ..., n]."""
+    n = int(rot["dims"])
+    perm = np.arange(x.shape[-1])
+    perm[0:n:2], perm[1:n:2] = np.arange(n // 2), np.arange(n // 2, n)
+    out = np.empty_like(np.asarray(x, np.float64))
+    out[..., perm] = rotate_pairs(np.asarray(x)[..., perm], positions, rot)
+    return out
 
 
-def feed_forward(x, w, p):
-    return squared_relu(x @ w[p + "up"].T) @ w[p + "down"].T
+def window_mask(T, window):
+    """[T, T]: row i sees itself and the window - 1 columns before it (None: all before it)."""
+    d = np.arange(T)[:, None] - np.arange(T)[None, :]
+    return (d >= 0) & (d < (window if window else T + 1))
+
+
+def softmax_with_sink(scores, seen, sink=1.0):
+    """Weights of the seen columns; `sink` is added to the sum of exponentials."""
+    s = np.where(seen, scores, -np.inf)
+    m = np.maximum(s.max(axis=-1, keepdims=True), 0.0)
+    p = np.exp(s - m)
+    return p / (p.sum(axis=-1, keepdims=True) + sink * np.exp(-m))
+
+
+def window_attention(h, w, p, m, eps):
+    """Grouped-query attention over a sliding window; the raw keys are the values."""
+    T, H, G, dim = len(h), m["heads"], m["kv_heads"], m["dim"]
+    q = (h @ w[p + "q"].T + w[p + "q.b"]).reshape(T, H, dim)
+    k = (h @ w[p + "k"].T + w[p + "k.b"]).reshape(T, G, dim)
+    src = np.arange(H) // (H // G)
+    pos = np.arange(T)
+    v = k[:, src]
+    q = rotate_halves(rms_norm(q, w[p + "q.norm"], eps), pos, m["rot"])
+    k = rotate_halves(rms_norm(k, w[p + "k.norm"], eps), pos, m["rot"])[:, src]
+    a = softmax_with_sink(np.einsum("ihd,jhd->hij", q, k) * m["scale"], window_mask(T, m["mask"]["size"]))
+    return np.einsum("hij,jhd->ihd", a, v).reshape(T, -1) @ w[p + "o"].T
+
+
+def decayed_outer_products(q, k, v, decay):
+    """S_t = decay_t S_(t-1) + k_t v_t^T, o_t = S_t^T q_t: q, k [T, H, dk], v [T, H, dv], decay [T, H]."""
+    T, H, dk = q.shape
+    S = np.zeros((H, dk, v.shape[-1]))
+    out = np.empty(v.shape)
+    for t in range(T):
+        S = decay[t][:, None, None] * S + k[t][:, :, None] * v[t][:, None, :]
+        out[t] = np.einsum("hkv,hk->hv", S, q[t])
+    return out
+
+
+def retention(h, w, p, m, eps):
+    T, H, dk, dv = len(h), m["heads"], m["dim"], m["vdim"]
+    q, k, v = (h @ w[p + n].T for n in "qkv")
+    decay = np.broadcast_to(np.asarray(m["decay"], np.float64), (T, H))
+    o = decayed_outer_products(q.reshape(T, H, dk), k.reshape(T, H, dk) * dk ** -0.5, v.reshape(T, H, dv), decay)
+    return (divide_by_rms(o, eps).reshape(T, H * dv) * silu(h @ w[p + "g"].T)) @ w[p + "o"].T
+
+
+def parallel(h, w, p, m, eps):
+    return (m["left_scale"] * window_attention(h, w, p + "left.", m["left"], eps)
+            + m["right_scale"] * retention(h, w, p + "right.", m["right"], eps))
+
+
+def matrix_memory(q, k, v, i, f):
+    """Exponential input gate i and log forget gate f [T, H] with a running maximum from 0; q is scaled."""
+    T, H, dk = q.shape
+    S, n, m = np.zeros((H, dk, v.shape[-1])), np.zeros((H, dk)), np.zeros(H)
+    out = np.empty(v.shape)
+    for t in range(T):
+        m_new = np.maximum(f[t] + m, i[t])
+        keep, write = np.exp(f[t] + m - m_new), np.exp(i[t] - m_new)
+        S = keep[:, None, None] * S + write[:, None, None] * k[t][:, :, None] * v[t][:, None, :]
+        n = keep[:, None] * n + write[:, None] * k[t]
+        m = m_new
+        out[t] = np.einsum("hkv,hk->hv", S, q[t]) / (np.maximum(np.abs((n * q[t]).sum(-1)), np.exp(-m)) + 1e-6)[:, None]
+    return out
+
+
+def mlstm(h, w, p, m, eps):
+    T, H, dk, dv, cap = len(h), m["heads"], m["dim"], m["vdim"], m["gate_cap"]
+    q, k, v = (h @ w[p + n].T for n in "qkv")
+    i, f = (cap * np.tanh((h @ w[p + n].T + w[p + n + ".b"]) / cap) for n in "if")
+    o = matrix_memory(q.reshape(T, H, dk) * dk ** -0.5, k.reshape(T, H, dk), v.reshape(T, H, dv), i, log_sigmoid(f))
+    return (divide_by_rms(o, eps).reshape(T, H * dv) * w[p + "norm"] * sigmoid(h @ w[p + "g"].T)) @ w[p + "o"].T
+
+
+def mamba2(h, w, p, m, eps):
+    T, H, dv, N, G = len(h), m["heads"], m["vdim"], m["state"], m["groups"]
+    inner = H * dv
+    z, xbc, dt = np.split(h @ w[p + "in"].T, [inner, 2 * inner + 2 * G * N], axis=-1)
+    x, B, C = np.split(silu(causal_conv(xbc, w[p + "conv"]) + w[p + "conv.b"]), [inner, inner + G * N], axis=-1)
+    x, B, C = x.reshape(T, H, dv), B.reshape(T, G, N), C.reshape(T, G, N)
+    src = np.arange(H) // (H // G)
+    dt = softplus(dt + w[p + "dt_bias"])
+    y = decayed_outer_products(C[:, src], B[:, src], dt[:, :, None] * x, np.exp(-np.exp(w[p + "A_log"]) * dt))
+    y = (y + w[p + "D"][:, None] * x).reshape(T, inner) * silu(z)
+    y = divide_by_rms(y.reshape(T, m["norm_groups"], -1), eps).reshape(T, inner) * w[p + "norm"]
+    return y @ w[p + "o"].T
+
+
+MIXERS = {"latent_attention": latent_attention, "channel_delta": channel_delta, "parallel": parallel, "mlstm": mlstm,
+          "mamba2": mamba2}
+
+
+def feed_forward(x, w, p, act=squared_relu):
+    return act(x @ w[p + "up"].T) @ w[p + "down"].T
+
+
+def layer_runs(cfg):
+    """(layer, number of its pass, whether a looped pass begins here) in the order they are run."""
+    n = len(cfg["layers"])
+    loop = cfg.get("loop") or dict(start=n, stop=n, times=1)
+    a, b = loop["start"], loop["stop"]
+    looped = [(i, t, i == a) for t in range(loop["times"]) for i in range(a, b)]
+    return [(i, 0, False) for i in range(a)] + looped + [(i, 0, False) for i in range(b, n)]
+
+
+def forward_sandwich(cfg, w, tokens, want_layers=False):
+    """Norms ahead of and after every sublayer, some layers run several times with the same weights."""
+    eps = cfg["norm"]["eps"]
+    e = np.asarray(w["embed"], np.float64)[np.asarray(tokens)]
+    x, states = e, []
+    for i, t, begins in layer_runs(cfg):
+        layer, p = cfg["layers"][i], f"l{i}."
+        if begins:
+            x = x + (e if t > 0 else 0.0) + w["loop.step"][t]
+        y = MIXERS[layer["type"]](rms_norm(x, w[p + "norm1"], eps), w, p + "mix.", layer["mixer"], eps)
+        x = x + rms_norm(y, w[p + "norm1b"], eps)
+        if layer.get("mlp"):
+            y = feed_forward(rms_norm(x, w[p + "norm2"], eps), w, p + "mlp.", gelu_erf)
+            x = x + rms_norm(y, w[p + "norm2b"], eps)
+        states.append(x)
+    logits = rms_norm(x, w["final.norm"], eps) @ w["head"].T
+    return (logits, np.stack(states)) if want_layers else logits
 
 
 def forward(cfg, w, tokens, want_layers=False):
     """Logits [T, vocab] of one sequence (and the residual stream after every layer)."""
+    if cfg["architecture"] == "Lofudra":
+        return forward_sandwich(cfg, w, tokens, want_layers)
     eps = cfg["norm"]["eps"]
     x = np.asarray(w["embed"], np.float64)[np.asarray(tokens)]
     states = []
