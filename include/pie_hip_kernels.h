@@ -46,9 +46,11 @@ extern "C" {
  *      [pages, hk, page_size] (were [pages, page_size, hk]); int4 tile-major weights in decode
  *      order (pie_hip_repack_mfma_tiles_int4); pie_hip_gemv_time_next removed
  *   3  lm_head argmax pairs, attention merge in the output projection, uniform-row hints
- *   4  current: the `swiglu` argument of the linears is an epilogue code (PIE_HIP_EPI_*: 0 and 1
- *      mean what they did, 2 is the squared ReLU); the layer-stack kernels */
-#define PIE_HIP_ABI_VERSION 4
+ *   4  the `swiglu` argument of the linears is an epilogue code (PIE_HIP_EPI_*: 0 and 1
+ *      mean what they did, 2 is the squared ReLU); the layer-stack kernels
+ *   5  current: epilogue code 3 (exact GELU); grouped attention with windows and sinks, memories with
+ *      one decay per head, residual_norm */
+#define PIE_HIP_ABI_VERSION 5
 int pie_hip_abi_version(void);
 
 /* ---- W4A16 ("int4b8", symmetric, group-quantised) ------------------------- */
@@ -109,10 +111,12 @@ int pie_hip_gemv_w4a16_tuned(const uint16_t* act_bf16, const uint32_t* packed,
  * driver/cuda/src/model/llama_like.cpp:370-705.
  */
 /* Epilogue codes, the `swiglu` argument of every linear entry point: PIE_HIP_EPI_RELU2 stores
- * y[m, n] = bf16( max(sum, 0)^2 ) (all N columns; not combinable with beta). */
+ * y[m, n] = bf16( max(sum, 0)^2 ), PIE_HIP_EPI_GELU bf16( sum/2 (1 + erf(sum / sqrt 2)) ) (all N columns;
+ * not combinable with beta; GELU over bf16 weights only). */
 #define PIE_HIP_EPI_NONE 0
 #define PIE_HIP_EPI_SWIGLU 1
 #define PIE_HIP_EPI_RELU2 2
+#define PIE_HIP_EPI_GELU 3
 #define PIE_HIP_FMT_INT4B8 0
 #define PIE_HIP_FMT_INT8 1
 #define PIE_HIP_FMT_FP8 2
@@ -909,6 +913,132 @@ int pie_hip_delta_step(int dtype, const void* fused, const float* conv_w, const 
                        size_t conv_offset, const int32_t* rs_slot, const int32_t* rs_fresh, int num_requests, int ld,
                        int ld_gate, int ld_y, int heads, int kv_heads, int dim, int vdim, int taps, int write_conv,
                        float eps, void* stream);
+
+/* One step of the residual stream of layers with norms ahead of and after their sublayers:
+ *   x[n] = (read_x ? x[n] : 0) + y[n] / sqrt(mean(y[n]^2) + eps) * post_weight + table[token_ids[n]] + add
+ *   x_act[n] = x[n] / sqrt(mean(x[n]^2) + eps) * next_weight        (compute type)
+ * y with post_weight, token_ids with table_bf16, and add [width] may each be NULL (left out);
+ * next_weight NULL: x_act = x.  ids >= vocab read row 0.  Columns from the width to ld are not touched. */
+int pie_hip_residual_norm(int dtype, const void* y, const float* post_weight, float* x, int read_x,
+                          const uint32_t* token_ids, const uint16_t* table_bf16, int vocab, const float* add,
+                          const float* next_weight, void* x_act, int rows, int width, int ldy, int ld, float eps,
+                          void* stream);
+/* y[M, N] fp32 = act[M, K] . W[N, K]^T over bf16 weights (fp32 sums, not rounded): the few columns that
+ * drive a recurrence.  K % 32 == 0, N % 16 == 0. */
+int pie_hip_linear_f32out(int dtype, const void* act, const uint16_t* w_bf16, float* y, int M, int N, int K,
+                          void* stream);
+
+/*
+ * Grouped-query attention with an optional sliding window (a row sees its last `window` keys, itself
+ * included; 0: all), an optional sink (`sink` is added to the sum of exponentials; 0: none), and any
+ * head size.  Cache rows: [kv_heads][key dimp | value dimp], dim padded with zeros to dimp; the pool is
+ * [pages * page_size, row], one per layer run.
+ * pie_hip_group_attn_prep: fused[n] holds q (heads * dim from q_off), k and v (kv_heads * dim from k_off /
+ *   v_off; v_off < 0: the values are the keys as projected).  Biases (or NULL) are added, q and k are
+ *   normed per head (weights [dim], or NULL) and rotated over their first rot_dims entries, entry i
+ *   with entry i + rot_dims / 2 (table of pie_hip_rotary_table); q goes to q_out [N, heads, dimp].
+ * pie_hip_group_attn_rows: one query row per block row; rows NULL: rows 0 .. num_rows - 1, else the
+ *   listed ones.  o[row, h * dimp ..] * out_scale, rows of ld_o.  bf16; dimp / 32 in {1, 2, 3, 4, 6, 8};
+ *   page_size % 16 == 0.  Workspace pie_hip_group_attn_rows_workspace_bytes.
+ * pie_hip_group_attn_tiles: tiles [num_tiles][2] = (first row, rows) of consecutive rows of one request,
+ *   at most pie_hip_group_attn_tile_rows(heads, kv_heads, half) of them; half tiles only for dimp > 128.
+ * pie_hip_group_attn_plain: any size and compute type, dimp <= 1024.
+ */
+int pie_hip_group_attn_prep(int dtype, const void* fused, int q_off, int k_off, int v_off, const float* q_bias,
+                            const float* k_bias, const float* q_norm, const float* k_norm, const float* rope_table,
+                            int rot_dims, const int64_t* kv_slots, void* q_out, void* pool, int num_tokens,
+                            int ld_fused, int heads, int kv_heads, int dim, int dimp, float eps, void* stream);
+int pie_hip_group_attn_supported(int dimp);
+size_t pie_hip_group_attn_rows_workspace_bytes(int num_rows, int heads, int kv_heads, int dimp, int max_kv_len, int window);
+int pie_hip_group_attn_rows(const uint16_t* q, const uint16_t* pool, uint16_t* o, const uint32_t* kv_page_indices,
+                            const uint32_t* row_page_begin, const int32_t* row_kv_len, const int32_t* rows,
+                            int num_rows, int heads, int kv_heads, int dimp, int ld_o, int page_size, float scale,
+                            int window, float sink, float out_scale, int max_kv_len, void* workspace,
+                            size_t workspace_bytes, void* stream);
+int pie_hip_group_attn_tile_rows(int heads, int kv_heads, int half);
+int pie_hip_group_attn_tiles(const uint16_t* q, const uint16_t* pool, uint16_t* o, const uint32_t* kv_page_indices,
+                             const uint32_t* row_page_begin, const int32_t* row_kv_len, const int32_t* tiles,
+                             int num_tiles, int half, int heads, int kv_heads, int dimp, int ld_o, int page_size,
+                             float scale, int window, float sink, float out_scale, void* stream);
+int pie_hip_group_attn_plain(int dtype, const void* q, const void* pool, void* o, const uint32_t* kv_page_indices,
+                             const uint32_t* row_page_begin, const int32_t* row_kv_len, int num_rows, int heads,
+                             int kv_heads, int dimp, int ld_o, int page_size, float scale, int window, float sink,
+                             float out_scale, void* stream);
+
+/*
+ * Memories with one decay per head and token: S_t = d_t S_(t-1) + w_t k_t v_t^T (S [dim, vdim] fp32),
+ * o_t = S_t^T q_t.  Query and key heads may be shared: head h uses head h / (heads / kv_heads).
+ * The rule gives d_t and w_t (gates: fp32 rows of ld_gates values per token):
+ *   FIXED      d = 2^decay[head], w = k_scale                                         (retention)
+ *   EXP_GATES  i = cap tanh((gates[h] + gate_bias[h]) / cap), f = log sigmoid(cap tanh((gates[heads + h] +
+ *              gate_bias[heads + h]) / cap)), m_t = max(f + m_(t-1), i), d = exp(f + m_(t-1) - m_t), w =
+ *              exp(i - m_t); a vector n with v = 1 beside S; o is divided by max(|n . q|, exp(-m_t)) +
+ *              1e-6 in pie_hip_decay_out                                                       (mLSTM)
+ *   STEP       dt = softplus(gates[h] + gate_bias[h]), d = 2^(decay[h] dt), w = dt            (Mamba-2)
+ * o is also multiplied by q_scale.  A request's state: S [heads, dim, vdim], then (EXP_GATES) n [heads,
+ * dim] and m [heads] in units of log 2, at state_offset of its slot; the last taps - 1 inputs of a
+ * convolution ([taps - 1, channels], compute type) at conv_offset.
+ */
+#define PIE_HIP_DECAY_FIXED 0
+#define PIE_HIP_DECAY_EXP_GATES 1
+#define PIE_HIP_DECAY_STEP 2
+typedef struct {
+    int kind, heads, kv_heads, dim, vdim;
+    float q_scale, k_scale, gate_cap;
+    const float* decay;       /* [heads]: FIXED log2 of the decay; STEP -exp(A_log) log2(e) */
+    const float* gate_bias;   /* EXP_GATES [2 heads]; STEP [heads] */
+} PieHipDecayRule;
+/* Which rows of the batch a request owns and where its state lives. */
+typedef struct {
+    const int32_t* row_req;     /* [num_tokens] */
+    const int32_t* qo_indptr;   /* [num_requests + 1] */
+    const int32_t* rs_slot;     /* [num_requests] */
+    const int32_t* rs_fresh;    /* [num_requests] 1: starts from zero */
+    void* rs_base;
+    size_t rs_stride, state_offset, conv_offset;   /* bytes */
+    int num_tokens, num_requests;
+} PieHipStateRows;
+/* out[n, c] = silu(bias[c] + sum_j conv_w[c, j] * input_(n - (taps - 1) + j)[c]) for the first `channels`
+ * columns of fused (earlier inputs from the state, zeros before the start); rows of ld_out. */
+int pie_hip_conv_silu(int dtype, const void* fused, const float* conv_w, const float* conv_bias,
+                      const PieHipStateRows* rows, void* out, int ld, int channels, int taps, int ld_out, void* stream);
+/* Token by token, any compute type: q, k, v rows of ld values.  o [N, heads * vdim] fp32; den [N, heads, 2]
+ * (EXP_GATES: n . q and m_t).  dim <= 512. */
+int pie_hip_decay_scan(int dtype, const PieHipDecayRule* rule, const PieHipStateRows* rows, const void* q,
+                       const void* k, const void* v, int ld, const float* gates, int ld_gates, float* o, float* den,
+                       void* stream);
+/* 64 tokens at a time on the matrix cores (bf16).  chunks [num_chunks][2] = (first row, rows <= 64), a
+ * request's in order; req_chunks [num_requests + 1].  dim <= 512. */
+size_t pie_hip_decay_chunked_workspace_bytes(const PieHipDecayRule* rule, int num_chunks);
+int pie_hip_decay_chunked(const PieHipDecayRule* rule, const PieHipStateRows* rows, const uint16_t* q,
+                          const uint16_t* k, const uint16_t* v, int ld, const float* gates, int ld_gates, float* o,
+                          float* den, const int32_t* chunks, const int32_t* req_chunks, int num_chunks,
+                          void* workspace, size_t workspace_bytes, void* stream);
+/* y[n, h * vdim + c] = out_scale * o' / sqrt(mean(o'^2) + eps) * norm_w[h * vdim + c] * act(gate[n, h * vdim + c]),
+ * o' = o, divided for EXP_GATES as above (and m_t of a request's last row goes to its state).  norm_w may
+ * be NULL; gate_act 0: sigmoid, 1: silu. */
+int pie_hip_decay_out(int dtype, const PieHipDecayRule* rule, const PieHipStateRows* rows, const float* o,
+                      const float* den, const void* gate, int ld_gate, int gate_act, const float* norm_w, void* y,
+                      int ld_y, float out_scale, float eps, void* stream);
+/* One token per request (row r = request r), one launch: the state is read and written once.  conv_w not
+ * NULL: q, k, v are columns q_off, k_off, v_off of `fused` ahead of the convolution (conv_w [channels, taps] indexed
+ * by the same columns, the state is read, not moved on) and skip[head] * v is added to o.  y not NULL: with
+ * pie_hip_decay_out's norm and gate fused (one block per head then), else o and den.
+ * vdim % 4 == 0, dim <= 512, vdim <= 1024 (pie_hip_decay_step_supported). */
+int pie_hip_decay_step_supported(int dim, int vdim);
+int pie_hip_decay_step_fuses(const PieHipDecayRule* rule, int num_requests);
+int pie_hip_decay_step(int dtype, const PieHipDecayRule* rule, const PieHipStateRows* rows, const void* fused,
+                       int q_off, int k_off, int v_off, int ld, const float* gates, int ld_gates, const float* conv_w,
+                       const float* conv_bias, int channels, int taps, const float* skip, float* o, float* den,
+                       const void* gate, int ld_gate, int gate_act, const float* norm_w, void* y, int ld_y,
+                       float out_scale, float eps, void* stream);
+/* y = g / sqrt(mean over its part (g^2) + eps) * norm_w, g = (o + skip[head] * x) * silu(z), the heads * vdim
+ * values of a row in `parts` equal parts; x NULL: o as it is.  conv_w taps > 1 and conv_fused not NULL (one row
+ * per request): the convolution's state also moves on by the row's inputs. */
+int pie_hip_gated_part_norm(int dtype, const float* o, const void* x, int ld_x, const float* skip, const void* z,
+                            int ld_z, const float* norm_w, void* y, int ld_y, int heads, int vdim, int parts,
+                            const PieHipStateRows* rows, const void* conv_fused, int ld_fused, int channels, int taps,
+                            float eps, void* stream);
 
 /* pie_hip_sample_gather_logits over fp32 logits. */
 int pie_hip_sample_gather_logits_f32(const float* logits, const int32_t* rows, float* out_f32,

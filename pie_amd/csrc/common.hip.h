@@ -265,6 +265,30 @@ __device__ __forceinline__ void kv_decode_bf16_pairs(const typename KvVec<KVF>::
     }
 }
 
+// The epilogues of the linears that act on one value: the codes from PIE_HIP_EPI_RELU2 on (0: none).
+// Outputs are bf16, so erf is the five-term rational approximation of Abramowitz and Stegun, Handbook
+// of Mathematical Functions, 7.1.26 (absolute error under 1.5e-7): a quarter of the registers of the
+// library function, which the weight-streaming kernels need for loads in flight.  GELU: whether the
+// instance takes that code at all (linears over bf16 weights do).
+inline int pointwise_code(int epilogue) { return epilogue >= PIE_HIP_EPI_RELU2 ? epilogue : 0; }
+template <bool GELU>
+__device__ __forceinline__ float epilogue_pointwise(float v, int code) {
+    if (code == PIE_HIP_EPI_RELU2) {
+        v = fmaxf(v, 0.f);
+        v *= v;
+    } else if (GELU && code == PIE_HIP_EPI_GELU) {
+        const float x = fabsf(v) * 0.70710678118654752f;
+        const float t = __builtin_amdgcn_rcpf(fmaf(0.3275911f, x, 1.f));
+        float p = fmaf(1.061405429f, t, -1.453152027f);
+        p = fmaf(p, t, 1.421413741f);
+        p = fmaf(p, t, -0.284496736f);
+        p = fmaf(p, t, 0.254829592f);
+        const float q = 0.5f * p * t * __builtin_amdgcn_exp2f(-1.4426950408889634f * x * x);   // (1 - erf |x|) / 2
+        v *= v < 0.f ? q : 1.f - q;
+    }
+    return v;
+}
+
 inline int launch_status() {
     return hipGetLastError() == hipSuccess ? PIE_HIP_OK : PIE_HIP_ERR_LAUNCH;
 }

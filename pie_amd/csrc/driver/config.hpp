@@ -21,7 +21,7 @@ namespace pie_hip_driver {
 // Each layer names a mixer (what exchanges information between tokens) with its own sizes, and an
 // optional feed-forward.  Mixers are listed here once, with every constant a parameter.
 
-// Rotary embedding of the first `dims` entries of a vector, adjacent pairs.
+// Rotary embedding of the first `dims` entries of a vector (which entries pair up is the mixer's).
 struct RotarySpec {
     int dims = 0;
     double base = 10000.0;
@@ -46,18 +46,58 @@ struct ChannelDeltaSpec {
     int decay_rank = 0, gate_rank = 0;   // low-rank decay and output gate (a checkpoint's tensors fix them)
 };
 
-enum class MixerKind { LatentAttention, ChannelDelta };
+// Grouped-query attention: optional sliding window (0: none), optional sink (added to the sum of
+// exponentials), projections with biases, norms per head before a half-split rotation, values that are
+// the keys as projected.
+struct GroupAttentionSpec {
+    int heads = 0, kv_heads = 0, dim = 0, vdim = 0, window = 0;
+    double scale = 0.0;
+    float sink = 0.f;
+    RotarySpec rot;
+};
+
+// A memory S [dim, vdim] with one decay per head and token.  Retention: constant decays; MatrixLstm:
+// exponential gates with a running maximum and a normaliser; StateSpace (Mamba-2): step sizes, query and
+// key heads shared by groups, a short convolution with biases, a skip per head.
+enum class DecayKind { Retention, MatrixLstm, StateSpace };
+struct DecayMemorySpec {
+    DecayKind kind = DecayKind::Retention;
+    int heads = 0, kv_heads = 0, dim = 0, vdim = 0, taps = 1;
+    int norm_parts = 1;            // StateSpace: equal parts of the gated output that are normed on their own
+    double gate_cap = 0.0;         // MatrixLstm
+    std::vector<double> decay;     // Retention, one per head
+};
+
+// Attention and a memory side by side on the same input: attention_scale * a + memory_scale * m.
+enum class MixerKind { LatentAttention, ChannelDelta, DecayMemory, Parallel };
 
 struct LayerSpec {
     MixerKind mixer = MixerKind::LatentAttention;
     LatentAttentionSpec latent;
     ChannelDeltaSpec delta;
-    int ff = 0;   // squared-ReLU feed-forward of this width; 0: the layer has none
+    GroupAttentionSpec attn;       // Parallel
+    DecayMemorySpec memory;        // DecayMemory, Parallel
+    float attention_scale = 1.f, memory_scale = 1.f;
+    int ff = 0;   // width of the feed-forward (ModelConfig::ff_act between its two matrices); 0: the layer has none
+    bool has_attn() const { return mixer == MixerKind::Parallel; }
+    bool has_memory() const { return mixer == MixerKind::Parallel || mixer == MixerKind::DecayMemory; }
 };
+
+// Layers start .. stop - 1 run `times` times in a row with the same weights; every pass keeps its own
+// cache and state.
+struct LayerLoop {
+    int start = 0, stop = 0, times = 1;
+};
+struct LayerRun {
+    int layer, pass;
+    bool begins_pass;   // first layer of a pass of the loop
+};
+
+enum class FeedForwardAct { SquaredRelu, Gelu };
 
 struct ModelConfig {
     // architecture: "llama3" (dense, adjacent-pair RoPE) | "qwen3" (dense, qk-norm, half-split
-    // RoPE) | "qwen3_moe" | "varasun" (layer stack)
+    // RoPE) | "qwen3_moe" | "varasun", "lofudra" (layer stacks)
     std::string arch = "llama3";
     int hidden = 0, layers = 0, q_heads = 0, kv_heads = 0, head_dim = 0, intermediate = 0;
     int vocab = 0;
@@ -95,6 +135,23 @@ struct ModelConfig {
     // layer stacks: the layers, and what follows the last one (logits = cap * tanh(scale * y / cap);
     // cap 0: no cap).  Empty for the uniform architectures above.
     std::vector<LayerSpec> stack;
+    LayerLoop loop;                // stop 0: none
+    bool sandwich_norms = false;   // a norm ahead of every sublayer besides the one on its output
+    FeedForwardAct ff_act = FeedForwardAct::SquaredRelu;
+    std::vector<LayerRun> layer_runs() const {
+        std::vector<LayerRun> runs;
+        const int n = static_cast<int>(stack.size());
+        for (int l = 0; l < n; ++l) {
+            if (loop.stop > loop.start && l == loop.start) {
+                for (int t = 0; t < loop.times; ++t)
+                    for (int k = loop.start; k < loop.stop; ++k) runs.push_back({k, t, k == loop.start});
+                l = loop.stop - 1;
+            } else {
+                runs.push_back({l, 0, false});
+            }
+        }
+        return runs;
+    }
     float logit_scale = 1.f, logit_softcap = 0.f;
     bool is_stack() const { return !stack.empty(); }
     // activations and products: "bfloat16" | "float32" (layer stacks only: true 32-bit throughout)
@@ -258,12 +315,41 @@ inline void finalize_stack(DriverConfig& c) {
             if (a.rot.dims < 0 || a.rot.dims % 2 != 0 || a.rot.dims > a.rot_dim)
                 throw std::runtime_error(at + "rot.dims must be even and at most rot_dim");
             if (a.rot.dims > 0 && !(a.rot.base > 0.0)) throw std::runtime_error(at + "rot.base must be positive");
-        } else {
+        } else if (l.mixer == MixerKind::ChannelDelta) {
             const auto& d = l.delta;
             if (d.heads <= 0 || d.kv_heads <= 0 || d.dim <= 0 || d.vdim <= 0 || d.taps <= 0)
                 throw std::runtime_error(at + "channel_delta needs heads, kv_heads, dim, vdim, conv");
             if (d.heads % d.kv_heads != 0) throw std::runtime_error(at + "heads must be a multiple of kv_heads");
         }
+        if (l.has_attn()) {
+            const auto& a = l.attn;
+            if (a.heads <= 0 || a.kv_heads <= 0 || a.dim <= 0 || a.window < 0)
+                throw std::runtime_error(at + "attention needs heads, kv_heads, dim and a window that is not negative");
+            if (a.heads % a.kv_heads != 0) throw std::runtime_error(at + "heads must be a multiple of kv_heads");
+            if (a.vdim != a.dim) throw std::runtime_error(at + "values that are the keys have the keys' size");
+            if (a.dim > 1024) throw std::runtime_error(at + "attention heads are limited to 1024 values");
+            if (a.rot.dims < 0 || a.rot.dims % 2 != 0 || a.rot.dims > a.dim)
+                throw std::runtime_error(at + "rot.dims must be even and at most dim");
+            if (a.rot.dims > 0 && !(a.rot.base > 0.0)) throw std::runtime_error(at + "rot.base must be positive");
+        }
+        if (l.has_memory()) {
+            const auto& d = l.memory;
+            if (d.heads <= 0 || d.kv_heads <= 0 || d.dim <= 0 || d.vdim <= 0 || d.taps <= 0)
+                throw std::runtime_error(at + "a memory needs heads, key heads, dim, vdim (and conv)");
+            if (d.heads % d.kv_heads != 0) throw std::runtime_error(at + "heads must be a multiple of the groups");
+            if (d.dim > 512) throw std::runtime_error(at + "memories are limited to 512 key channels");
+            if (d.kind == DecayKind::Retention && d.decay.size() != static_cast<size_t>(d.heads))
+                throw std::runtime_error(at + "retention needs one decay per head");
+            for (double v : d.decay)
+                if (!(v >= 0.0 && v <= 1.0)) throw std::runtime_error(at + "decays must be between 0 and 1");
+            if (d.kind == DecayKind::MatrixLstm && !(d.gate_cap > 0.0)) throw std::runtime_error(at + "gate_cap must be positive");
+            if (d.norm_parts <= 0 || (d.heads * d.vdim) % d.norm_parts != 0)
+                throw std::runtime_error(at + "norm_groups must divide heads * vdim");
+        }
+    }
+    if (m.loop.stop != 0 || m.loop.start != 0) {
+        if (m.loop.start < 0 || m.loop.stop <= m.loop.start || m.loop.stop > static_cast<int>(m.stack.size()) || m.loop.times <= 0)
+            throw std::runtime_error("config: loop needs 0 <= start < stop <= layers and times > 0");
     }
     if (m.compute_dtype != "bfloat16" && m.compute_dtype != "float32")
         throw std::runtime_error("config: compute_dtype must be bfloat16 or float32");

@@ -864,7 +864,8 @@ extern "C" long long pie_hip_driver_snapshot_info(const char* dir, char* out, si
           << ",\"rope_factor\":" << m.rope_factor << ",\"tie_embeddings\":" << (m.tie_embeddings ? "true" : "false")
           << ",\"num_experts\":" << m.num_experts << ",\"top_k\":" << m.top_k
           << ",\"expert_intermediate\":" << m.expert_intermediate << ",\"logit_scale\":" << m.logit_scale
-          << ",\"logit_softcap\":" << m.logit_softcap << ",\"stack\":[";
+          << ",\"logit_softcap\":" << m.logit_softcap << ",\"loop\":[" << m.loop.start << "," << m.loop.stop << ","
+          << m.loop.times << "],\"stack\":[";
         for (size_t i = 0; i < m.stack.size(); ++i) {
             const LayerSpec& l = m.stack[i];
             j << (i ? ",{" : "{") << "\"ff\":" << l.ff;
@@ -873,9 +874,24 @@ extern "C" long long pie_hip_driver_snapshot_info(const char* dir, char* out, si
                   << ",\"rot_dim\":" << l.latent.rot_dim << ",\"vdim\":" << l.latent.vdim << ",\"q_rank\":" << l.latent.q_rank
                   << ",\"kv_rank\":" << l.latent.kv_rank << ",\"scale\":" << l.latent.scale << ",\"rot_dims\":" << l.latent.rot.dims
                   << ",\"rot_base\":" << l.latent.rot.base << ",\"yarn\":" << (l.latent.rot.yarn ? "true" : "false");
-            else
+            else if (l.mixer == MixerKind::ChannelDelta)
                 j << ",\"type\":\"channel_delta\",\"heads\":" << l.delta.heads << ",\"kv_heads\":" << l.delta.kv_heads
                   << ",\"dim\":" << l.delta.dim << ",\"vdim\":" << l.delta.vdim << ",\"conv\":" << l.delta.taps;
+            if (l.has_attn())
+                j << ",\"attention\":{\"heads\":" << l.attn.heads << ",\"kv_heads\":" << l.attn.kv_heads << ",\"dim\":" << l.attn.dim
+                  << ",\"vdim\":" << l.attn.vdim << ",\"window\":" << l.attn.window << ",\"scale\":" << l.attn.scale << ",\"sink\":" << l.attn.sink
+                  << ",\"rot_dims\":" << l.attn.rot.dims << ",\"rot_base\":" << l.attn.rot.base << "},\"attention_scale\":"
+                  << l.attention_scale << ",\"memory_scale\":" << l.memory_scale;
+            if (l.has_memory()) {
+                const DecayMemorySpec& d = l.memory;
+                static const char* kinds[] = {"retention", "mlstm", "mamba2"};
+                j << ",\"type\":\"" << (l.has_attn() ? "parallel" : kinds[static_cast<int>(d.kind)]) << "\",\"memory\":{\"kind\":\""
+                  << kinds[static_cast<int>(d.kind)] << "\",\"heads\":" << d.heads << ",\"kv_heads\":" << d.kv_heads << ",\"dim\":" << d.dim
+                  << ",\"vdim\":" << d.vdim << ",\"conv\":" << d.taps << ",\"norm_groups\":" << d.norm_parts << ",\"gate_cap\":" << d.gate_cap
+                  << ",\"decay\":[";
+                for (size_t k = 0; k < d.decay.size(); ++k) j << (k ? "," : "") << d.decay[k];
+                j << "]}";
+            }
             j << "}";
         }
         j << "],\"tensors\":{";

@@ -321,7 +321,7 @@ Executor::~Executor() {
     if (kv_shadow_k_) (void)hipFree(kv_shadow_k_);
     if (kv_shadow_v_) (void)hipFree(kv_shadow_v_);
     for (Growable* g : {&mask_in_host_, &mask_in_dev_, &mask_bitmap_, &tile_in_host_, &tile_in_dev_, &expand_lat_, &expand_rot_,
-                        &expand_kv_, &chunk_host_, &chunk_dev_, &delta_ws_}) g->release();
+                        &expand_kv_, &list_host_, &list_dev_, &record_ws_}) g->release();
     for (Growable* g : {&samp_f32_, &samp_ws_, &samp_in_dev_, &samp_in_host_, &samp_out_dev_, &samp_out_host_})
         g->release();
     if (swap_pool_) (void)hipHostFree(swap_pool_);
@@ -488,16 +488,20 @@ bool Executor::alloc_pools() {
         v_pool_.clear();
         k_scale_pool_.clear();
         v_scale_pool_.clear();
-        latent_pool_.clear();
+        run_pool_.clear();
         return false;
     };
     if (m.is_stack()) {
-        for (const LayerSpec& l : m.stack) {
-            latent_pool_.push_back(nullptr);
-            if (l.mixer != MixerKind::LatentAttention) continue;
+        for (const LayerRun& run : m.layer_runs()) {   // every pass of a looped layer has its own
+            const LayerSpec& l = m.stack[static_cast<size_t>(run.layer)];
+            run_pool_.push_back(nullptr);
+            const int row = l.mixer == MixerKind::LatentAttention ? LatentShape(l.latent).ld_row
+                            : l.has_attn()                        ? l.attn.kv_heads * 2 * pad_head(l.attn.dim)
+                                                                  : 0;
+            if (row == 0) continue;
             const size_t esize = m.f32() ? 4 : 2;
-            latent_pool_.back() = pool(static_cast<size_t>(page_size_) * LatentShape(l.latent).ld_row * esize);
-            if (!latent_pool_.back()) return give_up();
+            run_pool_.back() = pool(static_cast<size_t>(page_size_) * row * esize);
+            if (!run_pool_.back()) return give_up();
         }
         return true;
     }

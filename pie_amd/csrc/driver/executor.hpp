@@ -19,6 +19,11 @@
 //                     over the latent pool, out-projection
 //   channel delta     in-projection, convolution + unit vectors, decay and gate projections, the
 //                     recurrence over the request's state slot, norm + gate, out-projection
+//   decay memory      in-projection, fp32 gate columns, (convolution,) the recurrence over the request's
+//                     state slot, norm + gate, out-projection
+//   parallel          one in-projection, grouped attention and a decay memory on it, one out-projection
+// Architectures with norms ahead of their sublayers have the stream normed by the kernel that last
+// changed it; looped layers run several times, each pass with its own cache and state.
 //
 // Split into a host `prepare` (plan upload, outside any capture) and a device-only `body`
 // that is captured into a HIP graph per (rows, sampled rows, context bucket) for pure decode,
@@ -141,10 +146,15 @@ class Executor {
     void alloc_uniform();
     void alloc_stack();
     void prepare_stack(const BatchPlan& plan, const Inputs& in);   // host half: checks, state slots, row ranges
+    void prepare_lists(const BatchPlan& plan);
     void commit_stack(const BatchPlan& plan);                      // after success: the slots' new positions
     void stack_body(int N, int S, int max_kv_len);
     void stack_latent(const StackLayer& w, int layer, int N, int max_kv_len, const Inputs& in);
     void stack_delta(const StackLayer& w, int layer, int N, const Inputs& in);
+    void stack_mix(const StackLayer& w, int run, int N, int max_kv_len, const Inputs& in);
+    void stack_attention(const StackLayer& w, int run, int N, int max_kv_len, const Inputs& in);
+    void stack_memory(const StackLayer& w, int run, int N, const Inputs& in);
+    PieHipStateRows state_rows(int run, int N, const Inputs& in) const;
     void stack_linear(const Linear& w, const void* act, void* y, int M, int epilogue = PIE_HIP_EPI_NONE);
     void tune_linears();
 
@@ -215,9 +225,23 @@ class Executor {
     int n_tiles_ = 0, tile_rows_ = 0;
     // keys and values projected out of cached latents (the longest portion so far)
     Growable expand_lat_, expand_rot_, expand_kv_;
-    // delta rule over portions: the step's chunks and the chunk records
-    Growable chunk_host_, chunk_dev_, delta_ws_;
-    int n_chunks_ = 0;
+    // Recurrences and attention over portions: lists of the step (int32, back to back in one block) and
+    // the chunk records.  A chunk list is (first row, rows) per chunk, then each request's first chunk;
+    // attention tiles are (first row, rows), with the requests of one row listed apart.
+    struct ChunkList {
+        int n = 0;
+        size_t chunks = 0, first = 0;   // places in the block
+    };
+    struct TileList {
+        int n = 0, half = 0;
+        size_t tiles = 0;
+    };
+    Growable list_host_, list_dev_, record_ws_;
+    ChunkList chunks16_, chunks64_;     // of the delta rule, of the decay memories
+    std::map<std::tuple<int, int, int>, TileList> tile_lists_;   // by (heads, kv heads, padded head size)
+    size_t single_rows_ = 0;            // rows of the requests that bring one token
+    int n_single_ = 0;
+    const int32_t* list_at(size_t place) const { return static_cast<const int32_t*>(list_dev_.ptr) + place; }
     // custom attention masks of the current forward (never part of a captured graph)
     Growable mask_in_host_, mask_in_dev_, mask_bitmap_;
     int mask_stride_ = 0;
@@ -240,17 +264,19 @@ class Executor {
              *o = nullptr, *act = nullptr, *gate = nullptr,
              *xs = nullptr, *raw_logits = nullptr;
         float *dq = nullptr, *dk = nullptr, *dv = nullptr, *dg = nullptr, *d_beta = nullptr, *d_o = nullptr;
+        void* conv = nullptr;                                      // compute type: after a memory's convolution
+        float *gates = nullptr, *mem_o = nullptr, *den = nullptr;  // decay memories: gate columns, read-outs, divisors
         std::vector<float*> rotary;              // tables of the step, one per distinct rotation
         std::vector<void*> allocs;
     } stack_;
     int dt_ = PIE_HIP_DT_BF16;
     const BatchPlan* plan_ = nullptr;            // (while a forward is being enqueued)
     int n_requests_ = 0;
-    std::vector<unsigned char*> latent_pool_;    // per layer (null: no latent cache)
+    std::vector<unsigned char*> run_pool_;       // per layer run (null: no paged cache)
     unsigned char *rs_base_ = nullptr, *rs_host_ = nullptr;
     int rs_slots_ = 0, cpu_rs_slots_ = 0;
     size_t rs_stride_ = 0;                       // bytes per slot
-    std::vector<size_t> rs_state_off_, rs_conv_off_;   // per layer
+    std::vector<size_t> rs_state_off_, rs_conv_off_;   // per layer run
     std::vector<int64_t> rs_pos_, rs_host_pos_;  // tokens a slot's state has seen (-1: nothing)
 
     std::map<std::tuple<int, int, int, int>, hipGraphExec_t> graphs_;   // (rows, sampling slots, context bucket, rows equally long)

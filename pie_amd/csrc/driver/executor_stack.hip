@@ -1,6 +1,7 @@
 // Layer stacks in the executor: workspaces, recurrent-state slots, and the forward body of models
 // whose layers are listed one by one (ModelConfig::stack).
 #include <algorithm>
+#include <cmath>
 #include <cstring>
 #include <set>
 #include <stdexcept>
@@ -33,8 +34,15 @@ void Executor::alloc_stack() {
     const size_t ld_x = static_cast<size_t>(model_.ld_x());
     size_t in = 0, cq = 0, q = 0, q_lat = 0, o_lat = 0, o = 0, act = 0, gate = 0;
     size_t kd = 0, vd = 0, gd = 0, heads = 0, state = 0;
+    size_t conv = 0, gates = 0, mem_o = 0, den = 0, head_pad = 0;
     auto up = [](size_t& v, int n) { v = std::max(v, static_cast<size_t>(n)); };
-    for (const StackLayer& l : model_.stack) {
+    auto place = [&](size_t bytes) {
+        const size_t at = state;
+        state = (state + bytes + 255) / 256 * 256;
+        return at;
+    };
+    for (const LayerRun& run : model_.runs) {
+        const StackLayer& l = model_.stack[static_cast<size_t>(run.layer)];
         rs_state_off_.push_back(0);
         rs_conv_off_.push_back(0);
         up(act, l.spec.ff > 0 ? pad_to(l.spec.ff, 128) : 0);
@@ -46,7 +54,7 @@ void Executor::alloc_stack() {
             up(q_lat, s.heads * s.ld_row);
             up(o_lat, s.heads * s.kvp);
             up(o, s.ld_o);
-        } else {
+        } else if (l.spec.mixer == MixerKind::ChannelDelta) {
             const ChannelDeltaSpec& d = l.spec.delta;
             const DeltaShape s(d);
             up(in, s.ld_in);
@@ -56,13 +64,26 @@ void Executor::alloc_stack() {
             up(vd, s.vd);
             up(gd, d.heads * d.dim);
             up(heads, d.heads);
-            auto place = [&](size_t bytes) {
-                const size_t at = state;
-                state = (state + bytes + 255) / 256 * 256;
-                return at;
-            };
             rs_state_off_.back() = place(static_cast<size_t>(d.heads) * d.dim * d.vdim * 4);
             rs_conv_off_.back() = place(static_cast<size_t>(d.taps - 1) * s.channels * esize);
+        } else {
+            const MixShape s(l.spec);
+            const DecayMemorySpec& d = l.spec.memory;
+            up(in, s.ld_in);
+            up(o, s.ld_o);
+            if (l.spec.has_attn()) {
+                up(q, l.spec.attn.heads * s.dimp);
+                up(head_pad, s.dimp);
+            }
+            if (l.spec.has_memory()) {
+                up(conv, s.ld_conv);
+                up(gates, s.gates);
+                up(mem_o, d.heads * d.vdim);
+                up(den, 2 * d.heads);
+                const size_t per_head = static_cast<size_t>(d.dim) * d.vdim + (d.kind == DecayKind::MatrixLstm ? d.dim + 1 : 0);
+                rs_state_off_.back() = place(d.heads * per_head * 4);
+                if (s.channels) rs_conv_off_.back() = place(static_cast<size_t>(d.taps - 1) * s.channels * esize);
+            }
         }
     }
     // Zeroed: columns that pad a row to its product's K are written by nobody.
@@ -92,6 +113,10 @@ void Executor::alloc_stack() {
     stack_.dg = f32(T * gd);
     stack_.d_beta = f32(T * heads);
     stack_.d_o = f32(T * vd);
+    stack_.conv = compute(T * conv);
+    stack_.gates = f32(T * gates);
+    stack_.mem_o = f32(T * mem_o);
+    stack_.den = f32(T * den);
     const size_t srows = std::min<size_t>(T, 2 * static_cast<size_t>(cfg_.batching.max_forward_requests));
     stack_.xs = compute(srows * ld_x);
     stack_.raw_logits = compute(srows * static_cast<size_t>(model_.head.N));
@@ -104,15 +129,16 @@ void Executor::alloc_stack() {
                     gemm_ws_bytes_ = std::max(gemm_ws_bytes_, pie_hip_gemm_mfma_workspace_bytes(rows, w->N, w->K));
     gemm_ws_bytes_ = std::min<size_t>(gemm_ws_bytes_, size_t(64) << 20);
     if (gemm_ws_bytes_) PIE_HIP_CHECK(hipMalloc(&gemm_ws_, gemm_ws_bytes_));
-    // partial results of the latent attention's splits: a plan with more than one split has at most
-    // 512 (tile, split) blocks of 32 (token, head) pairs
+    // partial results of the attentions' splits: a plan with more than one split has at most 512 (tile,
+    // split) blocks of 32 (token, head) pairs (latent) or 16 heads (grouped)
     if (o_lat && !m.f32()) {
         size_t kvp = 0;
         for (const StackLayer& l : model_.stack)
             if (l.spec.mixer == MixerKind::LatentAttention) up(kvp, LatentShape(l.spec.latent).kvp);
         attn_ws_bytes_ = 512 * 32 * (kvp + 2) * sizeof(float);
-        PIE_HIP_CHECK(hipMalloc(&attn_ws_, attn_ws_bytes_));
     }
+    if (head_pad && !m.f32()) attn_ws_bytes_ = std::max(attn_ws_bytes_, 512 * 16 * (head_pad + 2) * sizeof(float));
+    if (attn_ws_bytes_) PIE_HIP_CHECK(hipMalloc(&attn_ws_, attn_ws_bytes_));
     rs_stride_ = state;
     if (state) {
         rs_slots_ = cfg_.batching.rs_cache_slots;
@@ -203,25 +229,75 @@ void Executor::prepare_stack(const BatchPlan& plan, const Inputs& in) {
     qo[plan.R] = plan.N;
     if (recurrent)
         for (int r = 0; r < plan.R; ++r) rs_pos_[plan.rs_slots[r]] = -1;   // (until the pass has succeeded)
-    if (recurrent && !plan.pure_decode) {
-        // the requests' rows in chunks of sixteen: (first row, rows), then each request's first chunk
-        std::vector<int32_t> chunks, first(1, 0);
-        for (int r = 0; r < plan.R; ++r) {
-            for (int i = plan.qo_indptr[r]; i < plan.qo_indptr[r + 1]; i += 16) {
-                chunks.push_back(i);
-                chunks.push_back(std::min(16, plan.qo_indptr[r + 1] - i));
-            }
-            first.push_back(static_cast<int32_t>(chunks.size() / 2));
-        }
-        n_chunks_ = static_cast<int>(chunks.size() / 2);
-        chunks.insert(chunks.end(), first.begin(), first.end());
-        chunk_host_.pinned = true;
-        chunk_host_.ensure(chunks.size() * 4);
-        chunk_dev_.ensure(chunks.size() * 4);
-        std::memcpy(chunk_host_.ptr, chunks.data(), chunks.size() * 4);
-        PIE_HIP_CHECK(hipMemcpyAsync(chunk_dev_.ptr, chunk_host_.ptr, chunks.size() * 4, hipMemcpyHostToDevice, stream_));
-    }
+    if (!plan.pure_decode) prepare_lists(plan);
     plan_ = &plan;
+}
+
+// What the kernels for portions walk: chunks of the recurrences, tiles of the attention.
+void Executor::prepare_lists(const BatchPlan& plan) {
+    bool delta = false, memory = false;
+    tile_lists_.clear();
+    std::vector<int32_t> all;
+    auto chunk_list = [&](int size) {
+        ChunkList l;
+        std::vector<int32_t> first(1, 0);
+        l.chunks = all.size();
+        for (int r = 0; r < plan.R; ++r) {
+            for (int i = plan.qo_indptr[r]; i < plan.qo_indptr[r + 1]; i += size) {
+                all.push_back(i);
+                all.push_back(std::min(size, plan.qo_indptr[r + 1] - i));
+                ++l.n;
+            }
+            first.push_back(l.n);
+        }
+        l.first = all.size();
+        all.insert(all.end(), first.begin(), first.end());
+        return l;
+    };
+    for (const StackLayer& l : model_.stack) {
+        delta |= l.spec.mixer == MixerKind::ChannelDelta;
+        memory |= l.spec.has_memory();
+        if (!l.spec.has_attn() || dt_ != PIE_HIP_DT_BF16) continue;
+        const GroupAttentionSpec& a = l.spec.attn;
+        const auto key = std::make_tuple(a.heads, a.kv_heads, pad_head(a.dim));
+        if (tile_lists_.count(key)) continue;
+        TileList t;
+        std::vector<std::pair<int, int>> tiles;   // (first row, rows)
+        // half tiles while whole ones would not give every CU two blocks, and for the widest heads
+        for (t.half = std::get<2>(key) > 128 ? 1 : 0;; t.half = 1) {
+            const int per = pie_hip_group_attn_tile_rows(a.heads, a.kv_heads, t.half);
+            tiles.clear();
+            for (int r = 0; r < plan.R; ++r) {
+                const int q0 = plan.qo_indptr[r], q1 = plan.qo_indptr[r + 1];
+                if (q1 - q0 < 2) continue;
+                for (int i = q0; i < q1; i += per) tiles.emplace_back(i, std::min(per, q1 - i));
+            }
+            if (t.half || tiles.size() * static_cast<size_t>(a.kv_heads) >= 512) break;
+        }
+        // (the ones that see most keys start first)
+        std::stable_sort(tiles.begin(), tiles.end(), [&](const auto& x, const auto& y) {
+            return plan.row_kv_len[x.first + x.second - 1] > plan.row_kv_len[y.first + y.second - 1];
+        });
+        t.n = static_cast<int>(tiles.size());
+        t.tiles = all.size();
+        for (const auto& [row, n] : tiles) {
+            all.push_back(row);
+            all.push_back(n);
+        }
+        tile_lists_[key] = t;
+    }
+    if (delta) chunks16_ = chunk_list(16);
+    if (memory) chunks64_ = chunk_list(64);
+    single_rows_ = all.size();
+    for (int r = 0; r < plan.R; ++r)
+        if (plan.qo_indptr[r + 1] - plan.qo_indptr[r] == 1) all.push_back(plan.qo_indptr[r]);
+    n_single_ = static_cast<int>(all.size() - single_rows_);
+    if (all.empty()) return;
+    list_host_.pinned = true;
+    list_host_.ensure(all.size() * 4);
+    list_dev_.ensure(all.size() * 4);
+    std::memcpy(list_host_.ptr, all.data(), all.size() * 4);
+    PIE_HIP_CHECK(hipMemcpyAsync(list_dev_.ptr, list_host_.ptr, all.size() * 4, hipMemcpyHostToDevice, stream_));
 }
 
 void Executor::commit_stack(const BatchPlan& plan) {
@@ -248,7 +324,7 @@ void Executor::stack_latent(const StackLayer& w, int layer, int N, int max_kv_le
     const auto* pages = reinterpret_cast<const uint32_t*>(in_dev_ + in.off_pages);
     const float* rope = w.rotary >= 0 ? stack_.rotary[static_cast<size_t>(w.rotary)] : nullptr;
     stack_linear(w.w_in, stack_.xa, stack_.in, N);
-    PIE_KERNEL(pie_hip_latent_prep(dt_, stack_.in, w.q_norm, w.kv_norm, rope, slots, stack_.cq, latent_pool_[layer], N,
+    PIE_KERNEL(pie_hip_latent_prep(dt_, stack_.in, w.q_norm, w.kv_norm, rope, slots, stack_.cq, run_pool_[layer], N,
                                    s.ld_in, s.kv_off, a.q_rank, s.ld_cq, a.kv_rank, s.kvp, a.rot_dim, a.rot.dims,
                                    s.ld_row, model_.cfg().rms_eps, stream_));
     stack_linear(w.w_uq, stack_.cq, stack_.q, N);
@@ -264,14 +340,14 @@ void Executor::stack_latent(const StackLayer& w, int layer, int N, int max_kv_le
                                        s.ld_q, s.hd, s.heads * s.ld_row, s.ld_row, s.dimp, a.rot_dim, a.rot.dims, s.rotp, stream_));
         if (matrix)
             PIE_KERNEL(pie_hip_latent_attn_rows(static_cast<const uint16_t*>(stack_.q_lat),
-                                                reinterpret_cast<const uint16_t*>(latent_pool_[layer]),
+                                                reinterpret_cast<const uint16_t*>(run_pool_[layer]),
                                                 static_cast<uint16_t*>(stack_.o_lat), pages, row_begin, row_len,
                                                 reinterpret_cast<const int32_t*>(in_dev_ + in.off_row_req),
                                                 reinterpret_cast<const int32_t*>(in_dev_ + in.off_qo), r0, n, s.heads, s.kvp,
                                                 s.rotp, page_size_, static_cast<float>(a.scale), max_len, max_tokens, attn_ws_,
                                                 attn_ws_bytes_, stream_));
         else
-            PIE_KERNEL(pie_hip_latent_attn_rows_plain(dt_, rows_of(stack_.q_lat, r0, s.heads * s.ld_row), latent_pool_[layer],
+            PIE_KERNEL(pie_hip_latent_attn_rows_plain(dt_, rows_of(stack_.q_lat, r0, s.heads * s.ld_row), run_pool_[layer],
                                                       rows_of(stack_.o_lat, r0, s.heads * s.kvp), pages, row_begin + r0, row_len + r0, n,
                                                       s.heads, s.kvp, s.ld_row, page_size_, static_cast<float>(a.scale), stream_));
         PIE_KERNEL(pie_hip_head_linear(dt_, rows_of(stack_.o_lat, r0, s.heads * s.kvp), w.w_uv, rows_of(stack_.o, r0, s.ld_o), nullptr, n,
@@ -305,7 +381,7 @@ void Executor::stack_latent(const StackLayer& w, int layer, int N, int max_kv_le
             auto* lat = static_cast<uint16_t*>(expand_lat_.ptr);
             auto* rot = static_cast<uint16_t*>(expand_rot_.ptr);
             auto* kv = static_cast<uint16_t*>(expand_kv_.ptr);
-            PIE_KERNEL(pie_hip_latent_gather(reinterpret_cast<const uint16_t*>(latent_pool_[layer]),
+            PIE_KERNEL(pie_hip_latent_gather(reinterpret_cast<const uint16_t*>(run_pool_[layer]),
                                              pages + plan_->row_page_begin[q0], lat, rot, ctx, s.kvp, s.rotp, page_size_, stream_));
             PIE_KERNEL(pie_hip_gemm_mfma(PIE_HIP_FMT_BF16, lat, w.w_ukv.data, nullptr, 0, 0, kv, ctx, w.w_ukv.N, w.w_ukv.K, 0,
                                          PIE_HIP_EPI_NONE, stream_));
@@ -351,17 +427,142 @@ void Executor::stack_delta(const StackLayer& w, int layer, int N, const Inputs& 
                                           rs_stride_, rs_state_off_[layer], qo, slot, fresh, n_requests_, d.heads, d.kv_heads,
                                           d.dim, d.vdim, stream_));
         } else {
-            delta_ws_.ensure(pie_hip_delta_chunked_workspace_bytes(n_chunks_, d.heads, d.dim));
-            const auto* chunks = static_cast<const int32_t*>(chunk_dev_.ptr);
+            record_ws_.ensure(pie_hip_delta_chunked_workspace_bytes(chunks16_.n, d.heads, d.dim));
             PIE_KERNEL(pie_hip_delta_chunked(stack_.dq, stack_.dk, stack_.dv, stack_.dg, stack_.d_beta, stack_.d_o, rs_base_,
-                                             rs_stride_, rs_state_off_[layer], chunks, chunks + 2 * n_chunks_, qo, slot, fresh,
-                                             n_chunks_, n_requests_, d.heads, d.kv_heads, d.dim, d.vdim, delta_ws_.ptr,
-                                             delta_ws_.cap, stream_));
+                                             rs_stride_, rs_state_off_[layer], list_at(chunks16_.chunks), list_at(chunks16_.first),
+                                             qo, slot, fresh, chunks16_.n, n_requests_, d.heads, d.kv_heads, d.dim, d.vdim,
+                                             record_ws_.ptr, record_ws_.cap, stream_));
         }
         PIE_KERNEL(pie_hip_delta_out(dt_, stack_.d_o, stack_.gate, w.out_norm, stack_.o, N, s.ld_gate, s.ld_o, d.heads, d.vdim,
                                      eps, stream_));
     }
     stack_linear(w.wo, stack_.o, stack_.y, N);
+}
+
+PieHipStateRows Executor::state_rows(int run, int N, const Inputs& in) const {
+    PieHipStateRows r{};
+    r.row_req = reinterpret_cast<const int32_t*>(in_dev_ + in.off_row_req);
+    r.qo_indptr = reinterpret_cast<const int32_t*>(in_dev_ + in.off_qo);
+    r.rs_slot = reinterpret_cast<const int32_t*>(in_dev_ + in.off_rs_slot);
+    r.rs_fresh = reinterpret_cast<const int32_t*>(in_dev_ + in.off_rs_fresh);
+    r.rs_base = rs_base_;
+    r.rs_stride = rs_stride_;
+    r.state_offset = rs_state_off_[static_cast<size_t>(run)];
+    r.conv_offset = rs_conv_off_[static_cast<size_t>(run)];
+    r.num_tokens = N;
+    r.num_requests = n_requests_;
+    return r;
+}
+
+// Attention and memory write their columns of the rows that W_o reads, scaled.
+void Executor::stack_mix(const StackLayer& w, int run, int N, int max_kv_len, const Inputs& in) {
+    const MixShape s(w.spec);
+    stack_linear(w.w_in, stack_.xa, stack_.in, N);
+    if (s.gates)
+        PIE_KERNEL(pie_hip_linear_f32out(dt_, stack_.xa, w.w_gates, stack_.gates, N, s.gates, w.w_in.K, stream_));
+    if (w.spec.has_attn()) stack_attention(w, run, N, max_kv_len, in);
+    if (w.spec.has_memory()) stack_memory(w, run, N, in);
+    stack_linear(w.wo, stack_.o, stack_.y, N);
+}
+
+void Executor::stack_attention(const StackLayer& w, int run, int N, int max_kv_len, const Inputs& in) {
+    const GroupAttentionSpec& a = w.spec.attn;
+    const MixShape s(w.spec);
+    const auto* row_begin = reinterpret_cast<const uint32_t*>(in_dev_ + in.off_row_begin);
+    const auto* row_len = reinterpret_cast<const int32_t*>(in_dev_ + in.off_row_len);
+    const auto* pages = reinterpret_cast<const uint32_t*>(in_dev_ + in.off_pages);
+    const float* rope = w.rotary >= 0 ? stack_.rotary[static_cast<size_t>(w.rotary)] : nullptr;
+    const float scale = static_cast<float>(a.scale), out_scale = w.spec.attention_scale;
+    unsigned char* pool = run_pool_[static_cast<size_t>(run)];
+    PIE_KERNEL(pie_hip_group_attn_prep(dt_, stack_.in, s.q_off, s.k_off, -1, w.q_bias, w.k_bias, w.q_norm, w.k_norm, rope, a.rot.dims,
+                                       reinterpret_cast<const int64_t*>(in_dev_ + in.off_slots), stack_.q, pool, N, s.ld_in, a.heads,
+                                       a.kv_heads, a.dim, s.dimp, model_.cfg().rms_eps, stream_));
+    if (dt_ != PIE_HIP_DT_BF16 || !pie_hip_group_attn_supported(s.dimp)) {
+        PIE_KERNEL(pie_hip_group_attn_plain(dt_, stack_.q, pool, stack_.o, pages, row_begin, row_len, N, a.heads, a.kv_heads, s.dimp, s.ld_o,
+                                            page_size_, scale, a.window, a.sink, out_scale, stream_));
+        return;
+    }
+    const auto* q = static_cast<const uint16_t*>(stack_.q);
+    const auto* kv = reinterpret_cast<const uint16_t*>(pool);
+    auto* o = static_cast<uint16_t*>(stack_.o);
+    auto rows_form = [&](const int32_t* rows, int n) {
+        PIE_KERNEL(pie_hip_group_attn_rows(q, kv, o, pages, row_begin, row_len, rows, n, a.heads, a.kv_heads, s.dimp, s.ld_o, page_size_,
+                                           scale, a.window, a.sink, out_scale, max_kv_len, attn_ws_, attn_ws_bytes_, stream_));
+    };
+    if (plan_->pure_decode) return rows_form(nullptr, N);
+    const TileList& t = tile_lists_.at(std::make_tuple(a.heads, a.kv_heads, s.dimp));
+    if (t.n)
+        PIE_KERNEL(pie_hip_group_attn_tiles(q, kv, o, pages, row_begin, row_len, list_at(t.tiles), t.n, t.half, a.heads, a.kv_heads, s.dimp,
+                                            s.ld_o, page_size_, scale, a.window, a.sink, out_scale, stream_));
+    if (n_single_) rows_form(list_at(single_rows_), n_single_);
+}
+
+void Executor::stack_memory(const StackLayer& w, int run, int N, const Inputs& in) {
+    const DecayMemorySpec& d = w.spec.memory;
+    const MixShape s(w.spec);
+    const bool ssm = d.kind == DecayKind::StateSpace;
+    const float head_scale = static_cast<float>(1.0 / std::sqrt(static_cast<double>(d.dim)));
+    PieHipDecayRule rule{};
+    rule.kind = d.kind == DecayKind::Retention    ? PIE_HIP_DECAY_FIXED
+                : d.kind == DecayKind::MatrixLstm ? PIE_HIP_DECAY_EXP_GATES
+                                                  : PIE_HIP_DECAY_STEP;
+    rule.heads = d.heads;
+    rule.kv_heads = d.kv_heads;
+    rule.dim = d.dim;
+    rule.vdim = d.vdim;
+    rule.q_scale = d.kind == DecayKind::MatrixLstm ? head_scale : 1.f;
+    rule.k_scale = d.kind == DecayKind::Retention ? head_scale : 1.f;
+    rule.gate_cap = static_cast<float>(d.gate_cap);
+    rule.decay = w.decay_log2;
+    rule.gate_bias = w.gate_bias;
+    const PieHipStateRows rows = state_rows(run, N, in);
+    const float eps = model_.cfg().rms_eps;
+    const size_t esize = dt_ == PIE_HIP_DT_F32 ? 4 : 2;
+    auto at = [&](void* base, int col) { return static_cast<unsigned char*>(base) + static_cast<size_t>(col) * esize; };
+    const void* gate = at(stack_.in, s.gate_off);
+    void* y = at(stack_.o, s.out_off);
+    const int gate_act = d.kind == DecayKind::Retention ? 1 : 0;   // silu, else the logistic function
+    const float scale = w.spec.memory_scale;
+    auto out = [&] {
+        PIE_KERNEL(pie_hip_decay_out(dt_, &rule, &rows, stack_.mem_o, stack_.den, gate, s.ld_in, gate_act, w.out_norm, y, s.ld_o, scale, eps,
+                                     stream_));
+    };
+    auto part_norm = [&](const void* x, const void* conv_fused) {
+        PIE_KERNEL(pie_hip_gated_part_norm(dt_, stack_.mem_o, x, s.ld_conv, w.skip, gate, s.ld_in, w.out_norm, y, s.ld_o, d.heads, d.vdim,
+                                           d.norm_parts, &rows, conv_fused, s.ld_in, s.channels, d.taps, eps, stream_));
+    };
+    if (plan_->pure_decode && pie_hip_decay_step_supported(d.dim, d.vdim)) {
+        const bool fuse = !ssm && pie_hip_decay_step_fuses(&rule, rows.num_requests);
+        PIE_KERNEL(pie_hip_decay_step(dt_, &rule, &rows, stack_.in, s.mq_off, s.mk_off, s.mv_off, s.ld_in, stack_.gates, s.gates,
+                                      ssm ? w.conv_w : nullptr, ssm ? w.conv_b : nullptr, s.channels, d.taps, ssm ? w.skip : nullptr,
+                                      stack_.mem_o, stack_.den, gate, s.ld_in, gate_act, w.out_norm, fuse ? y : nullptr, s.ld_o, scale, eps,
+                                      stream_));
+        if (ssm) part_norm(nullptr, stack_.in);
+        else if (!fuse) out();
+        return;
+    }
+    const void *q = at(stack_.in, s.mq_off), *k = at(stack_.in, s.mk_off), *v = at(stack_.in, s.mv_off);
+    int ld = s.ld_in;
+    if (ssm) {
+        PIE_KERNEL(pie_hip_conv_silu(dt_, stack_.in, w.conv_w, w.conv_b, &rows, stack_.conv, s.ld_in, s.channels, d.taps, s.ld_conv, stream_));
+        PIE_KERNEL(pie_hip_delta_conv_state(dt_, stack_.in, rs_base_, rs_stride_, rows.conv_offset, rows.qo_indptr, rows.rs_slot,
+                                            rows.rs_fresh, rows.num_requests, s.ld_in, s.channels, d.taps, stream_));
+        q = at(stack_.conv, s.mq_off);
+        k = at(stack_.conv, s.mk_off);
+        v = at(stack_.conv, s.mv_off);
+        ld = s.ld_conv;
+    }
+    if (dt_ == PIE_HIP_DT_BF16 && !plan_->pure_decode) {
+        record_ws_.ensure(pie_hip_decay_chunked_workspace_bytes(&rule, chunks64_.n));
+        PIE_KERNEL(pie_hip_decay_chunked(&rule, &rows, static_cast<const uint16_t*>(q), static_cast<const uint16_t*>(k),
+                                         static_cast<const uint16_t*>(v), ld, stack_.gates, s.gates, stack_.mem_o, stack_.den,
+                                         list_at(chunks64_.chunks), list_at(chunks64_.first), chunks64_.n, record_ws_.ptr, record_ws_.cap,
+                                         stream_));
+    } else {
+        PIE_KERNEL(pie_hip_decay_scan(dt_, &rule, &rows, q, k, v, ld, stack_.gates, s.gates, stack_.mem_o, stack_.den, stream_));
+    }
+    if (ssm) part_norm(stack_.conv, nullptr);
+    else out();
 }
 
 void Executor::stack_body(int N, int S, int max_kv_len) {
@@ -370,21 +571,50 @@ void Executor::stack_body(int N, int S, int max_kv_len) {
     const int H = m.hidden, ld = model_.ld_x();
     hipStream_t s = stream_;
     n_requests_ = plan_->R;
-    PIE_KERNEL(pie_hip_embed_stream(dt_, reinterpret_cast<const uint32_t*>(in_dev_ + in.off_tokens), model_.embed,
-                                    stack_.x, stack_.xa, N, H, ld, m.vocab, s));
+    const auto* tokens = reinterpret_cast<const uint32_t*>(in_dev_ + in.off_tokens);
+    const size_t n_runs = model_.runs.size();
+    auto layer_of = [&](size_t run) -> const StackLayer& { return model_.stack[static_cast<size_t>(model_.runs[run].layer)]; };
+    // What the stream takes on ahead of run `run` besides the last sublayer's output (`y` null: nothing yet),
+    // and the norm it is read through: a looped pass adds its step vector and, from the second pass on, the
+    // embedding again.
+    auto enter = [&](size_t run, const void* y, const float* post, int ldy, bool read_x) {
+        const bool more = run < n_runs, begins = more && model_.runs[run].begins_pass;
+        const int pass = more ? model_.runs[run].pass : 0;
+        const bool embed = !read_x || (begins && pass > 0);
+        PIE_KERNEL(pie_hip_residual_norm(dt_, y, post, stack_.x, read_x ? 1 : 0, embed ? tokens : nullptr, model_.embed, m.vocab,
+                                         begins ? model_.loop_step + static_cast<size_t>(pass) * H : nullptr,
+                                         more ? layer_of(run).pre1 : nullptr, stack_.xa, N, H, ldy, ld, m.rms_eps, s));
+    };
+    if (m.sandwich_norms) enter(0, nullptr, nullptr, 0, false);
+    else PIE_KERNEL(pie_hip_embed_stream(dt_, tokens, model_.embed, stack_.x, stack_.xa, N, H, ld, m.vocab, s));
     for (size_t i = 0; i < model_.rotary.size(); ++i)
         PIE_KERNEL(pie_hip_rotary_table(reinterpret_cast<const int32_t*>(in_dev_ + in.off_positions),
                                         model_.rotary[i].freq, stack_.rotary[i], N, model_.rotary[i].spec.dims,
                                         model_.rotary[i].mscale, s));
-    for (size_t l = 0; l < model_.stack.size(); ++l) {
-        const StackLayer& w = model_.stack[l];
-        if (w.spec.mixer == MixerKind::LatentAttention) stack_latent(w, static_cast<int>(l), N, max_kv_len, in);
-        else stack_delta(w, static_cast<int>(l), N, in);
-        PIE_KERNEL(pie_hip_norm_add(dt_, stack_.y, w.norm1, stack_.x, stack_.xa, N, H, w.wo.N, ld, m.rms_eps, s));
+    const int act = m.ff_act == FeedForwardAct::Gelu ? PIE_HIP_EPI_GELU : PIE_HIP_EPI_RELU2;
+    for (size_t r = 0; r < n_runs; ++r) {
+        const StackLayer& w = layer_of(r);
+        const int run = static_cast<int>(r);
+        switch (w.spec.mixer) {
+            case MixerKind::LatentAttention: stack_latent(w, run, N, max_kv_len, in); break;
+            case MixerKind::ChannelDelta: stack_delta(w, run, N, in); break;
+            default: stack_mix(w, run, N, max_kv_len, in); break;
+        }
+        // y joins the stream; `last`: the layer's last sublayer
+        auto finish = [&](const float* post, int ldy, bool last) {
+            if (!m.sandwich_norms)
+                PIE_KERNEL(pie_hip_norm_add(dt_, stack_.y, post, stack_.x, stack_.xa, N, H, ldy, ld, m.rms_eps, s));
+            else if (last)
+                enter(r + 1, stack_.y, post, ldy, true);
+            else
+                PIE_KERNEL(pie_hip_residual_norm(dt_, stack_.y, post, stack_.x, 1, nullptr, nullptr, 0, nullptr, w.pre2, stack_.xa, N, H,
+                                                 ldy, ld, m.rms_eps, s));
+        };
+        finish(w.norm1, w.wo.N, w.spec.ff == 0);
         if (w.spec.ff > 0) {
-            stack_linear(w.w_up, stack_.xa, stack_.act, N, PIE_HIP_EPI_RELU2);
+            stack_linear(w.w_up, stack_.xa, stack_.act, N, act);
             stack_linear(w.w_down, stack_.act, stack_.y, N);
-            PIE_KERNEL(pie_hip_norm_add(dt_, stack_.y, w.norm2, stack_.x, stack_.xa, N, H, w.w_down.N, ld, m.rms_eps, s));
+            finish(w.norm2, w.w_down.N, true);
         }
     }
     // the output norm and the head on the sampled rows only

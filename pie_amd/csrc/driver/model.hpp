@@ -96,9 +96,58 @@ struct DeltaShape {
           ld_gate(pad_to(vd, 16)), ld_o(pad_to(vd, 128)) {}
 };
 
+// (the head sizes the matrix-core attention is built for; wider ones take the plain kernel)
+constexpr int pad_head(int v) { return v <= 128 ? pad_to(v, 32) : v <= 256 ? pad_to(v, 64) : pad_to(v, 32); }
+// Grouped attention beside or without a memory, and a memory alone, behind one fused projection.
+struct MixShape {
+    int q_off = 0, k_off = 0, dimp = 0, ld_attn = 0;   // attention: query and key columns; output heads of dimp
+    int mq_off = 0, mk_off = 0, mv_off = 0, gate_off = 0;   // memory: columns of the fused projection
+    int channels = 0, ld_conv = 0;                     // StateSpace: convolved columns [values | keys | queries]
+    int gates = 0;                                     // fp32 gate columns, a product of their own
+    int out_off = 0, ld_in = 0, ld_o = 0;              // where the memory's output starts in the rows of W_o's input
+    explicit MixShape(const LayerSpec& l) {
+        int at = 0, out = 0;
+        auto place = [&](int n) {
+            const int here = at;
+            at = pad_to(at + n, 8);
+            return here;
+        };
+        const auto& d = l.memory;
+        const int kd = d.kv_heads * d.dim, vd = d.heads * d.vdim;
+        if (l.has_attn()) {
+            dimp = pad_head(l.attn.dim);
+            q_off = place(l.attn.heads * l.attn.dim);
+            k_off = place(l.attn.kv_heads * l.attn.dim);
+            out = ld_attn = pad_to(l.attn.heads * dimp, 16);
+        }
+        if (l.has_memory()) {
+            if (d.kind == DecayKind::StateSpace) {   // contiguous, so that one convolution covers them
+                mv_off = at;
+                mk_off = mv_off + vd;
+                mq_off = mk_off + kd;
+                channels = vd + 2 * kd;
+                ld_conv = pad_to(channels, 8);
+                at = pad_to(at + channels, 8);
+                gates = pad_to(d.heads, 16);
+            } else {
+                mq_off = place(kd);
+                mk_off = place(kd);
+                mv_off = place(vd);
+                if (d.kind == DecayKind::MatrixLstm) gates = pad_to(2 * d.heads, 16);
+            }
+            gate_off = place(vd);
+            out_off = out;
+            out += vd;
+        }
+        ld_in = pad_to(at, 16);
+        ld_o = pad_to(out, 128);
+    }
+};
+
 struct StackLayer {
     LayerSpec spec;
-    float *norm1 = nullptr, *norm2 = nullptr;
+    float *norm1 = nullptr, *norm2 = nullptr;   // on the sublayers' outputs
+    float *pre1 = nullptr, *pre2 = nullptr;     // ahead of the sublayers (null: none)
     Linear w_in;            // everything the mixer projects its input to, fused
     Linear wo;
     Linear w_up, w_down;    // feed-forward (none: data null)
@@ -110,6 +159,10 @@ struct StackLayer {
     int rotary = -1;                             // index into Model::rotary
     // channel delta
     uint16_t *w_decay = nullptr, *w_gate = nullptr;   // second factors of the low-rank decay and output gate
+    // grouped attention, decay memories (conv_w, dt_bias and out_norm as below)
+    float *q_bias = nullptr, *k_bias = nullptr, *k_norm = nullptr;
+    uint16_t* w_gates = nullptr;                     // [MixShape::gates, width]: the products that drive the recurrence
+    float *conv_b = nullptr, *skip = nullptr, *gate_bias = nullptr, *decay_log2 = nullptr;
     float *conv_w = nullptr, *decay_rate = nullptr /* -exp(A_log) log2(e) */, *dt_bias = nullptr, *out_norm = nullptr;
 };
 
@@ -166,6 +219,8 @@ class Model {
     std::vector<RotaryTable> rotary;   // the stack's distinct rotations
     Linear head;                       // lm_head, padded
     float* stack_norm = nullptr;       // norm ahead of it
+    float* loop_step = nullptr;        // [times, hidden]: added ahead of every pass of the loop
+    std::vector<LayerRun> runs;        // the layers in the order they are run
     int ld_x() const { return pad_to(cfg_.hidden, 128); }
 
     // bytes streamed from HBM by one decode step at batch 1 (every weight once)

@@ -161,12 +161,17 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
     linear(head, "head", pad_to(V, 16), Hp, H, [&](auto put) { plain_rows(put, "head", 0, V, H); });
     stack_norm = vec("final.norm", H, ones);
 
+    runs = cfg.layer_runs();
+    if (cfg.loop.stop > cfg.loop.start)
+        loop_step = vec("loop.step", static_cast<size_t>(cfg.loop.times) * H, [](size_t) { return 0.f; });
     stack.resize(cfg.stack.size());
     for (size_t l = 0; l < stack.size(); ++l) {
         StackLayer& w = stack[l];
         w.spec = cfg.stack[l];
+        const char *post1 = cfg.sandwich_norms ? "norm1b" : "norm1", *post2 = cfg.sandwich_norms ? "norm2b" : "norm2";
         const std::string p = "l" + std::to_string(l) + ".", mix = p + "mix.";
-        w.norm1 = vec(p + "norm1", H, ones);
+        w.norm1 = vec(p + post1, H, ones);
+        if (cfg.sandwich_norms) w.pre1 = vec(p + "norm1", H, ones);
         if (w.spec.mixer == MixerKind::LatentAttention) {
             const LatentAttentionSpec& a = w.spec.latent;
             const LatentShape s(a);
@@ -216,7 +221,7 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
                 for (int r = 0; r < H; ++r)
                     for (int h = 0; h < a.heads; ++h) put(r, h * s.vdp, m.row(r) + h * a.vdim, a.vdim);
             });
-        } else {
+        } else if (w.spec.mixer == MixerKind::ChannelDelta) {
             ChannelDeltaSpec& d = w.spec.delta;
             // the ranks of the decay and the output gate are the shapes of their first factors
             auto rank_of = [&](const std::string& name, int dflt) {
@@ -264,9 +269,106 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
             PIE_HIP_CHECK(hipMemcpyAsync(w.conv_w, conv.data(), conv.size() * 4, hipMemcpyHostToDevice, stream));
             PIE_HIP_CHECK(hipStreamSynchronize(stream));
         }
+        if (w.spec.has_attn() || w.spec.has_memory()) {
+            const MixShape s(w.spec);
+            const GroupAttentionSpec& a = w.spec.attn;
+            const DecayMemorySpec& d = w.spec.memory;
+            const int kd = d.kv_heads * d.dim, vd = d.heads * d.vdim;
+            const std::string left = mix + "left.", mem = w.spec.has_attn() ? mix + "right." : mix;
+            const bool ssm = w.spec.has_memory() && d.kind == DecayKind::StateSpace;
+            if (w.spec.has_attn()) {
+                w.rotary = rotary_of(a.rot);
+                auto zeros = [](size_t) { return 0.f; };
+                w.q_bias = vec(left + "q.b", static_cast<size_t>(a.heads) * a.dim, zeros);
+                w.k_bias = vec(left + "k.b", static_cast<size_t>(a.kv_heads) * a.dim, zeros);
+                w.q_norm = vec(left + "q.norm", a.dim, ones);
+                w.k_norm = vec(left + "k.norm", a.dim, ones);
+            }
+            // a state-space checkpoint's one projection: gate | values | keys | queries | step sizes
+            HostMatrix in;
+            if (ssm && !random) in = matrix(mem + "in", 2 * vd + 2 * kd + d.heads, H);
+            linear(w.w_in, mix + "in", s.ld_in, Hp, H, [&](auto put) {
+                if (w.spec.has_attn()) {
+                    plain_rows(put, left + "q", s.q_off, a.heads * a.dim, H);
+                    plain_rows(put, left + "k", s.k_off, a.kv_heads * a.dim, H);
+                }
+                if (ssm) {
+                    for (int r = 0; r < s.channels; ++r) put(s.mv_off + r, 0, in.row(vd + r), H);
+                    for (int r = 0; r < vd; ++r) put(s.gate_off + r, 0, in.row(r), H);
+                } else if (w.spec.has_memory()) {
+                    plain_rows(put, mem + "q", s.mq_off, kd, H);
+                    plain_rows(put, mem + "k", s.mk_off, kd, H);
+                    plain_rows(put, mem + "v", s.mv_off, vd, H);
+                    plain_rows(put, mem + "g", s.gate_off, vd, H);
+                }
+            });
+            if (s.gates) {
+                decode_bytes_ += static_cast<size_t>(s.gates) * Hp * 2;
+                w.w_gates = device_matrix(mix + "gates", static_cast<size_t>(s.gates) * Hp, H, [&](std::vector<uint16_t>& host) {
+                    auto rows = [&](const HostMatrix& m, int from, int to) {
+                        for (int r = 0; r < d.heads; ++r)
+                            std::memcpy(&host[static_cast<size_t>(to + r) * Hp], m.row(from + r), static_cast<size_t>(H) * 2);
+                    };
+                    if (ssm) {
+                        rows(in, vd + s.channels, 0);
+                    } else {
+                        rows(matrix(mem + "i", d.heads, H), 0, 0);
+                        rows(matrix(mem + "f", d.heads, H), 0, d.heads);
+                    }
+                });
+            }
+            auto upload_f32 = [&](const std::string& name, const std::vector<float>& v) {
+                float* dst = static_cast<float*>(alloc(v.size() * 4, name));
+                PIE_HIP_CHECK(hipMemcpyAsync(dst, v.data(), v.size() * 4, hipMemcpyHostToDevice, stream));
+                PIE_HIP_CHECK(hipStreamSynchronize(stream));
+                return dst;
+            };
+            if (w.spec.has_memory() && d.kind == DecayKind::Retention) {
+                // (a decay of 0 becomes a power of two that is 0 in fp32)
+                std::vector<float> lg;
+                for (double v : d.decay) lg.push_back(v > 0.0 ? static_cast<float>(std::max(std::log2(v), -1000.0)) : -1000.f);
+                w.decay_log2 = upload_f32("", lg);
+            } else if (w.spec.has_memory() && d.kind == DecayKind::MatrixLstm) {
+                std::vector<float> b(static_cast<size_t>(2 * d.heads), 0.f);
+                if (random) {
+                    std::fill(b.begin() + d.heads, b.end(), 3.f);
+                } else {
+                    size_t at = 0;
+                    for (const char* n : {"i.b", "f.b"}) {
+                        const StTensor& t = snap->at(mem + n);
+                        expect_shape(t, mem + n, d.heads, -1);
+                        std::vector<uint16_t> staging;
+                        const uint16_t* src = as_bf16(t, staging);
+                        for (int h = 0; h < d.heads; ++h) b[at++] = bf16_value(src[h]);
+                    }
+                }
+                w.gate_bias = upload_f32("", b);
+                w.out_norm = vec(mem + "norm", vd, ones);
+            } else if (ssm) {
+                w.decay_log2 = vec_mapped(mem + "A_log", d.heads, [&](size_t i) { return std::log(1.f + static_cast<float>(i % 8)); },
+                                          [](float v) { return static_cast<float>(-std::exp(static_cast<double>(v)) * 1.4426950408889634074); });
+                w.gate_bias = vec(mem + "dt_bias", d.heads, [](size_t) { return -3.f; });
+                w.skip = vec(mem + "D", d.heads, ones);
+                w.out_norm = vec(mem + "norm", vd, ones);
+                w.conv_b = vec(mem + "conv.b", s.channels, [](size_t) { return 0.f; });
+                w.conv_w = vec(mem + "conv", static_cast<size_t>(s.channels) * d.taps, [](size_t) { return 0.5f; });
+            }
+            linear(w.wo, mix + "o", Hp, s.ld_o, a.heads * a.vdim + vd, [&](auto put) {
+                if (w.spec.has_attn()) {
+                    const HostMatrix m = matrix(left + "o", H, a.heads * a.vdim);
+                    for (int r = 0; r < H; ++r)
+                        for (int h = 0; h < a.heads; ++h) put(r, h * s.dimp, m.row(r) + h * a.vdim, a.vdim);
+                }
+                if (w.spec.has_memory()) {
+                    const HostMatrix m = matrix(mem + "o", H, vd);
+                    for (int r = 0; r < H; ++r) put(r, s.out_off, m.row(r), vd);
+                }
+            });
+        }
         if (w.spec.ff > 0) {
             const int ff = w.spec.ff, ffp = pad_to(ff, 128);
-            w.norm2 = vec(p + "norm2", H, ones);
+            w.norm2 = vec(p + post2, H, ones);
+            if (cfg.sandwich_norms) w.pre2 = vec(p + "norm2", H, ones);
             linear(w.w_up, p + "mlp.up", ffp, Hp, H, [&](auto put) { plain_rows(put, p + "mlp.up", 0, ff, H); });
             linear(w.w_down, p + "mlp.down", Hp, ffp, ff, [&](auto put) { plain_rows(put, p + "mlp.down", 0, H, ff); });
         }

@@ -380,6 +380,44 @@ inline RotarySpec parse_rotary(const Json& j, const std::string& at) {
     return r;
 }
 
+// A mixer's sub-object (or the error that it is missing).
+inline const Json& json_object(const Json& j, const std::string& key, const std::string& at) {
+    const Json* v = j.get(key);
+    if (!v || v->kind != Json::Object) throw std::runtime_error("snapshot: " + at + " needs '" + key + "'");
+    return *v;
+}
+
+inline GroupAttentionSpec parse_group_attention(const Json& j, const std::string& at) {
+    GroupAttentionSpec a;
+    a.heads = json_size(j, "heads", at);
+    a.kv_heads = json_size(j, "kv_heads", at);
+    a.dim = json_size(j, "dim", at);
+    a.vdim = json_size(j, "vdim", at);
+    a.scale = json_number(j, "scale", at);
+    a.sink = 1.f;   // a sink of score 0
+    if (const Json* m = j.get("mask"); m && m->kind == Json::Object) {
+        a.window = json_size(*m, "size", at + " mask");
+        if (a.window <= 0) throw std::runtime_error("snapshot: " + at + ": mask.size must be positive");
+    }
+    if (const Json* r = j.get("rot"); r && r->kind == Json::Object) a.rot = parse_rotary(*r, at + " rot");
+    return a;
+}
+
+inline DecayMemorySpec parse_retention(const Json& j, const std::string& at) {
+    DecayMemorySpec d;
+    d.kind = DecayKind::Retention;
+    d.heads = d.kv_heads = json_size(j, "heads", at);
+    d.dim = json_size(j, "dim", at);
+    d.vdim = json_size(j, "vdim", at);
+    const Json* list = j.get("decay");
+    if (!list || list->kind != Json::Array) throw std::runtime_error("snapshot: " + at + " needs a list 'decay'");
+    for (const Json& v : list->arr) {
+        if (v.kind != Json::Number) throw std::runtime_error("snapshot: " + at + ": decay must hold numbers");
+        d.decay.push_back(v.num);
+    }
+    return d;
+}
+
 // One entry per mixer kind: config name -> reader of its sizes.
 struct MixerReader {
     const char* type;
@@ -411,14 +449,62 @@ inline const std::vector<MixerReader>& mixer_registry() {
              d.vdim = json_size(j, "vdim", at);
              d.taps = json_size(j, "conv", at);
          }},
+        {"parallel",
+         [](LayerSpec& l, const Json& j, const std::string& at) {
+             l.mixer = MixerKind::Parallel;
+             l.attn = parse_group_attention(json_object(j, "left", at), at + " left");
+             l.memory = parse_retention(json_object(j, "right", at), at + " right");
+             l.attention_scale = static_cast<float>(json_number(j, "left_scale", at));
+             l.memory_scale = static_cast<float>(json_number(j, "right_scale", at));
+         }},
+        {"mlstm",
+         [](LayerSpec& l, const Json& j, const std::string& at) {
+             l.mixer = MixerKind::DecayMemory;
+             auto& d = l.memory;
+             d.kind = DecayKind::MatrixLstm;
+             d.heads = d.kv_heads = json_size(j, "heads", at);
+             d.dim = json_size(j, "dim", at);
+             d.vdim = json_size(j, "vdim", at);
+             d.gate_cap = json_number(j, "gate_cap", at);
+         }},
+        {"mamba2",
+         [](LayerSpec& l, const Json& j, const std::string& at) {
+             l.mixer = MixerKind::DecayMemory;
+             auto& d = l.memory;
+             d.kind = DecayKind::StateSpace;
+             d.heads = json_size(j, "heads", at);
+             d.kv_heads = json_size(j, "groups", at);
+             d.dim = json_size(j, "state", at);
+             d.vdim = json_size(j, "vdim", at);
+             d.taps = json_size(j, "conv", at);
+             d.norm_parts = json_size(j, "norm_groups", at);
+         }},
+    };
+    return table;
+}
+
+// What sets one layer-stack architecture apart from another besides the mixers its layers name.
+struct StackArchitecture {
+    const char* name;   // config.json's "architecture"
+    const char* arch;
+    bool sandwich_norms;
+    FeedForwardAct ff_act;
+};
+inline const std::vector<StackArchitecture>& stack_registry() {
+    static const std::vector<StackArchitecture> table = {
+        {"Varasun", "varasun", false, FeedForwardAct::SquaredRelu},
+        {"Lofudra", "lofudra", true, FeedForwardAct::Gelu},
     };
     return table;
 }
 
 // {"architecture", "width", "vocab", "norm": {"eps"}, "logit_scale", "logit_softcap",
+//  "loop": {"start", "stop", "times"},
 //  "layers": [{"type", "mixer": {...}, "mlp": {"kind", "ff"} | null}, ...]}
-inline void apply_stack_config(ModelConfig& m, const Json& c) {
-    m.arch = "varasun";
+inline void apply_stack_config(ModelConfig& m, const Json& c, const StackArchitecture& a) {
+    m.arch = a.arch;
+    m.sandwich_norms = a.sandwich_norms;
+    m.ff_act = a.ff_act;
     m.hidden = json_size(c, "width", "config.json");
     m.vocab = json_size(c, "vocab", "config.json");
     const Json* norm = c.get("norm");
@@ -426,6 +512,12 @@ inline void apply_stack_config(ModelConfig& m, const Json& c) {
     m.rms_eps = static_cast<float>(json_number(*norm, "eps", "norm"));
     m.logit_scale = static_cast<float>(c.number_or("logit_scale", 1.0));
     m.logit_softcap = static_cast<float>(c.number_or("logit_softcap", 0.0));
+    m.loop = LayerLoop{};
+    if (const Json* loop = c.get("loop"); loop && loop->kind == Json::Object) {
+        m.loop.start = json_size(*loop, "start", "loop");
+        m.loop.stop = json_size(*loop, "stop", "loop");
+        m.loop.times = json_size(*loop, "times", "loop");
+    }
     const Json* layers = c.get("layers");
     if (!layers || layers->kind != Json::Array || layers->arr.empty())
         throw std::runtime_error("snapshot: config.json needs a list 'layers'");
@@ -510,7 +602,8 @@ inline void apply_hf_fields(ModelConfig& m, const Json& c, const std::string& ty
 inline void apply_hf_config(ModelConfig& m, const std::string& dir) {
     const Json c = parse_json_file(dir + "/config.json");
     const std::string arch = c.string_or("architecture", "");
-    if (arch == "Varasun") return apply_stack_config(m, c);
+    for (const StackArchitecture& a : stack_registry())
+        if (arch == a.name) return apply_stack_config(m, c, a);
     const std::string type = c.string_or("model_type", "");
     if (type.empty() && !arch.empty()) throw std::runtime_error("snapshot: unsupported architecture '" + arch + "'");
     apply_hf_fields(m, c, type);

@@ -50,7 +50,7 @@ struct GemmArgs {
     const unsigned char* scale;
     uint16_t* y;
     int M, N, K, g_shift, beta, swiglu, scale_is_bf16;
-    int relu2;        // 1: y = bf16(max(sum, 0)^2)
+    int pointwise;        // PIE_HIP_EPI_RELU2 and above: applied to the sum (0: nothing)
     float* partial;   // split-K: fp32 [gridDim.z][M][N] partial sums (row scale applied), else null
 };
 
@@ -381,10 +381,7 @@ __global__ __launch_bounds__(SH::kNW* kWave) void gemm_mfma_kernel(const GemmArg
                     }
                 } else if (ok) {
                     const size_t o = static_cast<size_t>(m) * nout + n;
-                    if (a.relu2) {
-                        v = fmaxf(v, 0.f);
-                        v *= v;
-                    }
+                    v = epilogue_pointwise<true>(v, a.pointwise);
                     if (a.beta) v += bf16_bits_to_f32(a.y[o]);
                     a.y[o] = f32_to_bf16_bits(v);
                 }
@@ -396,7 +393,7 @@ __global__ __launch_bounds__(SH::kNW* kWave) void gemm_mfma_kernel(const GemmArg
 // (residual add, or SwiGLU over adjacent (gate, up) columns with both rounded to bf16 first).
 __global__ __launch_bounds__(256) void gemm_splitk_reduce_kernel(const float* partial, uint16_t* y,
                                                                  int M, int N, int splits, int beta,
-                                                                 int swiglu, int relu2) {
+                                                                 int swiglu, int pointwise) {
     const int nout = swiglu ? N / 2 : N;
     const size_t idx = static_cast<size_t>(blockIdx.x) * 256 + threadIdx.x;
     if (idx >= static_cast<size_t>(M) * nout) return;
@@ -417,10 +414,7 @@ __global__ __launch_bounds__(256) void gemm_splitk_reduce_kernel(const float* pa
         const float* p = partial + static_cast<size_t>(m) * N + c;
         float v = 0.f;
         for (int z = 0; z < splits; ++z) v += p[z * plane];
-        if (relu2) {
-            v = fmaxf(v, 0.f);
-            v *= v;
-        }
+        v = epilogue_pointwise<true>(v, pointwise);
         if (beta) v += bf16_bits_to_f32(y[idx]);
         y[idx] = f32_to_bf16_bits(v);
     }
@@ -479,16 +473,16 @@ int splitk_shares(int M, int N, int K) {
 
 template <class F>
 int launch_gemm_splitk(GemmArgs a, int splits, float* ws, hipStream_t stream) {
-    const int beta = a.beta, swiglu = a.swiglu, relu2 = a.relu2;
+    const int beta = a.beta, swiglu = a.swiglu, pointwise = a.pointwise;
     a.partial = ws;
     a.beta = 0;
     a.swiglu = 0;
-    a.relu2 = 0;
+    a.pointwise = 0;
     const int st = a.M <= 64 ? launch_gemm_mt<F, 1, 8>(a, splits, stream) : launch_gemm_mt<F, 2, 8>(a, splits, stream);
     if (st != PIE_HIP_OK) return st;
     const size_t outs = static_cast<size_t>(a.M) * (swiglu ? a.N / 2 : a.N);
     hipLaunchKernelGGL(gemm_splitk_reduce_kernel, dim3(static_cast<unsigned>((outs + 255) / 256)), dim3(256), 0,
-                       stream, ws, a.y, a.M, a.N, splits, beta, swiglu, relu2);
+                       stream, ws, a.y, a.M, a.N, splits, beta, swiglu, pointwise);
     return launch_status();
 }
 
@@ -503,10 +497,10 @@ int gemm_entry(int format, const uint16_t* act_bf16, const void* weight, const v
     if (!act_bf16 || !weight || !y_bf16 || M <= 0 || N <= 0 || K <= 0) return PIE_HIP_ERR_INVALID;
     if (format != PIE_HIP_FMT_BF16 && !scale) return PIE_HIP_ERR_INVALID;
     if (K % BK != 0) return PIE_HIP_ERR_UNSUPPORTED;
-    const int relu2 = swiglu == PIE_HIP_EPI_RELU2 ? 1 : 0;
+    const int pointwise = pointwise_code(swiglu);
     swiglu = swiglu == PIE_HIP_EPI_SWIGLU ? 1 : 0;
     if (swiglu && (N % 2 != 0 || beta)) return PIE_HIP_ERR_INVALID;
-    if (relu2 && beta) return PIE_HIP_ERR_INVALID;
+    if (pointwise && beta) return PIE_HIP_ERR_INVALID;
     GemmArgs a{};
     a.act = act_bf16;
     a.w = static_cast<const unsigned char*>(weight);
@@ -517,7 +511,7 @@ int gemm_entry(int format, const uint16_t* act_bf16, const void* weight, const v
     a.K = K;
     a.beta = beta;
     a.swiglu = swiglu;
-    a.relu2 = relu2;
+    a.pointwise = pointwise;
     a.scale_is_bf16 = scale_is_bf16;
     hipStream_t st = static_cast<hipStream_t>(stream);
     if (format == PIE_HIP_FMT_INT4B8) {

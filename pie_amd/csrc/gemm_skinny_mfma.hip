@@ -31,6 +31,8 @@
 //     with one DPP move.
 #include "common.hip.h"
 
+#include <type_traits>
+
 namespace pie_hip {
 namespace {
 
@@ -125,7 +127,7 @@ struct SkinnyArgs {
     const int32_t* offsets;     // grouped: [P+1] first row of each problem; null: one problem
     int M;                      // rows when offsets == null
     int N, K, G, g_shift, beta, swiglu, scale_is_bf16;
-    int relu2;                  // 1: y = bf16(max(sum, 0)^2)
+    int pointwise;                  // PIE_HIP_EPI_RELU2 and above: applied to the sum (0: nothing)
     int m_split;                // dense only: blockIdx.y = 16-row pass
     int tiled;                  // weights (and int4 group scales) in the tile-major layout
     size_t w_stride, scale_stride;  // bytes between problems
@@ -401,10 +403,7 @@ __global__ __launch_bounds__(KP* kWave) void skinny_kernel(const SkinnyArgs a) {
                 }
             } else if (ok) {
                 const size_t o = static_cast<size_t>(m) * nout + n;
-                if (a.relu2) {
-                    v = fmaxf(v, 0.f);
-                    v *= v;
-                }
+                v = epilogue_pointwise<std::is_same<F, SkBf16>::value>(v, a.pointwise);
                 if (a.beta) v += bf16_bits_to_f32(a.y[o]);
                 a.y[o] = f32_to_bf16_bits(v);
             }
@@ -757,10 +756,7 @@ __global__ __launch_bounds__(kSwWaves* kWave, NG == 1 && MT == 1 ? 4 : 2) void s
                 }
             } else if (ok) {
                 const size_t o = static_cast<size_t>(m) * nout + n;
-                if (a.relu2) {
-                    v = fmaxf(v, 0.f);
-                    v *= v;
-                }
+                v = epilogue_pointwise<std::is_same<F, SkBf16>::value>(v, a.pointwise);
                 if (a.beta) v += bf16_bits_to_f32(a.y[o]);
                 a.y[o] = f32_to_bf16_bits(v);
             }
@@ -876,7 +872,7 @@ int launch_skinny(SkinnyArgs a, int problems, hipStream_t stream) {
         a.g_shift = __builtin_ctz(static_cast<unsigned>(a.G));
     }
     if (a.swiglu && (a.N % 2 != 0 || a.beta)) return PIE_HIP_ERR_INVALID;
-    if (a.relu2 && a.beta) return PIE_HIP_ERR_INVALID;
+    if (a.pointwise && a.beta) return PIE_HIP_ERR_INVALID;
     if (problems > 65535) return PIE_HIP_ERR_UNSUPPORTED;
     // Dense matrices with more than one 16-row pass: one block per (tile group, pass) instead
     // of a pass loop inside the block.  The passes then read the same weights at about the same
@@ -957,6 +953,7 @@ __global__ __launch_bounds__(256) void repack_scale_tiles_kernel(const uint16_t*
 }
 
 int dispatch_skinny(int format, const SkinnyArgs& a, int problems, hipStream_t st) {
+    if (a.pointwise == PIE_HIP_EPI_GELU && format != PIE_HIP_FMT_BF16) return PIE_HIP_ERR_UNSUPPORTED;
     switch (format) {
         case PIE_HIP_FMT_INT4B8: return launch_skinny<SkInt4>(a, problems, st);
         case PIE_HIP_FMT_INT8: return launch_skinny<SkInt8>(a, problems, st);
@@ -987,7 +984,7 @@ extern "C" int pie_hip_gemm_skinny(int format, const uint16_t* act_bf16, const v
     a.G = group_size;
     a.beta = beta;
     a.swiglu = swiglu == PIE_HIP_EPI_SWIGLU ? 1 : 0;
-    a.relu2 = swiglu == PIE_HIP_EPI_RELU2 ? 1 : 0;
+    a.pointwise = pointwise_code(swiglu);
     a.scale_is_bf16 = scale_is_bf16;
     return dispatch_skinny(format, a, 1, static_cast<hipStream_t>(stream));
 }
@@ -1016,7 +1013,7 @@ extern "C" int pie_hip_moe_grouped_gemm(int format, const uint16_t* act_bf16,
     a.K = K;
     a.G = group_size;
     a.swiglu = swiglu == PIE_HIP_EPI_SWIGLU ? 1 : 0;
-    a.relu2 = swiglu == PIE_HIP_EPI_RELU2 ? 1 : 0;
+    a.pointwise = pointwise_code(swiglu);
     a.scale_is_bf16 = scale_is_bf16;
     a.w_stride = weight_stride_bytes;
     a.scale_stride = scale_stride_bytes;
@@ -1042,7 +1039,7 @@ extern "C" int pie_hip_gemm_skinny_tiled(int format, const uint16_t* act_bf16, c
     a.G = group_size;
     a.beta = beta;
     a.swiglu = swiglu == PIE_HIP_EPI_SWIGLU ? 1 : 0;
-    a.relu2 = swiglu == PIE_HIP_EPI_RELU2 ? 1 : 0;
+    a.pointwise = pointwise_code(swiglu);
     a.scale_is_bf16 = scale_is_bf16;
     a.tiled = 1;
     return dispatch_skinny(format, a, 1, static_cast<hipStream_t>(stream));
@@ -1109,7 +1106,7 @@ extern "C" int pie_hip_moe_grouped_gemm_tiled(int format, const uint16_t* act_bf
     a.K = K;
     a.G = group_size;
     a.swiglu = swiglu == PIE_HIP_EPI_SWIGLU ? 1 : 0;
-    a.relu2 = swiglu == PIE_HIP_EPI_RELU2 ? 1 : 0;
+    a.pointwise = pointwise_code(swiglu);
     a.scale_is_bf16 = scale_is_bf16;
     a.tiled = 1;
     a.w_stride = weight_stride_bytes;

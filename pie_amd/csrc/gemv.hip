@@ -280,7 +280,7 @@ struct GemvArgs {
     const float* mg_part_ml;     // [M, hq, nsplit, 2] f32 (max, sum)
     const int32_t* mg_row_len;   // visible keys per row
     int mg_nsplit, mg_units_per_split, mg_hq, mg_d;
-    int relu2;   // 1: y = bf16(max(sum, 0)^2)
+    int pointwise;   // PIE_HIP_EPI_RELU2 and above: applied to the sum (0: nothing)
 };
 
 // attn_decode_merge_kernel's arithmetic for the eight output dimensions d0 .. d0 + 7 of one
@@ -762,10 +762,7 @@ __global__ __launch_bounds__(kBlock) void gemv_kernel(const GemvArgs a) {
                 const int row = row_begin + g * R + lane / M;
                 if (lane < R * M && row < row_end) {
                     if constexpr (F::kRowScale) mine *= u.rs;
-                    if (a.relu2) {
-                        mine = fmaxf(mine, 0.f);
-                        mine *= mine;
-                    }
+                    mine = epilogue_pointwise<std::is_same<F, FmtBf16>::value>(mine, a.pointwise);
                     const float prev = a.beta ? bf16_bits_to_f32(u.prev) : 0.f;
                     const uint16_t out = f32_to_bf16_bits(mine + prev);
                     a.y[static_cast<size_t>(lane % M) * N + row] = out;
@@ -1119,8 +1116,9 @@ extern "C" int pie_hip_linear_fused(int format, const uint16_t* act_bf16,
     using namespace pie_hip;
     GemvArgs a{act_bf16, static_cast<const u32x4_t*>(weight), nullptr, nullptr, y_bf16, N, K,
                group_size, beta, norm_weight_bf16, eps, swiglu == PIE_HIP_EPI_SWIGLU ? 1 : 0};
-    a.relu2 = swiglu == PIE_HIP_EPI_RELU2 ? 1 : 0;
-    if (a.relu2 && beta) return PIE_HIP_ERR_INVALID;
+    a.pointwise = pointwise_code(swiglu);
+    if (a.pointwise && beta) return PIE_HIP_ERR_INVALID;
+    if (a.pointwise == PIE_HIP_EPI_GELU && format != PIE_HIP_FMT_BF16) return PIE_HIP_ERR_UNSUPPORTED;
     hipStream_t st = static_cast<hipStream_t>(stream);
     switch (format) {
         case PIE_HIP_FMT_INT4B8:

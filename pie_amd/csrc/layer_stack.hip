@@ -95,6 +95,146 @@ __global__ __launch_bounds__(BLOCK) void norm_add_kernel(const T* __restrict__ y
     }
 }
 
+// Layers with norms ahead of and after their sublayers: x takes a sublayer's normed output and whatever
+// else enters the stream (a row of the embedding table, a vector), and its compute-type copy is normed
+// for the next sublayer.  One block per row, up to 8192 values of the row in registers between the
+// passes; wider rows go through memory again.
+struct ResidualArgs {
+    const void* y;
+    const float *post_w, *add, *next_w;
+    float* x;
+    const uint32_t* tokens;
+    const uint16_t* table;
+    void* xa;
+    int read_x, vocab, width, ldy, ld;
+    float eps;
+};
+template <class T, int BLOCK>
+__global__ __launch_bounds__(BLOCK) void residual_norm_kernel(const ResidualArgs a) {
+    __shared__ float red[BLOCK / kWave];
+    const size_t n = blockIdx.x;
+    const T* yr = a.y ? static_cast<const T*>(a.y) + n * a.ldy : nullptr;
+    float* xr = a.x + n * a.ld;
+    T* ar = static_cast<T*>(a.xa) + n * a.ld;
+    const uint16_t* er = nullptr;
+    if (a.tokens) {
+        const uint32_t t = a.tokens[n];
+        er = a.table + static_cast<size_t>(t < static_cast<uint32_t>(a.vocab) ? t : 0) * a.width;
+    }
+    constexpr int kCache = 2048 / BLOCK;   // groups of four
+    const int n4 = a.width % 4 == 0 ? a.width / 4 : 0;   // (a table row of another width is not aligned)
+    const int done = min(n4, kCache * BLOCK) * 4;
+    f32x4_t yv[kCache], xv[kCache], wv[kCache], nv[kCache];
+    const f32x4_t zero = {0.f, 0.f, 0.f, 0.f};
+    float local = 0.f;
+#pragma unroll
+    for (int c = 0; c < kCache; ++c) {
+        const int i = threadIdx.x + c * BLOCK;
+        if (i >= n4) break;
+        yv[c] = wv[c] = zero;
+        if (yr) {
+            if constexpr (sizeof(T) == 2) {
+                const u32x2_t r = *reinterpret_cast<const u32x2_t*>(yr + 4 * i);
+                yv[c] = f32x4_t{bf16_lo(r.x), bf16_hi(r.x), bf16_lo(r.y), bf16_hi(r.y)};
+            } else {
+                yv[c] = *reinterpret_cast<const f32x4_t*>(yr + 4 * i);
+            }
+            wv[c] = *reinterpret_cast<const f32x4_t*>(a.post_w + 4 * i);
+        }
+        xv[c] = a.read_x ? *reinterpret_cast<const f32x4_t*>(xr + 4 * i) : zero;
+        if (er) {
+            const u32x2_t r = *reinterpret_cast<const u32x2_t*>(er + 4 * i);
+            xv[c] += f32x4_t{bf16_lo(r.x), bf16_hi(r.x), bf16_lo(r.y), bf16_hi(r.y)};
+        }
+        if (a.next_w) nv[c] = *reinterpret_cast<const f32x4_t*>(a.next_w + 4 * i);
+    }
+    auto other = [&](int i) {   // what joins x besides the sublayer's output, beyond the cached part
+        return (a.read_x ? xr[i] : 0.f) + (er ? bf16_bits_to_f32(er[i]) : 0.f) + (a.add ? a.add[i] : 0.f);
+    };
+    float inv = 0.f;
+    if (yr) {
+#pragma unroll
+        for (int c = 0; c < kCache; ++c)
+            if (threadIdx.x + c * BLOCK < n4)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) local += yv[c][e] * yv[c][e];
+        for (int i = done + threadIdx.x; i < a.width; i += BLOCK) {
+            const float v = act_get<T>(yr[i]);
+            local += v * v;
+        }
+        inv = 1.f / sqrtf(block_total(local, red) / static_cast<float>(a.width) + a.eps);
+    }
+    local = 0.f;
+#pragma unroll
+    for (int c = 0; c < kCache; ++c) {
+        const int i = threadIdx.x + c * BLOCK;
+        if (i >= n4) break;
+        if (a.add) xv[c] += *reinterpret_cast<const f32x4_t*>(a.add + 4 * i);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            xv[c][e] += yv[c][e] * inv * wv[c][e];
+            local += xv[c][e] * xv[c][e];
+        }
+        *reinterpret_cast<f32x4_t*>(xr + 4 * i) = xv[c];
+    }
+    for (int i = done + threadIdx.x; i < a.width; i += BLOCK) {
+        const float v = other(i) + (yr ? act_get<T>(yr[i]) * inv * a.post_w[i] : 0.f);
+        xr[i] = v;
+        local += v * v;
+    }
+    const float scale = a.next_w ? 1.f / sqrtf(block_total(local, red) / static_cast<float>(a.width) + a.eps) : 1.f;
+#pragma unroll
+    for (int c = 0; c < kCache; ++c) {
+        const int i = threadIdx.x + c * BLOCK;
+        if (i >= n4) break;
+        f32x4_t o = xv[c];
+        if (a.next_w)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) o[e] *= scale * nv[c][e];
+        if constexpr (sizeof(T) == 2)
+            *reinterpret_cast<u32x2_t*>(ar + 4 * i) = u32x2_t{pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3])};
+        else *reinterpret_cast<f32x4_t*>(ar + 4 * i) = o;
+    }
+    for (int i = done + threadIdx.x; i < a.width; i += BLOCK)   // (a thread reads what it wrote)
+        ar[i] = act_put<T>(a.next_w ? xr[i] * scale * a.next_w[i] : xr[i]);
+}
+
+// y = act . W^T with fp32 outputs: eight waves share the K of a 16 x 16 tile.
+typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
+constexpr int kThinWaves = 8;
+__global__ __launch_bounds__(kThinWaves* kWave) void linear_f32out_kernel(const uint16_t* __restrict__ act,
+                                                                          const uint16_t* __restrict__ w, float* __restrict__ y,
+                                                                          int M, int N, int K) {
+    __shared__ __attribute__((aligned(16))) float part[kThinWaves][kWave * 4];
+    const int n0 = blockIdx.x * 16, m0 = blockIdx.y * 16, lane = threadIdx.x & (kWave - 1), l16 = lane & 15, g = lane >> 4;
+    const int wv = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave);
+    const uint16_t* wp = w + static_cast<size_t>(n0 + l16) * K + 8 * g;
+    const uint16_t* ap = act + static_cast<size_t>(min(m0 + l16, M - 1)) * K + 8 * g;
+    f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
+    constexpr int U = 4;   // k-steps requested together
+    const int steps = K / 32;
+    for (int s0 = wv; s0 < steps; s0 += U * kThinWaves) {
+        u32x4_t a[U], b[U];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const int k = 32 * min(s0 + u * kThinWaves, steps - 1);
+            a[u] = *reinterpret_cast<const u32x4_t*>(ap + k);
+            b[u] = *reinterpret_cast<const u32x4_t*>(wp + k);
+        }
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+            if (s0 + u * kThinWaves < steps)
+                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, b[u]), __builtin_bit_cast(bf16x8_t, a[u]), acc, 0, 0, 0);
+    }
+    *reinterpret_cast<f32x4_t*>(&part[wv][lane * 4]) = acc;
+    __syncthreads();
+    if (wv != 0) return;
+    f32x4_t v = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < kThinWaves; ++i) v += *reinterpret_cast<const f32x4_t*>(&part[i][lane * 4]);
+    if (m0 + l16 < M) *reinterpret_cast<f32x4_t*>(y + static_cast<size_t>(m0 + l16) * N + n0 + 4 * g) = v;
+}
+
 // out[s] = rmsnorm(x[rows[s]]) * w in the compute type; columns past the width are zero
 template <class T>
 __global__ __launch_bounds__(1024) void norm_rows_kernel(const float* __restrict__ x, const uint32_t* __restrict__ rows,
@@ -195,7 +335,7 @@ __global__ void rotary_table_kernel(const int32_t* __restrict__ positions, const
 // 16-wide K steps through LDS, 4 x 4 outputs per thread.
 constexpr int kFT = 64, kFK = 16;
 __global__ __launch_bounds__(256) void linear_f32_kernel(const float* __restrict__ act, const uint16_t* __restrict__ w,
-                                                         float* __restrict__ y, int M, int N, int K, int relu2) {
+                                                         float* __restrict__ y, int M, int N, int K, int pointwise) {
     __shared__ float as[kFK][kFT + 4];
     __shared__ float ws[kFK][kFT + 4];
     const int n0 = blockIdx.x * kFT, m0 = blockIdx.y * kFT;
@@ -233,10 +373,8 @@ __global__ __launch_bounds__(256) void linear_f32_kernel(const float* __restrict
             const int m = m0 + ty * 4 + i, n = n0 + tx * 4 + j;
             if (m >= M || n >= N) continue;
             float v = acc[i][j];
-            if (relu2) {
-                v = fmaxf(v, 0.f);
-                v *= v;
-            }
+            if (pointwise == PIE_HIP_EPI_GELU) v = 0.5f * v * (1.f + erff(v * 0.70710678118654752f));
+            else v = epilogue_pointwise<false>(v, pointwise);
             y[static_cast<size_t>(m) * N + n] = v;
         }
 }
@@ -274,6 +412,35 @@ extern "C" int pie_hip_norm_add(int dtype, const void* y, const float* weight, f
     return launch_status();
 }
 
+extern "C" int pie_hip_residual_norm(int dtype, const void* y, const float* post_weight, float* x, int read_x,
+                                     const uint32_t* token_ids, const uint16_t* table_bf16, int vocab, const float* add,
+                                     const float* next_weight, void* x_act, int rows, int width, int ldy, int ld,
+                                     float eps, void* stream) {
+    if (!x || !x_act || rows <= 0 || width <= 0 || ld < width || (y && (!post_weight || ldy < width)) ||
+        (token_ids && (!table_bf16 || vocab <= 0)))
+        return PIE_HIP_ERR_INVALID;
+    if ((y && ldy % 8 != 0) || ld % 8 != 0) return PIE_HIP_ERR_UNSUPPORTED;
+    const ResidualArgs a{y, post_weight, add, next_weight, x, token_ids, table_bf16, x_act, read_x ? 1 : 0, vocab, width, ldy, ld, eps};
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    if (width >= 2048 && rows < 512)
+        PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL((residual_norm_kernel<T, 1024>), dim3(rows), dim3(1024), 0, s, a));
+    else
+        PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL((residual_norm_kernel<T, 256>), dim3(rows), dim3(256), 0, s, a));
+    return launch_status();
+}
+
+extern "C" int pie_hip_linear_f32out(int dtype, const void* act, const uint16_t* w_bf16, float* y, int M, int N, int K,
+                                     void* stream) {
+    if (dtype == PIE_HIP_DT_F32)
+        return pie_hip_linear_f32(static_cast<const float*>(act), w_bf16, y, M, N, K, PIE_HIP_EPI_NONE, stream);
+    if (dtype != PIE_HIP_DT_BF16 || !act || !w_bf16 || !y || M <= 0 || N <= 0 || K <= 0) return PIE_HIP_ERR_INVALID;
+    const int gy = (M + 15) / 16;
+    if (K % 32 != 0 || N % 16 != 0 || gy > 65535) return PIE_HIP_ERR_UNSUPPORTED;
+    hipLaunchKernelGGL(linear_f32out_kernel, dim3(N / 16, gy), dim3(kThinWaves * kWave), 0, static_cast<hipStream_t>(stream),
+                       static_cast<const uint16_t*>(act), w_bf16, y, M, N, K);
+    return launch_status();
+}
+
 extern "C" int pie_hip_norm_rows(int dtype, const float* x, const uint32_t* rows, const float* weight, void* out,
                                  int num_out, int width, int ld, int num_rows, float eps, void* stream) {
     if (!x || !rows || !weight || !out || num_out <= 0 || width <= 0 || ld < width || num_rows <= 0)
@@ -304,10 +471,10 @@ extern "C" int pie_hip_rotary_table(const int32_t* positions, const double* freq
 extern "C" int pie_hip_linear_f32(const float* act, const uint16_t* w_bf16, float* y, int M, int N, int K,
                                   int epilogue, void* stream) {
     if (!act || !w_bf16 || !y || M <= 0 || N <= 0 || K <= 0) return PIE_HIP_ERR_INVALID;
-    if (epilogue != PIE_HIP_EPI_NONE && epilogue != PIE_HIP_EPI_RELU2) return PIE_HIP_ERR_UNSUPPORTED;
+    if (epilogue != PIE_HIP_EPI_NONE && epilogue != PIE_HIP_EPI_RELU2 && epilogue != PIE_HIP_EPI_GELU) return PIE_HIP_ERR_UNSUPPORTED;
     const int gy = (M + kFT - 1) / kFT;
     if (gy > 65535) return PIE_HIP_ERR_UNSUPPORTED;
     hipLaunchKernelGGL(linear_f32_kernel, dim3((N + kFT - 1) / kFT, gy), dim3(256), 0, static_cast<hipStream_t>(stream),
-                       act, w_bf16, y, M, N, K, epilogue == PIE_HIP_EPI_RELU2 ? 1 : 0);
+                       act, w_bf16, y, M, N, K, pointwise_code(epilogue));
     return launch_status();
 }
