@@ -343,17 +343,24 @@ def other_configs_extra(drvmod):
     return out
 
 
-# --layer-stack: layers of a layer-stack model (latent attention, one channel-delta layer in three,
-# squared-ReLU feed-forward) beside bf16 llama-type layers of the same width, heads and feed-forward.
+# --layer-stack: layers of the layer-stack models beside bf16 llama-type layers of the same width and
+# feed-forward width.  Varasun: latent attention, one channel-delta layer in three, squared-ReLU
+# feed-forward.  Lofudra: mLSTM, Mamba-2, windowed attention beside retention in turn, GELU feed-forward.
 STACK_SIZES = {
     "width4096": dict(width=4096, heads=32, dim=128, rot_dim=64, vdim=128, q_rank=1536, kv_rank=512, ff=14336,
-                      kv_heads=8, vocab=32000, layers=6),
+                      kv_heads=8, vocab=32000, layers=6, window=1024,
+                      mlstm=dict(heads=8, dim=256, vdim=512, gate_cap=15.0),
+                      mamba2=dict(heads=128, vdim=64, state=128, groups=8, conv=4, norm_groups=8),
+                      retention=dict(heads=16, dim=128, vdim=256)),
     "width2048": dict(width=2048, heads=16, dim=128, rot_dim=64, vdim=128, q_rank=768, kv_rank=512, ff=8192,
-                      kv_heads=4, vocab=32000, layers=6),
+                      kv_heads=4, vocab=32000, layers=6, window=4096,
+                      mlstm=dict(heads=8, dim=128, vdim=256, gate_cap=15.0),
+                      mamba2=dict(heads=64, vdim=64, state=128, groups=4, conv=4, norm_groups=4),
+                      retention=dict(heads=8, dim=128, vdim=256)),
 }
 
 
-def stack_config(z: dict) -> dict:
+def varasun_config(z: dict) -> dict:
     rot = dict(dims=z["rot_dim"], base=10000.0, scaling=dict(factor=4.0, original=4096, fast=24.0, slow=2.0))
     latent = dict(type="latent_attention", mlp=dict(kind="dense", ff=z["ff"]),
                   mixer=dict(heads=z["heads"], dim=z["dim"], rot_dim=z["rot_dim"], vdim=z["vdim"], q_rank=z["q_rank"],
@@ -363,6 +370,19 @@ def stack_config(z: dict) -> dict:
     layers = [delta if l % 3 == 2 else latent for l in range(z["layers"])]
     return dict(architecture="Varasun", layers=layers, width=z["width"], vocab=z["vocab"], norm=dict(eps=1e-6),
                 logit_scale=0.25, logit_softcap=30.0)
+
+
+def lofudra_config(z: dict) -> dict:
+    left = dict(heads=z["heads"], kv_heads=z["kv_heads"], dim=z["dim"], vdim=z["dim"], scale=z["dim"] ** -0.5,
+                mask=dict(size=z["window"]), rot=dict(dims=z["dim"], base=500000.0))
+    right = dict(z["retention"], decay=[1.0 - 2.0 ** (-5.0 - 0.5 * h) for h in range(z["retention"]["heads"])])
+    kinds = [("mlstm", z["mlstm"]), ("mamba2", z["mamba2"]),
+             ("parallel", dict(left=left, right=right, left_scale=0.75, right_scale=0.75))]
+    layers = [dict(type=t, mixer=m, mlp=dict(kind="dense", ff=z["ff"])) for t, m in (kinds * z["layers"])[:z["layers"]]]
+    return dict(architecture="Lofudra", layers=layers, width=z["width"], vocab=z["vocab"], norm=dict(eps=1e-6))
+
+
+STACKS = {"varasun": varasun_config, "lofudra": lofudra_config}
 
 
 def stack_workload(args):
@@ -381,9 +401,12 @@ def stack_workload(args):
         max_new = args.warmup + args.steps + 1
         pages = (n_prompt + max_new + page - 1) // page * 64 + 8
         with tempfile.TemporaryDirectory() as td:
-            (Path(td) / "config.json").write_text(json.dumps(stack_config(z)))
-            models = {
-                "varasun": dict(hf_path=td, random_weights=True, quant="bf16"),
+            models = {}
+            for stack, config in STACKS.items():
+                (Path(td) / stack).mkdir()
+                (Path(td) / stack / "config.json").write_text(json.dumps(config(z)))
+                models[stack] = dict(hf_path=str(Path(td) / stack), random_weights=True, quant="bf16")
+            models |= {
                 "llama": dict(arch="llama3", hidden=z["width"], layers=z["layers"], q_heads=z["heads"],
                               kv_heads=z["kv_heads"], head_dim=z["dim"], intermediate=z["ff"], vocab=z["vocab"],
                               quant="bf16"),
@@ -588,7 +611,7 @@ def main():
     ap.add_argument("--layer-stack", default=None, choices=["all", *STACK_SIZES],
                     help="measure layer-stack models (prefill and decode at batch 1, 16, 64) beside the llama-type "
                          "model of equal size instead of the headline workload")
-    ap.add_argument("--layer-stack-only", default=None, choices=["varasun", "llama"],
+    ap.add_argument("--layer-stack-only", default=None, choices=[*STACKS, "llama"],
                     help="with --layer-stack: only this side (for profiles)")
     args = ap.parse_args()
     if args.gpus != 1:

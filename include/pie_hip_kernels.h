@@ -999,9 +999,12 @@ typedef struct {
     int num_tokens, num_requests;
 } PieHipStateRows;
 /* out[n, c] = silu(bias[c] + sum_j conv_w[c, j] * input_(n - (taps - 1) + j)[c]) for the first `channels`
- * columns of fused (earlier inputs from the state, zeros before the start); rows of ld_out. */
+ * columns of fused (earlier inputs from the state, zeros before the start); rows of ld_out.
+ * move_state (one row per request only): the state also moves on by that row; elsewhere
+ * pie_hip_delta_conv_state does it afterwards. */
 int pie_hip_conv_silu(int dtype, const void* fused, const float* conv_w, const float* conv_bias,
-                      const PieHipStateRows* rows, void* out, int ld, int channels, int taps, int ld_out, void* stream);
+                      const PieHipStateRows* rows, void* out, int ld, int channels, int taps, int ld_out,
+                      int move_state, void* stream);
 /* Token by token, any compute type: q, k, v rows of ld values.  o [N, heads * vdim] fp32; den [N, heads, 2]
  * (EXP_GATES: n . q and m_t).  dim <= 512. */
 int pie_hip_decay_scan(int dtype, const PieHipDecayRule* rule, const PieHipStateRows* rows, const void* q,
@@ -1022,7 +1025,7 @@ int pie_hip_decay_out(int dtype, const PieHipDecayRule* rule, const PieHipStateR
                       int ld_y, float out_scale, float eps, void* stream);
 /* One token per request (row r = request r), one launch: the state is read and written once.  conv_w not
  * NULL: q, k, v are columns q_off, k_off, v_off of `fused` ahead of the convolution (conv_w [channels, taps] indexed
- * by the same columns, the state is read, not moved on) and skip[head] * v is added to o.  y not NULL: with
+ * by the same columns; the state is read, not moved on).  skip not NULL: skip[head] * v is added to o.  y not NULL: with
  * pie_hip_decay_out's norm and gate fused (one block per head then), else o and den.
  * vdim % 4 == 0, dim <= 512, vdim <= 1024 (pie_hip_decay_step_supported). */
 int pie_hip_decay_step_supported(int dim, int vdim);

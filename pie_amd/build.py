@@ -76,7 +76,7 @@ def build_kernels(force: bool = False, jobs: int | None = None) -> Path:
     jobs = jobs or _jobs()
     with ThreadPoolExecutor(max_workers=jobs) as pool:
         list(pool.map(_run, todo))
-    if force or todo or not KERNEL_LIB.exists():
+    if force or todo or not _newer(KERNEL_LIB, objs):
         _run([HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", str(KERNEL_LIB),
               *map(str, objs)])
     return KERNEL_LIB

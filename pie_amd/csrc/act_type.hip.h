@@ -51,7 +51,10 @@ struct ActVec<float> {
     }
 };
 
-__device__ __forceinline__ float sigmoid_f32(float z) { return 1.f / (1.f + expf(-z)); }
+// (the bare exponential and reciprocal: a few units in the last place)
+__device__ __forceinline__ float sigmoid_f32(float z) {
+    return __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+}
 
 // Sum over a block of up to 1024 threads (a multiple of 64); every thread gets the total.
 // `smem`: one float per wave.

@@ -533,18 +533,24 @@ void Executor::stack_memory(const StackLayer& w, int run, int N, const Inputs& i
     };
     if (plan_->pure_decode && pie_hip_decay_step_supported(d.dim, d.vdim)) {
         const bool fuse = !ssm && pie_hip_decay_step_fuses(&rule, rows.num_requests);
-        PIE_KERNEL(pie_hip_decay_step(dt_, &rule, &rows, stack_.in, s.mq_off, s.mk_off, s.mv_off, s.ld_in, stack_.gates, s.gates,
-                                      ssm ? w.conv_w : nullptr, ssm ? w.conv_b : nullptr, s.channels, d.taps, ssm ? w.skip : nullptr,
-                                      stack_.mem_o, stack_.den, gate, s.ld_in, gate_act, w.out_norm, fuse ? y : nullptr, s.ld_o, scale, eps,
-                                      stream_));
-        if (ssm) part_norm(nullptr, stack_.in);
+        // (the heads of a group convolve the same keys and queries again: worth a launch of its own once
+        // the batch fills the device)
+        const bool conv_first = ssm && rows.num_requests * d.heads >= 1024;
+        if (conv_first)
+            PIE_KERNEL(pie_hip_conv_silu(dt_, stack_.in, w.conv_w, w.conv_b, &rows, stack_.conv, s.ld_in, s.channels, d.taps, s.ld_conv, 1, stream_));
+        const bool conv_in = ssm && !conv_first;
+        PIE_KERNEL(pie_hip_decay_step(dt_, &rule, &rows, conv_first ? stack_.conv : stack_.in, s.mq_off, s.mk_off, s.mv_off,
+                                      conv_first ? s.ld_conv : s.ld_in, stack_.gates, s.gates, conv_in ? w.conv_w : nullptr,
+                                      conv_in ? w.conv_b : nullptr, s.channels, d.taps, ssm ? w.skip : nullptr, stack_.mem_o, stack_.den, gate,
+                                      s.ld_in, gate_act, w.out_norm, fuse ? y : nullptr, s.ld_o, scale, eps, stream_));
+        if (ssm) part_norm(nullptr, conv_first ? nullptr : stack_.in);
         else if (!fuse) out();
         return;
     }
     const void *q = at(stack_.in, s.mq_off), *k = at(stack_.in, s.mk_off), *v = at(stack_.in, s.mv_off);
     int ld = s.ld_in;
     if (ssm) {
-        PIE_KERNEL(pie_hip_conv_silu(dt_, stack_.in, w.conv_w, w.conv_b, &rows, stack_.conv, s.ld_in, s.channels, d.taps, s.ld_conv, stream_));
+        PIE_KERNEL(pie_hip_conv_silu(dt_, stack_.in, w.conv_w, w.conv_b, &rows, stack_.conv, s.ld_in, s.channels, d.taps, s.ld_conv, 0, stream_));
         PIE_KERNEL(pie_hip_delta_conv_state(dt_, stack_.in, rs_base_, rs_stride_, rows.conv_offset, rows.qo_indptr, rows.rs_slot,
                                             rows.rs_fresh, rows.num_requests, s.ld_in, s.channels, d.taps, stream_));
         q = at(stack_.conv, s.mq_off);

@@ -89,6 +89,83 @@ __global__ __launch_bounds__(256) void group_prep_kernel(const PrepArgs a) {
     }
 }
 
+// The same for heads of whole 8-value pieces: a lane takes eight neighbouring values, LPH lanes a head, 64 / LPH
+// heads a wave; a rotated value's partner is half / 8 lanes away.
+template <class T>
+__device__ __forceinline__ void load8(const T* p, float* f) {
+    if constexpr (sizeof(T) == 2) {
+        ActVec<T>::load(p, f);
+    } else {
+        ActVec<T>::load(p, f);
+        ActVec<T>::load(p + 4, f + 4);
+    }
+}
+template <class T>
+__device__ __forceinline__ void store8(T* p, const float* f) {
+    if constexpr (sizeof(T) == 2) {
+        *reinterpret_cast<u32x4_t*>(p) = u32x4_t{pack_bf16x2(f[0], f[1]), pack_bf16x2(f[2], f[3]), pack_bf16x2(f[4], f[5]), pack_bf16x2(f[6], f[7])};
+    } else {
+        *reinterpret_cast<f32x4_t*>(p) = f32x4_t{f[0], f[1], f[2], f[3]};
+        *reinterpret_cast<f32x4_t*>(p + 4) = f32x4_t{f[4], f[5], f[6], f[7]};
+    }
+}
+template <class T, int LPH>
+__global__ __launch_bounds__(256) void group_prep_vec_kernel(const PrepArgs a) {
+    const int units = a.heads + a.kv_heads, lane = threadIdx.x & (kWave - 1);
+    const long long unit = static_cast<long long>(blockIdx.x) * (256 / LPH) + threadIdx.x / LPH;
+    const bool on = unit < static_cast<long long>(a.num_tokens) * units;   // (every lane takes part in the exchanges)
+    const size_t n = on ? unit / units : 0;
+    const int u = on ? static_cast<int>(unit % units) : 0;
+    const bool is_q = u < a.heads;
+    const int h = is_q ? u : u - a.heads, d = 8 * (lane & (LPH - 1));
+    const bool in = on && d < a.dim, rotated = in && d < a.rot_dims;
+    const T* row = static_cast<const T*>(a.fused) + n * a.ld;
+    const int half = a.rot_dims / 2, t = d < half ? d : d - half;
+    const float* bias = is_q ? a.q_bias : a.k_bias;
+    const float* norm = is_q ? a.q_norm : a.k_norm;
+    float x[8] = {}, raw[8], b[8] = {}, w[8] = {}, c[8] = {}, s[8] = {}, v[8] = {}, local = 0.f;
+    const int64_t slot = on && !is_q ? a.slots[n] : -1;
+    if (in) {
+        load8(row + (is_q ? a.q_off : a.k_off) + h * a.dim + d, x);
+        if (bias) load8(bias + h * a.dim + d, b);
+        if (norm) load8(norm + d, w);
+        if (!is_q && a.v_off >= 0) load8(row + a.v_off + h * a.dim + d, v);
+    }
+    if (rotated) {
+        load8(a.rope + n * a.rot_dims + t, c);
+        load8(a.rope + n * a.rot_dims + half + t, s);
+    }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+        x[e] += b[e];
+        raw[e] = x[e];
+        local += x[e] * x[e];
+    }
+    if (norm) {
+#pragma unroll
+        for (int off = 1; off < LPH; off <<= 1) local += __shfl_xor(local, off, kWave);
+        const float inv = 1.f / sqrtf(local / static_cast<float>(a.dim) + a.eps);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[e] *= inv * w[e];
+    }
+    if (a.rot_dims > 0) {
+        const int from = lane + (d < half ? half / 8 : -half / 8);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            const float other = __shfl(x[e], from, kWave);
+            if (rotated) x[e] = d < half ? x[e] * c[e] - other * s[e] : x[e] * c[e] + other * s[e];
+        }
+    }
+    if (!on || d >= a.dimp) return;
+    if (is_q) {
+        store8(static_cast<T*>(a.q) + (n * a.heads + h) * a.dimp + d, x);
+    } else if (slot >= 0) {
+        T* k = static_cast<T*>(a.pool) + (static_cast<size_t>(slot) * a.kv_heads + h) * 2 * a.dimp + d;
+        store8(k, x);
+        store8(k + a.dimp, a.v_off < 0 ? raw : v);
+    }
+}
+
 // ---- any size, any compute type --------------------------------------------------------------------
 struct PlainArgs {
     const void *q, *pool;
@@ -229,30 +306,42 @@ __global__ __launch_bounds__(kBlock, 2) void group_rows_kernel(const AttnArgs a)
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks) qf[ks] = __builtin_bit_cast(bf16x8_t, *reinterpret_cast<const u32x4_t*>(qp + 32 * ks));
     }
-    auto row_of = [&](int j) {   // (keys past the end repeat the last: their weights are zero)
-        j = min(j, len - 1);
-        const int page = a.ps_shift >= 0 ? j >> a.ps_shift : j / a.ps;
-        return a.pool + ((static_cast<size_t>(pages[page]) * a.ps + (j - page * a.ps)) * a.kv_heads + kvh) * 2 * D;
+    // Places of this lane's rows of a step: two keys and a value row.  Their pages are asked for one step of
+    // this wave ahead of the rows, so that the two requests do not stand in line.
+    uint32_t pid[3];
+    int in_page[3];
+    auto fetch_pages = [&](int step) {
+        const int j0 = begin + step * kStep;
+#pragma unroll
+        for (int i = 0; i < 3; ++i) {   // (keys past the end repeat the last: their weights are zero)
+            const int j = min(j0 + (i < 2 ? 16 * i + l16 : lane >> 1), len - 1);
+            const int page = a.ps_shift >= 0 ? j >> a.ps_shift : j / a.ps;
+            pid[i] = pages[page];
+            in_page[i] = j - page * a.ps;
+        }
     };
     u32x4_t kr[2][KS], vr[NP];
     auto issue = [&](int step) {
-        const int j0 = begin + step * kStep;
+        const uint16_t* row[3];
 #pragma unroll
-        for (int nt = 0; nt < 2; ++nt) {
-            const uint16_t* p = row_of(j0 + 16 * nt + l16) + 8 * g;
+        for (int i = 0; i < 3; ++i) row[i] = a.pool + ((static_cast<size_t>(pid[i]) * a.ps + in_page[i]) * a.kv_heads + kvh) * 2 * D;
+        fetch_pages(step + kWaves);
 #pragma unroll
-            for (int ks = 0; ks < KS; ++ks) kr[nt][ks] = *reinterpret_cast<const u32x4_t*>(p + 32 * ks);
-        }
+        for (int nt = 0; nt < 2; ++nt)
+#pragma unroll
+            for (int ks = 0; ks < KS; ++ks) kr[nt][ks] = *reinterpret_cast<const u32x4_t*>(row[nt] + 8 * g + 32 * ks);
         // values: two lanes per key, NP pieces each
-        const uint16_t* p = row_of(j0 + (lane >> 1)) + D + (lane & 1) * 8;
 #pragma unroll
-        for (int u = 0; u < NP; ++u) vr[u] = *reinterpret_cast<const u32x4_t*>(p + 16 * u);
+        for (int u = 0; u < NP; ++u) vr[u] = *reinterpret_cast<const u32x4_t*>(row[2] + D + (lane & 1) * 8 + 16 * u);
     };
     f32x4_t acc[DT];
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) acc[dt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     float mx = -INFINITY, lsum = 0.f;   // (raw score units)
-    if (s_lo + wv < s_hi) issue(s_lo + wv);
+    if (s_lo + wv < s_hi) {
+        fetch_pages(s_lo + wv);
+        issue(s_lo + wv);
+    }
     for (int st = s_lo + wv; st < s_hi; st += kWaves) {
         const int j0 = begin + st * kStep;
         f32x4_t sc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
@@ -568,6 +657,21 @@ extern "C" int pie_hip_group_attn_prep(int dtype, const void* fused, int q_off, 
     const long long units = static_cast<long long>(num_tokens) * (heads + kv_heads);
     const dim3 grid(static_cast<unsigned>((units + 3) / 4));
     hipStream_t s = static_cast<hipStream_t>(stream);
+    auto whole = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
+    if (dim % 8 == 0 && dimp % 8 == 0 && rot_dims % 16 == 0 && q_off % 8 == 0 && k_off % 8 == 0 && (v_off < 0 || v_off % 8 == 0) &&
+        ld_fused % 8 == 0 && dimp <= 512 && whole(fused) && whole(q_out) && whole(pool) && whole(rope_table) && whole(q_bias) &&
+        whole(k_bias) && whole(q_norm) && whole(k_norm)) {
+        const int pieces = dimp / 8, lph = pieces <= 4 ? 4 : pieces <= 8 ? 8 : pieces <= 16 ? 16 : pieces <= 32 ? 32 : 64;
+        const dim3 vgrid(static_cast<unsigned>((units + 256 / lph - 1) / (256 / lph)));
+        PIE_ACT_DISPATCH(dtype, T, switch (lph) {
+            case 4: hipLaunchKernelGGL((group_prep_vec_kernel<T, 4>), vgrid, dim3(256), 0, s, a); break;
+            case 8: hipLaunchKernelGGL((group_prep_vec_kernel<T, 8>), vgrid, dim3(256), 0, s, a); break;
+            case 16: hipLaunchKernelGGL((group_prep_vec_kernel<T, 16>), vgrid, dim3(256), 0, s, a); break;
+            case 32: hipLaunchKernelGGL((group_prep_vec_kernel<T, 32>), vgrid, dim3(256), 0, s, a); break;
+            default: hipLaunchKernelGGL((group_prep_vec_kernel<T, 64>), vgrid, dim3(256), 0, s, a); break;
+        });
+        return launch_status();
+    }
     PIE_ACT_DISPATCH(dtype, T, {
         if (dimp <= 64) hipLaunchKernelGGL((group_prep_kernel<T, 1>), grid, dim3(256), 0, s, a);
         else if (dimp <= 128) hipLaunchKernelGGL((group_prep_kernel<T, 2>), grid, dim3(256), 0, s, a);

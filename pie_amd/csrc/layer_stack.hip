@@ -199,40 +199,49 @@ __global__ __launch_bounds__(BLOCK) void residual_norm_kernel(const ResidualArgs
         ar[i] = act_put<T>(a.next_w ? xr[i] * scale * a.next_w[i] : xr[i]);
 }
 
-// y = act . W^T with fp32 outputs: eight waves share the K of a 16 x 16 tile.
+// y = act . W^T with fp32 outputs: the waves of a block share the K of a row tile and NT column tiles, each
+// requesting U of its k-steps at once.
 typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
-constexpr int kThinWaves = 8;
-__global__ __launch_bounds__(kThinWaves* kWave) void linear_f32out_kernel(const uint16_t* __restrict__ act,
-                                                                          const uint16_t* __restrict__ w, float* __restrict__ y,
-                                                                          int M, int N, int K) {
-    __shared__ __attribute__((aligned(16))) float part[kThinWaves][kWave * 4];
-    const int n0 = blockIdx.x * 16, m0 = blockIdx.y * 16, lane = threadIdx.x & (kWave - 1), l16 = lane & 15, g = lane >> 4;
+template <int WAVES, int NT, int U>
+__global__ __launch_bounds__(WAVES* kWave) void linear_f32out_kernel(const uint16_t* __restrict__ act,
+                                                                     const uint16_t* __restrict__ w, float* __restrict__ y,
+                                                                     int M, int N, int K) {
+    __shared__ __attribute__((aligned(16))) float part[NT][WAVES][kWave * 4];
+    const int n0 = blockIdx.x * 16 * NT, m0 = blockIdx.y * 16, lane = threadIdx.x & (kWave - 1), l16 = lane & 15, g = lane >> 4;
     const int wv = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave);
-    const uint16_t* wp = w + static_cast<size_t>(n0 + l16) * K + 8 * g;
     const uint16_t* ap = act + static_cast<size_t>(min(m0 + l16, M - 1)) * K + 8 * g;
-    f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
-    constexpr int U = 4;   // k-steps requested together
+    const uint16_t* wp[NT];
+    f32x4_t acc[NT];
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+        wp[t] = w + static_cast<size_t>(min(n0 + 16 * t, N - 16) + l16) * K + 8 * g;   // (a tile past N repeats the last one)
+        acc[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    }
     const int steps = K / 32;
-    for (int s0 = wv; s0 < steps; s0 += U * kThinWaves) {
-        u32x4_t a[U], b[U];
+    for (int s0 = wv; s0 < steps; s0 += U * WAVES) {
+        u32x4_t a[U], b[NT][U];
 #pragma unroll
         for (int u = 0; u < U; ++u) {
-            const int k = 32 * min(s0 + u * kThinWaves, steps - 1);
+            const int k = 32 * min(s0 + u * WAVES, steps - 1);
             a[u] = *reinterpret_cast<const u32x4_t*>(ap + k);
-            b[u] = *reinterpret_cast<const u32x4_t*>(wp + k);
+#pragma unroll
+            for (int t = 0; t < NT; ++t) b[t][u] = *reinterpret_cast<const u32x4_t*>(wp[t] + k);
         }
 #pragma unroll
         for (int u = 0; u < U; ++u)
-            if (s0 + u * kThinWaves < steps)
-                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, b[u]), __builtin_bit_cast(bf16x8_t, a[u]), acc, 0, 0, 0);
+            if (s0 + u * WAVES < steps)
+#pragma unroll
+                for (int t = 0; t < NT; ++t)
+                    acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, b[t][u]), __builtin_bit_cast(bf16x8_t, a[u]), acc[t], 0, 0, 0);
     }
-    *reinterpret_cast<f32x4_t*>(&part[wv][lane * 4]) = acc;
+#pragma unroll
+    for (int t = 0; t < NT; ++t) *reinterpret_cast<f32x4_t*>(&part[t][wv][lane * 4]) = acc[t];
     __syncthreads();
-    if (wv != 0) return;
+    if (wv >= NT || n0 + 16 * wv >= N) return;   // wave t adds tile t up
     f32x4_t v = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int i = 0; i < kThinWaves; ++i) v += *reinterpret_cast<const f32x4_t*>(&part[i][lane * 4]);
-    if (m0 + l16 < M) *reinterpret_cast<f32x4_t*>(y + static_cast<size_t>(m0 + l16) * N + n0 + 4 * g) = v;
+    for (int i = 0; i < WAVES; ++i) v += *reinterpret_cast<const f32x4_t*>(&part[wv][i][lane * 4]);
+    if (m0 + l16 < M) *reinterpret_cast<f32x4_t*>(y + static_cast<size_t>(m0 + l16) * N + n0 + 16 * wv + 4 * g) = v;
 }
 
 // out[s] = rmsnorm(x[rows[s]]) * w in the compute type; columns past the width are zero
@@ -436,8 +445,12 @@ extern "C" int pie_hip_linear_f32out(int dtype, const void* act, const uint16_t*
     if (dtype != PIE_HIP_DT_BF16 || !act || !w_bf16 || !y || M <= 0 || N <= 0 || K <= 0) return PIE_HIP_ERR_INVALID;
     const int gy = (M + 15) / 16;
     if (K % 32 != 0 || N % 16 != 0 || gy > 65535) return PIE_HIP_ERR_UNSUPPORTED;
-    hipLaunchKernelGGL(linear_f32out_kernel, dim3(N / 16, gy), dim3(kThinWaves * kWave), 0, static_cast<hipStream_t>(stream),
-                       static_cast<const uint16_t*>(act), w_bf16, y, M, N, K);
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    const auto* x = static_cast<const uint16_t*>(act);
+    if (M >= 512 && N > 16)   // (row tiles fill the device: column tiles share their activations)
+        hipLaunchKernelGGL((linear_f32out_kernel<8, 4, 2>), dim3((N + 63) / 64, gy), dim3(512), 0, s, x, w_bf16, y, M, N, K);
+    else
+        hipLaunchKernelGGL((linear_f32out_kernel<16, 1, 8>), dim3(N / 16, gy), dim3(1024), 0, s, x, w_bf16, y, M, N, K);
     return launch_status();
 }
 
