@@ -248,8 +248,12 @@ MIXERS = {"latent_attention": latent_attention, "channel_delta": channel_delta, 
           "mamba2": mamba2}
 
 
-def feed_forward(x, w, p, act=squared_relu):
-    return act(x @ w[p + "up"].T) @ w[p + "down"].T
+def feed_forward(x, w, p):
+    return squared_relu(x @ w[p + "up"].T) @ w[p + "down"].T
+
+
+def gelu_feed_forward(x, w, p):
+    return gelu_erf(x @ w[p + "up"].T) @ w[p + "down"].T
 
 
 def layer_runs(cfg):
@@ -273,7 +277,7 @@ def forward_sandwich(cfg, w, tokens, want_layers=False):
         y = MIXERS[layer["type"]](rms_norm(x, w[p + "norm1"], eps), w, p + "mix.", layer["mixer"], eps)
         x = x + rms_norm(y, w[p + "norm1b"], eps)
         if layer.get("mlp"):
-            y = feed_forward(rms_norm(x, w[p + "norm2"], eps), w, p + "mlp.", gelu_erf)
+            y = gelu_feed_forward(rms_norm(x, w[p + "norm2"], eps), w, p + "mlp.")
             x = x + rms_norm(y, w[p + "norm2b"], eps)
         states.append(x)
     logits = rms_norm(x, w["final.norm"], eps) @ w["head"].T

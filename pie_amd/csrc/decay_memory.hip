@@ -368,7 +368,7 @@ __device__ __forceinline__ f32x4_t mfma_bf16(const u32x4_t a, const bf16x8_t b, 
 
 __global__ __launch_bounds__(256) void decay_chunk_kernel(const ChunkArgs a) {
     __shared__ __attribute__((aligned(16))) uint16_t tiles[2][2][kChunk * kPieceStride];   // two steps' queries and keys, or values
-    __shared__ __attribute__((aligned(16))) float s_f[kChunk], s_in[kChunk], s_m[kChunk], s_u[kChunk], s_w[kChunk];
+    __shared__ __attribute__((aligned(16))) float s_top[kChunk], s_top_lo[kChunk], s_in[kChunk], s_in_lo[kChunk], s_u[kChunk], s_w[kChunk];
     const PieHipDecayRule& r = a.rule;
     const int h = blockIdx.x, ch = blockIdx.y, tid = threadIdx.x, lane = tid & (kWave - 1);
     const int wv = __builtin_amdgcn_readfirstlane(tid / kWave), l16 = lane & 15, g = lane >> 4;
@@ -380,35 +380,38 @@ __global__ __launch_bounds__(256) void decay_chunk_kernel(const ChunkArgs a) {
     if (wv == 0) {
         TokenGate tg{0.f, stab ? -INFINITY : 0.f, 0.f};   // tokens past the portion: decay 1, weight 0
         if (lane < nt) tg = token_gate(r, a.gates + static_cast<size_t>(row0 + lane) * a.ld_gates, h);
-        float F = tg.keep;
+        // (running sums in double: differences of two of them stay right to the last bit however fast the
+        // head forgets)
+        double F = tg.keep;
 #pragma unroll
         for (int off = 1; off < kWave; off <<= 1) {
-            const float up = __shfl_up(F, off, kWave);
+            const double up = __shfl_up(F, off, kWave);
             if (lane >= off) F += up;
         }
-        const float in = tg.in - F;
-        float M = 0.f;
+        const double in = static_cast<double>(tg.in) - F;
+        double M = 0.0;
         if (stab) {
-            float mx = in;
+            double mx = in;
 #pragma unroll
             for (int off = 1; off < kWave; off <<= 1) {
-                const float up = __shfl_up(mx, off, kWave);
-                if (lane >= off) mx = fmaxf(mx, up);
+                const double up = __shfl_up(mx, off, kWave);
+                if (lane >= off) mx = fmax(mx, up);
             }
             M = F + mx;
         }
-        const float F_end = __shfl(F, kWave - 1, kWave), M_end = __shfl(M, kWave - 1, kWave);
-        s_f[lane] = F;
-        s_in[lane] = in;
-        s_m[lane] = M;
+        const double F_end = __shfl(F, kWave - 1, kWave), M_end = __shfl(M, kWave - 1, kWave), top = F - M;
+        s_top[lane] = static_cast<float>(top);
+        s_top_lo[lane] = static_cast<float>(top - s_top[lane]);
+        s_in[lane] = static_cast<float>(in);
+        s_in_lo[lane] = lane < nt ? static_cast<float>(in - s_in[lane]) : 0.f;
         s_u[lane] = tg.weight;
-        s_w[lane] = tg.weight * exp2f(F_end + in - M_end);
+        s_w[lane] = tg.weight * exp2f(static_cast<float>(F_end + in - M_end));
         float* meta = a.meta + rec * a.lay.meta_elems;
-        meta[lane] = stab ? F : r.q_scale * exp2f(F);
-        meta[kChunk + lane] = M;
+        meta[lane] = stab ? static_cast<float>(F) : r.q_scale * exp2f(static_cast<float>(F));
+        meta[kChunk + lane] = static_cast<float>(M);
         if (lane == 0) {
-            meta[2 * kChunk] = stab ? F_end : exp2f(F_end);
-            meta[2 * kChunk + 1] = M_end;
+            meta[2 * kChunk] = stab ? static_cast<float>(F_end) : exp2f(static_cast<float>(F_end));
+            meta[2 * kChunk + 1] = static_cast<float>(M_end);
         }
     }
     // scores: wave w takes query tile w against key tiles 0 .. w
@@ -460,14 +463,14 @@ __global__ __launch_bounds__(256) void decay_chunk_kernel(const ChunkArgs a) {
     u32x4_t p_hi[2], p_lo[2];
     {
         const int t = 16 * wv + l16;
-        const float top = s_f[t] - s_m[t];
+        const float top = s_top[t], top_lo = s_top_lo[t];
 #pragma unroll
         for (int ks = 0; ks < 2; ++ks) {
             float x[8];
 #pragma unroll
             for (int e = 0; e < 8; ++e) {
                 const int s = 32 * ks + 16 * (e >> 2) + 4 * g + (e & 3);
-                x[e] = s <= t ? acc[2 * ks + (e >> 2)][e & 3] * (r.q_scale * s_u[s] * exp2f(top + s_in[s])) : 0.f;
+                x[e] = s <= t ? acc[2 * ks + (e >> 2)][e & 3] * (r.q_scale * s_u[s] * exp2f((top + s_in[s]) + (top_lo + s_in_lo[s]))) : 0.f;
             }
             split8(x, p_hi[ks], p_lo[ks]);
         }

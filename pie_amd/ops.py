@@ -354,6 +354,7 @@ def copy_kv_pages(pool: torch.Tensor, srcs: torch.Tensor, dsts: torch.Tensor) ->
 
 
 RELU2 = 2   # `swiglu` argument of the linears: squared-ReLU epilogue, all N columns
+GELU = 3    # exact GELU, all N columns (bf16 weights)
 
 FMT = {"int4b8": 0, "int8": 1, "fp8": 2, "bf16": 3}
 
@@ -1118,12 +1119,12 @@ def rotary_table(positions: torch.Tensor, freq: torch.Tensor, mscale: float) -> 
     return table
 
 
-def linear_f32(act: torch.Tensor, w: torch.Tensor, relu2: bool = False) -> torch.Tensor:
+def linear_f32(act: torch.Tensor, w: torch.Tensor, relu2: bool = False, epilogue: int = 0) -> torch.Tensor:
     _dev(act, torch.float32, "act")
     _dev(w, torch.bfloat16, "w")
     y = torch.empty((act.shape[0], w.shape[0]), dtype=torch.float32, device=act.device)
     _check(kernels().pie_hip_linear_f32(_ptr(act), _ptr(w), _ptr(y), act.shape[0], w.shape[0], act.shape[1],
-                                        2 if relu2 else 0, _stream()), "pie_hip_linear_f32")
+                                        RELU2 if relu2 else epilogue, _stream()), "pie_hip_linear_f32")
     return y
 
 
@@ -1212,3 +1213,172 @@ def delta_scan(q, k, v, log2_decay, beta, state, qo_indptr, slots, fresh, heads,
                                      C.c_size_t(0), _ptr(ct), _ptr(ft), _ptr(qo_indptr), _ptr(slots), _ptr(fresh), len(chunks), R,
                                      heads, kv_heads, dim, vdim, _ptr(ws), C.c_size_t(need), _stream()), "pie_hip_delta_chunked")
     return o
+
+
+def residual_norm(x: torch.Tensor, width: int, eps: float, dtype, y=None, post_weight=None, read_x: bool = True, tokens=None,
+                  table=None, add=None, next_weight=None) -> torch.Tensor:
+    """x takes rmsnorm(y) * post_weight, table[tokens] and add (each optional) in place; returns x, normed with
+    next_weight if given, in `dtype`."""
+    _dev(x, torch.float32, "x")
+    xa = torch.zeros(x.shape, dtype=dtype, device=x.device)
+    _check(kernels().pie_hip_residual_norm(_dt(xa), _ptr(y), _ptr(post_weight), _ptr(x), int(read_x), _ptr(tokens), _ptr(table),
+                                           0 if table is None else table.shape[0], _ptr(add), _ptr(next_weight), _ptr(xa), x.shape[0],
+                                           width, 0 if y is None else y.shape[1], x.shape[1], C.c_float(eps), _stream()),
+           "pie_hip_residual_norm")
+    return xa
+
+
+def linear_f32out(act: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    _dev(w, torch.bfloat16, "w")
+    y = torch.empty((act.shape[0], w.shape[0]), dtype=torch.float32, device=act.device)
+    _check(kernels().pie_hip_linear_f32out(_dt(act), _ptr(act), _ptr(w), _ptr(y), act.shape[0], w.shape[0], act.shape[1], _stream()),
+           "pie_hip_linear_f32out")
+    return y
+
+
+def group_attn_prep(fused, q_off, k_off, v_off, q_bias, k_bias, q_norm, k_norm, rope, rot_dims, slots, pool, heads, kv_heads, dim, dimp,
+                    eps) -> torch.Tensor:
+    """q [N, heads, dimp]; the rows' keys and values go to pool [slots, kv_heads, 2 dimp]."""
+    q = torch.full((fused.shape[0], heads, dimp), 3.0, dtype=fused.dtype, device=fused.device)
+    _check(kernels().pie_hip_group_attn_prep(_dt(fused), _ptr(fused), q_off, k_off, v_off, _ptr(q_bias), _ptr(k_bias), _ptr(q_norm),
+                                             _ptr(k_norm), _ptr(rope), rot_dims, _ptr(slots), _ptr(q), _ptr(pool), fused.shape[0],
+                                             fused.shape[1], heads, kv_heads, dim, dimp, C.c_float(eps), _stream()),
+           "pie_hip_group_attn_prep")
+    return q
+
+
+def group_attn(form: str, q, pool, page_indices, row_begin, row_len, page_size, scale, window=0, sink=0.0, out_scale=1.0, ld_o=None,
+               rows=None, tiles=None, half: int = 0, max_kv_len: Optional[int] = None) -> torch.Tensor:
+    """q [N, heads, dimp], pool [slots, kv_heads, 2 dimp] -> o [N, ld_o] (heads dimp apart); form "rows" (all rows,
+    or the listed ones), "tiles" or "plain"."""
+    n, heads, dimp = q.shape
+    kv_heads = pool.shape[1]
+    ld_o = ld_o or heads * dimp
+    o = torch.full((n, ld_o), 3.0, dtype=q.dtype, device=q.device)
+    longest = int(row_len.max()) if max_kv_len is None else max_kv_len
+    lib = kernels()
+    tail = (heads, kv_heads, dimp, ld_o, page_size, C.c_float(scale), window, C.c_float(sink), C.c_float(out_scale))
+    head = (_ptr(q), _ptr(pool), _ptr(o), _ptr(page_indices), _ptr(row_begin), _ptr(row_len))
+    if form == "plain":
+        _check(lib.pie_hip_group_attn_plain(_dt(q), *head, n, *tail, _stream()), "pie_hip_group_attn_plain")
+    elif form == "tiles":
+        _check(lib.pie_hip_group_attn_tiles(*head, _ptr(tiles), tiles.shape[0], half, *tail, _stream()), "pie_hip_group_attn_tiles")
+    else:
+        count = n if rows is None else rows.numel()
+        lib.pie_hip_group_attn_rows_workspace_bytes.restype = C.c_size_t
+        need = int(lib.pie_hip_group_attn_rows_workspace_bytes(count, heads, kv_heads, dimp, longest, window))
+        ws = torch.empty(max(need, 16), dtype=torch.uint8, device=q.device)
+        _check(lib.pie_hip_group_attn_rows(*head, _ptr(rows), count, *tail, longest, _ptr(ws), C.c_size_t(need), _stream()),
+               "pie_hip_group_attn_rows")
+    return o
+
+
+def group_attn_tile_rows(heads: int, kv_heads: int, half: int) -> int:
+    return int(kernels().pie_hip_group_attn_tile_rows(heads, kv_heads, half))
+
+
+class DecayRule(C.Structure):
+    """PieHipDecayRule: kind 0 retention, 1 mLSTM, 2 Mamba-2."""
+    _fields_ = [("kind", C.c_int), ("heads", C.c_int), ("kv_heads", C.c_int), ("dim", C.c_int), ("vdim", C.c_int),
+                ("q_scale", C.c_float), ("k_scale", C.c_float), ("gate_cap", C.c_float), ("decay", C.c_void_p), ("gate_bias", C.c_void_p)]
+
+
+class StateRows(C.Structure):
+    """PieHipStateRows: the batch's rows, their requests, and where the requests' states live."""
+    _fields_ = [("row_req", C.c_void_p), ("qo_indptr", C.c_void_p), ("rs_slot", C.c_void_p), ("rs_fresh", C.c_void_p), ("rs_base", C.c_void_p),
+                ("rs_stride", C.c_size_t), ("state_offset", C.c_size_t), ("conv_offset", C.c_size_t), ("num_tokens", C.c_int),
+                ("num_requests", C.c_int)]
+
+
+def decay_rule(kind, heads, kv_heads, dim, vdim, q_scale=1.0, k_scale=1.0, gate_cap=0.0, decay=None, gate_bias=None) -> DecayRule:
+    address = lambda x: None if x is None else x.data_ptr()
+    return DecayRule(kind, heads, kv_heads, dim, vdim, q_scale, k_scale, gate_cap, address(decay), address(gate_bias))
+
+
+def state_rows(row_req, qo_indptr, slots, fresh, state, state_offset: int = 0, conv_offset: int = 0) -> StateRows:
+    """state: [slots, bytes] uint8."""
+    return StateRows(row_req.data_ptr(), qo_indptr.data_ptr(), slots.data_ptr(), fresh.data_ptr(), state.data_ptr(), state.stride(0),
+                     state_offset, conv_offset, row_req.numel(), slots.numel())
+
+
+def conv_silu(fused, w, bias, rows: StateRows, channels: int, move_state: bool = False) -> torch.Tensor:
+    out = torch.full((fused.shape[0], -(-channels // 8) * 8), 3.0, dtype=fused.dtype, device=fused.device)
+    _check(kernels().pie_hip_conv_silu(_dt(fused), _ptr(fused), _ptr(w), _ptr(bias), C.byref(rows), _ptr(out), fused.shape[1], channels,
+                                       w.shape[1], out.shape[1], int(move_state), _stream()), "pie_hip_conv_silu")
+    return out
+
+
+def conv_state(fused, rows: StateRows, channels: int, taps: int) -> None:
+    base = C.c_void_p(rows.rs_base)
+    _check(kernels().pie_hip_delta_conv_state(_dt(fused), _ptr(fused), base, C.c_size_t(rows.rs_stride), C.c_size_t(rows.conv_offset),
+                                              C.c_void_p(rows.qo_indptr), C.c_void_p(rows.rs_slot), C.c_void_p(rows.rs_fresh),
+                                              rows.num_requests, fused.shape[1], channels, taps, _stream()), "pie_hip_delta_conv_state")
+
+
+def decay_memory(form: str, rule: DecayRule, rows: StateRows, fused, q_off: int, k_off: int, v_off: int, gates, qo_indptr=None):
+    """(o [N, heads * vdim], den [N, heads, 2]) by "scan", "chunked" or "step" (one row per request)."""
+    n, lib = fused.shape[0], kernels()
+    o = torch.full((n, rule.heads * rule.vdim), 3.0, dtype=torch.float32, device=fused.device)
+    den = torch.full((n, rule.heads, 2), 3.0, dtype=torch.float32, device=fused.device)
+    ldg = 0 if gates is None else gates.shape[1]
+    if form == "step":
+        _check(lib.pie_hip_decay_step(_dt(fused), C.byref(rule), C.byref(rows), _ptr(fused), q_off, k_off, v_off, fused.shape[1],
+                                      _ptr(gates), ldg, None, None, 0, 0, None, _ptr(o), _ptr(den), None, 0, 0, None, None, 0,
+                                      C.c_float(1.0), C.c_float(0.0), _stream()), "pie_hip_decay_step")
+        return o, den
+    at = lambda off: C.c_void_p(fused.data_ptr() + off * fused.element_size())
+    if form == "scan":
+        _check(lib.pie_hip_decay_scan(_dt(fused), C.byref(rule), C.byref(rows), at(q_off), at(k_off), at(v_off), fused.shape[1], _ptr(gates),
+                                      ldg, _ptr(o), _ptr(den), _stream()), "pie_hip_decay_scan")
+        return o, den
+    qo = qo_indptr.tolist()
+    chunks, first = [], [0]
+    for r in range(len(qo) - 1):
+        chunks += [(i, min(64, qo[r + 1] - i)) for i in range(qo[r], qo[r + 1], 64)]
+        first.append(len(chunks))
+    lib.pie_hip_decay_chunked_workspace_bytes.restype = C.c_size_t
+    need = int(lib.pie_hip_decay_chunked_workspace_bytes(C.byref(rule), len(chunks)))
+    ws = torch.empty(max(need, 16), dtype=torch.uint8, device=fused.device)
+    ct = torch.tensor(chunks, dtype=torch.int32, device=fused.device)
+    ft = torch.tensor(first, dtype=torch.int32, device=fused.device)
+    _check(lib.pie_hip_decay_chunked(C.byref(rule), C.byref(rows), at(q_off), at(k_off), at(v_off), fused.shape[1], _ptr(gates), ldg, _ptr(o),
+                                     _ptr(den), _ptr(ct), _ptr(ft), len(chunks), _ptr(ws), C.c_size_t(need), _stream()),
+           "pie_hip_decay_chunked")
+    return o, den
+
+
+def decay_out(rule: DecayRule, rows: StateRows, o, den, gate, gate_act: int, norm_w, out_scale: float, eps: float) -> torch.Tensor:
+    y = torch.full(gate.shape, 3.0, dtype=gate.dtype, device=gate.device)
+    _check(kernels().pie_hip_decay_out(_dt(gate), C.byref(rule), C.byref(rows), _ptr(o), _ptr(den), _ptr(gate), gate.shape[1], gate_act,
+                                       _ptr(norm_w), _ptr(y), y.shape[1], C.c_float(out_scale), C.c_float(eps), _stream()),
+           "pie_hip_decay_out")
+    return y
+
+
+def decay_step_fused(rule: DecayRule, rows: StateRows, fused, q_off, k_off, v_off, gates, gate, gate_act, norm_w, out_scale, eps) -> torch.Tensor:
+    """The step with norm and gate in the same launch (a block per head)."""
+    y = torch.full(gate.shape, 3.0, dtype=gate.dtype, device=gate.device)
+    _check(kernels().pie_hip_decay_step(_dt(fused), C.byref(rule), C.byref(rows), _ptr(fused), q_off, k_off, v_off, fused.shape[1],
+                                        _ptr(gates), 0 if gates is None else gates.shape[1], None, None, 0, 0, None, None, None, _ptr(gate),
+                                        gate.shape[1], gate_act, _ptr(norm_w), _ptr(y), y.shape[1], C.c_float(out_scale), C.c_float(eps),
+                                        _stream()), "pie_hip_decay_step")
+    return y
+
+
+def decay_step_conv(rule: DecayRule, rows: StateRows, fused, q_off, k_off, v_off, gates, conv_w, conv_b, skip) -> torch.Tensor:
+    """The step with the convolution ahead of it in the same launch; o with the skip added."""
+    o = torch.full((fused.shape[0], rule.heads * rule.vdim), 3.0, dtype=torch.float32, device=fused.device)
+    _check(kernels().pie_hip_decay_step(_dt(fused), C.byref(rule), C.byref(rows), _ptr(fused), q_off, k_off, v_off, fused.shape[1],
+                                        _ptr(gates), gates.shape[1], _ptr(conv_w), _ptr(conv_b), conv_w.shape[0], conv_w.shape[1], _ptr(skip),
+                                        _ptr(o), None, None, 0, 0, None, None, 0, C.c_float(1.0), C.c_float(0.0), _stream()),
+           "pie_hip_decay_step")
+    return o
+
+
+def gated_part_norm(o, x, skip, z, norm_w, heads, vdim, parts, rows: StateRows, eps, conv_fused=None, channels=0, taps=1) -> torch.Tensor:
+    y = torch.full(z.shape, 3.0, dtype=z.dtype, device=z.device)
+    _check(kernels().pie_hip_gated_part_norm(_dt(z), _ptr(o), _ptr(x), 0 if x is None else x.shape[1], _ptr(skip), _ptr(z), z.shape[1],
+                                             _ptr(norm_w), _ptr(y), y.shape[1], heads, vdim, parts, C.byref(rows), _ptr(conv_fused),
+                                             0 if conv_fused is None else conv_fused.shape[1], channels, taps, C.c_float(eps), _stream()),
+           "pie_hip_gated_part_norm")
+    return y

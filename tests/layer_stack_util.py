@@ -46,6 +46,110 @@ ATTENTION_ONLY = stack([latent(heads=4, dim=32, rot_dim=16, vdim=32, kv_rank=64,
 DELTA_ONLY = stack([delta(heads=4, kv_heads=4, dim=32, vdim=32, conv=4, ff=48), delta(heads=2, kv_heads=1, dim=64, vdim=16, conv=2)])
 
 
+# ---- Lofudra -----------------------------------------------------------------------------------------
+def dense(ff):
+    return dict(kind="dense", ff=ff) if ff else None
+
+
+def parallel(heads=6, kv_heads=2, dim=40, rot_dims=24, window=9, base=500.0, scale=None, r_heads=3, r_dim=20, r_vdim=12, decay=None,
+             left_scale=0.7, right_scale=1.2, ff=56):
+    left = dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, scale=scale if scale is not None else dim ** -0.5,
+                mask=dict(size=window), rot=dict(dims=rot_dims, base=base))
+    right = dict(heads=r_heads, dim=r_dim, vdim=r_vdim, decay=decay or [1.0 - 0.5 ** (2 + 3 * h) for h in range(r_heads)])
+    return dict(type="parallel", mlp=dense(ff), mixer=dict(left=left, right=right, left_scale=left_scale, right_scale=right_scale))
+
+
+def mlstm(heads=3, dim=20, vdim=24, gate_cap=9.0, ff=72):
+    return dict(type="mlstm", mlp=dense(ff), mixer=dict(heads=heads, dim=dim, vdim=vdim, gate_cap=gate_cap))
+
+
+def mamba2(heads=6, vdim=12, state=20, groups=3, conv=4, norm_groups=4, ff=40):
+    return dict(type="mamba2", mlp=dense(ff),
+                mixer=dict(heads=heads, vdim=vdim, state=state, groups=groups, conv=conv, norm_groups=norm_groups))
+
+
+def lofudra(layers, loop=None, width=112, vocab=97, eps=1e-4):
+    cfg = dict(architecture="Lofudra", layers=layers, width=width, vocab=vocab, norm=dict(eps=eps))
+    if loop:
+        cfg["loop"] = dict(zip(("start", "stop", "times"), loop))
+    return cfg
+
+
+# sizes off every padding unit, heads shared and not, norm parts that cut heads, convolutions of one to six
+# taps, windows of one token and wider than the prompts, no loop, a loop over some and over all layers, layers
+# without a feed-forward, sizes of every matrix-core form and of the plain ones
+LOFUDRA_CONFIGS = {
+    "trio": lofudra([mlstm(), mamba2(), parallel()], loop=(0, 2, 2)),
+    "first_attention": lofudra([parallel(heads=5, kv_heads=5, dim=18, rot_dims=18, window=1, r_heads=1, r_dim=7, r_vdim=9, ff=0),
+                                mamba2(heads=4, vdim=10, state=9, groups=4, conv=1, norm_groups=1, ff=31),
+                                mlstm(heads=1, dim=33, vdim=30, ff=0), mamba2(heads=2, vdim=18, state=40, groups=1, conv=6, norm_groups=6, ff=0)],
+                               loop=(1, 3, 3), width=75, vocab=130),
+    "all_looped": lofudra([parallel(heads=7, kv_heads=1, dim=64, rot_dims=32, window=33, left_scale=1.0, right_scale=1.0),
+                           mlstm(heads=2, dim=64, vdim=40), mamba2(heads=8, vdim=16, state=64, groups=2, conv=2, norm_groups=2)], loop=(0, 3, 2)),
+    "wide": lofudra([parallel(heads=20, kv_heads=1, dim=96, rot_dims=96, window=500, r_heads=2, r_dim=128, r_vdim=64, ff=64),
+                     mlstm(heads=2, dim=130, vdim=68, gate_cap=15.0), mamba2(heads=4, vdim=64, state=128, groups=1, conv=3, norm_groups=4),
+                     parallel(heads=4, kv_heads=2, dim=192, rot_dims=64, window=70, r_heads=2, r_dim=256, r_vdim=40)], width=160, vocab=64),
+    "wider": lofudra([parallel(heads=2, kv_heads=1, dim=300, rot_dims=100, window=40, r_heads=1, r_dim=40, r_vdim=300, ff=0),
+                      mlstm(heads=1, dim=260, vdim=36), mlstm(heads=2, dim=24, vdim=264),
+                      parallel(heads=3, kv_heads=3, dim=250, rot_dims=250, window=64, ff=0)], loop=(1, 2, 1), width=128, vocab=80),
+}
+
+
+def lofudra_weights(cfg, seed=0, sharp=1.0):
+    """`sharp` scales the attention's query norms: large values make single keys stand out."""
+    rng = np.random.default_rng(seed)
+    w, H = {}, cfg["width"]
+
+    def lin(name, rows, cols, gain=1.0):
+        w[name] = bf16(rng.standard_normal((rows, cols)) * gain / np.sqrt(cols))
+
+    def vec(name, n, lo=0.7, hi=1.3):
+        w[name] = bf16(rng.uniform(lo, hi, n))
+
+    w["embed"] = bf16(rng.standard_normal((cfg["vocab"], H)))
+    if "loop" in cfg:
+        w["loop.step"] = bf16(rng.standard_normal((cfg["loop"]["times"], H)) * 0.5)
+    for i, layer in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", layer["mixer"]
+        x = p + "mix."
+        for n in ("norm1", "norm1b") + (("norm2", "norm2b") if layer["mlp"] else ()):
+            vec(p + n, H)
+        if layer["type"] == "parallel":
+            a, r = m["left"], m["right"]
+            for n, heads in (("q", a["heads"]), ("k", a["kv_heads"])):
+                lin(x + f"left.{n}", heads * a["dim"], H)
+                w[x + f"left.{n}.b"] = bf16(rng.standard_normal(heads * a["dim"]) * 0.5)
+                vec(x + f"left.{n}.norm", a["dim"], *((0.7 * sharp, 1.3 * sharp) if n == "q" else (0.7, 1.3)))
+            lin(x + "left.o", H, a["heads"] * a["dim"])
+            for n, rows in (("q", r["dim"]), ("k", r["dim"]), ("v", r["vdim"]), ("g", r["vdim"])):
+                lin(x + f"right.{n}", r["heads"] * rows, H)
+            lin(x + "right.o", H, r["heads"] * r["vdim"])
+        elif layer["type"] == "mlstm":
+            for n, rows in (("q", m["dim"]), ("k", m["dim"]), ("v", m["vdim"]), ("g", m["vdim"])):
+                lin(x + n, m["heads"] * rows, H)
+            lin(x + "o", H, m["heads"] * m["vdim"])
+            vec(x + "norm", m["heads"] * m["vdim"])
+            for n, mean in (("i", -1.0), ("f", 3.0)):
+                lin(x + n, m["heads"], H, 3.0)
+                w[x + n + ".b"] = bf16(mean + rng.standard_normal(m["heads"]))
+        else:
+            inner, bc = m["heads"] * m["vdim"], m["groups"] * m["state"]
+            lin(x + "in", 2 * inner + 2 * bc + m["heads"], H)
+            w[x + "conv"] = bf16(rng.standard_normal((inner + 2 * bc, m["conv"])) * 0.6)
+            w[x + "conv.b"] = bf16(rng.standard_normal(inner + 2 * bc) * 0.3)
+            w[x + "dt_bias"] = bf16(rng.uniform(-3.0, 0.5, m["heads"]))
+            w[x + "A_log"] = bf16(rng.uniform(-2.0, 1.0, m["heads"]))
+            w[x + "D"] = bf16(rng.standard_normal(m["heads"]))
+            vec(x + "norm", inner)
+            lin(x + "o", H, inner)
+        if layer["mlp"]:
+            lin(p + "mlp.up", layer["mlp"]["ff"], H)
+            lin(p + "mlp.down", H, layer["mlp"]["ff"])
+    vec("final.norm", H)
+    lin("head", cfg["vocab"], H, 3.0)
+    return w
+
+
 def bf16(a):
     """Rounds to the nearest bf16 value (ties to even); returns float32."""
     u = np.ascontiguousarray(a, np.float32).view(np.uint32)
@@ -159,3 +263,31 @@ def assert_close(got, want, dtype, what=""):
         assert e.max() < F32_TOL, (what, e.max(), int(e.argmax()))
     else:
         assert e.max() < BF16_TOL and (len(e) < 8 or np.median(e) < BF16_MEDIAN), (what, np.median(e), e.max(), int(e.argmax()))
+
+
+def engine(directory, dtype, **kw):
+    from pie_amd.driver import Driver
+    from pie_amd.engine import Engine
+
+    d = Driver(stack_toml(directory, dtype, **kw))
+    return d, Engine(d)
+
+
+def tokens(cfg, n, seed=0):
+    return [int(x) for x in np.random.default_rng(seed).integers(0, cfg["vocab"], n)]
+
+
+def run(e, rid, toks, portions):
+    """Logits of every position, the request cut into `portions` (the last one repeats)."""
+    got, at, i = [], 0, 0
+    while at < len(toks):
+        n = min(portions[min(i, len(portions) - 1)], len(toks) - at)
+        got.append(e.step([(rid, toks[at:at + n], list(range(n)))])[0])
+        at += n
+        i += 1
+    return np.concatenate(got)
+
+
+def close_tie(logits):
+    top = np.sort(logits, axis=-1)[..., -2:]
+    return top[..., 1] - top[..., 0]

@@ -9,7 +9,8 @@ from pathlib import Path
 import numpy as np
 import pytest
 
-from layer_stack_util import (ATTENTION_ONLY, CONFIGS, DELTA_ONLY, assert_close, delta, latent, random_weights, stack, stack_toml, write_stack)
+from layer_stack_util import (ATTENTION_ONLY, CONFIGS, DELTA_ONLY, assert_close, close_tie, delta, engine, latent, random_weights, run, stack,
+                              tokens, write_stack)
 from oracle import layer_stack as ls
 
 pytestmark = pytest.mark.gpu
@@ -38,29 +39,6 @@ def models(tmp_path_factory):
             return cache[key]
         out[name] = (cfg, w, write_stack(tmp_path_factory.mktemp(name), cfg, w), ref)
     return out
-
-
-def engine(directory, dtype, **kw):
-    from pie_amd.driver import Driver
-    from pie_amd.engine import Engine
-
-    d = Driver(stack_toml(directory, dtype, **kw))
-    return d, Engine(d)
-
-
-def tokens(cfg, n, seed=0):
-    return [int(x) for x in np.random.default_rng(seed).integers(0, cfg["vocab"], n)]
-
-
-def run(e, rid, toks, portions):
-    """Logits of every position, the request cut into `portions` (the last one repeats)."""
-    got, at, i = [], 0, 0
-    while at < len(toks):
-        n = min(portions[min(i, len(portions) - 1)], len(toks) - at)
-        got.append(e.step([(rid, toks[at:at + n], list(range(n)))])[0])
-        at += n
-        i += 1
-    return np.concatenate(got)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -178,11 +156,6 @@ def test_weights_come_from_the_file_to_the_last_bit(gpu, models):
         assert np.array_equal(rows[:m["q_rank"], :112], w["l0.mix.dq"])
         kv_off = -(-m["q_rank"] // 16) * 16
         assert np.array_equal(rows[kv_off:kv_off + m["kv_rank"] + m["rot_dim"], :112], w["l0.mix.dkv"])
-
-
-def close_tie(logits):
-    top = np.sort(logits, axis=-1)[..., -2:]
-    return top[..., 1] - top[..., 0]
 
 
 @pytest.mark.parametrize("name", ["mixed", "expanded", "attention_only"])
