@@ -448,7 +448,7 @@ extern "C" int pie_hip_linear_f32out(int dtype, const void* act, const uint16_t*
     hipStream_t s = static_cast<hipStream_t>(stream);
     const auto* x = static_cast<const uint16_t*>(act);
     if (M >= 512 && N > 16)   // (row tiles fill the device: column tiles share their activations)
-        hipLaunchKernelGGL((linear_f32out_kernel<8, 4, 2>), dim3((N + 63) / 64, gy), dim3(512), 0, s, x, w_bf16, y, M, N, K);
+        hipLaunchKernelGGL((linear_f32out_kernel<8, 4, 8>), dim3((N + 63) / 64, gy), dim3(512), 0, s, x, w_bf16, y, M, N, K);
     else
         hipLaunchKernelGGL((linear_f32out_kernel<16, 1, 8>), dim3(N / 16, gy), dim3(1024), 0, s, x, w_bf16, y, M, N, K);
     return launch_status();

@@ -86,16 +86,27 @@ def test_unequal_batches_equal_each_request_alone(gpu, models, name, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-def test_a_wide_decode_batch(gpu, models, dtype):
-    """Many requests of unequal length decoded together: the launches that other batch sizes take."""
-    cfg, directory, ref = models["wide"]
+@pytest.mark.parametrize("which", ["wide", "many_heads"])
+def test_a_wide_decode_batch(gpu, models, tmp_path, which, dtype):
+    """Many requests of unequal length decoded together: the launches that other batch sizes take (whole heads
+    per block, the convolution ahead of the step)."""
+    if which == "wide":
+        cfg, directory, ref = models["wide"]
+    else:
+        cfg = lofudra([mamba2(heads=32, vdim=8, state=16, groups=2, conv=4, norm_groups=2), mlstm(heads=12, dim=16, vdim=48)], width=96, vocab=70)
+        w = lofudra_weights(cfg, 9)
+        directory, w64 = write_stack(tmp_path, cfg, w), {k: v.astype(np.float64) for k, v in w.items()}
+        ref = lambda toks: ls.forward(cfg, w64, toks)
     seqs = {r: tokens(cfg, 20 + 7 * (r % 5), 50 + r % 3) for r in range(40)}
     d, e = engine(directory, dtype, total_pages=160, max_tokens=2048, slots=40, requests=40)
     with d:
         e.step([(r, s[:-6], []) for r, s in seqs.items()])
         got = [e.step([(r, [s[len(s) - 6 + i]], [0]) for r, s in seqs.items()]) for i in range(6)]
     for r, s in seqs.items():
-        assert_close(np.concatenate([g[r] for g in got]), ref(s)[-6:], dtype, r)
+        if r < 15:   # (the others repeat them)
+            assert_close(np.concatenate([g[r] for g in got]), ref(s)[-6:], dtype, r)
+        else:
+            assert_close(np.concatenate([g[r] for g in got]), np.concatenate([g[r % 15] for g in got]), dtype, r)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
