@@ -284,10 +284,125 @@ def forward_sandwich(cfg, w, tokens, want_layers=False):
     return (logits, np.stack(states)) if want_layers else logits
 
 
+# ---- Fobanex ---------------------------------------------------------------------------------------
+def grouped_attention(q, k, v, scale):
+    """q [T, H, d], k [T, G, d], v [T, G, dv]; query head h reads key head h // (H / G) -> [T, H, dv]."""
+    src = np.arange(q.shape[1]) // (q.shape[1] // k.shape[1])
+    return causal_softmax_attention(np.einsum("ihd,jhd->hij", q, k[:, src]) * scale, v[:, src])
+
+
+def rotate_heads(x, rot):
+    """Interleaved rotation of [T, heads, d] by each row's place (no spec: as it is)."""
+    return rotate_pairs(x, np.arange(len(x)), rot) if rot else x
+
+
+def normed_attention(h, w, p, m, eps, shared=None):
+    """One norm over all query rows and one over all key rows, ahead of the split into heads."""
+    T, dim = len(h), m["dim"]
+    q = rms_norm(h @ w[p + "q"].T, w[p + "q.norm"], eps).reshape(T, m["heads"], dim)
+    k = rms_norm(h @ w[p + "k"].T, w[p + "k.norm"], eps).reshape(T, m["kv_heads"], dim)
+    v = (h @ w[p + "v"].T).reshape(T, m["kv_heads"], m["vdim"])
+    o = grouped_attention(rotate_heads(q, m.get("rot")), rotate_heads(k, m.get("rot")), v, m["scale"])
+    return o.reshape(T, -1) @ w[p + "o"].T
+
+
+def key_value_attention(h, w, p, m, eps, shared=None):
+    """The keys as projected are the values; a logistic gate on the concatenated heads."""
+    T = len(h)
+    q, k = (h @ w[p + "q"].T).reshape(T, m["heads"], m["dim"]), (h @ w[p + "k"].T).reshape(T, m["kv_heads"], m["dim"])
+    o = grouped_attention(rotate_heads(q, m.get("rot")), rotate_heads(k, m.get("rot")), k, m["scale"])
+    return (o.reshape(T, -1) * sigmoid(h @ w[p + "g"].T)) @ w[p + "o"].T
+
+
+def latent_of(h, w, p, m, eps):
+    """What a latent layer caches per token: the normed latent and the rotated key part."""
+    rank = m["kv_rank"]
+    kv = h @ w[p + "dkv"].T
+    return rms_norm(kv[:, :rank], w[p + "dkv.norm"], eps), rotate_halves(kv[:, rank:], np.arange(len(h)), m["rot"])
+
+
+def gated_latent_attention(h, w, p, m, eps, shared=None):
+    """Half-split rotation and a logistic gate; `shared`: another layer's latents and rotated key parts."""
+    T = len(h)
+    H, dim, rd, dv = m["heads"], m["dim"], m["rot_dim"], m["vdim"]
+    c, kr = shared if shared is not None else latent_of(h, w, p, m, eps)
+    cq = rms_norm(h @ w[p + "dq"].T, w[p + "dq.norm"], eps)
+    q = (cq @ w[p + "uq"].T).reshape(T, H, dim + rd)
+    qr = rotate_halves(q[..., dim:], np.arange(T), m["rot"])
+    kn, v = (c @ w[p + "uk"].T).reshape(T, H, dim), (c @ w[p + "uv"].T).reshape(T, H, dv)
+    scores = (np.einsum("ihd,jhd->hij", q[..., :dim], kn) + np.einsum("ihd,jd->hij", qr, kr)) * m["scale"]
+    o = causal_softmax_attention(scores, v).reshape(T, H * dv)
+    return (o * sigmoid(h @ w[p + "g"].T)) @ w[p + "o"].T
+
+
+def gated_feed_forward(h, w, p):
+    g, u = (h @ w[p + n].T + w[p + n + ".b"] for n in ("gate", "up"))
+    return (silu(g) * u) @ w[p + "down"].T + w[p + "down.b"]
+
+
+def clamped_expert(h, w, p, limit):
+    g, u = np.minimum(h @ w[p + "gate"].T, limit), np.clip(h @ w[p + "up"].T, -limit, limit)
+    return (g * sigmoid(1.702 * g) * (u + 1.0)) @ w[p + "down"].T
+
+
+def route(z, r):
+    """Router logits [T, E] -> weights [T, E], zero where an expert is not chosen."""
+    T, E = z.shape
+    s = np.exp(z - z.max(axis=-1, keepdims=True))
+    s /= s.sum(axis=-1, keepdims=True)
+    out = np.zeros_like(s)
+    groups = r.get("groups") or dict(count=1, keep=1)
+    size = E // groups["count"]
+    for t in range(T):
+        best = np.argsort(-s[t].reshape(groups["count"], size).max(axis=-1), kind="stable")[:groups["keep"]]
+        open_to = np.where(np.isin(np.arange(E) // size, best), s[t], -1.0)
+        chosen = np.argsort(-open_to, kind="stable")[:r["top"]]
+        out[t, chosen] = s[t, chosen] / (s[t, chosen].sum() + 1e-20) * r["scale"]
+    return out
+
+
+def mixture(h, w, p, mlp):
+    r = mlp["router"]
+    weight = route(h @ w[p + "router"].T, r)
+    y = np.zeros_like(h)
+    for e in range(r["experts"]):
+        t = np.nonzero(weight[:, e])[0]
+        if len(t):
+            y[t] += weight[t, e, None] * clamped_expert(h[t], w, f"{p}e{e}.", mlp["expert"]["limit"])
+    return y
+
+
+SHARED_AHEAD_MIXERS = {"attention": normed_attention, "attention_2": key_value_attention, "latent_attention": gated_latent_attention}
+
+
+def forward_shared_norm(cfg, w, tokens, want_layers=False):
+    """One norm ahead of each layer; the mixer and the feed-forward both read it and join the stream together."""
+    eps = cfg["norm"]["eps"]
+    x = np.asarray(w["embed"], np.float64)[np.asarray(tokens)] * cfg["embedding"]["scale"]
+    states, latents = [], {}
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, mlp = f"l{i}.", layer["mixer"], layer.get("mlp")
+        h = rms_norm(x, w[p + "norm1"], eps)
+        shared = None
+        if layer["type"] == "latent_attention":
+            if m.get("kv_from") is None:
+                latents[i] = latent_of(h, w, p + "mix.", m, eps)
+            shared = latents[i if m.get("kv_from") is None else m["kv_from"]]
+        y = SHARED_AHEAD_MIXERS[layer["type"]](h, w, p + "mix.", m, eps, shared)
+        if mlp:
+            y = y + (gated_feed_forward(h, w, p + "mlp.") if mlp["kind"] == "dense" else mixture(h, w, p + "mlp.", mlp))
+        x = x + y
+        states.append(x)
+    logits = rms_norm(x, w["final.norm"], eps) @ w["head"].T
+    return (logits, np.stack(states)) if want_layers else logits
+
+
 def forward(cfg, w, tokens, want_layers=False):
     """Logits [T, vocab] of one sequence (and the residual stream after every layer)."""
     if cfg["architecture"] == "Lofudra":
         return forward_sandwich(cfg, w, tokens, want_layers)
+    if cfg["architecture"] == "Fobanex":
+        return forward_shared_norm(cfg, w, tokens, want_layers)
     eps = cfg["norm"]["eps"]
     x = np.asarray(w["embed"], np.float64)[np.asarray(tokens)]
     states = []
