@@ -48,9 +48,12 @@ extern "C" {
  *   3  lm_head argmax pairs, attention merge in the output projection, uniform-row hints
  *   4  the `swiglu` argument of the linears is an epilogue code (PIE_HIP_EPI_*: 0 and 1
  *      mean what they did, 2 is the squared ReLU); the layer-stack kernels
- *   5  current: epilogue code 3 (exact GELU); grouped attention with windows and sinks, memories with
- *      one decay per head, residual_norm */
-#define PIE_HIP_ABI_VERSION 5
+ *   5  epilogue code 3 (exact GELU); grouped attention with windows and sinks, memories with
+ *      one decay per head, residual_norm
+ *   6  current: gated products with biases and clamps (PieHipGlu, the *_glu entry points); gates on the
+ *      outputs of grouped and latent attention; norms over whole projections; expert groups;
+ *      residual_join */
+#define PIE_HIP_ABI_VERSION 6
 int pie_hip_abi_version(void);
 
 /* ---- W4A16 ("int4b8", symmetric, group-quantised) ------------------------- */
@@ -117,6 +120,15 @@ int pie_hip_gemv_w4a16_tuned(const uint16_t* act_bf16, const uint32_t* packed,
 #define PIE_HIP_EPI_SWIGLU 1
 #define PIE_HIP_EPI_RELU2 2
 #define PIE_HIP_EPI_GELU 3
+/* What a gated product (PIE_HIP_EPI_SWIGLU) does with its column pairs besides the plain rule:
+ *   g = min(g + bias, limit), u = clamp(u + bias, -limit, limit),
+ *   y = g / (1 + exp(-alpha g)) * (u + shift)
+ * bias: fp32 [N] in the order of the weight rows (NULL: none), added to the fp32 sums before they are
+ * rounded to the output type.  {NULL, INFINITY, 1, 0} is the plain rule. */
+typedef struct {
+    const float* bias;
+    float limit, alpha, shift;
+} PieHipGlu;
 #define PIE_HIP_FMT_INT4B8 0
 #define PIE_HIP_FMT_INT8 1
 #define PIE_HIP_FMT_FP8 2
@@ -125,6 +137,11 @@ int pie_hip_linear_fused(int format, const uint16_t* act_bf16, const uint16_t* n
                          float eps, const void* weight, const void* scale, int scale_is_bf16,
                          int group_size, uint16_t* y_bf16, int M, int N, int K, int beta,
                          int swiglu, void* stream);
+/* The same with `glu` (NULL: the plain rule), PIE_HIP_EPI_SWIGLU only. */
+int pie_hip_linear_fused_glu(int format, const uint16_t* act_bf16, const uint16_t* norm_weight_bf16,
+                             float eps, const void* weight, const void* scale, int scale_is_bf16,
+                             int group_size, uint16_t* y_bf16, int M, int N, int K, int beta,
+                             int swiglu, const PieHipGlu* glu, void* stream);
 
 /*
  * The attention output projection of a decode step with the attention's split merge in its
@@ -202,6 +219,11 @@ int pie_hip_lm_head_argmax(const uint16_t* act_bf16, const uint16_t* norm_weight
 int pie_hip_gemm_skinny(int format, const uint16_t* act_bf16, const void* weight,
                         const void* scale, int scale_is_bf16, int group_size, uint16_t* y_bf16,
                         int M, int N, int K, int beta, int swiglu, void* stream);
+/* The same with `glu` (NULL: the plain rule), over row-major or (`tiled`) tile-major weights. */
+int pie_hip_gemm_skinny_glu(int format, const uint16_t* act_bf16, const void* weight,
+                            const void* scale, int scale_is_bf16, int group_size, uint16_t* y_bf16,
+                            int M, int N, int K, int beta, int swiglu, int tiled, const PieHipGlu* glu,
+                            void* stream);
 
 /*
  * Tiled weight-only GEMM on the matrix cores for prefill and large batches (compute-bound M):
@@ -233,6 +255,11 @@ int pie_hip_gemm_mfma_splitk(int format, const uint16_t* act_bf16, const void* w
                              const void* scale, int scale_is_bf16, int group_size,
                              uint16_t* y_bf16, int M, int N, int K, int beta, int swiglu,
                              void* workspace, size_t workspace_bytes, void* stream);
+/* Either of the two (workspace NULL: not split) with `glu` (NULL: the plain rule). */
+int pie_hip_gemm_mfma_glu(int format, const uint16_t* act_bf16, const void* weight,
+                          const void* scale, int scale_is_bf16, int group_size,
+                          uint16_t* y_bf16, int M, int N, int K, int beta, int swiglu,
+                          const PieHipGlu* glu, void* workspace, size_t workspace_bytes, void* stream);
 
 /*
  * MoE grouped weight-only GEMM: one skinny problem per expert in a single launch.
@@ -252,6 +279,15 @@ int pie_hip_moe_grouped_gemm(int format, const uint16_t* act_bf16, const int32_t
                              size_t weight_stride_bytes, const void* scales,
                              size_t scale_stride_bytes, int scale_is_bf16, int group_size,
                              uint16_t* y_bf16, int N, int K, int swiglu, void* stream);
+/* The same with `glu` (NULL: the plain rule; its bias is [N], the same for every expert), over row-major or
+ * (`tiled`) tile-major weights. */
+int pie_hip_moe_grouped_gemm_glu(int format, const uint16_t* act_bf16, const int32_t* route_act_rows,
+                                 const int32_t* expert_offsets, int num_experts,
+                                 int max_rows_per_expert, const void* weights,
+                                 size_t weight_stride_bytes, const void* scales,
+                                 size_t scale_stride_bytes, int scale_is_bf16, int group_size,
+                                 uint16_t* y_bf16, int N, int K, int swiglu, int tiled,
+                                 const PieHipGlu* glu, void* stream);
 
 /*
  * Tile-major weight layout for the skinny and grouped GEMMs.  The 16 bytes that lane (j, q) of a
@@ -312,6 +348,14 @@ int pie_hip_moe_route(const uint16_t* router_logits_bf16, int32_t* topk_idx, flo
 int pie_hip_moe_route_opt(const uint16_t* router_logits_bf16, int32_t* topk_idx, float* topk_weight,
                       int32_t* expert_offsets, int32_t* route_token, int32_t* route_pos,
                       int num_tokens, int num_experts, int top_k, int renormalize, void* stream);
+/* The same from fp32 logits (rows of ld_logits), with the experts in num_groups equal groups of neighbours:
+ * a token chooses among the experts of the keep_groups groups whose best expert has the largest probability
+ * (ties to the lowest group); weight = p / (sum of the chosen p + 1e-20) * weight_scale.  top_k <= 64 and at most
+ * keep_groups * num_experts / num_groups.  Up to sixteen tokens take one launch. */
+int pie_hip_moe_route_groups(const float* router_logits, int ld_logits, int32_t* topk_idx, float* topk_weight,
+                             int32_t* expert_offsets, int32_t* route_token, int32_t* route_pos, int num_tokens,
+                             int num_experts, int top_k, int num_groups, int keep_groups, float weight_scale,
+                             void* stream);
 
 /*
  * A decode batch's way into the MoE block in two launches instead of four: per token the RMSNorm
@@ -809,10 +853,11 @@ int pie_hip_linear_f32(const float* act, const uint16_t* w_bf16, float* y, int M
  * pie_hip_latent_prep: fused[n] = [query latent q_rank | .. | kv_off: latent kv_rank, rot_dim key
  *   values]; cq[n] = the query latent normed (compact rows of ld_cq, zero padded); the token's
  *   cache row = the normed latent and the key values rotated in adjacent pairs (first rot_dims of
- *   them, table of pie_hip_rotary_table).
+ *   them, table of pie_hip_rotary_table).  kv_norm NULL: only the query latent (fused holds nothing else).
  * pie_hip_head_linear: y[n, h, c] = sum_k W[h, c, k] act[n, h, k] (heads act_stride / y_stride
  *   apart in rows of ld_act / ld_y; C % 16 == 0, K % 32 == 0).  With rotp > 0 also
- *   y[n, h, C + i] = the rotated act[n, h, rot_off + i], i < rot_dim, zeros to rotp.
+ *   y[n, h, C + i] = the rotated act[n, h, rot_off + i], i < rot_dim, zeros to rotp.  With gate,
+ *   y[n, h, c] is multiplied by the logistic function of gate[n, h * C + c] (rows of ld_gate).
  * pie_hip_latent_attn_rows_plain: o[n, h, :] = softmax_j(q[n, h, :] . row_j * scale) . row_j[:kvp]
  *   over the first row_kv_len[n] keys; q [rows, heads, ld_row], o [rows, heads, kvp].  Any sizes
  *   (kvp <= 2048).
@@ -823,7 +868,8 @@ int pie_hip_latent_prep(int dtype, const void* fused, const float* q_norm, const
                         int rot_dims, int ld_row, float eps, void* stream);
 int pie_hip_head_linear(int dtype, const void* act, const uint16_t* w_bf16, void* y, const float* rope_table,
                         int M, int heads, int C, int K, int ld_act, int act_stride, int ld_y, int y_stride,
-                        int rot_off, int rot_dim, int rot_dims, int rotp, void* stream);
+                        int rot_off, int rot_dim, int rot_dims, int rotp, const void* gate, int ld_gate,
+                        void* stream);
 int pie_hip_latent_attn_rows_plain(int dtype, const void* q, const void* pool, void* o,
                                    const uint32_t* kv_page_indices, const uint32_t* row_page_begin,
                                    const int32_t* row_kv_len, int num_rows, int heads, int kvp, int ld_row,
@@ -848,7 +894,8 @@ int pie_hip_latent_attn_rows(const uint16_t* q, const uint16_t* pool, uint16_t* 
  * pie_hip_latent_attn_prefill: rows [row0, row0 + num_rows) of one request, q [rows, heads, dimp +
  *   rotp] (the rotated part not yet rotated: rope_table rows as for pie_hip_latent_prep), kv
  *   [num_keys, heads, dimp + vdp] the projected keys and values, rot as gathered; row n sees its
- *   first row_kv_len[n] keys; o [rows, ld_o], heads vdp apart.  (dimp + rotp) / 32 in 2..6, vdp / 32
+ *   first row_kv_len[n] keys; o [rows, ld_o], heads vdp apart, times the logistic function of
+ *   gate[n, h * vdp + c] (rows of ld_gate; NULL: none).  (dimp + rotp) / 32 in 2..6, vdp / 32
  *   in 1..4 (pie_hip_latent_attn_prefill_supported). */
 int pie_hip_latent_gather(const uint16_t* pool, const uint32_t* pages, uint16_t* lat, uint16_t* rot, int num_keys,
                           int kvp, int rotp, int page_size, void* stream);
@@ -856,7 +903,7 @@ int pie_hip_latent_attn_prefill_supported(int dimp, int rotp, int vdp);
 int pie_hip_latent_attn_prefill(const uint16_t* q, const uint16_t* kv, const uint16_t* rot, uint16_t* o,
                                 const float* rope_table, const int32_t* row_kv_len, int row0, int num_rows,
                                 int num_keys, int heads, int dimp, int rotp, int rot_dims, int vdp, int ld_o,
-                                float scale, void* stream);
+                                float scale, const uint16_t* gate, int ld_gate, void* stream);
 
 /*
  * Gated delta rule with a decay per head and key channel.  row_req [N]: request of each row;
@@ -923,6 +970,32 @@ int pie_hip_residual_norm(int dtype, const void* y, const float* post_weight, fl
                           const uint32_t* token_ids, const uint16_t* table_bf16, int vocab, const float* add,
                           const float* next_weight, void* x_act, int rows, int width, int ldy, int ld, float eps,
                           void* stream);
+/* What a mixture of experts leaves per token: its routes' rows y (compute type, rows of ld), the row pos[t, k]
+ * of each route and its weight [t, k]. */
+typedef struct {
+    const void* y;
+    const int32_t* pos;
+    const float* weight;
+    int top_k, ld;
+} PieHipRoutes;
+/* One step of the residual stream of layers whose sublayers read one norm and join the stream together:
+ *   x[n] = (read_x ? x[n] : 0) + y[n] + y2[n] + add + sum_k weight[n, k] routes.y[pos[n, k]] + table[token_ids[n]] *
+ *          table_scale
+ *   x_act[n] = x[n] / sqrt(mean(x[n]^2) + eps) * next_weight        (compute type)
+ * y (rows of ldy), y2 (rows of ldy2), add [width], routes and token_ids with table_bf16 may each be NULL (left
+ * out); next_weight NULL: x_act = x.  ids >= vocab read row 0.  Columns from the width to ld are not touched. */
+int pie_hip_residual_join(int dtype, const void* y, int ldy, const void* y2, int ldy2, const float* add,
+                          const PieHipRoutes* routes, float* x, int read_x, const uint32_t* token_ids,
+                          const uint16_t* table_bf16, int vocab, float table_scale, const float* next_weight,
+                          void* x_act, int rows, int width, int ld, float eps, void* stream);
+/* The fp32 forms of a mixture's products and of the gated rule:
+ * pie_hip_moe_grouped_linear_f32: rows expert_offsets[e] .. expert_offsets[e + 1] of y [routes, N] are
+ *   act[route_act_rows[r]] (or act[r]) . W_e^T, W_e bf16 [N, K] at w + e * N * K; no expert has more than max_rows.
+ * pie_hip_glu_f32: y[m, i] = the rule of PieHipGlu on columns (2i, 2i + 1) of x [M, 2 n]. */
+int pie_hip_moe_grouped_linear_f32(const float* act, const int32_t* route_act_rows, const int32_t* expert_offsets,
+                                   int num_experts, int max_rows, const uint16_t* w_bf16, float* y, int N, int K,
+                                   void* stream);
+int pie_hip_glu_f32(const float* x, const PieHipGlu* glu, float* y, int M, int n, void* stream);
 /* y[M, N] fp32 = act[M, K] . W[N, K]^T over bf16 weights (fp32 sums, not rounded): the few columns that
  * drive a recurrence.  K % 32 == 0, N % 16 == 0. */
 int pie_hip_linear_f32out(int dtype, const void* act, const uint16_t* w_bf16, float* y, int M, int N, int K,
@@ -938,32 +1011,43 @@ int pie_hip_linear_f32out(int dtype, const void* act, const uint16_t* w_bf16, fl
  *   normed per head (weights [dim], or NULL) and rotated over their first rot_dims entries, entry i
  *   with entry i + rot_dims / 2 (table of pie_hip_rotary_table); q goes to q_out [N, heads, dimp].
  * pie_hip_group_attn_rows: one query row per block row; rows NULL: rows 0 .. num_rows - 1, else the
- *   listed ones.  o[row, h * dimp ..] * out_scale, rows of ld_o.  bf16; dimp / 32 in {1, 2, 3, 4, 6, 8};
+ *   listed ones.  o[row, h * dimp ..] * out_scale, rows of ld_o, in all three forms also times the
+ *   logistic function of gate[row, h * dimp ..] (rows of ld_gate; NULL: none).  bf16; dimp / 32 in {1, 2, 3, 4, 6, 8};
  *   page_size % 16 == 0.  Workspace pie_hip_group_attn_rows_workspace_bytes.
  * pie_hip_group_attn_tiles: tiles [num_tiles][2] = (first row, rows) of consecutive rows of one request,
  *   at most pie_hip_group_attn_tile_rows(heads, kv_heads, half) of them; half tiles only for dimp > 128.
  * pie_hip_group_attn_plain: any size and compute type, dimp <= 1024.
+ * pie_hip_group_attn_prep_joint: as pie_hip_group_attn_prep without biases, with one norm over a row's whole
+ *   query projection and one over its whole key projection (weights [heads * dim] and [kv_heads * dim], or
+ *   NULL), values of their own size vdim <= dimp, and either pairing of the rotated entries
+ *   (PIE_HIP_ROPE_HALF or PIE_HIP_ROPE_ADJACENT).
  */
 int pie_hip_group_attn_prep(int dtype, const void* fused, int q_off, int k_off, int v_off, const float* q_bias,
                             const float* k_bias, const float* q_norm, const float* k_norm, const float* rope_table,
                             int rot_dims, const int64_t* kv_slots, void* q_out, void* pool, int num_tokens,
                             int ld_fused, int heads, int kv_heads, int dim, int dimp, float eps, void* stream);
+int pie_hip_group_attn_prep_joint(int dtype, const void* fused, int q_off, int k_off, int v_off, const float* q_norm,
+                                  const float* k_norm, const float* rope_table, int rot_dims, int pairing,
+                                  const int64_t* kv_slots, void* q_out, void* pool, int num_tokens, int ld_fused,
+                                  int heads, int kv_heads, int dim, int vdim, int dimp, float eps, void* stream);
 int pie_hip_group_attn_supported(int dimp);
 size_t pie_hip_group_attn_rows_workspace_bytes(int num_rows, int heads, int kv_heads, int dimp, int max_kv_len, int window);
 int pie_hip_group_attn_rows(const uint16_t* q, const uint16_t* pool, uint16_t* o, const uint32_t* kv_page_indices,
                             const uint32_t* row_page_begin, const int32_t* row_kv_len, const int32_t* rows,
                             int num_rows, int heads, int kv_heads, int dimp, int ld_o, int page_size, float scale,
-                            int window, float sink, float out_scale, int max_kv_len, void* workspace,
+                            int window, float sink, float out_scale, const uint16_t* gate, int ld_gate,
+                            int max_kv_len, void* workspace,
                             size_t workspace_bytes, void* stream);
 int pie_hip_group_attn_tile_rows(int heads, int kv_heads, int half);
 int pie_hip_group_attn_tiles(const uint16_t* q, const uint16_t* pool, uint16_t* o, const uint32_t* kv_page_indices,
                              const uint32_t* row_page_begin, const int32_t* row_kv_len, const int32_t* tiles,
                              int num_tiles, int half, int heads, int kv_heads, int dimp, int ld_o, int page_size,
-                             float scale, int window, float sink, float out_scale, void* stream);
+                             float scale, int window, float sink, float out_scale, const uint16_t* gate,
+                             int ld_gate, void* stream);
 int pie_hip_group_attn_plain(int dtype, const void* q, const void* pool, void* o, const uint32_t* kv_page_indices,
                              const uint32_t* row_page_begin, const int32_t* row_kv_len, int num_rows, int heads,
                              int kv_heads, int dimp, int ld_o, int page_size, float scale, int window, float sink,
-                             float out_scale, void* stream);
+                             float out_scale, const void* gate, int ld_gate, void* stream);
 
 /*
  * Memories with one decay per head and token: S_t = d_t S_(t-1) + w_t k_t v_t^T (S [dim, vdim] fp32),

@@ -289,6 +289,15 @@ __device__ __forceinline__ float epilogue_pointwise(float v, int code) {
     return v;
 }
 
+// The gated rule on a column pair whose biases are in; {NULL, INFINITY, 1, 0} is the plain one.
+constexpr PieHipGlu kPlainGlu = {nullptr, __builtin_inff(), 1.f, 0.f};
+__device__ __forceinline__ float glu_value(float g, float u, const PieHipGlu& r) {
+    g = fminf(g, r.limit);
+    u = fminf(fmaxf(u, -r.limit), r.limit);
+    return g / (1.f + expf(-r.alpha * g)) * (u + r.shift);
+}
+inline bool glu_ok(const PieHipGlu* r, int epilogue) { return !r || (epilogue == PIE_HIP_EPI_SWIGLU && r->limit >= 0.f); }
+
 inline int launch_status() {
     return hipGetLastError() == hipSuccess ? PIE_HIP_OK : PIE_HIP_ERR_LAUNCH;
 }

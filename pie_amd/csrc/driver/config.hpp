@@ -21,7 +21,8 @@ namespace pie_hip_driver {
 // Each layer names a mixer (what exchanges information between tokens) with its own sizes, and an
 // optional feed-forward.  Mixers are listed here once, with every constant a parameter.
 
-// Rotary embedding of the first `dims` entries of a vector (which entries pair up is the mixer's).
+// Rotary embedding of the first `dims` entries of a vector (which entries pair up is the mixer's: neighbours,
+// or entry i with entry i + dims / 2).
 struct RotarySpec {
     int dims = 0;
     double base = 10000.0;
@@ -33,11 +34,15 @@ struct RotarySpec {
     }
 };
 
-// Attention over a cached low-rank latent per token and one rotated key part shared by the heads.
+// Attention over a cached low-rank latent per token and one rotated key part shared by the heads; optionally
+// on another layer's cached latents, and with a logistic gate on the concatenated heads.
 struct LatentAttentionSpec {
     int heads = 0, dim = 0, rot_dim = 0, vdim = 0, q_rank = 0, kv_rank = 0;
     double scale = 0.0;
     RotarySpec rot;
+    bool half_split = false;   // rotated pairs (i, i + dims / 2) instead of neighbours
+    bool gate = false;
+    int kv_from = -1;          // the layer whose cache rows this one reads (-1: its own)
 };
 
 // Gated delta rule with one decay per head and key channel; a short causal convolution before it.
@@ -47,13 +52,18 @@ struct ChannelDeltaSpec {
 };
 
 // Grouped-query attention: optional sliding window (0: none), optional sink (added to the sum of
-// exponentials), projections with biases, norms per head before a half-split rotation, values that are
-// the keys as projected.
+// exponentials), query and key projections with or without biases, normed per head, over the whole projection
+// or not at all before the rotation, values of their own or the keys as projected, an optional logistic gate on
+// the concatenated heads.
+enum class QueryKeyNorm { None, PerHead, WholeProjection };
 struct GroupAttentionSpec {
     int heads = 0, kv_heads = 0, dim = 0, vdim = 0, window = 0;
     double scale = 0.0;
     float sink = 0.f;
     RotarySpec rot;
+    bool half_split = true, biases = true, own_values = false, gate = false;
+    QueryKeyNorm norm = QueryKeyNorm::PerHead;
+    int widest() const { return dim > vdim ? dim : vdim; }
 };
 
 // A memory S [dim, vdim] with one decay per head and token.  Retention: constant decays; MatrixLstm:
@@ -68,18 +78,27 @@ struct DecayMemorySpec {
     std::vector<double> decay;     // Retention, one per head
 };
 
-// Attention and a memory side by side on the same input: attention_scale * a + memory_scale * m.
-enum class MixerKind { LatentAttention, ChannelDelta, DecayMemory, Parallel };
+// Parallel: attention and a memory side by side on the same input, attention_scale * a + memory_scale * m.
+enum class MixerKind { LatentAttention, ChannelDelta, DecayMemory, Parallel, Attention };
+
+// A mixture of gated feed-forwards: a softmax router over `experts`, of which a token uses `top`, chosen from
+// the best `keep` of `groups` equal groups of neighbours; the chosen probabilities are divided by their sum and
+// multiplied by `scale`.  Expert: g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(alpha g) (u + shift).
+struct MixtureSpec {
+    int experts = 0, top = 0, ff = 0, groups = 1, keep = 1;
+    float scale = 1.f, limit = 0.f, alpha = 1.f, shift = 0.f;
+};
 
 struct LayerSpec {
     MixerKind mixer = MixerKind::LatentAttention;
     LatentAttentionSpec latent;
     ChannelDeltaSpec delta;
-    GroupAttentionSpec attn;       // Parallel
+    GroupAttentionSpec attn;       // Parallel, Attention
     DecayMemorySpec memory;        // DecayMemory, Parallel
     float attention_scale = 1.f, memory_scale = 1.f;
-    int ff = 0;   // width of the feed-forward (ModelConfig::ff_act between its two matrices); 0: the layer has none
-    bool has_attn() const { return mixer == MixerKind::Parallel; }
+    int ff = 0;   // width of the dense feed-forward (ModelConfig::ff_act); 0: the layer has none
+    MixtureSpec moe;   // experts 0: the layer has none
+    bool has_attn() const { return mixer == MixerKind::Parallel || mixer == MixerKind::Attention; }
     bool has_memory() const { return mixer == MixerKind::Parallel || mixer == MixerKind::DecayMemory; }
 };
 
@@ -93,11 +112,12 @@ struct LayerRun {
     bool begins_pass;   // first layer of a pass of the loop
 };
 
-enum class FeedForwardAct { SquaredRelu, Gelu };
+// (GatedSilu: silu(gate) * up between three matrices with biases)
+enum class FeedForwardAct { SquaredRelu, Gelu, GatedSilu };
 
 struct ModelConfig {
     // architecture: "llama3" (dense, adjacent-pair RoPE) | "qwen3" (dense, qk-norm, half-split
-    // RoPE) | "qwen3_moe" | "varasun", "lofudra" (layer stacks)
+    // RoPE) | "qwen3_moe" | "varasun", "lofudra", "fobanex" (layer stacks)
     std::string arch = "llama3";
     int hidden = 0, layers = 0, q_heads = 0, kv_heads = 0, head_dim = 0, intermediate = 0;
     int vocab = 0;
@@ -137,6 +157,8 @@ struct ModelConfig {
     std::vector<LayerSpec> stack;
     LayerLoop loop;                // stop 0: none
     bool sandwich_norms = false;   // a norm ahead of every sublayer besides the one on its output
+    bool shared_norm = false;      // one norm per layer: mixer and feed-forward read it and join the stream together
+    float embed_scale = 1.f;       // (with shared_norm)
     FeedForwardAct ff_act = FeedForwardAct::SquaredRelu;
     std::vector<LayerRun> layer_runs() const {
         std::vector<LayerRun> runs;
@@ -315,6 +337,15 @@ inline void finalize_stack(DriverConfig& c) {
             if (a.rot.dims < 0 || a.rot.dims % 2 != 0 || a.rot.dims > a.rot_dim)
                 throw std::runtime_error(at + "rot.dims must be even and at most rot_dim");
             if (a.rot.dims > 0 && !(a.rot.base > 0.0)) throw std::runtime_error(at + "rot.base must be positive");
+            if (a.kv_from >= 0) {
+                const LayerSpec* from = a.kv_from < static_cast<int>(i) ? &m.stack[static_cast<size_t>(a.kv_from)] : nullptr;
+                if (!from || from->mixer != MixerKind::LatentAttention || from->latent.kv_from >= 0)
+                    throw std::runtime_error(at + "kv_from must name an earlier latent_attention layer with latents of its own");
+                const auto& b = from->latent;
+                if (b.kv_rank != a.kv_rank || b.rot_dim != a.rot_dim || !(b.rot == a.rot) || b.half_split != a.half_split)
+                    throw std::runtime_error(at + "kv_from: kv_rank, rot_dim and the rotation must be equal");
+                if (m.loop.stop != 0) throw std::runtime_error(at + "kv_from cannot be combined with a loop");
+            }
         } else if (l.mixer == MixerKind::ChannelDelta) {
             const auto& d = l.delta;
             if (d.heads <= 0 || d.kv_heads <= 0 || d.dim <= 0 || d.vdim <= 0 || d.taps <= 0)
@@ -326,11 +357,21 @@ inline void finalize_stack(DriverConfig& c) {
             if (a.heads <= 0 || a.kv_heads <= 0 || a.dim <= 0 || a.window < 0)
                 throw std::runtime_error(at + "attention needs heads, kv_heads, dim and a window that is not negative");
             if (a.heads % a.kv_heads != 0) throw std::runtime_error(at + "heads must be a multiple of kv_heads");
-            if (a.vdim != a.dim) throw std::runtime_error(at + "values that are the keys have the keys' size");
-            if (a.dim > 1024) throw std::runtime_error(at + "attention heads are limited to 1024 values");
+            if (a.vdim <= 0) throw std::runtime_error(at + "attention needs a positive vdim");
+            if (!a.own_values && a.vdim != a.dim) throw std::runtime_error(at + "values that are the keys have the keys' size");
+            if (a.widest() > 1024) throw std::runtime_error(at + "attention heads are limited to 1024 values");
             if (a.rot.dims < 0 || a.rot.dims % 2 != 0 || a.rot.dims > a.dim)
                 throw std::runtime_error(at + "rot.dims must be even and at most dim");
             if (a.rot.dims > 0 && !(a.rot.base > 0.0)) throw std::runtime_error(at + "rot.base must be positive");
+        }
+        if (l.moe.experts != 0) {
+            const auto& e = l.moe;
+            if (!m.shared_norm) throw std::runtime_error(at + "a mixture needs an architecture whose sublayers share a norm");
+            if (e.experts <= 0 || e.ff <= 0 || e.top <= 0 || e.groups <= 0 || e.keep <= 0 || e.keep > e.groups || e.experts % e.groups != 0)
+                throw std::runtime_error(at + "a mixture needs experts in equal groups, a positive width, top and kept groups");
+            if (e.top > e.keep * (e.experts / e.groups)) throw std::runtime_error(at + "fewer experts in the kept groups than a token uses");
+            if (e.experts > 512 || e.top > 64) throw std::runtime_error(at + "mixtures are limited to 512 experts, 64 per token");
+            if (!(e.limit >= 0.f)) throw std::runtime_error(at + "expert.limit must not be negative");
         }
         if (l.has_memory()) {
             const auto& d = l.memory;

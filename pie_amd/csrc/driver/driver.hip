@@ -864,24 +864,32 @@ extern "C" long long pie_hip_driver_snapshot_info(const char* dir, char* out, si
           << ",\"rope_factor\":" << m.rope_factor << ",\"tie_embeddings\":" << (m.tie_embeddings ? "true" : "false")
           << ",\"num_experts\":" << m.num_experts << ",\"top_k\":" << m.top_k
           << ",\"expert_intermediate\":" << m.expert_intermediate << ",\"logit_scale\":" << m.logit_scale
-          << ",\"logit_softcap\":" << m.logit_softcap << ",\"loop\":[" << m.loop.start << "," << m.loop.stop << ","
+          << ",\"logit_softcap\":" << m.logit_softcap << ",\"embed_scale\":" << m.embed_scale << ",\"loop\":[" << m.loop.start << "," << m.loop.stop << ","
           << m.loop.times << "],\"stack\":[";
         for (size_t i = 0; i < m.stack.size(); ++i) {
             const LayerSpec& l = m.stack[i];
             j << (i ? ",{" : "{") << "\"ff\":" << l.ff;
+            if (l.moe.experts)
+                j << ",\"mixture\":{\"experts\":" << l.moe.experts << ",\"top\":" << l.moe.top << ",\"ff\":" << l.moe.ff << ",\"groups\":"
+                  << l.moe.groups << ",\"keep\":" << l.moe.keep << ",\"scale\":" << l.moe.scale << ",\"limit\":" << l.moe.limit << "}";
             if (l.mixer == MixerKind::LatentAttention)
                 j << ",\"type\":\"latent_attention\",\"heads\":" << l.latent.heads << ",\"dim\":" << l.latent.dim
                   << ",\"rot_dim\":" << l.latent.rot_dim << ",\"vdim\":" << l.latent.vdim << ",\"q_rank\":" << l.latent.q_rank
                   << ",\"kv_rank\":" << l.latent.kv_rank << ",\"scale\":" << l.latent.scale << ",\"rot_dims\":" << l.latent.rot.dims
-                  << ",\"rot_base\":" << l.latent.rot.base << ",\"yarn\":" << (l.latent.rot.yarn ? "true" : "false");
+                  << ",\"rot_base\":" << l.latent.rot.base << ",\"yarn\":" << (l.latent.rot.yarn ? "true" : "false")
+                  << ",\"half_split\":" << (l.latent.half_split ? "true" : "false") << ",\"gate\":" << (l.latent.gate ? "true" : "false")
+                  << ",\"kv_from\":" << l.latent.kv_from;
             else if (l.mixer == MixerKind::ChannelDelta)
                 j << ",\"type\":\"channel_delta\",\"heads\":" << l.delta.heads << ",\"kv_heads\":" << l.delta.kv_heads
                   << ",\"dim\":" << l.delta.dim << ",\"vdim\":" << l.delta.vdim << ",\"conv\":" << l.delta.taps;
             if (l.has_attn())
                 j << ",\"attention\":{\"heads\":" << l.attn.heads << ",\"kv_heads\":" << l.attn.kv_heads << ",\"dim\":" << l.attn.dim
                   << ",\"vdim\":" << l.attn.vdim << ",\"window\":" << l.attn.window << ",\"scale\":" << l.attn.scale << ",\"sink\":" << l.attn.sink
-                  << ",\"rot_dims\":" << l.attn.rot.dims << ",\"rot_base\":" << l.attn.rot.base << "},\"attention_scale\":"
-                  << l.attention_scale << ",\"memory_scale\":" << l.memory_scale;
+                  << ",\"rot_dims\":" << l.attn.rot.dims << ",\"rot_base\":" << l.attn.rot.base << ",\"half_split\":"
+                  << (l.attn.half_split ? "true" : "false") << ",\"biases\":" << (l.attn.biases ? "true" : "false") << ",\"own_values\":"
+                  << (l.attn.own_values ? "true" : "false") << ",\"gate\":" << (l.attn.gate ? "true" : "false") << ",\"norm\":"
+                  << static_cast<int>(l.attn.norm) << "},\"attention_scale\":" << l.attention_scale << ",\"memory_scale\":" << l.memory_scale;
+            if (l.mixer == MixerKind::Attention) j << ",\"type\":\"attention\"";
             if (l.has_memory()) {
                 const DecayMemorySpec& d = l.memory;
                 static const char* kinds[] = {"retention", "mlstm", "mamba2"};

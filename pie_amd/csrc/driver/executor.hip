@@ -134,7 +134,7 @@ bool routes_to_gemv(const Linear& w, int M, bool has_norm, size_t ws_bytes) {
 
 bool linear_fused(const Linear& w, const uint16_t* act, const uint16_t* norm_w, float eps,
                   uint16_t* y, int M, int beta, int swiglu, uint16_t* norm_tmp, void* gemm_ws,
-                  size_t gemm_ws_bytes, hipStream_t s, int force) {
+                  size_t gemm_ws_bytes, hipStream_t s, int force, const PieHipGlu* glu) {
     const int fmt = fmt_code(w.kind);
     const int sbf = w.scale_bf16 ? 1 : 0;
     const int forced_rows = forced_gemv_rows();
@@ -149,8 +149,8 @@ bool linear_fused(const Linear& w, const uint16_t* act, const uint16_t* norm_w, 
         gemv = tuned == 0;
     }
     if (gemv) {
-        const int st = pie_hip_linear_fused(fmt, act, norm_w, eps, w.data, w.scale, sbf, w.group, y, M, w.N, w.K,
-                                            beta, swiglu, s);
+        const int st = pie_hip_linear_fused_glu(fmt, act, norm_w, eps, w.data, w.scale, sbf, w.group, y, M, w.N, w.K,
+                                                beta, swiglu, glu, s);
         if (st == PIE_HIP_OK) return true;
         if (st != PIE_HIP_ERR_UNSUPPORTED) PIE_KERNEL(st);
         if (force >= 0) return false;
@@ -169,25 +169,21 @@ bool linear_fused(const Linear& w, const uint16_t* act, const uint16_t* norm_w, 
         if (path != GemmPath::Skinny) {
             // the tiled GEMM (weights dequantised to bf16 while staged), in K shares for a
             // decode batch whose output has few tiles
-            const int sg = path == GemmPath::TiledSplitK
-                               ? pie_hip_gemm_mfma_splitk(fmt, a, w.data, w.scale, sbf, w.group, y, M, w.N,
-                                                          w.K, beta, swiglu, gemm_ws, gemm_ws_bytes, s)
-                               : pie_hip_gemm_mfma(fmt, a, w.data, w.scale, sbf, w.group, y, M, w.N, w.K,
-                                                   beta, swiglu, s);
+            const bool split = path == GemmPath::TiledSplitK;
+            const int sg = pie_hip_gemm_mfma_glu(fmt, a, w.data, w.scale, sbf, w.group, y, M, w.N, w.K, beta, swiglu, glu,
+                                                 split ? gemm_ws : nullptr, split ? gemm_ws_bytes : 0, s);
             if (sg == PIE_HIP_OK) return true;
             if (sg != PIE_HIP_ERR_UNSUPPORTED) PIE_KERNEL(sg);
             if (force >= 0) return false;
         }
-        const int st = w.data_tiled
-                           ? pie_hip_gemm_skinny_tiled(fmt, a, w.data_tiled, w.scale_tiled ? w.scale_tiled : w.scale,
-                                                       sbf, w.group, y, M, w.N, w.K, beta, swiglu, s)
-                           : pie_hip_gemm_skinny(fmt, a, w.data, w.scale, sbf, w.group, y, M, w.N, w.K, beta,
-                                                 swiglu, s);
+        const int st = pie_hip_gemm_skinny_glu(fmt, a, w.data_tiled ? w.data_tiled : w.data,
+                                               w.data_tiled && w.scale_tiled ? w.scale_tiled : w.scale, sbf, w.group, y, M,
+                                               w.N, w.K, beta, swiglu, w.data_tiled ? 1 : 0, glu, s);
         if (st == PIE_HIP_OK) return true;
         if (st != PIE_HIP_ERR_UNSUPPORTED) PIE_KERNEL(st);
         if (force >= 0) return false;
-        PIE_KERNEL(pie_hip_linear_fused(fmt, a, nullptr, eps, w.data, w.scale, sbf, w.group, y, M,
-                                        w.N, w.K, beta, swiglu, s));
+        PIE_KERNEL(pie_hip_linear_fused_glu(fmt, a, nullptr, eps, w.data, w.scale, sbf, w.group, y, M,
+                                            w.N, w.K, beta, swiglu, glu, s));
     }
     return true;
 }
@@ -494,9 +490,13 @@ bool Executor::alloc_pools() {
     if (m.is_stack()) {
         for (const LayerRun& run : m.layer_runs()) {   // every pass of a looped layer has its own
             const LayerSpec& l = m.stack[static_cast<size_t>(run.layer)];
+            if (l.mixer == MixerKind::LatentAttention && l.latent.kv_from >= 0) {   // (without loops layers are runs)
+                run_pool_.push_back(run_pool_[static_cast<size_t>(l.latent.kv_from)]);
+                continue;
+            }
             run_pool_.push_back(nullptr);
             const int row = l.mixer == MixerKind::LatentAttention ? LatentShape(l.latent).ld_row
-                            : l.has_attn()                        ? l.attn.kv_heads * 2 * pad_head(l.attn.dim)
+                            : l.has_attn()                        ? l.attn.kv_heads * 2 * pad_head(l.attn.widest())
                                                                   : 0;
             if (row == 0) continue;
             const size_t esize = m.f32() ? 4 : 2;

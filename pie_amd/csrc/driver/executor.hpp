@@ -21,7 +21,11 @@
 //                     recurrence over the request's state slot, norm + gate, out-projection
 //   decay memory      in-projection, fp32 gate columns, (convolution,) the recurrence over the request's
 //                     state slot, norm + gate, out-projection
+//   attention         in-projection, norms + rotation + cache write, grouped attention, out-projection
 //   parallel          one in-projection, grouped attention and a decay memory on it, one out-projection
+// A mixture of experts: fp32 router logits, the choice of experts and the sorted layout, two grouped products.
+// Architectures whose sublayers share a norm join both outputs (a mixture's routes weighted on the way) and norm
+// the stream for the next layer in one kernel; latent layers may read another layer's cache rows.
 // Architectures with norms ahead of their sublayers have the stream normed by the kernel that last
 // changed it; looped layers run several times, each pass with its own cache and state.
 //
@@ -63,7 +67,7 @@ struct SampleOutputs {
 // y = epilogue(rmsnorm?(act) . W^T) through the bf16 / quantised kernels (executor.hip).
 bool linear_fused(const Linear& w, const uint16_t* act, const uint16_t* norm_w, float eps,
                   uint16_t* y, int M, int beta, int epilogue, uint16_t* norm_tmp, void* gemm_ws,
-                  size_t gemm_ws_bytes, hipStream_t s, int force = -1);
+                  size_t gemm_ws_bytes, hipStream_t s, int force = -1, const PieHipGlu* glu = nullptr);
 
 class Executor {
   public:
@@ -155,7 +159,11 @@ class Executor {
     void stack_attention(const StackLayer& w, int run, int N, int max_kv_len, const Inputs& in);
     void stack_memory(const StackLayer& w, int run, int N, const Inputs& in);
     PieHipStateRows state_rows(int run, int N, const Inputs& in) const;
-    void stack_linear(const Linear& w, const void* act, void* y, int M, int epilogue = PIE_HIP_EPI_NONE);
+    void stack_mixture(const StackLayer& w, int N);
+    void stack_shared_norm(int N, int max_kv_len, const Inputs& in);
+    void stack_mixer(const StackLayer& w, int run, int N, int max_kv_len, const Inputs& in);
+    void stack_linear(const Linear& w, const void* act, void* y, int M, int epilogue = PIE_HIP_EPI_NONE,
+                      const PieHipGlu* glu = nullptr);
     void tune_linears();
 
     DriverConfig cfg_;
@@ -265,6 +273,9 @@ class Executor {
              *xs = nullptr, *raw_logits = nullptr;
         float *dq = nullptr, *dk = nullptr, *dv = nullptr, *dg = nullptr, *d_beta = nullptr, *d_o = nullptr;
         void* conv = nullptr;                                      // compute type: after a memory's convolution
+        void *y2 = nullptr, *routes = nullptr;                     // compute type: a feed-forward's rows, a mixture's routes' rows
+        float *router = nullptr, *route_w = nullptr, *glu = nullptr;   // router logits, weights, fp32 pairs ahead of the gated rule
+        int32_t *route_idx = nullptr, *route_offsets = nullptr, *route_token = nullptr, *route_pos = nullptr;
         float *gates = nullptr, *mem_o = nullptr, *den = nullptr;  // decay memories: gate columns, read-outs, divisors
         std::vector<float*> rotary;              // tables of the step, one per distinct rotation
         std::vector<void*> allocs;

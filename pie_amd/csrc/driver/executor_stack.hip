@@ -35,6 +35,7 @@ void Executor::alloc_stack() {
     size_t in = 0, cq = 0, q = 0, q_lat = 0, o_lat = 0, o = 0, act = 0, gate = 0;
     size_t kd = 0, vd = 0, gd = 0, heads = 0, state = 0;
     size_t conv = 0, gates = 0, mem_o = 0, den = 0, head_pad = 0;
+    size_t y2 = 0, top = 0, router = 0, experts = 0, glu = 0;
     auto up = [](size_t& v, int n) { v = std::max(v, static_cast<size_t>(n)); };
     auto place = [&](size_t bytes) {
         const size_t at = state;
@@ -46,6 +47,18 @@ void Executor::alloc_stack() {
         rs_state_off_.push_back(0);
         rs_conv_off_.push_back(0);
         up(act, l.spec.ff > 0 ? pad_to(l.spec.ff, 128) : 0);
+        if (m.shared_norm && l.spec.ff > 0) {
+            up(y2, model_.ld_x());
+            up(glu, 2 * pad_to(l.spec.ff, 128));
+        }
+        if (l.spec.moe.experts > 0) {
+            const int width = l.spec.moe.top * pad_to(l.spec.moe.ff, 128);
+            up(act, width);
+            up(glu, 2 * width);
+            up(top, l.spec.moe.top);
+            up(router, pad_to(l.spec.moe.experts, 16));
+            up(experts, l.spec.moe.experts);
+        }
         if (l.spec.mixer == MixerKind::LatentAttention) {
             const LatentShape s(l.spec.latent);
             up(in, s.ld_in);
@@ -107,6 +120,18 @@ void Executor::alloc_stack() {
     stack_.o = compute(T * o);
     stack_.act = compute(T * act);
     stack_.gate = compute(T * gate);
+    stack_.y2 = compute(T * y2);
+    if (top) {
+        stack_.routes = compute(T * top * ld_x);
+        stack_.router = f32(T * router);
+        stack_.route_w = f32(T * top);
+        auto i32 = [&](size_t n) { return static_cast<int32_t*>(take(n * 4)); };
+        stack_.route_idx = i32(T * top);
+        stack_.route_offsets = i32(experts + 1);
+        stack_.route_token = i32(T * top);
+        stack_.route_pos = i32(T * top);
+    }
+    if (m.f32()) stack_.glu = f32(T * glu);
     stack_.dq = f32(T * kd);
     stack_.dk = f32(T * kd);
     stack_.dv = f32(T * vd);
@@ -123,7 +148,7 @@ void Executor::alloc_stack() {
     stack_.logits = f32(srows * static_cast<size_t>(m.vocab));
     for (const RotaryTable& r : model_.rotary) stack_.rotary.push_back(f32(T * static_cast<size_t>(r.spec.dims)));
     for (StackLayer& l : model_.stack)
-        for (const Linear* w : {&l.w_in, &l.w_uq, &l.wo, &l.w_up, &l.w_down})
+        for (const Linear* w : {&l.w_in, &l.w_uq, &l.wo, l.spec.moe.experts ? &l.wo : &l.w_up, l.spec.moe.experts ? &l.wo : &l.w_down})
             for (int rows : {64, 128})
                 if (!m.f32() && w->data && w->K % 64 == 0)
                     gemm_ws_bytes_ = std::max(gemm_ws_bytes_, pie_hip_gemm_mfma_workspace_bytes(rows, w->N, w->K));
@@ -257,9 +282,9 @@ void Executor::prepare_lists(const BatchPlan& plan) {
     for (const StackLayer& l : model_.stack) {
         delta |= l.spec.mixer == MixerKind::ChannelDelta;
         memory |= l.spec.has_memory();
-        if (!l.spec.has_attn() || dt_ != PIE_HIP_DT_BF16) continue;
+        if (!l.spec.has_attn() || dt_ != PIE_HIP_DT_BF16 || !pie_hip_group_attn_supported(pad_head(l.spec.attn.widest()))) continue;
         const GroupAttentionSpec& a = l.spec.attn;
-        const auto key = std::make_tuple(a.heads, a.kv_heads, pad_head(a.dim));
+        const auto key = std::make_tuple(a.heads, a.kv_heads, pad_head(a.widest()));
         if (tile_lists_.count(key)) continue;
         TileList t;
         std::vector<std::pair<int, int>> tiles;   // (first row, rows)
@@ -306,13 +331,45 @@ void Executor::commit_stack(const BatchPlan& plan) {
     for (int r = 0; r < plan.R; ++r) rs_pos_[plan.rs_slots[r]] = plan.positions[plan.qo_indptr[r + 1] - 1] + 1;
 }
 
-void Executor::stack_linear(const Linear& w, const void* act, void* y, int M, int epilogue) {
-    if (dt_ == PIE_HIP_DT_F32)
+void Executor::stack_linear(const Linear& w, const void* act, void* y, int M, int epilogue, const PieHipGlu* glu) {
+    if (dt_ == PIE_HIP_DT_F32 && epilogue == PIE_HIP_EPI_SWIGLU) {
+        PIE_KERNEL(pie_hip_linear_f32(static_cast<const float*>(act), static_cast<const uint16_t*>(w.data), stack_.glu, M, w.N, w.K,
+                                      PIE_HIP_EPI_NONE, stream_));
+        PIE_KERNEL(pie_hip_glu_f32(stack_.glu, glu, static_cast<float*>(y), M, w.N / 2, stream_));
+    } else if (dt_ == PIE_HIP_DT_F32)
         PIE_KERNEL(pie_hip_linear_f32(static_cast<const float*>(act), static_cast<const uint16_t*>(w.data),
                                       static_cast<float*>(y), M, w.N, w.K, epilogue, stream_));
     else
         linear_fused(w, static_cast<const uint16_t*>(act), nullptr, 0.f, static_cast<uint16_t*>(y), M, 0, epilogue,
-                     nullptr, gemm_ws_, gemm_ws_bytes_, stream_);
+                     nullptr, gemm_ws_, gemm_ws_bytes_, stream_, -1, glu);
+}
+
+// Each token's row through its experts: routes' rows in stack_.routes, their places and weights beside them.
+void Executor::stack_mixture(const StackLayer& w, int N) {
+    const MixtureSpec& e = w.spec.moe;
+    const int Hp = model_.ld_x(), ffp = w.w_down.K, ld = pad_to(e.experts, 16);
+    PIE_KERNEL(pie_hip_linear_f32out(dt_, stack_.xa, w.w_router, stack_.router, N, ld, Hp, stream_));
+    PIE_KERNEL(pie_hip_moe_route_groups(stack_.router, ld, stack_.route_idx, stack_.route_w, stack_.route_offsets, stack_.route_token,
+                                        stack_.route_pos, N, e.experts, e.top, e.groups, e.keep, e.scale, stream_));
+    const PieHipGlu glu{nullptr, e.limit, e.alpha, e.shift};
+    if (dt_ == PIE_HIP_DT_F32) {
+        PIE_KERNEL(pie_hip_moe_grouped_linear_f32(static_cast<const float*>(stack_.xa), stack_.route_token, stack_.route_offsets, e.experts, N,
+                                                  static_cast<const uint16_t*>(w.w_up.data), stack_.glu, 2 * ffp, Hp, stream_));
+        PIE_KERNEL(pie_hip_glu_f32(stack_.glu, &glu, static_cast<float*>(stack_.act), N * e.top, ffp, stream_));
+        PIE_KERNEL(pie_hip_moe_grouped_linear_f32(static_cast<const float*>(stack_.act), nullptr, stack_.route_offsets, e.experts, N,
+                                                  static_cast<const uint16_t*>(w.w_down.data), static_cast<float*>(stack_.routes), Hp, ffp,
+                                                  stream_));
+        return;
+    }
+    const int hint = std::max(1, std::min(N, 2 * ((N * e.top + e.experts - 1) / e.experts)));
+    auto grouped = [&](const Linear& l, const void* act, const int32_t* rows, void* y, int epilogue, const PieHipGlu* rule) {
+        PIE_KERNEL(pie_hip_moe_grouped_gemm_glu(PIE_HIP_FMT_BF16, static_cast<const uint16_t*>(act), rows, stack_.route_offsets, e.experts,
+                                                hint, l.data_tiled ? l.data_tiled : l.data, l.data_bytes() / e.experts, nullptr, 0, 0, 0,
+                                                static_cast<uint16_t*>(y), l.N / e.experts, l.K, epilogue, l.data_tiled ? 1 : 0, rule,
+                                                stream_));
+    };
+    grouped(w.w_up, stack_.xa, stack_.route_token, stack_.act, PIE_HIP_EPI_SWIGLU, &glu);
+    grouped(w.w_down, stack_.act, nullptr, stack_.routes, PIE_HIP_EPI_NONE, nullptr);
 }
 
 void Executor::stack_latent(const StackLayer& w, int layer, int N, int max_kv_len, const Inputs& in) {
@@ -324,20 +381,21 @@ void Executor::stack_latent(const StackLayer& w, int layer, int N, int max_kv_le
     const auto* pages = reinterpret_cast<const uint32_t*>(in_dev_ + in.off_pages);
     const float* rope = w.rotary >= 0 ? stack_.rotary[static_cast<size_t>(w.rotary)] : nullptr;
     stack_linear(w.w_in, stack_.xa, stack_.in, N);
+    const size_t esize = dt_ == PIE_HIP_DT_F32 ? 4 : 2;
+    auto rows_of = [&](void* buf, int row, int ld) { return static_cast<unsigned char*>(buf) + static_cast<size_t>(row) * ld * esize; };
+    auto gate_of = [&](int row) { return a.gate ? rows_of(stack_.in, row, s.ld_in) + static_cast<size_t>(s.gate_off) * esize : nullptr; };
     PIE_KERNEL(pie_hip_latent_prep(dt_, stack_.in, w.q_norm, w.kv_norm, rope, slots, stack_.cq, run_pool_[layer], N,
                                    s.ld_in, s.kv_off, a.q_rank, s.ld_cq, a.kv_rank, s.kvp, a.rot_dim, a.rot.dims,
                                    s.ld_row, model_.cfg().rms_eps, stream_));
     stack_linear(w.w_uq, stack_.cq, stack_.q, N);
 
-    const size_t esize = dt_ == PIE_HIP_DT_F32 ? 4 : 2;
-    auto rows_of = [&](void* buf, int row, int ld) { return static_cast<unsigned char*>(buf) + static_cast<size_t>(row) * ld * esize; };
     const bool matrix = dt_ == PIE_HIP_DT_BF16 && pie_hip_latent_attn_rows_supported(s.kvp, s.rotp);
     // rows [r0, r0 + n): through the latent space
     auto rows_form = [&](int r0, int n, int max_len, int max_tokens) {
         if (n <= 0) return;
         PIE_KERNEL(pie_hip_head_linear(dt_, rows_of(stack_.q, r0, s.ld_q), w.w_uk_t, rows_of(stack_.q_lat, r0, s.heads * s.ld_row),
                                        rope ? rope + static_cast<size_t>(r0) * a.rot.dims : nullptr, n, s.heads, s.kvp, s.dimp,
-                                       s.ld_q, s.hd, s.heads * s.ld_row, s.ld_row, s.dimp, a.rot_dim, a.rot.dims, s.rotp, stream_));
+                                       s.ld_q, s.hd, s.heads * s.ld_row, s.ld_row, s.dimp, a.rot_dim, a.rot.dims, s.rotp, nullptr, 0, stream_));
         if (matrix)
             PIE_KERNEL(pie_hip_latent_attn_rows(static_cast<const uint16_t*>(stack_.q_lat),
                                                 reinterpret_cast<const uint16_t*>(run_pool_[layer]),
@@ -351,7 +409,7 @@ void Executor::stack_latent(const StackLayer& w, int layer, int N, int max_kv_le
                                                       rows_of(stack_.o_lat, r0, s.heads * s.kvp), pages, row_begin + r0, row_len + r0, n,
                                                       s.heads, s.kvp, s.ld_row, page_size_, static_cast<float>(a.scale), stream_));
         PIE_KERNEL(pie_hip_head_linear(dt_, rows_of(stack_.o_lat, r0, s.heads * s.kvp), w.w_uv, rows_of(stack_.o, r0, s.ld_o), nullptr, n,
-                                       s.heads, s.vdp, s.kvp, s.heads * s.kvp, s.kvp, s.ld_o, s.vdp, 0, 0, 0, 0, stream_));
+                                       s.heads, s.vdp, s.kvp, s.heads * s.kvp, s.kvp, s.ld_o, s.vdp, 0, 0, 0, 0, gate_of(r0), s.ld_in, stream_));
     };
     if (plan_->pure_decode) {
         rows_form(0, N, max_kv_len, 1);
@@ -387,7 +445,8 @@ void Executor::stack_latent(const StackLayer& w, int layer, int N, int max_kv_le
                                          PIE_HIP_EPI_NONE, stream_));
             PIE_KERNEL(pie_hip_latent_attn_prefill(static_cast<const uint16_t*>(stack_.q), kv, rot, static_cast<uint16_t*>(stack_.o),
                                                    rope, row_len, q0, q1 - q0, ctx, s.heads, s.dimp, s.rotp, a.rot.dims, s.vdp,
-                                                   s.ld_o, static_cast<float>(a.scale), stream_));
+                                                   s.ld_o, static_cast<float>(a.scale), reinterpret_cast<const uint16_t*>(gate_of(0)),
+                                                   s.ld_in, stream_));
         }
         rows_form(run0, N - run0, run_len, run_tokens);
     }
@@ -474,26 +533,35 @@ void Executor::stack_attention(const StackLayer& w, int run, int N, int max_kv_l
     const float* rope = w.rotary >= 0 ? stack_.rotary[static_cast<size_t>(w.rotary)] : nullptr;
     const float scale = static_cast<float>(a.scale), out_scale = w.spec.attention_scale;
     unsigned char* pool = run_pool_[static_cast<size_t>(run)];
-    PIE_KERNEL(pie_hip_group_attn_prep(dt_, stack_.in, s.q_off, s.k_off, -1, w.q_bias, w.k_bias, w.q_norm, w.k_norm, rope, a.rot.dims,
-                                       reinterpret_cast<const int64_t*>(in_dev_ + in.off_slots), stack_.q, pool, N, s.ld_in, a.heads,
-                                       a.kv_heads, a.dim, s.dimp, model_.cfg().rms_eps, stream_));
+    const size_t esize = dt_ == PIE_HIP_DT_F32 ? 4 : 2;
+    const void* gate = a.gate ? static_cast<unsigned char*>(stack_.in) + static_cast<size_t>(s.attn_gate_off) * esize : nullptr;
+    const auto* slots = reinterpret_cast<const int64_t*>(in_dev_ + in.off_slots);
+    // (the kernel for norms per head rotates half-split vectors and knows biases)
+    if (a.norm == QueryKeyNorm::PerHead || a.biases)
+        PIE_KERNEL(pie_hip_group_attn_prep(dt_, stack_.in, s.q_off, s.k_off, s.v_off, w.q_bias, w.k_bias, w.q_norm, w.k_norm, rope, a.rot.dims,
+                                           slots, stack_.q, pool, N, s.ld_in, a.heads, a.kv_heads, a.dim, s.dimp, model_.cfg().rms_eps, stream_));
+    else
+        PIE_KERNEL(pie_hip_group_attn_prep_joint(dt_, stack_.in, s.q_off, s.k_off, s.v_off, w.q_norm, w.k_norm, rope, a.rot.dims,
+                                                 a.half_split ? PIE_HIP_ROPE_HALF : PIE_HIP_ROPE_ADJACENT, slots, stack_.q, pool, N, s.ld_in,
+                                                 a.heads, a.kv_heads, a.dim, a.vdim, s.dimp, model_.cfg().rms_eps, stream_));
     if (dt_ != PIE_HIP_DT_BF16 || !pie_hip_group_attn_supported(s.dimp)) {
         PIE_KERNEL(pie_hip_group_attn_plain(dt_, stack_.q, pool, stack_.o, pages, row_begin, row_len, N, a.heads, a.kv_heads, s.dimp, s.ld_o,
-                                            page_size_, scale, a.window, a.sink, out_scale, stream_));
+                                            page_size_, scale, a.window, a.sink, out_scale, gate, s.ld_in, stream_));
         return;
     }
     const auto* q = static_cast<const uint16_t*>(stack_.q);
     const auto* kv = reinterpret_cast<const uint16_t*>(pool);
     auto* o = static_cast<uint16_t*>(stack_.o);
+    const auto* g = static_cast<const uint16_t*>(gate);
     auto rows_form = [&](const int32_t* rows, int n) {
         PIE_KERNEL(pie_hip_group_attn_rows(q, kv, o, pages, row_begin, row_len, rows, n, a.heads, a.kv_heads, s.dimp, s.ld_o, page_size_,
-                                           scale, a.window, a.sink, out_scale, max_kv_len, attn_ws_, attn_ws_bytes_, stream_));
+                                           scale, a.window, a.sink, out_scale, g, s.ld_in, max_kv_len, attn_ws_, attn_ws_bytes_, stream_));
     };
     if (plan_->pure_decode) return rows_form(nullptr, N);
     const TileList& t = tile_lists_.at(std::make_tuple(a.heads, a.kv_heads, s.dimp));
     if (t.n)
         PIE_KERNEL(pie_hip_group_attn_tiles(q, kv, o, pages, row_begin, row_len, list_at(t.tiles), t.n, t.half, a.heads, a.kv_heads, s.dimp,
-                                            s.ld_o, page_size_, scale, a.window, a.sink, out_scale, stream_));
+                                            s.ld_o, page_size_, scale, a.window, a.sink, out_scale, g, s.ld_in, stream_));
     if (n_single_) rows_form(list_at(single_rows_), n_single_);
 }
 
@@ -571,6 +639,43 @@ void Executor::stack_memory(const StackLayer& w, int run, int N, const Inputs& i
     else out();
 }
 
+void Executor::stack_mixer(const StackLayer& w, int run, int N, int max_kv_len, const Inputs& in) {
+    switch (w.spec.mixer) {
+        case MixerKind::LatentAttention: stack_latent(w, run, N, max_kv_len, in); break;
+        case MixerKind::ChannelDelta: stack_delta(w, run, N, in); break;
+        default: stack_mix(w, run, N, max_kv_len, in); break;
+    }
+}
+
+// Layers whose mixer and feed-forward read one norm: both outputs join the stream in one kernel, which norms it
+// for the next layer.
+void Executor::stack_shared_norm(int N, int max_kv_len, const Inputs& in) {
+    const ModelConfig& m = model_.cfg();
+    const int ld = model_.ld_x();
+    const size_t n_runs = model_.runs.size();
+    auto layer_of = [&](size_t run) -> const StackLayer& { return model_.stack[static_cast<size_t>(model_.runs[run].layer)]; };
+    PIE_KERNEL(pie_hip_residual_join(dt_, nullptr, 0, nullptr, 0, nullptr, nullptr, stack_.x, 0,
+                                     reinterpret_cast<const uint32_t*>(in_dev_ + in.off_tokens), model_.embed, m.vocab, m.embed_scale,
+                                     layer_of(0).pre1, stack_.xa, N, m.hidden, ld, m.rms_eps, stream_));
+    for (size_t r = 0; r < n_runs; ++r) {
+        const StackLayer& w = layer_of(r);
+        stack_mixer(w, static_cast<int>(r), N, max_kv_len, in);
+        const bool dense = w.spec.ff > 0, mixture = w.spec.moe.experts > 0;
+        if (dense && w.up_bias) {
+            const PieHipGlu glu{w.up_bias, INFINITY, 1.f, 0.f};
+            stack_linear(w.w_up, stack_.xa, stack_.act, N, PIE_HIP_EPI_SWIGLU, &glu);
+        } else if (dense) {
+            stack_linear(w.w_up, stack_.xa, stack_.act, N, m.ff_act == FeedForwardAct::Gelu ? PIE_HIP_EPI_GELU : PIE_HIP_EPI_RELU2);
+        }
+        if (dense) stack_linear(w.w_down, stack_.act, stack_.y2, N);
+        if (mixture) stack_mixture(w, N);
+        const PieHipRoutes routes{stack_.routes, stack_.route_pos, stack_.route_w, w.spec.moe.top, ld};
+        PIE_KERNEL(pie_hip_residual_join(dt_, stack_.y, w.wo.N, dense ? stack_.y2 : nullptr, w.w_down.N, w.down_bias,
+                                         mixture ? &routes : nullptr, stack_.x, 1, nullptr, nullptr, 0, 0.f,
+                                         r + 1 < n_runs ? layer_of(r + 1).pre1 : nullptr, stack_.xa, N, m.hidden, ld, m.rms_eps, stream_));
+    }
+}
+
 void Executor::stack_body(int N, int S, int max_kv_len) {
     const Inputs in = input_layout(N, S);
     const ModelConfig& m = model_.cfg();
@@ -591,21 +696,18 @@ void Executor::stack_body(int N, int S, int max_kv_len) {
                                          begins ? model_.loop_step + static_cast<size_t>(pass) * H : nullptr,
                                          more ? layer_of(run).pre1 : nullptr, stack_.xa, N, H, ldy, ld, m.rms_eps, s));
     };
-    if (m.sandwich_norms) enter(0, nullptr, nullptr, 0, false);
+    if (m.shared_norm) {
+    } else if (m.sandwich_norms) enter(0, nullptr, nullptr, 0, false);
     else PIE_KERNEL(pie_hip_embed_stream(dt_, tokens, model_.embed, stack_.x, stack_.xa, N, H, ld, m.vocab, s));
     for (size_t i = 0; i < model_.rotary.size(); ++i)
         PIE_KERNEL(pie_hip_rotary_table(reinterpret_cast<const int32_t*>(in_dev_ + in.off_positions),
                                         model_.rotary[i].freq, stack_.rotary[i], N, model_.rotary[i].spec.dims,
                                         model_.rotary[i].mscale, s));
     const int act = m.ff_act == FeedForwardAct::Gelu ? PIE_HIP_EPI_GELU : PIE_HIP_EPI_RELU2;
-    for (size_t r = 0; r < n_runs; ++r) {
+    if (m.shared_norm) stack_shared_norm(N, max_kv_len, in);
+    for (size_t r = 0; r < n_runs && !m.shared_norm; ++r) {
         const StackLayer& w = layer_of(r);
-        const int run = static_cast<int>(r);
-        switch (w.spec.mixer) {
-            case MixerKind::LatentAttention: stack_latent(w, run, N, max_kv_len, in); break;
-            case MixerKind::ChannelDelta: stack_delta(w, run, N, in); break;
-            default: stack_mix(w, run, N, max_kv_len, in); break;
-        }
+        stack_mixer(w, static_cast<int>(r), N, max_kv_len, in);
         // y joins the stream; `last`: the layer's last sublayer
         auto finish = [&](const float* post, int ldy, bool last) {
             if (!m.sandwich_norms)

@@ -75,13 +75,15 @@ constexpr int pad_latent(int v) {
 }
 struct LatentShape {
     int heads, dimp, rotp, vdp, kvp;   // per-head sizes and the latent, rounded up
-    int kv_off, ld_in;                 // fused down projection: query latent | (kv_off) latent, rotated key part
+    int kv_off, gate_off, ld_in;       // fused projection: query latent | latent, rotated key part | gates (heads of vdp)
     int ld_cq, hd, ld_q;               // query latent rows; q rows: heads of [dimp | rotp]
     int ld_row;                        // cache row: [kvp | rotp]
     int ld_o;                          // attention output rows: heads of vdp
     explicit LatentShape(const LatentAttentionSpec& a)
         : heads(a.heads), dimp(pad_to(a.dim, 32)), rotp(a.rot_dim > 0 ? pad_to(a.rot_dim, 32) : 32), vdp(pad_to(a.vdim, 32)),
-          kvp(pad_latent(a.kv_rank)), kv_off(pad_to(a.q_rank, 16)), ld_in(pad_to(kv_off + a.kv_rank + a.rot_dim, 16)),
+          kvp(pad_latent(a.kv_rank)), kv_off(pad_to(a.q_rank, 16)),
+          gate_off(pad_to(kv_off + (a.kv_from < 0 ? a.kv_rank + a.rot_dim : 0), 8)),
+          ld_in(pad_to(gate_off + (a.gate ? heads * vdp : 0), 16)),
           ld_cq(pad_to(a.q_rank, 128)), hd(dimp + rotp), ld_q(heads * hd), ld_row(kvp + rotp),
           ld_o(pad_to(heads * vdp, 128)) {}
 };
@@ -101,6 +103,7 @@ constexpr int pad_head(int v) { return v <= 128 ? pad_to(v, 32) : v <= 256 ? pad
 // Grouped attention beside or without a memory, and a memory alone, behind one fused projection.
 struct MixShape {
     int q_off = 0, k_off = 0, dimp = 0, ld_attn = 0;   // attention: query and key columns; output heads of dimp
+    int v_off = -1, attn_gate_off = -1;                // its own values, its gates (heads of dimp)
     int mq_off = 0, mk_off = 0, mv_off = 0, gate_off = 0;   // memory: columns of the fused projection
     int channels = 0, ld_conv = 0;                     // StateSpace: convolved columns [values | keys | queries]
     int gates = 0;                                     // fp32 gate columns, a product of their own
@@ -115,9 +118,11 @@ struct MixShape {
         const auto& d = l.memory;
         const int kd = d.kv_heads * d.dim, vd = d.heads * d.vdim;
         if (l.has_attn()) {
-            dimp = pad_head(l.attn.dim);
+            dimp = pad_head(l.attn.widest());
             q_off = place(l.attn.heads * l.attn.dim);
             k_off = place(l.attn.kv_heads * l.attn.dim);
+            if (l.attn.own_values) v_off = place(l.attn.kv_heads * l.attn.vdim);
+            if (l.attn.gate) attn_gate_off = place(l.attn.heads * dimp);
             out = ld_attn = pad_to(l.attn.heads * dimp, 16);
         }
         if (l.has_memory()) {
@@ -150,7 +155,10 @@ struct StackLayer {
     float *pre1 = nullptr, *pre2 = nullptr;     // ahead of the sublayers (null: none)
     Linear w_in;            // everything the mixer projects its input to, fused
     Linear wo;
-    Linear w_up, w_down;    // feed-forward (none: data null)
+    Linear w_up, w_down;    // feed-forward (none: data null).  Gated: w_up's rows are (gate_i, up_i) pairs; a mixture's
+                            // experts are stacked along the rows
+    float *up_bias = nullptr, *down_bias = nullptr;   // gated: in the order of the rows
+    uint16_t* w_router = nullptr;                     // mixture: [experts rounded up to 16, width]
     // latent attention
     Linear w_uq;
     Linear w_ukv;                                // [heads * (dimp + vdp), kvp]: keys and values out of the latent

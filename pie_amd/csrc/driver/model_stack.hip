@@ -168,25 +168,48 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
     for (size_t l = 0; l < stack.size(); ++l) {
         StackLayer& w = stack[l];
         w.spec = cfg.stack[l];
+        // a gated pair of matrices as rows (gate_0, up_0, gate_1, ..)
+        auto paired_rows = [&](const auto& put, const std::string& at, int row0, int ff) {
+            int half = 0;
+            for (const char* name : {"gate", "up"}) {
+                const HostMatrix mat = matrix(at + name, ff, H);
+                for (int r = 0; r < ff; ++r) put(row0 + 2 * r + half, 0, mat.row(r), H);
+                ++half;
+            }
+        };
         const char *post1 = cfg.sandwich_norms ? "norm1b" : "norm1", *post2 = cfg.sandwich_norms ? "norm2b" : "norm2";
         const std::string p = "l" + std::to_string(l) + ".", mix = p + "mix.";
-        w.norm1 = vec(p + post1, H, ones);
-        if (cfg.sandwich_norms) w.pre1 = vec(p + "norm1", H, ones);
+        if (!cfg.shared_norm) w.norm1 = vec(p + post1, H, ones);
+        if (cfg.sandwich_norms || cfg.shared_norm) w.pre1 = vec(p + "norm1", H, ones);
         if (w.spec.mixer == MixerKind::LatentAttention) {
             const LatentAttentionSpec& a = w.spec.latent;
             const LatentShape s(a);
             w.rotary = rotary_of(a.rot);
             w.q_norm = vec(mix + "dq.norm", a.q_rank, ones);
-            w.kv_norm = vec(mix + "dkv.norm", a.kv_rank, ones);
+            if (a.kv_from < 0) w.kv_norm = vec(mix + "dkv.norm", a.kv_rank, ones);
+            // The kernels rotate neighbours: of half-split vectors entry i goes to place 2 i and entry i + dims / 2 to
+            // 2 i + 1, in queries and keys alike (scores do not change).
+            auto rotated_place = [&](int i) {
+                const int half = a.rot.dims / 2;
+                return !a.half_split || i >= a.rot.dims ? i : i < half ? 2 * i : 2 * (i - half) + 1;
+            };
             linear(w.w_in, mix + "in", s.ld_in, Hp, H, [&](auto put) {
                 plain_rows(put, mix + "dq", 0, a.q_rank, H);
-                plain_rows(put, mix + "dkv", s.kv_off, a.kv_rank + a.rot_dim, H);
+                if (a.kv_from < 0) {
+                    const HostMatrix m = matrix(mix + "dkv", a.kv_rank + a.rot_dim, H);
+                    for (int r = 0; r < a.kv_rank + a.rot_dim; ++r)
+                        put(s.kv_off + (r < a.kv_rank ? r : a.kv_rank + rotated_place(r - a.kv_rank)), 0, m.row(r), H);
+                }
+                if (a.gate) {
+                    const HostMatrix m = matrix(mix + "g", a.heads * a.vdim, H);
+                    for (int r = 0; r < a.heads * a.vdim; ++r) put(s.gate_off + r / a.vdim * s.vdp + r % a.vdim, 0, m.row(r), H);
+                }
             });
             linear(w.w_uq, mix + "uq", s.ld_q, s.ld_cq, a.q_rank, [&](auto put) {
                 const HostMatrix m = matrix(mix + "uq", a.heads * (a.dim + a.rot_dim), a.q_rank);
                 for (int h = 0; h < a.heads; ++h)
                     for (int i = 0; i < a.dim + a.rot_dim; ++i)
-                        put(h * s.hd + (i < a.dim ? i : s.dimp + i - a.dim), 0, m.row(h * (a.dim + a.rot_dim) + i), a.q_rank);
+                        put(h * s.hd + (i < a.dim ? i : s.dimp + rotated_place(i - a.dim)), 0, m.row(h * (a.dim + a.rot_dim) + i), a.q_rank);
             });
             HostMatrix uk, uv;
             if (!random) {
@@ -274,15 +297,22 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
             const GroupAttentionSpec& a = w.spec.attn;
             const DecayMemorySpec& d = w.spec.memory;
             const int kd = d.kv_heads * d.dim, vd = d.heads * d.vdim;
-            const std::string left = mix + "left.", mem = w.spec.has_attn() ? mix + "right." : mix;
+            const bool both = w.spec.has_attn() && w.spec.has_memory();
+            const std::string left = both ? mix + "left." : mix, mem = both ? mix + "right." : mix;
             const bool ssm = w.spec.has_memory() && d.kind == DecayKind::StateSpace;
             if (w.spec.has_attn()) {
                 w.rotary = rotary_of(a.rot);
                 auto zeros = [](size_t) { return 0.f; };
-                w.q_bias = vec(left + "q.b", static_cast<size_t>(a.heads) * a.dim, zeros);
-                w.k_bias = vec(left + "k.b", static_cast<size_t>(a.kv_heads) * a.dim, zeros);
-                w.q_norm = vec(left + "q.norm", a.dim, ones);
-                w.k_norm = vec(left + "k.norm", a.dim, ones);
+                const size_t qd = static_cast<size_t>(a.heads) * a.dim, kd_attn = static_cast<size_t>(a.kv_heads) * a.dim;
+                if (a.biases) {
+                    w.q_bias = vec(left + "q.b", qd, zeros);
+                    w.k_bias = vec(left + "k.b", kd_attn, zeros);
+                }
+                if (a.norm != QueryKeyNorm::None) {
+                    const bool whole = a.norm == QueryKeyNorm::WholeProjection;
+                    w.q_norm = vec(left + "q.norm", whole ? qd : a.dim, ones);
+                    w.k_norm = vec(left + "k.norm", whole ? kd_attn : a.dim, ones);
+                }
             }
             // a state-space checkpoint's one projection: gate | values | keys | queries | step sizes
             HostMatrix in;
@@ -291,6 +321,11 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
                 if (w.spec.has_attn()) {
                     plain_rows(put, left + "q", s.q_off, a.heads * a.dim, H);
                     plain_rows(put, left + "k", s.k_off, a.kv_heads * a.dim, H);
+                    if (a.own_values) plain_rows(put, left + "v", s.v_off, a.kv_heads * a.vdim, H);
+                    if (a.gate) {
+                        const HostMatrix m = matrix(left + "g", a.heads * a.vdim, H);
+                        for (int r = 0; r < a.heads * a.vdim; ++r) put(s.attn_gate_off + r / a.vdim * s.dimp + r % a.vdim, 0, m.row(r), H);
+                    }
                 }
                 if (ssm) {
                     for (int r = 0; r < s.channels; ++r) put(s.mv_off + r, 0, in.row(vd + r), H);
@@ -365,9 +400,43 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
                 }
             });
         }
-        if (w.spec.ff > 0) {
+        if (w.spec.moe.experts > 0) {
+            const MixtureSpec& e = w.spec.moe;
+            const int ff = e.ff, ffp = pad_to(ff, 128), rows = pad_to(e.experts, 16);
+            decode_bytes_ += static_cast<size_t>(rows) * Hp * 2;
+            w.w_router = device_matrix(p + "mlp.router", static_cast<size_t>(rows) * Hp, H, [&](std::vector<uint16_t>& host) {
+                const HostMatrix m = matrix(p + "mlp.router", e.experts, H);
+                for (int r = 0; r < e.experts; ++r) std::memcpy(&host[static_cast<size_t>(r) * Hp], m.row(r), static_cast<size_t>(H) * 2);
+            });
+            linear(w.w_up, p + "mlp.experts.up", e.experts * 2 * ffp, Hp, H, [&](auto put) {
+                for (int i = 0; i < e.experts; ++i) paired_rows(put, p + "mlp.e" + std::to_string(i) + ".", i * 2 * ffp, ff);
+            });
+            linear(w.w_down, p + "mlp.experts.down", e.experts * Hp, ffp, ff, [&](auto put) {
+                for (int i = 0; i < e.experts; ++i) plain_rows(put, p + "mlp.e" + std::to_string(i) + ".down", i * Hp, H, ff);
+            });
+        } else if (w.spec.ff > 0 && cfg.ff_act == FeedForwardAct::GatedSilu) {
             const int ff = w.spec.ff, ffp = pad_to(ff, 128);
-            w.norm2 = vec(p + post2, H, ones);
+            linear(w.w_up, p + "mlp.up", 2 * ffp, Hp, H, [&](auto put) { paired_rows(put, p + "mlp.", 0, ff); });
+            linear(w.w_down, p + "mlp.down", Hp, ffp, ff, [&](auto put) { plain_rows(put, p + "mlp.down", 0, H, ff); });
+            std::vector<float> b(static_cast<size_t>(2 * ffp), 0.f);
+            if (!random) {
+                int half = 0;
+                for (const char* name : {"mlp.gate.b", "mlp.up.b"}) {
+                    const StTensor& t = snap->at(p + name);
+                    expect_shape(t, p + name, ff, -1);
+                    std::vector<uint16_t> staging;
+                    const uint16_t* src = as_bf16(t, staging);
+                    for (int r = 0; r < ff; ++r) b[static_cast<size_t>(2 * r + half)] = bf16_value(src[r]);
+                    ++half;
+                }
+            }
+            w.up_bias = static_cast<float*>(alloc(b.size() * 4, ""));
+            PIE_HIP_CHECK(hipMemcpyAsync(w.up_bias, b.data(), b.size() * 4, hipMemcpyHostToDevice, stream));
+            PIE_HIP_CHECK(hipStreamSynchronize(stream));
+            w.down_bias = vec(p + "mlp.down.b", H, [](size_t) { return 0.f; });
+        } else if (w.spec.ff > 0) {
+            const int ff = w.spec.ff, ffp = pad_to(ff, 128);
+            if (!cfg.shared_norm) w.norm2 = vec(p + post2, H, ones);
             if (cfg.sandwich_norms) w.pre2 = vec(p + "norm2", H, ones);
             linear(w.w_up, p + "mlp.up", ffp, Hp, H, [&](auto put) { plain_rows(put, p + "mlp.up", 0, ff, H); });
             linear(w.w_down, p + "mlp.down", Hp, ffp, ff, [&](auto put) { plain_rows(put, p + "mlp.down", 0, H, ff); });

@@ -403,6 +403,17 @@ inline GroupAttentionSpec parse_group_attention(const Json& j, const std::string
     return a;
 }
 
+// Attention as a mixer of its own: interleaved rotation, no biases, no sink.
+inline void read_attention(LayerSpec& l, const Json& j, const std::string& at, QueryKeyNorm norm, bool own_values, bool gate) {
+    l.mixer = MixerKind::Attention;
+    l.attn = parse_group_attention(j, at);
+    l.attn.sink = 0.f;
+    l.attn.half_split = l.attn.biases = false;
+    l.attn.norm = norm;
+    l.attn.own_values = own_values;
+    l.attn.gate = gate;
+}
+
 inline DecayMemorySpec parse_retention(const Json& j, const std::string& at) {
     DecayMemorySpec d;
     d.kind = DecayKind::Retention;
@@ -416,6 +427,24 @@ inline DecayMemorySpec parse_retention(const Json& j, const std::string& at) {
         d.decay.push_back(v.num);
     }
     return d;
+}
+
+inline MixtureSpec parse_mixture(const Json& j, const std::string& at) {
+    MixtureSpec e;
+    const Json &expert = json_object(j, "expert", at), &router = json_object(j, "router", at);
+    e.ff = json_size(expert, "ff", at + " expert");
+    e.limit = static_cast<float>(json_number(expert, "limit", at + " expert"));
+    e.alpha = 1.702f;
+    e.shift = 1.f;
+    e.experts = json_size(router, "experts", at + " router");
+    e.top = json_size(router, "top", at + " router");
+    e.scale = static_cast<float>(router.number_or("scale", 1.0));
+    if (const Json* g = router.get("groups"); g && g->kind == Json::Object) {
+        e.groups = json_size(*g, "count", at + " groups");
+        e.keep = json_size(*g, "keep", at + " groups");
+    }
+    if (e.experts <= 0) throw std::runtime_error("snapshot: " + at + ": router.experts must be positive");
+    return e;
 }
 
 // One entry per mixer kind: config name -> reader of its sizes.
@@ -438,7 +467,17 @@ inline const std::vector<MixerReader>& mixer_registry() {
              a.scale = json_number(j, "scale", at);
              const Json* rot = j.get("rot");
              if (rot && rot->kind == Json::Object) a.rot = parse_rotary(*rot, at + " rot");
+             if (const Json* from = j.get("kv_from"); from && from->kind == Json::Number) {
+                 a.kv_from = json_size(j, "kv_from", at);
+                 if (a.kv_from < 0) throw std::runtime_error("snapshot: " + at + ": kv_from must not be negative");
+             }
          }},
+        {"attention",
+         [](LayerSpec& l, const Json& j, const std::string& at) {
+             read_attention(l, j, at, QueryKeyNorm::WholeProjection, true, false);
+         }},
+        {"attention_2",
+         [](LayerSpec& l, const Json& j, const std::string& at) { read_attention(l, j, at, QueryKeyNorm::None, false, true); }},
         {"channel_delta",
          [](LayerSpec& l, const Json& j, const std::string& at) {
              l.mixer = MixerKind::ChannelDelta;
@@ -489,22 +528,30 @@ struct StackArchitecture {
     const char* arch;
     bool sandwich_norms;
     FeedForwardAct ff_act;
+    bool shared_norm = false;
+    bool gated_latents = false;   // latent attention with an output gate and half-split rotation
 };
 inline const std::vector<StackArchitecture>& stack_registry() {
     static const std::vector<StackArchitecture> table = {
         {"Varasun", "varasun", false, FeedForwardAct::SquaredRelu},
         {"Lofudra", "lofudra", true, FeedForwardAct::Gelu},
+        {"Fobanex", "fobanex", false, FeedForwardAct::GatedSilu, true, true},
     };
     return table;
 }
 
 // {"architecture", "width", "vocab", "norm": {"eps"}, "logit_scale", "logit_softcap",
-//  "loop": {"start", "stop", "times"},
-//  "layers": [{"type", "mixer": {...}, "mlp": {"kind", "ff"} | null}, ...]}
+//  "loop": {"start", "stop", "times"}, "embedding": {"scale"},
+//  "layers": [{"type", "mixer": {...}, "mlp": {"kind": "dense", "ff"} | {"kind": "moe", "expert": {"ff", "limit"},
+//              "router": {"experts", "top", "scale", "groups": {"count", "keep"}}} | null}, ...]}
 inline void apply_stack_config(ModelConfig& m, const Json& c, const StackArchitecture& a) {
     m.arch = a.arch;
     m.sandwich_norms = a.sandwich_norms;
     m.ff_act = a.ff_act;
+    m.shared_norm = a.shared_norm;
+    m.embed_scale = 1.f;
+    if (const Json* e = c.get("embedding"); a.shared_norm && e && e->kind == Json::Object)
+        m.embed_scale = static_cast<float>(e->number_or("scale", 1.0));
     m.hidden = json_size(c, "width", "config.json");
     m.vocab = json_size(c, "vocab", "config.json");
     const Json* norm = c.get("norm");
@@ -535,11 +582,17 @@ inline void apply_stack_config(ModelConfig& m, const Json& c, const StackArchite
                 known = true;
             }
         if (!known) throw std::runtime_error("snapshot: " + at + ": unknown mixer '" + type + "'");
+        l.latent.gate = l.latent.half_split = a.gated_latents;
         if (const Json* mlp = j.get("mlp"); mlp && mlp->kind == Json::Object) {
             const std::string kind = mlp->string_or("kind", "");
-            if (kind != "dense") throw std::runtime_error("snapshot: " + at + ": unknown mlp kind '" + kind + "'");
-            l.ff = json_size(*mlp, "ff", at + " mlp");
-            if (l.ff <= 0) throw std::runtime_error("snapshot: " + at + ": mlp.ff must be positive");
+            if (kind == "dense") {
+                l.ff = json_size(*mlp, "ff", at + " mlp");
+                if (l.ff <= 0) throw std::runtime_error("snapshot: " + at + ": mlp.ff must be positive");
+            } else if (kind == "moe" && a.shared_norm) {
+                l.moe = parse_mixture(*mlp, at + " mlp");
+            } else {
+                throw std::runtime_error("snapshot: " + at + ": unknown mlp kind '" + kind + "'");
+            }
         }
         m.stack.push_back(l);
     }

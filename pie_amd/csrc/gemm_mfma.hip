@@ -51,6 +51,7 @@ struct GemmArgs {
     uint16_t* y;
     int M, N, K, g_shift, beta, swiglu, scale_is_bf16;
     int pointwise;        // PIE_HIP_EPI_RELU2 and above: applied to the sum (0: nothing)
+    PieHipGlu glu = kPlainGlu;   // swiglu
     float* partial;   // split-K: fp32 [gridDim.z][M][N] partial sums (row scale applied), else null
 };
 
@@ -372,13 +373,12 @@ __global__ __launch_bounds__(SH::kNW* kWave) void gemm_mfma_kernel(const GemmArg
                 if (a.partial) {
                     if (ok) a.partial[(static_cast<size_t>(blockIdx.z) * M + m) * N + n] = v;
                 } else if (a.swiglu) {
+                    if (a.glu.bias) v += a.glu.bias[min(n, N - 1)];
                     const float gb = bf16_bits_to_f32(f32_to_bf16_bits(v));
                     const float other = __int_as_float(__builtin_amdgcn_update_dpp(
                         0, __float_as_int(gb), 0xB1, 0xF, 0xF, true));  // quad_perm [1,0,3,2]
-                    if ((j & 1) == 0 && ok) {
-                        const float silu = gb / (1.f + expf(-gb));
-                        a.y[static_cast<size_t>(m) * nout + n / 2] = f32_to_bf16_bits(silu * other);
-                    }
+                    if ((j & 1) == 0 && ok)
+                        a.y[static_cast<size_t>(m) * nout + n / 2] = f32_to_bf16_bits(glu_value(gb, other, a.glu));
                 } else if (ok) {
                     const size_t o = static_cast<size_t>(m) * nout + n;
                     v = epilogue_pointwise<true>(v, a.pointwise);
@@ -393,7 +393,7 @@ __global__ __launch_bounds__(SH::kNW* kWave) void gemm_mfma_kernel(const GemmArg
 // (residual add, or SwiGLU over adjacent (gate, up) columns with both rounded to bf16 first).
 __global__ __launch_bounds__(256) void gemm_splitk_reduce_kernel(const float* partial, uint16_t* y,
                                                                  int M, int N, int splits, int beta,
-                                                                 int swiglu, int pointwise) {
+                                                                 int swiglu, int pointwise, const PieHipGlu glu) {
     const int nout = swiglu ? N / 2 : N;
     const size_t idx = static_cast<size_t>(blockIdx.x) * 256 + threadIdx.x;
     if (idx >= static_cast<size_t>(M) * nout) return;
@@ -406,10 +406,13 @@ __global__ __launch_bounds__(256) void gemm_splitk_reduce_kernel(const float* pa
             g += p[z * plane];
             u += p[z * plane + 1];
         }
+        if (glu.bias) {
+            g += glu.bias[2 * c];
+            u += glu.bias[2 * c + 1];
+        }
         const float gb = bf16_bits_to_f32(f32_to_bf16_bits(g));
         const float ub = bf16_bits_to_f32(f32_to_bf16_bits(u));
-        const float silu = gb / (1.f + expf(-gb));
-        y[idx] = f32_to_bf16_bits(silu * ub);
+        y[idx] = f32_to_bf16_bits(glu_value(gb, ub, glu));
     } else {
         const float* p = partial + static_cast<size_t>(m) * N + c;
         float v = 0.f;
@@ -482,7 +485,7 @@ int launch_gemm_splitk(GemmArgs a, int splits, float* ws, hipStream_t stream) {
     if (st != PIE_HIP_OK) return st;
     const size_t outs = static_cast<size_t>(a.M) * (swiglu ? a.N / 2 : a.N);
     hipLaunchKernelGGL(gemm_splitk_reduce_kernel, dim3(static_cast<unsigned>((outs + 255) / 256)), dim3(256), 0,
-                       stream, ws, a.y, a.M, a.N, splits, beta, swiglu, pointwise);
+                       stream, ws, a.y, a.M, a.N, splits, beta, swiglu, pointwise, a.glu);
     return launch_status();
 }
 
@@ -493,7 +496,8 @@ namespace pie_hip {
 namespace {
 int gemm_entry(int format, const uint16_t* act_bf16, const void* weight, const void* scale,
                int scale_is_bf16, int group_size, uint16_t* y_bf16, int M, int N, int K, int beta,
-               int swiglu, void* workspace, size_t workspace_bytes, void* stream) {
+               int swiglu, const PieHipGlu* glu, void* workspace, size_t workspace_bytes, void* stream) {
+    if (!glu_ok(glu, swiglu)) return PIE_HIP_ERR_INVALID;
     if (!act_bf16 || !weight || !y_bf16 || M <= 0 || N <= 0 || K <= 0) return PIE_HIP_ERR_INVALID;
     if (format != PIE_HIP_FMT_BF16 && !scale) return PIE_HIP_ERR_INVALID;
     if (K % BK != 0) return PIE_HIP_ERR_UNSUPPORTED;
@@ -512,6 +516,7 @@ int gemm_entry(int format, const uint16_t* act_bf16, const void* weight, const v
     a.beta = beta;
     a.swiglu = swiglu;
     a.pointwise = pointwise;
+    if (glu) a.glu = *glu;
     a.scale_is_bf16 = scale_is_bf16;
     hipStream_t st = static_cast<hipStream_t>(stream);
     if (format == PIE_HIP_FMT_INT4B8) {
@@ -548,7 +553,7 @@ extern "C" int pie_hip_gemm_mfma(int format, const uint16_t* act_bf16, const voi
                                  uint16_t* y_bf16, int M, int N, int K, int beta, int swiglu,
                                  void* stream) {
     return pie_hip::gemm_entry(format, act_bf16, weight, scale, scale_is_bf16, group_size, y_bf16, M, N,
-                               K, beta, swiglu, nullptr, 0, stream);
+                               K, beta, swiglu, nullptr, nullptr, 0, stream);
 }
 
 extern "C" size_t pie_hip_gemm_mfma_workspace_bytes(int M, int N, int K) {
@@ -562,5 +567,13 @@ extern "C" int pie_hip_gemm_mfma_splitk(int format, const uint16_t* act_bf16, co
                                         uint16_t* y_bf16, int M, int N, int K, int beta, int swiglu,
                                         void* workspace, size_t workspace_bytes, void* stream) {
     return pie_hip::gemm_entry(format, act_bf16, weight, scale, scale_is_bf16, group_size, y_bf16, M, N,
-                               K, beta, swiglu, workspace, workspace_bytes, stream);
+                               K, beta, swiglu, nullptr, workspace, workspace_bytes, stream);
+}
+
+extern "C" int pie_hip_gemm_mfma_glu(int format, const uint16_t* act_bf16, const void* weight,
+                                     const void* scale, int scale_is_bf16, int group_size,
+                                     uint16_t* y_bf16, int M, int N, int K, int beta, int swiglu,
+                                     const PieHipGlu* glu, void* workspace, size_t workspace_bytes, void* stream) {
+    return pie_hip::gemm_entry(format, act_bf16, weight, scale, scale_is_bf16, group_size, y_bf16, M, N,
+                               K, beta, swiglu, glu, workspace, workspace_bytes, stream);
 }

@@ -140,6 +140,7 @@ struct SkinnyArgs {
     uint16_t* v_pages;
     int hq, hk, d;
     int half_out;   // q / k rows re-ordered at load: pair (2i, 2i+1) goes to positions (i, i + d/2)
+    PieHipGlu glu = kPlainGlu;   // swiglu
 };
 
 constexpr int gcd_c(int a, int b) { return b == 0 ? a : gcd_c(b, a % b); }
@@ -394,13 +395,12 @@ __global__ __launch_bounds__(KP* kWave) void skinny_kernel(const SkinnyArgs a) {
             float v = (total(i) + bias) * row_scale[i];
             if (a.swiglu) {
                 // columns (2i, 2i+1) = (gate_i, up_i) sit in adjacent lanes
+                if (a.glu.bias) v += a.glu.bias[min(n, N - 1)];
                 const float gb = bf16_bits_to_f32(f32_to_bf16_bits(v));
                 const float other = __int_as_float(__builtin_amdgcn_update_dpp(
                     0, __float_as_int(gb), 0xB1, 0xF, 0xF, true));  // quad_perm [1,0,3,2]
-                if ((j & 1) == 0 && ok) {
-                    const float silu = gb / (1.f + expf(-gb));
-                    a.y[static_cast<size_t>(m) * nout + n / 2] = f32_to_bf16_bits(silu * other);
-                }
+                if ((j & 1) == 0 && ok)
+                    a.y[static_cast<size_t>(m) * nout + n / 2] = f32_to_bf16_bits(glu_value(gb, other, a.glu));
             } else if (ok) {
                 const size_t o = static_cast<size_t>(m) * nout + n;
                 v = epilogue_pointwise<std::is_same<F, SkBf16>::value>(v, a.pointwise);
@@ -747,13 +747,12 @@ __global__ __launch_bounds__(kSwWaves* kWave, NG == 1 && MT == 1 ? 4 : 2) void s
                     }
                 }
             } else if (a.swiglu) {
+                if (a.glu.bias) v += a.glu.bias[min(n, N - 1)];
                 const float gb = bf16_bits_to_f32(f32_to_bf16_bits(v));
                 const float other = __int_as_float(__builtin_amdgcn_update_dpp(
                     0, __float_as_int(gb), 0xB1, 0xF, 0xF, true));  // quad_perm [1,0,3,2]
-                if ((j & 1) == 0 && ok) {
-                    const float silu = gb / (1.f + expf(-gb));
-                    a.y[static_cast<size_t>(m) * nout + n / 2] = f32_to_bf16_bits(silu * other);
-                }
+                if ((j & 1) == 0 && ok)
+                    a.y[static_cast<size_t>(m) * nout + n / 2] = f32_to_bf16_bits(glu_value(gb, other, a.glu));
             } else if (ok) {
                 const size_t o = static_cast<size_t>(m) * nout + n;
                 v = epilogue_pointwise<std::is_same<F, SkBf16>::value>(v, a.pointwise);
@@ -966,12 +965,12 @@ int dispatch_skinny(int format, const SkinnyArgs& a, int problems, hipStream_t s
 }  // namespace
 }  // namespace pie_hip
 
-extern "C" int pie_hip_gemm_skinny(int format, const uint16_t* act_bf16, const void* weight,
-                                   const void* scale, int scale_is_bf16, int group_size,
-                                   uint16_t* y_bf16, int M, int N, int K, int beta, int swiglu,
-                                   void* stream) {
-    using namespace pie_hip;
-    if (!act_bf16 || !weight || !y_bf16 || M <= 0) return PIE_HIP_ERR_INVALID;
+namespace pie_hip {
+namespace {
+int skinny_entry(int format, const uint16_t* act_bf16, const void* weight, const void* scale, int scale_is_bf16,
+                 int group_size, uint16_t* y_bf16, int M, int N, int K, int beta, int swiglu, int tiled,
+                 const PieHipGlu* glu, void* stream) {
+    if (!act_bf16 || !weight || !y_bf16 || M <= 0 || !glu_ok(glu, swiglu)) return PIE_HIP_ERR_INVALID;
     if (format != PIE_HIP_FMT_BF16 && !scale) return PIE_HIP_ERR_INVALID;
     SkinnyArgs a{};
     a.act = act_bf16;
@@ -985,21 +984,18 @@ extern "C" int pie_hip_gemm_skinny(int format, const uint16_t* act_bf16, const v
     a.beta = beta;
     a.swiglu = swiglu == PIE_HIP_EPI_SWIGLU ? 1 : 0;
     a.pointwise = pointwise_code(swiglu);
+    if (glu) a.glu = *glu;
     a.scale_is_bf16 = scale_is_bf16;
+    a.tiled = tiled ? 1 : 0;
     return dispatch_skinny(format, a, 1, static_cast<hipStream_t>(stream));
 }
 
-extern "C" int pie_hip_moe_grouped_gemm(int format, const uint16_t* act_bf16,
-                                        const int32_t* route_act_rows,
-                                        const int32_t* expert_offsets, int num_experts,
-                                        int max_rows_per_expert, const void* weights,
-                                        size_t weight_stride_bytes, const void* scales,
-                                        size_t scale_stride_bytes, int scale_is_bf16,
-                                        int group_size, uint16_t* y_bf16, int N, int K, int swiglu,
-                                        void* stream) {
-    using namespace pie_hip;
-    if (!act_bf16 || !expert_offsets || !weights || !y_bf16 || num_experts <= 0 ||
-        max_rows_per_expert <= 0)
+int grouped_entry(int format, const uint16_t* act_bf16, const int32_t* route_act_rows, const int32_t* expert_offsets,
+                  int num_experts, int max_rows_per_expert, const void* weights, size_t weight_stride_bytes,
+                  const void* scales, size_t scale_stride_bytes, int scale_is_bf16, int group_size, uint16_t* y_bf16,
+                  int N, int K, int swiglu, int tiled, const PieHipGlu* glu, void* stream) {
+    if (!act_bf16 || !expert_offsets || !weights || !y_bf16 || num_experts <= 0 || max_rows_per_expert <= 0 ||
+        !glu_ok(glu, swiglu))
         return PIE_HIP_ERR_INVALID;
     if (format != PIE_HIP_FMT_BF16 && !scales) return PIE_HIP_ERR_INVALID;
     SkinnyArgs a{};
@@ -1014,35 +1010,56 @@ extern "C" int pie_hip_moe_grouped_gemm(int format, const uint16_t* act_bf16,
     a.G = group_size;
     a.swiglu = swiglu == PIE_HIP_EPI_SWIGLU ? 1 : 0;
     a.pointwise = pointwise_code(swiglu);
+    if (glu) a.glu = *glu;
     a.scale_is_bf16 = scale_is_bf16;
+    a.tiled = tiled ? 1 : 0;
     a.w_stride = weight_stride_bytes;
     a.scale_stride = scale_stride_bytes;
     return dispatch_skinny(format, a, num_experts, static_cast<hipStream_t>(stream));
 }
+}  // namespace
+}  // namespace pie_hip
 
-// ---- the same two entry points over weights in the tile-major layout ----------------------
-extern "C" int pie_hip_gemm_skinny_tiled(int format, const uint16_t* act_bf16, const void* weight,
-                                   const void* scale, int scale_is_bf16, int group_size,
-                                   uint16_t* y_bf16, int M, int N, int K, int beta, int swiglu,
-                                   void* stream) {
-    using namespace pie_hip;
-    if (!act_bf16 || !weight || !y_bf16 || M <= 0) return PIE_HIP_ERR_INVALID;
-    if (format != PIE_HIP_FMT_BF16 && !scale) return PIE_HIP_ERR_INVALID;
-    SkinnyArgs a{};
-    a.act = act_bf16;
-    a.w = static_cast<const unsigned char*>(weight);
-    a.scale = static_cast<const unsigned char*>(scale);
-    a.y = y_bf16;
-    a.M = M;
-    a.N = N;
-    a.K = K;
-    a.G = group_size;
-    a.beta = beta;
-    a.swiglu = swiglu == PIE_HIP_EPI_SWIGLU ? 1 : 0;
-    a.pointwise = pointwise_code(swiglu);
-    a.scale_is_bf16 = scale_is_bf16;
-    a.tiled = 1;
-    return dispatch_skinny(format, a, 1, static_cast<hipStream_t>(stream));
+extern "C" int pie_hip_gemm_skinny(int format, const uint16_t* act_bf16, const void* weight, const void* scale,
+                                   int scale_is_bf16, int group_size, uint16_t* y_bf16, int M, int N, int K,
+                                   int beta, int swiglu, void* stream) {
+    return pie_hip::skinny_entry(format, act_bf16, weight, scale, scale_is_bf16, group_size, y_bf16, M, N, K, beta, swiglu,
+                                 0, nullptr, stream);
+}
+
+extern "C" int pie_hip_gemm_skinny_glu(int format, const uint16_t* act_bf16, const void* weight, const void* scale,
+                                       int scale_is_bf16, int group_size, uint16_t* y_bf16, int M, int N, int K,
+                                       int beta, int swiglu, int tiled, const PieHipGlu* glu, void* stream) {
+    return pie_hip::skinny_entry(format, act_bf16, weight, scale, scale_is_bf16, group_size, y_bf16, M, N, K, beta, swiglu,
+                                 tiled, glu, stream);
+}
+
+extern "C" int pie_hip_moe_grouped_gemm(int format, const uint16_t* act_bf16, const int32_t* route_act_rows,
+                                        const int32_t* expert_offsets, int num_experts, int max_rows_per_expert,
+                                        const void* weights, size_t weight_stride_bytes, const void* scales,
+                                        size_t scale_stride_bytes, int scale_is_bf16, int group_size, uint16_t* y_bf16,
+                                        int N, int K, int swiglu, void* stream) {
+    return pie_hip::grouped_entry(format, act_bf16, route_act_rows, expert_offsets, num_experts, max_rows_per_expert, weights,
+                                  weight_stride_bytes, scales, scale_stride_bytes, scale_is_bf16, group_size, y_bf16, N, K,
+                                  swiglu, 0, nullptr, stream);
+}
+
+extern "C" int pie_hip_moe_grouped_gemm_glu(int format, const uint16_t* act_bf16, const int32_t* route_act_rows,
+                                            const int32_t* expert_offsets, int num_experts, int max_rows_per_expert,
+                                            const void* weights, size_t weight_stride_bytes, const void* scales,
+                                            size_t scale_stride_bytes, int scale_is_bf16, int group_size, uint16_t* y_bf16,
+                                            int N, int K, int swiglu, int tiled, const PieHipGlu* glu, void* stream) {
+    return pie_hip::grouped_entry(format, act_bf16, route_act_rows, expert_offsets, num_experts, max_rows_per_expert, weights,
+                                  weight_stride_bytes, scales, scale_stride_bytes, scale_is_bf16, group_size, y_bf16, N, K,
+                                  swiglu, tiled, glu, stream);
+}
+
+// ---- over weights in the tile-major layout ----------------------
+extern "C" int pie_hip_gemm_skinny_tiled(int format, const uint16_t* act_bf16, const void* weight, const void* scale,
+                                         int scale_is_bf16, int group_size, uint16_t* y_bf16, int M, int N, int K,
+                                         int beta, int swiglu, void* stream) {
+    return pie_hip::skinny_entry(format, act_bf16, weight, scale, scale_is_bf16, group_size, y_bf16, M, N, K, beta, swiglu,
+                                 1, nullptr, stream);
 }
 
 // q|k|v projection over tile-major weights with RoPE and the KV write in the epilogue (more rows
@@ -1082,36 +1099,14 @@ extern "C" int pie_hip_qkv_rope_skinny_tiled(int format, const uint16_t* act_bf1
     return dispatch_skinny(format, a, 1, static_cast<hipStream_t>(stream));
 }
 
-extern "C" int pie_hip_moe_grouped_gemm_tiled(int format, const uint16_t* act_bf16,
-                                        const int32_t* route_act_rows,
-                                        const int32_t* expert_offsets, int num_experts,
-                                        int max_rows_per_expert, const void* weights,
-                                        size_t weight_stride_bytes, const void* scales,
-                                        size_t scale_stride_bytes, int scale_is_bf16,
-                                        int group_size, uint16_t* y_bf16, int N, int K, int swiglu,
-                                        void* stream) {
-    using namespace pie_hip;
-    if (!act_bf16 || !expert_offsets || !weights || !y_bf16 || num_experts <= 0 ||
-        max_rows_per_expert <= 0)
-        return PIE_HIP_ERR_INVALID;
-    if (format != PIE_HIP_FMT_BF16 && !scales) return PIE_HIP_ERR_INVALID;
-    SkinnyArgs a{};
-    a.act = act_bf16;
-    a.act_rows = route_act_rows;
-    a.w = static_cast<const unsigned char*>(weights);
-    a.scale = static_cast<const unsigned char*>(scales);
-    a.y = y_bf16;
-    a.offsets = expert_offsets;
-    a.N = N;
-    a.K = K;
-    a.G = group_size;
-    a.swiglu = swiglu == PIE_HIP_EPI_SWIGLU ? 1 : 0;
-    a.pointwise = pointwise_code(swiglu);
-    a.scale_is_bf16 = scale_is_bf16;
-    a.tiled = 1;
-    a.w_stride = weight_stride_bytes;
-    a.scale_stride = scale_stride_bytes;
-    return dispatch_skinny(format, a, num_experts, static_cast<hipStream_t>(stream));
+extern "C" int pie_hip_moe_grouped_gemm_tiled(int format, const uint16_t* act_bf16, const int32_t* route_act_rows,
+                                              const int32_t* expert_offsets, int num_experts, int max_rows_per_expert,
+                                              const void* weights, size_t weight_stride_bytes, const void* scales,
+                                              size_t scale_stride_bytes, int scale_is_bf16, int group_size, uint16_t* y_bf16,
+                                              int N, int K, int swiglu, void* stream) {
+    return pie_hip::grouped_entry(format, act_bf16, route_act_rows, expert_offsets, num_experts, max_rows_per_expert, weights,
+                                  weight_stride_bytes, scales, scale_stride_bytes, scale_is_bf16, group_size, y_bf16, N, K,
+                                  swiglu, 1, nullptr, stream);
 }
 
 namespace {

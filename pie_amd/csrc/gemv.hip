@@ -281,6 +281,7 @@ struct GemvArgs {
     const int32_t* mg_row_len;   // visible keys per row
     int mg_nsplit, mg_units_per_split, mg_hq, mg_d;
     int pointwise;   // PIE_HIP_EPI_RELU2 and above: applied to the sum (0: nothing)
+    PieHipGlu glu = kPlainGlu;   // swiglu
 };
 
 // attn_decode_merge_kernel's arithmetic for the eight output dimensions d0 .. d0 + 7 of one
@@ -713,12 +714,15 @@ __global__ __launch_bounds__(kBlock) void gemv_kernel(const GemvArgs a) {
                             gv *= u.rs;
                             uv *= u.rs2;
                         }
+                        if (!ROPE && a.glu.bias) {
+                            gv += a.glu.bias[row];
+                            uv += a.glu.bias[row + 1];
+                        }
                         const float gb = bf16_bits_to_f32(f32_to_bf16_bits(gv));
                         const float ub = bf16_bits_to_f32(f32_to_bf16_bits(uv));
                         const int m = lane % M;
                         if (!ROPE) {
-                            const float silu = gb / (1.f + expf(-gb));
-                            a.y[static_cast<size_t>(m) * (N / 2) + row / 2] = f32_to_bf16_bits(silu * ub);
+                            a.y[static_cast<size_t>(m) * (N / 2) + row / 2] = f32_to_bf16_bits(glu_value(gb, ub, a.glu));
                         } else {
                             // the projection's bf16 values, then the rotation of
                             // qkv_rope_kvwrite_kernel with the same operations and rounding
@@ -1113,9 +1117,20 @@ extern "C" int pie_hip_linear_fused(int format, const uint16_t* act_bf16,
                                     const void* weight, const void* scale, int scale_is_bf16,
                                     int group_size, uint16_t* y_bf16, int M, int N, int K,
                                     int beta, int swiglu, void* stream) {
+    return pie_hip_linear_fused_glu(format, act_bf16, norm_weight_bf16, eps, weight, scale, scale_is_bf16, group_size, y_bf16,
+                                    M, N, K, beta, swiglu, nullptr, stream);
+}
+
+extern "C" int pie_hip_linear_fused_glu(int format, const uint16_t* act_bf16,
+                                        const uint16_t* norm_weight_bf16, float eps,
+                                        const void* weight, const void* scale, int scale_is_bf16,
+                                        int group_size, uint16_t* y_bf16, int M, int N, int K,
+                                        int beta, int swiglu, const PieHipGlu* glu, void* stream) {
     using namespace pie_hip;
+    if (!glu_ok(glu, swiglu)) return PIE_HIP_ERR_INVALID;
     GemvArgs a{act_bf16, static_cast<const u32x4_t*>(weight), nullptr, nullptr, y_bf16, N, K,
                group_size, beta, norm_weight_bf16, eps, swiglu == PIE_HIP_EPI_SWIGLU ? 1 : 0};
+    if (glu) a.glu = *glu;
     a.pointwise = pointwise_code(swiglu);
     if (a.pointwise && beta) return PIE_HIP_ERR_INVALID;
     if (a.pointwise == PIE_HIP_EPI_GELU && format != PIE_HIP_FMT_BF16) return PIE_HIP_ERR_UNSUPPORTED;

@@ -1,5 +1,6 @@
 // Grouped-query attention of the layer stacks: any head size, any number of query heads per key head, an
-// optional sliding window, an optional sink (a constant added to the sum of exponentials).
+// optional sliding window, an optional sink (a constant added to the sum of exponentials), an optional gate
+// on the output.
 //   o[n, h, :] = sum_j p_j v_j,  p_j = exp(s_j) / (sink + sum exp(s)),  s_j = q[n, h, :] . k_j * scale,
 //   len - window <= j < len = row_kv_len[n]
 // A cache row holds, per key head, the key and the value next to each other: [kv_heads][dimp | dimp].
@@ -166,6 +167,163 @@ __global__ __launch_bounds__(256) void group_prep_vec_kernel(const PrepArgs a) {
     }
 }
 
+// One norm over a row's whole query projection and one over its whole key projection, values of their own
+// size, either pairing of the rotated entries.  One block per row.
+struct JointPrepArgs {
+    const void* fused;
+    const float *q_norm, *k_norm, *rope;
+    const int64_t* slots;
+    void *q, *pool;
+    int q_off, k_off, v_off, rot_dims, adjacent, ld, heads, kv_heads, dim, vdim, dimp;
+    float eps;
+};
+// Eight neighbouring values per thread and unit (pairs of neighbours rotate inside one): the first kCache units
+// of a thread stay in registers between the sums and the stores.
+template <class T>
+__global__ __launch_bounds__(256) void group_prep_joint_vec_kernel(const JointPrepArgs a) {
+    __shared__ float red[2][256 / kWave];
+    constexpr int kCache = 4;
+    const size_t n = blockIdx.x;
+    const int tid = threadIdx.x, lane = tid & (kWave - 1), wv = tid / kWave;
+    const T* row = static_cast<const T*>(a.fused) + n * a.ld;
+    const int per = a.dimp / 8, nq = a.heads * per, nk = a.kv_heads * per, total = nq + 2 * nk;   // q | k | v
+    const int64_t slot = a.slots[n];
+    // where unit u's values are (null: padding), and its place
+    auto source = [&](int u, int& h, int& d) -> const T* {
+        const int part = u < nq ? 0 : u < nq + nk ? 1 : 2;
+        const int w = u - (part == 0 ? 0 : part == 1 ? nq : nq + nk);
+        h = w / per;
+        d = 8 * (w - h * per);
+        if (d >= (part == 2 ? a.vdim : a.dim)) return nullptr;
+        if (part == 0) return row + a.q_off + h * a.dim + d;
+        if (part == 1 || a.v_off < 0) return row + a.k_off + h * a.dim + d;   // (values that are the keys as projected)
+        return row + a.v_off + h * a.vdim + d;
+    };
+    float x[kCache][8], sq = 0.f, sk = 0.f;
+    auto add_up = [&](int u, const float* f) {
+        float s = 0.f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) s += f[e] * f[e];
+        if (u < nq) sq += s;
+        else if (u < nq + nk) sk += s;
+    };
+#pragma unroll
+    for (int c = 0; c < kCache; ++c) {
+        const int u = tid + 256 * c;
+        int h, d;
+        const T* p = u < total ? source(u, h, d) : nullptr;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[c][e] = 0.f;
+        if (p) load8(p, x[c]);
+    }
+    float inv_q = 1.f, inv_k = 1.f;
+    if (a.q_norm || a.k_norm) {
+#pragma unroll
+        for (int c = 0; c < kCache; ++c)
+            if (tid + 256 * c < nq + nk) add_up(tid + 256 * c, x[c]);
+        for (int u = tid + 256 * kCache; u < nq + nk; u += 256) {
+            int h, d;
+            float f[8];
+            if (const T* p = source(u, h, d)) {
+                load8(p, f);
+                add_up(u, f);
+            }
+        }
+        sq = wave_sum(sq);
+        sk = wave_sum(sk);
+        if (lane == 0) {
+            red[0][wv] = sq;
+            red[1][wv] = sk;
+        }
+        __syncthreads();
+        sq = sk = 0.f;
+#pragma unroll
+        for (int w = 0; w < 256 / kWave; ++w) {
+            sq += red[0][w];
+            sk += red[1][w];
+        }
+        if (a.q_norm) inv_q = 1.f / sqrtf(sq / static_cast<float>(a.heads * a.dim) + a.eps);
+        if (a.k_norm) inv_k = 1.f / sqrtf(sk / static_cast<float>(a.kv_heads * a.dim) + a.eps);
+    }
+    const float* tab = a.rope + n * a.rot_dims;
+    const int half = a.rot_dims / 2;
+    auto finish = [&](int u, float* f) {
+        int h, d;
+        const bool in = source(u, h, d) != nullptr;
+        if (u < nq + nk && in) {
+            const float* norm = u < nq ? a.q_norm : a.k_norm;
+            const float inv = u < nq ? inv_q : inv_k;
+            if (norm) {
+                float w[8];
+                load8(norm + h * a.dim + d, w);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) f[e] *= inv * w[e];
+            }
+#pragma unroll
+            for (int e = 0; e < 8; e += 2)
+                if (d + e < a.rot_dims) {
+                    const float c = tab[(d + e) >> 1], s = tab[half + ((d + e) >> 1)], u0 = f[e], u1 = f[e + 1];
+                    f[e] = u0 * c - u1 * s;
+                    f[e + 1] = u1 * c + u0 * s;
+                }
+        }
+        if (u < nq) {
+            store8(static_cast<T*>(a.q) + (n * a.heads + h) * a.dimp + d, f);
+        } else if (slot >= 0) {
+            T* k = static_cast<T*>(a.pool) + (static_cast<size_t>(slot) * a.kv_heads + h) * 2 * a.dimp + d;
+            store8(u < nq + nk ? k : k + a.dimp, f);
+        }
+    };
+#pragma unroll
+    for (int c = 0; c < kCache; ++c)
+        if (tid + 256 * c < total) finish(tid + 256 * c, x[c]);
+    for (int u = tid + 256 * kCache; u < total; u += 256) {
+        int h, d;
+        float f[8] = {};
+        if (const T* p = source(u, h, d)) load8(p, f);
+        finish(u, f);
+    }
+}
+// Any size and pairing, a value per thread.
+template <class T>
+__global__ __launch_bounds__(256) void group_prep_joint_kernel(const JointPrepArgs a) {
+    __shared__ float red[256 / kWave];
+    const size_t n = blockIdx.x;
+    const T *row = static_cast<const T*>(a.fused) + n * a.ld, *q = row + a.q_off, *k = row + a.k_off;
+    const int Q = a.heads * a.dim, K = a.kv_heads * a.dim;
+    auto inverse = [&](const T* p, int len) {
+        float s = 0.f;
+        for (int i = threadIdx.x; i < len; i += 256) {
+            const float v = act_get<T>(p[i]);
+            s += v * v;
+        }
+        return 1.f / sqrtf(block_total(s, red) / static_cast<float>(len) + a.eps);
+    };
+    const float inv_q = a.q_norm ? inverse(q, Q) : 1.f, inv_k = a.k_norm ? inverse(k, K) : 1.f;
+    const int64_t slot = a.slots[n];
+    const float* tab = a.rope + n * a.rot_dims;
+    const int half = a.rot_dims / 2;
+    auto rotated = [&](const T* p, const float* norm, float inv, int h, int d) {
+        auto value = [&](int i) { return act_get<T>(p[h * a.dim + i]) * (norm ? inv * norm[h * a.dim + i] : 1.f); };
+        if (d >= a.rot_dims) return value(d);
+        const bool first = a.adjacent ? (d & 1) == 0 : d < half;
+        const int t = a.adjacent ? d >> 1 : first ? d : d - half, other = a.adjacent ? d ^ 1 : first ? d + half : d - half;
+        return first ? value(d) * tab[t] - value(other) * tab[half + t] : value(d) * tab[t] + value(other) * tab[half + t];
+    };
+    for (int i = threadIdx.x; i < a.heads * a.dimp; i += 256) {
+        const int h = i / a.dimp, d = i % a.dimp;
+        static_cast<T*>(a.q)[n * a.heads * a.dimp + i] = act_put<T>(d < a.dim ? rotated(q, a.q_norm, inv_q, h, d) : 0.f);
+    }
+    if (slot < 0) return;
+    T* pool = static_cast<T*>(a.pool) + static_cast<size_t>(slot) * a.kv_heads * 2 * a.dimp;
+    for (int i = threadIdx.x; i < a.kv_heads * a.dimp; i += 256) {
+        const int h = i / a.dimp, d = i % a.dimp;
+        const T zero = act_put<T>(0.f);
+        pool[h * 2 * a.dimp + d] = d < a.dim ? act_put<T>(rotated(k, a.k_norm, inv_k, h, d)) : zero;
+        pool[(h * 2 + 1) * a.dimp + d] = d >= a.vdim ? zero : a.v_off < 0 ? k[h * a.dim + d] : row[a.v_off + h * a.vdim + d];
+    }
+}
+
 // ---- any size, any compute type --------------------------------------------------------------------
 struct PlainArgs {
     const void *q, *pool;
@@ -174,6 +332,8 @@ struct PlainArgs {
     const int32_t* row_len;
     int heads, kv_heads, dimp, ld_o, ps, window;
     float scale, sink, out_scale;
+    const void* gate;   // null: none
+    int ld_gate;
 };
 // One block per (row, head): 64 keys at a time, a wave per key for the scores, a thread per column for the
 // sums.
@@ -238,7 +398,9 @@ __global__ __launch_bounds__(256) void group_attn_plain_kernel(const PlainArgs a
 #pragma unroll
     for (int c = 0; c < 4; ++c) {
         const int d = tid + 256 * c;
-        if (d < D) static_cast<T*>(a.o)[n * a.ld_o + h * D + d] = act_put<T>(acc[c] * s_stat[0]);
+        if (d >= D) break;
+        const float f = a.gate ? s_stat[0] / (1.f + expf(-act_get<T>(static_cast<const T*>(a.gate)[n * a.ld_gate + h * D + d]))) : s_stat[0];
+        static_cast<T*>(a.o)[n * a.ld_o + h * D + d] = act_put<T>(acc[c] * f);
     }
 }
 
@@ -251,7 +413,17 @@ struct AttnArgs {
     const int32_t *row_len, *list;   // rows of the rows form (null: 0, 1, ..); (first row, rows) of the tiles form
     int heads, kv_heads, ratio, heads_per_tile, head_groups, ld_o, ps, ps_shift, window, nsplit;
     float scale_log2e, sink, out_scale;
+    const uint16_t* gate;      // logistic gates of the outputs, null: none
+    int ld_gate;
 };
+// Four neighbouring outputs, times the logistic function of their gates.
+__device__ __forceinline__ void store_gated(uint16_t* o, f32x4_t v, const uint16_t* gate) {
+    if (gate) {
+        const u32x2_t r = *reinterpret_cast<const u32x2_t*>(gate);
+        v *= f32x4_t{sigmoid_f32(bf16_lo(r.x)), sigmoid_f32(bf16_hi(r.x)), sigmoid_f32(bf16_lo(r.y)), sigmoid_f32(bf16_hi(r.y))};
+    }
+    *reinterpret_cast<u32x2_t*>(o) = u32x2_t{pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3])};
+}
 __device__ __forceinline__ void split_weights(const float* s, float off, float c, float& sum, bf16x8_t& hi_out, bf16x8_t& lo_out) {
     uint32_t hi[4], lo[4];
 #pragma unroll
@@ -413,8 +585,8 @@ __global__ __launch_bounds__(kBlock, 2) void group_rows_kernel(const AttnArgs a)
 #pragma unroll
         for (int w = 0; w < kWaves; ++w) v += *reinterpret_cast<const f32x4_t*>(&sums[(w * 16 + hd) * D + d]);
         if (a.o)
-            *reinterpret_cast<u32x2_t*>(a.o + static_cast<size_t>(n) * a.ld_o + (h0 + hd) * D + d) =
-                u32x2_t{pack_bf16x2(v[0] * inv, v[1] * inv), pack_bf16x2(v[2] * inv, v[3] * inv)};
+            store_gated(a.o + static_cast<size_t>(n) * a.ld_o + (h0 + hd) * D + d, v * inv,
+                        a.gate ? a.gate + static_cast<size_t>(n) * a.ld_gate + (h0 + hd) * D + d : nullptr);
         else
             *reinterpret_cast<f32x4_t*>(a.part_o + (out * a.nsplit + blockIdx.y) * D + d) = v;
     }
@@ -444,8 +616,8 @@ __global__ void group_merge_kernel(const AttnArgs a, uint16_t* __restrict__ o, i
         v += *reinterpret_cast<const f32x4_t*>(po + static_cast<size_t>(s) * D) * w;
     }
     const float inv = a.out_scale * normaliser(l, mx, a.sink);
-    *reinterpret_cast<u32x2_t*>(o + static_cast<size_t>(n) * a.ld_o + h * D + 4 * threadIdx.x) =
-        u32x2_t{pack_bf16x2(v[0] * inv, v[1] * inv), pack_bf16x2(v[2] * inv, v[3] * inv)};
+    store_gated(o + static_cast<size_t>(n) * a.ld_o + h * D + 4 * threadIdx.x, v * inv,
+                a.gate ? a.gate + static_cast<size_t>(n) * a.ld_gate + h * D + 4 * threadIdx.x : nullptr);
 }
 
 // Tiles form: a block takes 64 QT (token, head) pairs of one key head — pair m is token m / heads_per_tile,
@@ -606,10 +778,9 @@ __global__ __launch_bounds__(kBlock, KS > 4 ? 1 : 2) void group_tiles_kernel(con
         const float inv = a.out_scale * normaliser(l, mx[t] * a.scale_log2e, a.sink);
         uint16_t* op = a.o + static_cast<size_t>(my_row[t]) * a.ld_o + my_head[t] * D + 4 * g;
 #pragma unroll
-        for (int dt = 0; dt < DT; ++dt) {
-            const f32x4_t v = acc[t][dt];
-            *reinterpret_cast<u32x2_t*>(op + 16 * dt) = u32x2_t{pack_bf16x2(v[0] * inv, v[1] * inv), pack_bf16x2(v[2] * inv, v[3] * inv)};
-        }
+        for (int dt = 0; dt < DT; ++dt)
+            store_gated(op + 16 * dt, acc[t][dt] * inv,
+                        a.gate ? a.gate + static_cast<size_t>(my_row[t]) * a.ld_gate + my_head[t] * D + 4 * g + 16 * dt : nullptr);
     }
 }
 
@@ -633,6 +804,10 @@ int rows_splits(int num_rows, int heads, int kv_heads, int max_kv_len, int windo
     return ns < 1 ? 1 : static_cast<int>(ns);
 }
 int shift_of(int ps) { return (ps & (ps - 1)) == 0 ? __builtin_ctz(static_cast<unsigned>(ps)) : -1; }
+// gates: none, or rows of all heads; eight-byte pieces where four outputs are stored together
+bool gate_ok(const void* gate, int ld_gate, int heads, int dimp, bool pieces) {
+    return !gate || (ld_gate >= heads * dimp && (!pieces || (ld_gate % 4 == 0 && reinterpret_cast<uintptr_t>(gate) % 8 == 0)));
+}
 bool sizes_ok(int heads, int kv_heads, int dimp, int ld_o, int ps, int window, float sink) {
     return heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && dimp > 0 && ld_o >= heads * dimp && ps > 0 && window >= 0 && sink >= 0.f;
 }
@@ -681,6 +856,29 @@ extern "C" int pie_hip_group_attn_prep(int dtype, const void* fused, int q_off, 
     return launch_status();
 }
 
+extern "C" int pie_hip_group_attn_prep_joint(int dtype, const void* fused, int q_off, int k_off, int v_off, const float* q_norm,
+                                             const float* k_norm, const float* rope_table, int rot_dims, int pairing,
+                                             const int64_t* kv_slots, void* q_out, void* pool, int num_tokens,
+                                             int ld_fused, int heads, int kv_heads, int dim, int vdim, int dimp,
+                                             float eps, void* stream) {
+    if (!fused || !kv_slots || !q_out || !pool || num_tokens <= 0 || heads <= 0 || kv_heads <= 0 || dim <= 0 || vdim <= 0 || dimp < dim ||
+        dimp < vdim || q_off < 0 || k_off < 0 || q_off + heads * dim > ld_fused || k_off + kv_heads * dim > ld_fused ||
+        (v_off < 0 && vdim != dim) || v_off + kv_heads * vdim > ld_fused || rot_dims < 0 || rot_dims % 2 != 0 || rot_dims > dim ||
+        (rot_dims > 0 && !rope_table) || (pairing != PIE_HIP_ROPE_HALF && pairing != PIE_HIP_ROPE_ADJACENT))
+        return PIE_HIP_ERR_INVALID;
+    const bool adjacent = pairing == PIE_HIP_ROPE_ADJACENT;
+    const JointPrepArgs a{fused, q_norm, k_norm, rope_table, kv_slots, q_out, pool, q_off, k_off, v_off, rot_dims, adjacent ? 1 : 0,
+                          ld_fused, heads, kv_heads, dim, vdim, dimp, eps};
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    auto whole = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
+    if (dim % 8 == 0 && vdim % 8 == 0 && dimp % 8 == 0 && (adjacent || rot_dims == 0) && q_off % 8 == 0 && k_off % 8 == 0 &&
+        (v_off < 0 || v_off % 8 == 0) && ld_fused % 8 == 0 && whole(fused) && whole(q_out) && whole(pool) && whole(q_norm) && whole(k_norm))
+        PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL(group_prep_joint_vec_kernel<T>, dim3(num_tokens), dim3(256), 0, s, a));
+    else
+        PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL(group_prep_joint_kernel<T>, dim3(num_tokens), dim3(256), 0, s, a));
+    return launch_status();
+}
+
 extern "C" int pie_hip_group_attn_supported(int dimp) {
     return dimp == 32 || dimp == 64 || dimp == 96 || dimp == 128 || dimp == 192 || dimp == 256;
 }
@@ -696,15 +894,15 @@ extern "C" size_t pie_hip_group_attn_rows_workspace_bytes(int num_rows, int head
 extern "C" int pie_hip_group_attn_rows(const uint16_t* q, const uint16_t* pool, uint16_t* o, const uint32_t* kv_page_indices,
                                        const uint32_t* row_page_begin, const int32_t* row_kv_len, const int32_t* rows,
                                        int num_rows, int heads, int kv_heads, int dimp, int ld_o, int page_size, float scale,
-                                       int window, float sink, float out_scale, int max_kv_len, void* workspace,
-                                       size_t workspace_bytes, void* stream) {
+                                       int window, float sink, float out_scale, const uint16_t* gate, int ld_gate,
+                                       int max_kv_len, void* workspace, size_t workspace_bytes, void* stream) {
     if (!q || !pool || !o || !kv_page_indices || !row_page_begin || !row_kv_len || num_rows <= 0 || max_kv_len <= 0 ||
-        !sizes_ok(heads, kv_heads, dimp, ld_o, page_size, window, sink))
+        !sizes_ok(heads, kv_heads, dimp, ld_o, page_size, window, sink) || !gate_ok(gate, ld_gate, heads, dimp, true))
         return PIE_HIP_ERR_INVALID;
     if (!pie_hip_group_attn_supported(dimp) || ld_o % 4 != 0) return PIE_HIP_ERR_UNSUPPORTED;
     const int ratio = heads / kv_heads, ns = rows_splits(num_rows, heads, kv_heads, max_kv_len, window);
     AttnArgs a{q, pool, o, nullptr, nullptr, kv_page_indices, row_page_begin, row_kv_len, rows, heads, kv_heads, ratio, 16,
-               (ratio + 15) / 16, ld_o, page_size, shift_of(page_size), window, ns, scale * kLog2e, sink, out_scale};
+               (ratio + 15) / 16, ld_o, page_size, shift_of(page_size), window, ns, scale * kLog2e, sink, out_scale, gate, ld_gate};
     if (ns > 1) {
         if (!workspace || workspace_bytes < pie_hip_group_attn_rows_workspace_bytes(num_rows, heads, kv_heads, dimp, max_kv_len, window))
             return PIE_HIP_ERR_INVALID;
@@ -736,14 +934,16 @@ extern "C" int pie_hip_group_attn_tile_rows(int heads, int kv_heads, int half) {
 extern "C" int pie_hip_group_attn_tiles(const uint16_t* q, const uint16_t* pool, uint16_t* o, const uint32_t* kv_page_indices,
                                         const uint32_t* row_page_begin, const int32_t* row_kv_len, const int32_t* tiles,
                                         int num_tiles, int half, int heads, int kv_heads, int dimp, int ld_o, int page_size,
-                                        float scale, int window, float sink, float out_scale, void* stream) {
+                                        float scale, int window, float sink, float out_scale, const uint16_t* gate,
+                                        int ld_gate, void* stream) {
     if (!q || !pool || !o || !kv_page_indices || !row_page_begin || !row_kv_len || !tiles || num_tiles <= 0 ||
-        !sizes_ok(heads, kv_heads, dimp, ld_o, page_size, window, sink))
+        !sizes_ok(heads, kv_heads, dimp, ld_o, page_size, window, sink) || !gate_ok(gate, ld_gate, heads, dimp, true))
         return PIE_HIP_ERR_INVALID;
     if (!pie_hip_group_attn_supported(dimp) || ld_o % 4 != 0) return PIE_HIP_ERR_UNSUPPORTED;
     const int ratio = heads / kv_heads, hpt = ratio >= 64 ? 64 : ratio;
     const AttnArgs a{q, pool, o, nullptr, nullptr, kv_page_indices, row_page_begin, row_kv_len, tiles, heads, kv_heads, ratio, hpt,
-                     (ratio + hpt - 1) / hpt, ld_o, page_size, shift_of(page_size), window, 1, scale * kLog2e, sink, out_scale};
+                     (ratio + hpt - 1) / hpt, ld_o, page_size, shift_of(page_size), window, 1, scale * kLog2e, sink, out_scale,
+                     gate, ld_gate};
     if (static_cast<long long>(num_tiles) * kv_heads * a.head_groups > 0x7FFFFFFF) return PIE_HIP_ERR_UNSUPPORTED;
     hipStream_t s = static_cast<hipStream_t>(stream);
     switch (dimp / 32) {
@@ -761,12 +961,12 @@ extern "C" int pie_hip_group_attn_tiles(const uint16_t* q, const uint16_t* pool,
 extern "C" int pie_hip_group_attn_plain(int dtype, const void* q, const void* pool, void* o, const uint32_t* kv_page_indices,
                                         const uint32_t* row_page_begin, const int32_t* row_kv_len, int num_rows, int heads,
                                         int kv_heads, int dimp, int ld_o, int page_size, float scale, int window, float sink,
-                                        float out_scale, void* stream) {
+                                        float out_scale, const void* gate, int ld_gate, void* stream) {
     if (!q || !pool || !o || !kv_page_indices || !row_page_begin || !row_kv_len || num_rows <= 0 ||
-        !sizes_ok(heads, kv_heads, dimp, ld_o, page_size, window, sink))
+        !sizes_ok(heads, kv_heads, dimp, ld_o, page_size, window, sink) || !gate_ok(gate, ld_gate, heads, dimp, false))
         return PIE_HIP_ERR_INVALID;
     if (dimp > 1024 || heads > 65535) return PIE_HIP_ERR_UNSUPPORTED;
-    const PlainArgs a{q, pool, o, kv_page_indices, row_page_begin, row_kv_len, heads, kv_heads, dimp, ld_o, page_size, window, scale, sink, out_scale};
+    const PlainArgs a{q, pool, o, kv_page_indices, row_page_begin, row_kv_len, heads, kv_heads, dimp, ld_o, page_size, window, scale, sink, out_scale, gate, ld_gate};
     PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL(group_attn_plain_kernel<T>, dim3(num_rows, heads), dim3(256), 0,
                                                   static_cast<hipStream_t>(stream), a));
     return launch_status();

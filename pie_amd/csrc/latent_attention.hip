@@ -29,7 +29,8 @@ __device__ __forceinline__ float rotated_entry(int i, int dims, const float* tab
 }
 
 // The fused down projection's row -> the normed query latent (compact, padded with zeros) and the
-// token's cache row: normed latent, rotated key part.  One block per token.
+// token's cache row: normed latent, rotated key part (`kv_norm` null: only the query latent, the cache rows
+// are another layer's).  One block per token.
 template <class T>
 __global__ __launch_bounds__(256) void latent_prep_kernel(
     const T* __restrict__ fused, const float* __restrict__ q_norm, const float* __restrict__ kv_norm,
@@ -43,7 +44,7 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
     // both sums of squares: waves 0-1 the query latent, waves 2-3 the key/value latent
     const int half = threadIdx.x >> 7, t = threadIdx.x & 127;
     const T* src = half ? fk : fq;
-    const int len = half ? kv_rank : q_rank;
+    const int len = half ? (kv_norm ? kv_rank : 0) : q_rank;
     float local = 0.f;
     for (int i = t; i < len; i += 128) {
         const float v = act_get<T>(src[i]);
@@ -56,6 +57,7 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
     const float inv_k = 1.f / sqrtf((red[2] + red[3]) / static_cast<float>(kv_rank) + eps);
     for (int i = threadIdx.x; i < ld_cq; i += 256)
         cq[n * ld_cq + i] = act_put<T>(i < q_rank ? act_get<T>(fq[i]) * inv_q * q_norm[i] : 0.f);
+    if (!kv_norm) return;
     const int64_t slot = kv_slots[n];
     if (slot < 0) return;
     T* row = pool + static_cast<size_t>(slot) * ld_row;
@@ -81,6 +83,8 @@ struct HeadArgs {
     const float* rope_table;   // (used when rotp > 0 and rot_dims > 0)
     int M, heads, C, K, ld_act, act_stride, ld_y, y_stride;
     int rot_off, rot_dim, rot_dims, rotp;
+    const void* gate;          // logistic gates of the outputs [M, ld_gate], heads C apart (null: none)
+    int ld_gate;
 };
 
 template <class T>
@@ -146,7 +150,13 @@ __global__ __launch_bounds__(kWave) void head_linear_mfma_kernel(const HeadArgs 
         const int m = m0 + 16 * t + l16;
         if (m >= a.M) continue;
         uint16_t* yp = static_cast<uint16_t*>(a.y) + static_cast<size_t>(m) * a.ld_y + static_cast<size_t>(h) * a.y_stride + c0 + 4 * g;
-        *reinterpret_cast<u32x2_t*>(yp) = u32x2_t{pack_bf16x2(acc[t][0], acc[t][1]), pack_bf16x2(acc[t][2], acc[t][3])};
+        f32x4_t v = acc[t];
+        if (a.gate) {
+            const u32x2_t r = *reinterpret_cast<const u32x2_t*>(static_cast<const uint16_t*>(a.gate) + static_cast<size_t>(m) * a.ld_gate +
+                                                                h * a.C + c0 + 4 * g);
+            v *= f32x4_t{sigmoid_f32(bf16_lo(r.x)), sigmoid_f32(bf16_hi(r.x)), sigmoid_f32(bf16_lo(r.y)), sigmoid_f32(bf16_hi(r.y))};
+        }
+        *reinterpret_cast<u32x2_t*>(yp) = u32x2_t{pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3])};
     }
 }
 
@@ -167,6 +177,7 @@ __global__ __launch_bounds__(256) void head_linear_f32_kernel(const HeadArgs a) 
 #pragma unroll
             for (int e = 0; e < 8; ++e) acc = fmaf(row[k + e], w[e], acc);
         }
+        if (a.gate) acc /= 1.f + expf(-static_cast<const float*>(a.gate)[static_cast<size_t>(m) * a.ld_gate + h * a.C + c]);
         dst[c] = acc;
     }
     if (a.rotp > 0) head_rotated_part<float>(a, h, m, m + 1, 0, 1);
@@ -251,10 +262,10 @@ extern "C" int pie_hip_latent_prep(int dtype, const void* fused, const float* q_
                                    const float* rope_table, const int64_t* kv_slots, void* cq, void* pool,
                                    int num_tokens, int ld_fused, int kv_off, int q_rank, int ld_cq, int kv_rank,
                                    int kvp, int rot_dim, int rot_dims, int ld_row, float eps, void* stream) {
-    if (!fused || !q_norm || !kv_norm || !kv_slots || !cq || !pool || num_tokens <= 0 || q_rank <= 0 || kv_rank <= 0 ||
-        (rot_dims > 0 && !rope_table))
+    if (!fused || !q_norm || !cq || num_tokens <= 0 || q_rank <= 0 || kv_rank <= 0 ||
+        (kv_norm && (!kv_slots || !pool || (rot_dims > 0 && !rope_table))))
         return PIE_HIP_ERR_INVALID;
-    if (kv_off < q_rank || kv_off + kv_rank + rot_dim > ld_fused || ld_cq < q_rank || kvp < kv_rank ||
+    if (kv_off < q_rank || q_rank > ld_fused || (kv_norm && kv_off + kv_rank + rot_dim > ld_fused) || ld_cq < q_rank || kvp < kv_rank ||
         ld_row < kvp + rot_dim || rot_dims > rot_dim || rot_dims % 2 != 0)
         return PIE_HIP_ERR_INVALID;
     PIE_ACT_DISPATCH(dtype, T,
@@ -268,7 +279,7 @@ extern "C" int pie_hip_latent_prep(int dtype, const void* fused, const float* q_
 extern "C" int pie_hip_head_linear(int dtype, const void* act, const uint16_t* w_bf16, void* y,
                                    const float* rope_table, int M, int heads, int C, int K, int ld_act,
                                    int act_stride, int ld_y, int y_stride, int rot_off, int rot_dim, int rot_dims,
-                                   int rotp, void* stream) {
+                                   int rotp, const void* gate, int ld_gate, void* stream) {
     if (!act || !w_bf16 || !y || M <= 0 || heads <= 0 || C <= 0 || K <= 0) return PIE_HIP_ERR_INVALID;
     if (C % 16 != 0 || K % 32 != 0 || ld_act % 8 != 0 || act_stride % 8 != 0 || ld_y % 8 != 0 || y_stride % 8 != 0)
         return PIE_HIP_ERR_UNSUPPORTED;
@@ -276,8 +287,9 @@ extern "C" int pie_hip_head_linear(int dtype, const void* act, const uint16_t* w
     if (rotp > 0 && ((rot_dims > 0 && !rope_table) || rot_dims > rot_dim || rot_dims % 2 != 0 || rotp < rot_dim || y_stride < C + rotp ||
                        act_stride < rot_off + rot_dim))
         return PIE_HIP_ERR_INVALID;
+    if (gate && (ld_gate < heads * C || ld_gate % 4 != 0 || reinterpret_cast<uintptr_t>(gate) % 8 != 0)) return PIE_HIP_ERR_INVALID;
     const HeadArgs a{act, w_bf16, y, rope_table, M, heads, C, K, ld_act, act_stride, ld_y, y_stride, rot_off, rot_dim,
-                     rot_dims, rotp};
+                     rot_dims, rotp, gate, ld_gate};
     hipStream_t s = static_cast<hipStream_t>(stream);
     if (heads > 65535) return PIE_HIP_ERR_UNSUPPORTED;
     if (dtype == PIE_HIP_DT_F32) {

@@ -13,7 +13,7 @@
 // Queries sit on the lane%16 axis of both products, so the softmax state is per lane.  A wave skips
 // the steps past its own last query.  Blocks of one head follow each other eight apart in launch
 // order, so a head's keys stay in one XCD's L2; the longest tiles start first.
-#include "common.hip.h"
+#include "act_type.hip.h"
 
 #include <type_traits>
 
@@ -48,6 +48,8 @@ struct LatentPrefillArgs {
     const int32_t* row_len;
     int row0, num_rows, heads, dimp, rotp, rot_dims, ld_o;
     float scale_log2e;
+    const uint16_t* gate;   // logistic gates of the outputs [rows, ld_gate] (null: none)
+    int ld_gate;
 };
 
 template <int KS, int VT, int QT>
@@ -251,8 +253,12 @@ __global__ __launch_bounds__(kBlock, 2) void latent_prefill_kernel(const LatentP
         uint16_t* op = a.o + static_cast<size_t>(a.row0 + t0 + m) * a.ld_o + h * DV + 4 * g;
 #pragma unroll
         for (int dt = 0; dt < DT; ++dt) {
-            const f32x4_t v = acc[t][dt];
-            *reinterpret_cast<u32x2_t*>(op + 16 * dt) = u32x2_t{pack_bf16x2(v[0] * inv, v[1] * inv), pack_bf16x2(v[2] * inv, v[3] * inv)};
+            f32x4_t v = acc[t][dt] * inv;
+            if (a.gate) {
+                const u32x2_t r = *reinterpret_cast<const u32x2_t*>(a.gate + static_cast<size_t>(a.row0 + t0 + m) * a.ld_gate + h * DV + 4 * g + 16 * dt);
+                v *= f32x4_t{sigmoid_f32(bf16_lo(r.x)), sigmoid_f32(bf16_hi(r.x)), sigmoid_f32(bf16_lo(r.y)), sigmoid_f32(bf16_hi(r.y))};
+            }
+            *reinterpret_cast<u32x2_t*>(op + 16 * dt) = u32x2_t{pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3])};
         }
     }
 }
@@ -292,13 +298,14 @@ extern "C" int pie_hip_latent_attn_prefill_supported(int dimp, int rotp, int vdp
 extern "C" int pie_hip_latent_attn_prefill(const uint16_t* q, const uint16_t* kv, const uint16_t* rot, uint16_t* o,
                                            const float* rope_table, const int32_t* row_kv_len, int row0, int num_rows,
                                            int num_keys, int heads, int dimp, int rotp, int rot_dims, int vdp, int ld_o,
-                                           float scale, void* stream) {
+                                           float scale, const uint16_t* gate, int ld_gate, void* stream) {
     if (!q || !kv || !rot || !o || !row_kv_len || row0 < 0 || num_rows <= 0 || num_keys <= 0 || heads <= 0 ||
-        (rot_dims > 0 && !rope_table) || rot_dims > rotp || rot_dims % 2 != 0 || ld_o < heads * vdp)
+        (rot_dims > 0 && !rope_table) || rot_dims > rotp || rot_dims % 2 != 0 || ld_o < heads * vdp ||
+        (gate && (ld_gate < heads * vdp || ld_gate % 4 != 0 || reinterpret_cast<uintptr_t>(gate) % 8 != 0)))
         return PIE_HIP_ERR_INVALID;
     if (!pie_hip_latent_attn_prefill_supported(dimp, rotp, vdp) || ld_o % 8 != 0 || num_rows > 64 * 65535) return PIE_HIP_ERR_UNSUPPORTED;
     const LatentPrefillArgs a{q, kv, rot, o, rope_table, row_kv_len, row0, num_rows, heads, dimp, rotp, rot_dims, ld_o,
-                              scale * 1.4426950408889634f};
+                              scale * 1.4426950408889634f, gate, ld_gate};
     hipStream_t s = static_cast<hipStream_t>(stream);
     const int ks = (dimp + rotp) / 32, vt = vdp / 32;
 #define PIE_PREFILL_CASE(KK, VV) \

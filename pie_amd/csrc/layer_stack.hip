@@ -1,6 +1,7 @@
 // The kernels every layer of a layer-stack model shares: embedding into an fp32 residual stream,
-// the norm-and-add that ends a sublayer, the output norm, the logit finish (scale, soft cap,
-// argmax), the rotation table, and the fp32 linear of the 32-bit compute type.
+// the norm-and-add that ends a sublayer, the join of sublayers that share a norm, the output norm, the
+// logit finish (scale, soft cap, argmax), the rotation table, and the fp32 linears of the 32-bit compute
+// type.
 //
 // The residual stream x is fp32 [rows, ld]; the activations the products read are a copy of it in
 // the compute type, written by the kernel that last changed x, so no product starts with a
@@ -199,6 +200,104 @@ __global__ __launch_bounds__(BLOCK) void residual_norm_kernel(const ResidualArgs
         ar[i] = act_put<T>(a.next_w ? xr[i] * scale * a.next_w[i] : xr[i]);
 }
 
+// Layers whose sublayers read one norm: x takes what they give together — up to two rows, a vector, a
+// token's routes through a mixture, a row of the embedding table — and its compute-type copy is normed for
+// the next layer.  One block per row, as above.
+struct JoinArgs {
+    const void *y, *y2;
+    const float *add, *next_w;
+    PieHipRoutes routes;
+    float* x;
+    const uint32_t* tokens;
+    const uint16_t* table;
+    void* xa;
+    int ldy, ldy2, read_x, vocab, width, ld;
+    float table_scale, eps;
+};
+template <class T>
+__device__ __forceinline__ f32x4_t load4(const T* p) {
+    if constexpr (sizeof(T) == 2) {
+        const u32x2_t r = *reinterpret_cast<const u32x2_t*>(p);
+        return f32x4_t{bf16_lo(r.x), bf16_hi(r.x), bf16_lo(r.y), bf16_hi(r.y)};
+    } else {
+        return *reinterpret_cast<const f32x4_t*>(p);
+    }
+}
+template <class T, int BLOCK>
+__global__ __launch_bounds__(BLOCK) void residual_join_kernel(const JoinArgs a) {
+    __shared__ float red[BLOCK / kWave];
+    const size_t n = blockIdx.x;
+    const T* yr = a.y ? static_cast<const T*>(a.y) + n * a.ldy : nullptr;
+    const T* y2r = a.y2 ? static_cast<const T*>(a.y2) + n * a.ldy2 : nullptr;
+    float* xr = a.x + n * a.ld;
+    T* ar = static_cast<T*>(a.xa) + n * a.ld;
+    const uint16_t* er = nullptr;
+    if (a.tokens) {
+        const uint32_t t = a.tokens[n];
+        er = a.table + static_cast<size_t>(t < static_cast<uint32_t>(a.vocab) ? t : 0) * a.width;
+    }
+    const int K = a.routes.y ? a.routes.top_k : 0;
+    const int32_t* pos = K ? a.routes.pos + n * K : nullptr;
+    const float* weight = K ? a.routes.weight + n * K : nullptr;
+    const T* ry = static_cast<const T*>(a.routes.y);
+    constexpr int kCache = 2048 / BLOCK;   // groups of four
+    const int n4 = a.width % 4 == 0 ? a.width / 4 : 0;
+    const int done = min(n4, kCache * BLOCK) * 4;
+    f32x4_t v[kCache];
+    float local = 0.f;
+#pragma unroll
+    for (int c = 0; c < kCache; ++c) {
+        const int i = 4 * (threadIdx.x + c * BLOCK);
+        if (i >= 4 * n4) break;
+        f32x4_t s = {0.f, 0.f, 0.f, 0.f};   // (the sublayers' sum first, then the stream)
+        if (yr) s += load4(yr + i);
+        if (y2r) s += load4(y2r + i);
+        if (a.add) s += *reinterpret_cast<const f32x4_t*>(a.add + i);
+        for (int k0 = 0; k0 < K; k0 += 4) {   // (four routes requested together)
+            f32x4_t r[4];
+            float w[4];
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                const int k = min(k0 + u, K - 1);
+                w[u] = k0 + u < K ? weight[k] : 0.f;
+                r[u] = load4(ry + static_cast<size_t>(pos[k]) * a.routes.ld + i);
+            }
+#pragma unroll
+            for (int u = 0; u < 4; ++u)
+                if (k0 + u < K) s += r[u] * w[u];
+        }
+        if (er) s += load4(er + i) * a.table_scale;
+        if (a.read_x) s += *reinterpret_cast<const f32x4_t*>(xr + i);
+        v[c] = s;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) local += s[e] * s[e];
+        *reinterpret_cast<f32x4_t*>(xr + i) = s;
+    }
+    for (int i = done + threadIdx.x; i < a.width; i += BLOCK) {
+        float s = 0.f;
+        if (yr) s += act_get<T>(yr[i]);
+        if (y2r) s += act_get<T>(y2r[i]);
+        if (a.add) s += a.add[i];
+        for (int k = 0; k < K; ++k) s += act_get<T>(ry[static_cast<size_t>(pos[k]) * a.routes.ld + i]) * weight[k];
+        if (er) s += bf16_bits_to_f32(er[i]) * a.table_scale;
+        if (a.read_x) s += xr[i];
+        xr[i] = s;
+        local += s * s;
+    }
+    const float scale = a.next_w ? 1.f / sqrtf(block_total(local, red) / static_cast<float>(a.width) + a.eps) : 1.f;
+#pragma unroll
+    for (int c = 0; c < kCache; ++c) {
+        const int i = 4 * (threadIdx.x + c * BLOCK);
+        if (i >= 4 * n4) break;
+        f32x4_t o = v[c];
+        if (a.next_w) o *= *reinterpret_cast<const f32x4_t*>(a.next_w + i) * scale;
+        if constexpr (sizeof(T) == 2) *reinterpret_cast<u32x2_t*>(ar + i) = u32x2_t{pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3])};
+        else *reinterpret_cast<f32x4_t*>(ar + i) = o;
+    }
+    for (int i = done + threadIdx.x; i < a.width; i += BLOCK)   // (a thread reads what it wrote)
+        ar[i] = act_put<T>(a.next_w ? xr[i] * (scale * a.next_w[i]) : xr[i]);
+}
+
 // y = act . W^T with fp32 outputs: the waves of a block share the K of a row tile and NT column tiles, each
 // requesting U of its k-steps at once.
 typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
@@ -343,20 +442,29 @@ __global__ void rotary_table_kernel(const int32_t* __restrict__ positions, const
 // y[M, N] = epilogue(act[M, K] fp32 . W[N, K]^T bf16), fp32 products and sums: 64 x 64 tiles of
 // 16-wide K steps through LDS, 4 x 4 outputs per thread.
 constexpr int kFT = 64, kFK = 16;
+// With `offsets` one of several problems (blockIdx.z): rows offsets[z] .. offsets[z + 1] of y, its weights
+// N * K further, its rows of act as `act_rows` lists them.
 __global__ __launch_bounds__(256) void linear_f32_kernel(const float* __restrict__ act, const uint16_t* __restrict__ w,
-                                                         float* __restrict__ y, int M, int N, int K, int pointwise) {
+                                                         float* __restrict__ y, int M, int N, int K, int pointwise,
+                                                         const int32_t* __restrict__ offsets, const int32_t* __restrict__ act_rows) {
     __shared__ float as[kFK][kFT + 4];
     __shared__ float ws[kFK][kFT + 4];
-    const int n0 = blockIdx.x * kFT, m0 = blockIdx.y * kFT;
+    const int n0 = blockIdx.x * kFT, m0 = blockIdx.y * kFT + (offsets ? offsets[blockIdx.z] : 0);
+    if (offsets) {
+        M = offsets[blockIdx.z + 1];
+        if (m0 >= M) return;
+        w += static_cast<size_t>(blockIdx.z) * N * K;
+    }
     const int tid = threadIdx.x, tx = tid & 15, ty = tid >> 4;
     const int lr = tid >> 2, lk = (tid & 3) * 4;   // the row and the four k-values this thread stages
+    const size_t arow = m0 + lr >= M ? 0 : act_rows ? act_rows[m0 + lr] : m0 + lr;
     float acc[4][4] = {};
     for (int k0 = 0; k0 < K; k0 += kFK) {
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
             const int k = k0 + lk + e;
             const bool kin = k < K;
-            as[lk + e][lr] = kin && m0 + lr < M ? act[static_cast<size_t>(m0 + lr) * K + k] : 0.f;
+            as[lk + e][lr] = kin && m0 + lr < M ? act[arow * K + k] : 0.f;
             ws[lk + e][lr] = kin && n0 + lr < N ? bf16_bits_to_f32(w[static_cast<size_t>(n0 + lr) * K + k]) : 0.f;
         }
         __syncthreads();
@@ -386,6 +494,20 @@ __global__ __launch_bounds__(256) void linear_f32_kernel(const float* __restrict
             else v = epilogue_pointwise<false>(v, pointwise);
             y[static_cast<size_t>(m) * N + n] = v;
         }
+}
+
+// y[m, i] = the gated rule on columns (2i, 2i + 1) of x
+__global__ __launch_bounds__(256) void glu_f32_kernel(const float* __restrict__ x, const PieHipGlu glu, float* __restrict__ y,
+                                                      size_t total, int n) {
+    const size_t idx = static_cast<size_t>(blockIdx.x) * 256 + threadIdx.x;
+    if (idx >= total) return;
+    const size_t m = idx / n, i = idx % n;
+    float g = x[m * 2 * n + 2 * i], u = x[m * 2 * n + 2 * i + 1];
+    if (glu.bias) {
+        g += glu.bias[2 * i];
+        u += glu.bias[2 * i + 1];
+    }
+    y[idx] = glu_value(g, u, glu);
 }
 
 }  // namespace
@@ -435,6 +557,25 @@ extern "C" int pie_hip_residual_norm(int dtype, const void* y, const float* post
         PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL((residual_norm_kernel<T, 1024>), dim3(rows), dim3(1024), 0, s, a));
     else
         PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL((residual_norm_kernel<T, 256>), dim3(rows), dim3(256), 0, s, a));
+    return launch_status();
+}
+
+extern "C" int pie_hip_residual_join(int dtype, const void* y, int ldy, const void* y2, int ldy2, const float* add,
+                                     const PieHipRoutes* routes, float* x, int read_x, const uint32_t* token_ids,
+                                     const uint16_t* table_bf16, int vocab, float table_scale, const float* next_weight,
+                                     void* x_act, int rows, int width, int ld, float eps, void* stream) {
+    if (!x || !x_act || rows <= 0 || width <= 0 || ld < width || (y && ldy < width) || (y2 && ldy2 < width) ||
+        (token_ids && (!table_bf16 || vocab <= 0)) ||
+        (routes && (!routes->y || !routes->pos || !routes->weight || routes->top_k <= 0 || routes->ld < width)))
+        return PIE_HIP_ERR_INVALID;
+    if ((y && ldy % 8 != 0) || (y2 && ldy2 % 8 != 0) || (routes && routes->ld % 8 != 0) || ld % 8 != 0) return PIE_HIP_ERR_UNSUPPORTED;
+    const JoinArgs a{y, y2, add, next_weight, routes ? *routes : PieHipRoutes{}, x, token_ids, table_bf16, x_act, ldy, ldy2,
+                     read_x ? 1 : 0, vocab, width, ld, table_scale, eps};
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    if (width >= 2048 && rows < 512)
+        PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL((residual_join_kernel<T, 1024>), dim3(rows), dim3(1024), 0, s, a));
+    else
+        PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL((residual_join_kernel<T, 256>), dim3(rows), dim3(256), 0, s, a));
     return launch_status();
 }
 
@@ -488,6 +629,26 @@ extern "C" int pie_hip_linear_f32(const float* act, const uint16_t* w_bf16, floa
     const int gy = (M + kFT - 1) / kFT;
     if (gy > 65535) return PIE_HIP_ERR_UNSUPPORTED;
     hipLaunchKernelGGL(linear_f32_kernel, dim3((N + kFT - 1) / kFT, gy), dim3(256), 0, static_cast<hipStream_t>(stream),
-                       act, w_bf16, y, M, N, K, pointwise_code(epilogue));
+                       act, w_bf16, y, M, N, K, pointwise_code(epilogue), nullptr, nullptr);
+    return launch_status();
+}
+
+extern "C" int pie_hip_moe_grouped_linear_f32(const float* act, const int32_t* route_act_rows, const int32_t* expert_offsets,
+                                              int num_experts, int max_rows, const uint16_t* w_bf16, float* y, int N,
+                                              int K, void* stream) {
+    if (!act || !expert_offsets || !w_bf16 || !y || num_experts <= 0 || max_rows <= 0 || N <= 0 || K <= 0) return PIE_HIP_ERR_INVALID;
+    const int gy = (max_rows + kFT - 1) / kFT;
+    if (gy > 65535 || num_experts > 65535) return PIE_HIP_ERR_UNSUPPORTED;
+    hipLaunchKernelGGL(linear_f32_kernel, dim3((N + kFT - 1) / kFT, gy, num_experts), dim3(256), 0, static_cast<hipStream_t>(stream),
+                       act, w_bf16, y, 0, N, K, 0, expert_offsets, route_act_rows);
+    return launch_status();
+}
+
+extern "C" int pie_hip_glu_f32(const float* x, const PieHipGlu* glu, float* y, int M, int n, void* stream) {
+    if (!x || !y || M <= 0 || n <= 0 || !glu_ok(glu, PIE_HIP_EPI_SWIGLU)) return PIE_HIP_ERR_INVALID;
+    const size_t total = static_cast<size_t>(M) * n;
+    if ((total + 255) / 256 > 0x7FFFFFFFull) return PIE_HIP_ERR_UNSUPPORTED;
+    hipLaunchKernelGGL(glu_f32_kernel, dim3(static_cast<unsigned>((total + 255) / 256)), dim3(256), 0,
+                       static_cast<hipStream_t>(stream), x, glu ? *glu : kPlainGlu, y, total, n);
     return launch_status();
 }

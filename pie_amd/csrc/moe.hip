@@ -8,10 +8,15 @@
 //   each sorted route, the sorted position of each (token, k) route).  The reference instead
 //   launches one GEMV per route (driver/cuda/src/model/kimi_forward.cpp:662-714).
 //
+//   pie_hip_moe_route_groups: the same from fp32 logits, with the choice limited to the experts of
+//   a token's best groups and the weights scaled.
+//
 //   pie_hip_moe_combine: out[t] (+)= sum_k w[t, k] * y_route[pos[t, k]] in top-k order, fp32,
 //   one rounding (token_batched_weighted_sum[_add]_bf16_kernel,
 //   driver/cuda/src/kernels/moe_dispatch.cu:152-196).
 #include "common.hip.h"
+
+#include <type_traits>
 
 namespace pie_hip {
 namespace {
@@ -50,12 +55,47 @@ __device__ __forceinline__ void wave_argmax(float& v, int& i) {
     argmax_pick(v, i, __uint_as_float(v32[0]), static_cast<int>(i32[0]), __uint_as_float(v32[1]), static_cast<int>(i32[1]));
 }
 
+// Experts in `count` equal groups of neighbours, of which a token keeps the `keep` whose best expert has
+// the largest probability; weight = p / (sum of the chosen p + 1e-20) * scale.
+struct GroupRule {
+    int count, keep;
+    float scale;
+};
+struct NoGroups {};
+
+// Leaves -2 in place of the probabilities outside the kept groups (one wave; `bits`: kMaxExperts words of LDS
+// that only this wave touches — probabilities are not negative, so they order like their bits).
+__device__ __forceinline__ void mask_groups(float (&p)[kMaxExperts / kWave], int lane, int E, const GroupRule& r, int* bits) {
+    constexpr int kPer = kMaxExperts / kWave;
+    const int size = E / r.count, nper = (E + kWave - 1) / kWave;
+    for (int g = lane; g < r.count; g += kWave) bits[g] = 0;
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");   // (the wave's LDS operations are in order)
+#pragma unroll
+    for (int j = 0; j < kPer; ++j)
+        if (j < nper && lane + kWave * j < E) atomicMax(&bits[(lane + kWave * j) / size], __float_as_int(p[j]));
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+#pragma unroll
+    for (int j = 0; j < kPer; ++j) {
+        const int e = lane + kWave * j;
+        if (j >= nper || e >= E) continue;
+        const int g = e / size;
+        const float mine = __int_as_float(bits[g]);
+        int before = 0;
+        for (int o = 0; o < r.count; ++o) {
+            const float other = __int_as_float(bits[o]);
+            before += other > mine || (other == mine && o < g) ? 1 : 0;
+        }
+        if (before >= r.keep) p[j] = -2.f;
+    }
+}
+
 // One wave: softmax over one token's experts, top-k with exclusion, renormalise (`renorm`; without
 // it the chosen experts keep their softmax probabilities, driver/portable/src/graph_common.cpp:279-283).
 // logit(e) returns expert e's router logit (a bf16 value widened to float).
-template <class Logit>
+template <class Logit, class Groups = NoGroups>
 __device__ __forceinline__ void topk_of_token(Logit logit, int lane, int t, int32_t* __restrict__ topk_idx,
-                                              float* __restrict__ topk_w, int E, int K, int renorm) {
+                                              float* __restrict__ topk_w, int E, int K, int renorm,
+                                              const Groups groups = {}, int* lds = nullptr) {
     // (entries j >= nper hold no expert: the passes below skip them)
     const int nper = (E + kWave - 1) / kWave;
     float p[kPerLane];
@@ -80,6 +120,9 @@ __device__ __forceinline__ void topk_of_token(Logit logit, int lane, int t, int3
     const float inv_z = 1.f / sum;
 #pragma unroll
     for (int j = 0; j < kPerLane; ++j) p[j] = (lane + kWave * j < E) ? p[j] * inv_z : -2.f;
+    constexpr bool kGroups = std::is_same<Groups, GroupRule>::value;
+    if constexpr (kGroups)
+        if (groups.count > 1) mask_groups(p, lane, E, groups, lds);
     float w_sum = 0.f, my_w = 0.f;   // lane k keeps the k-th weight
     int my_e = 0;
     for (int k = 0; k < K; ++k) {
@@ -102,7 +145,8 @@ __device__ __forceinline__ void topk_of_token(Logit logit, int lane, int t, int3
             my_e = bi;
         }
     }
-    const float inv_w = 1.f / w_sum;
+    float inv_w = 1.f / w_sum;
+    if constexpr (kGroups) inv_w = groups.scale / (w_sum + 1e-20f);
     if (lane < K) {
         topk_idx[static_cast<size_t>(t) * K + lane] = my_e;
         topk_w[static_cast<size_t>(t) * K + lane] = renorm ? my_w * inv_w : my_w;
@@ -303,9 +347,9 @@ __global__ __launch_bounds__(kNormRouteThreads) void moe_norm_route_kernel(
 }
 
 // One block: rank of every route inside its expert, expert offsets, sorted positions.
-__global__ __launch_bounds__(kRouteThreads) void moe_sort_kernel(
-    const int32_t* __restrict__ topk_idx, int32_t* __restrict__ expert_offsets,
-    int32_t* __restrict__ route_token, int32_t* __restrict__ route_pos, int N, int E, int K) {
+__device__ __forceinline__ void sort_routes(const int32_t* topk_idx, int32_t* __restrict__ expert_offsets,
+                                            int32_t* __restrict__ route_token, int32_t* __restrict__ route_pos, int N, int E,
+                                            int K) {
     __shared__ int cnt[kMaxExperts];
     __shared__ int base[kMaxExperts + 1];
     const int tid = threadIdx.x, lane = tid & (kWave - 1), wv = tid / kWave;
@@ -345,6 +389,39 @@ __global__ __launch_bounds__(kRouteThreads) void moe_sort_kernel(
         route_pos[r] = pos;
         route_token[pos] = r / K;
     }
+}
+__global__ __launch_bounds__(kRouteThreads) void moe_sort_kernel(
+    const int32_t* __restrict__ topk_idx, int32_t* __restrict__ expert_offsets,
+    int32_t* __restrict__ route_token, int32_t* __restrict__ route_pos, int N, int E, int K) {
+    sort_routes(topk_idx, expert_offsets, route_token, route_pos, N, E, K);
+}
+
+// fp32 logits and groups of experts: one wave per token, four to a block.
+__global__ __launch_bounds__(256) void moe_topk_groups_kernel(const float* __restrict__ logits, int ld,
+                                                              int32_t* __restrict__ topk_idx, float* __restrict__ topk_w, int N,
+                                                              int E, int K, const GroupRule groups) {
+    __shared__ int best[4][kMaxExperts];
+    const int lane = threadIdx.x & (kWave - 1), wv = threadIdx.x / kWave, t = blockIdx.x * 4 + wv;
+    if (t >= N) return;
+    const float* row = logits + static_cast<size_t>(t) * ld;
+    topk_of_token([&](int e) { return row[e]; }, lane, t, topk_idx, topk_w, E, K, 1, groups, best[wv]);
+}
+// The same and the sorted layout in one block, a wave per token.
+constexpr int kFusedTokens = kRouteThreads / kWave;
+__global__ __launch_bounds__(kRouteThreads) void moe_route_groups_kernel(const float* __restrict__ logits, int ld,
+                                                                         int32_t* topk_idx, float* __restrict__ topk_w,
+                                                                         int32_t* __restrict__ expert_offsets,
+                                                                         int32_t* __restrict__ route_token,
+                                                                         int32_t* __restrict__ route_pos, int N, int E, int K,
+                                                                         const GroupRule groups) {
+    __shared__ int best[kFusedTokens][kMaxExperts];
+    const int lane = threadIdx.x & (kWave - 1), t = threadIdx.x / kWave;
+    if (t < N) {
+        const float* row = logits + static_cast<size_t>(t) * ld;
+        topk_of_token([&](int e) { return row[e]; }, lane, t, topk_idx, topk_w, E, K, 1, groups, best[t]);
+    }
+    __syncthreads();   // (a block's stores are seen by its own threads after the barrier)
+    sort_routes(topk_idx, expert_offsets, route_token, route_pos, N, E, K);
 }
 
 __global__ __launch_bounds__(256) void moe_combine_kernel(
@@ -526,6 +603,30 @@ extern "C" int pie_hip_moe_route_opt(const uint16_t* router_logits_bf16, int32_t
                        renormalize ? 1 : 0);
     hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(kRouteThreads), 0, st, topk_idx, expert_offsets,
                        route_token, route_pos, num_tokens, num_experts, top_k);
+    return launch_status();
+}
+
+extern "C" int pie_hip_moe_route_groups(const float* router_logits, int ld_logits, int32_t* topk_idx, float* topk_weight,
+                                        int32_t* expert_offsets, int32_t* route_token, int32_t* route_pos,
+                                        int num_tokens, int num_experts, int top_k, int num_groups, int keep_groups,
+                                        float weight_scale, void* stream) {
+    using namespace pie_hip;
+    if (!router_logits || !topk_idx || !topk_weight || !expert_offsets || !route_token || !route_pos || num_tokens <= 0 ||
+        num_experts <= 0 || ld_logits < num_experts || top_k <= 0 || num_groups <= 0 || num_experts % num_groups != 0 ||
+        keep_groups <= 0 || keep_groups > num_groups || top_k > keep_groups * (num_experts / num_groups))
+        return PIE_HIP_ERR_INVALID;
+    if (num_experts > kMaxExperts || top_k > kWave) return PIE_HIP_ERR_UNSUPPORTED;
+    hipStream_t st = static_cast<hipStream_t>(stream);
+    const GroupRule groups{num_groups, keep_groups, weight_scale};
+    if (num_tokens <= kFusedTokens) {
+        hipLaunchKernelGGL(moe_route_groups_kernel, dim3(1), dim3(kRouteThreads), 0, st, router_logits, ld_logits, topk_idx,
+                           topk_weight, expert_offsets, route_token, route_pos, num_tokens, num_experts, top_k, groups);
+        return launch_status();
+    }
+    hipLaunchKernelGGL(moe_topk_groups_kernel, dim3((num_tokens + 3) / 4), dim3(256), 0, st, router_logits, ld_logits, topk_idx,
+                       topk_weight, num_tokens, num_experts, top_k, groups);
+    hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(kRouteThreads), 0, st, topk_idx, expert_offsets, route_token, route_pos,
+                       num_tokens, num_experts, top_k);
     return launch_status();
 }
 

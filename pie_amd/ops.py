@@ -1129,13 +1129,15 @@ def linear_f32(act: torch.Tensor, w: torch.Tensor, relu2: bool = False, epilogue
 
 
 def head_linear(act: torch.Tensor, w: torch.Tensor, rope_table: Optional[torch.Tensor] = None, rot_dim: int = 0,
-                rot_dims: int = 0, rotp: int = 0) -> torch.Tensor:
-    """act [M, heads, A], w [heads, C, K] -> [M, heads, C + rotp]; the rotated part starts at K."""
+                rot_dims: int = 0, rotp: int = 0, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """act [M, heads, A], w [heads, C, K] -> [M, heads, C + rotp]; the rotated part starts at K.  gate [M, ld]:
+    logistic gates of the outputs."""
     M, heads, A = act.shape
     _, n, k = w.shape
     y = torch.full((M, heads, n + rotp), 3.0, dtype=act.dtype, device=act.device)
     _check(kernels().pie_hip_head_linear(_dt(act), _ptr(act), _ptr(w), _ptr(y), _ptr(rope_table), M, heads, n, k,
-                                         heads * A, A, heads * (n + rotp), n + rotp, k, rot_dim, rot_dims, rotp, _stream()),
+                                         heads * A, A, heads * (n + rotp), n + rotp, k, rot_dim, rot_dims, rotp, _ptr(gate),
+                                         0 if gate is None else gate.shape[1], _stream()),
            "pie_hip_head_linear")
     return y
 
@@ -1174,8 +1176,10 @@ def latent_gather(pool: torch.Tensor, pages: torch.Tensor, num_keys: int, kvp: i
 
 
 def latent_attn_prefill(q: torch.Tensor, kv: torch.Tensor, rot: torch.Tensor, rope_table: Optional[torch.Tensor],
-                        rot_dims: int, row_len: torch.Tensor, dimp: int, scale: float) -> torch.Tensor:
-    """q [rows, heads, dimp + rotp], kv [keys, heads, dimp + vdp], rot [keys, rotp] -> o [rows, heads * vdp]."""
+                        rot_dims: int, row_len: torch.Tensor, dimp: int, scale: float,
+                        gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """q [rows, heads, dimp + rotp], kv [keys, heads, dimp + vdp], rot [keys, rotp] -> o [rows, heads * vdp], times
+    the logistic function of gate [rows, ld]."""
     rows, heads, _ = q.shape
     vdp = kv.shape[2] - dimp
     o = torch.full((rows, heads * vdp), 3.0, dtype=torch.bfloat16, device=q.device)
@@ -1183,7 +1187,8 @@ def latent_attn_prefill(q: torch.Tensor, kv: torch.Tensor, rot: torch.Tensor, ro
         raise KernelError("a row sees more keys than there are")
     _check(kernels().pie_hip_latent_attn_prefill(_ptr(q), _ptr(kv), _ptr(rot), _ptr(o), _ptr(rope_table), _ptr(row_len), 0, rows,
                                                  kv.shape[0], heads, dimp, rot.shape[1], rot_dims, vdp, heads * vdp,
-                                                 C.c_float(scale), _stream()), "pie_hip_latent_attn_prefill")
+                                                 C.c_float(scale), _ptr(gate), 0 if gate is None else gate.shape[1], _stream()),
+           "pie_hip_latent_attn_prefill")
     return o
 
 
@@ -1248,16 +1253,17 @@ def group_attn_prep(fused, q_off, k_off, v_off, q_bias, k_bias, q_norm, k_norm, 
 
 
 def group_attn(form: str, q, pool, page_indices, row_begin, row_len, page_size, scale, window=0, sink=0.0, out_scale=1.0, ld_o=None,
-               rows=None, tiles=None, half: int = 0, max_kv_len: Optional[int] = None) -> torch.Tensor:
-    """q [N, heads, dimp], pool [slots, kv_heads, 2 dimp] -> o [N, ld_o] (heads dimp apart); form "rows" (all rows,
-    or the listed ones), "tiles" or "plain"."""
+               rows=None, tiles=None, half: int = 0, max_kv_len: Optional[int] = None, gate=None) -> torch.Tensor:
+    """q [N, heads, dimp], pool [slots, kv_heads, 2 dimp] -> o [N, ld_o] (heads dimp apart), times the logistic
+    function of gate [N, ld]; form "rows" (all rows, or the listed ones), "tiles" or "plain"."""
     n, heads, dimp = q.shape
     kv_heads = pool.shape[1]
     ld_o = ld_o or heads * dimp
     o = torch.full((n, ld_o), 3.0, dtype=q.dtype, device=q.device)
     longest = int(row_len.max()) if max_kv_len is None else max_kv_len
     lib = kernels()
-    tail = (heads, kv_heads, dimp, ld_o, page_size, C.c_float(scale), window, C.c_float(sink), C.c_float(out_scale))
+    tail = (heads, kv_heads, dimp, ld_o, page_size, C.c_float(scale), window, C.c_float(sink), C.c_float(out_scale), _ptr(gate),
+            0 if gate is None else gate.shape[1])
     head = (_ptr(q), _ptr(pool), _ptr(o), _ptr(page_indices), _ptr(row_begin), _ptr(row_len))
     if form == "plain":
         _check(lib.pie_hip_group_attn_plain(_dt(q), *head, n, *tail, _stream()), "pie_hip_group_attn_plain")
@@ -1275,6 +1281,107 @@ def group_attn(form: str, q, pool, page_indices, row_begin, row_len, page_size, 
 
 def group_attn_tile_rows(heads: int, kv_heads: int, half: int) -> int:
     return int(kernels().pie_hip_group_attn_tile_rows(heads, kv_heads, half))
+
+
+def group_attn_prep_joint(fused, q_off, k_off, v_off, q_norm, k_norm, rope, rot_dims, adjacent: bool, slots, pool, heads, kv_heads, dim,
+                          vdim, dimp, eps) -> torch.Tensor:
+    """As group_attn_prep with norms over whole projections (or none), no biases, values of vdim entries, and
+    neighbours rotated together if `adjacent`."""
+    q = torch.full((fused.shape[0], heads, dimp), 3.0, dtype=fused.dtype, device=fused.device)
+    _check(kernels().pie_hip_group_attn_prep_joint(_dt(fused), _ptr(fused), q_off, k_off, v_off, _ptr(q_norm), _ptr(k_norm), _ptr(rope),
+                                                   rot_dims, int(adjacent), _ptr(slots), _ptr(q), _ptr(pool), fused.shape[0],
+                                                   fused.shape[1], heads, kv_heads, dim, vdim, dimp, C.c_float(eps), _stream()),
+           "pie_hip_group_attn_prep_joint")
+    return q
+
+
+class Glu(C.Structure):
+    """PieHipGlu: biases of the column pairs, clamp, slope of the logistic function, what is added to the second."""
+    _fields_ = [("bias", C.c_void_p), ("limit", C.c_float), ("alpha", C.c_float), ("shift", C.c_float)]
+
+
+def glu(bias=None, limit=float("inf"), alpha=1.0, shift=0.0) -> Glu:
+    return Glu(None if bias is None else bias.data_ptr(), limit, alpha, shift)
+
+
+def linear_glu(form: str, act: torch.Tensor, w: torch.Tensor, rule: Glu) -> torch.Tensor:
+    """The gated rule on act . w^T (rows of w: gate_0, up_0, gate_1, ..) by one of the bf16 products: "gemv", "skinny",
+    "tiled", "splitk", or in fp32 by "f32"."""
+    M, K = act.shape
+    N, lib = w.shape[0], kernels()
+    _dev(w, torch.bfloat16, "w")
+    if form == "f32":
+        x = linear_f32(act, w)
+        y = torch.empty((M, N // 2), dtype=torch.float32, device=act.device)
+        _check(lib.pie_hip_glu_f32(_ptr(x), C.byref(rule), _ptr(y), M, N // 2, _stream()), "pie_hip_glu_f32")
+        return y
+    y = torch.empty((M, N // 2), dtype=torch.bfloat16, device=act.device)
+    head = (3, _ptr(act))
+    if form == "gemv":
+        st = lib.pie_hip_linear_fused_glu(*head, None, C.c_float(0.0), _ptr(w), None, 0, 0, _ptr(y), M, N, K, 0, 1, C.byref(rule), _stream())
+    elif form == "skinny":
+        st = lib.pie_hip_gemm_skinny_glu(*head, _ptr(w), None, 0, 0, _ptr(y), M, N, K, 0, 1, 0, C.byref(rule), _stream())
+    else:
+        lib.pie_hip_gemm_mfma_workspace_bytes.restype = C.c_size_t
+        need = int(lib.pie_hip_gemm_mfma_workspace_bytes(M, N, K)) if form == "splitk" else 0
+        ws = torch.empty(max(need, 16), dtype=torch.uint8, device=act.device)
+        st = lib.pie_hip_gemm_mfma_glu(*head, _ptr(w), None, 0, 0, _ptr(y), M, N, K, 0, 1, C.byref(rule), _ptr(ws) if need else None,
+                                       C.c_size_t(need), _stream())
+    _check(st, f"gated product ({form})")
+    return y
+
+
+def moe_route_groups(logits: torch.Tensor, experts: int, top: int, groups: int, keep: int, scale: float):
+    """fp32 logits [T, ld] -> (experts [T, top], weights [T, top], offsets [experts + 1], token of each sorted route,
+    place of each route [T, top])."""
+    _dev(logits, torch.float32, "logits")
+    T = logits.shape[0]
+    i32 = lambda *shape: torch.empty(shape, dtype=torch.int32, device=logits.device)
+    idx, offsets, token, pos = i32(T, top), i32(experts + 1), i32(T * top), i32(T, top)
+    weight = torch.empty((T, top), dtype=torch.float32, device=logits.device)
+    _check(kernels().pie_hip_moe_route_groups(_ptr(logits), logits.shape[1], _ptr(idx), _ptr(weight), _ptr(offsets), _ptr(token), _ptr(pos),
+                                              T, experts, top, groups, keep, C.c_float(scale), _stream()), "pie_hip_moe_route_groups")
+    return idx, weight, offsets, token, pos
+
+
+def moe_grouped_glu(act: torch.Tensor, rows, offsets: torch.Tensor, w: torch.Tensor, routes: int, rule: Optional[Glu]) -> torch.Tensor:
+    """Rows sorted by expert times w [experts, N, K] (gated if there is a rule); bf16 or fp32 by act's type."""
+    E, N, K = w.shape
+    lib = kernels()
+    if act.dtype == torch.float32:
+        y = torch.empty((routes, N), dtype=torch.float32, device=act.device)
+        _check(lib.pie_hip_moe_grouped_linear_f32(_ptr(act), _ptr(rows), _ptr(offsets), E, routes, _ptr(w), _ptr(y), N, K, _stream()),
+               "pie_hip_moe_grouped_linear_f32")
+        if rule is None:
+            return y
+        z = torch.empty((routes, N // 2), dtype=torch.float32, device=act.device)
+        _check(lib.pie_hip_glu_f32(_ptr(y), C.byref(rule), _ptr(z), routes, N // 2, _stream()), "pie_hip_glu_f32")
+        return z
+    y = torch.empty((routes, N if rule is None else N // 2), dtype=torch.bfloat16, device=act.device)
+    _check(lib.pie_hip_moe_grouped_gemm_glu(3, _ptr(act), _ptr(rows), _ptr(offsets), E, max(1, routes), _ptr(w), C.c_size_t(N * K * 2), None,
+                                            C.c_size_t(0), 0, 0, _ptr(y), N, K, 0 if rule is None else 1, 0,
+                                            None if rule is None else C.byref(rule), _stream()), "pie_hip_moe_grouped_gemm_glu")
+    return y
+
+
+class Routes(C.Structure):
+    """PieHipRoutes: the rows a mixture left, each token's places among them and their weights."""
+    _fields_ = [("y", C.c_void_p), ("pos", C.c_void_p), ("weight", C.c_void_p), ("top_k", C.c_int), ("ld", C.c_int)]
+
+
+def residual_join(x: torch.Tensor, width: int, eps: float, dtype, y=None, y2=None, add=None, routes=None, read_x: bool = True, tokens=None,
+                  table=None, table_scale: float = 1.0, next_weight=None) -> torch.Tensor:
+    """x takes y, y2, add, routes = (rows, places [n, k], weights [n, k]) and table[tokens] * table_scale (each
+    optional) in place; returns x, normed with next_weight if given, in `dtype`."""
+    _dev(x, torch.float32, "x")
+    xa = torch.zeros(x.shape, dtype=dtype, device=x.device)
+    r = None if routes is None else Routes(routes[0].data_ptr(), routes[1].data_ptr(), routes[2].data_ptr(), routes[1].shape[1],
+                                           routes[0].shape[1])
+    _check(kernels().pie_hip_residual_join(_dt(xa), _ptr(y), 0 if y is None else y.shape[1], _ptr(y2), 0 if y2 is None else y2.shape[1],
+                                           _ptr(add), None if r is None else C.byref(r), _ptr(x), int(read_x), _ptr(tokens), _ptr(table),
+                                           0 if table is None else table.shape[0], C.c_float(table_scale), _ptr(next_weight), _ptr(xa),
+                                           x.shape[0], width, x.shape[1], C.c_float(eps), _stream()), "pie_hip_residual_join")
+    return xa
 
 
 class DecayRule(C.Structure):
