@@ -1137,7 +1137,7 @@ def head_linear(act: torch.Tensor, w: torch.Tensor, rope_table: Optional[torch.T
     y = torch.full((M, heads, n + rotp), 3.0, dtype=act.dtype, device=act.device)
     _check(kernels().pie_hip_head_linear(_dt(act), _ptr(act), _ptr(w), _ptr(y), _ptr(rope_table), M, heads, n, k,
                                          heads * A, A, heads * (n + rotp), n + rotp, k, rot_dim, rot_dims, rotp, _ptr(gate),
-                                         0 if gate is None else gate.shape[1], _stream()),
+                                         0 if gate is None else gate.stride(0), _stream()),
            "pie_hip_head_linear")
     return y
 
@@ -1187,7 +1187,7 @@ def latent_attn_prefill(q: torch.Tensor, kv: torch.Tensor, rot: torch.Tensor, ro
         raise KernelError("a row sees more keys than there are")
     _check(kernels().pie_hip_latent_attn_prefill(_ptr(q), _ptr(kv), _ptr(rot), _ptr(o), _ptr(rope_table), _ptr(row_len), 0, rows,
                                                  kv.shape[0], heads, dimp, rot.shape[1], rot_dims, vdp, heads * vdp,
-                                                 C.c_float(scale), _ptr(gate), 0 if gate is None else gate.shape[1], _stream()),
+                                                 C.c_float(scale), _ptr(gate), 0 if gate is None else gate.stride(0), _stream()),
            "pie_hip_latent_attn_prefill")
     return o
 
@@ -1263,7 +1263,7 @@ def group_attn(form: str, q, pool, page_indices, row_begin, row_len, page_size, 
     longest = int(row_len.max()) if max_kv_len is None else max_kv_len
     lib = kernels()
     tail = (heads, kv_heads, dimp, ld_o, page_size, C.c_float(scale), window, C.c_float(sink), C.c_float(out_scale), _ptr(gate),
-            0 if gate is None else gate.shape[1])
+            0 if gate is None else gate.stride(0))
     head = (_ptr(q), _ptr(pool), _ptr(o), _ptr(page_indices), _ptr(row_begin), _ptr(row_len))
     if form == "plain":
         _check(lib.pie_hip_group_attn_plain(_dt(q), *head, n, *tail, _stream()), "pie_hip_group_attn_plain")

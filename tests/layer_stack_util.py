@@ -150,6 +150,109 @@ def lofudra_weights(cfg, seed=0, sharp=1.0):
     return w
 
 
+# ---- Fobanex -----------------------------------------------------------------------------------------
+def moe(experts=9, top=3, ff=40, groups=3, keep=2, limit=1.5, scale=1.7):
+    router = dict(experts=experts, top=top, scale=scale)
+    if groups:
+        router["groups"] = dict(count=groups, keep=keep)
+    return dict(kind="moe", expert=dict(ff=ff, limit=limit), router=router)
+
+
+def normed_attention(heads=6, kv_heads=2, dim=40, vdim=24, rot=None, scale=None, mlp=None):
+    return dict(type="attention", mlp=mlp,
+                mixer=dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, rot=rot or rotary(16), scale=scale if scale is not None else dim ** -0.5))
+
+
+def key_value_attention(heads=6, kv_heads=3, dim=32, rot=None, scale=None, mlp=None):
+    return dict(type="attention_2", mlp=mlp,
+                mixer=dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, rot=rot or rotary(20), scale=scale if scale is not None else dim ** -0.5))
+
+
+def shared_latent(kv_from=None, mlp=None, heads=3, dim=24, rot_dim=8, vdim=20, q_rank=40, kv_rank=48, base=500.0):
+    m = dict(heads=heads, dim=dim, rot_dim=rot_dim, vdim=vdim, q_rank=q_rank, kv_rank=kv_rank, rot=dict(dims=rot_dim, base=base),
+             scale=(dim + rot_dim) ** -0.5)
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return dict(type="latent_attention", mlp=mlp, mixer=m)
+
+
+def fobanex(layers, width=112, vocab=97, eps=1e-4, scale=3.0):
+    return dict(architecture="Fobanex", layers=layers, width=width, vocab=vocab, norm=dict(eps=eps), embedding=dict(scale=scale))
+
+
+# sizes off every padding unit, values wider and narrower than the keys, head counts shared and not, latents read by
+# a neighbour, across other layers and by layers of other head counts, rotations with and without scaling, one
+# expert, one group, all groups, all experts, layers without a feed-forward, sizes of every matrix-core form and of
+# the plain ones
+FOBANEX_CONFIGS = {
+    "quartet": fobanex([shared_latent(mlp=dense(72)), shared_latent(0, moe()), normed_attention(mlp=moe(groups=0, top=2)), key_value_attention(mlp=dense(56))]),
+    "dense": fobanex([normed_attention(mlp=dense(100)), shared_latent(heads=5, dim=40, rot_dim=16, vdim=33, kv_rank=100), key_value_attention(mlp=dense(31)),
+                      shared_latent(1, dense(64), heads=2, dim=16, rot_dim=16, vdim=64, kv_rank=100, q_rank=64)], scale=1.0),
+    "odd": fobanex([key_value_attention(heads=5, kv_heads=5, dim=18, rot=rotary(18), mlp=moe(experts=1, top=1, ff=17, groups=1, keep=1)),
+                    normed_attention(heads=4, kv_heads=1, dim=20, vdim=28, rot=rotary(10, scaling=False)),
+                    shared_latent(heads=2, dim=9, rot_dim=6, vdim=7, q_rank=11, kv_rank=13, mlp=moe(experts=20, top=5, ff=33, groups=4, keep=4, scale=1.0)),
+                    shared_latent(2, heads=3, dim=12, rot_dim=6, vdim=5, q_rank=30, kv_rank=13)], width=75, vocab=130, scale=0.5),
+    "wide": fobanex([normed_attention(heads=20, kv_heads=1, dim=96, vdim=64, rot=rotary(96, 300.0), mlp=moe(experts=40, top=8, ff=64, groups=5, keep=1)),
+                     shared_latent(heads=17, dim=64, rot_dim=32, vdim=64, q_rank=96, kv_rank=128, mlp=dense(200)),
+                     key_value_attention(heads=4, kv_heads=2, dim=192, rot=rotary(64)),
+                     shared_latent(1, moe(experts=6, top=6, ff=128, groups=2, keep=2, limit=0.5), heads=33, dim=32, rot_dim=32, vdim=32, kv_rank=128),
+                     shared_latent(heads=2, dim=32, rot_dim=16, vdim=16, kv_rank=520), shared_latent(1, heads=1, dim=64, rot_dim=32, vdim=40, kv_rank=128)],
+                    width=160, vocab=64),
+    "wider": fobanex([normed_attention(heads=2, kv_heads=1, dim=300, vdim=120, rot=rotary(100), mlp=dense(40)),
+                      key_value_attention(heads=3, kv_heads=3, dim=264, rot=rotary(264, scaling=False)),
+                      normed_attention(heads=3, kv_heads=3, dim=24, vdim=130, rot=rotary(24))], width=128, vocab=80),
+}
+
+
+def fobanex_weights(cfg, seed=0, sharp=1.0):
+    """`sharp` scales the queries (through their norms where they have some): large values make single keys stand out."""
+    rng = np.random.default_rng(seed)
+    w, H = {}, cfg["width"]
+
+    def lin(name, rows, cols, gain=1.0):
+        w[name] = bf16(rng.standard_normal((rows, cols)) * gain / np.sqrt(cols))
+
+    def vec(name, n, lo=0.7, hi=1.3):
+        w[name] = bf16(rng.uniform(lo, hi, n))
+
+    lin("embed", cfg["vocab"], H, np.sqrt(H))
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, mlp = f"l{i}.", layer["mixer"], layer["mlp"]
+        x = p + "mix."
+        vec(p + "norm1", H)
+        if layer["type"] == "latent_attention":
+            lin(x + "dq", m["q_rank"], H)
+            vec(x + "dq.norm", m["q_rank"])
+            lin(x + "uq", m["heads"] * (m["dim"] + m["rot_dim"]), m["q_rank"], sharp)
+            if "kv_from" not in m:
+                lin(x + "dkv", m["kv_rank"] + m["rot_dim"], H)
+                vec(x + "dkv.norm", m["kv_rank"])
+            lin(x + "uk", m["heads"] * m["dim"], m["kv_rank"])
+            lin(x + "uv", m["heads"] * m["vdim"], m["kv_rank"])
+        else:
+            lin(x + "q", m["heads"] * m["dim"], H, sharp if layer["type"] == "attention_2" else 1.0)
+            lin(x + "k", m["kv_heads"] * m["dim"], H)
+            if layer["type"] == "attention":
+                lin(x + "v", m["kv_heads"] * m["vdim"], H)
+                vec(x + "q.norm", m["heads"] * m["dim"], 0.7 * sharp, 1.3 * sharp)
+                vec(x + "k.norm", m["kv_heads"] * m["dim"])
+        if layer["type"] != "attention":
+            lin(x + "g", m["heads"] * m["vdim"], H, 1.5)
+        lin(x + "o", H, m["heads"] * m["vdim"], 2.0)
+        if mlp and mlp["kind"] == "dense":
+            for n, rows, cols in (("gate", mlp["ff"], H), ("up", mlp["ff"], H), ("down", H, mlp["ff"])):
+                lin(p + "mlp." + n, rows, cols, 1.5)
+                w[p + "mlp." + n + ".b"] = bf16(rng.standard_normal(rows) * 0.5)
+        elif mlp:
+            lin(p + "mlp.router", mlp["router"]["experts"], H, 2.0)
+            for e in range(mlp["router"]["experts"]):
+                for n, rows, cols in (("gate", mlp["expert"]["ff"], H), ("up", mlp["expert"]["ff"], H), ("down", H, mlp["expert"]["ff"])):
+                    lin(f"{p}mlp.e{e}.{n}", rows, cols, 1.5)
+    vec("final.norm", H)
+    lin("head", cfg["vocab"], H, 3.0)
+    return w
+
+
 def bf16(a):
     """Rounds to the nearest bf16 value (ties to even); returns float32."""
     u = np.ascontiguousarray(a, np.float32).view(np.uint32)
@@ -263,6 +366,18 @@ def assert_close(got, want, dtype, what=""):
         assert e.max() < F32_TOL, (what, e.max(), int(e.argmax()))
     else:
         assert e.max() < BF16_TOL and (len(e) < 8 or np.median(e) < BF16_MEDIAN), (what, np.median(e), e.max(), int(e.argmax()))
+
+
+def assert_close_routed(got, want, dtype, what=""):
+    """For mixtures: where two experts are all but equally probable, rounding decides between them, at that token and
+    a little at those that read it.  fp32: one position in fifty may be such a one; bf16: one in six."""
+    e = np.sort(position_errors(got, want))
+    assert np.isfinite(e).all(), what
+    n = len(e)
+    if dtype == "float32":
+        assert e[n - 1 - n // 50] < F32_TOL, (what, e[-1])
+    else:
+        assert e[-1] < 1.0 and e[n - 1 - n // 6] < BF16_TOL and (n < 8 or np.median(e) < BF16_MEDIAN), (what, np.median(e), e[-5:])
 
 
 def engine(directory, dtype, **kw):
