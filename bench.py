@@ -346,17 +346,22 @@ def other_configs_extra(drvmod):
 # --layer-stack: layers of the layer-stack models beside bf16 llama-type layers of the same width and
 # feed-forward width.  Varasun: latent attention, one channel-delta layer in three, squared-ReLU
 # feed-forward.  Lofudra: mLSTM, Mamba-2, windowed attention beside retention in turn, GELU feed-forward.
+# Fobanex: gated latent attention (the second layer on the first one's latents), attention normed over whole
+# projections, attention on its keys; two dense layers and four mixtures.  "moe" is the qwen3_moe-type model,
+# a mixture of the same experts in every layer.
 STACK_SIZES = {
     "width4096": dict(width=4096, heads=32, dim=128, rot_dim=64, vdim=128, q_rank=1536, kv_rank=512, ff=14336,
                       kv_heads=8, vocab=32000, layers=6, window=1024,
                       mlstm=dict(heads=8, dim=256, vdim=512, gate_cap=15.0),
                       mamba2=dict(heads=128, vdim=64, state=128, groups=8, conv=4, norm_groups=8),
-                      retention=dict(heads=16, dim=128, vdim=256)),
+                      retention=dict(heads=16, dim=128, vdim=256),
+                      experts=64, top=8, expert_ff=1536, groups=8, keep=4),
     "width2048": dict(width=2048, heads=16, dim=128, rot_dim=64, vdim=128, q_rank=768, kv_rank=512, ff=8192,
                       kv_heads=4, vocab=32000, layers=6, window=4096,
                       mlstm=dict(heads=8, dim=128, vdim=256, gate_cap=15.0),
                       mamba2=dict(heads=64, vdim=64, state=128, groups=4, conv=4, norm_groups=4),
-                      retention=dict(heads=8, dim=128, vdim=256)),
+                      retention=dict(heads=8, dim=128, vdim=256),
+                      experts=64, top=8, expert_ff=768, groups=8, keep=4),
 }
 
 
@@ -382,12 +387,31 @@ def lofudra_config(z: dict) -> dict:
     return dict(architecture="Lofudra", layers=layers, width=z["width"], vocab=z["vocab"], norm=dict(eps=1e-6))
 
 
-STACKS = {"varasun": varasun_config, "lofudra": lofudra_config}
+def fobanex_config(z: dict) -> dict:
+    def rot(base):
+        return dict(dims=z["rot_dim"], base=base, scaling=dict(factor=4.0, original=4096, fast=24.0, slow=2.0))
+
+    latent = dict(heads=z["heads"], dim=z["dim"], rot_dim=z["rot_dim"], vdim=z["vdim"], q_rank=z["q_rank"],
+                  kv_rank=z["kv_rank"], rot=dict(dims=z["rot_dim"], base=10000.0), scale=(z["dim"] + z["rot_dim"]) ** -0.5)
+    heads = dict(heads=z["heads"], kv_heads=z["kv_heads"], dim=z["dim"], vdim=z["dim"], scale=z["dim"] ** -0.5)
+    kinds = [("latent_attention", latent), ("latent_attention", dict(latent, kv_from=0)),
+             ("attention", dict(heads, rot=rot(500000.0))), ("attention", dict(heads, rot=rot(500000.0))),
+             ("attention_2", dict(heads, rot=rot(10000.0))), ("attention_2", dict(heads, rot=rot(10000.0)))]
+    dense = dict(kind="dense", ff=z["ff"])
+    moe = dict(kind="moe", expert=dict(ff=z["expert_ff"], limit=7.0),
+               router=dict(experts=z["experts"], top=z["top"], scale=1.5, groups=dict(count=z["groups"], keep=z["keep"])))
+    layers = [dict(type=t, mixer=m, mlp=dense if l % 5 == 0 else moe) for l, (t, m) in enumerate(kinds[:z["layers"]])]
+    return dict(architecture="Fobanex", layers=layers, width=z["width"], vocab=z["vocab"], norm=dict(eps=1e-6),
+                embedding=dict(scale=z["width"] ** 0.5))
+
+
+STACKS = {"varasun": varasun_config, "lofudra": lofudra_config, "fobanex": fobanex_config}
+STACK_SIDES = [*STACKS, "llama", "moe"]
 
 
 def stack_workload(args):
-    """Prefill and decode throughput of the layer stacks above and of the llama-type model of equal
-    size, both through the driver boundary on random bf16 weights."""
+    """Prefill and decode throughput of the layer stacks above and of the llama-type and qwen3_moe-type models of
+    equal size, all through the driver boundary on random bf16 weights."""
     import tempfile
 
     from pie_amd import driver as drvmod
@@ -410,10 +434,13 @@ def stack_workload(args):
                 "llama": dict(arch="llama3", hidden=z["width"], layers=z["layers"], q_heads=z["heads"],
                               kv_heads=z["kv_heads"], head_dim=z["dim"], intermediate=z["ff"], vocab=z["vocab"],
                               quant="bf16"),
+                "moe": dict(arch="qwen3_moe", hidden=z["width"], layers=z["layers"], q_heads=z["heads"],
+                            kv_heads=z["kv_heads"], head_dim=z["dim"], intermediate=z["expert_ff"], vocab=z["vocab"],
+                            num_experts=z["experts"], top_k=z["top"], expert_intermediate=z["expert_ff"], quant="bf16"),
             }
             res = {}
             for which, model in models.items():
-                if args.layer_stack_only and which != args.layer_stack_only:
+                if args.layer_stack_only and which not in args.layer_stack_only.split(","):
                     continue
                 drv = drvmod.Driver(toml(model, page, pages, 2048, 64))
                 try:
@@ -428,6 +455,7 @@ def stack_workload(args):
                         wall = tm["decode_wall_us"] * 1e-6 / tm["decode_steps"]
                         r[f"decode_batch{batch}"] = dict(tokens_per_s=round(batch / wall, 1), ms_per_step=round(wall * 1e3, 4))
                     res[which] = r
+                    print(f"# {name} {which}: {json.dumps(r)}", file=sys.stderr, flush=True)
                 finally:
                     drv.close()
             out[name] = dict(sizes=z, **res)
@@ -609,11 +637,13 @@ def main():
                     help="only launch what a `rocprofv3 --pmc FETCH_SIZE|WRITE_SIZE` run needs: a "
                          "256 MiB device copy (the counter's scale) and the four int4 GEMV shapes")
     ap.add_argument("--layer-stack", default=None, choices=["all", *STACK_SIZES],
-                    help="measure layer-stack models (prefill and decode at batch 1, 16, 64) beside the llama-type "
-                         "model of equal size instead of the headline workload")
-    ap.add_argument("--layer-stack-only", default=None, choices=[*STACKS, "llama"],
-                    help="with --layer-stack: only this side (for profiles)")
+                    help="measure layer-stack models (prefill and decode at batch 1, 16, 64) beside the llama-type and "
+                         "qwen3_moe-type models of equal size instead of the headline workload")
+    ap.add_argument("--layer-stack-only", default=None, metavar="SIDE[,SIDE]",
+                    help=f"with --layer-stack: only these sides ({', '.join(STACK_SIDES)})")
     args = ap.parse_args()
+    if args.layer_stack_only and not set(args.layer_stack_only.split(",")) <= set(STACK_SIDES):
+        ap.error(f"--layer-stack-only: sides are {', '.join(STACK_SIDES)}")
     if args.gpus != 1:
         print("bench.py: this driver path is built and measured on one GPU; "
               f"--gpus {args.gpus} is not supported (run with --gpus 1).", file=sys.stderr)

@@ -288,6 +288,13 @@ int pie_hip_moe_grouped_gemm_glu(int format, const uint16_t* act_bf16, const int
                                  size_t scale_stride_bytes, int scale_is_bf16, int group_size,
                                  uint16_t* y_bf16, int N, int K, int swiglu, int tiled,
                                  const PieHipGlu* glu, void* stream);
+/* bf16 experts with many routes each (a prompt's tokens): the tiled GEMM's blocks of block_rows (64, 128, 256; 0:
+ * chosen from the routes per expert) routes of one expert, whose weights are read once per block.  num_routes =
+ * expert_offsets[num_experts].  K % 64 == 0, tile-major weights need N % 16 == 0. */
+int pie_hip_moe_grouped_gemm_mfma(const uint16_t* act_bf16, const int32_t* route_act_rows, const int32_t* expert_offsets,
+                                  int num_experts, int num_routes, const void* weights_bf16, size_t weight_stride_bytes,
+                                  uint16_t* y_bf16, int N, int K, int epilogue, int tiled, const PieHipGlu* glu,
+                                  int block_rows, void* stream);
 
 /*
  * Tile-major weight layout for the skinny and grouped GEMMs.  The 16 bytes that lane (j, q) of a

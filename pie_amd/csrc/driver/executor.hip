@@ -570,11 +570,20 @@ void Executor::moe_block(const LayerWeights& w, int N, const uint16_t* next_norm
     auto grouped = tiled ? pie_hip_moe_grouped_gemm_tiled : pie_hip_moe_grouped_gemm;
     auto wptr = [&](const Linear& l) { return tiled ? l.data_tiled : l.data; };
     auto sptr = [&](const Linear& l) { return tiled && l.scale_tiled ? l.scale_tiled : l.scale; };
-    PIE_KERNEL(grouped(fmt, xn_, moe_route_token_, moe_offsets_, E, hint, wptr(w.wgu),
-                       w.wgu.data_bytes() / E, sptr(w.wgu), w.wgu.scale_bytes() / E, sbf, w.wgu.group,
-                       act_, 2 * Ie, H, 1, s));
-    PIE_KERNEL(grouped(fmt, act_, nullptr, moe_offsets_, E, hint, wptr(w.wdown), w.wdown.data_bytes() / E,
-                       sptr(w.wdown), w.wdown.scale_bytes() / E, sbf, w.wdown.group, moe_y_, H, Ie, 0, s));
+    if (w.wgu.kind == Quant::Bf16 && w.wdown.kind == Quant::Bf16 && H % 64 == 0 && Ie % 64 == 0 && grouped_in_blocks(N * K, E)) {
+        auto blocks = [&](const Linear& l, const uint16_t* act, const int32_t* rows, uint16_t* y, int rows_out, int cols, int epilogue) {
+            PIE_KERNEL(pie_hip_moe_grouped_gemm_mfma(act, rows, moe_offsets_, E, N * K, wptr(l), l.data_bytes() / E, y, rows_out, cols,
+                                                     epilogue, tiled ? 1 : 0, nullptr, 0, s));
+        };
+        blocks(w.wgu, xn_, moe_route_token_, act_, 2 * Ie, H, PIE_HIP_EPI_SWIGLU);
+        blocks(w.wdown, act_, nullptr, moe_y_, H, Ie, PIE_HIP_EPI_NONE);
+    } else {
+        PIE_KERNEL(grouped(fmt, xn_, moe_route_token_, moe_offsets_, E, hint, wptr(w.wgu),
+                           w.wgu.data_bytes() / E, sptr(w.wgu), w.wgu.scale_bytes() / E, sbf, w.wgu.group,
+                           act_, 2 * Ie, H, 1, s));
+        PIE_KERNEL(grouped(fmt, act_, nullptr, moe_offsets_, E, hint, wptr(w.wdown), w.wdown.data_bytes() / E,
+                           sptr(w.wdown), w.wdown.scale_bytes() / E, sbf, w.wdown.group, moe_y_, H, Ie, 0, s));
+    }
     // with the next layer's attention norm riding along when that layer takes its rows normalised
     int combined = PIE_HIP_ERR_UNSUPPORTED;
     if (next_norm)

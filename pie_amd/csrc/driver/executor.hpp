@@ -142,6 +142,9 @@ class Executor {
     void enqueue_samplers();
     void collect_samplers(const BatchPlan& plan, SampleOutputs& out);
     void moe_block(const LayerWeights& w, int N, const uint16_t* next_norm, hipStream_t s);
+    // bf16 experts: from this many routes per expert on, blocks of routes beat passes of 16 over an expert's weights
+    static bool grouped_in_blocks(long long routes, int experts) { return routes >= kBlockRoutes * static_cast<long long>(experts); }
+    static constexpr int kBlockRoutes = 12;
     static constexpr int kFusedRouteRows = 256;   // batches up to this size take pie_hip_moe_norm_route
     static constexpr size_t kMergeProjMaxBytes = 64 * 1024;   // partial results a merging output projection reads per block
     bool xn_holds_next_norm_ = false;             // (while a forward is being enqueued) xn_ = the coming layer's normalised rows

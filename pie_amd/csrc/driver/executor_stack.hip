@@ -362,7 +362,15 @@ void Executor::stack_mixture(const StackLayer& w, int N) {
         return;
     }
     const int hint = std::max(1, std::min(N, 2 * ((N * e.top + e.experts - 1) / e.experts)));
+    const bool blocks = grouped_in_blocks(N * e.top, e.experts);
     auto grouped = [&](const Linear& l, const void* act, const int32_t* rows, void* y, int epilogue, const PieHipGlu* rule) {
+        if (blocks) {
+            PIE_KERNEL(pie_hip_moe_grouped_gemm_mfma(static_cast<const uint16_t*>(act), rows, stack_.route_offsets, e.experts, N * e.top,
+                                                     l.data_tiled ? l.data_tiled : l.data, l.data_bytes() / e.experts,
+                                                     static_cast<uint16_t*>(y), l.N / e.experts, l.K, epilogue, l.data_tiled ? 1 : 0, rule, 0,
+                                                     stream_));
+            return;
+        }
         PIE_KERNEL(pie_hip_moe_grouped_gemm_glu(PIE_HIP_FMT_BF16, static_cast<const uint16_t*>(act), rows, stack_.route_offsets, e.experts,
                                                 hint, l.data_tiled ? l.data_tiled : l.data, l.data_bytes() / e.experts, nullptr, 0, 0, 0,
                                                 static_cast<uint16_t*>(y), l.N / e.experts, l.K, epilogue, l.data_tiled ? 1 : 0, rule,

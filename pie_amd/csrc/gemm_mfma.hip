@@ -26,6 +26,10 @@
 //   * activations are the MFMA A operand, weights the B operand: an accumulator lane holds one
 //     weight row n (column of y) for four consecutive activation rows, so row scales are
 //     per-lane scalars and the SwiGLU partner (gate_i, up_i interleaved) is the neighbour lane.
+// Grouped form (the experts of a mixture, bf16): a block finds its problem from the route offsets — row
+// blocks are numbered through all problems, no problem's rows share a block with another's — and gathers
+// its activation rows; weights may be in the tile-major order of the skinny kernels, of which a transfer
+// takes the same 16-byte granules from other places.
 #include "common.hip.h"
 
 #include <type_traits>
@@ -53,7 +57,41 @@ struct GemmArgs {
     int pointwise;        // PIE_HIP_EPI_RELU2 and above: applied to the sum (0: nothing)
     PieHipGlu glu = kPlainGlu;   // swiglu
     float* partial;   // split-K: fp32 [gridDim.z][M][N] partial sums (row scale applied), else null
+    // grouped: rows offsets[p] .. offsets[p + 1] of y belong to problem p (of `problems`), whose weights start
+    // w_stride bytes after the one before; act_rows: the activation row of each (null: the same row)
+    const int32_t* offsets;
+    const int32_t* act_rows;
+    size_t w_stride;
+    int problems, tiled;
 };
+
+// The problem and the rows [m0, m1) of block row `t` when problems are cut into blocks of `rows` rows one after
+// another; false behind the last.  Every lane of the wave calls it and gets the same answer.
+__device__ __forceinline__ bool grouped_place(const int32_t* __restrict__ offsets, int problems, int rows, int t, int lane,
+                                              int& p, int& m0, int& m1) {
+    int before = 0;
+    for (int base = 0; base < problems; base += kWave) {
+        const int e = base + lane;
+        const int lo = e < problems ? offsets[e] : 0, hi = e < problems ? offsets[e + 1] : 0;
+        const int n = (hi - lo + rows - 1) / rows;
+        int sum = n;
+#pragma unroll
+        for (int d = 1; d < kWave; d <<= 1) {
+            const int o = __shfl_up(sum, d);
+            if (lane >= d) sum += o;
+        }
+        const unsigned long long past = __ballot(before + sum > t);
+        if (past) {
+            const int at = __ffsll(past) - 1;
+            p = __builtin_amdgcn_readfirstlane(base + at);
+            m0 = __builtin_amdgcn_readfirstlane(__shfl(lo, at) + (t - before - __shfl(sum - n, at)) * rows);
+            m1 = __builtin_amdgcn_readfirstlane(__shfl(hi, at));
+            return true;
+        }
+        before += __shfl(sum, kWave - 1);
+    }
+    return false;
+}
 
 __device__ __forceinline__ uint32_t pack_trunc(float lo, float hi) {
     return __builtin_amdgcn_perm(__float_as_uint(hi), __float_as_uint(lo), 0x07060302u);
@@ -194,10 +232,11 @@ struct GBf16 {
 // MT: 16-row activation tiles per wave (4: 64 x 64 per wave; 2: 32 x 64 for small batches).
 // NW: waves per block, 4 (2 x 2 quadrants) or 8 (4 x 2: two waves per SIMD, so one wave's
 // barrier and operand-read waits sit in the other's MFMAs).
-template <class Base, int MT_, int NW_ = 4>
+template <class Base, int MT_, int NW_ = 4, bool GROUPED = false>
 struct Shape {
     using Format = Base;
     static constexpr int kMT = MT_, kNW = NW_;
+    static constexpr bool kGrouped = GROUPED;
 };
 
 template <class SH>
@@ -215,8 +254,13 @@ __global__ __launch_bounds__(SH::kNW* kWave) void gemm_mfma_kernel(const GemmArg
     const int wv = __builtin_amdgcn_readfirstlane(tid / kWave);
     const int j = lane & 15, q = lane >> 4;
     const int wm = wv >> 1, wn = wv & 1;
-    const int M = a.M, N = a.N, K = a.K;
-    const int n0 = blockIdx.x * BN, m0 = blockIdx.y * BMv;
+    const int N = a.N, K = a.K;
+    const int n0 = blockIdx.x * BN;
+    int M = a.M, m0 = blockIdx.y * BMv, problem = 0;
+    if constexpr (SH::kGrouped)
+        if (!grouped_place(a.offsets, a.problems, BMv, blockIdx.y, lane, problem, m0, M)) return;
+    const unsigned char* w = a.w + (SH::kGrouped ? static_cast<size_t>(problem) * a.w_stride : 0);
+    const int wstep = SH::kGrouped && a.tiled ? 16 : 1;   // values between a granule and the one a k-value further, per k-value
     // split-K: block z owns the K steps [kbeg, kbeg + nk) (the host makes every share non-empty)
     const int nk_all = K / BK;
     const int per_split = (nk_all + static_cast<int>(gridDim.z) - 1) / static_cast<int>(gridDim.z);
@@ -232,9 +276,19 @@ __global__ __launch_bounds__(SH::kNW* kWave) void gemm_mfma_kernel(const GemmArg
     for (int u = 0; u < (MT > 4 ? MT : 4); ++u) {
         const int r = (u * NW + wv) * 8 + (lane >> 3);
         const int g = (lane & 7) ^ ((r >> 1) & 7);
-        if (u < MT) aptr[u] = a.act + static_cast<size_t>(min(m0 + r, M - 1)) * K + g * 8;
-        if (u < TB)
-            bptr[u] = reinterpret_cast<const uint16_t*>(a.w) + static_cast<size_t>(min(n0 + r, N - 1)) * K + g * 8;
+        if (u < MT) {
+            int row = min(m0 + r, M - 1);
+            if (SH::kGrouped && a.act_rows) row = a.act_rows[row];
+            aptr[u] = a.act + static_cast<size_t>(row) * K + g * 8;
+        }
+        if (u < TB) {
+            const int n = min(n0 + r, N - 1);
+            // (tile-major: granule g of a row in 32-value blocks of [k / 8 % 4][16 rows])
+            const size_t at = SH::kGrouped && a.tiled
+                                  ? ((static_cast<size_t>(n >> 4) * (K >> 5) + (g >> 2)) * 64 + (g & 3) * 16 + (n & 15)) * 8
+                                  : static_cast<size_t>(n) * K + g * 8;
+            bptr[u] = reinterpret_cast<const uint16_t*>(w) + at;
+        }
     }
     auto issue_direct = [&](int kt) {
         const int k0 = (kbeg + min(kt, nk - 1)) * BK;
@@ -242,7 +296,7 @@ __global__ __launch_bounds__(SH::kNW* kWave) void gemm_mfma_kernel(const GemmArg
         if (F::kDirect) {
 #pragma unroll
             for (int u = 0; u < TB; ++u)
-                __builtin_amdgcn_global_load_lds(bptr[u] + k0, PIE_LDS_PTR(lds_b + st * kTileVecs + (u * NW + wv) * 64), 16, 0, 0);
+                __builtin_amdgcn_global_load_lds(bptr[u] + static_cast<size_t>(k0) * wstep, PIE_LDS_PTR(lds_b + st * kTileVecs + (u * NW + wv) * 64), 16, 0, 0);
         }
 #pragma unroll
         for (int u = 0; u < MT; ++u)
@@ -545,8 +599,61 @@ int gemm_entry(int format, const uint16_t* act_bf16, const void* weight, const v
         default: return PIE_HIP_ERR_INVALID;
     }
 }
+
+template <int MT>
+int launch_grouped(const GemmArgs& a, int routes, hipStream_t stream) {
+    constexpr int NW = 8, BMv = 16 * MT * (NW / 2);
+    using SH = Shape<GBf16, MT, NW, true>;
+    constexpr size_t smem = static_cast<size_t>(kStages) * (BMv * (BK / 8) + kTileVecs) * sizeof(u32x4_t);
+    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&gemm_mfma_kernel<SH>),
+                                                       hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(smem));
+    if (attr != hipSuccess) return PIE_HIP_ERR_LAUNCH;
+    // (no cut of the routes into problems makes more row blocks)
+    const int blocks = routes / BMv + (routes < a.problems ? routes : a.problems);
+    if (blocks > 65535) return PIE_HIP_ERR_UNSUPPORTED;
+    hipLaunchKernelGGL((gemm_mfma_kernel<SH>), dim3((a.N + BN - 1) / BN, blocks), dim3(NW * kWave), smem, stream, a);
+    return launch_status();
+}
 }  // namespace
 }  // namespace pie_hip
+
+extern "C" int pie_hip_moe_grouped_gemm_mfma(const uint16_t* act_bf16, const int32_t* route_act_rows, const int32_t* expert_offsets,
+                                             int num_experts, int num_routes, const void* weights_bf16, size_t weight_stride_bytes,
+                                             uint16_t* y_bf16, int N, int K, int epilogue, int tiled, const PieHipGlu* glu,
+                                             int block_rows, void* stream) {
+    using namespace pie_hip;
+    if (!act_bf16 || !expert_offsets || !weights_bf16 || !y_bf16 || num_experts <= 0 || num_routes <= 0 || N <= 0 || K <= 0 ||
+        !glu_ok(glu, epilogue))
+        return PIE_HIP_ERR_INVALID;
+    GemmArgs a{};
+    a.swiglu = epilogue == PIE_HIP_EPI_SWIGLU ? 1 : 0;
+    a.pointwise = pointwise_code(epilogue);
+    if (a.swiglu && N % 2 != 0) return PIE_HIP_ERR_INVALID;
+    if (K % BK != 0 || (tiled && N % 16 != 0)) return PIE_HIP_ERR_UNSUPPORTED;
+    a.act = act_bf16;
+    a.act_rows = route_act_rows;
+    a.offsets = expert_offsets;
+    a.problems = num_experts;
+    a.w = static_cast<const unsigned char*>(weights_bf16);
+    a.w_stride = weight_stride_bytes;
+    a.tiled = tiled ? 1 : 0;
+    a.y = y_bf16;
+    a.M = num_routes;
+    a.N = N;
+    a.K = K;
+    if (glu) a.glu = *glu;
+    // (64 experts of 3072 x 4096, routes per expert 16 / 64 / 256: 295 / 367 / 985 us in blocks of 64, 310 / 324 / 746 of
+    // 128, 377 / 412 / 679 of 256; passes of 16 rows: 390 / 1161 / 4300)
+    const int each = num_routes / num_experts;
+    if (block_rows == 0) block_rows = each < 48 ? 64 : each < 112 ? 128 : 256;
+    hipStream_t st = static_cast<hipStream_t>(stream);
+    switch (block_rows) {
+        case 64: return launch_grouped<1>(a, num_routes, st);
+        case 128: return launch_grouped<2>(a, num_routes, st);
+        case 256: return launch_grouped<4>(a, num_routes, st);
+        default: return PIE_HIP_ERR_UNSUPPORTED;
+    }
+}
 
 extern "C" int pie_hip_gemm_mfma(int format, const uint16_t* act_bf16, const void* weight,
                                  const void* scale, int scale_is_bf16, int group_size,

@@ -214,18 +214,25 @@ struct JoinArgs {
     int ldy, ldy2, read_x, vocab, width, ld;
     float table_scale, eps;
 };
+// Eight values at a time, still in the compute type.
 template <class T>
-__device__ __forceinline__ f32x4_t load4(const T* p) {
-    if constexpr (sizeof(T) == 2) {
-        const u32x2_t r = *reinterpret_cast<const u32x2_t*>(p);
-        return f32x4_t{bf16_lo(r.x), bf16_hi(r.x), bf16_lo(r.y), bf16_hi(r.y)};
-    } else {
-        return *reinterpret_cast<const f32x4_t*>(p);
+struct Eight {
+    u32x4_t r[sizeof(T) / 2];
+    __device__ __forceinline__ void load(const T* p) {
+#pragma unroll
+        for (int h = 0; h < static_cast<int>(sizeof(T)) / 2; ++h) r[h] = reinterpret_cast<const u32x4_t*>(p)[h];
     }
-}
+    __device__ __forceinline__ float get(int e) const {
+        if constexpr (sizeof(T) == 2) return e & 1 ? bf16_hi(r[0][e / 2]) : bf16_lo(r[0][e / 2]);
+        else return __uint_as_float(r[e / 4][e % 4]);
+    }
+};
+constexpr int kJoinRoutes = 64;   // places and weights of a token's first routes wait in LDS
 template <class T, int BLOCK>
 __global__ __launch_bounds__(BLOCK) void residual_join_kernel(const JoinArgs a) {
     __shared__ float red[BLOCK / kWave];
+    __shared__ int pos[kJoinRoutes];
+    __shared__ float weight[kJoinRoutes];
     const size_t n = blockIdx.x;
     const T* yr = a.y ? static_cast<const T*>(a.y) + n * a.ldy : nullptr;
     const T* y2r = a.y2 ? static_cast<const T*>(a.y2) + n * a.ldy2 : nullptr;
@@ -237,41 +244,67 @@ __global__ __launch_bounds__(BLOCK) void residual_join_kernel(const JoinArgs a) 
         er = a.table + static_cast<size_t>(t < static_cast<uint32_t>(a.vocab) ? t : 0) * a.width;
     }
     const int K = a.routes.y ? a.routes.top_k : 0;
-    const int32_t* pos = K ? a.routes.pos + n * K : nullptr;
-    const float* weight = K ? a.routes.weight + n * K : nullptr;
     const T* ry = static_cast<const T*>(a.routes.y);
-    constexpr int kCache = 2048 / BLOCK;   // groups of four
-    const int n4 = a.width % 4 == 0 ? a.width / 4 : 0;
-    const int done = min(n4, kCache * BLOCK) * 4;
-    f32x4_t v[kCache];
+    if (K) {
+        if (threadIdx.x < static_cast<unsigned>(K)) {
+            pos[threadIdx.x] = a.routes.pos[n * K + threadIdx.x];
+            weight[threadIdx.x] = a.routes.weight[n * K + threadIdx.x];
+        }
+        __syncthreads();
+    }
+    constexpr int kCache = 8192 / (8 * BLOCK);   // groups of eight
+    const int n8 = a.width % 8 == 0 ? a.width / 8 : 0;
+    const int done = min(n8, kCache * BLOCK) * 8;
+    float v[kCache][8];
     float local = 0.f;
 #pragma unroll
     for (int c = 0; c < kCache; ++c) {
-        const int i = 4 * (threadIdx.x + c * BLOCK);
-        if (i >= 4 * n4) break;
-        f32x4_t s = {0.f, 0.f, 0.f, 0.f};   // (the sublayers' sum first, then the stream)
-        if (yr) s += load4(yr + i);
-        if (y2r) s += load4(y2r + i);
-        if (a.add) s += *reinterpret_cast<const f32x4_t*>(a.add + i);
-        for (int k0 = 0; k0 < K; k0 += 4) {   // (four routes requested together)
-            f32x4_t r[4];
-            float w[4];
+        const int i = 8 * (threadIdx.x + c * BLOCK);
+        if (i >= 8 * n8) break;
+        // (what a group reads is requested before any of it is used; the sublayers' sum first, then the stream)
+        Eight<T> g1, g2;
+        Eight<uint16_t> ge;
+        Eight<float> gx, gadd;
+        if (yr) g1.load(yr + i);
+        if (y2r) g2.load(y2r + i);
+        if (er) ge.load(er + i);
+        if (a.read_x) gx.load(xr + i);
+        if (a.add) gadd.load(a.add + i);
+        float (&s)[8] = v[c];
 #pragma unroll
-            for (int u = 0; u < 4; ++u) {
-                const int k = min(k0 + u, K - 1);
-                w[u] = k0 + u < K ? weight[k] : 0.f;
-                r[u] = load4(ry + static_cast<size_t>(pos[k]) * a.routes.ld + i);
+        for (int e = 0; e < 8; ++e) s[e] = 0.f;
+        if (yr)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) s[e] += g1.get(e);
+        if (y2r)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) s[e] += g2.get(e);
+        if (a.add)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) s[e] += gadd.get(e);
+        for (int k0 = 0; k0 < K; k0 += 8) {
+            Eight<T> r[8];
+#pragma unroll
+            for (int u = 0; u < 8; ++u) r[u].load(ry + static_cast<size_t>(pos[min(k0 + u, K - 1)]) * a.routes.ld + i);
+#pragma unroll
+            for (int u = 0; u < 8; ++u) {
+                const float w = k0 + u < K ? weight[min(k0 + u, K - 1)] : 0.f;
+                if (k0 + u < K)
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) s[e] = fmaf(r[u].get(e), w, s[e]);
             }
-#pragma unroll
-            for (int u = 0; u < 4; ++u)
-                if (k0 + u < K) s += r[u] * w[u];
         }
-        if (er) s += load4(er + i) * a.table_scale;
-        if (a.read_x) s += *reinterpret_cast<const f32x4_t*>(xr + i);
-        v[c] = s;
+        if (er)
 #pragma unroll
-        for (int e = 0; e < 4; ++e) local += s[e] * s[e];
-        *reinterpret_cast<f32x4_t*>(xr + i) = s;
+            for (int e = 0; e < 8; ++e) s[e] = fmaf(ge.get(e), a.table_scale, s[e]);
+        if (a.read_x)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) s[e] += gx.get(e);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) local += s[e] * s[e];
+#pragma unroll
+        for (int h = 0; h < 2; ++h)
+            *reinterpret_cast<f32x4_t*>(xr + i + 4 * h) = f32x4_t{s[4 * h], s[4 * h + 1], s[4 * h + 2], s[4 * h + 3]};
     }
     for (int i = done + threadIdx.x; i < a.width; i += BLOCK) {
         float s = 0.f;
@@ -287,12 +320,23 @@ __global__ __launch_bounds__(BLOCK) void residual_join_kernel(const JoinArgs a) 
     const float scale = a.next_w ? 1.f / sqrtf(block_total(local, red) / static_cast<float>(a.width) + a.eps) : 1.f;
 #pragma unroll
     for (int c = 0; c < kCache; ++c) {
-        const int i = 4 * (threadIdx.x + c * BLOCK);
-        if (i >= 4 * n4) break;
-        f32x4_t o = v[c];
-        if (a.next_w) o *= *reinterpret_cast<const f32x4_t*>(a.next_w + i) * scale;
-        if constexpr (sizeof(T) == 2) *reinterpret_cast<u32x2_t*>(ar + i) = u32x2_t{pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3])};
-        else *reinterpret_cast<f32x4_t*>(ar + i) = o;
+        const int i = 8 * (threadIdx.x + c * BLOCK);
+        if (i >= 8 * n8) break;
+        float (&o)[8] = v[c];
+        if (a.next_w) {
+            Eight<float> w;
+            w.load(a.next_w + i);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) o[e] *= w.get(e) * scale;
+        }
+        if constexpr (sizeof(T) == 2) {
+            *reinterpret_cast<u32x4_t*>(ar + i) =
+                u32x4_t{pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3]), pack_bf16x2(o[4], o[5]), pack_bf16x2(o[6], o[7])};
+        } else {
+#pragma unroll
+            for (int h = 0; h < 2; ++h)
+                *reinterpret_cast<f32x4_t*>(ar + i + 4 * h) = f32x4_t{o[4 * h], o[4 * h + 1], o[4 * h + 2], o[4 * h + 3]};
+        }
     }
     for (int i = done + threadIdx.x; i < a.width; i += BLOCK)   // (a thread reads what it wrote)
         ar[i] = act_put<T>(a.next_w ? xr[i] * (scale * a.next_w[i]) : xr[i]);
@@ -568,12 +612,13 @@ extern "C" int pie_hip_residual_join(int dtype, const void* y, int ldy, const vo
         (token_ids && (!table_bf16 || vocab <= 0)) ||
         (routes && (!routes->y || !routes->pos || !routes->weight || routes->top_k <= 0 || routes->ld < width)))
         return PIE_HIP_ERR_INVALID;
-    if ((y && ldy % 8 != 0) || (y2 && ldy2 % 8 != 0) || (routes && routes->ld % 8 != 0) || ld % 8 != 0) return PIE_HIP_ERR_UNSUPPORTED;
+    if ((y && ldy % 8 != 0) || (y2 && ldy2 % 8 != 0) || (routes && (routes->ld % 8 != 0 || routes->top_k > kJoinRoutes)) || ld % 8 != 0)
+        return PIE_HIP_ERR_UNSUPPORTED;
     const JoinArgs a{y, y2, add, next_weight, routes ? *routes : PieHipRoutes{}, x, token_ids, table_bf16, x_act, ldy, ldy2,
                      read_x ? 1 : 0, vocab, width, ld, table_scale, eps};
     hipStream_t s = static_cast<hipStream_t>(stream);
-    if (width >= 2048 && rows < 512)
-        PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL((residual_join_kernel<T, 1024>), dim3(rows), dim3(1024), 0, s, a));
+    if (width > 2048 && rows < 512)
+        PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL((residual_join_kernel<T, 512>), dim3(rows), dim3(512), 0, s, a));
     else
         PIE_ACT_DISPATCH(dtype, T, hipLaunchKernelGGL((residual_join_kernel<T, 256>), dim3(rows), dim3(256), 0, s, a));
     return launch_status();

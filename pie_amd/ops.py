@@ -1344,8 +1344,10 @@ def moe_route_groups(logits: torch.Tensor, experts: int, top: int, groups: int, 
     return idx, weight, offsets, token, pos
 
 
-def moe_grouped_glu(act: torch.Tensor, rows, offsets: torch.Tensor, w: torch.Tensor, routes: int, rule: Optional[Glu]) -> torch.Tensor:
-    """Rows sorted by expert times w [experts, N, K] (gated if there is a rule); bf16 or fp32 by act's type."""
+def moe_grouped_glu(act: torch.Tensor, rows, offsets: torch.Tensor, w: torch.Tensor, routes: int, rule: Optional[Glu],
+                    block_rows: Optional[int] = None, tiled: bool = False) -> torch.Tensor:
+    """Rows sorted by expert times w [experts, N, K] (gated if there is a rule); bf16 or fp32 by act's type.  bf16 with
+    block_rows: in blocks of that many routes (0: the library's choice), `tiled`: over tile-major weights."""
     E, N, K = w.shape
     lib = kernels()
     if act.dtype == torch.float32:
@@ -1358,9 +1360,15 @@ def moe_grouped_glu(act: torch.Tensor, rows, offsets: torch.Tensor, w: torch.Ten
         _check(lib.pie_hip_glu_f32(_ptr(y), C.byref(rule), _ptr(z), routes, N // 2, _stream()), "pie_hip_glu_f32")
         return z
     y = torch.empty((routes, N if rule is None else N // 2), dtype=torch.bfloat16, device=act.device)
+    glu_arg = None if rule is None else C.byref(rule)
+    if block_rows is not None:
+        _check(lib.pie_hip_moe_grouped_gemm_mfma(_ptr(act), _ptr(rows), _ptr(offsets), E, routes, _ptr(w), C.c_size_t(N * K * 2), _ptr(y), N, K,
+                                                 0 if rule is None else 1, int(tiled), glu_arg, block_rows, _stream()),
+               "pie_hip_moe_grouped_gemm_mfma")
+        return y
     _check(lib.pie_hip_moe_grouped_gemm_glu(3, _ptr(act), _ptr(rows), _ptr(offsets), E, max(1, routes), _ptr(w), C.c_size_t(N * K * 2), None,
-                                            C.c_size_t(0), 0, 0, _ptr(y), N, K, 0 if rule is None else 1, 0,
-                                            None if rule is None else C.byref(rule), _stream()), "pie_hip_moe_grouped_gemm_glu")
+                                            C.c_size_t(0), 0, 0, _ptr(y), N, K, 0 if rule is None else 1, int(tiled), glu_arg, _stream()),
+           "pie_hip_moe_grouped_gemm_glu")
     return y
 
 

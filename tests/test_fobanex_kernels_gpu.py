@@ -91,8 +91,39 @@ def test_grouped_products(gpu, bf, T, E, top, K, N):
             assert np.abs(gated[pos[n, k]] - rule(x[0::2], x[1::2], 0.75, 1.702, 1.0)).max() < (5e-2 if bf else 1e-4)
 
 
+@pytest.mark.parametrize("T,E,top,K,N", [(1, 5, 2, 128, 64), (1, 1, 1, 64, 16), (9, 5, 2, 256, 96), (120, 3, 2, 128, 160), (70, 17, 4, 384, 32),
+                                         (700, 2, 1, 192, 272), (300, 130, 8, 64, 128), (257, 70, 1, 128, 48)])
+@pytest.mark.parametrize("block_rows", [0, 64, 128, 256])
+def test_grouped_products_in_blocks_of_routes(gpu, T, E, top, K, N, block_rows):
+    """Blocks of one expert's routes, over row-major and tile-major weights; some experts without routes, some with many
+    blocks, more experts than a wave has lanes."""
+    import torch
+    from pie_amd import ops
+
+    rng = np.random.default_rng(T + E)
+    act, w = t(rng.standard_normal((T, K)), gpu, torch.bfloat16), t(rng.standard_normal((E, N, K)) * 2 / np.sqrt(K), gpu, torch.bfloat16)
+    ld = -(-E // 16) * 16
+    z = (rng.standard_normal((T, ld)) + (np.arange(ld) % 3 == 1) * 2.0).astype(np.float32)   # (an uneven choice)
+    idx, _, offsets, token, pos = ops.moe_route_groups(t(z, gpu), E, top, 1, 1, 1.0)
+    wt = ops.repack_mfma_tiles(ops.WeightView("bf16", w.reshape(E * N, K), None, 0, E * N, K)).data.reshape(E, N, K)
+    glu = ops.glu(None, 0.75, 1.702, 1.0)
+    a, wh, idx, pos = host(act), host(w), host(idx).astype(int), host(pos).astype(int)
+    want = np.zeros((T * top, N), np.float32)
+    for e in range(E):
+        n, k = np.nonzero(idx == e)
+        want[pos[n, k]] = a[n] @ wh[e].T
+    sorted_act = act[torch.as_tensor(host(token).astype(np.int64), device=gpu)].contiguous()
+    for weights, tiled in ((w, False), (wt, True)):
+        plain = host(ops.moe_grouped_glu(act, token, offsets, weights, T * top, None, block_rows, tiled))
+        assert np.abs(plain - want).max() < 5e-2
+        assert np.array_equal(plain, host(ops.moe_grouped_glu(sorted_act, None, offsets, weights, T * top, None, block_rows, tiled)))
+        gated = host(ops.moe_grouped_glu(act, token, offsets, weights, T * top, glu, block_rows, tiled))
+        assert np.abs(gated - rule(want[:, 0::2], want[:, 1::2], 0.75, 1.702, 1.0)).max() < 5e-2
+
+
 @pytest.mark.parametrize("bf", [False, True])
-@pytest.mark.parametrize("width,ld,rows,top", [(96, 128, 5, 3), (75, 128, 9, 1), (2048, 2048, 3, 8), (4098, 4224, 2, 5), (9000, 9088, 2, 2), (256, 256, 600, 4)])
+@pytest.mark.parametrize("width,ld,rows,top", [(96, 128, 5, 3), (75, 128, 9, 1), (2048, 2048, 3, 8), (4098, 4224, 2, 5), (9000, 9088, 2, 2), (256, 256, 600, 4),
+                                               (4096, 4096, 3, 11), (4104, 4224, 520, 9)])
 def test_residual_join(gpu, bf, width, ld, rows, top):
     import torch
     from pie_amd import ops
