@@ -605,15 +605,33 @@ __global__ void group_merge_kernel(const AttnArgs a, uint16_t* __restrict__ o, i
     const int steps = (len - begin + kStep - 1) / kStep, per = max(1, (steps + a.nsplit - 1) / a.nsplit);
     const int ns = min(a.nsplit, (steps + per - 1) / per);
     const float* ml = a.part_ml + out * a.nsplit * 2;
-    float mx = -INFINITY;
-    for (int s = 0; s < ns; ++s) mx = fmaxf(mx, ml[2 * s]);
-    float l = 0.f;
+    float mx = -INFINITY, l = 0.f;
     f32x4_t v = {0.f, 0.f, 0.f, 0.f};
     const float* po = a.part_o + out * a.nsplit * D + 4 * threadIdx.x;
-    for (int s = 0; s < ns; ++s) {
-        const float w = mx == -INFINITY ? 0.f : exp2f(ml[2 * s] - mx);
-        l = fmaf(ml[2 * s + 1], w, l);
-        v += *reinterpret_cast<const f32x4_t*>(po + static_cast<size_t>(s) * D) * w;
+    constexpr int kAhead = 8;   // splits requested together (those behind the last read it again and weigh nothing)
+    for (int s0 = 0; s0 < ns; s0 += kAhead) {
+        float m[kAhead];
+#pragma unroll
+        for (int u = 0; u < kAhead; ++u) m[u] = ml[2 * min(s0 + u, ns - 1)];
+#pragma unroll
+        for (int u = 0; u < kAhead; ++u) mx = fmaxf(mx, m[u]);
+    }
+    for (int s0 = 0; s0 < ns; s0 += kAhead) {
+        f32x4_t p[kAhead];
+        float w[kAhead], sum[kAhead];
+#pragma unroll
+        for (int u = 0; u < kAhead; ++u) {
+            const int s = min(s0 + u, ns - 1);
+            p[u] = *reinterpret_cast<const f32x4_t*>(po + static_cast<size_t>(s) * D);
+            w[u] = ml[2 * s];
+            sum[u] = ml[2 * s + 1];
+        }
+#pragma unroll
+        for (int u = 0; u < kAhead; ++u) {
+            const float e = mx == -INFINITY || s0 + u >= ns ? 0.f : exp2f(w[u] - mx);
+            l = fmaf(sum[u], e, l);
+            v += p[u] * e;
+        }
     }
     const float inv = a.out_scale * normaliser(l, mx, a.sink);
     store_gated(o + static_cast<size_t>(n) * a.ld_o + h * D + 4 * threadIdx.x, v * inv,
