@@ -369,13 +369,13 @@ def assert_close(got, want, dtype, what=""):
 
 
 def assert_close_routed(got, want, dtype, what=""):
-    """For mixtures: where two experts are all but equally probable, rounding decides between them, at that token and
-    a little at those that read it.  fp32: one position in fifty may be such a one; bf16: one in six."""
+    """For mixtures: where two experts are all but equally probable, rounding to bf16 decides between them, at that token
+    and a little at those that read it.  fp32: every position; bf16: one in six may be such a one."""
     e = np.sort(position_errors(got, want))
     assert np.isfinite(e).all(), what
     n = len(e)
     if dtype == "float32":
-        assert e[n - 1 - n // 50] < F32_TOL, (what, e[-1])
+        assert e[-1] < F32_TOL, (what, e[-5:])
     else:
         assert e[-1] < 1.0 and e[n - 1 - n // 6] < BF16_TOL and (n < 8 or np.median(e) < BF16_MEDIAN), (what, np.median(e), e[-5:])
 
