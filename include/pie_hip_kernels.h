@@ -50,10 +50,12 @@ extern "C" {
  *      mean what they did, 2 is the squared ReLU); the layer-stack kernels
  *   5  epilogue code 3 (exact GELU); grouped attention with windows and sinks, memories with
  *      one decay per head, residual_norm
- *   6  current: gated products with biases and clamps (PieHipGlu, the *_glu entry points); gates on the
+ *   6  gated products with biases and clamps (PieHipGlu, the *_glu entry points); gates on the
  *      outputs of grouped and latent attention; norms over whole projections; expert groups;
- *      residual_join */
-#define PIE_HIP_ABI_VERSION 6
+ *      residual_join
+ *   7  current: `sinks` of latent attention, gates per head (`gate_cols`), latents without a rotated part;
+ *      epilogues of the fp32 grouped product; corrected routes, gated joins behind convolutions */
+#define PIE_HIP_ABI_VERSION 7
 int pie_hip_abi_version(void);
 
 /* ---- W4A16 ("int4b8", symmetric, group-quantised) ------------------------- */
@@ -864,10 +866,12 @@ int pie_hip_linear_f32(const float* act, const uint16_t* w_bf16, float* y, int M
  * pie_hip_head_linear: y[n, h, c] = sum_k W[h, c, k] act[n, h, k] (heads act_stride / y_stride
  *   apart in rows of ld_act / ld_y; C % 16 == 0, K % 32 == 0).  With rotp > 0 also
  *   y[n, h, C + i] = the rotated act[n, h, rot_off + i], i < rot_dim, zeros to rotp.  With gate,
- *   y[n, h, c] is multiplied by the logistic function of gate[n, h * C + c] (rows of ld_gate).
+ *   y[n, h, c] is multiplied by the logistic function of gate[n, h * gate_cols + c % gate_cols] (rows of
+ *   ld_gate; gate_cols C: one per value, 1: one per head).
  * pie_hip_latent_attn_rows_plain: o[n, h, :] = softmax_j(q[n, h, :] . row_j * scale) . row_j[:kvp]
  *   over the first row_kv_len[n] keys; q [rows, heads, ld_row], o [rows, heads, kvp].  Any sizes
- *   (kvp <= 2048).
+ *   (kvp <= 2048).  sinks [heads] fp32 (NULL: none), in all forms of the attention: exp(sinks[h]) joins head
+ *   h's sum of exponentials.
  */
 int pie_hip_latent_prep(int dtype, const void* fused, const float* q_norm, const float* kv_norm,
                         const float* rope_table, const int64_t* kv_slots, void* cq, void* pool, int num_tokens,
@@ -876,14 +880,14 @@ int pie_hip_latent_prep(int dtype, const void* fused, const float* q_norm, const
 int pie_hip_head_linear(int dtype, const void* act, const uint16_t* w_bf16, void* y, const float* rope_table,
                         int M, int heads, int C, int K, int ld_act, int act_stride, int ld_y, int y_stride,
                         int rot_off, int rot_dim, int rot_dims, int rotp, const void* gate, int ld_gate,
-                        void* stream);
+                        int gate_cols, void* stream);
 int pie_hip_latent_attn_rows_plain(int dtype, const void* q, const void* pool, void* o,
                                    const uint32_t* kv_page_indices, const uint32_t* row_page_begin,
                                    const int32_t* row_kv_len, int num_rows, int heads, int kvp, int ld_row,
-                                   int page_size, float scale, void* stream);
+                                   int page_size, float scale, const float* sinks, void* stream);
 
 /* The same function on the matrix cores over bf16 pools, rows [row0, row0 + num_rows): weights
- * enter the second product as hi + lo bf16 pairs.  rotp in {32, 64}, kvp in {64, 128, 192, 256, 384,
+ * enter the second product as hi + lo bf16 pairs.  rotp in {0, 32, 64}, kvp in {64, 128, 192, 256, 384,
  * 512} (pie_hip_latent_attn_rows_supported), page_size % 16 == 0.  max_tokens_per_req: the most
  * rows a request brings (1: a decode batch; more: row_req / qo_indptr must cover the rows, whole
  * requests only).  workspace: pie_hip_latent_attn_rows_workspace_bytes. */
@@ -893,8 +897,8 @@ size_t pie_hip_latent_attn_rows_workspace_bytes(int num_rows, int heads, int kvp
 int pie_hip_latent_attn_rows(const uint16_t* q, const uint16_t* pool, uint16_t* o, const uint32_t* kv_page_indices,
                              const uint32_t* row_page_begin, const int32_t* row_kv_len, const int32_t* row_req,
                              const int32_t* qo_indptr, int row0, int num_rows, int heads, int kvp, int rotp,
-                             int page_size, float scale, int max_kv_len, int max_tokens_per_req, void* workspace,
-                             size_t workspace_bytes, void* stream);
+                             int page_size, float scale, const float* sinks, int max_kv_len,
+                             int max_tokens_per_req, void* workspace, size_t workspace_bytes, void* stream);
 /* Long portions: keys and values projected out of the latents, then ordinary causal attention.
  * pie_hip_latent_gather: the first num_keys cache rows of a page list as compact rows, lat [num_keys,
  *   kvp] and rot [num_keys, rotp].
@@ -902,15 +906,17 @@ int pie_hip_latent_attn_rows(const uint16_t* q, const uint16_t* pool, uint16_t* 
  *   rotp] (the rotated part not yet rotated: rope_table rows as for pie_hip_latent_prep), kv
  *   [num_keys, heads, dimp + vdp] the projected keys and values, rot as gathered; row n sees its
  *   first row_kv_len[n] keys; o [rows, ld_o], heads vdp apart, times the logistic function of
- *   gate[n, h * vdp + c] (rows of ld_gate; NULL: none).  (dimp + rotp) / 32 in 2..6, vdp / 32
- *   in 1..4 (pie_hip_latent_attn_prefill_supported). */
+ *   gate[n, h * gate_cols + c % gate_cols] (rows of ld_gate, gate_cols vdp or 1; NULL: none).  rot may be
+ *   NULL with rotp 0.  (dimp + rotp) / 32 in 1..6, vdp / 32 in 1..4
+ *   (pie_hip_latent_attn_prefill_supported). */
 int pie_hip_latent_gather(const uint16_t* pool, const uint32_t* pages, uint16_t* lat, uint16_t* rot, int num_keys,
                           int kvp, int rotp, int page_size, void* stream);
 int pie_hip_latent_attn_prefill_supported(int dimp, int rotp, int vdp);
 int pie_hip_latent_attn_prefill(const uint16_t* q, const uint16_t* kv, const uint16_t* rot, uint16_t* o,
                                 const float* rope_table, const int32_t* row_kv_len, int row0, int num_rows,
                                 int num_keys, int heads, int dimp, int rotp, int rot_dims, int vdp, int ld_o,
-                                float scale, const uint16_t* gate, int ld_gate, void* stream);
+                                float scale, const float* sinks, const uint16_t* gate, int ld_gate,
+                                int gate_cols, void* stream);
 
 /*
  * Gated delta rule with a decay per head and key channel.  row_req [N]: request of each row;
@@ -997,11 +1003,12 @@ int pie_hip_residual_join(int dtype, const void* y, int ldy, const void* y2, int
                           void* x_act, int rows, int width, int ld, float eps, void* stream);
 /* The fp32 forms of a mixture's products and of the gated rule:
  * pie_hip_moe_grouped_linear_f32: rows expert_offsets[e] .. expert_offsets[e + 1] of y [routes, N] are
- *   act[route_act_rows[r]] (or act[r]) . W_e^T, W_e bf16 [N, K] at w + e * N * K; no expert has more than max_rows.
+ *   act[route_act_rows[r]] (or act[r]) . W_e^T, W_e bf16 [N, K] at w + e * N * K; no expert has more than
+ *   max_rows; epilogue as for pie_hip_linear_f32.
  * pie_hip_glu_f32: y[m, i] = the rule of PieHipGlu on columns (2i, 2i + 1) of x [M, 2 n]. */
 int pie_hip_moe_grouped_linear_f32(const float* act, const int32_t* route_act_rows, const int32_t* expert_offsets,
                                    int num_experts, int max_rows, const uint16_t* w_bf16, float* y, int N, int K,
-                                   void* stream);
+                                   int epilogue, void* stream);
 int pie_hip_glu_f32(const float* x, const PieHipGlu* glu, float* y, int M, int n, void* stream);
 /* y[M, N] fp32 = act[M, K] . W[N, K]^T over bf16 weights (fp32 sums, not rounded): the few columns that
  * drive a recurrence.  K % 32 == 0, N % 16 == 0. */
@@ -1133,6 +1140,39 @@ int pie_hip_gated_part_norm(int dtype, const float* o, const void* x, int ld_x, 
                             int ld_z, const float* norm_w, void* y, int ld_y, int heads, int vdim, int parts,
                             const PieHipStateRows* rows, const void* conv_fused, int ld_fused, int channels, int taps,
                             float eps, void* stream);
+
+/*
+ * Layers whose sublayers' outputs pass a logistic gate and whose sublayers read a short convolution of the normed
+ * stream: h = norm(x), the sublayer reads h + conv(h), x += sublayer * sigmoid(gate), the gate a product of h.
+ * pie_hip_embed_bigram: x[n] = e / sqrt(mean(e^2) + eps) * norm_weight, e = table[token_ids[n]] * table_scale +
+ *   bigram[row], row = (prev_ids[n] * mul_prev + token_ids[n] * mul_cur) mod buckets in 64 bits, row `buckets`
+ *   where prev_ids[n] < 0 (a sequence's first token); bigram NULL: left out; ids >= vocab read row 0 of table.
+ * pie_hip_gated_join: x[n] += (y[n] or a mixture's routes, see PieHipRoutes) * sigmoid(gate[n] + gate_bias) (neither y
+ *   nor routes: x as it is); h[n] = x[n] / sqrt(mean(x[n]^2) + eps) * next_weight in the compute type (next_weight
+ *   NULL: x only).  With conv_w (one row per request, taps <= 4) also recent[n] = h[n] + the convolution, whose
+ *   state moves on by the row.  Rows of ld; columns from the width on are not touched.
+ * pie_hip_recent_rows: recent[n, c] = h[n, c] + sum_j conv_w[j, c] h_(n - (taps - 1) + j)[c], earlier rows from the
+ *   request's state, zeros before its start; pie_hip_delta_conv_state (channels = width) moves the state on
+ *   afterwards.  conv_w [taps, width] fp32; the state is [taps - 1, width] in the compute type at conv_offset.
+ */
+int pie_hip_embed_bigram(const uint32_t* token_ids, const int32_t* prev_ids, const uint16_t* table_bf16, int vocab,
+                         float table_scale, const uint16_t* bigram_bf16, unsigned long long buckets,
+                         unsigned long long mul_prev, unsigned long long mul_cur, const float* norm_weight, float* x,
+                         int num_tokens, int width, int ld, float eps, void* stream);
+int pie_hip_gated_join(int dtype, const void* y, int ldy, const PieHipRoutes* routes, const void* gate, int ld_gate,
+                       const float* gate_bias, float* x, const float* next_weight, void* h, void* recent,
+                       const float* conv_w, int taps, const PieHipStateRows* state, int rows, int width, int ld,
+                       float eps, void* stream);
+int pie_hip_recent_rows(int dtype, const void* h, const float* conv_w, int taps, const PieHipStateRows* state, void* recent,
+                        int width, int ld, void* stream);
+/* The sorted layout of pie_hip_moe_route_groups for a router of logistic scores s = sigmoid(logit): a token uses the
+ * top_k experts with the largest s + correction (lowest index among equals), weighted by their s.  `shared` experts
+ * that every token uses come ahead of them, as experts 0 .. shared - 1, weighted by sigmoid(logits[t, num_experts]);
+ * the routed ones are numbered from `shared` on.  topk_idx and topk_weight [T, shared + top_k],
+ * expert_offsets [shared + num_experts + 1]. */
+int pie_hip_moe_route_corrected(const float* router_logits, int ld_logits, const float* correction, int32_t* topk_idx,
+                                float* topk_weight, int32_t* expert_offsets, int32_t* route_token, int32_t* route_pos,
+                                int num_tokens, int num_experts, int top_k, int shared, void* stream);
 
 /* pie_hip_sample_gather_logits over fp32 logits. */
 int pie_hip_sample_gather_logits_f32(const float* logits, const int32_t* rows, float* out_f32,

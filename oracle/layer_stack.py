@@ -1,6 +1,7 @@
 """Plain, slow statement of the layer-stack models in numpy double precision: Varasun (latent attention,
 the channel-decay delta rule) and Lofudra (windowed attention beside retention, mLSTM, Mamba-2, a loop
-over some of the layers).
+over some of the layers), Fobanex (normed and gated attention, shared latents, mixtures) and Minodra (latent
+attention without positions, gated sublayers behind short convolutions, mixtures with a corrected choice).
 
 One function per mechanism, whole sequences only: no cache, no pages, no batches.  Nothing here is
 shared with the product path; the tests compare the driver with it and plant their mistakes here.
@@ -397,8 +398,96 @@ def forward_shared_norm(cfg, w, tokens, want_layers=False):
     return (logits, np.stack(states)) if want_layers else logits
 
 
+# ---- Minodra ---------------------------------------------------------------------------------------
+def bigram_rows(tokens, buckets, mul_prev, mul_cur):
+    """Row of the bigram table per place: a hash of the previous and the own token; the last row at the start."""
+    t = [int(x) for x in tokens]
+    return np.array([buckets] + [(a * mul_prev + b * mul_cur) % buckets for a, b in zip(t, t[1:])])
+
+
+def scalar_norm(x, g, eps):
+    """Divided by its root mean square, times one number."""
+    return divide_by_rms(np.asarray(x, np.float64), eps) * float(np.asarray(g).reshape(()))
+
+
+def with_recent(h, w):
+    """A row plus a causal convolution over it and the rows before it."""
+    return h + causal_conv(h, w)
+
+
+def softmax_with_learned_sink(scores, seen, sink):
+    """scores [H, T, T], sink [H] in score units: exp(sink) joins the sum, without key or value."""
+    s = np.where(seen, scores, -np.inf)
+    m = np.maximum(s.max(axis=-1, keepdims=True), sink[:, None, None])
+    p = np.exp(s - m)
+    return p / (p.sum(axis=-1, keepdims=True) + np.exp(sink[:, None, None] - m))
+
+
+def sink_latent_attention(h, w, p, m, eps):
+    """No rotation; a learned sink and one logistic output gate per head."""
+    T, H, dim, dv = len(h), m["heads"], m["dim"], m["vdim"]
+    cq = rms_norm(h @ w[p + "dq"].T, w[p + "dq.norm"], eps)
+    c = rms_norm(h @ w[p + "dkv"].T, w[p + "dkv.norm"], eps)
+    q, k, v = ((x @ w[p + n].T).reshape(T, H, d) for x, n, d in ((cq, "uq", dim), (c, "uk", dim), (c, "uv", dv)))
+    a = softmax_with_learned_sink(np.einsum("ihd,jhd->hij", q, k) * m["scale"], window_mask(T, None), w[p + "sink"])
+    o = np.einsum("hij,jhd->ihd", a, v) * sigmoid(h @ w[p + "g"].T)[:, :, None]
+    return o.reshape(T, H * dv) @ w[p + "o"].T
+
+
+def silu_pair_feed_forward(h, w, p):
+    return (silu(h @ w[p + "gate"].T) * (h @ w[p + "up"].T)) @ w[p + "down"].T
+
+
+def corrected_route(z, correction, top):
+    """Logistic scores; the largest scores plus correction are chosen, the plain scores are the weights."""
+    s = sigmoid(z)
+    out = np.zeros_like(s)
+    for t in range(len(z)):
+        chosen = np.argsort(-(s[t] + correction), kind="stable")[:top]
+        out[t, chosen] = s[t, chosen]
+    return out
+
+
+def shared_mixture(h, w, p, mlp):
+    """Squared-ReLU experts, the chosen ones weighted; one more for every token behind a logistic gate."""
+    weight = corrected_route(h @ w[p + "router"].T, w[p + "correction"], mlp["router"]["top"])
+    y = np.zeros_like(h)
+    for e in range(mlp["router"]["experts"]):
+        t = np.nonzero(weight[:, e])[0]
+        if len(t):
+            y[t] += weight[t, e, None] * feed_forward(h[t], w, f"{p}e{e}.")
+    if mlp.get("shared"):
+        y += sigmoid(h @ w[p + "shared.sg"].T) * feed_forward(h, w, p + "shared.")
+    return y
+
+
+def gated_sublayer(x, w, p, n, sublayer, eps):
+    """x plus the sublayer's output through a logistic gate; both read the normed stream, the sublayer behind a convolution."""
+    h = scalar_norm(x, w[f"{p}norm{n}"], eps)
+    return x + sublayer(with_recent(h, w[f"{p}canon{n}"])) * sigmoid(h @ w[f"{p}rg{n}"].T + w[f"{p}rg{n}.b"])
+
+
+def forward_gated(cfg, w, tokens, want_layers=False):
+    eps, b = cfg["norm"]["eps"], cfg["embedding"]["bigram"]
+    x = np.asarray(w["embed"], np.float64)[np.asarray(tokens)] * cfg["embedding"]["scale"]
+    x = scalar_norm(x + w["bigram"][bigram_rows(tokens, b["buckets"], b["mul_prev"], b["mul_cur"])], w["embed.norm"], eps)
+    states = []
+    for i, layer in enumerate(cfg["layers"]):
+        p, mlp = f"l{i}.", layer.get("mlp")
+        x = gated_sublayer(x, w, p, 1, lambda h: sink_latent_attention(h, w, p + "mix.", layer["mixer"], eps), eps)
+        if mlp:
+            ff = silu_pair_feed_forward if mlp["kind"] == "dense" else (lambda h, w, q: shared_mixture(h, w, q, mlp))
+            x = gated_sublayer(x, w, p, 2, lambda h: ff(h, w, p + "mlp."), eps)
+        states.append(x)
+    cap = cfg["logit_softcap"]
+    logits = cap * np.tanh(scalar_norm(x, w["final.norm"], eps) @ w["head"].T / cap)
+    return (logits, np.stack(states)) if want_layers else logits
+
+
 def forward(cfg, w, tokens, want_layers=False):
     """Logits [T, vocab] of one sequence (and the residual stream after every layer)."""
+    if cfg["architecture"] == "Minodra":
+        return forward_gated(cfg, w, tokens, want_layers)
     if cfg["architecture"] == "Lofudra":
         return forward_sandwich(cfg, w, tokens, want_layers)
     if cfg["architecture"] == "Fobanex":

@@ -51,6 +51,21 @@ struct ActVec<float> {
     }
 };
 
+// Eight values at a time, still in the compute type.
+template <class T>
+struct Eight {
+    u32x4_t r[sizeof(T) / 2];
+    __device__ __forceinline__ void load(const T* p) {
+#pragma unroll
+        for (int h = 0; h < static_cast<int>(sizeof(T)) / 2; ++h) r[h] = reinterpret_cast<const u32x4_t*>(p)[h];
+    }
+    __device__ __forceinline__ float get(int e) const {
+        if constexpr (sizeof(T) == 2) return e & 1 ? bf16_hi(r[0][e / 2]) : bf16_lo(r[0][e / 2]);
+        else return __uint_as_float(r[e / 4][e % 4]);
+    }
+};
+constexpr int kJoinRoutes = 64;   // places and weights of a token's routes through a mixture wait in LDS
+
 // (the bare exponential and reciprocal: a few units in the last place)
 __device__ __forceinline__ float sigmoid_f32(float z) {
     return __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));

@@ -34,14 +34,17 @@ struct RotarySpec {
     }
 };
 
-// Attention over a cached low-rank latent per token and one rotated key part shared by the heads; optionally
-// on another layer's cached latents, and with a logistic gate on the concatenated heads.
+// Attention over a cached low-rank latent per token and one rotated key part shared by the heads (or none);
+// optionally on another layer's cached latents, with a learned sink per head (exp(sink) joins the sum of
+// exponentials), and with logistic gates on the heads' outputs: one per value or one per head.
+enum class OutputGate { None, PerValue, PerHead };
 struct LatentAttentionSpec {
     int heads = 0, dim = 0, rot_dim = 0, vdim = 0, q_rank = 0, kv_rank = 0;
     double scale = 0.0;
     RotarySpec rot;
     bool half_split = false;   // rotated pairs (i, i + dims / 2) instead of neighbours
-    bool gate = false;
+    bool sinks = false;
+    OutputGate gate = OutputGate::None;
     int kv_from = -1;          // the layer whose cache rows this one reads (-1: its own)
 };
 
@@ -81,12 +84,25 @@ struct DecayMemorySpec {
 // Parallel: attention and a memory side by side on the same input, attention_scale * a + memory_scale * m.
 enum class MixerKind { LatentAttention, ChannelDelta, DecayMemory, Parallel, Attention };
 
-// A mixture of gated feed-forwards: a softmax router over `experts`, of which a token uses `top`, chosen from
-// the best `keep` of `groups` equal groups of neighbours; the chosen probabilities are divided by their sum and
-// multiplied by `scale`.  Expert: g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(alpha g) (u + shift).
+// A mixture of feed-forwards: a router over `experts`, of which a token uses `top`.
+// GroupSoftmax: chosen from the best `keep` of `groups` equal groups of neighbours; the chosen probabilities are
+// divided by their sum and multiplied by `scale`.  CorrectedScores: logistic scores, the largest after a learned
+// correction are chosen, the scores themselves are the weights.
+// Expert, ClampedPair: g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(alpha g) (u + shift);
+// SquaredRelu: max(up, 0)^2.  `shared_ff`: width of one more expert that every token uses, behind a logistic gate
+// (0: none); it is cut into parts as wide as the (padded) experts, which then run and join like chosen ones.
+enum class RouterKind { GroupSoftmax, CorrectedScores };
+enum class ExpertKind { ClampedPair, SquaredRelu };
 struct MixtureSpec {
-    int experts = 0, top = 0, ff = 0, groups = 1, keep = 1;
+    RouterKind router = RouterKind::GroupSoftmax;
+    ExpertKind expert = ExpertKind::ClampedPair;
+    int experts = 0, top = 0, ff = 0, groups = 1, keep = 1, shared_ff = 0;
     float scale = 1.f, limit = 0.f, alpha = 1.f, shift = 0.f;
+    int padded_ff() const { return (ff + 127) / 128 * 128; }
+    int shared_parts() const { return shared_ff > 0 ? (shared_ff + padded_ff() - 1) / padded_ff() : 0; }
+    int all_experts() const { return experts + shared_parts(); }   // shared parts first
+    int routes() const { return top + shared_parts(); }            // of a token
+    int router_columns() const { return experts + (shared_ff > 0 ? 1 : 0); }   // the last: the shared expert's gate
 };
 
 struct LayerSpec {
@@ -112,12 +128,18 @@ struct LayerRun {
     bool begins_pass;   // first layer of a pass of the loop
 };
 
-// (GatedSilu: silu(gate) * up between three matrices with biases)
+// (GatedSilu: silu(gate) * up between three matrices, with biases or without)
 enum class FeedForwardAct { SquaredRelu, Gelu, GatedSilu };
+
+// A second embedding row per token, by a hash of the previous token and its own: row (previous * mul_prev + token *
+// mul_cur) mod buckets, row `buckets` for a sequence's first token (buckets 0: none).
+struct BigramSpec {
+    std::uint64_t buckets = 0, mul_prev = 0, mul_cur = 0;
+};
 
 struct ModelConfig {
     // architecture: "llama3" (dense, adjacent-pair RoPE) | "qwen3" (dense, qk-norm, half-split
-    // RoPE) | "qwen3_moe" | "varasun", "lofudra", "fobanex" (layer stacks)
+    // RoPE) | "qwen3_moe" | "varasun", "lofudra", "fobanex", "minodra" (layer stacks)
     std::string arch = "llama3";
     int hidden = 0, layers = 0, q_heads = 0, kv_heads = 0, head_dim = 0, intermediate = 0;
     int vocab = 0;
@@ -158,8 +180,14 @@ struct ModelConfig {
     LayerLoop loop;                // stop 0: none
     bool sandwich_norms = false;   // a norm ahead of every sublayer besides the one on its output
     bool shared_norm = false;      // one norm per layer: mixer and feed-forward read it and join the stream together
-    float embed_scale = 1.f;       // (with shared_norm)
+    // sublayers read a normed row plus a convolution over it and its last canon_taps - 1 predecessors; their outputs
+    // pass a logistic gate of the normed row; norms have one weight for all columns; the embedding is normed
+    bool gated_sublayers = false;
+    int canon_taps = 0;
+    BigramSpec bigram;
+    float embed_scale = 1.f;       // (with shared_norm or gated_sublayers)
     FeedForwardAct ff_act = FeedForwardAct::SquaredRelu;
+    bool ff_biases = false;        // GatedSilu
     std::vector<LayerRun> layer_runs() const {
         std::vector<LayerRun> runs;
         const int n = static_cast<int>(stack.size());
@@ -366,11 +394,14 @@ inline void finalize_stack(DriverConfig& c) {
         }
         if (l.moe.experts != 0) {
             const auto& e = l.moe;
-            if (!m.shared_norm) throw std::runtime_error(at + "a mixture needs an architecture whose sublayers share a norm");
+            if (!m.shared_norm && !m.gated_sublayers)
+                throw std::runtime_error(at + "this architecture has no mixtures");
             if (e.experts <= 0 || e.ff <= 0 || e.top <= 0 || e.groups <= 0 || e.keep <= 0 || e.keep > e.groups || e.experts % e.groups != 0)
                 throw std::runtime_error(at + "a mixture needs experts in equal groups, a positive width, top and kept groups");
             if (e.top > e.keep * (e.experts / e.groups)) throw std::runtime_error(at + "fewer experts in the kept groups than a token uses");
-            if (e.experts > 512 || e.top > 64) throw std::runtime_error(at + "mixtures are limited to 512 experts, 64 per token");
+            if (e.shared_ff < 0) throw std::runtime_error(at + "shared.ff must not be negative");
+            if (e.all_experts() > 512 || e.routes() > 64)
+                throw std::runtime_error(at + "mixtures are limited to 512 experts, 64 per token (a shared expert counts by its parts)");
             if (!(e.limit >= 0.f)) throw std::runtime_error(at + "expert.limit must not be negative");
         }
         if (l.has_memory()) {
@@ -392,6 +423,7 @@ inline void finalize_stack(DriverConfig& c) {
         if (m.loop.start < 0 || m.loop.stop <= m.loop.start || m.loop.stop > static_cast<int>(m.stack.size()) || m.loop.times <= 0)
             throw std::runtime_error("config: loop needs 0 <= start < stop <= layers and times > 0");
     }
+    if (m.gated_sublayers && m.canon_taps <= 0) throw std::runtime_error("config: canon.taps must be positive");
     if (m.compute_dtype != "bfloat16" && m.compute_dtype != "float32")
         throw std::runtime_error("config: compute_dtype must be bfloat16 or float32");
     m.quant = "bf16";   // the linears of layer stacks are kept as stored

@@ -864,20 +864,24 @@ extern "C" long long pie_hip_driver_snapshot_info(const char* dir, char* out, si
           << ",\"rope_factor\":" << m.rope_factor << ",\"tie_embeddings\":" << (m.tie_embeddings ? "true" : "false")
           << ",\"num_experts\":" << m.num_experts << ",\"top_k\":" << m.top_k
           << ",\"expert_intermediate\":" << m.expert_intermediate << ",\"logit_scale\":" << m.logit_scale
-          << ",\"logit_softcap\":" << m.logit_softcap << ",\"embed_scale\":" << m.embed_scale << ",\"loop\":[" << m.loop.start << "," << m.loop.stop << ","
+          << ",\"logit_softcap\":" << m.logit_softcap << ",\"embed_scale\":" << m.embed_scale << ",\"canon_taps\":" << m.canon_taps
+          << ",\"bigram\":[" << m.bigram.buckets << "," << m.bigram.mul_prev << "," << m.bigram.mul_cur << "],\"loop\":[" << m.loop.start << "," << m.loop.stop << ","
           << m.loop.times << "],\"stack\":[";
         for (size_t i = 0; i < m.stack.size(); ++i) {
             const LayerSpec& l = m.stack[i];
             j << (i ? ",{" : "{") << "\"ff\":" << l.ff;
             if (l.moe.experts)
                 j << ",\"mixture\":{\"experts\":" << l.moe.experts << ",\"top\":" << l.moe.top << ",\"ff\":" << l.moe.ff << ",\"groups\":"
-                  << l.moe.groups << ",\"keep\":" << l.moe.keep << ",\"scale\":" << l.moe.scale << ",\"limit\":" << l.moe.limit << "}";
+                  << l.moe.groups << ",\"keep\":" << l.moe.keep << ",\"scale\":" << l.moe.scale << ",\"limit\":" << l.moe.limit << ",\"shared_ff\":"
+                  << l.moe.shared_ff << ",\"router\":" << static_cast<int>(l.moe.router) << ",\"expert\":" << static_cast<int>(l.moe.expert) << "}";
             if (l.mixer == MixerKind::LatentAttention)
                 j << ",\"type\":\"latent_attention\",\"heads\":" << l.latent.heads << ",\"dim\":" << l.latent.dim
                   << ",\"rot_dim\":" << l.latent.rot_dim << ",\"vdim\":" << l.latent.vdim << ",\"q_rank\":" << l.latent.q_rank
                   << ",\"kv_rank\":" << l.latent.kv_rank << ",\"scale\":" << l.latent.scale << ",\"rot_dims\":" << l.latent.rot.dims
                   << ",\"rot_base\":" << l.latent.rot.base << ",\"yarn\":" << (l.latent.rot.yarn ? "true" : "false")
-                  << ",\"half_split\":" << (l.latent.half_split ? "true" : "false") << ",\"gate\":" << (l.latent.gate ? "true" : "false")
+                  << ",\"half_split\":" << (l.latent.half_split ? "true" : "false") << ",\"gate\":" << (l.latent.gate != OutputGate::None ? "true" : "false")
+                  << ",\"gate_per_head\":" << (l.latent.gate == OutputGate::PerHead ? "true" : "false") << ",\"sinks\":"
+                  << (l.latent.sinks ? "true" : "false")
                   << ",\"kv_from\":" << l.latent.kv_from;
             else if (l.mixer == MixerKind::ChannelDelta)
                 j << ",\"type\":\"channel_delta\",\"heads\":" << l.delta.heads << ",\"kv_heads\":" << l.delta.kv_heads

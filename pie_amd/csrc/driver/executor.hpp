@@ -23,6 +23,8 @@
 //                     state slot, norm + gate, out-projection
 //   attention         in-projection, norms + rotation + cache write, grouped attention, out-projection
 //   parallel          one in-projection, grouped attention and a decay memory on it, one out-projection
+// Gated sublayers: the embedding normed, then per sublayer the stream normed, a short convolution over the normed
+// rows (state in the request's slot), the sublayer on it, and a logistic gate of the normed row on its output.
 // A mixture of experts: fp32 router logits, the choice of experts and the sorted layout, two grouped products.
 // Architectures whose sublayers share a norm join both outputs (a mixture's routes weighted on the way) and norm
 // the stream for the next layer in one kernel; latent layers may read another layer's cache rows.
@@ -131,7 +133,7 @@ class Executor {
     // rows' requests and the requests' row ranges and state slots.
     struct Inputs {
         size_t off_tokens, off_positions, off_slots, off_row_begin, off_row_len, off_sample_rows,
-            off_row_req, off_qo, off_rs_slot, off_rs_fresh, off_pages, total;
+            off_row_req, off_prev, off_qo, off_rs_slot, off_rs_fresh, off_pages, total;
     };
     Inputs input_layout(int N, int S) const;
     void body(int N, int S, int max_kv_len);
@@ -163,7 +165,9 @@ class Executor {
     void stack_memory(const StackLayer& w, int run, int N, const Inputs& in);
     PieHipStateRows state_rows(int run, int N, const Inputs& in) const;
     void stack_mixture(const StackLayer& w, int N);
+    void stack_dense(const StackLayer& w, void* y, int N);
     void stack_shared_norm(int N, int max_kv_len, const Inputs& in);
+    void stack_gated(int N, int max_kv_len, const Inputs& in);
     void stack_mixer(const StackLayer& w, int run, int N, int max_kv_len, const Inputs& in);
     void stack_linear(const Linear& w, const void* act, void* y, int M, int epilogue = PIE_HIP_EPI_NONE,
                       const PieHipGlu* glu = nullptr);
@@ -277,6 +281,7 @@ class Executor {
         float *dq = nullptr, *dk = nullptr, *dv = nullptr, *dg = nullptr, *d_beta = nullptr, *d_o = nullptr;
         void* conv = nullptr;                                      // compute type: after a memory's convolution
         void *y2 = nullptr, *routes = nullptr;                     // compute type: a feed-forward's rows, a mixture's routes' rows
+        void *h = nullptr, *sub_gate = nullptr;                    // compute type: normed rows ahead of their convolution, gates of a sublayer
         float *router = nullptr, *route_w = nullptr, *glu = nullptr;   // router logits, weights, fp32 pairs ahead of the gated rule
         int32_t *route_idx = nullptr, *route_offsets = nullptr, *route_token = nullptr, *route_pos = nullptr;
         float *gates = nullptr, *mem_o = nullptr, *den = nullptr;  // decay memories: gate columns, read-outs, divisors
@@ -291,7 +296,9 @@ class Executor {
     int rs_slots_ = 0, cpu_rs_slots_ = 0;
     size_t rs_stride_ = 0;                       // bytes per slot
     std::vector<size_t> rs_state_off_, rs_conv_off_;   // per layer run
+    std::vector<std::array<size_t, 2>> rs_canon_off_;  // per layer run: inputs of the convolutions ahead of its sublayers
     std::vector<int64_t> rs_pos_, rs_host_pos_;  // tokens a slot's state has seen (-1: nothing)
+    std::vector<int32_t> rs_last_, rs_host_last_;   // the last of them
 
     std::map<std::tuple<int, int, int, int>, hipGraphExec_t> graphs_;   // (rows, sampling slots, context bucket, rows equally long)
     bool uniform_rows_ = false;   // this step's rows are about equally long (decode batches)

@@ -46,18 +46,20 @@ void Executor::alloc_stack() {
         const StackLayer& l = model_.stack[static_cast<size_t>(run.layer)];
         rs_state_off_.push_back(0);
         rs_conv_off_.push_back(0);
+        rs_canon_off_.push_back({0, 0});
+        if (m.gated_sublayers)
+            for (int n = 0; n < (l.pre2 ? 2 : 1) && m.canon_taps > 1; ++n)
+                rs_canon_off_.back()[n] = place(static_cast<size_t>(m.canon_taps - 1) * m.hidden * esize);
         up(act, l.spec.ff > 0 ? pad_to(l.spec.ff, 128) : 0);
-        if (m.shared_norm && l.spec.ff > 0) {
-            up(y2, model_.ld_x());
-            up(glu, 2 * pad_to(l.spec.ff, 128));
-        }
+        if (m.shared_norm && l.spec.ff > 0) up(y2, model_.ld_x());
+        if (m.ff_act == FeedForwardAct::GatedSilu && l.spec.ff > 0) up(glu, 2 * pad_to(l.spec.ff, 128));
         if (l.spec.moe.experts > 0) {
-            const int width = l.spec.moe.top * pad_to(l.spec.moe.ff, 128);
-            up(act, width);
-            up(glu, 2 * width);
-            up(top, l.spec.moe.top);
-            up(router, pad_to(l.spec.moe.experts, 16));
-            up(experts, l.spec.moe.experts);
+            const MixtureSpec& e = l.spec.moe;
+            up(act, e.routes() * e.padded_ff());
+            if (e.expert == ExpertKind::ClampedPair) up(glu, 2 * e.routes() * e.padded_ff());
+            up(top, e.routes());
+            up(router, pad_to(e.router_columns(), 16));
+            up(experts, e.all_experts());
         }
         if (l.spec.mixer == MixerKind::LatentAttention) {
             const LatentShape s(l.spec.latent);
@@ -99,6 +101,7 @@ void Executor::alloc_stack() {
             }
         }
     }
+    if (m.bigram.buckets > 0 && state == 0) place(4);   // (a request's previous token is state: it needs a slot)
     // Zeroed: columns that pad a row to its product's K are written by nobody.
     auto take = [&](size_t bytes) {
         void* p = nullptr;
@@ -121,6 +124,10 @@ void Executor::alloc_stack() {
     stack_.act = compute(T * act);
     stack_.gate = compute(T * gate);
     stack_.y2 = compute(T * y2);
+    if (m.gated_sublayers) {
+        stack_.h = compute(T * ld_x);
+        stack_.sub_gate = compute(T * ld_x);
+    }
     if (top) {
         stack_.routes = compute(T * top * ld_x);
         stack_.router = f32(T * router);
@@ -148,7 +155,7 @@ void Executor::alloc_stack() {
     stack_.logits = f32(srows * static_cast<size_t>(m.vocab));
     for (const RotaryTable& r : model_.rotary) stack_.rotary.push_back(f32(T * static_cast<size_t>(r.spec.dims)));
     for (StackLayer& l : model_.stack)
-        for (const Linear* w : {&l.w_in, &l.w_uq, &l.wo, l.spec.moe.experts ? &l.wo : &l.w_up, l.spec.moe.experts ? &l.wo : &l.w_down})
+        for (const Linear* w : {&l.w_in, &l.w_uq, &l.wo, &l.w_gate1, l.spec.moe.experts ? &l.wo : &l.w_up, l.spec.moe.experts ? &l.wo : &l.w_down})
             for (int rows : {64, 128})
                 if (!m.f32() && w->data && w->K % 64 == 0)
                     gemm_ws_bytes_ = std::max(gemm_ws_bytes_, pie_hip_gemm_mfma_workspace_bytes(rows, w->N, w->K));
@@ -179,6 +186,8 @@ void Executor::alloc_stack() {
         }
         rs_pos_.assign(static_cast<size_t>(rs_slots_), -1);
         rs_host_pos_.assign(static_cast<size_t>(cpu_rs_slots_), -1);
+        rs_last_.assign(static_cast<size_t>(rs_slots_), -1);
+        rs_host_last_.assign(static_cast<size_t>(cpu_rs_slots_), -1);
     }
     PIE_HIP_CHECK(hipStreamSynchronize(stream_));
 }
@@ -190,6 +199,7 @@ void Executor::copy_rs_d2d(const uint32_t* srcs, const uint32_t* dsts, size_t n)
         PIE_HIP_CHECK(hipMemcpyAsync(rs_base_ + dsts[i] * rs_stride_, rs_base_ + srcs[i] * rs_stride_, rs_stride_,
                                      hipMemcpyDeviceToDevice, stream_));
         rs_pos_[dsts[i]] = rs_pos_[srcs[i]];
+        rs_last_[dsts[i]] = rs_last_[srcs[i]];
     }
     PIE_HIP_CHECK(hipStreamSynchronize(stream_));
 }
@@ -198,6 +208,7 @@ void Executor::copy_rs_d2h(const uint32_t* srcs, const uint32_t* dsts, size_t n)
         PIE_HIP_CHECK(hipMemcpyAsync(rs_host_ + dsts[i] * rs_stride_, rs_base_ + srcs[i] * rs_stride_, rs_stride_,
                                      hipMemcpyDeviceToHost, stream_));
         rs_host_pos_[dsts[i]] = rs_pos_[srcs[i]];
+        rs_host_last_[dsts[i]] = rs_last_[srcs[i]];
     }
     PIE_HIP_CHECK(hipStreamSynchronize(stream_));
 }
@@ -206,6 +217,7 @@ void Executor::copy_rs_h2d(const uint32_t* srcs, const uint32_t* dsts, size_t n)
         PIE_HIP_CHECK(hipMemcpyAsync(rs_base_ + dsts[i] * rs_stride_, rs_host_ + srcs[i] * rs_stride_, rs_stride_,
                                      hipMemcpyHostToDevice, stream_));
         rs_pos_[dsts[i]] = rs_host_pos_[srcs[i]];
+        rs_last_[dsts[i]] = rs_host_last_[srcs[i]];
     }
     PIE_HIP_CHECK(hipStreamSynchronize(stream_));
 }
@@ -213,6 +225,7 @@ void Executor::copy_rs_h2h(const uint32_t* srcs, const uint32_t* dsts, size_t n)
     for (size_t i = 0; i < n; ++i) {
         std::memmove(rs_host_ + dsts[i] * rs_stride_, rs_host_ + srcs[i] * rs_stride_, rs_stride_);
         rs_host_pos_[dsts[i]] = rs_host_pos_[srcs[i]];
+        rs_host_last_[dsts[i]] = rs_host_last_[srcs[i]];
     }
 }
 
@@ -220,6 +233,7 @@ void Executor::copy_rs_h2h(const uint32_t* srcs, const uint32_t* dsts, size_t n)
 void Executor::prepare_stack(const BatchPlan& plan, const Inputs& in) {
     if (plan.has_user_masks) throw std::runtime_error("executor: layer stacks take no custom attention masks");
     auto* row_req = reinterpret_cast<int32_t*>(in_host_ + in.off_row_req);
+    auto* prev = reinterpret_cast<int32_t*>(in_host_ + in.off_prev);
     auto* qo = reinterpret_cast<int32_t*>(in_host_ + in.off_qo);
     auto* slot = reinterpret_cast<int32_t*>(in_host_ + in.off_rs_slot);
     auto* fresh = reinterpret_cast<int32_t*>(in_host_ + in.off_rs_fresh);
@@ -232,6 +246,7 @@ void Executor::prepare_stack(const BatchPlan& plan, const Inputs& in) {
         qo[r] = q0;
         for (int i = q0; i < q1; ++i) {
             row_req[i] = r;
+            prev[i] = i > q0 ? static_cast<int32_t>(plan.tokens[i - 1]) : -1;
             if (i > q0 && plan.positions[i] != plan.positions[i - 1] + 1)
                 throw std::runtime_error("executor: a request's rows must be consecutive positions");
         }
@@ -250,6 +265,7 @@ void Executor::prepare_stack(const BatchPlan& plan, const Inputs& in) {
                                      std::to_string(plan.positions[q0]));
         slot[r] = static_cast<int32_t>(s);
         fresh[r] = reset ? 1 : 0;
+        if (!reset) prev[q0] = rs_last_[s];
     }
     qo[plan.R] = plan.N;
     if (recurrent)
@@ -328,7 +344,11 @@ void Executor::prepare_lists(const BatchPlan& plan) {
 void Executor::commit_stack(const BatchPlan& plan) {
     plan_ = nullptr;
     if (rs_slots_ == 0) return;
-    for (int r = 0; r < plan.R; ++r) rs_pos_[plan.rs_slots[r]] = plan.positions[plan.qo_indptr[r + 1] - 1] + 1;
+    for (int r = 0; r < plan.R; ++r) {
+        const int last = plan.qo_indptr[r + 1] - 1;
+        rs_pos_[plan.rs_slots[r]] = plan.positions[last] + 1;
+        rs_last_[plan.rs_slots[r]] = static_cast<int32_t>(plan.tokens[last]);
+    }
 }
 
 void Executor::stack_linear(const Linear& w, const void* act, void* y, int M, int epilogue, const PieHipGlu* glu) {
@@ -347,36 +367,46 @@ void Executor::stack_linear(const Linear& w, const void* act, void* y, int M, in
 // Each token's row through its experts: routes' rows in stack_.routes, their places and weights beside them.
 void Executor::stack_mixture(const StackLayer& w, int N) {
     const MixtureSpec& e = w.spec.moe;
-    const int Hp = model_.ld_x(), ffp = w.w_down.K, ld = pad_to(e.experts, 16);
+    const int Hp = model_.ld_x(), ffp = w.w_down.K, ld = pad_to(e.router_columns(), 16), E = e.all_experts(), routes = N * e.routes();
     PIE_KERNEL(pie_hip_linear_f32out(dt_, stack_.xa, w.w_router, stack_.router, N, ld, Hp, stream_));
-    PIE_KERNEL(pie_hip_moe_route_groups(stack_.router, ld, stack_.route_idx, stack_.route_w, stack_.route_offsets, stack_.route_token,
-                                        stack_.route_pos, N, e.experts, e.top, e.groups, e.keep, e.scale, stream_));
+    if (e.router == RouterKind::CorrectedScores)
+        PIE_KERNEL(pie_hip_moe_route_corrected(stack_.router, ld, w.correction, stack_.route_idx, stack_.route_w, stack_.route_offsets,
+                                               stack_.route_token, stack_.route_pos, N, e.experts, e.top, e.shared_parts(), stream_));
+    else
+        PIE_KERNEL(pie_hip_moe_route_groups(stack_.router, ld, stack_.route_idx, stack_.route_w, stack_.route_offsets, stack_.route_token,
+                                            stack_.route_pos, N, e.experts, e.top, e.groups, e.keep, e.scale, stream_));
+    const bool pair = e.expert == ExpertKind::ClampedPair;
     const PieHipGlu glu{nullptr, e.limit, e.alpha, e.shift};
     if (dt_ == PIE_HIP_DT_F32) {
-        PIE_KERNEL(pie_hip_moe_grouped_linear_f32(static_cast<const float*>(stack_.xa), stack_.route_token, stack_.route_offsets, e.experts, N,
-                                                  static_cast<const uint16_t*>(w.w_up.data), stack_.glu, 2 * ffp, Hp, stream_));
-        PIE_KERNEL(pie_hip_glu_f32(stack_.glu, &glu, static_cast<float*>(stack_.act), N * e.top, ffp, stream_));
-        PIE_KERNEL(pie_hip_moe_grouped_linear_f32(static_cast<const float*>(stack_.act), nullptr, stack_.route_offsets, e.experts, N,
-                                                  static_cast<const uint16_t*>(w.w_down.data), static_cast<float*>(stack_.routes), Hp, ffp,
-                                                  stream_));
+        auto product = [&](const void* act, const int32_t* rows, const Linear& l, float* y, int n, int k, int epilogue) {
+            PIE_KERNEL(pie_hip_moe_grouped_linear_f32(static_cast<const float*>(act), rows, stack_.route_offsets, E, N,
+                                                      static_cast<const uint16_t*>(l.data), y, n, k, epilogue, stream_));
+        };
+        if (pair) {
+            product(stack_.xa, stack_.route_token, w.w_up, stack_.glu, 2 * ffp, Hp, PIE_HIP_EPI_NONE);
+            PIE_KERNEL(pie_hip_glu_f32(stack_.glu, &glu, static_cast<float*>(stack_.act), routes, ffp, stream_));
+        } else {
+            product(stack_.xa, stack_.route_token, w.w_up, static_cast<float*>(stack_.act), ffp, Hp, PIE_HIP_EPI_RELU2);
+        }
+        product(stack_.act, nullptr, w.w_down, static_cast<float*>(stack_.routes), Hp, ffp, PIE_HIP_EPI_NONE);
         return;
     }
-    const int hint = std::max(1, std::min(N, 2 * ((N * e.top + e.experts - 1) / e.experts)));
-    const bool blocks = grouped_in_blocks(N * e.top, e.experts);
+    const int hint = std::max(1, std::min(N, 2 * ((routes + E - 1) / E)));
+    const bool blocks = grouped_in_blocks(routes, E);
     auto grouped = [&](const Linear& l, const void* act, const int32_t* rows, void* y, int epilogue, const PieHipGlu* rule) {
         if (blocks) {
-            PIE_KERNEL(pie_hip_moe_grouped_gemm_mfma(static_cast<const uint16_t*>(act), rows, stack_.route_offsets, e.experts, N * e.top,
-                                                     l.data_tiled ? l.data_tiled : l.data, l.data_bytes() / e.experts,
-                                                     static_cast<uint16_t*>(y), l.N / e.experts, l.K, epilogue, l.data_tiled ? 1 : 0, rule, 0,
+            PIE_KERNEL(pie_hip_moe_grouped_gemm_mfma(static_cast<const uint16_t*>(act), rows, stack_.route_offsets, E, routes,
+                                                     l.data_tiled ? l.data_tiled : l.data, l.data_bytes() / E,
+                                                     static_cast<uint16_t*>(y), l.N / E, l.K, epilogue, l.data_tiled ? 1 : 0, rule, 0,
                                                      stream_));
             return;
         }
-        PIE_KERNEL(pie_hip_moe_grouped_gemm_glu(PIE_HIP_FMT_BF16, static_cast<const uint16_t*>(act), rows, stack_.route_offsets, e.experts,
-                                                hint, l.data_tiled ? l.data_tiled : l.data, l.data_bytes() / e.experts, nullptr, 0, 0, 0,
-                                                static_cast<uint16_t*>(y), l.N / e.experts, l.K, epilogue, l.data_tiled ? 1 : 0, rule,
+        PIE_KERNEL(pie_hip_moe_grouped_gemm_glu(PIE_HIP_FMT_BF16, static_cast<const uint16_t*>(act), rows, stack_.route_offsets, E,
+                                                hint, l.data_tiled ? l.data_tiled : l.data, l.data_bytes() / E, nullptr, 0, 0, 0,
+                                                static_cast<uint16_t*>(y), l.N / E, l.K, epilogue, l.data_tiled ? 1 : 0, rule,
                                                 stream_));
     };
-    grouped(w.w_up, stack_.xa, stack_.route_token, stack_.act, PIE_HIP_EPI_SWIGLU, &glu);
+    grouped(w.w_up, stack_.xa, stack_.route_token, stack_.act, pair ? PIE_HIP_EPI_SWIGLU : PIE_HIP_EPI_RELU2, pair ? &glu : nullptr);
     grouped(w.w_down, stack_.act, nullptr, stack_.routes, PIE_HIP_EPI_NONE, nullptr);
 }
 
@@ -391,7 +421,7 @@ void Executor::stack_latent(const StackLayer& w, int layer, int N, int max_kv_le
     stack_linear(w.w_in, stack_.xa, stack_.in, N);
     const size_t esize = dt_ == PIE_HIP_DT_F32 ? 4 : 2;
     auto rows_of = [&](void* buf, int row, int ld) { return static_cast<unsigned char*>(buf) + static_cast<size_t>(row) * ld * esize; };
-    auto gate_of = [&](int row) { return a.gate ? rows_of(stack_.in, row, s.ld_in) + static_cast<size_t>(s.gate_off) * esize : nullptr; };
+    auto gate_of = [&](int row) { return s.gate_cols ? rows_of(stack_.in, row, s.ld_in) + static_cast<size_t>(s.gate_off) * esize : nullptr; };
     PIE_KERNEL(pie_hip_latent_prep(dt_, stack_.in, w.q_norm, w.kv_norm, rope, slots, stack_.cq, run_pool_[layer], N,
                                    s.ld_in, s.kv_off, a.q_rank, s.ld_cq, a.kv_rank, s.kvp, a.rot_dim, a.rot.dims,
                                    s.ld_row, model_.cfg().rms_eps, stream_));
@@ -403,21 +433,22 @@ void Executor::stack_latent(const StackLayer& w, int layer, int N, int max_kv_le
         if (n <= 0) return;
         PIE_KERNEL(pie_hip_head_linear(dt_, rows_of(stack_.q, r0, s.ld_q), w.w_uk_t, rows_of(stack_.q_lat, r0, s.heads * s.ld_row),
                                        rope ? rope + static_cast<size_t>(r0) * a.rot.dims : nullptr, n, s.heads, s.kvp, s.dimp,
-                                       s.ld_q, s.hd, s.heads * s.ld_row, s.ld_row, s.dimp, a.rot_dim, a.rot.dims, s.rotp, nullptr, 0, stream_));
+                                       s.ld_q, s.hd, s.heads * s.ld_row, s.ld_row, s.dimp, a.rot_dim, a.rot.dims, s.rotp, nullptr, 0, 0, stream_));
         if (matrix)
             PIE_KERNEL(pie_hip_latent_attn_rows(static_cast<const uint16_t*>(stack_.q_lat),
                                                 reinterpret_cast<const uint16_t*>(run_pool_[layer]),
                                                 static_cast<uint16_t*>(stack_.o_lat), pages, row_begin, row_len,
                                                 reinterpret_cast<const int32_t*>(in_dev_ + in.off_row_req),
                                                 reinterpret_cast<const int32_t*>(in_dev_ + in.off_qo), r0, n, s.heads, s.kvp,
-                                                s.rotp, page_size_, static_cast<float>(a.scale), max_len, max_tokens, attn_ws_,
+                                                s.rotp, page_size_, static_cast<float>(a.scale), w.sinks, max_len, max_tokens, attn_ws_,
                                                 attn_ws_bytes_, stream_));
         else
             PIE_KERNEL(pie_hip_latent_attn_rows_plain(dt_, rows_of(stack_.q_lat, r0, s.heads * s.ld_row), run_pool_[layer],
                                                       rows_of(stack_.o_lat, r0, s.heads * s.kvp), pages, row_begin + r0, row_len + r0, n,
-                                                      s.heads, s.kvp, s.ld_row, page_size_, static_cast<float>(a.scale), stream_));
+                                                      s.heads, s.kvp, s.ld_row, page_size_, static_cast<float>(a.scale), w.sinks, stream_));
         PIE_KERNEL(pie_hip_head_linear(dt_, rows_of(stack_.o_lat, r0, s.heads * s.kvp), w.w_uv, rows_of(stack_.o, r0, s.ld_o), nullptr, n,
-                                       s.heads, s.vdp, s.kvp, s.heads * s.kvp, s.kvp, s.ld_o, s.vdp, 0, 0, 0, 0, gate_of(r0), s.ld_in, stream_));
+                                       s.heads, s.vdp, s.kvp, s.heads * s.kvp, s.kvp, s.ld_o, s.vdp, 0, 0, 0, 0, gate_of(r0), s.ld_in,
+                                       s.gate_cols, stream_));
     };
     if (plan_->pure_decode) {
         rows_form(0, N, max_kv_len, 1);
@@ -442,10 +473,10 @@ void Executor::stack_latent(const StackLayer& w, int layer, int N, int max_kv_le
             run_tokens = 1;
             const int ctx = plan_->row_kv_len[q1 - 1];
             expand_lat_.ensure(static_cast<size_t>(ctx) * s.kvp * 2);
-            expand_rot_.ensure(static_cast<size_t>(ctx) * s.rotp * 2);
+            if (s.rotp) expand_rot_.ensure(static_cast<size_t>(ctx) * s.rotp * 2);
             expand_kv_.ensure(static_cast<size_t>(ctx) * w.w_ukv.N * 2);
             auto* lat = static_cast<uint16_t*>(expand_lat_.ptr);
-            auto* rot = static_cast<uint16_t*>(expand_rot_.ptr);
+            auto* rot = s.rotp ? static_cast<uint16_t*>(expand_rot_.ptr) : nullptr;
             auto* kv = static_cast<uint16_t*>(expand_kv_.ptr);
             PIE_KERNEL(pie_hip_latent_gather(reinterpret_cast<const uint16_t*>(run_pool_[layer]),
                                              pages + plan_->row_page_begin[q0], lat, rot, ctx, s.kvp, s.rotp, page_size_, stream_));
@@ -453,8 +484,8 @@ void Executor::stack_latent(const StackLayer& w, int layer, int N, int max_kv_le
                                          PIE_HIP_EPI_NONE, stream_));
             PIE_KERNEL(pie_hip_latent_attn_prefill(static_cast<const uint16_t*>(stack_.q), kv, rot, static_cast<uint16_t*>(stack_.o),
                                                    rope, row_len, q0, q1 - q0, ctx, s.heads, s.dimp, s.rotp, a.rot.dims, s.vdp,
-                                                   s.ld_o, static_cast<float>(a.scale), reinterpret_cast<const uint16_t*>(gate_of(0)),
-                                                   s.ld_in, stream_));
+                                                   s.ld_o, static_cast<float>(a.scale), w.sinks, reinterpret_cast<const uint16_t*>(gate_of(0)),
+                                                   s.ld_in, s.gate_cols, stream_));
         }
         rows_form(run0, N - run0, run_len, run_tokens);
     }
@@ -655,6 +686,20 @@ void Executor::stack_mixer(const StackLayer& w, int run, int N, int max_kv_len, 
     }
 }
 
+// A layer's dense feed-forward on stack_.xa (its down projection's bias is left to what adds y).
+void Executor::stack_dense(const StackLayer& w, void* y, int N) {
+    switch (model_.cfg().ff_act) {
+        case FeedForwardAct::GatedSilu: {
+            const PieHipGlu glu{w.up_bias, INFINITY, 1.f, 0.f};
+            stack_linear(w.w_up, stack_.xa, stack_.act, N, PIE_HIP_EPI_SWIGLU, &glu);
+            break;
+        }
+        case FeedForwardAct::Gelu: stack_linear(w.w_up, stack_.xa, stack_.act, N, PIE_HIP_EPI_GELU); break;
+        case FeedForwardAct::SquaredRelu: stack_linear(w.w_up, stack_.xa, stack_.act, N, PIE_HIP_EPI_RELU2); break;
+    }
+    stack_linear(w.w_down, stack_.act, y, N);
+}
+
 // Layers whose mixer and feed-forward read one norm: both outputs join the stream in one kernel, which norms it
 // for the next layer.
 void Executor::stack_shared_norm(int N, int max_kv_len, const Inputs& in) {
@@ -669,18 +714,78 @@ void Executor::stack_shared_norm(int N, int max_kv_len, const Inputs& in) {
         const StackLayer& w = layer_of(r);
         stack_mixer(w, static_cast<int>(r), N, max_kv_len, in);
         const bool dense = w.spec.ff > 0, mixture = w.spec.moe.experts > 0;
-        if (dense && w.up_bias) {
-            const PieHipGlu glu{w.up_bias, INFINITY, 1.f, 0.f};
-            stack_linear(w.w_up, stack_.xa, stack_.act, N, PIE_HIP_EPI_SWIGLU, &glu);
-        } else if (dense) {
-            stack_linear(w.w_up, stack_.xa, stack_.act, N, m.ff_act == FeedForwardAct::Gelu ? PIE_HIP_EPI_GELU : PIE_HIP_EPI_RELU2);
-        }
-        if (dense) stack_linear(w.w_down, stack_.act, stack_.y2, N);
+        if (dense) stack_dense(w, stack_.y2, N);
         if (mixture) stack_mixture(w, N);
-        const PieHipRoutes routes{stack_.routes, stack_.route_pos, stack_.route_w, w.spec.moe.top, ld};
+        const PieHipRoutes routes{stack_.routes, stack_.route_pos, stack_.route_w, w.spec.moe.routes(), ld};
         PIE_KERNEL(pie_hip_residual_join(dt_, stack_.y, w.wo.N, dense ? stack_.y2 : nullptr, w.w_down.N, w.down_bias,
                                          mixture ? &routes : nullptr, stack_.x, 1, nullptr, nullptr, 0, 0.f,
                                          r + 1 < n_runs ? layer_of(r + 1).pre1 : nullptr, stack_.xa, N, m.hidden, ld, m.rms_eps, stream_));
+    }
+}
+
+// Layers of gated sublayers: the kernel that ends one norms the stream for the next, whose input is the normed row
+// plus a convolution over it and the rows before it — in the same launch where every request brings one row.
+void Executor::stack_gated(int N, int max_kv_len, const Inputs& in) {
+    const ModelConfig& m = model_.cfg();
+    const int H = m.hidden, ld = model_.ld_x(), taps = m.canon_taps;
+    PIE_KERNEL(pie_hip_embed_bigram(reinterpret_cast<const uint32_t*>(in_dev_ + in.off_tokens),
+                                    reinterpret_cast<const int32_t*>(in_dev_ + in.off_prev), model_.embed, m.vocab, m.embed_scale,
+                                    model_.bigram, m.bigram.buckets, m.bigram.mul_prev, m.bigram.mul_cur, model_.embed_norm, stack_.x, N, H,
+                                    ld, m.rms_eps, stream_));
+    struct Sublayer {
+        const float *norm, *canon, *gate_bias;
+        const Linear* gate;
+        size_t state;   // of the convolution
+    };
+    auto sublayer = [&](size_t run, int n) {
+        const StackLayer& w = model_.stack[static_cast<size_t>(model_.runs[run].layer)];
+        return n == 0 ? Sublayer{w.pre1, w.canon1, w.gate1_bias, &w.w_gate1, rs_canon_off_[run][0]}
+                      : Sublayer{w.pre2, w.canon2, w.gate2_bias, &w.w_gate2, rs_canon_off_[run][1]};
+    };
+    // the output of `from` (none at the start: y and routes null) joins the stream, which `to` (null: the last one
+    // has ended) reads
+    auto join = [&](const Sublayer* from, const void* y, const PieHipRoutes* routes, const Sublayer* to) {
+        if (!from && !to) return;
+        PieHipStateRows state{};
+        if (to) {
+            state = state_rows(0, N, in);
+            state.conv_offset = to->state;
+        }
+        const bool fused = to && plan_->pure_decode && taps <= 4;
+        PIE_KERNEL(pie_hip_gated_join(dt_, y, ld, routes, from ? stack_.sub_gate : nullptr, ld, from ? from->gate_bias : nullptr, stack_.x,
+                                      to ? to->norm : nullptr, stack_.h, stack_.xa, fused ? to->canon : nullptr, taps, &state, N, H, ld,
+                                      m.rms_eps, stream_));
+        if (!to) return;
+        if (!fused) {
+            PIE_KERNEL(pie_hip_recent_rows(dt_, stack_.h, to->canon, taps, &state, stack_.xa, H, ld, stream_));
+            if (taps > 1)
+                PIE_KERNEL(pie_hip_delta_conv_state(dt_, stack_.h, rs_base_, rs_stride_, state.conv_offset, state.qo_indptr, state.rs_slot,
+                                                    state.rs_fresh, state.num_requests, ld, H, taps, stream_));
+        }
+        stack_linear(*to->gate, stack_.h, stack_.sub_gate, N);
+    };
+    const size_t n_runs = model_.runs.size();
+    Sublayer now = sublayer(0, 0);
+    join(nullptr, nullptr, nullptr, &now);
+    for (size_t r = 0; r < n_runs; ++r) {
+        const StackLayer& w = model_.stack[static_cast<size_t>(model_.runs[r].layer)];
+        auto finish = [&](const void* y, const PieHipRoutes* routes, bool layer_ends) {
+            const bool more = !layer_ends || r + 1 < n_runs;
+            const Sublayer next = !more ? Sublayer{} : layer_ends ? sublayer(r + 1, 0) : sublayer(r, 1);
+            join(&now, y, routes, more ? &next : nullptr);
+            now = next;
+        };
+        stack_mixer(w, static_cast<int>(r), N, max_kv_len, in);
+        const bool dense = w.spec.ff > 0, mixture = w.spec.moe.experts > 0;
+        finish(stack_.y, nullptr, !dense && !mixture);
+        if (dense) {
+            stack_dense(w, stack_.y, N);
+            finish(stack_.y, nullptr, true);
+        } else if (mixture) {
+            stack_mixture(w, N);
+            const PieHipRoutes routes{stack_.routes, stack_.route_pos, stack_.route_w, w.spec.moe.routes(), ld};
+            finish(nullptr, &routes, true);
+        }
     }
 }
 
@@ -704,16 +809,16 @@ void Executor::stack_body(int N, int S, int max_kv_len) {
                                          begins ? model_.loop_step + static_cast<size_t>(pass) * H : nullptr,
                                          more ? layer_of(run).pre1 : nullptr, stack_.xa, N, H, ldy, ld, m.rms_eps, s));
     };
-    if (m.shared_norm) {
+    if (m.shared_norm || m.gated_sublayers) {
     } else if (m.sandwich_norms) enter(0, nullptr, nullptr, 0, false);
     else PIE_KERNEL(pie_hip_embed_stream(dt_, tokens, model_.embed, stack_.x, stack_.xa, N, H, ld, m.vocab, s));
     for (size_t i = 0; i < model_.rotary.size(); ++i)
         PIE_KERNEL(pie_hip_rotary_table(reinterpret_cast<const int32_t*>(in_dev_ + in.off_positions),
                                         model_.rotary[i].freq, stack_.rotary[i], N, model_.rotary[i].spec.dims,
                                         model_.rotary[i].mscale, s));
-    const int act = m.ff_act == FeedForwardAct::Gelu ? PIE_HIP_EPI_GELU : PIE_HIP_EPI_RELU2;
     if (m.shared_norm) stack_shared_norm(N, max_kv_len, in);
-    for (size_t r = 0; r < n_runs && !m.shared_norm; ++r) {
+    else if (m.gated_sublayers) stack_gated(N, max_kv_len, in);
+    for (size_t r = 0; r < n_runs && !m.shared_norm && !m.gated_sublayers; ++r) {
         const StackLayer& w = layer_of(r);
         stack_mixer(w, static_cast<int>(r), N, max_kv_len, in);
         // y joins the stream; `last`: the layer's last sublayer
@@ -728,8 +833,7 @@ void Executor::stack_body(int N, int S, int max_kv_len) {
         };
         finish(w.norm1, w.wo.N, w.spec.ff == 0);
         if (w.spec.ff > 0) {
-            stack_linear(w.w_up, stack_.xa, stack_.act, N, act);
-            stack_linear(w.w_down, stack_.act, stack_.y, N);
+            stack_dense(w, stack_.y, N);
             finish(w.norm2, w.w_down.N, true);
         }
     }

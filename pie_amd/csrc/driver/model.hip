@@ -139,7 +139,7 @@ void Model::build_tiled_copies(hipStream_t stream) {
         for (Linear* w : {&l.wqkv, &l.wo, &l.wgu, &l.wdown}) linears.push_back(w);
     if (!cfg_.f32())   // (the fp32 products read the row-major weights)
         for (StackLayer& l : stack)
-            for (Linear* w : {&l.w_in, &l.w_uq, &l.wo, &l.w_up, &l.w_down}) linears.push_back(w);
+            for (Linear* w : {&l.w_in, &l.w_uq, &l.wo, &l.w_up, &l.w_down, &l.w_gate1, &l.w_gate2}) linears.push_back(w);
     for (Linear* w : linears) {
         if (!w->data || w->data_tiled || w->N <= 0 || w->N % 16 != 0) continue;
         const size_t row_bytes = w->data_bytes() / static_cast<size_t>(w->N);

@@ -75,15 +75,16 @@ constexpr int pad_latent(int v) {
 }
 struct LatentShape {
     int heads, dimp, rotp, vdp, kvp;   // per-head sizes and the latent, rounded up
-    int kv_off, gate_off, ld_in;       // fused projection: query latent | latent, rotated key part | gates (heads of vdp)
+    int kv_off, gate_off, gate_cols, ld_in;   // fused projection: query latent | latent, rotated key part | gates (heads of
+                                              // gate_cols: vdp, 1 or 0)
     int ld_cq, hd, ld_q;               // query latent rows; q rows: heads of [dimp | rotp]
-    int ld_row;                        // cache row: [kvp | rotp]
+    int ld_row;                        // cache row: [kvp | rotp] (rotp 0: no rotated part)
     int ld_o;                          // attention output rows: heads of vdp
     explicit LatentShape(const LatentAttentionSpec& a)
-        : heads(a.heads), dimp(pad_to(a.dim, 32)), rotp(a.rot_dim > 0 ? pad_to(a.rot_dim, 32) : 32), vdp(pad_to(a.vdim, 32)),
+        : heads(a.heads), dimp(pad_to(a.dim, 32)), rotp(pad_to(a.rot_dim, 32)), vdp(pad_to(a.vdim, 32)),
           kvp(pad_latent(a.kv_rank)), kv_off(pad_to(a.q_rank, 16)),
           gate_off(pad_to(kv_off + (a.kv_from < 0 ? a.kv_rank + a.rot_dim : 0), 8)),
-          ld_in(pad_to(gate_off + (a.gate ? heads * vdp : 0), 16)),
+          gate_cols(a.gate == OutputGate::PerValue ? vdp : a.gate == OutputGate::PerHead ? 1 : 0), ld_in(pad_to(gate_off + heads * gate_cols, 16)),
           ld_cq(pad_to(a.q_rank, 128)), hd(dimp + rotp), ld_q(heads * hd), ld_row(kvp + rotp),
           ld_o(pad_to(heads * vdp, 128)) {}
 };
@@ -158,12 +159,16 @@ struct StackLayer {
     Linear w_up, w_down;    // feed-forward (none: data null).  Gated: w_up's rows are (gate_i, up_i) pairs; a mixture's
                             // experts are stacked along the rows
     float *up_bias = nullptr, *down_bias = nullptr;   // gated: in the order of the rows
-    uint16_t* w_router = nullptr;                     // mixture: [experts rounded up to 16, width]
+    uint16_t* w_router = nullptr;                     // mixture: [router columns rounded up to 16, width]
+    float* correction = nullptr;                      // mixture: added to the scores for the choice (CorrectedScores)
+    // gated sublayers: gate product and bias, convolution [taps, width] ahead of mixer and feed-forward
+    Linear w_gate1, w_gate2;
+    float *gate1_bias = nullptr, *gate2_bias = nullptr, *canon1 = nullptr, *canon2 = nullptr;
     // latent attention
     Linear w_uq;
     Linear w_ukv;                                // [heads * (dimp + vdp), kvp]: keys and values out of the latent
     uint16_t *w_uk_t = nullptr, *w_uv = nullptr; // per head [kvp, dimp] (transposed keys) and [vdp, kvp]
-    float *q_norm = nullptr, *kv_norm = nullptr;
+    float *q_norm = nullptr, *kv_norm = nullptr, *sinks = nullptr;
     int rotary = -1;                             // index into Model::rotary
     // channel delta
     uint16_t *w_decay = nullptr, *w_gate = nullptr;   // second factors of the low-rank decay and output gate
@@ -227,6 +232,8 @@ class Model {
     std::vector<RotaryTable> rotary;   // the stack's distinct rotations
     Linear head;                       // lm_head, padded
     float* stack_norm = nullptr;       // norm ahead of it
+    uint16_t* bigram = nullptr;        // [buckets + 1, hidden]
+    float* embed_norm = nullptr;       // norm of the embedding (gated sublayers)
     float* loop_step = nullptr;        // [times, hidden]: added ahead of every pass of the loop
     std::vector<LayerRun> runs;        // the layers in the order they are run
     int ld_x() const { return pad_to(cfg_.hidden, 128); }

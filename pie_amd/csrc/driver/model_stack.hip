@@ -159,7 +159,42 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
     embed = device_matrix("embed", static_cast<size_t>(V) * H, 1,
                           [&](std::vector<uint16_t>& host) { host = matrix("embed", V, H).v; });
     linear(head, "head", pad_to(V, 16), Hp, H, [&](auto put) { plain_rows(put, "head", 0, V, H); });
-    stack_norm = vec("final.norm", H, ones);
+    // a norm with one weight for all columns, spread over them
+    auto scalar_norm = [&](const std::string& name) {
+        float g = 1.f;
+        if (!random) {
+            const StTensor& t = snap->at(name);
+            if (t.elems() != 1) throw std::runtime_error("snapshot: tensor '" + name + "' has an unexpected shape");
+            std::vector<uint16_t> staging;
+            if (t.dtype == "F32") std::memcpy(&g, t.data, 4);
+            else g = bf16_value(as_bf16(t, staging)[0]);
+        }
+        const std::vector<float> v(static_cast<size_t>(H), g);
+        float* d = static_cast<float*>(alloc(4 * v.size(), name));
+        PIE_HIP_CHECK(hipMemcpyAsync(d, v.data(), 4 * v.size(), hipMemcpyHostToDevice, stream));
+        PIE_HIP_CHECK(hipStreamSynchronize(stream));
+        return d;
+    };
+    // a convolution's taps, one after the other: [width, taps] -> [taps, width] fp32
+    auto tap_major = [&](const std::string& name, int taps) {
+        std::vector<float> v(static_cast<size_t>(taps) * H, 0.25f);
+        if (!random) {
+            const HostMatrix m = matrix(name, H, taps);
+            for (int c = 0; c < H; ++c)
+                for (int j = 0; j < taps; ++j) v[static_cast<size_t>(j) * H + c] = bf16_value(m.row(c)[j]);
+        }
+        float* d = static_cast<float*>(alloc(4 * v.size(), name));
+        PIE_HIP_CHECK(hipMemcpyAsync(d, v.data(), 4 * v.size(), hipMemcpyHostToDevice, stream));
+        PIE_HIP_CHECK(hipStreamSynchronize(stream));
+        return d;
+    };
+    stack_norm = cfg.gated_sublayers ? scalar_norm("final.norm") : vec("final.norm", H, ones);
+    if (cfg.gated_sublayers) embed_norm = scalar_norm("embed.norm");
+    if (cfg.bigram.buckets > 0) {
+        if (cfg.bigram.buckets >= (1ull << 31) - 1) throw std::runtime_error("model: too many bigram buckets");
+        const int rows = static_cast<int>(cfg.bigram.buckets) + 1;
+        bigram = device_matrix("bigram", static_cast<size_t>(rows) * H, 1, [&](std::vector<uint16_t>& host) { host = matrix("bigram", rows, H).v; });
+    }
 
     runs = cfg.layer_runs();
     if (cfg.loop.stop > cfg.loop.start)
@@ -179,7 +214,17 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
         };
         const char *post1 = cfg.sandwich_norms ? "norm1b" : "norm1", *post2 = cfg.sandwich_norms ? "norm2b" : "norm2";
         const std::string p = "l" + std::to_string(l) + ".", mix = p + "mix.";
-        if (!cfg.shared_norm) w.norm1 = vec(p + post1, H, ones);
+        // what surrounds sublayer n of a gated pair
+        auto gated_sublayer = [&](const std::string& n, float*& norm, float*& canon, Linear& gate, float*& bias) {
+            norm = scalar_norm(p + "norm" + n);
+            canon = tap_major(p + "canon" + n, cfg.canon_taps);
+            linear(gate, p + "rg" + n, Hp, Hp, H, [&](auto put) { plain_rows(put, p + "rg" + n, 0, H, H); });
+            bias = vec(p + "rg" + n + ".b", H, [](size_t) { return 0.f; });
+        };
+        if (cfg.gated_sublayers) {
+            gated_sublayer("1", w.pre1, w.canon1, w.w_gate1, w.gate1_bias);
+            if (w.spec.ff > 0 || w.spec.moe.experts > 0) gated_sublayer("2", w.pre2, w.canon2, w.w_gate2, w.gate2_bias);
+        } else if (!cfg.shared_norm) w.norm1 = vec(p + post1, H, ones);
         if (cfg.sandwich_norms || cfg.shared_norm) w.pre1 = vec(p + "norm1", H, ones);
         if (w.spec.mixer == MixerKind::LatentAttention) {
             const LatentAttentionSpec& a = w.spec.latent;
@@ -200,7 +245,8 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
                     for (int r = 0; r < a.kv_rank + a.rot_dim; ++r)
                         put(s.kv_off + (r < a.kv_rank ? r : a.kv_rank + rotated_place(r - a.kv_rank)), 0, m.row(r), H);
                 }
-                if (a.gate) {
+                if (a.gate == OutputGate::PerHead) plain_rows(put, mix + "g", s.gate_off, a.heads, H);
+                if (a.gate == OutputGate::PerValue) {
                     const HostMatrix m = matrix(mix + "g", a.heads * a.vdim, H);
                     for (int r = 0; r < a.heads * a.vdim; ++r) put(s.gate_off + r / a.vdim * s.vdp + r % a.vdim, 0, m.row(r), H);
                 }
@@ -211,6 +257,7 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
                     for (int i = 0; i < a.dim + a.rot_dim; ++i)
                         put(h * s.hd + (i < a.dim ? i : s.dimp + rotated_place(i - a.dim)), 0, m.row(h * (a.dim + a.rot_dim) + i), a.q_rank);
             });
+            if (a.sinks) w.sinks = vec(mix + "sink", a.heads, [](size_t) { return 0.f; });
             HostMatrix uk, uv;
             if (!random) {
                 uk = matrix(mix + "uk", a.heads * a.dim, a.kv_rank);
@@ -402,22 +449,41 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
         }
         if (w.spec.moe.experts > 0) {
             const MixtureSpec& e = w.spec.moe;
-            const int ff = e.ff, ffp = pad_to(ff, 128), rows = pad_to(e.experts, 16);
+            const int ff = e.ff, ffp = e.padded_ff(), rows = pad_to(e.router_columns(), 16), parts = e.shared_parts();
+            const std::string sh = p + "mlp.shared.";
             decode_bytes_ += static_cast<size_t>(rows) * Hp * 2;
             w.w_router = device_matrix(p + "mlp.router", static_cast<size_t>(rows) * Hp, H, [&](std::vector<uint16_t>& host) {
                 const HostMatrix m = matrix(p + "mlp.router", e.experts, H);
                 for (int r = 0; r < e.experts; ++r) std::memcpy(&host[static_cast<size_t>(r) * Hp], m.row(r), static_cast<size_t>(H) * 2);
+                if (parts) std::memcpy(&host[static_cast<size_t>(e.experts) * Hp], matrix(sh + "sg", 1, H).row(0), static_cast<size_t>(H) * 2);
             });
-            linear(w.w_up, p + "mlp.experts.up", e.experts * 2 * ffp, Hp, H, [&](auto put) {
-                for (int i = 0; i < e.experts; ++i) paired_rows(put, p + "mlp.e" + std::to_string(i) + ".", i * 2 * ffp, ff);
+            if (e.router == RouterKind::CorrectedScores) w.correction = vec(p + "mlp.correction", e.experts, [](size_t) { return 0.f; });
+            const bool pair = e.expert == ExpertKind::ClampedPair;
+            const int up_rows = (pair ? 2 : 1) * ffp;   // of an expert
+            linear(w.w_up, p + "mlp.experts.up", e.all_experts() * up_rows, Hp, H, [&](auto put) {
+                if (parts) {   // (part i's rows follow part i - 1's: up_rows is ffp for experts of one matrix)
+                    if (pair) throw std::runtime_error("model: shared experts are of one matrix");
+                    plain_rows(put, sh + "up", 0, e.shared_ff, H);
+                }
+                for (int i = 0; i < e.experts; ++i) {
+                    const std::string at = p + "mlp.e" + std::to_string(i) + ".";
+                    if (pair) paired_rows(put, at, (parts + i) * up_rows, ff);
+                    else plain_rows(put, at + "up", (parts + i) * up_rows, ff, H);
+                }
             });
-            linear(w.w_down, p + "mlp.experts.down", e.experts * Hp, ffp, ff, [&](auto put) {
-                for (int i = 0; i < e.experts; ++i) plain_rows(put, p + "mlp.e" + std::to_string(i) + ".down", i * Hp, H, ff);
+            linear(w.w_down, p + "mlp.experts.down", e.all_experts() * Hp, ffp, ff, [&](auto put) {
+                if (parts) {
+                    const HostMatrix m = matrix(sh + "down", H, e.shared_ff);
+                    for (int i = 0; i < parts; ++i)
+                        for (int r = 0; r < H; ++r) put(i * Hp + r, 0, m.row(r) + i * ffp, std::min(ffp, e.shared_ff - i * ffp));
+                }
+                for (int i = 0; i < e.experts; ++i) plain_rows(put, p + "mlp.e" + std::to_string(i) + ".down", (parts + i) * Hp, H, ff);
             });
         } else if (w.spec.ff > 0 && cfg.ff_act == FeedForwardAct::GatedSilu) {
             const int ff = w.spec.ff, ffp = pad_to(ff, 128);
             linear(w.w_up, p + "mlp.up", 2 * ffp, Hp, H, [&](auto put) { paired_rows(put, p + "mlp.", 0, ff); });
             linear(w.w_down, p + "mlp.down", Hp, ffp, ff, [&](auto put) { plain_rows(put, p + "mlp.down", 0, H, ff); });
+            if (!cfg.ff_biases) continue;   // (nothing else of the layer is left to load)
             std::vector<float> b(static_cast<size_t>(2 * ffp), 0.f);
             if (!random) {
                 int half = 0;

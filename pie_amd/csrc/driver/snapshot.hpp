@@ -360,6 +360,12 @@ inline int json_size(const Json& j, const std::string& key, const std::string& a
         throw std::runtime_error("snapshot: " + at + " needs an integer '" + key + "'");
     return static_cast<int>(v->num);
 }
+inline std::uint64_t json_count(const Json& j, const std::string& key, const std::string& at) {
+    const Json* v = j.get(key);
+    if (!v || v->kind != Json::Number || !(v->num >= 0.0) || v->num > 9.0e15 || v->num != static_cast<double>(static_cast<std::uint64_t>(v->num)))
+        throw std::runtime_error("snapshot: " + at + " needs a whole number '" + key + "' that is not negative");
+    return static_cast<std::uint64_t>(v->num);
+}
 inline double json_number(const Json& j, const std::string& key, const std::string& at) {
     const Json* v = j.get(key);
     if (!v || v->kind != Json::Number) throw std::runtime_error("snapshot: " + at + " needs a number '" + key + "'");
@@ -429,10 +435,22 @@ inline DecayMemorySpec parse_retention(const Json& j, const std::string& at) {
     return d;
 }
 
-inline MixtureSpec parse_mixture(const Json& j, const std::string& at) {
+inline MixtureSpec parse_mixture(const Json& j, const std::string& at, RouterKind kind, ExpertKind form) {
     MixtureSpec e;
+    e.router = kind;
+    e.expert = form;
     const Json &expert = json_object(j, "expert", at), &router = json_object(j, "router", at);
     e.ff = json_size(expert, "ff", at + " expert");
+    if (kind == RouterKind::CorrectedScores) {
+        e.experts = json_size(router, "experts", at + " router");
+        e.top = json_size(router, "top", at + " router");
+        if (const Json* shared = j.get("shared"); shared && shared->kind == Json::Object) {
+            e.shared_ff = json_size(*shared, "ff", at + " shared");
+            if (e.shared_ff <= 0) throw std::runtime_error("snapshot: " + at + ": shared.ff must be positive");
+        }
+        if (e.experts <= 0) throw std::runtime_error("snapshot: " + at + ": router.experts must be positive");
+        return e;
+    }
     e.limit = static_cast<float>(json_number(expert, "limit", at + " expert"));
     e.alpha = 1.702f;
     e.shift = 1.f;
@@ -460,7 +478,7 @@ inline const std::vector<MixerReader>& mixer_registry() {
              auto& a = l.latent;
              a.heads = json_size(j, "heads", at);
              a.dim = json_size(j, "dim", at);
-             a.rot_dim = json_size(j, "rot_dim", at);
+             if (j.get("rot_dim")) a.rot_dim = json_size(j, "rot_dim", at);   // (left out: no rotated part)
              a.vdim = json_size(j, "vdim", at);
              a.q_rank = json_size(j, "q_rank", at);
              a.kv_rank = json_size(j, "kv_rank", at);
@@ -529,29 +547,49 @@ struct StackArchitecture {
     bool sandwich_norms;
     FeedForwardAct ff_act;
     bool shared_norm = false;
-    bool gated_latents = false;   // latent attention with an output gate and half-split rotation
+    bool half_split_latents = false;   // rotation of latent attention
+    OutputGate latent_gate = OutputGate::None;
+    bool latent_sinks = false;
+    bool ff_biases = false;
+    bool gated_sublayers = false;
+    RouterKind router = RouterKind::GroupSoftmax;
+    ExpertKind expert = ExpertKind::ClampedPair;
 };
 inline const std::vector<StackArchitecture>& stack_registry() {
     static const std::vector<StackArchitecture> table = {
         {"Varasun", "varasun", false, FeedForwardAct::SquaredRelu},
         {"Lofudra", "lofudra", true, FeedForwardAct::Gelu},
-        {"Fobanex", "fobanex", false, FeedForwardAct::GatedSilu, true, true},
+        {"Fobanex", "fobanex", false, FeedForwardAct::GatedSilu, true, true, OutputGate::PerValue, false, true},
+        {"Minodra", "minodra", false, FeedForwardAct::GatedSilu, false, false, OutputGate::PerHead, true, false, true, RouterKind::CorrectedScores,
+         ExpertKind::SquaredRelu},
     };
     return table;
 }
 
 // {"architecture", "width", "vocab", "norm": {"eps"}, "logit_scale", "logit_softcap",
-//  "loop": {"start", "stop", "times"}, "embedding": {"scale"},
+//  "loop": {"start", "stop", "times"}, "embedding": {"scale", "bigram": {"buckets", "mul_prev", "mul_cur"}},
+//  "canon": {"taps"},
 //  "layers": [{"type", "mixer": {...}, "mlp": {"kind": "dense", "ff"} | {"kind": "moe", "expert": {"ff", "limit"},
-//              "router": {"experts", "top", "scale", "groups": {"count", "keep"}}} | null}, ...]}
+//              "router": {"experts", "top", "scale", "groups": {"count", "keep"}}, "shared": {"ff"}} | null}, ...]}
 inline void apply_stack_config(ModelConfig& m, const Json& c, const StackArchitecture& a) {
     m.arch = a.arch;
     m.sandwich_norms = a.sandwich_norms;
     m.ff_act = a.ff_act;
     m.shared_norm = a.shared_norm;
+    m.ff_biases = a.ff_biases;
+    m.gated_sublayers = a.gated_sublayers;
+    m.canon_taps = a.gated_sublayers ? json_size(json_object(c, "canon", "config.json"), "taps", "canon") : 0;
     m.embed_scale = 1.f;
-    if (const Json* e = c.get("embedding"); a.shared_norm && e && e->kind == Json::Object)
+    m.bigram = BigramSpec{};
+    if (const Json* e = c.get("embedding"); (a.shared_norm || a.gated_sublayers) && e && e->kind == Json::Object) {
         m.embed_scale = static_cast<float>(e->number_or("scale", 1.0));
+        if (const Json* b = e->get("bigram"); a.gated_sublayers && b && b->kind == Json::Object) {
+            m.bigram.buckets = json_count(*b, "buckets", "embedding.bigram");
+            m.bigram.mul_prev = json_count(*b, "mul_prev", "embedding.bigram");
+            m.bigram.mul_cur = json_count(*b, "mul_cur", "embedding.bigram");
+            if (m.bigram.buckets == 0) throw std::runtime_error("snapshot: embedding.bigram.buckets must be positive");
+        }
+    }
     m.hidden = json_size(c, "width", "config.json");
     m.vocab = json_size(c, "vocab", "config.json");
     const Json* norm = c.get("norm");
@@ -582,14 +620,16 @@ inline void apply_stack_config(ModelConfig& m, const Json& c, const StackArchite
                 known = true;
             }
         if (!known) throw std::runtime_error("snapshot: " + at + ": unknown mixer '" + type + "'");
-        l.latent.gate = l.latent.half_split = a.gated_latents;
+        l.latent.half_split = a.half_split_latents;
+        l.latent.gate = a.latent_gate;
+        l.latent.sinks = a.latent_sinks;
         if (const Json* mlp = j.get("mlp"); mlp && mlp->kind == Json::Object) {
             const std::string kind = mlp->string_or("kind", "");
             if (kind == "dense") {
                 l.ff = json_size(*mlp, "ff", at + " mlp");
                 if (l.ff <= 0) throw std::runtime_error("snapshot: " + at + ": mlp.ff must be positive");
-            } else if (kind == "moe" && a.shared_norm) {
-                l.moe = parse_mixture(*mlp, at + " mlp");
+            } else if (kind == "moe" && (a.shared_norm || a.gated_sublayers)) {
+                l.moe = parse_mixture(*mlp, at + " mlp", a.router, a.expert);
             } else {
                 throw std::runtime_error("snapshot: " + at + ": unknown mlp kind '" + kind + "'");
             }

@@ -83,8 +83,8 @@ struct HeadArgs {
     const float* rope_table;   // (used when rotp > 0 and rot_dims > 0)
     int M, heads, C, K, ld_act, act_stride, ld_y, y_stride;
     int rot_off, rot_dim, rot_dims, rotp;
-    const void* gate;          // logistic gates of the outputs [M, ld_gate], heads C apart (null: none)
-    int ld_gate;
+    const void* gate;          // logistic gates of the outputs [M, ld_gate] (null: none)
+    int ld_gate, gate_cols;    // per head C (one per output) or 1
 };
 
 template <class T>
@@ -151,7 +151,9 @@ __global__ __launch_bounds__(kWave) void head_linear_mfma_kernel(const HeadArgs 
         if (m >= a.M) continue;
         uint16_t* yp = static_cast<uint16_t*>(a.y) + static_cast<size_t>(m) * a.ld_y + static_cast<size_t>(h) * a.y_stride + c0 + 4 * g;
         f32x4_t v = acc[t];
-        if (a.gate) {
+        if (a.gate && a.gate_cols == 1) {
+            v *= sigmoid_f32(bf16_bits_to_f32(static_cast<const uint16_t*>(a.gate)[static_cast<size_t>(m) * a.ld_gate + h]));
+        } else if (a.gate) {
             const u32x2_t r = *reinterpret_cast<const u32x2_t*>(static_cast<const uint16_t*>(a.gate) + static_cast<size_t>(m) * a.ld_gate +
                                                                 h * a.C + c0 + 4 * g);
             v *= f32x4_t{sigmoid_f32(bf16_lo(r.x)), sigmoid_f32(bf16_hi(r.x)), sigmoid_f32(bf16_lo(r.y)), sigmoid_f32(bf16_hi(r.y))};
@@ -177,7 +179,8 @@ __global__ __launch_bounds__(256) void head_linear_f32_kernel(const HeadArgs a) 
 #pragma unroll
             for (int e = 0; e < 8; ++e) acc = fmaf(row[k + e], w[e], acc);
         }
-        if (a.gate) acc /= 1.f + expf(-static_cast<const float*>(a.gate)[static_cast<size_t>(m) * a.ld_gate + h * a.C + c]);
+        if (a.gate)
+            acc /= 1.f + expf(-static_cast<const float*>(a.gate)[static_cast<size_t>(m) * a.ld_gate + (a.gate_cols == 1 ? h : h * a.C + c)]);
         dst[c] = acc;
     }
     if (a.rotp > 0) head_rotated_part<float>(a, h, m, m + 1, 0, 1);
@@ -190,7 +193,7 @@ template <class T>
 __global__ __launch_bounds__(kPlainThreads) void latent_rows_plain_kernel(
     const T* __restrict__ q, const T* __restrict__ pool, T* __restrict__ o, const uint32_t* __restrict__ page_indices,
     const uint32_t* __restrict__ row_begin, const int32_t* __restrict__ row_len, int heads, int kvp, int ld_row, int ps,
-    float scale) {
+    float scale, const float* __restrict__ sinks) {
     extern __shared__ float sm[];
     float* qrow = sm;                      // ld_row
     float* prob = sm + ld_row;             // kPlainThreads
@@ -244,7 +247,11 @@ __global__ __launch_bounds__(kPlainThreads) void latent_rows_plain_kernel(
             acc[c] = a;
         }
     }
-    const float inv = sum > 0.f ? 1.f / sum : 0.f;
+    float inv = sum > 0.f ? 1.f / sum : 0.f;
+    if (sinks) {   // (in the units of the larger of the two)
+        const float top = fmaxf(mx, sinks[h]), w = expf(mx - top);
+        inv = w / (sum * w + expf(sinks[h] - top));
+    }
     T* op = o + (static_cast<size_t>(n) * heads + h) * kvp;
 #pragma unroll
     for (int c = 0; c < kPlainCols; ++c) {
@@ -279,7 +286,7 @@ extern "C" int pie_hip_latent_prep(int dtype, const void* fused, const float* q_
 extern "C" int pie_hip_head_linear(int dtype, const void* act, const uint16_t* w_bf16, void* y,
                                    const float* rope_table, int M, int heads, int C, int K, int ld_act,
                                    int act_stride, int ld_y, int y_stride, int rot_off, int rot_dim, int rot_dims,
-                                   int rotp, const void* gate, int ld_gate, void* stream) {
+                                   int rotp, const void* gate, int ld_gate, int gate_cols, void* stream) {
     if (!act || !w_bf16 || !y || M <= 0 || heads <= 0 || C <= 0 || K <= 0) return PIE_HIP_ERR_INVALID;
     if (C % 16 != 0 || K % 32 != 0 || ld_act % 8 != 0 || act_stride % 8 != 0 || ld_y % 8 != 0 || y_stride % 8 != 0)
         return PIE_HIP_ERR_UNSUPPORTED;
@@ -287,9 +294,10 @@ extern "C" int pie_hip_head_linear(int dtype, const void* act, const uint16_t* w
     if (rotp > 0 && ((rot_dims > 0 && !rope_table) || rot_dims > rot_dim || rot_dims % 2 != 0 || rotp < rot_dim || y_stride < C + rotp ||
                        act_stride < rot_off + rot_dim))
         return PIE_HIP_ERR_INVALID;
-    if (gate && (ld_gate < heads * C || ld_gate % 4 != 0 || reinterpret_cast<uintptr_t>(gate) % 8 != 0)) return PIE_HIP_ERR_INVALID;
+    if (gate && ((gate_cols != 1 && gate_cols != C) || ld_gate < heads * gate_cols)) return PIE_HIP_ERR_INVALID;
+    if (gate && gate_cols == C && (ld_gate % 4 != 0 || reinterpret_cast<uintptr_t>(gate) % 8 != 0)) return PIE_HIP_ERR_INVALID;
     const HeadArgs a{act, w_bf16, y, rope_table, M, heads, C, K, ld_act, act_stride, ld_y, y_stride, rot_off, rot_dim,
-                     rot_dims, rotp, gate, ld_gate};
+                     rot_dims, rotp, gate, ld_gate, gate_cols};
     hipStream_t s = static_cast<hipStream_t>(stream);
     if (heads > 65535) return PIE_HIP_ERR_UNSUPPORTED;
     if (dtype == PIE_HIP_DT_F32) {
@@ -312,7 +320,7 @@ extern "C" int pie_hip_head_linear(int dtype, const void* act, const uint16_t* w
 extern "C" int pie_hip_latent_attn_rows_plain(int dtype, const void* q, const void* pool, void* o,
                                               const uint32_t* kv_page_indices, const uint32_t* row_page_begin,
                                               const int32_t* row_kv_len, int num_rows, int heads, int kvp, int ld_row,
-                                              int page_size, float scale, void* stream) {
+                                              int page_size, float scale, const float* sinks, void* stream) {
     if (!q || !pool || !o || !kv_page_indices || !row_page_begin || !row_kv_len || num_rows <= 0 || heads <= 0 ||
         kvp <= 0 || ld_row < kvp || page_size <= 0)
         return PIE_HIP_ERR_INVALID;
@@ -323,6 +331,6 @@ extern "C" int pie_hip_latent_attn_rows_plain(int dtype, const void* q, const vo
                      hipLaunchKernelGGL(latent_rows_plain_kernel<T>, dim3(heads, num_rows), dim3(kPlainThreads), smem,
                                         static_cast<hipStream_t>(stream), static_cast<const T*>(q),
                                         static_cast<const T*>(pool), static_cast<T*>(o), kv_page_indices,
-                                        row_page_begin, row_kv_len, heads, kvp, ld_row, page_size, scale));
+                                        row_page_begin, row_kv_len, heads, kvp, ld_row, page_size, scale, sinks));
     return launch_status();
 }

@@ -39,7 +39,15 @@ struct LatentRowsArgs {
     const int32_t* qo_indptr;
     int row0, num_rows, heads, head_groups, heads_per_tile, tokens_per_tile, ps, ps_shift, steps_per_split, nsplit;
     float scale_log2e;
+    const float* sinks;       // [heads] (null: none); with partial results the merge adds them
 };
+
+// What the weighted sum is multiplied by: its sum of exponentials l, taken at m (in powers of two), and a sink's
+// join in the units of the larger of m and the sink.
+__device__ __forceinline__ float sink_inverse(float m, float l, float sink_log2) {
+    const float top = fmaxf(m, sink_log2), w = exp2f(m - top);
+    return w / (l * w + exp2f(sink_log2 - top));
+}
 
 // Keys of one split: a decode row cuts its own keys evenly (steps_per_split 0), whatever the bound
 // the launch was planned with; portions take the planned length.
@@ -49,7 +57,7 @@ __device__ __forceinline__ int split_keys(int keys, int nsplit, int steps_per_sp
     return max(1, (steps + nsplit - 1) / nsplit) * kStep;
 }
 
-// C: latent columns / 64; R: rotated columns / 32; MT: 16-pair tiles per block
+// C: latent columns / 64; R: rotated columns / 32 (0: the rows are latents only); MT: 16-pair tiles per block
 template <int C, int R, int MT>
 __global__ __launch_bounds__(kBlock, 2) void latent_rows_kernel(const LatentRowsArgs a) {
     constexpr int LD = 64 * C + 32 * R, STRIDE = LD + 8, KS = 2 * C + R;
@@ -251,7 +259,8 @@ __global__ __launch_bounds__(kBlock, 2) void latent_rows_kernel(const LatentRows
         const size_t out = pair_out(m);
         const float l = s_l[m];
         if (a.o) {
-            const float inv = l > 0.f ? 1.f / l : 0.f;
+            const float inv = a.sinks ? sink_inverse(s_m[m], l, a.sinks[h0 + m % a.heads_per_tile] * 1.4426950408889634f)
+                              : l > 0.f ? 1.f / l : 0.f;
 #pragma unroll
             for (int c = 0; c < C; ++c) {
                 const f32x4_t v = acc[c][t];
@@ -275,15 +284,17 @@ __global__ __launch_bounds__(kBlock, 2) void latent_rows_kernel(const LatentRows
 // thread.  A row has as many pieces as splits start before its last key.
 __global__ void latent_merge_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
                                     const int32_t* __restrict__ row_len, uint16_t* __restrict__ o, int row0, int heads,
-                                    int kvp, int nsplit, int steps_per_split) {
+                                    int kvp, int nsplit, int steps_per_split, const float* __restrict__ sinks) {
     const size_t out = static_cast<size_t>(row0) * heads + blockIdx.x;
     const int len = row_len[out / heads], keys_per_split = split_keys(len, nsplit, steps_per_split);
     const int ns = min(nsplit, (len + keys_per_split - 1) / keys_per_split);
     const float* ml = part_ml + out * nsplit * 2;
     float mx = -INFINITY;
     for (int s = 0; s < ns; ++s) mx = fmaxf(mx, ml[2 * s]);
+    const float sink = sinks ? sinks[out % heads] * 1.4426950408889634f : -INFINITY;
+    mx = fmaxf(mx, sink);
     const float safe = mx == -INFINITY ? 0.f : mx;
-    float l = 0.f;
+    float l = exp2f(sink - safe);
     f32x4_t v = {0.f, 0.f, 0.f, 0.f};
     const float* po = part_o + out * nsplit * kvp + 4 * threadIdx.x;
 #pragma unroll 4
@@ -334,7 +345,7 @@ int launch_latent_rows(const LatentRowsArgs& a, const LatentPlan& p, hipStream_t
 using namespace pie_hip;
 
 extern "C" int pie_hip_latent_attn_rows_supported(int kvp, int rotp) {
-    if (rotp != 32 && rotp != 64) return 0;
+    if (rotp != 0 && rotp != 32 && rotp != 64) return 0;
     return kvp == 64 || kvp == 128 || kvp == 192 || kvp == 256 || kvp == 384 || kvp == 512;
 }
 
@@ -349,8 +360,8 @@ extern "C" int pie_hip_latent_attn_rows(const uint16_t* q, const uint16_t* pool,
                                         const uint32_t* kv_page_indices, const uint32_t* row_page_begin,
                                         const int32_t* row_kv_len, const int32_t* row_req, const int32_t* qo_indptr,
                                         int row0, int num_rows, int heads, int kvp, int rotp, int page_size,
-                                        float scale, int max_kv_len, int max_tokens_per_req, void* workspace,
-                                        size_t workspace_bytes, void* stream) {
+                                        float scale, const float* sinks, int max_kv_len, int max_tokens_per_req,
+                                        void* workspace, size_t workspace_bytes, void* stream) {
     if (!q || !pool || !o || !kv_page_indices || !row_page_begin || !row_kv_len || row0 < 0 || num_rows <= 0 ||
         heads <= 0 || page_size <= 0 || max_tokens_per_req <= 0)
         return PIE_HIP_ERR_INVALID;
@@ -362,7 +373,7 @@ extern "C" int pie_hip_latent_attn_rows(const uint16_t* q, const uint16_t* pool,
                      max_tokens_per_req > 1 ? row_req : nullptr, qo_indptr, row0, num_rows, heads, p.head_groups,
                      p.heads_per_tile, p.tokens_per_tile, page_size,
                      (page_size & (page_size - 1)) == 0 ? __builtin_ctz(static_cast<unsigned>(page_size)) : -1, p.steps_per_split, p.nsplit,
-                     scale * 1.4426950408889634f};
+                     scale * 1.4426950408889634f, sinks};
     if (p.nsplit > 1) {
         if (!workspace || workspace_bytes < pie_hip_latent_attn_rows_workspace_bytes(num_rows, heads, kvp, max_kv_len, max_tokens_per_req))
             return PIE_HIP_ERR_INVALID;
@@ -376,11 +387,12 @@ extern "C" int pie_hip_latent_attn_rows(const uint16_t* q, const uint16_t* pool,
     int st = PIE_HIP_ERR_UNSUPPORTED;
 #define PIE_LATENT_CASE(CC, RR) \
     if (kvp == 64 * CC && rotp == 32 * RR) st = launch_latent_rows<CC, RR>(a, p, s);
+    PIE_LATENT_CASE(1, 0) PIE_LATENT_CASE(2, 0) PIE_LATENT_CASE(3, 0) PIE_LATENT_CASE(4, 0) PIE_LATENT_CASE(6, 0) PIE_LATENT_CASE(8, 0)
     PIE_LATENT_CASE(1, 1) PIE_LATENT_CASE(2, 1) PIE_LATENT_CASE(3, 1) PIE_LATENT_CASE(4, 1) PIE_LATENT_CASE(6, 1) PIE_LATENT_CASE(8, 1)
     PIE_LATENT_CASE(1, 2) PIE_LATENT_CASE(2, 2) PIE_LATENT_CASE(3, 2) PIE_LATENT_CASE(4, 2) PIE_LATENT_CASE(6, 2) PIE_LATENT_CASE(8, 2)
 #undef PIE_LATENT_CASE
     if (st != PIE_HIP_OK || p.nsplit == 1) return st;
     hipLaunchKernelGGL(latent_merge_kernel, dim3(num_rows * heads), dim3(kvp / 4), 0, s, a.part_o, a.part_ml, row_kv_len, o,
-                       row0, heads, kvp, p.nsplit, p.steps_per_split);
+                       row0, heads, kvp, p.nsplit, p.steps_per_split, sinks);
     return launch_status();
 }

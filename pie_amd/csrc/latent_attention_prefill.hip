@@ -48,8 +48,9 @@ struct LatentPrefillArgs {
     const int32_t* row_len;
     int row0, num_rows, heads, dimp, rotp, rot_dims, ld_o;
     float scale_log2e;
+    const float* sinks;     // [heads] (null: none)
     const uint16_t* gate;   // logistic gates of the outputs [rows, ld_gate] (null: none)
-    int ld_gate;
+    int ld_gate, gate_cols;   // per head DV or 1
 };
 
 template <int KS, int VT, int QT>
@@ -119,7 +120,7 @@ __global__ __launch_bounds__(kBlock, 2) void latent_prefill_kernel(const LatentP
     for (int u = 0; u < NP; ++u) {
         const int p = min(piece0 + 8 * u, PPR - 1), e = p * 8;
         if (e < a.dimp) src[u] = a.kv + static_cast<size_t>(h) * per_head + e;
-        else if (p < PPK) src[u] = a.rot + (e - a.dimp);
+        else if (p < PPK) src[u] = a.rot + (e - a.dimp);   // (rotp 0: no such piece)
         else src[u] = a.kv + static_cast<size_t>(h) * per_head + a.dimp + (e - D);
         step_elems[u] = e >= a.dimp && p < PPK ? a.rotp : static_cast<int>(ld_kv);
     }
@@ -249,12 +250,19 @@ __global__ __launch_bounds__(kBlock, 2) void latent_prefill_kernel(const LatentP
         l += __shfl_xor(l, 32, kWave);
         const int m = wv * 16 * QT + t * 16 + l16;
         if (m >= rows) continue;
-        const float inv = l > 0.f ? 1.f / l : 0.f;
+        float inv = l > 0.f ? 1.f / l : 0.f;
+        if (a.sinks) {   // (in the units of the larger of the two)
+            const float m2 = mx[t] * a.scale_log2e, sink = a.sinks[h] * 1.4426950408889634f;
+            const float top = fmaxf(m2, sink), w = exp2f(m2 - top);
+            inv = w / (l * w + exp2f(sink - top));
+        }
+        if (a.gate && a.gate_cols == 1)
+            inv *= sigmoid_f32(bf16_bits_to_f32(a.gate[static_cast<size_t>(a.row0 + t0 + m) * a.ld_gate + h]));
         uint16_t* op = a.o + static_cast<size_t>(a.row0 + t0 + m) * a.ld_o + h * DV + 4 * g;
 #pragma unroll
         for (int dt = 0; dt < DT; ++dt) {
             f32x4_t v = acc[t][dt] * inv;
-            if (a.gate) {
+            if (a.gate && a.gate_cols != 1) {
                 const u32x2_t r = *reinterpret_cast<const u32x2_t*>(a.gate + static_cast<size_t>(a.row0 + t0 + m) * a.ld_gate + h * DV + 4 * g + 16 * dt);
                 v *= f32x4_t{sigmoid_f32(bf16_lo(r.x)), sigmoid_f32(bf16_hi(r.x)), sigmoid_f32(bf16_lo(r.y)), sigmoid_f32(bf16_hi(r.y))};
             }
@@ -281,7 +289,7 @@ using namespace pie_hip;
 
 extern "C" int pie_hip_latent_gather(const uint16_t* pool, const uint32_t* pages, uint16_t* lat, uint16_t* rot,
                                      int num_keys, int kvp, int rotp, int page_size, void* stream) {
-    if (!pool || !pages || !lat || !rot || num_keys <= 0 || kvp <= 0 || rotp < 0 || page_size <= 0) return PIE_HIP_ERR_INVALID;
+    if (!pool || !pages || !lat || (!rot && rotp > 0) || num_keys <= 0 || kvp <= 0 || rotp < 0 || page_size <= 0) return PIE_HIP_ERR_INVALID;
     if (kvp % 8 != 0 || rotp % 8 != 0) return PIE_HIP_ERR_UNSUPPORTED;
     const size_t pieces = static_cast<size_t>(num_keys) * ((kvp + rotp) / 8);
     const size_t blocks = (pieces + 255) / 256;
@@ -292,26 +300,28 @@ extern "C" int pie_hip_latent_gather(const uint16_t* pool, const uint32_t* pages
 
 extern "C" int pie_hip_latent_attn_prefill_supported(int dimp, int rotp, int vdp) {
     const int ks = (dimp + rotp) / 32, vt = vdp / 32;
-    return dimp > 0 && rotp > 0 && dimp % 32 == 0 && rotp % 32 == 0 && vdp % 32 == 0 && ks >= 2 && ks <= 6 && vt >= 1 && vt <= 4;
+    return dimp > 0 && rotp >= 0 && dimp % 32 == 0 && rotp % 32 == 0 && vdp % 32 == 0 && ks >= 1 && ks <= 6 && vt >= 1 && vt <= 4;
 }
 
 extern "C" int pie_hip_latent_attn_prefill(const uint16_t* q, const uint16_t* kv, const uint16_t* rot, uint16_t* o,
                                            const float* rope_table, const int32_t* row_kv_len, int row0, int num_rows,
                                            int num_keys, int heads, int dimp, int rotp, int rot_dims, int vdp, int ld_o,
-                                           float scale, const uint16_t* gate, int ld_gate, void* stream) {
-    if (!q || !kv || !rot || !o || !row_kv_len || row0 < 0 || num_rows <= 0 || num_keys <= 0 || heads <= 0 ||
+                                           float scale, const float* sinks, const uint16_t* gate, int ld_gate, int gate_cols,
+                                           void* stream) {
+    if (!q || !kv || (!rot && rotp > 0) || !o || !row_kv_len || row0 < 0 || num_rows <= 0 || num_keys <= 0 || heads <= 0 ||
         (rot_dims > 0 && !rope_table) || rot_dims > rotp || rot_dims % 2 != 0 || ld_o < heads * vdp ||
-        (gate && (ld_gate < heads * vdp || ld_gate % 4 != 0 || reinterpret_cast<uintptr_t>(gate) % 8 != 0)))
+        (gate && ((gate_cols != 1 && gate_cols != vdp) || ld_gate < heads * gate_cols)) ||
+        (gate && gate_cols == vdp && (ld_gate % 4 != 0 || reinterpret_cast<uintptr_t>(gate) % 8 != 0)))
         return PIE_HIP_ERR_INVALID;
     if (!pie_hip_latent_attn_prefill_supported(dimp, rotp, vdp) || ld_o % 8 != 0 || num_rows > 64 * 65535) return PIE_HIP_ERR_UNSUPPORTED;
     const LatentPrefillArgs a{q, kv, rot, o, rope_table, row_kv_len, row0, num_rows, heads, dimp, rotp, rot_dims, ld_o,
-                              scale * 1.4426950408889634f, gate, ld_gate};
+                              scale * 1.4426950408889634f, sinks, gate, ld_gate, gate_cols};
     hipStream_t s = static_cast<hipStream_t>(stream);
     const int ks = (dimp + rotp) / 32, vt = vdp / 32;
 #define PIE_PREFILL_CASE(KK, VV) \
     if (ks == KK && vt == VV) return launch_latent_prefill<KK, VV>(a, s);
 #define PIE_PREFILL_ROW(KK) PIE_PREFILL_CASE(KK, 1) PIE_PREFILL_CASE(KK, 2) PIE_PREFILL_CASE(KK, 3) PIE_PREFILL_CASE(KK, 4)
-    PIE_PREFILL_ROW(2) PIE_PREFILL_ROW(3) PIE_PREFILL_ROW(4) PIE_PREFILL_ROW(5) PIE_PREFILL_ROW(6)
+    PIE_PREFILL_ROW(1) PIE_PREFILL_ROW(2) PIE_PREFILL_ROW(3) PIE_PREFILL_ROW(4) PIE_PREFILL_ROW(5) PIE_PREFILL_ROW(6)
 #undef PIE_PREFILL_ROW
 #undef PIE_PREFILL_CASE
     return PIE_HIP_ERR_UNSUPPORTED;

@@ -214,20 +214,6 @@ struct JoinArgs {
     int ldy, ldy2, read_x, vocab, width, ld;
     float table_scale, eps;
 };
-// Eight values at a time, still in the compute type.
-template <class T>
-struct Eight {
-    u32x4_t r[sizeof(T) / 2];
-    __device__ __forceinline__ void load(const T* p) {
-#pragma unroll
-        for (int h = 0; h < static_cast<int>(sizeof(T)) / 2; ++h) r[h] = reinterpret_cast<const u32x4_t*>(p)[h];
-    }
-    __device__ __forceinline__ float get(int e) const {
-        if constexpr (sizeof(T) == 2) return e & 1 ? bf16_hi(r[0][e / 2]) : bf16_lo(r[0][e / 2]);
-        else return __uint_as_float(r[e / 4][e % 4]);
-    }
-};
-constexpr int kJoinRoutes = 64;   // places and weights of a token's first routes wait in LDS
 template <class T, int BLOCK>
 __global__ __launch_bounds__(BLOCK) void residual_join_kernel(const JoinArgs a) {
     __shared__ float red[BLOCK / kWave];
@@ -680,12 +666,13 @@ extern "C" int pie_hip_linear_f32(const float* act, const uint16_t* w_bf16, floa
 
 extern "C" int pie_hip_moe_grouped_linear_f32(const float* act, const int32_t* route_act_rows, const int32_t* expert_offsets,
                                               int num_experts, int max_rows, const uint16_t* w_bf16, float* y, int N,
-                                              int K, void* stream) {
+                                              int K, int epilogue, void* stream) {
     if (!act || !expert_offsets || !w_bf16 || !y || num_experts <= 0 || max_rows <= 0 || N <= 0 || K <= 0) return PIE_HIP_ERR_INVALID;
+    if (epilogue != PIE_HIP_EPI_NONE && epilogue != PIE_HIP_EPI_RELU2 && epilogue != PIE_HIP_EPI_GELU) return PIE_HIP_ERR_UNSUPPORTED;
     const int gy = (max_rows + kFT - 1) / kFT;
     if (gy > 65535 || num_experts > 65535) return PIE_HIP_ERR_UNSUPPORTED;
     hipLaunchKernelGGL(linear_f32_kernel, dim3((N + kFT - 1) / kFT, gy, num_experts), dim3(256), 0, static_cast<hipStream_t>(stream),
-                       act, w_bf16, y, 0, N, K, 0, expert_offsets, route_act_rows);
+                       act, w_bf16, y, 0, N, K, pointwise_code(epilogue), expert_offsets, route_act_rows);
     return launch_status();
 }
 

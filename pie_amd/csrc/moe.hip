@@ -11,6 +11,9 @@
 //   pie_hip_moe_route_groups: the same from fp32 logits, with the choice limited to the experts of
 //   a token's best groups and the weights scaled.
 //
+//   pie_hip_moe_route_corrected: logistic scores, the choice by score + correction, the scores as weights,
+//   and experts that every token uses ahead of the chosen ones.
+//
 //   pie_hip_moe_combine: out[t] (+)= sum_k w[t, k] * y_route[pos[t, k]] in top-k order, fp32,
 //   one rounding (token_batched_weighted_sum[_add]_bf16_kernel,
 //   driver/cuda/src/kernels/moe_dispatch.cu:152-196).
@@ -424,6 +427,80 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_groups_kernel(const f
     sort_routes(topk_idx, expert_offsets, route_token, route_pos, N, E, K);
 }
 
+// Logistic scores: one wave chooses a token's `top` experts by score + correction; `shared` experts that every
+// token uses come first, weighted by one more logit.
+struct CorrectedRule {
+    const float* logits;       // [N, ld], column E: the shared experts' gate
+    const float* correction;   // [E]
+    int ld, E, top, shared;
+};
+__device__ __forceinline__ float logistic(float z) { return 1.f / (1.f + expf(-z)); }
+__device__ __forceinline__ void corrected_of_token(const CorrectedRule& r, int lane, int t, int32_t* __restrict__ topk_idx,
+                                                   float* __restrict__ topk_w) {
+    const float* row = r.logits + static_cast<size_t>(t) * r.ld;
+    const int nper = (r.E + kWave - 1) / kWave, K = r.shared + r.top;
+    float s[kPerLane], c[kPerLane];
+#pragma unroll
+    for (int j = 0; j < kPerLane; ++j) {
+        const int e = lane + kWave * j;
+        s[j] = 0.f;
+        c[j] = -INFINITY;
+        if (j < nper && e < r.E) {
+            s[j] = logistic(row[e]);
+            c[j] = s[j] + r.correction[e];
+        }
+    }
+    float my_w = 0.f;   // lane k keeps the k-th expert and weight
+    int my_e = 0;
+    if (lane < r.shared) {
+        my_w = logistic(row[r.E]);
+        my_e = lane;
+    }
+    for (int k = r.shared; k < K; ++k) {
+        float bv = -INFINITY;
+        int bi = kMaxExperts;
+#pragma unroll
+        for (int j = 0; j < kPerLane; ++j)
+            if (j < nper && c[j] > bv) {
+                bv = c[j];
+                bi = lane + kWave * j;
+            }
+        wave_argmax(bv, bi);
+        bi = min(bi, r.E - 1);   // only reachable with NaN logits; keeps every index in range
+        float won = 0.f;
+#pragma unroll
+        for (int j = 0; j < kPerLane; ++j)
+            if (j < nper && bi == lane + kWave * j) {
+                won = s[j];
+                c[j] = -INFINITY;   // exclude on the next pass
+            }
+        won = __shfl(won, bi & (kWave - 1), kWave);
+        if (lane == k) {
+            my_w = won;
+            my_e = r.shared + bi;
+        }
+    }
+    if (lane < K) {
+        topk_idx[static_cast<size_t>(t) * K + lane] = my_e;
+        topk_w[static_cast<size_t>(t) * K + lane] = my_w;
+    }
+}
+__global__ __launch_bounds__(256) void moe_topk_corrected_kernel(const CorrectedRule r, int32_t* __restrict__ topk_idx,
+                                                                 float* __restrict__ topk_w, int N) {
+    const int lane = threadIdx.x & (kWave - 1), t = blockIdx.x * 4 + threadIdx.x / kWave;
+    if (t < N) corrected_of_token(r, lane, t, topk_idx, topk_w);
+}
+__global__ __launch_bounds__(kRouteThreads) void moe_route_corrected_kernel(const CorrectedRule r, int32_t* topk_idx,
+                                                                            float* __restrict__ topk_w,
+                                                                            int32_t* __restrict__ expert_offsets,
+                                                                            int32_t* __restrict__ route_token,
+                                                                            int32_t* __restrict__ route_pos, int N) {
+    const int lane = threadIdx.x & (kWave - 1), t = threadIdx.x / kWave;
+    if (t < N) corrected_of_token(r, lane, t, topk_idx, topk_w);
+    __syncthreads();   // (a block's stores are seen by its own threads after the barrier)
+    sort_routes(topk_idx, expert_offsets, route_token, route_pos, N, r.E + r.shared, r.top + r.shared);
+}
+
 __global__ __launch_bounds__(256) void moe_combine_kernel(
     const uint16_t* __restrict__ y_routes, const int32_t* __restrict__ route_pos,
     const float* __restrict__ topk_w, uint16_t* __restrict__ out, int K, int H, int add) {
@@ -627,6 +704,29 @@ extern "C" int pie_hip_moe_route_groups(const float* router_logits, int ld_logit
                        topk_weight, num_tokens, num_experts, top_k, groups);
     hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(kRouteThreads), 0, st, topk_idx, expert_offsets, route_token, route_pos,
                        num_tokens, num_experts, top_k);
+    return launch_status();
+}
+
+extern "C" int pie_hip_moe_route_corrected(const float* router_logits, int ld_logits, const float* correction,
+                                           int32_t* topk_idx, float* topk_weight, int32_t* expert_offsets,
+                                           int32_t* route_token, int32_t* route_pos, int num_tokens, int num_experts,
+                                           int top_k, int shared, void* stream) {
+    using namespace pie_hip;
+    if (!router_logits || !correction || !topk_idx || !topk_weight || !expert_offsets || !route_token || !route_pos ||
+        num_tokens <= 0 || num_experts <= 0 || top_k <= 0 || top_k > num_experts || shared < 0 ||
+        ld_logits < num_experts + (shared > 0 ? 1 : 0))
+        return PIE_HIP_ERR_INVALID;
+    if (num_experts + shared > kMaxExperts || top_k + shared > kWave) return PIE_HIP_ERR_UNSUPPORTED;
+    hipStream_t st = static_cast<hipStream_t>(stream);
+    const CorrectedRule r{router_logits, correction, ld_logits, num_experts, top_k, shared};
+    if (num_tokens <= kFusedTokens) {
+        hipLaunchKernelGGL(moe_route_corrected_kernel, dim3(1), dim3(kRouteThreads), 0, st, r, topk_idx, topk_weight,
+                           expert_offsets, route_token, route_pos, num_tokens);
+        return launch_status();
+    }
+    hipLaunchKernelGGL(moe_topk_corrected_kernel, dim3((num_tokens + 3) / 4), dim3(256), 0, st, r, topk_idx, topk_weight, num_tokens);
+    hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(kRouteThreads), 0, st, topk_idx, expert_offsets, route_token, route_pos,
+                       num_tokens, num_experts + shared, top_k + shared);
     return launch_status();
 }
 

@@ -1129,15 +1129,15 @@ def linear_f32(act: torch.Tensor, w: torch.Tensor, relu2: bool = False, epilogue
 
 
 def head_linear(act: torch.Tensor, w: torch.Tensor, rope_table: Optional[torch.Tensor] = None, rot_dim: int = 0,
-                rot_dims: int = 0, rotp: int = 0, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                rot_dims: int = 0, rotp: int = 0, gate: Optional[torch.Tensor] = None, gate_cols: Optional[int] = None) -> torch.Tensor:
     """act [M, heads, A], w [heads, C, K] -> [M, heads, C + rotp]; the rotated part starts at K.  gate [M, ld]:
-    logistic gates of the outputs."""
+    logistic gates, one per output or (gate_cols 1) one per head."""
     M, heads, A = act.shape
     _, n, k = w.shape
     y = torch.full((M, heads, n + rotp), 3.0, dtype=act.dtype, device=act.device)
     _check(kernels().pie_hip_head_linear(_dt(act), _ptr(act), _ptr(w), _ptr(y), _ptr(rope_table), M, heads, n, k,
                                          heads * A, A, heads * (n + rotp), n + rotp, k, rot_dim, rot_dims, rotp, _ptr(gate),
-                                         0 if gate is None else gate.stride(0), _stream()),
+                                         0 if gate is None else gate.stride(0), n if gate_cols is None else gate_cols, _stream()),
            "pie_hip_head_linear")
     return y
 
@@ -1145,15 +1145,15 @@ def head_linear(act: torch.Tensor, w: torch.Tensor, rope_table: Optional[torch.T
 def latent_attn_rows(q: torch.Tensor, pool: torch.Tensor, kvp: int, page_indices: torch.Tensor, row_begin: torch.Tensor,
                      row_len: torch.Tensor, page_size: int, scale: float, row_req: Optional[torch.Tensor] = None,
                      qo_indptr: Optional[torch.Tensor] = None, max_tokens: int = 1, plain: bool = False,
-                     max_kv_len: Optional[int] = None) -> torch.Tensor:
-    """q [rows, heads, ld], pool [slots, ld] -> o [rows, heads, kvp]."""
+                     max_kv_len: Optional[int] = None, sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """q [rows, heads, ld], pool [slots, ld], sinks [heads] -> o [rows, heads, kvp]."""
     rows, heads, ld = q.shape
     o = torch.full((rows, heads, kvp), 3.0, dtype=q.dtype, device=q.device)
     longest = int(row_len.max()) if max_kv_len is None else max_kv_len
     lib = kernels()
     if plain:
         _check(lib.pie_hip_latent_attn_rows_plain(_dt(q), _ptr(q), _ptr(pool), _ptr(o), _ptr(page_indices), _ptr(row_begin),
-                                                  _ptr(row_len), rows, heads, kvp, ld, page_size, C.c_float(scale), _stream()),
+                                                  _ptr(row_len), rows, heads, kvp, ld, page_size, C.c_float(scale), _ptr(sinks), _stream()),
                "pie_hip_latent_attn_rows_plain")
         return o
     lib.pie_hip_latent_attn_rows_workspace_bytes.restype = C.c_size_t
@@ -1161,7 +1161,7 @@ def latent_attn_rows(q: torch.Tensor, pool: torch.Tensor, kvp: int, page_indices
     ws = torch.empty(max(need, 16), dtype=torch.uint8, device=q.device)
     _check(lib.pie_hip_latent_attn_rows(_ptr(q), _ptr(pool), _ptr(o), _ptr(page_indices), _ptr(row_begin), _ptr(row_len),
                                         _ptr(row_req), _ptr(qo_indptr), 0, rows, heads, kvp, ld - kvp, page_size,
-                                        C.c_float(scale), longest, max_tokens, _ptr(ws), C.c_size_t(need), _stream()),
+                                        C.c_float(scale), _ptr(sinks), longest, max_tokens, _ptr(ws), C.c_size_t(need), _stream()),
            "pie_hip_latent_attn_rows")
     return o
 
@@ -1177,17 +1177,19 @@ def latent_gather(pool: torch.Tensor, pages: torch.Tensor, num_keys: int, kvp: i
 
 def latent_attn_prefill(q: torch.Tensor, kv: torch.Tensor, rot: torch.Tensor, rope_table: Optional[torch.Tensor],
                         rot_dims: int, row_len: torch.Tensor, dimp: int, scale: float,
-                        gate: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """q [rows, heads, dimp + rotp], kv [keys, heads, dimp + vdp], rot [keys, rotp] -> o [rows, heads * vdp], times
-    the logistic function of gate [rows, ld]."""
+                        gate: Optional[torch.Tensor] = None, gate_cols: Optional[int] = None,
+                        sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """q [rows, heads, dimp + rotp], kv [keys, heads, dimp + vdp], rot [keys, rotp] (or None), sinks [heads] ->
+    o [rows, heads * vdp], times the logistic function of gate [rows, ld], one per value or (gate_cols 1) per head."""
     rows, heads, _ = q.shape
     vdp = kv.shape[2] - dimp
     o = torch.full((rows, heads * vdp), 3.0, dtype=torch.bfloat16, device=q.device)
     if int(row_len.max()) > kv.shape[0]:
         raise KernelError("a row sees more keys than there are")
     _check(kernels().pie_hip_latent_attn_prefill(_ptr(q), _ptr(kv), _ptr(rot), _ptr(o), _ptr(rope_table), _ptr(row_len), 0, rows,
-                                                 kv.shape[0], heads, dimp, rot.shape[1], rot_dims, vdp, heads * vdp,
-                                                 C.c_float(scale), _ptr(gate), 0 if gate is None else gate.stride(0), _stream()),
+                                                 kv.shape[0], heads, dimp, 0 if rot is None else rot.shape[1], rot_dims, vdp,
+                                                 heads * vdp, C.c_float(scale), _ptr(sinks), _ptr(gate),
+                                                 0 if gate is None else gate.stride(0), vdp if gate_cols is None else gate_cols, _stream()),
            "pie_hip_latent_attn_prefill")
     return o
 
@@ -1345,14 +1347,15 @@ def moe_route_groups(logits: torch.Tensor, experts: int, top: int, groups: int, 
 
 
 def moe_grouped_glu(act: torch.Tensor, rows, offsets: torch.Tensor, w: torch.Tensor, routes: int, rule: Optional[Glu],
-                    block_rows: Optional[int] = None, tiled: bool = False) -> torch.Tensor:
-    """Rows sorted by expert times w [experts, N, K] (gated if there is a rule); bf16 or fp32 by act's type.  bf16 with
-    block_rows: in blocks of that many routes (0: the library's choice), `tiled`: over tile-major weights."""
+                    block_rows: Optional[int] = None, tiled: bool = False, epilogue: int = 0) -> torch.Tensor:
+    """Rows sorted by expert times w [experts, N, K] (gated if there is a rule, else with a pointwise epilogue); bf16 or
+    fp32 by act's type.  bf16 with block_rows: in blocks of that many routes (0: the library's choice), `tiled`: over
+    tile-major weights."""
     E, N, K = w.shape
     lib = kernels()
     if act.dtype == torch.float32:
         y = torch.empty((routes, N), dtype=torch.float32, device=act.device)
-        _check(lib.pie_hip_moe_grouped_linear_f32(_ptr(act), _ptr(rows), _ptr(offsets), E, routes, _ptr(w), _ptr(y), N, K, _stream()),
+        _check(lib.pie_hip_moe_grouped_linear_f32(_ptr(act), _ptr(rows), _ptr(offsets), E, routes, _ptr(w), _ptr(y), N, K, epilogue, _stream()),
                "pie_hip_moe_grouped_linear_f32")
         if rule is None:
             return y
@@ -1363,11 +1366,11 @@ def moe_grouped_glu(act: torch.Tensor, rows, offsets: torch.Tensor, w: torch.Ten
     glu_arg = None if rule is None else C.byref(rule)
     if block_rows is not None:
         _check(lib.pie_hip_moe_grouped_gemm_mfma(_ptr(act), _ptr(rows), _ptr(offsets), E, routes, _ptr(w), C.c_size_t(N * K * 2), _ptr(y), N, K,
-                                                 0 if rule is None else 1, int(tiled), glu_arg, block_rows, _stream()),
+                                                 epilogue if rule is None else 1, int(tiled), glu_arg, block_rows, _stream()),
                "pie_hip_moe_grouped_gemm_mfma")
         return y
     _check(lib.pie_hip_moe_grouped_gemm_glu(3, _ptr(act), _ptr(rows), _ptr(offsets), E, max(1, routes), _ptr(w), C.c_size_t(N * K * 2), None,
-                                            C.c_size_t(0), 0, 0, _ptr(y), N, K, 0 if rule is None else 1, int(tiled), glu_arg, _stream()),
+                                            C.c_size_t(0), 0, 0, _ptr(y), N, K, epilogue if rule is None else 1, int(tiled), glu_arg, _stream()),
            "pie_hip_moe_grouped_gemm_glu")
     return y
 
@@ -1497,3 +1500,50 @@ def gated_part_norm(o, x, skip, z, norm_w, heads, vdim, parts, rows: StateRows, 
                                              0 if conv_fused is None else conv_fused.shape[1], channels, taps, C.c_float(eps), _stream()),
            "pie_hip_gated_part_norm")
     return y
+
+
+def embed_bigram(tokens, prev, table, scale: float, bigram, buckets: int, mul_prev: int, mul_cur: int, norm_w, ld: int, eps: float) -> torch.Tensor:
+    """x [N, ld]: the normed sum of a token's row and the row of its pair with the previous one (prev < 0: none)."""
+    width = table.shape[1]
+    x = torch.zeros((tokens.numel(), ld), dtype=torch.float32, device=table.device)
+    u64 = C.c_ulonglong
+    _check(kernels().pie_hip_embed_bigram(_ptr(tokens), _ptr(prev), _ptr(table), table.shape[0], C.c_float(scale), _ptr(bigram), u64(buckets),
+                                          u64(mul_prev), u64(mul_cur), _ptr(norm_w), _ptr(x), tokens.numel(), width, ld, C.c_float(eps),
+                                          _stream()), "pie_hip_embed_bigram")
+    return x
+
+
+def gated_join(x: torch.Tensor, width: int, eps: float, dtype, y=None, routes=None, gate=None, gate_bias=None, next_weight=None, conv_w=None,
+               rows: Optional[StateRows] = None):
+    """x takes y (or routes, as in residual_join) times the logistic function of gate + gate_bias in place; returns
+    (h, recent): x normed, and with conv_w [taps, width] (one row per request) h plus its convolution."""
+    _dev(x, torch.float32, "x")
+    h, recent = (torch.zeros(x.shape, dtype=dtype, device=x.device) for _ in range(2))
+    r = None if routes is None else Routes(routes[0].data_ptr(), routes[1].data_ptr(), routes[2].data_ptr(), routes[1].shape[1],
+                                           routes[0].shape[1])
+    _check(kernels().pie_hip_gated_join(_dt(h), _ptr(y), 0 if y is None else y.shape[1], None if r is None else C.byref(r), _ptr(gate),
+                                        0 if gate is None else gate.shape[1], _ptr(gate_bias), _ptr(x), _ptr(next_weight), _ptr(h),
+                                        _ptr(recent) if conv_w is not None else None, _ptr(conv_w), 0 if conv_w is None else conv_w.shape[0],
+                                        None if rows is None else C.byref(rows), x.shape[0], width, x.shape[1], C.c_float(eps), _stream()),
+           "pie_hip_gated_join")
+    return h, recent
+
+
+def recent_rows(h: torch.Tensor, conv_w: torch.Tensor, rows: StateRows) -> torch.Tensor:
+    """h [N, ld] plus its convolution (conv_w [taps, width]) over each request's rows and state."""
+    out = torch.zeros_like(h)
+    _check(kernels().pie_hip_recent_rows(_dt(h), _ptr(h), _ptr(conv_w), conv_w.shape[0], C.byref(rows), _ptr(out), conv_w.shape[1], h.shape[1],
+                                         _stream()), "pie_hip_recent_rows")
+    return out
+
+
+def moe_route_corrected(logits: torch.Tensor, correction: torch.Tensor, top: int, shared: int):
+    """fp32 logits [T, ld] (column `experts`: the shared experts' gate) -> as moe_route_groups, the shared experts first."""
+    _dev(logits, torch.float32, "logits")
+    T, E, K = logits.shape[0], correction.numel(), top + shared
+    i32 = lambda *shape: torch.empty(shape, dtype=torch.int32, device=logits.device)
+    idx, offsets, token, pos = i32(T, K), i32(E + shared + 1), i32(T * K), i32(T, K)
+    weight = torch.empty((T, K), dtype=torch.float32, device=logits.device)
+    _check(kernels().pie_hip_moe_route_corrected(_ptr(logits), logits.shape[1], _ptr(correction), _ptr(idx), _ptr(weight), _ptr(offsets),
+                                                 _ptr(token), _ptr(pos), T, E, top, shared, _stream()), "pie_hip_moe_route_corrected")
+    return idx, weight, offsets, token, pos
