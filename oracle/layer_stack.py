@@ -410,6 +410,10 @@ def scalar_norm(x, g, eps):
     return divide_by_rms(np.asarray(x, np.float64), eps) * float(np.asarray(g).reshape(()))
 
 
+def softcap(logits, cap):
+    return cap * np.tanh(logits / cap)
+
+
 def with_recent(h, w):
     """A row plus a causal convolution over it and the rows before it."""
     return h + causal_conv(h, w)
@@ -468,9 +472,11 @@ def gated_sublayer(x, w, p, n, sublayer, eps):
 
 
 def forward_gated(cfg, w, tokens, want_layers=False):
-    eps, b = cfg["norm"]["eps"], cfg["embedding"]["bigram"]
+    eps, b = cfg["norm"]["eps"], cfg["embedding"].get("bigram")
     x = np.asarray(w["embed"], np.float64)[np.asarray(tokens)] * cfg["embedding"]["scale"]
-    x = scalar_norm(x + w["bigram"][bigram_rows(tokens, b["buckets"], b["mul_prev"], b["mul_cur"])], w["embed.norm"], eps)
+    if b:
+        x = x + w["bigram"][bigram_rows(tokens, b["buckets"], b["mul_prev"], b["mul_cur"])]
+    x = scalar_norm(x, w["embed.norm"], eps)
     states = []
     for i, layer in enumerate(cfg["layers"]):
         p, mlp = f"l{i}.", layer.get("mlp")
@@ -479,8 +485,7 @@ def forward_gated(cfg, w, tokens, want_layers=False):
             ff = silu_pair_feed_forward if mlp["kind"] == "dense" else (lambda h, w, q: shared_mixture(h, w, q, mlp))
             x = gated_sublayer(x, w, p, 2, lambda h: ff(h, w, p + "mlp."), eps)
         states.append(x)
-    cap = cfg["logit_softcap"]
-    logits = cap * np.tanh(scalar_norm(x, w["final.norm"], eps) @ w["head"].T / cap)
+    logits = softcap(scalar_norm(x, w["final.norm"], eps) @ w["head"].T, cfg["logit_softcap"])
     return (logits, np.stack(states)) if want_layers else logits
 
 

@@ -253,11 +253,105 @@ def fobanex_weights(cfg, seed=0, sharp=1.0):
     return w
 
 
+# ---- Minodra -----------------------------------------------------------------------------------------
+def sink_latent(mlp=None, heads=3, dim=24, vdim=20, q_rank=40, kv_rank=48, scale=None):
+    return dict(type="latent_attention", mlp=mlp,
+                mixer=dict(heads=heads, dim=dim, vdim=vdim, q_rank=q_rank, kv_rank=kv_rank, scale=scale if scale is not None else dim ** -0.5))
+
+
+def shared_moe(experts=9, top=3, ff=40, shared=56):
+    m = dict(kind="moe", expert=dict(ff=ff), router=dict(experts=experts, top=top))
+    if shared:
+        m["shared"] = dict(ff=shared)
+    return m
+
+
+def minodra(layers, width=112, vocab=97, eps=1e-4, scale=3.0, taps=3, softcap=11.0, bigram=(61, 97531, 2654435761)):
+    e = dict(scale=scale)
+    if bigram:
+        e["bigram"] = dict(zip(("buckets", "mul_prev", "mul_cur"), bigram))
+    return dict(architecture="Minodra", layers=layers, width=width, vocab=vocab, norm=dict(eps=eps), embedding=e, canon=dict(taps=taps),
+                logit_softcap=softcap)
+
+
+# sizes off every padding unit, values wider and narrower than the keys, convolutions of one to six taps, layers
+# without a feed-forward at the end and between others, one expert, all experts, a shared expert narrower than the
+# others, wider than one and than several, and none, multipliers beyond 32 bits, one bucket, no bigrams, widths of one
+# and several blocks, sizes of every matrix-core form and of the plain ones
+MINODRA_CONFIGS = {
+    "pair": minodra([sink_latent(dense(72)), sink_latent(shared_moe(), heads=5, dim=40, vdim=33, q_rank=52, kv_rank=100)]),
+    "odd": minodra([sink_latent(shared_moe(experts=1, top=1, ff=17, shared=0), heads=1, dim=9, vdim=7, q_rank=11, kv_rank=13), sink_latent(),
+                    sink_latent(dense(31), heads=4, dim=33, vdim=48, q_rank=30, kv_rank=65), sink_latent()],
+                   width=75, vocab=130, scale=0.5, taps=1, softcap=30.0, bigram=(1, 3, 5)),
+    "wide": minodra([sink_latent(shared_moe(experts=40, top=8, ff=64, shared=300), heads=17, dim=32, vdim=32, q_rank=64, kv_rank=520),
+                     sink_latent(shared_moe(experts=6, top=6, ff=150, shared=60), heads=33, dim=64, vdim=64, q_rank=96, kv_rank=200),
+                     sink_latent(dense(200), heads=2, dim=32, vdim=96, q_rank=130, kv_rank=380)], width=160, vocab=64, taps=6),
+    "broad": minodra([sink_latent(shared_moe(experts=5, top=2, ff=24, shared=24), heads=2, kv_rank=64),
+                      sink_latent(dense(64), heads=6, dim=16, vdim=16, kv_rank=128)], width=2056, vocab=50, taps=4, bigram=None),
+    "four": minodra([sink_latent(shared_moe(experts=20, top=5, ff=33, shared=33)), sink_latent(heads=2, dim=48, vdim=64, kv_rank=256),
+                     sink_latent(shared_moe(experts=4, top=2, shared=0)), sink_latent(dense(40), heads=16, dim=16, vdim=24, kv_rank=192)],
+                    width=96, taps=2, bigram=(2000, 1 << 40, 12345678901)),
+}
+
+
+def minodra_weights(cfg, seed=0, sharp=1.0, spread=0.4):
+    """`sharp` scales the query projections: large values make single keys stand out.  `spread` of the corrections: large
+    values make it rarer that two experts are all but equally good a choice, of which either weighs its whole score."""
+    rng = np.random.default_rng(seed)
+    w, H = {}, cfg["width"]
+
+    def lin(name, rows, cols, gain=1.0):
+        w[name] = bf16(rng.standard_normal((rows, cols)) * gain / np.sqrt(cols))
+
+    def vec(name, n, lo=0.7, hi=1.3):
+        w[name] = bf16(rng.uniform(lo, hi, n))
+
+    lin("embed", cfg["vocab"], H, np.sqrt(H))
+    if cfg["embedding"].get("bigram"):
+        lin("bigram", cfg["embedding"]["bigram"]["buckets"] + 1, H, 2.0 * np.sqrt(H))
+    vec("embed.norm", ())
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, mlp = f"l{i}.", layer["mixer"], layer["mlp"]
+        x, q = p + "mix.", p + "mlp."
+        lin(x + "dq", m["q_rank"], H)
+        vec(x + "dq.norm", m["q_rank"])
+        lin(x + "uq", m["heads"] * m["dim"], m["q_rank"], sharp)
+        lin(x + "dkv", m["kv_rank"], H)
+        vec(x + "dkv.norm", m["kv_rank"])
+        lin(x + "uk", m["heads"] * m["dim"], m["kv_rank"])
+        lin(x + "uv", m["heads"] * m["vdim"], m["kv_rank"])
+        w[x + "sink"] = bf16(rng.uniform(0.0, 4.0, m["heads"]))
+        lin(x + "g", m["heads"], H, 1.5)
+        lin(x + "o", H, m["heads"] * m["vdim"], 3.0)
+        for n in ("1", "2") if mlp else ("1",):
+            vec(p + "norm" + n, ())
+            w[p + "canon" + n] = bf16(rng.standard_normal((H, cfg["canon"]["taps"])) * 0.5)
+            lin(p + "rg" + n, H, H, 1.5)
+            w[p + "rg" + n + ".b"] = bf16(rng.standard_normal(H) * 0.7)
+        if mlp and mlp["kind"] == "dense":
+            for n, rows, cols in (("gate", mlp["ff"], H), ("up", mlp["ff"], H), ("down", H, mlp["ff"])):
+                lin(q + n, rows, cols, 1.5)
+        elif mlp:
+            E = mlp["router"]["experts"]
+            lin(q + "router", E, H, 1.5)
+            w[q + "correction"] = bf16(rng.uniform(-spread, spread, E))
+            sizes = [(f"e{e}.", mlp["expert"]["ff"]) for e in range(E)]
+            if mlp.get("shared"):
+                sizes.append(("shared.", mlp["shared"]["ff"]))
+                lin(q + "shared.sg", 1, H, 2.0)
+            for n, ff in sizes:
+                lin(q + n + "up", ff, H, 1.5)
+                lin(q + n + "down", H, ff, 1.5)
+    vec("final.norm", ())
+    lin("head", cfg["vocab"], H, 6.0)
+    return w
+
+
 def bf16(a):
     """Rounds to the nearest bf16 value (ties to even); returns float32."""
     u = np.ascontiguousarray(a, np.float32).view(np.uint32)
     r = (u + 0x7FFF + ((u >> 16) & 1)) & np.uint32(0xFFFF0000)
-    return r.view(np.float32)
+    return r.view(np.float32).reshape(np.shape(a))
 
 
 def random_weights(cfg, seed=0, low_rank=12, sharp=1.0):
@@ -314,7 +408,7 @@ def write_stack(directory, cfg, weights):
     from safetensors.torch import save_file
 
     os.makedirs(directory, exist_ok=True)
-    save_file({k: torch.from_numpy(np.ascontiguousarray(v)).to(torch.bfloat16) for k, v in weights.items()},
+    save_file({k: torch.from_numpy(np.array(v, order="C")).to(torch.bfloat16) for k, v in weights.items()},
               os.path.join(directory, "model.safetensors"))
     with open(os.path.join(directory, "config.json"), "w") as f:
         json.dump(cfg, f)
