@@ -347,8 +347,9 @@ def other_configs_extra(drvmod):
 # feed-forward width.  Varasun: latent attention, one channel-delta layer in three, squared-ReLU
 # feed-forward.  Lofudra: mLSTM, Mamba-2, windowed attention beside retention in turn, GELU feed-forward.
 # Fobanex: gated latent attention (the second layer on the first one's latents), attention normed over whole
-# projections, attention on its keys; two dense layers and four mixtures.  "moe" is the qwen3_moe-type model,
-# a mixture of the same experts in every layer.
+# projections, attention on its keys; two dense layers and four mixtures.  Minodra: latent attention without a
+# rotated part, gated sublayers behind convolutions; as many dense layers as mixtures, which have a shared expert.
+# "moe" is the qwen3_moe-type model, a mixture of the same experts in every layer.
 STACK_SIZES = {
     "width4096": dict(width=4096, heads=32, dim=128, rot_dim=64, vdim=128, q_rank=1536, kv_rank=512, ff=14336,
                       kv_heads=8, vocab=32000, layers=6, window=1024,
@@ -405,7 +406,16 @@ def fobanex_config(z: dict) -> dict:
                 embedding=dict(scale=z["width"] ** 0.5))
 
 
-STACKS = {"varasun": varasun_config, "lofudra": lofudra_config, "fobanex": fobanex_config}
+def minodra_config(z: dict) -> dict:
+    mixer = dict(heads=z["heads"], dim=z["dim"], vdim=z["vdim"], q_rank=z["q_rank"], kv_rank=z["kv_rank"], scale=z["dim"] ** -0.5)
+    dense = dict(kind="dense", ff=z["ff"])
+    moe = dict(kind="moe", expert=dict(ff=z["expert_ff"]), router=dict(experts=z["experts"], top=z["top"]), shared=dict(ff=z["expert_ff"]))
+    layers = [dict(type="latent_attention", mixer=mixer, mlp=moe if l % 2 else dense) for l in range(z["layers"])]
+    return dict(architecture="Minodra", layers=layers, width=z["width"], vocab=z["vocab"], norm=dict(eps=1e-6), canon=dict(taps=4),
+                embedding=dict(scale=z["width"] ** 0.5, bigram=dict(buckets=65521, mul_prev=92821, mul_cur=31)), logit_softcap=30.0)
+
+
+STACKS = {"varasun": varasun_config, "lofudra": lofudra_config, "fobanex": fobanex_config, "minodra": minodra_config}
 STACK_SIDES = [*STACKS, "llama", "moe"]
 
 

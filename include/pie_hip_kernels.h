@@ -270,7 +270,7 @@ int pie_hip_gemm_mfma_glu(int format, const uint16_t* act_bf16, const void* weig
  *   weights at weights + e*weight_stride_bytes (scales at scales + e*scale_stride_bytes).
  * Experts without routes cost nothing and their weights are never read; an expert's weights
  * are read once per 16 routes that hit it.  max_rows_per_expert is a hint (> 0) of the largest
- * per-expert row count.  With swiglu the weight rows are interleaved (gate_0, up_0, ...) and y
+ * per-expert row count; num_routes (0: not known) bounds how many experts have any.  With swiglu the weight rows are interleaved (gate_0, up_0, ...) and y
  * is [routes, N/2].  Same K requirements as pie_hip_gemm_skinny.
  * Replaces the per-route MoE decode GEMVs (driver/cuda/src/kernels/dequant_wna16.cu:59-169)
  * and the grouped GEMM of driver/cuda/src/ops/gemm.hpp:189-198.
@@ -285,7 +285,7 @@ int pie_hip_moe_grouped_gemm(int format, const uint16_t* act_bf16, const int32_t
  * (`tiled`) tile-major weights. */
 int pie_hip_moe_grouped_gemm_glu(int format, const uint16_t* act_bf16, const int32_t* route_act_rows,
                                  const int32_t* expert_offsets, int num_experts,
-                                 int max_rows_per_expert, const void* weights,
+                                 int max_rows_per_expert, int num_routes, const void* weights,
                                  size_t weight_stride_bytes, const void* scales,
                                  size_t scale_stride_bytes, int scale_is_bf16, int group_size,
                                  uint16_t* y_bf16, int N, int K, int swiglu, int tiled,
@@ -1144,24 +1144,27 @@ int pie_hip_gated_part_norm(int dtype, const float* o, const void* x, int ld_x, 
 /*
  * Layers whose sublayers' outputs pass a logistic gate and whose sublayers read a short convolution of the normed
  * stream: h = norm(x), the sublayer reads h + conv(h), x += sublayer * sigmoid(gate), the gate a product of h.
- * pie_hip_embed_bigram: x[n] = e / sqrt(mean(e^2) + eps) * norm_weight, e = table[token_ids[n]] * table_scale +
- *   bigram[row], row = (prev_ids[n] * mul_prev + token_ids[n] * mul_cur) mod buckets in 64 bits, row `buckets`
- *   where prev_ids[n] < 0 (a sequence's first token); bigram NULL: left out; ids >= vocab read row 0 of table.
  * pie_hip_gated_join: x[n] += (y[n] or a mixture's routes, see PieHipRoutes) * sigmoid(gate[n] + gate_bias) (neither y
- *   nor routes: x as it is); h[n] = x[n] / sqrt(mean(x[n]^2) + eps) * next_weight in the compute type (next_weight
+ *   nor routes: x as it is; with `start` x is set to an embedding, see PieHipEmbedding); h[n] = x[n] / sqrt(mean(x[n]^2) + eps) * next_weight in the compute type (next_weight
  *   NULL: x only).  With conv_w (one row per request, taps <= 4) also recent[n] = h[n] + the convolution, whose
  *   state moves on by the row.  Rows of ld; columns from the width on are not touched.
  * pie_hip_recent_rows: recent[n, c] = h[n, c] + sum_j conv_w[j, c] h_(n - (taps - 1) + j)[c], earlier rows from the
  *   request's state, zeros before its start; pie_hip_delta_conv_state (channels = width) moves the state on
  *   afterwards.  conv_w [taps, width] fp32; the state is [taps - 1, width] in the compute type at conv_offset.
  */
-int pie_hip_embed_bigram(const uint32_t* token_ids, const int32_t* prev_ids, const uint16_t* table_bf16, int vocab,
-                         float table_scale, const uint16_t* bigram_bf16, unsigned long long buckets,
-                         unsigned long long mul_prev, unsigned long long mul_cur, const float* norm_weight, float* x,
-                         int num_tokens, int width, int ld, float eps, void* stream);
+/* x[n] = e / sqrt(mean(e^2) + eps) * norm_weight, e = table[token_ids[n]] * scale + pair_table[pair_rows[n]] (pair_table
+ * NULL: left out; ids >= vocab read row 0 of table). */
+typedef struct {
+    const uint32_t* token_ids;
+    const int32_t* pair_rows;
+    const uint16_t *table, *pair_table;
+    const float* norm_weight;
+    int vocab;
+    float scale;
+} PieHipEmbedding;
 int pie_hip_gated_join(int dtype, const void* y, int ldy, const PieHipRoutes* routes, const void* gate, int ld_gate,
-                       const float* gate_bias, float* x, const float* next_weight, void* h, void* recent,
-                       const float* conv_w, int taps, const PieHipStateRows* state, int rows, int width, int ld,
+                       const float* gate_bias, const PieHipEmbedding* start, float* x, const float* next_weight,
+                       void* h, void* recent, const float* conv_w, int taps, const PieHipStateRows* state, int rows, int width, int ld,
                        float eps, void* stream);
 int pie_hip_recent_rows(int dtype, const void* h, const float* conv_w, int taps, const PieHipStateRows* state, void* recent,
                         int width, int ld, void* stream);

@@ -64,6 +64,16 @@ struct Eight {
         else return __uint_as_float(r[e / 4][e % 4]);
     }
 };
+// (rounded to the compute type; p 16-byte aligned)
+template <class T>
+__device__ __forceinline__ void store_eight(T* p, const float (&v)[8]) {
+    if constexpr (sizeof(T) == 2) {
+        *reinterpret_cast<u32x4_t*>(p) = u32x4_t{pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]), pack_bf16x2(v[4], v[5]), pack_bf16x2(v[6], v[7])};
+    } else {
+#pragma unroll
+        for (int h = 0; h < 2; ++h) *reinterpret_cast<f32x4_t*>(p + 4 * h) = f32x4_t{v[4 * h], v[4 * h + 1], v[4 * h + 2], v[4 * h + 3]};
+    }
+}
 constexpr int kJoinRoutes = 64;   // places and weights of a token's routes through a mixture wait in LDS
 
 // (the bare exponential and reciprocal: a few units in the last place)

@@ -202,7 +202,7 @@ Executor::Inputs Executor::input_layout(int N, int S) const {
     in.off_sample_rows = off;  off = align_up(off + static_cast<size_t>(S) * 4, 256);
     const size_t per_row = model_.cfg().is_stack() ? 4 : 0;
     in.off_row_req = off;      off = align_up(off + N * per_row, 256);
-    in.off_prev = off;         off = align_up(off + N * per_row, 256);
+    in.off_pair = off;         off = align_up(off + N * per_row, 256);
     in.off_qo = off;           off = align_up(off + (N + 1) * per_row, 256);
     in.off_rs_slot = off;      off = align_up(off + N * per_row, 256);
     in.off_rs_fresh = off;     off = align_up(off + N * per_row, 256);

@@ -133,7 +133,7 @@ class Executor {
     // rows' requests and the requests' row ranges and state slots.
     struct Inputs {
         size_t off_tokens, off_positions, off_slots, off_row_begin, off_row_len, off_sample_rows,
-            off_row_req, off_prev, off_qo, off_rs_slot, off_rs_fresh, off_pages, total;
+            off_row_req, off_pair, off_qo, off_rs_slot, off_rs_fresh, off_pages, total;
     };
     Inputs input_layout(int N, int S) const;
     void body(int N, int S, int max_kv_len);

@@ -233,7 +233,13 @@ void Executor::copy_rs_h2h(const uint32_t* srcs, const uint32_t* dsts, size_t n)
 void Executor::prepare_stack(const BatchPlan& plan, const Inputs& in) {
     if (plan.has_user_masks) throw std::runtime_error("executor: layer stacks take no custom attention masks");
     auto* row_req = reinterpret_cast<int32_t*>(in_host_ + in.off_row_req);
-    auto* prev = reinterpret_cast<int32_t*>(in_host_ + in.off_prev);
+    auto* pair = reinterpret_cast<int32_t*>(in_host_ + in.off_pair);
+    const BigramSpec& bigram = model_.cfg().bigram;
+    auto pair_row = [&](int32_t before, uint32_t token) {   // (before < 0: a sequence's first token)
+        if (bigram.buckets == 0) return 0;
+        if (before < 0) return static_cast<int32_t>(bigram.buckets);
+        return static_cast<int32_t>((static_cast<uint64_t>(before) * bigram.mul_prev + static_cast<uint64_t>(token) * bigram.mul_cur) % bigram.buckets);
+    };
     auto* qo = reinterpret_cast<int32_t*>(in_host_ + in.off_qo);
     auto* slot = reinterpret_cast<int32_t*>(in_host_ + in.off_rs_slot);
     auto* fresh = reinterpret_cast<int32_t*>(in_host_ + in.off_rs_fresh);
@@ -246,7 +252,7 @@ void Executor::prepare_stack(const BatchPlan& plan, const Inputs& in) {
         qo[r] = q0;
         for (int i = q0; i < q1; ++i) {
             row_req[i] = r;
-            prev[i] = i > q0 ? static_cast<int32_t>(plan.tokens[i - 1]) : -1;
+            pair[i] = pair_row(i > q0 ? static_cast<int32_t>(plan.tokens[i - 1]) : -1, plan.tokens[i]);
             if (i > q0 && plan.positions[i] != plan.positions[i - 1] + 1)
                 throw std::runtime_error("executor: a request's rows must be consecutive positions");
         }
@@ -265,7 +271,7 @@ void Executor::prepare_stack(const BatchPlan& plan, const Inputs& in) {
                                      std::to_string(plan.positions[q0]));
         slot[r] = static_cast<int32_t>(s);
         fresh[r] = reset ? 1 : 0;
-        if (!reset) prev[q0] = rs_last_[s];
+        if (!reset) pair[q0] = pair_row(rs_last_[s], plan.tokens[q0]);
     }
     qo[plan.R] = plan.N;
     if (recurrent)
@@ -402,7 +408,7 @@ void Executor::stack_mixture(const StackLayer& w, int N) {
             return;
         }
         PIE_KERNEL(pie_hip_moe_grouped_gemm_glu(PIE_HIP_FMT_BF16, static_cast<const uint16_t*>(act), rows, stack_.route_offsets, E,
-                                                hint, l.data_tiled ? l.data_tiled : l.data, l.data_bytes() / E, nullptr, 0, 0, 0,
+                                                hint, routes, l.data_tiled ? l.data_tiled : l.data, l.data_bytes() / E, nullptr, 0, 0, 0,
                                                 static_cast<uint16_t*>(y), l.N / E, l.K, epilogue, l.data_tiled ? 1 : 0, rule,
                                                 stream_));
     };
@@ -728,10 +734,9 @@ void Executor::stack_shared_norm(int N, int max_kv_len, const Inputs& in) {
 void Executor::stack_gated(int N, int max_kv_len, const Inputs& in) {
     const ModelConfig& m = model_.cfg();
     const int H = m.hidden, ld = model_.ld_x(), taps = m.canon_taps;
-    PIE_KERNEL(pie_hip_embed_bigram(reinterpret_cast<const uint32_t*>(in_dev_ + in.off_tokens),
-                                    reinterpret_cast<const int32_t*>(in_dev_ + in.off_prev), model_.embed, m.vocab, m.embed_scale,
-                                    model_.bigram, m.bigram.buckets, m.bigram.mul_prev, m.bigram.mul_cur, model_.embed_norm, stack_.x, N, H,
-                                    ld, m.rms_eps, stream_));
+    const PieHipEmbedding start{reinterpret_cast<const uint32_t*>(in_dev_ + in.off_tokens),
+                                reinterpret_cast<const int32_t*>(in_dev_ + in.off_pair), model_.embed, model_.bigram, model_.embed_norm, m.vocab,
+                                m.embed_scale};
     struct Sublayer {
         const float *norm, *canon, *gate_bias;
         const Linear* gate;
@@ -742,17 +747,17 @@ void Executor::stack_gated(int N, int max_kv_len, const Inputs& in) {
         return n == 0 ? Sublayer{w.pre1, w.canon1, w.gate1_bias, &w.w_gate1, rs_canon_off_[run][0]}
                       : Sublayer{w.pre2, w.canon2, w.gate2_bias, &w.w_gate2, rs_canon_off_[run][1]};
     };
-    // the output of `from` (none at the start: y and routes null) joins the stream, which `to` (null: the last one
+    // the output of `from` (null: the embedding starts the stream) joins the stream, which `to` (null: the last one
     // has ended) reads
     auto join = [&](const Sublayer* from, const void* y, const PieHipRoutes* routes, const Sublayer* to) {
-        if (!from && !to) return;
         PieHipStateRows state{};
         if (to) {
             state = state_rows(0, N, in);
             state.conv_offset = to->state;
         }
         const bool fused = to && plan_->pure_decode && taps <= 4;
-        PIE_KERNEL(pie_hip_gated_join(dt_, y, ld, routes, from ? stack_.sub_gate : nullptr, ld, from ? from->gate_bias : nullptr, stack_.x,
+        PIE_KERNEL(pie_hip_gated_join(dt_, y, ld, routes, from ? stack_.sub_gate : nullptr, ld, from ? from->gate_bias : nullptr, from ? nullptr : &start,
+                                      stack_.x,
                                       to ? to->norm : nullptr, stack_.h, stack_.xa, fused ? to->canon : nullptr, taps, &state, N, H, ld,
                                       m.rms_eps, stream_));
         if (!to) return;

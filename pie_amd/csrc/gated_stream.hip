@@ -1,9 +1,9 @@
 // The residual stream of layers whose sublayers' outputs pass a logistic gate and whose sublayers read a short
 // convolution of the normed stream:
 //   h = norm(x),  x += sublayer(h + conv(h)) * sigmoid(W h + b)
-//   embed_bigram   the stream's start: a token's row and the row of its pair with the previous token, normed
 //   gated_join     what ends a sublayer: the gated output joins the fp32 stream, which is normed for the next one;
-//                  with one row per request the convolution and the move of its state ride along
+//                  with one row per request the convolution and the move of its state ride along.  The stream's
+//                  start is the same kernel: the normed sum of up to two embedding rows instead of a stream
 //   recent_rows    the convolution of portions, over the requests' rows and states
 // The normed row is rounded to the compute type before anything reads it, so that the convolution of a row
 // does not depend on which of the two kernels formed it.
@@ -12,55 +12,11 @@
 namespace pie_hip {
 namespace {
 
-struct EmbedBigramArgs {
-    const uint32_t* tokens;
-    const int32_t* prev;
-    const uint16_t *table, *bigram;
-    const float* norm_w;
-    float* x;
-    unsigned long long buckets, mul_prev, mul_cur;
-    int vocab, width, ld;
-    float scale, eps;
-};
-__global__ __launch_bounds__(256) void embed_bigram_kernel(const EmbedBigramArgs a) {
-    __shared__ float red[4];
-    const size_t n = blockIdx.x;
-    const uint32_t t = a.tokens[n];
-    const uint16_t* er = a.table + static_cast<size_t>(t < static_cast<uint32_t>(a.vocab) ? t : 0) * a.width;
-    const uint16_t* br = nullptr;
-    if (a.bigram) {
-        const int32_t p = a.prev[n];
-        const unsigned long long row = p < 0 ? a.buckets
-                                             : (static_cast<unsigned long long>(p) * a.mul_prev + static_cast<unsigned long long>(t) * a.mul_cur) % a.buckets;
-        br = a.bigram + row * a.width;
-    }
-    float* xr = a.x + n * a.ld;
-    constexpr int kCache = 16;   // values of a thread that stay in registers
-    float v[kCache], local = 0.f;
-    auto value = [&](int i) { return bf16_bits_to_f32(er[i]) * a.scale + (br ? bf16_bits_to_f32(br[i]) : 0.f); };
-#pragma unroll
-    for (int c = 0; c < kCache; ++c) {
-        const int i = threadIdx.x + c * 256;
-        v[c] = i < a.width ? value(i) : 0.f;
-        local += v[c] * v[c];
-    }
-    for (int i = threadIdx.x + kCache * 256; i < a.width; i += 256) {
-        const float e = value(i);
-        local += e * e;
-    }
-    const float inv = 1.f / sqrtf(block_total(local, red) / static_cast<float>(a.width) + a.eps);
-#pragma unroll
-    for (int c = 0; c < kCache; ++c) {
-        const int i = threadIdx.x + c * 256;
-        if (i < a.width) xr[i] = v[c] * inv * a.norm_w[i];
-    }
-    for (int i = threadIdx.x + kCache * 256; i < a.width; i += 256) xr[i] = value(i) * inv * a.norm_w[i];
-}
-
 struct GatedJoinArgs {
     const void *y, *gate;
     const float *gate_bias, *next_w, *conv_w;
     PieHipRoutes routes;
+    PieHipEmbedding start;
     float* x;
     void *h, *recent;
     PieHipStateRows state;
@@ -81,7 +37,13 @@ __global__ __launch_bounds__(BLOCK) void gated_join_kernel(const GatedJoinArgs a
     const T* gr = a.gate ? static_cast<const T*>(a.gate) + n * a.ld_gate : nullptr;
     const T* ry = static_cast<const T*>(a.routes.y);
     const int K = ry ? a.routes.top_k : 0;
-    const bool joins = yr || K;
+    const bool joins = yr || K, starts = a.start.token_ids != nullptr;
+    const uint16_t *er = nullptr, *pr = nullptr;
+    if (starts) {
+        const uint32_t t = a.start.token_ids[n];
+        er = a.start.table + static_cast<size_t>(t < static_cast<uint32_t>(a.start.vocab) ? t : 0) * a.width;
+        if (a.start.pair_table) pr = a.start.pair_table + static_cast<size_t>(a.start.pair_rows[n]) * a.width;
+    }
     float* xr = a.x + n * a.ld;
     T* hr = static_cast<T*>(a.h) + n * a.ld;
     T* rr = static_cast<T*>(a.recent) + n * a.ld;
@@ -105,7 +67,14 @@ __global__ __launch_bounds__(BLOCK) void gated_join_kernel(const GatedJoinArgs a
     float v[8], local = 0.f;
     Eight<float> nw, cw[TAPS > 0 ? TAPS : 1];
     Eight<T> past[KEEP > 0 ? KEEP : 1];
+    Eight<float> sw;
     if (mine) {
+        Eight<uint16_t> ge, gp;
+        if (starts) {
+            ge.load(er + i8);
+            if (pr) gp.load(pr + i8);
+            sw.load(a.start.norm_weight + i8);
+        }
         Eight<T> gy, gz;
         Eight<float> gb, gx;
         if (yr) gy.load(yr + i8);
@@ -113,7 +82,7 @@ __global__ __launch_bounds__(BLOCK) void gated_join_kernel(const GatedJoinArgs a
             gz.load(gr + i8);
             gb.load(a.gate_bias + i8);
         }
-        gx.load(xr + i8);
+        if (!starts) gx.load(xr + i8);
         if (a.next_w) nw.load(a.next_w + i8);
         if constexpr (TAPS > 0) {
 #pragma unroll
@@ -138,14 +107,31 @@ __global__ __launch_bounds__(BLOCK) void gated_join_kernel(const GatedJoinArgs a
         }
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
-            v[e] = joins ? fmaf(v[e], sigmoid_f32(gz.get(e) + gb.get(e)), gx.get(e)) : gx.get(e);
+            if (!starts) v[e] = joins ? fmaf(v[e], sigmoid_f32(gz.get(e) + gb.get(e)), gx.get(e)) : gx.get(e);
+            else v[e] = ge.get(e) * a.start.scale + (pr ? gp.get(e) : 0.f);
             local += v[e] * v[e];
         }
-        if (joins)
-#pragma unroll
-            for (int p = 0; p < 2; ++p)
-                *reinterpret_cast<f32x4_t*>(xr + i8 + 4 * p) = f32x4_t{v[4 * p], v[4 * p + 1], v[4 * p + 2], v[4 * p + 3]};
     }
+    if (starts) {   // (uniform: the whole block)
+        for (int i = done + threadIdx.x; i < a.width; i += BLOCK) {
+            const float o = bf16_bits_to_f32(er[i]) * a.start.scale + (pr ? bf16_bits_to_f32(pr[i]) : 0.f);
+            xr[i] = o;
+            local += o * o;
+        }
+        const float inv = 1.f / sqrtf(block_total(local, red) / static_cast<float>(a.width) + a.eps);
+        local = 0.f;
+        if (mine)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                v[e] *= inv * sw.get(e);
+                local += v[e] * v[e];
+            }
+        for (int i = done + threadIdx.x; i < a.width; i += BLOCK) xr[i] *= inv * a.start.norm_weight[i];
+    }
+    if (mine && (joins || starts))
+#pragma unroll
+        for (int p = 0; p < 2; ++p)
+            *reinterpret_cast<f32x4_t*>(xr + i8 + 4 * p) = f32x4_t{v[4 * p], v[4 * p + 1], v[4 * p + 2], v[4 * p + 3]};
     for (int i = done + threadIdx.x; i < a.width; i += BLOCK) {
         float s = yr ? act_get<T>(yr[i]) : 0.f;
         for (int k = 0; k < K; ++k) s = fmaf(act_get<T>(ry[static_cast<size_t>(pos[k]) * a.routes.ld + i]), weight[k], s);
@@ -310,25 +296,13 @@ int launch_recent_rows(const T* h, const float* w, int taps, const PieHipStateRo
 
 using namespace pie_hip;
 
-extern "C" int pie_hip_embed_bigram(const uint32_t* token_ids, const int32_t* prev_ids, const uint16_t* table_bf16, int vocab,
-                                    float table_scale, const uint16_t* bigram_bf16, unsigned long long buckets,
-                                    unsigned long long mul_prev, unsigned long long mul_cur, const float* norm_weight,
-                                    float* x, int num_tokens, int width, int ld, float eps, void* stream) {
-    if (!token_ids || !table_bf16 || vocab <= 0 || !norm_weight || !x || num_tokens <= 0 || width <= 0 || ld < width ||
-        (bigram_bf16 && (!prev_ids || buckets == 0)))
-        return PIE_HIP_ERR_INVALID;
-    const EmbedBigramArgs a{token_ids, prev_ids, table_bf16, bigram_bf16, norm_weight, x, buckets, mul_prev, mul_cur, vocab, width, ld,
-                            table_scale, eps};
-    hipLaunchKernelGGL(embed_bigram_kernel, dim3(num_tokens), dim3(256), 0, static_cast<hipStream_t>(stream), a);
-    return launch_status();
-}
-
 extern "C" int pie_hip_gated_join(int dtype, const void* y, int ldy, const PieHipRoutes* routes, const void* gate, int ld_gate,
-                                  const float* gate_bias, float* x, const float* next_weight, void* h, void* recent,
-                                  const float* conv_w, int taps, const PieHipStateRows* state, int rows, int width, int ld,
+                                  const float* gate_bias, const PieHipEmbedding* start, float* x, const float* next_weight,
+                                  void* h, void* recent, const float* conv_w, int taps, const PieHipStateRows* state, int rows, int width, int ld,
                                   float eps, void* stream) {
     if (!x || rows <= 0 || width <= 0 || ld < width || (y && (routes || ldy < width)) || (next_weight && !h) ||
-        ((y || routes) && (!gate || !gate_bias || ld_gate < width)) || (!y && !routes && !next_weight) ||
+        ((y || routes) && (start || !gate || !gate_bias || ld_gate < width)) || (!y && !routes && !start && !next_weight) ||
+        (start && (!start->token_ids || !start->table || !start->norm_weight || start->vocab <= 0 || (start->pair_table && !start->pair_rows))) ||
         (routes && (!routes->y || !routes->pos || !routes->weight || routes->top_k <= 0 || routes->ld < width)))
         return PIE_HIP_ERR_INVALID;
     if (conv_w && (!next_weight || !recent || taps <= 0 || !state_ok(state) || state->num_tokens != rows || state->num_requests != rows ||
@@ -337,7 +311,7 @@ extern "C" int pie_hip_gated_join(int dtype, const void* y, int ldy, const PieHi
     if ((y && ldy % 8 != 0) || ((y || routes) && ld_gate % 8 != 0) || (routes && (routes->ld % 8 != 0 || routes->top_k > kJoinRoutes)) ||
         ld % 8 != 0 || (conv_w && taps > 4))
         return PIE_HIP_ERR_UNSUPPORTED;
-    const GatedJoinArgs a{y, gate, gate_bias, next_weight, conv_w, routes ? *routes : PieHipRoutes{}, x, h, recent,
+    const GatedJoinArgs a{y, gate, gate_bias, next_weight, conv_w, routes ? *routes : PieHipRoutes{}, start ? *start : PieHipEmbedding{}, x, h, recent,
                           conv_w ? *state : PieHipStateRows{}, ldy, ld_gate, width, ld, eps};
     hipStream_t s = static_cast<hipStream_t>(stream);
     PIE_ACT_DISPATCH(dtype, T, {

@@ -131,6 +131,7 @@ struct SkinnyArgs {
     int m_split;                // dense only: blockIdx.y = 16-row pass
     int tiled;                  // weights (and int4 group scales) in the tile-major layout
     size_t w_stride, scale_stride;  // bytes between problems
+    int busy;                       // at most this many problems have rows (0: not known)
     // q|k|v epilogue of the wave-private form (rope_table != null): rows of W are the q, k and
     // v heads; adjacent output pairs of q and k heads are rotated, q goes to y [rows, hq*d], k
     // and v to slot kv_slots[row] of the page pools
@@ -883,7 +884,7 @@ int launch_skinny(SkinnyArgs a, int problems, hipStream_t stream) {
     // tiles of 16 weight rows per block: as many as still leave two blocks per CU; with few
     // tiles, eight waves split K instead of four.  Paired loads (whole 128-byte lines per row
     // and wave) when K allows.
-    const long tiles = static_cast<long>((a.N + 15) / 16) * (a.m_split ? (a.M + 15) / 16 : problems);
+    const long tiles = static_cast<long>((a.N + 15) / 16) * (a.m_split ? (a.M + 15) / 16 : a.busy > 0 && a.busy < problems ? a.busy : problems);
     constexpr int W8 = (CK / (8 * LK) >= 2) ? 2 : 1;   // loads per step with eight waves
     static const bool old_form = getenv("PIE_SKINNY_OLD") != nullptr;
     // dense tile-major launches take the wave-private form (measured, 8B decode steps of 8 / 16 /
@@ -991,7 +992,7 @@ int skinny_entry(int format, const uint16_t* act_bf16, const void* weight, const
 }
 
 int grouped_entry(int format, const uint16_t* act_bf16, const int32_t* route_act_rows, const int32_t* expert_offsets,
-                  int num_experts, int max_rows_per_expert, const void* weights, size_t weight_stride_bytes,
+                  int num_experts, int max_rows_per_expert, int num_routes, const void* weights, size_t weight_stride_bytes,
                   const void* scales, size_t scale_stride_bytes, int scale_is_bf16, int group_size, uint16_t* y_bf16,
                   int N, int K, int swiglu, int tiled, const PieHipGlu* glu, void* stream) {
     if (!act_bf16 || !expert_offsets || !weights || !y_bf16 || num_experts <= 0 || max_rows_per_expert <= 0 ||
@@ -1015,6 +1016,7 @@ int grouped_entry(int format, const uint16_t* act_bf16, const int32_t* route_act
     a.tiled = tiled ? 1 : 0;
     a.w_stride = weight_stride_bytes;
     a.scale_stride = scale_stride_bytes;
+    a.busy = num_routes;
     return dispatch_skinny(format, a, num_experts, static_cast<hipStream_t>(stream));
 }
 }  // namespace
@@ -1039,17 +1041,18 @@ extern "C" int pie_hip_moe_grouped_gemm(int format, const uint16_t* act_bf16, co
                                         const void* weights, size_t weight_stride_bytes, const void* scales,
                                         size_t scale_stride_bytes, int scale_is_bf16, int group_size, uint16_t* y_bf16,
                                         int N, int K, int swiglu, void* stream) {
-    return pie_hip::grouped_entry(format, act_bf16, route_act_rows, expert_offsets, num_experts, max_rows_per_expert, weights,
+    return pie_hip::grouped_entry(format, act_bf16, route_act_rows, expert_offsets, num_experts, max_rows_per_expert, 0, weights,
                                   weight_stride_bytes, scales, scale_stride_bytes, scale_is_bf16, group_size, y_bf16, N, K,
                                   swiglu, 0, nullptr, stream);
 }
 
 extern "C" int pie_hip_moe_grouped_gemm_glu(int format, const uint16_t* act_bf16, const int32_t* route_act_rows,
                                             const int32_t* expert_offsets, int num_experts, int max_rows_per_expert,
-                                            const void* weights, size_t weight_stride_bytes, const void* scales,
-                                            size_t scale_stride_bytes, int scale_is_bf16, int group_size, uint16_t* y_bf16,
-                                            int N, int K, int swiglu, int tiled, const PieHipGlu* glu, void* stream) {
-    return pie_hip::grouped_entry(format, act_bf16, route_act_rows, expert_offsets, num_experts, max_rows_per_expert, weights,
+                                            int num_routes, const void* weights, size_t weight_stride_bytes,
+                                            const void* scales, size_t scale_stride_bytes, int scale_is_bf16,
+                                            int group_size, uint16_t* y_bf16, int N, int K, int swiglu, int tiled,
+                                            const PieHipGlu* glu, void* stream) {
+    return pie_hip::grouped_entry(format, act_bf16, route_act_rows, expert_offsets, num_experts, max_rows_per_expert, num_routes, weights,
                                   weight_stride_bytes, scales, scale_stride_bytes, scale_is_bf16, group_size, y_bf16, N, K,
                                   swiglu, tiled, glu, stream);
 }
@@ -1104,7 +1107,7 @@ extern "C" int pie_hip_moe_grouped_gemm_tiled(int format, const uint16_t* act_bf
                                               const void* weights, size_t weight_stride_bytes, const void* scales,
                                               size_t scale_stride_bytes, int scale_is_bf16, int group_size, uint16_t* y_bf16,
                                               int N, int K, int swiglu, void* stream) {
-    return pie_hip::grouped_entry(format, act_bf16, route_act_rows, expert_offsets, num_experts, max_rows_per_expert, weights,
+    return pie_hip::grouped_entry(format, act_bf16, route_act_rows, expert_offsets, num_experts, max_rows_per_expert, 0, weights,
                                   weight_stride_bytes, scales, scale_stride_bytes, scale_is_bf16, group_size, y_bf16, N, K,
                                   swiglu, 1, nullptr, stream);
 }

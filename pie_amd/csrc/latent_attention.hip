@@ -44,27 +44,50 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
     // both sums of squares: waves 0-1 the query latent, waves 2-3 the key/value latent
     const int half = threadIdx.x >> 7, t = threadIdx.x & 127;
     const T* src = half ? fk : fq;
-    const int len = half ? (kv_norm ? kv_rank : 0) : q_rank;
+    const float* wgt = half ? kv_norm : q_norm;
+    const int len = half ? (kv_norm ? kv_rank : 0) : q_rank, padded = half ? (kv_norm ? kvp : 0) : ld_cq;
+    const int64_t slot = kv_norm ? kv_slots[n] : -1;
+    // eight values at a time, up to two groups per thread in registers with their weights (the groups' starts are
+    // multiples of 16 bytes where a row is read or written; longer latents, and a length's last values, one by one)
+    const bool whole = kv_off % 8 == 0 && ld_fused % 8 == 0 && ld_cq % 8 == 0 && kvp % 8 == 0 && ld_row % 8 == 0;
+    const int groups = whole ? min(len / 8, 256) : 0, done = 8 * groups;
+    Eight<T> x[2];
+    Eight<float> w[2];
     float local = 0.f;
-    for (int i = t; i < len; i += 128) {
+#pragma unroll
+    for (int c = 0; c < 2; ++c)
+        if (t + 128 * c < groups) {
+            x[c].load(src + 8 * (t + 128 * c));
+            w[c].load(wgt + 8 * (t + 128 * c));
+        }
+#pragma unroll
+    for (int c = 0; c < 2; ++c)
+        if (t + 128 * c < groups)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) local += x[c].get(e) * x[c].get(e);
+    for (int i = done + t; i < len; i += 128) {
         const float v = act_get<T>(src[i]);
         local += v * v;
     }
     local = wave_sum(local);
     if ((threadIdx.x & (kWave - 1)) == 0) red[threadIdx.x / kWave] = local;
     __syncthreads();
-    const float inv_q = 1.f / sqrtf((red[0] + red[1]) / static_cast<float>(q_rank) + eps);
-    const float inv_k = 1.f / sqrtf((red[2] + red[3]) / static_cast<float>(kv_rank) + eps);
-    for (int i = threadIdx.x; i < ld_cq; i += 256)
-        cq[n * ld_cq + i] = act_put<T>(i < q_rank ? act_get<T>(fq[i]) * inv_q * q_norm[i] : 0.f);
-    if (!kv_norm) return;
-    const int64_t slot = kv_slots[n];
-    if (slot < 0) return;
-    T* row = pool + static_cast<size_t>(slot) * ld_row;
-    for (int i = threadIdx.x; i < kvp; i += 256)
-        row[i] = act_put<T>(i < kv_rank ? act_get<T>(fk[i]) * inv_k * kv_norm[i] : 0.f);
+    const float inv = 1.f / sqrtf((red[2 * half] + red[2 * half + 1]) / static_cast<float>(half ? kv_rank : q_rank) + eps);
+    if (half && slot < 0) return;
+    T* dst = half ? pool + static_cast<size_t>(slot) * ld_row : cq + n * ld_cq;
+#pragma unroll
+    for (int c = 0; c < 2; ++c)
+        if (t + 128 * c < groups) {
+            float o[8];
+#pragma unroll
+            for (int e = 0; e < 8; ++e) o[e] = x[c].get(e) * inv * w[c].get(e);
+            store_eight<T>(dst + 8 * (t + 128 * c), o);
+        }
+    for (int i = done + t; i < padded; i += 128) dst[i] = act_put<T>(i < len ? act_get<T>(src[i]) * inv * wgt[i] : 0.f);
+    if (!half) return;   // (the rotated key part: waves 2-3)
+    T* row = dst;
     const float* tab = rope_table + n * rot_dims;
-    for (int i = threadIdx.x; i < ld_row - kvp; i += 256) {
+    for (int i = t; i < ld_row - kvp; i += 128) {
         float v = 0.f;
         if (i < rot_dim)
             v = rotated_entry(i, rot_dims, tab, [&](int e) { return act_get<T>(fk[kv_rank + e]); });
@@ -122,6 +145,15 @@ __global__ __launch_bounds__(kWave) void head_linear_mfma_kernel(const HeadArgs 
     for (int t = 0; t < MT; ++t)
         ap[t] = static_cast<const uint16_t*>(a.act) + static_cast<size_t>(min(m0 + 16 * t + l16, a.M - 1)) * a.ld_act +
                 static_cast<size_t>(h) * a.act_stride + 8 * g;
+    // (requested ahead of the products)
+    float head_gate[MT];
+    u32x2_t value_gate[MT];
+#pragma unroll
+    for (int t = 0; t < MT; ++t) {
+        const uint16_t* gp = static_cast<const uint16_t*>(a.gate) + static_cast<size_t>(min(m0 + 16 * t + l16, a.M - 1)) * a.ld_gate;
+        if (a.gate && a.gate_cols == 1) head_gate[t] = bf16_bits_to_f32(gp[h]);
+        else if (a.gate) value_gate[t] = *reinterpret_cast<const u32x2_t*>(gp + h * a.C + c0 + 4 * g);
+    }
     f32x4_t acc[MT];
 #pragma unroll
     for (int t = 0; t < MT; ++t) acc[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
@@ -152,10 +184,9 @@ __global__ __launch_bounds__(kWave) void head_linear_mfma_kernel(const HeadArgs 
         uint16_t* yp = static_cast<uint16_t*>(a.y) + static_cast<size_t>(m) * a.ld_y + static_cast<size_t>(h) * a.y_stride + c0 + 4 * g;
         f32x4_t v = acc[t];
         if (a.gate && a.gate_cols == 1) {
-            v *= sigmoid_f32(bf16_bits_to_f32(static_cast<const uint16_t*>(a.gate)[static_cast<size_t>(m) * a.ld_gate + h]));
+            v *= sigmoid_f32(head_gate[t]);
         } else if (a.gate) {
-            const u32x2_t r = *reinterpret_cast<const u32x2_t*>(static_cast<const uint16_t*>(a.gate) + static_cast<size_t>(m) * a.ld_gate +
-                                                                h * a.C + c0 + 4 * g);
+            const u32x2_t r = value_gate[t];
             v *= f32x4_t{sigmoid_f32(bf16_lo(r.x)), sigmoid_f32(bf16_hi(r.x)), sigmoid_f32(bf16_lo(r.y)), sigmoid_f32(bf16_hi(r.y))};
         }
         *reinterpret_cast<u32x2_t*>(yp) = u32x2_t{pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3])};

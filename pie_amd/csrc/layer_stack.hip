@@ -315,14 +315,7 @@ __global__ __launch_bounds__(BLOCK) void residual_join_kernel(const JoinArgs a) 
 #pragma unroll
             for (int e = 0; e < 8; ++e) o[e] *= w.get(e) * scale;
         }
-        if constexpr (sizeof(T) == 2) {
-            *reinterpret_cast<u32x4_t*>(ar + i) =
-                u32x4_t{pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3]), pack_bf16x2(o[4], o[5]), pack_bf16x2(o[6], o[7])};
-        } else {
-#pragma unroll
-            for (int h = 0; h < 2; ++h)
-                *reinterpret_cast<f32x4_t*>(ar + i + 4 * h) = f32x4_t{o[4 * h], o[4 * h + 1], o[4 * h + 2], o[4 * h + 3]};
-        }
+        store_eight<T>(ar + i, o);
     }
     for (int i = done + threadIdx.x; i < a.width; i += BLOCK)   // (a thread reads what it wrote)
         ar[i] = act_put<T>(a.next_w ? xr[i] * (scale * a.next_w[i]) : xr[i]);

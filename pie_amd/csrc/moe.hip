@@ -349,17 +349,18 @@ __global__ __launch_bounds__(kNormRouteThreads) void moe_norm_route_kernel(
     }
 }
 
-// One block: rank of every route inside its expert, expert offsets, sorted positions.
+// One block: rank of every route inside its expert, expert offsets, sorted positions.  The first `shared` routes of
+// every token are experts 0 .. shared - 1: their ranks are the tokens.
 __device__ __forceinline__ void sort_routes(const int32_t* topk_idx, int32_t* __restrict__ expert_offsets,
                                             int32_t* __restrict__ route_token, int32_t* __restrict__ route_pos, int N, int E,
-                                            int K) {
+                                            int K, int shared = 0) {
     __shared__ int cnt[kMaxExperts];
     __shared__ int base[kMaxExperts + 1];
     const int tid = threadIdx.x, lane = tid & (kWave - 1), wv = tid / kWave;
-    for (int e = tid; e < E; e += kRouteThreads) cnt[e] = 0;
+    for (int e = tid; e < E; e += kRouteThreads) cnt[e] = e < shared ? N : 0;
     __syncthreads();
     const int R = N * K;
-    for (int r = tid; r < R; r += kRouteThreads) route_pos[r] = atomicAdd(&cnt[topk_idx[r]], 1);
+    for (int r = tid; r < R; r += kRouteThreads) route_pos[r] = r % K < shared ? r / K : atomicAdd(&cnt[topk_idx[r]], 1);
     __syncthreads();
     if (wv == 0) {
         // exclusive scan of cnt[0..E): each lane owns a run of consecutive experts
@@ -395,8 +396,8 @@ __device__ __forceinline__ void sort_routes(const int32_t* topk_idx, int32_t* __
 }
 __global__ __launch_bounds__(kRouteThreads) void moe_sort_kernel(
     const int32_t* __restrict__ topk_idx, int32_t* __restrict__ expert_offsets,
-    int32_t* __restrict__ route_token, int32_t* __restrict__ route_pos, int N, int E, int K) {
-    sort_routes(topk_idx, expert_offsets, route_token, route_pos, N, E, K);
+    int32_t* __restrict__ route_token, int32_t* __restrict__ route_pos, int N, int E, int K, int shared) {
+    sort_routes(topk_idx, expert_offsets, route_token, route_pos, N, E, K, shared);
 }
 
 // fp32 logits and groups of experts: one wave per token, four to a block.
@@ -498,7 +499,7 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_corrected_kernel(cons
     const int lane = threadIdx.x & (kWave - 1), t = threadIdx.x / kWave;
     if (t < N) corrected_of_token(r, lane, t, topk_idx, topk_w);
     __syncthreads();   // (a block's stores are seen by its own threads after the barrier)
-    sort_routes(topk_idx, expert_offsets, route_token, route_pos, N, r.E + r.shared, r.top + r.shared);
+    sort_routes(topk_idx, expert_offsets, route_token, route_pos, N, r.E + r.shared, r.top + r.shared, r.shared);
 }
 
 __global__ __launch_bounds__(256) void moe_combine_kernel(
@@ -635,7 +636,7 @@ extern "C" int pie_hip_moe_norm_route(const uint16_t* x_bf16, const uint16_t* no
                        norm_weight_bf16, router_bf16, norm_out_bf16, router_logits_bf16, topk_idx, topk_weight,
                        hidden, num_experts, top_k, eps, renormalize ? 1 : 0);
     hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(kRouteThreads), 0, st, topk_idx, expert_offsets,
-                       route_token, route_pos, num_tokens, num_experts, top_k);
+                       route_token, route_pos, num_tokens, num_experts, top_k, 0);
     return launch_status();
 }
 
@@ -679,7 +680,7 @@ extern "C" int pie_hip_moe_route_opt(const uint16_t* router_logits_bf16, int32_t
                        router_logits_bf16, topk_idx, topk_weight, num_tokens, num_experts, top_k,
                        renormalize ? 1 : 0);
     hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(kRouteThreads), 0, st, topk_idx, expert_offsets,
-                       route_token, route_pos, num_tokens, num_experts, top_k);
+                       route_token, route_pos, num_tokens, num_experts, top_k, 0);
     return launch_status();
 }
 
@@ -703,7 +704,7 @@ extern "C" int pie_hip_moe_route_groups(const float* router_logits, int ld_logit
     hipLaunchKernelGGL(moe_topk_groups_kernel, dim3((num_tokens + 3) / 4), dim3(256), 0, st, router_logits, ld_logits, topk_idx,
                        topk_weight, num_tokens, num_experts, top_k, groups);
     hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(kRouteThreads), 0, st, topk_idx, expert_offsets, route_token, route_pos,
-                       num_tokens, num_experts, top_k);
+                       num_tokens, num_experts, top_k, 0);
     return launch_status();
 }
 
@@ -726,7 +727,7 @@ extern "C" int pie_hip_moe_route_corrected(const float* router_logits, int ld_lo
     }
     hipLaunchKernelGGL(moe_topk_corrected_kernel, dim3((num_tokens + 3) / 4), dim3(256), 0, st, r, topk_idx, topk_weight, num_tokens);
     hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(kRouteThreads), 0, st, topk_idx, expert_offsets, route_token, route_pos,
-                       num_tokens, num_experts + shared, top_k + shared);
+                       num_tokens, num_experts + shared, top_k + shared, shared);
     return launch_status();
 }
 

@@ -1347,10 +1347,11 @@ def moe_route_groups(logits: torch.Tensor, experts: int, top: int, groups: int, 
 
 
 def moe_grouped_glu(act: torch.Tensor, rows, offsets: torch.Tensor, w: torch.Tensor, routes: int, rule: Optional[Glu],
-                    block_rows: Optional[int] = None, tiled: bool = False, epilogue: int = 0) -> torch.Tensor:
+                    block_rows: Optional[int] = None, tiled: bool = False, epilogue: int = 0,
+                    known: bool = True) -> torch.Tensor:
     """Rows sorted by expert times w [experts, N, K] (gated if there is a rule, else with a pointwise epilogue); bf16 or
     fp32 by act's type.  bf16 with block_rows: in blocks of that many routes (0: the library's choice), `tiled`: over
-    tile-major weights."""
+    tile-major weights, `known`: the library is told the number of routes."""
     E, N, K = w.shape
     lib = kernels()
     if act.dtype == torch.float32:
@@ -1369,7 +1370,7 @@ def moe_grouped_glu(act: torch.Tensor, rows, offsets: torch.Tensor, w: torch.Ten
                                                  epilogue if rule is None else 1, int(tiled), glu_arg, block_rows, _stream()),
                "pie_hip_moe_grouped_gemm_mfma")
         return y
-    _check(lib.pie_hip_moe_grouped_gemm_glu(3, _ptr(act), _ptr(rows), _ptr(offsets), E, max(1, routes), _ptr(w), C.c_size_t(N * K * 2), None,
+    _check(lib.pie_hip_moe_grouped_gemm_glu(3, _ptr(act), _ptr(rows), _ptr(offsets), E, max(1, routes), routes if known else 0, _ptr(w), C.c_size_t(N * K * 2), None,
                                             C.c_size_t(0), 0, 0, _ptr(y), N, K, epilogue if rule is None else 1, int(tiled), glu_arg, _stream()),
            "pie_hip_moe_grouped_gemm_glu")
     return y
@@ -1502,27 +1503,28 @@ def gated_part_norm(o, x, skip, z, norm_w, heads, vdim, parts, rows: StateRows, 
     return y
 
 
-def embed_bigram(tokens, prev, table, scale: float, bigram, buckets: int, mul_prev: int, mul_cur: int, norm_w, ld: int, eps: float) -> torch.Tensor:
-    """x [N, ld]: the normed sum of a token's row and the row of its pair with the previous one (prev < 0: none)."""
-    width = table.shape[1]
-    x = torch.zeros((tokens.numel(), ld), dtype=torch.float32, device=table.device)
-    u64 = C.c_ulonglong
-    _check(kernels().pie_hip_embed_bigram(_ptr(tokens), _ptr(prev), _ptr(table), table.shape[0], C.c_float(scale), _ptr(bigram), u64(buckets),
-                                          u64(mul_prev), u64(mul_cur), _ptr(norm_w), _ptr(x), tokens.numel(), width, ld, C.c_float(eps),
-                                          _stream()), "pie_hip_embed_bigram")
-    return x
+class Embedding(C.Structure):
+    """PieHipEmbedding: a table's rows, a second table's rows, the norm of their sum."""
+    _fields_ = [("token_ids", C.c_void_p), ("pair_rows", C.c_void_p), ("table", C.c_void_p), ("pair_table", C.c_void_p), ("norm_weight", C.c_void_p),
+                ("vocab", C.c_int), ("scale", C.c_float)]
+
+
+def embedding(tokens, table, scale: float, norm_weight, pair_rows=None, pair_table=None) -> Embedding:
+    address = lambda x: None if x is None else x.data_ptr()
+    return Embedding(tokens.data_ptr(), address(pair_rows), table.data_ptr(), address(pair_table), norm_weight.data_ptr(), table.shape[0], scale)
 
 
 def gated_join(x: torch.Tensor, width: int, eps: float, dtype, y=None, routes=None, gate=None, gate_bias=None, next_weight=None, conv_w=None,
-               rows: Optional[StateRows] = None):
-    """x takes y (or routes, as in residual_join) times the logistic function of gate + gate_bias in place; returns
-    (h, recent): x normed, and with conv_w [taps, width] (one row per request) h plus its convolution."""
+               rows: Optional[StateRows] = None, start: Optional[Embedding] = None):
+    """x takes y (or routes, as in residual_join) times the logistic function of gate + gate_bias in place, or is set to
+    an embedding; returns (h, recent): x normed, and with conv_w [taps, width] (one row per request) h plus its convolution."""
     _dev(x, torch.float32, "x")
     h, recent = (torch.zeros(x.shape, dtype=dtype, device=x.device) for _ in range(2))
     r = None if routes is None else Routes(routes[0].data_ptr(), routes[1].data_ptr(), routes[2].data_ptr(), routes[1].shape[1],
                                            routes[0].shape[1])
     _check(kernels().pie_hip_gated_join(_dt(h), _ptr(y), 0 if y is None else y.shape[1], None if r is None else C.byref(r), _ptr(gate),
-                                        0 if gate is None else gate.shape[1], _ptr(gate_bias), _ptr(x), _ptr(next_weight), _ptr(h),
+                                        0 if gate is None else gate.shape[1], _ptr(gate_bias),
+                                        None if start is None else C.byref(start), _ptr(x), _ptr(next_weight), _ptr(h),
                                         _ptr(recent) if conv_w is not None else None, _ptr(conv_w), 0 if conv_w is None else conv_w.shape[0],
                                         None if rows is None else C.byref(rows), x.shape[0], width, x.shape[1], C.c_float(eps), _stream()),
            "pie_hip_gated_join")

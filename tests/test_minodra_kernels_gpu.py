@@ -1,5 +1,5 @@
-"""GPU: the kernels of gated sublayers — bigram embedding, gated joins with the convolution behind them, convolutions of
-portions, corrected routes with shared experts — and of latent attention with sinks, gates per head and no rotated
+"""GPU: the kernels of gated sublayers — embeddings that start the stream, gated joins with the convolution behind them,
+convolutions of portions, corrected routes with shared experts — and of latent attention with sinks, gates per head and no rotated
 part, against double-precision statements."""
 import numpy as np
 import pytest
@@ -9,25 +9,6 @@ from test_decay_memory_gpu import host, i32, t
 from test_layer_stack_kernels_gpu import paged
 
 pytestmark = pytest.mark.gpu
-
-
-@pytest.mark.parametrize("width,ld", [(96, 128), (75, 128), (2048, 2048), (4098, 4224), (9000, 9088)])
-@pytest.mark.parametrize("buckets,mul_prev,mul_cur", [(37, 1 << 40, 12345678901), (1, 2, 3), (1000, 7, 9), (0, 0, 0)])
-def test_embed_bigram(gpu, width, ld, buckets, mul_prev, mul_cur):
-    import torch
-    from pie_amd import ops
-
-    rng = np.random.default_rng(width)
-    toks, prev = rng.integers(0, 50, 9), rng.integers(0, 50, 9)
-    prev[[0, 4]] = -1
-    toks[7] = 60   # (an id past the table reads row 0)
-    table, bigram = t(rng.standard_normal((50, width)), gpu, torch.bfloat16), t(rng.standard_normal((buckets + 1, width)), gpu, torch.bfloat16)
-    nw = rng.uniform(0.5, 1.5, width).astype(np.float32)
-    x = host(ops.embed_bigram(i32(toks, gpu), i32(prev, gpu), table, 2.5, bigram if buckets else None, buckets, mul_prev, mul_cur, t(nw, gpu), ld, 1e-3))
-    e = host(table)[np.where(toks < 50, toks, 0)] * 2.5
-    if buckets:
-        e = e + host(bigram)[[buckets if p < 0 else (int(p) * mul_prev + int(c) * mul_cur) % buckets for p, c in zip(prev, toks)]]
-    assert np.abs(x[:, :width] - ls.rms_norm(e, nw, 1e-3)).max() < 1e-5 and (x[:, width:] == 0).all()
 
 
 class Slots:
@@ -60,6 +41,35 @@ class Slots:
             states[self.slots[r]] = x[len(x) - self.keep:]
             at += n
         return out, states
+
+
+@pytest.mark.parametrize("bf", [False, True])
+@pytest.mark.parametrize("width,ld", [(96, 128), (75, 128), (2048, 2048), (4098, 4224), (9000, 9088)])
+@pytest.mark.parametrize("pairs", [0, 37])
+def test_an_embedding_starts_the_stream(gpu, bf, width, ld, pairs):
+    import torch
+    from pie_amd import ops
+
+    rng = np.random.default_rng(width)
+    dt, eps, rows = torch.bfloat16 if bf else torch.float32, 1e-3, 9
+    toks, pair = rng.integers(0, 50, rows), rng.integers(0, pairs + 1, rows)
+    toks[7] = 60   # (an id past the table reads row 0)
+    table, bigram = (t(rng.standard_normal((n, width)), gpu, torch.bfloat16) for n in (50, pairs + 1))
+    ew, nw = (rng.uniform(0.5, 1.5, width).astype(np.float32) for _ in range(2))
+    held = [i32(toks, gpu), i32(pair, gpu), t(ew, gpu)]
+    start = ops.embedding(held[0], table, 2.5, held[2], held[1] if pairs else None, bigram if pairs else None)
+    s, w = Slots(rng, gpu, dt, width, 3, [1] * rows, [1] * rows), rng.standard_normal((3, width)).astype(np.float32)
+    e = host(table)[np.where(toks < 50, toks, 0)] * 2.5 + (host(bigram)[pair] if pairs else 0.0)
+    want = ls.rms_norm(e, ew, eps)
+    for kw in (dict(next_weight=t(nw, gpu)), dict(next_weight=t(nw, gpu), conv_w=t(w, gpu), rows=s.rows), dict()):
+        x = t(np.full((rows, ld), 3.0, np.float32), gpu)   # (what was there before does not matter)
+        h, recent = (host(v) for v in ops.gated_join(x, width, eps, dt, start=start, **kw))
+        assert np.abs(host(x)[:, :width] - want).max() < 1e-5 and (host(x)[:, width:] == 3.0).all()
+        if kw:
+            assert np.abs(h[:, :width] - ls.rms_norm(want, nw, eps)).max() < (4e-2 if bf else 3e-5)
+        if "rows" in kw:
+            out, states = s.want(h[:, :width], w)
+            assert (np.abs(recent[:, :width] - out) < (5e-3 if bf else 1e-5) * (1.0 + np.abs(out))).all() and np.array_equal(host(s.view()), states)
 
 
 @pytest.mark.parametrize("bf", [False, True])
@@ -173,7 +183,7 @@ def test_grouped_products_with_squared_relu(gpu, form, T, E, top, shared, K, N):
     act, w = t(rng.standard_normal((T, K)), gpu, dt), t(rng.standard_normal((E + shared, N, K)) * 2 / np.sqrt(K), gpu, torch.bfloat16)
     z = rng.standard_normal((T, 32)).astype(np.float32)
     idx, _, offsets, token, pos = ops.moe_route_corrected(t(z, gpu), t(np.zeros(E, np.float32), gpu), top, shared)
-    kw = dict(block_rows=0) if form == "blocks" else {}
+    kw = dict(block_rows=0) if form == "blocks" else dict(known=T % 2 == 1)
     got = host(ops.moe_grouped_glu(act, token, offsets, w, T * (top + shared), None, epilogue=2, **kw))
     a, wh, idx, pos = host(act), host(w), host(idx).astype(int), host(pos).astype(int)
     for n in range(T):
@@ -302,7 +312,9 @@ def test_bad_arguments_are_refused(gpu):
             ops.moe_route_corrected(z, correction, top, shared)
     x, y = torch.zeros((2, 128), device=gpu), torch.zeros((2, 128), device=gpu)
     nw = torch.ones(96, device=gpu)
-    for kw in (dict(), dict(y=y, next_weight=nw), dict(next_weight=nw, conv_w=torch.zeros((3, 96), device=gpu)), dict(y=y, gate=y)):
+    tok, table = torch.zeros(2, dtype=torch.int32, device=gpu), torch.zeros((3, 96), dtype=torch.bfloat16, device=gpu)
+    start = ops.embedding(tok, table, 1.0, nw)
+    for kw in (dict(), dict(y=y, next_weight=nw), dict(y=y, gate=y, gate_bias=nw, start=start), dict(start=ops.embedding(tok, table, 1.0, nw, None, table)), dict(next_weight=nw, conv_w=torch.zeros((3, 96), device=gpu)), dict(y=y, gate=y)):
         with pytest.raises(KernelError):
             ops.gated_join(x, 96, 1e-5, torch.float32, **kw)
     rng = np.random.default_rng(0)
