@@ -1150,7 +1150,7 @@ int pie_hip_gated_part_norm(int dtype, const float* o, const void* x, int ld_x, 
  *   state moves on by the row.  Rows of ld; columns from the width on are not touched.
  * pie_hip_recent_rows: recent[n, c] = h[n, c] + sum_j conv_w[j, c] h_(n - (taps - 1) + j)[c], earlier rows from the
  *   request's state, zeros before its start; pie_hip_delta_conv_state (channels = width) moves the state on
- *   afterwards.  conv_w [taps, width] fp32; the state is [taps - 1, width] in the compute type at conv_offset.
+ *   afterwards.  conv_w [taps, width] bf16; the state is [taps - 1, width] in the compute type at conv_offset.
  */
 /* x[n] = e / sqrt(mean(e^2) + eps) * norm_weight, e = table[token_ids[n]] * scale + pair_table[pair_rows[n]] (pair_table
  * NULL: left out; ids >= vocab read row 0 of table). */
@@ -1164,9 +1164,9 @@ typedef struct {
 } PieHipEmbedding;
 int pie_hip_gated_join(int dtype, const void* y, int ldy, const PieHipRoutes* routes, const void* gate, int ld_gate,
                        const float* gate_bias, const PieHipEmbedding* start, float* x, const float* next_weight,
-                       void* h, void* recent, const float* conv_w, int taps, const PieHipStateRows* state, int rows, int width, int ld,
+                       void* h, void* recent, const uint16_t* conv_w, int taps, const PieHipStateRows* state, int rows, int width, int ld,
                        float eps, void* stream);
-int pie_hip_recent_rows(int dtype, const void* h, const float* conv_w, int taps, const PieHipStateRows* state, void* recent,
+int pie_hip_recent_rows(int dtype, const void* h, const uint16_t* conv_w, int taps, const PieHipStateRows* state, void* recent,
                         int width, int ld, void* stream);
 /* The sorted layout of pie_hip_moe_route_groups for a router of logistic scores s = sigmoid(logit): a token uses the
  * top_k experts with the largest s + correction (lowest index among equals), weighted by their s.  `shared` experts

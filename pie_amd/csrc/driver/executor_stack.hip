@@ -738,14 +738,15 @@ void Executor::stack_gated(int N, int max_kv_len, const Inputs& in) {
                                 reinterpret_cast<const int32_t*>(in_dev_ + in.off_pair), model_.embed, model_.bigram, model_.embed_norm, m.vocab,
                                 m.embed_scale};
     struct Sublayer {
-        const float *norm, *canon, *gate_bias;
+        const float *norm, *gate_bias;
+        const uint16_t* canon;
         const Linear* gate;
         size_t state;   // of the convolution
     };
     auto sublayer = [&](size_t run, int n) {
         const StackLayer& w = model_.stack[static_cast<size_t>(model_.runs[run].layer)];
-        return n == 0 ? Sublayer{w.pre1, w.canon1, w.gate1_bias, &w.w_gate1, rs_canon_off_[run][0]}
-                      : Sublayer{w.pre2, w.canon2, w.gate2_bias, &w.w_gate2, rs_canon_off_[run][1]};
+        return n == 0 ? Sublayer{w.pre1, w.gate1_bias, w.canon1, &w.w_gate1, rs_canon_off_[run][0]}
+                      : Sublayer{w.pre2, w.gate2_bias, w.canon2, &w.w_gate2, rs_canon_off_[run][1]};
     };
     // the output of `from` (null: the embedding starts the stream) joins the stream, which `to` (null: the last one
     // has ended) reads

@@ -163,7 +163,8 @@ struct StackLayer {
     float* correction = nullptr;                      // mixture: added to the scores for the choice (CorrectedScores)
     // gated sublayers: gate product and bias, convolution [taps, width] ahead of mixer and feed-forward
     Linear w_gate1, w_gate2;
-    float *gate1_bias = nullptr, *gate2_bias = nullptr, *canon1 = nullptr, *canon2 = nullptr;
+    float *gate1_bias = nullptr, *gate2_bias = nullptr;
+    uint16_t *canon1 = nullptr, *canon2 = nullptr;
     // latent attention
     Linear w_uq;
     Linear w_ukv;                                // [heads * (dimp + vdp), kvp]: keys and values out of the latent

@@ -175,18 +175,13 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
         PIE_HIP_CHECK(hipStreamSynchronize(stream));
         return d;
     };
-    // a convolution's taps, one after the other: [width, taps] -> [taps, width] fp32
+    // a convolution's taps, one after the other: [width, taps] -> [taps, width]
     auto tap_major = [&](const std::string& name, int taps) {
-        std::vector<float> v(static_cast<size_t>(taps) * H, 0.25f);
-        if (!random) {
+        return device_matrix(name, static_cast<size_t>(taps) * H, taps, [&](std::vector<uint16_t>& host) {
             const HostMatrix m = matrix(name, H, taps);
             for (int c = 0; c < H; ++c)
-                for (int j = 0; j < taps; ++j) v[static_cast<size_t>(j) * H + c] = bf16_value(m.row(c)[j]);
-        }
-        float* d = static_cast<float*>(alloc(4 * v.size(), name));
-        PIE_HIP_CHECK(hipMemcpyAsync(d, v.data(), 4 * v.size(), hipMemcpyHostToDevice, stream));
-        PIE_HIP_CHECK(hipStreamSynchronize(stream));
-        return d;
+                for (int j = 0; j < taps; ++j) host[static_cast<size_t>(j) * H + c] = m.row(c)[j];
+        });
     };
     stack_norm = cfg.gated_sublayers ? scalar_norm("final.norm") : vec("final.norm", H, ones);
     if (cfg.gated_sublayers) embed_norm = scalar_norm("embed.norm");
@@ -215,7 +210,7 @@ void Model::load_stack(const ModelConfig& cfg, hipStream_t stream) {
         const char *post1 = cfg.sandwich_norms ? "norm1b" : "norm1", *post2 = cfg.sandwich_norms ? "norm2b" : "norm2";
         const std::string p = "l" + std::to_string(l) + ".", mix = p + "mix.";
         // what surrounds sublayer n of a gated pair
-        auto gated_sublayer = [&](const std::string& n, float*& norm, float*& canon, Linear& gate, float*& bias) {
+        auto gated_sublayer = [&](const std::string& n, float*& norm, uint16_t*& canon, Linear& gate, float*& bias) {
             norm = scalar_norm(p + "norm" + n);
             canon = tap_major(p + "canon" + n, cfg.canon_taps);
             linear(gate, p + "rg" + n, Hp, Hp, H, [&](auto put) { plain_rows(put, p + "rg" + n, 0, H, H); });

@@ -145,14 +145,14 @@ __global__ __launch_bounds__(kWave) void head_linear_mfma_kernel(const HeadArgs 
     for (int t = 0; t < MT; ++t)
         ap[t] = static_cast<const uint16_t*>(a.act) + static_cast<size_t>(min(m0 + 16 * t + l16, a.M - 1)) * a.ld_act +
                 static_cast<size_t>(h) * a.act_stride + 8 * g;
-    // (requested ahead of the products)
-    float head_gate[MT];
-    u32x2_t value_gate[MT];
+    // (requested ahead of the products; without a gate infinities, whose logistic function is 1)
+    u32x2_t gates[MT];
 #pragma unroll
     for (int t = 0; t < MT; ++t) {
         const uint16_t* gp = static_cast<const uint16_t*>(a.gate) + static_cast<size_t>(min(m0 + 16 * t + l16, a.M - 1)) * a.ld_gate;
-        if (a.gate && a.gate_cols == 1) head_gate[t] = bf16_bits_to_f32(gp[h]);
-        else if (a.gate) value_gate[t] = *reinterpret_cast<const u32x2_t*>(gp + h * a.C + c0 + 4 * g);
+        gates[t] = u32x2_t{0x7F807F80u, 0x7F807F80u};
+        if (a.gate && a.gate_cols == 1) gates[t].x = gates[t].y = gp[h] * 0x10001u;
+        else if (a.gate) gates[t] = *reinterpret_cast<const u32x2_t*>(gp + h * a.C + c0 + 4 * g);
     }
     f32x4_t acc[MT];
 #pragma unroll
@@ -182,13 +182,8 @@ __global__ __launch_bounds__(kWave) void head_linear_mfma_kernel(const HeadArgs 
         const int m = m0 + 16 * t + l16;
         if (m >= a.M) continue;
         uint16_t* yp = static_cast<uint16_t*>(a.y) + static_cast<size_t>(m) * a.ld_y + static_cast<size_t>(h) * a.y_stride + c0 + 4 * g;
-        f32x4_t v = acc[t];
-        if (a.gate && a.gate_cols == 1) {
-            v *= sigmoid_f32(head_gate[t]);
-        } else if (a.gate) {
-            const u32x2_t r = value_gate[t];
-            v *= f32x4_t{sigmoid_f32(bf16_lo(r.x)), sigmoid_f32(bf16_hi(r.x)), sigmoid_f32(bf16_lo(r.y)), sigmoid_f32(bf16_hi(r.y))};
-        }
+        const u32x2_t r = gates[t];
+        const f32x4_t v = acc[t] * f32x4_t{sigmoid_f32(bf16_lo(r.x)), sigmoid_f32(bf16_hi(r.x)), sigmoid_f32(bf16_lo(r.y)), sigmoid_f32(bf16_hi(r.y))};
         *reinterpret_cast<u32x2_t*>(yp) = u32x2_t{pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3])};
     }
 }

@@ -4,6 +4,7 @@ part, against double-precision statements."""
 import numpy as np
 import pytest
 
+from layer_stack_util import bf16
 from oracle import layer_stack as ls
 from test_decay_memory_gpu import host, i32, t
 from test_layer_stack_kernels_gpu import paged
@@ -58,10 +59,10 @@ def test_an_embedding_starts_the_stream(gpu, bf, width, ld, pairs):
     ew, nw = (rng.uniform(0.5, 1.5, width).astype(np.float32) for _ in range(2))
     held = [i32(toks, gpu), i32(pair, gpu), t(ew, gpu)]
     start = ops.embedding(held[0], table, 2.5, held[2], held[1] if pairs else None, bigram if pairs else None)
-    s, w = Slots(rng, gpu, dt, width, 3, [1] * rows, [1] * rows), rng.standard_normal((3, width)).astype(np.float32)
+    s, w = Slots(rng, gpu, dt, width, 3, [1] * rows, [1] * rows), bf16(rng.standard_normal((3, width)))
     e = host(table)[np.where(toks < 50, toks, 0)] * 2.5 + (host(bigram)[pair] if pairs else 0.0)
     want = ls.rms_norm(e, ew, eps)
-    for kw in (dict(next_weight=t(nw, gpu)), dict(next_weight=t(nw, gpu), conv_w=t(w, gpu), rows=s.rows), dict()):
+    for kw in (dict(next_weight=t(nw, gpu)), dict(next_weight=t(nw, gpu), conv_w=t(w, gpu, torch.bfloat16), rows=s.rows), dict()):
         x = t(np.full((rows, ld), 3.0, np.float32), gpu)   # (what was there before does not matter)
         h, recent = (host(v) for v in ops.gated_join(x, width, eps, dt, start=start, **kw))
         assert np.abs(host(x)[:, :width] - want).max() < 1e-5 and (host(x)[:, width:] == 3.0).all()
@@ -91,7 +92,7 @@ def test_gated_join(gpu, bf, width, ld, taps):
         if use == "last" and taps:
             continue
         s = Slots(rng, gpu, dt, width, taps, [1] * rows, [0, 1, 0, 0, 1]) if taps else None
-        w = rng.standard_normal((taps, width)).astype(np.float32) if taps else None
+        w = bf16(rng.standard_normal((taps, width))) if taps else None
         x0 = rng.standard_normal((rows, ld)).astype(np.float32)
         x, kw, want = t(x0, gpu), {}, x0[:, :width].astype(np.float64)
         if use in ("sublayer", "last"):
@@ -100,7 +101,7 @@ def test_gated_join(gpu, bf, width, ld, taps):
         if use == "mixture":
             kw.update(routes=(ry, t(pos, gpu), t(weight, gpu)), gate=gate, gate_bias=t(bias, gpu))
             want = want + mix * g
-        h, recent = ops.gated_join(x, width, eps, dt, next_weight=None if use == "last" else t(nw, gpu), conv_w=t(w, gpu) if taps else None,
+        h, recent = ops.gated_join(x, width, eps, dt, next_weight=None if use == "last" else t(nw, gpu), conv_w=t(w, gpu, torch.bfloat16) if taps else None,
                                    rows=s.rows if taps else None, **kw)
         assert np.abs(host(x)[:, :width] - want).max() < 3e-5 and np.array_equal(host(x)[:, width:], x0[:, width:])
         if use == "last":
@@ -125,8 +126,8 @@ def test_recent_rows(gpu, bf, width, ld, taps, lens):
     rng = np.random.default_rng(width + taps + len(lens))
     dt = torch.bfloat16 if bf else torch.float32
     s = Slots(rng, gpu, dt, width, taps, lens, [r % 3 == 1 for r in range(len(lens))])
-    h, w = t(rng.standard_normal((sum(lens), ld)), gpu, dt), rng.standard_normal((taps, width)).astype(np.float32)
-    got = host(ops.recent_rows(h, t(w, gpu), s.rows))
+    h, w = t(rng.standard_normal((sum(lens), ld)), gpu, dt), bf16(rng.standard_normal((taps, width)))
+    got = host(ops.recent_rows(h, t(w, gpu, torch.bfloat16), s.rows))
     out, states = s.want(host(h)[:, :width], w)
     assert (np.abs(got[:, :width] - out) < (5e-3 if bf else 1e-5) * (1.0 + np.abs(out))).all() and (got[:, width:] == 0).all()
     if taps > 1:
@@ -314,12 +315,12 @@ def test_bad_arguments_are_refused(gpu):
     nw = torch.ones(96, device=gpu)
     tok, table = torch.zeros(2, dtype=torch.int32, device=gpu), torch.zeros((3, 96), dtype=torch.bfloat16, device=gpu)
     start = ops.embedding(tok, table, 1.0, nw)
-    for kw in (dict(), dict(y=y, next_weight=nw), dict(y=y, gate=y, gate_bias=nw, start=start), dict(start=ops.embedding(tok, table, 1.0, nw, None, table)), dict(next_weight=nw, conv_w=torch.zeros((3, 96), device=gpu)), dict(y=y, gate=y)):
+    for kw in (dict(), dict(y=y, next_weight=nw), dict(y=y, gate=y, gate_bias=nw, start=start), dict(start=ops.embedding(tok, table, 1.0, nw, None, table)), dict(next_weight=nw, conv_w=torch.zeros((3, 96), dtype=torch.bfloat16, device=gpu)), dict(y=y, gate=y)):
         with pytest.raises(KernelError):
             ops.gated_join(x, 96, 1e-5, torch.float32, **kw)
     rng = np.random.default_rng(0)
     s = Slots(rng, gpu, torch.float32, 96, 3, [2], [0])   # (two rows of one request: not one each)
     with pytest.raises(KernelError):
-        ops.gated_join(x, 96, 1e-5, torch.float32, next_weight=nw, conv_w=torch.zeros((3, 96), device=gpu), rows=s.rows)
+        ops.gated_join(x, 96, 1e-5, torch.float32, next_weight=nw, conv_w=torch.zeros((3, 96), dtype=torch.bfloat16, device=gpu), rows=s.rows)
     with pytest.raises(KernelError):
         ops.head_linear(torch.zeros((1, 2, 32), device=gpu), torch.zeros((2, 16, 32), dtype=torch.bfloat16, device=gpu), gate=z[:1], gate_cols=2)
